@@ -96,10 +96,19 @@ def _build_lib(sources: list[Path], headers: list[Path], compiler: str, flags: l
     return out
 
 
-def build_kernels(jobs: int | None = None, verbose: bool = True) -> Path:
+def kernel_subset_lib(names) -> Path:
+    """Library of the given csrc/kernels sources alone (a model that runs before the whole is built)."""
+    return LIB_DIR / ("libcfc_kernels_" + "_".join(sorted(names)) + ".so")
+
+
+def build_kernels(jobs: int | None = None, verbose: bool = True, names=None) -> Path:
+    """The kernels library, or with ``names`` a library of those sources only."""
     srcs = sorted((CSRC / "kernels").glob("*.hip"))
+    if names is not None:
+        srcs = [s for s in srcs if s.stem in names]
     hdrs = sorted((CSRC / "kernels").glob("*.h"))
-    return _build_lib(srcs, hdrs, HIPCC, HIP_FLAGS, KERNELS_LIB, [f"--offload-arch={OFFLOAD_ARCH}"],
+    out = KERNELS_LIB if names is None else kernel_subset_lib(names)
+    return _build_lib(srcs, hdrs, HIPCC, HIP_FLAGS, out, [f"--offload-arch={OFFLOAD_ARCH}"],
                       jobs or min(8, os.cpu_count() or 4), verbose)
 
 

@@ -25,6 +25,7 @@ import math
 import os
 from pathlib import Path
 
+import numpy as np
 import torch
 import torch.nn.functional as F
 
@@ -497,6 +498,31 @@ class DecoderModel:
             self.fused_decode = True
             self.prefill_gemm = "hip"
 
+    # ---------------------------------------------------------------- engine interface
+    # kernel sources (csrc/kernels/<name>.hip) a run of this family loads
+    kernel_sources = None        # the whole library
+
+    def new_cache(self, num_blocks: int, dtype=None, device=None):
+        from ..runtime.kv_cache import PagedKVCache
+        return PagedKVCache(self.cfg.layers, num_blocks, self.w.kv_heads, self.cfg.head_dim, device or self.w.device,
+                            dtype=dtype or torch.bfloat16)
+
+    def decode_groups(self) -> int:
+        """Attention workgroups per sequence and KV partition of a decode step."""
+        return self.w.kv_heads
+
+    def decode_workspace(self, B: int, P: int) -> int:
+        """fp32 elements of the split-KV partials of a B-row decode step over P partitions."""
+        return B * self.w.heads * P * (self.cfg.head_dim + 2) if P > 1 else 1
+
+    def plan_prefill(self, cu, ctx, slots) -> dict:
+        """Host-side launch plan of a packed prefill (int32 arrays): the attention's query tiles and the
+        per-block runs of the V write."""
+        # query rows per prefill attention tile (the GQA-packed kernel takes 256 / G)
+        rows = K.prefill_rows(self.w.heads, self.w.kv_heads) if self.w.device.type == "cuda" else K.PREFILL_TILE_ROWS
+        seq, q0 = K.prefill_tiles(cu, rows, ctx)
+        return {"tile_seq": np.asarray(seq, np.int32), "tile_q0": np.asarray(q0, np.int32), "v_runs": K.v_runs(slots)}
+
     PACKED_FREE_FRACTION = 0.3   # HBM left free after packing when both copies are kept
     PREFILL_GEMM_DEFAULT = "hip"
     # "ppp": the persistent ping-pong kernel (one workgroup per CU walking the tiles, the DMA
@@ -649,10 +675,13 @@ class DecoderModel:
         return self._all_reduce(self._plin(i, "down", a))
 
     def forward_prefill(self, ids, positions, slots, cu_q, ctx_lens, block_tables, kv, tiles=None,
-                        last_idx=None, v_runs=None) -> torch.Tensor:
+                        last_idx=None, v_runs=None, plan=None) -> torch.Tensor:
         """Packed varlen prefill. Returns hidden states of rows ``last_idx`` (or all rows).
-        ``v_runs`` (ops.kernels.v_runs of the slots, on device): V written per cache block."""
+        ``v_runs`` (ops.kernels.v_runs of the slots, on device): V written per cache block.  ``plan``:
+        :meth:`plan_prefill`'s arrays on the device (``tiles`` and ``v_runs`` from it)."""
         cfg, w = self.cfg, self.w
+        if plan is not None:
+            tiles, v_runs = (plan["tile_seq"], plan["tile_q0"]), plan["v_runs"]
         x = K.embedding(w.embed, ids)
         residual = None
         x32 = None                     # TP fp32: this rank's fp32 partial of the previous layer's down
@@ -700,6 +729,8 @@ class DecoderModel:
         about as long as the rank's GEMMs, which would otherwise wait for it."""
         cfg, w = self.cfg, self.w
         dist = torch.distributed
+        halves = [dict(m, tiles=(m["plan"]["tile_seq"], m["plan"]["tile_q0"]), v_runs=m["plan"]["v_runs"])
+                  if m.get("plan") is not None else m for m in halves]
         st = [{"m": m, "x": K.embedding(w.embed, m["ids"]), "res": None, "work": None} for m in halves]
         f32 = self.tp_fp32
         eps = cfg.rms_eps

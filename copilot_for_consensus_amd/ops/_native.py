@@ -50,9 +50,17 @@ _KERNEL_SIGS = {
     "cfc_silu_mul_fp8": [P, P, P, I, I, I, P],
     "cfc_bias_gelu": [P, P, P, I, I, P],
     "cfc_embedding": [P, P, P, I, I, P],
-    "cfc_sample": [P, I, I, F, c_uint32, P, P, P],
-    "cfc_sample_truncated": [P, I, I, F, I, F, F, c_uint32, P, P, P],
+    "cfc_sample": [P, I, I, I, F, c_uint32, P, P, P],
+    "cfc_sample_truncated": [P, I, I, I, F, I, F, F, c_uint32, P, P, P],
     "cfc_decode_advance": [P, P, I, P, P, P, P, P, P, I, P, P, I, I] + [P] * 6 + [I] * 4 + [P] * 4,
+    "cfc_embed_f32": [P, P, P, I, I, I, I, P],
+    "cfc_depth_norm": [I, I, I, P, P, P, P, I, P, P, I, P, F, P, P, I, I, P, I, P, I, P, P, I, P, P, I, P, I, P],
+    "cfc_input_conv": [I, I, P, P, P, P, P, P, I, P, I, P, I, I, P, I, P, I, P],
+    "cfc_clamped_glu": [I, I, P, I, P, P, P, I, I, I, F, F, F, P],
+    "cfc_softcap": [P, c_int64, F, P],
+    "cfc_latent_norm": [I, P, I, I, I, I, P, P, F, P, P, I, P, I, P],
+    "cfc_head_linear": [I, P, c_int64, c_int64, P, I, I, I, I, I, I, P, c_int64, c_int64, P],
+    "cfc_latent_attention": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, P, P, P],
     "cfc_knn_scores": [P, P, I, I, I, P, P, P, P],
     "cfc_topk_pass": [P, P, I, I, I, I, P, P, P],
     "cfc_knn_topk": [P, P, I, I, I, I, P, P, P, I, P, P, P],
@@ -150,6 +158,19 @@ def kernels():
                         "`python -c 'import __graft_entry__ as g; g.build()'` (hipcc, gfx950).")
                 _kernels = _bind(ctypes.CDLL(str(lib), mode=os.RTLD_LOCAL), _KERNEL_SIGS)
     return _kernels
+
+
+def ensure_kernels(names=None):
+    """Load the kernels library, compiling what is needed first when the library is not built: the sources
+    ``names`` of csrc/kernels (None: all of them), as a library of their own."""
+    global _kernels
+    if _kernels is None and not os.environ.get("CFC_KERNELS_LIB") and not KERNELS_LIB.exists():
+        from .._build import build_kernels
+        lib = build_kernels(verbose=False, names=names)
+        with _lock:
+            if _kernels is None:
+                _kernels = _bind(ctypes.CDLL(str(lib), mode=os.RTLD_LOCAL), _KERNEL_SIGS)
+    return kernels()
 
 
 def runtime():

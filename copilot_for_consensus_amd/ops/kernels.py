@@ -1215,14 +1215,15 @@ def sample(logits, out_ids, temperature=0.0, seed=0, step=None):
                 p = torch.softmax(logits.float() / sp.temperature, -1)
                 out_ids.copy_(torch.multinomial(p, 1, generator=g)[:, 0].to(torch.int32))
         return out_ids
-    _req(logits, torch.bfloat16, "logits")
+    f32 = int(logits.dtype == torch.float32)
+    _req(logits, torch.float32 if f32 else torch.bfloat16, "logits")
     B, V = logits.shape
     if sp.truncated:
-        check(kernels().cfc_sample_truncated(logits.data_ptr(), B, V, sp.temperature, int(sp.top_k), float(sp.top_p),
+        check(kernels().cfc_sample_truncated(logits.data_ptr(), f32, B, V, sp.temperature, int(sp.top_k), float(sp.top_p),
                                              float(sp.min_p), int(seed) & 0xFFFFFFFF, _p(step), out_ids.data_ptr(),
                                              _stream(logits)), "cfc_sample_truncated")
         return out_ids
-    check(kernels().cfc_sample(logits.data_ptr(), B, V, float(sp.temperature), int(seed) & 0xFFFFFFFF, _p(step),
+    check(kernels().cfc_sample(logits.data_ptr(), f32, B, V, float(sp.temperature), int(seed) & 0xFFFFFFFF, _p(step),
                                out_ids.data_ptr(), _stream(logits)), "cfc_sample")
     return out_ids
 

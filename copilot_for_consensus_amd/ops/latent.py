@@ -1,0 +1,143 @@
+"""Latent attention ops (csrc/kernels/latent.hip): the norms of both latents with the cache write, the
+per-head products around the attention, and attention over the paged latents.
+
+GPU tensors go to the native library (which must be built), CPU tensors to the fp32 reference.
+"""
+from __future__ import annotations
+
+import math
+
+import torch
+
+from . import reference as ref
+from ._native import check, kernels
+from .kernels import _p, _req, _stream, _workspace
+from .stream import _act
+
+MFMA_MAX_RANK = 512       # latent ranks the MFMA attention kernel is built for
+ANY_ROWS = 4              # rows per tile of the general kernel
+
+
+def padded_rank(rank: int) -> int:
+    """Latent row stride: the rank rounded up to one MFMA step (32); the pad columns stay zero."""
+    return 32 * math.ceil(rank / 32)
+
+
+class HeadWeight:
+    """Per-head matrices [H, N, K] zero-padded to [H, 64 x, 32 y] for :func:`head_linear`."""
+
+    __slots__ = ("data", "H", "N", "K")
+
+    def __init__(self, w: torch.Tensor, n_out: int | None = None, k_in: int | None = None):
+        H, N, K = w.shape
+        self.H, self.N, self.K = H, n_out or N, k_in or K
+        self.data = torch.zeros(H, 64 * math.ceil(self.N / 64), 32 * math.ceil(self.K / 32), dtype=w.dtype, device=w.device)
+        self.data[:, :N, :K] = w
+
+    def nbytes(self) -> int:
+        return self.data.numel() * self.data.element_size()
+
+
+def head_linear(x: torch.Tensor, w: HeadWeight, out: torch.Tensor) -> torch.Tensor:
+    """out[t, h, :N] = w[h] x[t, h, :K].  x [T, H, >= K], out [T, H, >= N]: any row / head strides, last dim dense."""
+    T, H = x.shape[0], x.shape[1]
+    if H != w.H or out.shape[:2] != (T, H) or x.shape[2] < w.K or out.shape[2] < w.N:
+        raise ValueError(f"head_linear: x {tuple(x.shape)} w {w.H} x {w.N} x {w.K} out {tuple(out.shape)}")
+    if not x.is_cuda:
+        y = torch.matmul(x[:, :, :w.K].float().transpose(0, 1), w.data[:, :w.N, :w.K].float().transpose(1, 2))
+        out[:, :, :w.N] = y.transpose(0, 1).to(out.dtype)
+        return out
+    if x.stride(2) != 1 or out.stride(2) != 1 or x.dtype != out.dtype or x.dtype != w.data.dtype:
+        raise ValueError("head_linear: dense last dimensions and one dtype needed")
+    check(kernels().cfc_head_linear(_act(x.dtype), x.data_ptr(), x.stride(0), x.stride(1), w.data.data_ptr(),
+                                    w.data.shape[1], w.data.shape[2], T, H, w.N, w.K, out.data_ptr(), out.stride(0),
+                                    out.stride(1), _stream(x)), "cfc_head_linear")
+    return out
+
+
+def latent_norm(part, nq: int, wq, wc, eps: float, slots, cache, dtype) -> torch.Tensor:
+    """part: fp32 slabs [split, T, nq + rank] of the joint down projection.  Writes the normed cached
+    latent into ``cache`` [blocks, 32, RS] at ``slots``; returns the normed query latent [T, nq]."""
+    T, N = part.shape[1], part.shape[2]
+    RS = cache.shape[-1]
+    if not part.is_cuda:
+        q, c = ref.latent_norm(part, nq, wq, wc, eps)
+        cache.view(-1, RS)[slots.long(), :N - nq] = c.to(cache.dtype)
+        return q.to(dtype)
+    _req(part, torch.float32, "part")
+    _req(slots, torch.int32, "slots")
+    if cache.dtype != dtype:
+        raise TypeError(f"latent cache {cache.dtype}, activations {dtype}")
+    out = torch.empty(T, nq, dtype=dtype, device=part.device)
+    check(kernels().cfc_latent_norm(_act(dtype), part.data_ptr(), part.shape[0], T, nq, N - nq, wq.data_ptr(),
+                                    wc.data_ptr(), float(eps), slots.data_ptr(), out.data_ptr(), nq, cache.data_ptr(), RS,
+                                    _stream(part)), "cfc_latent_norm")
+    return out
+
+
+def rows_per_tile(dtype, RS: int, heads: int, decode: bool) -> int:
+    """(token, head) rows of one attention work item: the general kernel's 4, or 16 / 32 / 64 on MFMA."""
+    if dtype != torch.bfloat16 or RS > MFMA_MAX_RANK:
+        return ANY_ROWS
+    if not decode:
+        return 64
+    return 16 if heads <= 16 else (32 if heads <= 32 else 64)
+
+
+def attn_tiles(cu_q, heads: int, rows: int, ctx_lens=None):
+    """(sequence, first row) of every work item of a packed batch; with ``ctx_lens`` those with the most
+    keys first, so the long ones do not end the grid alone."""
+    tiles = []
+    for s in range(len(cu_q) - 1):
+        n = cu_q[s + 1] - cu_q[s]
+        base = ctx_lens[s] - n if ctx_lens is not None else 0
+        for m0 in range(0, n * heads, rows):
+            tiles.append((base + (min(m0 + rows, n * heads) - 1) // heads, s, m0))
+    if ctx_lens is not None:
+        tiles.sort(key=lambda t: -t[0])
+    return [t[1] for t in tiles], [t[2] for t in tiles]
+
+
+def partitions(n_tiles: int, max_ctx: int, target: int = 512) -> int:
+    """Key slices per work item: enough workgroups to fill the chip, at least four 64-key tiles each."""
+    return max(1, min(math.ceil(target / max(1, n_tiles)), math.ceil(max_ctx / 256)))
+
+
+def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles=None, rows: int | None = None,
+                     P: int = 1, workspace=None) -> torch.Tensor:
+    """Softmax attention of q [T, H, RS] over the paged latents [blocks, 32, RS], causal inside each
+    sequence's portion.  ``cu_q`` None: one token per sequence.  ``tiles``: device (tile_seq, tile_m0) of
+    :func:`attn_tiles` cut for ``rows``; P key slices per tile merged at the end."""
+    T, H, RS = q.shape
+    B = ctx_lens.numel()
+    if not q.is_cuda:
+        cu = cu_q if cu_q is not None else torch.arange(B + 1)
+        return ref.latent_attention(q, cache, block_tables, cu, ctx_lens, scale)
+    if not q.is_contiguous() or not cache.is_contiguous() or cache.shape[-1] != RS or cache.dtype != q.dtype:
+        raise ValueError(f"latent_attention: q {tuple(q.shape)} {q.dtype}, cache {tuple(cache.shape)} {cache.dtype}")
+    for name, t in (("block_tables", block_tables), ("ctx_lens", ctx_lens)):
+        _req(t, torch.int32, name)
+    rows = rows or rows_per_tile(q.dtype, RS, H, cu_q is None)
+    if cu_q is None:
+        if T != B:
+            raise ValueError(f"latent_attention: {T} rows for {B} sequences")
+        per_seq = math.ceil(H / rows)
+        ts = tm = None
+        n_tiles = B * per_seq
+    else:
+        if tiles is None:
+            a, b = attn_tiles(cu_q.tolist(), H, rows, ctx_lens.tolist())
+            tiles = tuple(torch.tensor(v, dtype=torch.int32, device=q.device) for v in (a, b))
+        ts, tm = tiles
+        per_seq, n_tiles = 0, ts.numel()
+    out = torch.empty_like(q)
+    po = pm = None
+    if P > 1:
+        need = T * H * P * (RS + 2)
+        ws = workspace if workspace is not None and workspace.numel() >= need else _workspace(q.device, need)
+        po, pm = ws[:T * H * P * RS], ws[T * H * P * RS:need]
+    check(kernels().cfc_latent_attention(_act(q.dtype), q.data_ptr(), cache.data_ptr(), block_tables.data_ptr(), _p(cu_q),
+                                         ctx_lens.data_ptr(), _p(ts), _p(tm), n_tiles, per_seq, rows, H, RS,
+                                         block_tables.shape[1], float(scale), P, T * H, _p(po), _p(pm), out.data_ptr(),
+                                         _stream(q)), "cfc_latent_attention")
+    return out

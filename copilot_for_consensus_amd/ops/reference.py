@@ -315,3 +315,74 @@ def quant_fp8_rows(x: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor]:
     amax = xf.abs().amax(1, keepdim=True)
     s = torch.where(amax > 0, amax / 448.0, torch.ones_like(amax))
     return (xf / s).clamp(-448.0, 448.0).to(torch.float8_e4m3fn), s
+
+
+# ----------------------------------------------------- 32-bit residual stream (stream.hip)
+def tail_slots(taps: int) -> int:
+    """Convolution inputs a cache block keeps per layer: the taps - 1 live ones and two spare rows (a
+    position that is run again must not overwrite what it reads), never more than the block's positions."""
+    return 0 if taps <= 1 else min(taps + 1, KV_BLOCK)
+
+
+def depth_norm(x, hist, part, bias, dwa, n, eps):
+    """X_n = x + sum of part slabs + bias into hist[n]; returns (sum_j dwa[j] X_j, 1 / rms of it)."""
+    if part is not None:
+        new = x + part.sum(0) + (bias if bias is not None else 0.0)
+        hist[n].copy_(new)
+        x = torch.einsum("j,jtw->tw", dwa[:n + 1].float(), hist[:n + 1])
+    return x, 1.0 / torch.sqrt((x * x).mean(-1) + eps)
+
+
+def input_conv(h, portions, block_tables, tail, weights):
+    """h [T, W] fp32 convolution inputs of packed portions [(first row, rows, first position, sequence)];
+    tail [blocks, slots, W] read for positions before a portion and updated.  weights: per sublayer
+    [W, taps].  Returns one h + conv(h) per sublayer."""
+    outs = [h.clone() for _ in weights]
+    taps = weights[0].shape[1]
+    for row0, n, pos0, seq in portions:
+        past = []
+        for q in range(pos0 - taps + 1, pos0):
+            if q < 0:
+                past.append(torch.zeros_like(h[0]))
+            else:
+                past.append(tail[int(block_tables[seq, q // KV_BLOCK]), q % tail.shape[1]])
+        ext = torch.cat([torch.stack(past), h[row0:row0 + n]]) if past else h[row0:row0 + n]
+        for o, w in zip(outs, weights):
+            for j in range(taps):
+                o[row0:row0 + n] += w[:, j] * ext[j:j + n]
+        for r in range(n):
+            q = pos0 + r
+            # the last inputs of the portion and of every block it crosses
+            if taps > 1 and (r >= n - (taps - 1) or KV_BLOCK - q % KV_BLOCK <= taps - 1):
+                tail[int(block_tables[seq, q // KV_BLOCK]), q % tail.shape[1]] = h[row0 + r]
+    return outs
+
+
+def clamped_glu(g, u, limit, alpha, beta):
+    g = torch.clamp(g, max=limit)
+    u = torch.clamp(u, min=-limit, max=limit)
+    return g * torch.sigmoid(alpha * g) * (u + beta)
+
+
+# ----------------------------------------------------- latent attention (latent.hip)
+def latent_norm(part, nq, wq, wc, eps):
+    """(normed query latent, normed cached latent) of the joint down projection's fp32 slabs."""
+    y = part.sum(0)
+    q, c = y[:, :nq], y[:, nq:]
+    q = q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * wq
+    c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * wc
+    return q, c
+
+
+def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale):
+    """q [T, H, RS]; cache [blocks, 32, RS]: softmax over the sequence's latents, per row causal."""
+    out = torch.empty_like(q)
+    for s in range(len(ctx_lens)):
+        a, b, ctx = int(cu_q[s]), int(cu_q[s + 1]), int(ctx_lens[s])
+        nb = -(-ctx // KV_BLOCK)
+        c = cache[block_tables[s, :nb].long()].reshape(nb * KV_BLOCK, -1)[:ctx].float()
+        sc = torch.matmul(q[a:b].float(), c.t()) * scale                        # [n, H, ctx]
+        pos = torch.arange(ctx - (b - a), ctx)
+        sc.masked_fill_((torch.arange(ctx)[None] > pos[:, None])[:, None], float("-inf"))
+        out[a:b] = torch.matmul(torch.softmax(sc, -1), c).to(q.dtype)
+    return out

@@ -35,9 +35,9 @@ class BenchPipeline:
                  max_new_tokens=512, tp=1, prefill_tokens=16384, llm_only=False, use_graph=True, seed=0,
                  index_prefill=1_000_000, groups=None, kv_dtype="bf16", weight_dtype="bf16", kv_max_prompt=4096,
                  index_group=None, overlap_prefill=False):
-        from ..models.decoder import DecoderModel, DecoderWeights, get_config
+        from ..models import registry
         from ..runtime.engine import LLMEngine
-        from ..runtime.kv_cache import PagedKVCache, blocks_needed
+        from ..runtime.kv_cache import blocks_needed
 
         self.groups = groups
         tp_rank = groups.tp_rank if groups is not None else 0
@@ -48,20 +48,20 @@ class BenchPipeline:
         # TP followers run the LLM only; the leader prepares the batch and broadcasts the prompts
         self.follower = tp > 1 and tp_rank != 0
         self.device = torch.device(device)
-        self.cfg = get_config(model)
+        self.cfg = registry.get_config(model)
         self.threads_per_step = threads_per_step
         self.max_new = max_new_tokens
         self.llm_only = llm_only
         self.rng = random.Random(seed)
         self.seed = seed
-        w = DecoderWeights.random(self.cfg, self.device, seed=1234, tp_rank=tp_rank, tp_size=tp)
+        w = registry.random_weights(self.cfg, self.device, seed=1234, tp_rank=tp_rank, tp_size=tp)
         if weight_dtype == "fp8":
             w.to_fp8()           # opt-in W8A8 FP8 projections (precision trade-off, not the headline)
         custom_ar = None
         if tp > 1:
             from ..parallel.custom_ar import maybe_create
             custom_ar = maybe_create(groups.tp_group, self.device, exchange_group=groups.tp_cpu_group)
-        self.model = DecoderModel(w, tp_group=groups.tp_group if tp > 1 else None, custom_ar=custom_ar)
+        self.model = registry.build_model(w, tp_group=groups.tp_group if tp > 1 else None, custom_ar=custom_ar)
         # KV budget: every thread of a step at ``kv_max_prompt`` prompt tokens + max_new, x1.1 (the
         # prompts this pipeline builds stay near 2.6k; a 70B model on one GPU needs the tighter bound)
         max_prompt = int(kv_max_prompt)
@@ -70,8 +70,7 @@ class BenchPipeline:
         nblk = int(1.1 * threads_per_step * blocks_needed(max_prompt + max_new_tokens)) + 64
         if self.overlap_prefill:
             nblk *= 2
-        kvd = {"bf16": torch.bfloat16, "fp8": torch.float8_e4m3fn}[kv_dtype]
-        self.kv = PagedKVCache(self.cfg.layers, nblk, w.kv_heads, self.cfg.head_dim, self.device, dtype=kvd)
+        self.kv = self.model.new_cache(nblk, dtype={"bf16": None, "fp8": torch.float8_e4m3fn}[kv_dtype])
         self.engine = LLMEngine(self.model, self.kv, max_prefill_tokens=prefill_tokens, use_graph=use_graph)
         self.rag = None
         # the next batch's encoder / kNN work runs on this stream beside the decode graph.  Its kernels

@@ -117,8 +117,7 @@ class ContinuousEngine:
         # workspace per width.
         self.widths = sorted({w for w in (1, 2, 4, 8, 16, 32, 64) if w < B} | {B})
         self._pb = {w: engine._part_blocks(w, self.max_blocks) for w in self.widths}
-        ws = max(w * self.model.w.heads * -pb * (self.model.cfg.head_dim + 2) if -pb > 1 else 1
-                 for w, pb in self._pb.items())
+        ws = max(self.model.decode_workspace(w, -pb) for w, pb in self._pb.items())
         self.workspace = torch.empty(max(1, ws), dtype=torch.float32, device=dev)
         self.part_blocks = self._pb[B]
         self.use_graph = engine._graph_for(B, self.sampling)
@@ -269,7 +268,7 @@ class ContinuousEngine:
                 tables.append(shared + new)
                 fresh.append(new)
                 start.append(len(shared) * KV_BLOCK)
-                if pc is not None:
+                if pc is not None and not self.engine.share_late:
                     pc.insert(r.prompt, tables[-1])
         except BaseException:
             self.engine._release(tables, fresh, failed=True)
@@ -291,6 +290,7 @@ class ContinuousEngine:
             self.engine._release(tables, fresh, failed=True)
             self.queue.extendleft(reversed(take))
             raise
+        self.engine._share_computed([r.prompt for r in take], tables)
         now = time.perf_counter()
         self.stats["prefill_s"] += now - t
         slots = [self.free.pop() for _ in take]

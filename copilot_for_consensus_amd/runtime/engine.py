@@ -109,9 +109,6 @@ class LLMEngine:
             import torch.distributed as dist
             self._gloo_tp = dist.get_backend(tp_group) == "gloo"
         self.last_used_graph = False
-        # query rows per prefill attention tile (the GQA-packed kernel takes 256 / G)
-        self._prefill_rows = (K.prefill_rows(model.w.heads, model.w.kv_heads) if kv.device.type == "cuda"
-                              else K.PREFILL_TILE_ROWS)
         self.stop_check_interval = stop_check_interval
         # host-side forward-progress counter (prefill chunks + decode steps issued): read by the DP
         # heartbeat (parallel/dp_node.py), it freezes when a GPU call hangs and the host blocks
@@ -122,6 +119,8 @@ class LLMEngine:
         if prefix_cache is None:
             prefix_cache = os.environ.get("CFC_PREFIX_CACHE", "1") != "0"
         self.prefix_cache = PrefixCache(kv.pool) if prefix_cache else None
+        # a cache whose blocks may be mapped by another sequence only once they are computed
+        self.share_late = getattr(kv, "share_after_compute", False)
         # CFC_DECODE_SHARED_CACHED=0: every KV block nontemporal, shared prefix included
         self.shared_cached = os.environ.get("CFC_DECODE_SHARED_CACHED", "1") != "0"
         # slots filled longest prompt first (CFC_DECODE_LPT=0: caller order).  The decode attention
@@ -153,7 +152,7 @@ class LLMEngine:
         CU).  Long KV runs per workgroup win: at B=128 P=1 streams 6.5 TB/s vs 5.0-5.4 for fixed
         26-block partitions (scripts/bench_decode_attn.py, profiles/decode_attn_partitions_r01.log)."""
         target = int(os.environ.get("CFC_DECODE_WGS", "512"))
-        P = max(1, math.ceil(target / max(1, B * self.model.w.kv_heads)))
+        P = max(1, math.ceil(target / max(1, B * self.model.decode_groups())))
         return -min(P, max(1, max_blocks // 2))
 
     def _i32(self, x):
@@ -224,41 +223,88 @@ class LLMEngine:
     def _chunk_meta(self, prompts, tables, chunk):
         """Device metadata of one packed prefill pass over ``chunk`` [(seq, first, end)]: the
         forward_prefill keyword arguments, the sequences finishing in it, and their ids on device."""
-        cu, ctx, rows, last_rows, finishing = [0], [], [], [], []
-        ids_np, pos_np, slot_np = [], [], []
+        finishing, last_rows, row = [], [], 0
         for (s, a, b) in chunk:
-            ids_np.append(np.asarray(prompts[s][a:b], dtype=np.int32))
-            p = np.arange(a, b, dtype=np.int32)
-            pos_np.append(p)
-            slot_np.append(np.asarray(tables[s], dtype=np.int32)[p // KV_BLOCK] * KV_BLOCK + p % KV_BLOCK)
-            cu.append(cu[-1] + (b - a))
-            ctx.append(b)
-            rows.append(s)
+            row += b - a
             if b == len(prompts[s]):
-                last_rows.append(cu[-1] - 1)
+                last_rows.append(row - 1)
                 finishing.append(s)
-        maxb = max(len(tables[s]) for s in rows)
-        bt = np.zeros((len(rows), maxb), dtype=np.int32)
-        for r, s in enumerate(rows):
-            bt[r, :len(tables[s])] = tables[s]
-        tseq, tq0 = K.prefill_tiles(cu, self._prefill_rows, ctx)
+        kw, extra = self._pass_meta([(prompts[s][a:b], a) for (s, a, b) in chunk], [tables[s] for (s, _, _) in chunk],
+                                    last_rows, np.asarray(finishing, np.int32))
+        return kw, finishing, extra
+
+    def _pass_meta(self, portions, tables, last_rows, extra=np.zeros(0, np.int32)):
+        """Device metadata of one packed pass over ``portions`` [(tokens, first position)] with their block
+        tables: the forward_prefill keyword arguments for the rows ``last_rows``, and ``extra`` (int32) on
+        the device."""
+        cu, ctx = [0], []
+        ids_np, pos_np, slot_np = [], [], []
+        for (toks, a), tbl in zip(portions, tables):
+            ids_np.append(np.asarray(toks, dtype=np.int32))
+            p = np.arange(a, a + len(toks), dtype=np.int32)
+            pos_np.append(p)
+            slot_np.append(np.asarray(tbl, dtype=np.int32)[p // KV_BLOCK] * KV_BLOCK + p % KV_BLOCK)
+            cu.append(cu[-1] + len(toks))
+            ctx.append(a + len(toks))
+        maxb = max(len(t) for t in tables)
+        bt = np.zeros((len(tables), maxb), dtype=np.int32)
+        for r, t in enumerate(tables):
+            bt[r, :len(t)] = t
         # everything the pass needs in ONE pinned host buffer and one non-blocking copy: a
         # pageable torch.tensor(..., device=cuda) synchronises the stream, so the GPU would idle
         # while the host builds the next chunk
         slots_np = np.concatenate(slot_np)
-        runs = K.v_runs(slots_np)
+        plan = self.model.plan_prefill(cu, ctx, slots_np)
+        arrays = [k for k, v in plan.items() if isinstance(v, np.ndarray)]
         parts = [np.concatenate(ids_np), np.concatenate(pos_np), slots_np,
-                 np.asarray(cu, np.int32), np.asarray(ctx, np.int32), np.asarray(tseq, np.int32),
-                 np.asarray(tq0, np.int32), np.asarray(last_rows, np.int32),
-                 np.asarray(finishing, np.int32), bt.reshape(-1), runs.reshape(-1)]
-        dev = self._h2d(np.concatenate(parts))
-        offs = np.cumsum([0] + [len(x) for x in parts]).tolist()
-        d_ids, d_pos, d_slots, d_cu, d_ctx, d_tseq, d_tq0, d_last, d_fin, d_bt, d_runs = (
-            dev[offs[i]:offs[i + 1]] for i in range(len(parts)))
+                 np.asarray(cu, np.int32), np.asarray(ctx, np.int32), np.asarray(last_rows, np.int32), extra,
+                 bt.reshape(-1)] + [plan[k].reshape(-1) for k in arrays]
+        # every array at a 16-byte offset of the buffer
+        offs = np.cumsum([0] + [-(-len(x) // 4) * 4 for x in parts]).tolist()
+        buf = np.zeros(offs[-1], np.int32)
+        for o, x in zip(offs, parts):
+            buf[o:o + len(x)] = x
+        dev = self._h2d(buf)
+        views = [dev[o:o + len(x)] for o, x in zip(offs, parts)]
+        d_ids, d_pos, d_slots, d_cu, d_ctx, d_last, d_extra, d_bt = views[:8]
+        plan.update((k, v.view(plan[k].shape)) for k, v in zip(arrays, views[8:]))
         kw = dict(ids=d_ids, positions=d_pos, slots=d_slots, cu_q=d_cu, ctx_lens=d_ctx,
-                  block_tables=d_bt.view(len(rows), maxb), tiles=(d_tseq, d_tq0),
-                  last_idx=d_last.long() if last_rows else None, v_runs=d_runs.view(-1, 4))
-        return kw, finishing, d_fin
+                  block_tables=d_bt.view(len(tables), maxb), plan=plan, last_idx=d_last.long() if last_rows else None)
+        return kw, d_extra
+
+    # ------------------------------------------------------------------ single steps
+    @torch.inference_mode()
+    def forward_step(self, entries) -> torch.Tensor | None:
+        """One forward pass over a mixed batch: ``entries`` [(tokens, first position, block table, wanted
+        rows)], portions of prompts beside single decoded tokens, the tables already holding a block for
+        every position.  Returns the logits at the wanted rows, in order (None if there are none).  A batch
+        of single later tokens takes the decode step's kernels, any other the packed pass."""
+        rows, base = [], 0
+        for toks, _, _, want in entries:
+            rows += [base + r for r in want]
+            base += len(toks)
+        if all(len(toks) == 1 and first > 0 for toks, first, _, _ in entries):
+            B = len(entries)
+            maxb = 8 * math.ceil(max(len(t) for _, _, t, _ in entries) / 8)
+            bt = np.zeros((B, maxb), np.int32)
+            meta = np.zeros((4, B), np.int32)
+            for b, (toks, first, tbl, _) in enumerate(entries):
+                bt[b, :len(tbl)] = tbl
+                meta[:, b] = (toks[0], first, tbl[first // KV_BLOCK] * KV_BLOCK + first % KV_BLOCK, first + 1)
+            dev = self._h2d(np.concatenate([bt.reshape(-1), meta.reshape(-1)]))
+            d_bt, d_meta = dev[:B * maxb].view(B, maxb), dev[B * maxb:].view(4, B).clone()
+            pb = self._part_blocks(B, maxb)
+            ws = torch.empty(max(1, self.model.decode_workspace(B, -pb)), dtype=torch.float32, device=self.device)
+            hidden = self.model.forward_decode(d_meta[0], d_meta[1], d_meta[2], d_meta[3], d_bt, self.kv,
+                                               attn_workspace=ws, part_blocks=pb)
+            if len(rows) < B:
+                hidden = hidden.index_select(0, torch.tensor(rows, dtype=torch.long, device=self.device)) if rows else None
+        else:
+            kw, _ = self._pass_meta([(toks, first) for toks, first, _, _ in entries], [t for _, _, t, _ in entries],
+                                    rows or [base - 1])
+            hidden = self.model.forward_prefill(**kw, kv=self.kv)
+        self.progress += 1
+        return self.model.logits(hidden) if rows else None
 
     def _h2d(self, a: np.ndarray) -> torch.Tensor:
         t = torch.from_numpy(a)
@@ -296,8 +342,7 @@ class LLMEngine:
         st = self._states.get(key)
         if st is None:
             P = -part_blocks if part_blocks < 0 else math.ceil(max_blocks / part_blocks)
-            ws = B * self.model.w.heads * P * (self.cfg.head_dim + 2) if P > 1 else 1
-            st = _DecodeState(B, max_blocks, max_new, self.device, ws)
+            st = _DecodeState(B, max_blocks, max_new, self.device, self.model.decode_workspace(B, P))
             # persistent: a captured graph holds these pointers
             st.stop_ids = torch.tensor(list(stop_ids), dtype=torch.int32, device=self.device)
             if stop_strings is not None:
@@ -396,7 +441,7 @@ class LLMEngine:
                     fresh.append(new)
                     tables[-1] = shared + new
                     start.append(len(shared) * KV_BLOCK)
-                    if pc is not None:
+                    if pc is not None and not self.share_late:
                         pc.insert(p, tables[-1])
             except BaseException:
                 self._release(tables, fresh, failed=True)
@@ -415,6 +460,7 @@ class LLMEngine:
             with span("llm.prefill"):
                 first = self._prefill(prompts, tables, temperature, seed, start)
             barrier()
+            self._share_computed(prompts, tables)
             t1 = time.perf_counter()
             self._ar_trace(f"after prefill of {B} x {sum(lens)} tokens")
 
@@ -536,6 +582,13 @@ class LLMEngine:
             out, lens = [out[inv[i]] for i in range(B)], [lens[inv[i]] for i in range(B)]
         return GenerationResult(out, lens, prefill_s=job.prefill_s, decode_s=t2 - t1, ttft_s=job.prefill_s,
                                 decode_steps=steps, cached_prompt_tokens=sum(job.start))
+
+    def _share_computed(self, prompts, tables):
+        """After a prefill: publish its full prompt blocks (caches that share only computed blocks)."""
+        if self.prefix_cache is not None and self.share_late:
+            with self._alloc_lock:
+                for p, t in zip(prompts, tables):
+                    self.prefix_cache.insert(p, t)
 
     def _release(self, tables, fresh, failed: bool = False):
         if self.prefix_cache is None:

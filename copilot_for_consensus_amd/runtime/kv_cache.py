@@ -108,5 +108,31 @@ class PagedKVCache:
         return self._k.numel() * self._k.element_size() * 2
 
 
+class LatentKVCache:
+    """Paged cache of a latent-attention decoder, on the same blocks and :class:`BlockPool` as
+    :class:`PagedKVCache`.  Per layer:
+      latents [blocks, 32, rank rounded up to 32]   normed latents, pad columns zero
+      tails   [blocks, slots, width] fp32           last inputs of the layer's causal convolution inside the
+                                                    block, row = position % slots (None without history)
+    A block holds all a sequence continuing after it needs, so prefix sharing works on whole blocks."""
+
+    # another sequence may map a block only after the pass that computes it (its tail is read in the
+    # launch that writes tails)
+    share_after_compute = True
+
+    def __init__(self, ranks: list[int], num_blocks: int, width: int, slots: int, device, dtype=torch.bfloat16):
+        self.layers, self.num_blocks, self.width, self.slots = len(ranks), num_blocks, width, slots
+        self.dtype, self.device = dtype, torch.device(device)
+        # zero-initialised: the slots of a partly filled block are read (then masked)
+        self.latents = [torch.zeros(num_blocks, KV_BLOCK, 32 * math.ceil(r / 32), dtype=dtype, device=self.device)
+                        for r in ranks]
+        self.tails = [torch.zeros(num_blocks, slots, width, dtype=torch.float32, device=self.device) if slots else None
+                      for _ in ranks]
+        self.pool = BlockPool(num_blocks)
+
+    def nbytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in (*self.latents, *self.tails) if t is not None)
+
+
 def blocks_needed(n_tokens: int) -> int:
     return math.ceil(n_tokens / KV_BLOCK)

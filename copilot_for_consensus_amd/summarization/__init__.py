@@ -83,9 +83,10 @@ class HipLLMSummarizer(Summarizer):
                  tp_rank: int = 0, ignore_eos: bool = False, top_k: int = 40, top_p: float = 0.95,
                  min_p: float = 0.05, stop_sequences=("</s>", "\n\n\n"), weight_dtype: str = "bf16",
                  kv_cache_dtype: str = "bf16", **_):
-        from ..models.decoder import DecoderModel, DecoderWeights, get_config, load_config_json
+        from ..models import registry
+        from ..models.decoder import DecoderWeights
         from ..runtime.engine import LLMEngine
-        from ..runtime.kv_cache import PagedKVCache
+        from ..runtime.kv_cache import blocks_needed
         from ..runtime.tokenizer import load_hf_tokenizer, synthetic_bpe
         dev = torch.device(device if (not str(device).startswith("cuda") or torch.cuda.is_available()) else "cpu")
         if gguf_path is None and checkpoint_dir and str(checkpoint_dir).endswith(".gguf"):
@@ -101,14 +102,19 @@ class HipLLMSummarizer(Summarizer):
             self.tokenizer = G.tokenizer_from_gguf(G.GGUFReader(gguf_path).metadata)
         elif checkpoint_dir:
             from pathlib import Path
-            cfg = load_config_json(Path(checkpoint_dir) / "config.json")
-            w = DecoderWeights.from_safetensors(cfg, checkpoint_dir, dev, tp_rank, tensor_parallel)
-            self.tokenizer = load_hf_tokenizer(Path(checkpoint_dir) / "tokenizer.json")
+            cfg = registry.load_config_json(Path(checkpoint_dir) / "config.json")
+            w = registry.load_weights(cfg, checkpoint_dir, dev, tp_rank, tensor_parallel)
+            tok = Path(checkpoint_dir) / "tokenizer.json"
+            # a family without special tokens may ship none (random / research weights)
+            self.tokenizer = load_hf_tokenizer(tok) if tok.exists() or isinstance(w, DecoderWeights) \
+                else synthetic_bpe(cfg.vocab_size)
         else:
-            cfg = get_config(model)
-            w = DecoderWeights.random(cfg, dev, seed=seed, tp_rank=tp_rank, tp_size=tensor_parallel)
+            cfg = registry.get_config(model)
+            w = registry.random_weights(cfg, dev, seed=seed, tp_rank=tp_rank, tp_size=tensor_parallel)
             self.tokenizer = synthetic_bpe(cfg.vocab_size)
         if weight_dtype == "fp8":
+            if not hasattr(w, "to_fp8"):
+                raise ValueError(f"{cfg.name}: no FP8 weights in this model family")
             w.to_fp8()           # opt-in W8A8 FP8 projections (LLM_WEIGHT_DTYPE=fp8)
         self.cfg = cfg
         self.model = cfg.name
@@ -116,9 +122,9 @@ class HipLLMSummarizer(Summarizer):
         if tp_group is not None and tensor_parallel > 1:
             from ..parallel.custom_ar import maybe_create
             custom_ar = maybe_create(tp_group, dev)
-        self.decoder = DecoderModel(w, tp_group=tp_group, custom_ar=custom_ar)
-        kvd = torch.float8_e4m3fn if kv_cache_dtype == "fp8" else torch.bfloat16
-        self.kv = PagedKVCache.for_budget(cfg.layers, w.kv_heads, cfg.head_dim, dev, kv_cache_tokens, dtype=kvd)
+        self.decoder = registry.build_model(w, tp_group=tp_group, custom_ar=custom_ar)
+        self.kv = self.decoder.new_cache(blocks_needed(kv_cache_tokens) + 1,
+                                         dtype=torch.float8_e4m3fn if kv_cache_dtype == "fp8" else None)
         self.engine = LLMEngine(self.decoder, self.kv)
         self.max_new_tokens, self.temperature = int(max_new_tokens), float(temperature)
         # llama.cpp server sampling defaults + the reference's stop sequences (llamacpp_summarizer.py:111-113)

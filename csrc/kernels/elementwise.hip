@@ -260,18 +260,24 @@ __device__ __forceinline__ uint32_t hash_u32(uint32_t x) {
 // lowest index) instead of an index that matched no comparison.
 __device__ __forceinline__ float logit_nan_as_ninf(float x) { return x != x ? -INFINITY : x; }
 
+// logits are bf16 bits (uint16_t) or fp32
+__device__ __forceinline__ float logit_f(uint16_t v) { return bf2f(v); }
+__device__ __forceinline__ float logit_f(float v) { return v; }
+
 // One workgroup per row. temperature <= 0 => greedy argmax (lowest index wins ties);
 // otherwise Gumbel-max sampling: argmax(logit/T + Gumbel(seed, step, row, idx)), which draws
 // exactly from softmax(logit/T).  `step` is read from device memory so graph replays advance it.
-__global__ void __launch_bounds__(1024) sample_kernel(const uint16_t* __restrict__ logits, int V, float temperature,
+template <typename LT>
+__global__ void __launch_bounds__(1024) sample_kernel(const LT* __restrict__ logits, int V, float temperature,
                                                      uint32_t seed, const int32_t* __restrict__ step_ptr,
                                                      int32_t* __restrict__ out_ids) {
   const int row = blockIdx.x;
-  const uint16_t* lr = logits + (size_t)row * V;
+  const LT* lr = logits + (size_t)row * V;
   const uint32_t step = step_ptr ? (uint32_t)*step_ptr : 0u;
   float best = -INFINITY;
   int best_i = 0x7fffffff;
-  const int nvec = (V % 8 == 0) ? V / 8 : 0;  // 16-byte row alignment needed for vector loads
+  constexpr int VE = 16 / sizeof(LT);               // elements of a 16-byte load
+  const int nvec = (V % VE == 0) ? V / VE : 0;  // 16-byte row alignment needed for vector loads
   const bool sample = temperature > 0.f;
   const float inv_t = sample ? 1.f / temperature : 1.f;
   auto score = [&](float x, int idx) -> float {
@@ -294,18 +300,23 @@ __global__ void __launch_bounds__(1024) sample_kernel(const uint16_t* __restrict
     for (int u = 0; u < 4; ++u) {
       const int c = c0 + u * blockDim.x;
       if (c >= nvec) break;
-      float v[8];
-      unpack8(raw[u], v);
+      float v[VE];
+      if constexpr (VE == 8) {
+        unpack8(raw[u], v);
+      } else {
+        v[0] = __uint_as_float(raw[u].x); v[1] = __uint_as_float(raw[u].y);
+        v[2] = __uint_as_float(raw[u].z); v[3] = __uint_as_float(raw[u].w);
+      }
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int idx = c * 8 + j;
+      for (int j = 0; j < VE; ++j) {
+        const int idx = c * VE + j;
         const float x = score(v[j], idx);
         if (x > best || (x == best && idx < best_i)) { best = x; best_i = idx; }
       }
     }
   }
-  for (int idx = nvec * 8 + threadIdx.x; idx < V; idx += blockDim.x) {  // tail (V % 8)
-    const float x = score(bf2f(lr[idx]), idx);
+  for (int idx = nvec * VE + threadIdx.x; idx < V; idx += blockDim.x) {  // tail
+    const float x = score(logit_f(lr[idx]), idx);
     if (x > best || (x == best && idx < best_i)) { best = x; best_i = idx; }
   }
   __shared__ float sb[16];
@@ -343,12 +354,13 @@ __device__ __forceinline__ uint32_t order_key(float f) {
   return (u & 0x80000000u) ? ~u : (u | 0x80000000u);
 }
 
-__global__ void __launch_bounds__(256) sample_topk_kernel(const uint16_t* __restrict__ logits, int V, float temperature,
+template <typename LT>
+__global__ void __launch_bounds__(256) sample_topk_kernel(const LT* __restrict__ logits, int V, float temperature,
                                                           int top_k, float top_p, float min_p, uint32_t seed,
                                                           const int32_t* __restrict__ step_ptr,
                                                           int32_t* __restrict__ out_ids) {
   const int row = blockIdx.x, tid = threadIdx.x;
-  const uint16_t* lr = logits + (size_t)row * V;
+  const LT* lr = logits + (size_t)row * V;
   const uint32_t step = step_ptr ? (uint32_t)*step_ptr : 0u;
   const int K = max(1, min(top_k > 0 ? top_k : SK_CAP, min(V, SK_CAP)));
   __shared__ uint32_t hist[256];
@@ -368,7 +380,7 @@ __global__ void __launch_bounds__(256) sample_topk_kernel(const uint16_t* __rest
     hist[tid] = 0;
     __syncthreads();
     for (int i = tid; i < V; i += 256) {
-      const uint32_t k = order_key(logit_nan_as_ninf(bf2f(lr[i])));
+      const uint32_t k = order_key(logit_nan_as_ninf(logit_f(lr[i])));
       if ((k & mask) == prefix) atomicAdd(&hist[(k >> shift) & 0xFF], 1u);
     }
     __syncthreads();
@@ -393,7 +405,7 @@ __global__ void __launch_bounds__(256) sample_topk_kernel(const uint16_t* __rest
   if (tid == 0) s_n = 0;
   __syncthreads();
   for (int i = tid; i < V; i += 256) {
-    const float f = logit_nan_as_ninf(bf2f(lr[i]));
+    const float f = logit_nan_as_ninf(logit_f(lr[i]));
     if (order_key(f) > prefix) {
       const int slot = atomicAdd(&s_n, 1);
       cv[slot] = f;
@@ -406,7 +418,7 @@ __global__ void __launch_bounds__(256) sample_topk_kernel(const uint16_t* __rest
     int found = 0;
     for (int base = lo; base < hi && found < (int)remaining; base += 64) {
       const int i = base + lane;
-      const bool tie = i < hi && order_key(logit_nan_as_ninf(bf2f(lr[i]))) == prefix;
+      const bool tie = i < hi && order_key(logit_nan_as_ninf(logit_f(lr[i]))) == prefix;
       const unsigned long long m = __ballot(tie);
       if (tie) {
         const int pos = found + __popcll(m & ((1ull << lane) - 1ull));
@@ -420,7 +432,7 @@ __global__ void __launch_bounds__(256) sample_topk_kernel(const uint16_t* __rest
   if (tid == 0) {
     int n0 = s_n;
     for (int w = 0; w < 4 && n0 < K; ++w)
-      for (int j = 0; j < tie_n[w] && n0 < K; ++j) { ci[n0] = tie_i[w][j]; cv[n0] = logit_nan_as_ninf(bf2f(lr[tie_i[w][j]])); ++n0; }
+      for (int j = 0; j < tie_n[w] && n0 < K; ++j) { ci[n0] = tie_i[w][j]; cv[n0] = logit_nan_as_ninf(logit_f(lr[tie_i[w][j]])); ++n0; }
     s_n = n0;
   }
   __syncthreads();
@@ -718,20 +730,26 @@ CFC_API int cfc_embedding(void* out, const void* table, const int32_t* ids, int 
 }
 
 // top_k <= 0: no top-k cut (candidates still capped at SK_CAP = 256); top_p >= 1 / min_p <= 0 disable those.
-CFC_API int cfc_sample_truncated(const void* logits, int B, int V, float temperature, int top_k, float top_p,
+// f32: the logits are fp32 (else bf16)
+CFC_API int cfc_sample_truncated(const void* logits, int f32, int B, int V, float temperature, int top_k, float top_p,
                                  float min_p, uint32_t seed, const int32_t* step_ptr, int32_t* out_ids,
                                  hipStream_t stream) {
   if (B == 0) return 0;
   if (V <= 0 || top_p <= 0.f) return -1;
-  sample_topk_kernel<<<B, 256, 0, stream>>>((const uint16_t*)logits, V, temperature, top_k, top_p, min_p, seed,
-                                            step_ptr, out_ids);
+  if (f32)
+    sample_topk_kernel<float><<<B, 256, 0, stream>>>((const float*)logits, V, temperature, top_k, top_p, min_p, seed,
+                                                     step_ptr, out_ids);
+  else
+    sample_topk_kernel<uint16_t><<<B, 256, 0, stream>>>((const uint16_t*)logits, V, temperature, top_k, top_p, min_p, seed,
+                                                        step_ptr, out_ids);
   return CFC_CHECK_LAUNCH();
 }
 
-CFC_API int cfc_sample(const void* logits, int B, int V, float temperature, uint32_t seed, const int32_t* step_ptr,
-                       int32_t* out_ids, hipStream_t stream) {
+CFC_API int cfc_sample(const void* logits, int f32, int B, int V, float temperature, uint32_t seed,
+                       const int32_t* step_ptr, int32_t* out_ids, hipStream_t stream) {
   if (B == 0) return 0;
-  sample_kernel<<<B, 1024, 0, stream>>>((const uint16_t*)logits, V, temperature, seed, step_ptr, out_ids);
+  if (f32) sample_kernel<float><<<B, 1024, 0, stream>>>((const float*)logits, V, temperature, seed, step_ptr, out_ids);
+  else sample_kernel<uint16_t><<<B, 1024, 0, stream>>>((const uint16_t*)logits, V, temperature, seed, step_ptr, out_ids);
   return CFC_CHECK_LAUNCH();
 }
 

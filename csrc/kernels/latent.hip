@@ -1,0 +1,581 @@
+// Latent attention for gfx950: every head's keys and values are products of ONE cached latent row per
+// token, so the paged cache holds [blocks][32][RS] latents (RS = rank rounded up to 32, zero-filled)
+// and attention runs in the latent space: with q' = W_uk^T q per head, score = q' . c and the head's
+// output is W_uv (sum p c).  All heads of a token then read the same rows (a multi-query attention
+// whose key and value are the same bytes, loaded once).
+//
+//   * latent_norm     RMS norms of the query latent and the cached latent from the fp32 slabs of the
+//                     joint down projection; the latter goes straight into the cache slot
+//   * head_linear     out[t][h] = W[h] in[t][h], the per-head products on both sides of the attention
+//   * latent_attn     flash-style attention over the paged latents.  A work item is 16 MR rows of the
+//                     flattened (token, head) rows of one sequence -- one decoded token's heads and a
+//                     prompt portion's rows are the same thing to it -- and a slice of its keys
+//   * latent_combine  merges the slices
+//   * latent_expand   a sequence's latents as per-head K / V blocks in the layout of the paged prefill
+//                     attention (attention.hip), for long portions where that costs fewer flops
+#include "common.h"
+
+namespace {
+
+typedef short i16x4_t __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) i16x4_t lds_i16x4_t;
+
+__device__ __forceinline__ float ldf(const uint16_t* p) { return bf2f(*p); }
+__device__ __forceinline__ float ldf(const float* p) { return *p; }
+__device__ __forceinline__ void stf(uint16_t* p, float v) { *p = f2bf(v); }
+__device__ __forceinline__ void stf(float* p, float v) { *p = v; }
+
+// ---------------------------------------------------------------------------------- latent_norm
+// part: fp32 slabs [split][T][NQ + NC] of the joint projection (query latent | cached latent).
+// One workgroup per row; the row's sums are kept in LDS.
+template <typename ACT>
+__global__ void __launch_bounds__(256) latent_norm_kernel(const float* __restrict__ part, int split, int T, int NQ, int NC,
+                                                         const float* __restrict__ wq, const float* __restrict__ wc,
+                                                         float eps, const int32_t* __restrict__ slots,
+                                                         ACT* __restrict__ q_out, int ldq, ACT* __restrict__ cache,
+                                                         int RS) {
+  extern __shared__ float row[];
+  __shared__ float red[16];
+  const int t = blockIdx.x, N = NQ + NC;
+  float sq = 0.f, sc = 0.f;
+  for (int c = threadIdx.x; c < N; c += 256) {
+    float v = 0.f;
+    for (int p = 0; p < split; ++p) v += part[((size_t)p * T + t) * N + c];
+    row[c] = v;
+    if (c < NQ) sq += v * v;
+    else sc += v * v;
+  }
+  sq = block_sum(sq, red);
+  sc = block_sum(sc, red);
+  const float rq = 1.f / sqrtf(sq / (float)NQ + eps), rc = 1.f / sqrtf(sc / (float)NC + eps);
+  ACT* dst = cache + (size_t)slots[t] * RS;
+  for (int c = threadIdx.x; c < N; c += 256) {      // each thread reads back only what it wrote
+    if (c < NQ) stf(q_out + (size_t)t * ldq + c, row[c] * rq * wq[c]);
+    else stf(dst + (c - NQ), row[c] * rc * wc[c - NQ]);
+  }
+}
+
+// ---------------------------------------------------------------------------------- head_linear
+// W [H][NP][KP] zero-padded (NP % 64 == 0, KP % 32 == 0).  Operands: A = W rows, B = token rows, so a
+// lane ends with four consecutive outputs of one token.  grid (token tiles, NP / (16 NT 4), H), four
+// waves side by side over the outputs, each with TT x NT 16 x 16 tiles.
+__device__ __forceinline__ f32x4_t mfma16(uint4 a, uint4 b, f32x4_t c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0,
+                                                 0, 0);
+}
+
+template <bool VEC>
+__device__ __forceinline__ uint4 ld_frag(const uint16_t* p, int k, int K) {
+  if constexpr (VEC) {
+    return k < K ? *reinterpret_cast<const uint4*>(p + k) : make_uint4(0, 0, 0, 0);
+  } else {
+    uint32_t w[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const uint32_t lo = k + 2 * i < K ? p[k + 2 * i] : 0, hi = k + 2 * i + 1 < K ? p[k + 2 * i + 1] : 0;
+      w[i] = lo | (hi << 16);
+    }
+    return make_uint4(w[0], w[1], w[2], w[3]);
+  }
+}
+
+template <int TT, int NT, bool VEC>
+__global__ void __launch_bounds__(256) head_linear_kernel(const uint16_t* __restrict__ x, int64_t ldx, int64_t hsx,
+                                                         const uint16_t* __restrict__ w, int NP, int KP, int T, int N,
+                                                         int K, uint16_t* __restrict__ out, int64_t ldo, int64_t hso) {
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
+  const int h = blockIdx.z, t0 = blockIdx.x * 16 * TT, n0 = (blockIdx.y * 4 + wv) * 16 * NT;
+  if (n0 >= NP) return;
+  const uint16_t* wp = w + ((size_t)h * NP + n0 + col) * KP + 8 * kq;
+  const uint16_t* xp[TT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) xp[i] = x + (int64_t)min(t0 + 16 * i + col, T - 1) * ldx + h * hsx;
+  f32x4_t acc[NT][TT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j)
+#pragma unroll
+    for (int i = 0; i < TT; ++i) acc[j][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < KP; k += 32) {
+    uint4 a[NT], b[TT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) a[j] = *reinterpret_cast<const uint4*>(wp + (size_t)16 * j * KP + k);
+#pragma unroll
+    for (int i = 0; i < TT; ++i) b[i] = ld_frag<VEC>(xp[i], k + 8 * kq, K);
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+      for (int i = 0; i < TT; ++i) acc[j][i] = mfma16(a[j], b[i], acc[j][i]);
+  }
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    const int t = t0 + 16 * i + col;
+    if (t >= T) continue;
+    uint16_t* o = out + (int64_t)t * ldo + h * hso;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      const int n = n0 + 16 * j + 4 * kq;
+      if constexpr (VEC) {
+        if (n < N)
+          *reinterpret_cast<uint2*>(o + n) =
+              make_uint2(pack2bf(acc[j][i][0], acc[j][i][1]), pack2bf(acc[j][i][2], acc[j][i][3]));
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float v = acc[j][i][e];
+          if (n + e < N) o[n + e] = f2bf(v);
+        }
+      }
+    }
+  }
+}
+
+__global__ void __launch_bounds__(256) head_linear_f32_kernel(const float* __restrict__ x, int64_t ldx, int64_t hsx,
+                                                             const float* __restrict__ w, int NP, int KP, int N, int K,
+                                                             float* __restrict__ out, int64_t ldo, int64_t hso) {
+  const int n = blockIdx.y * 256 + threadIdx.x, t = blockIdx.x, h = blockIdx.z;
+  if (n >= N) return;
+  const float* xr = x + t * ldx + h * hsx;
+  const float* wr = w + ((size_t)h * NP + n) * KP;
+  float s = 0.f;
+  for (int k = 0; k < K; ++k) s += xr[k] * wr[k];
+  out[t * ldo + h * hso + n] = s;
+}
+
+// ---------------------------------------------------------------------------------- latent_attn
+struct LatArgs {
+  const int32_t* block_tables;
+  const int32_t* cu_q;        // null: one token per sequence
+  const int32_t* ctx_lens;    // cached + new tokens
+  const int32_t* tile_seq;    // null: tile b is rows 16 MR (b % tiles_per_seq) of sequence b / tiles_per_seq
+  const int32_t* tile_m0;
+  int tiles_per_seq, H, RS, max_blocks, P;
+  float scale;
+  float* part_o;              // [rows][P][RS], unnormalised
+  float* part_ml;             // [rows][P][2]: running maximum (log2 domain), sum
+};
+
+struct LatTile { int m0, rows, q_row, pos_base, kt0, kt1, kend; const int32_t* bt; };
+
+// the tile's rows and its slice of 64-key tiles
+__device__ __forceinline__ LatTile lat_tile(const LatArgs& a, int tile, int p, int rows_per_tile) {
+  LatTile r;
+  const int s = a.tile_seq ? a.tile_seq[tile] : tile / a.tiles_per_seq;
+  r.m0 = a.tile_m0 ? a.tile_m0[tile] : (tile % a.tiles_per_seq) * rows_per_tile;
+  const int q0 = a.cu_q ? a.cu_q[s] : s, n = a.cu_q ? a.cu_q[s + 1] - q0 : 1;
+  r.rows = n * a.H;
+  r.q_row = q0 * a.H;
+  r.pos_base = a.ctx_lens[s] - n;
+  r.kend = r.pos_base + (min(r.m0 + rows_per_tile, r.rows) - 1) / a.H + 1;
+  const int nt = (r.kend + 63) / 64;
+  r.kt0 = (int)((int64_t)nt * p / a.P);
+  r.kt1 = (int)((int64_t)nt * (p + 1) / a.P);
+  r.bt = a.block_tables + (size_t)s * a.max_blocks;
+  return r;
+}
+
+constexpr int LP = 72;      // P row stride in LDS, elements (64 keys + 8 against bank conflicts)
+
+// Eight waves, a 64-key x R64 tile of latents double-buffered in LDS (row-major, 16-byte chunks
+// XOR-swizzled by the key).
+//   scores   S^T = C q'^T: wave (row group rg, key group) multiplies 16-key A fragments from LDS with
+//            its 16 rows' q' held in registers; a lane owns one row's scores for 4 (or 8) keys
+//   softmax  per row across the lane groups by lane swaps, across the waves of a row group through LDS
+//   output   O^T += C^T P^T: wave w owns latent columns 16 (w + 8 j) of every row; the C^T fragments
+//            are transposing LDS reads (ds_read_b64_tr_b16) of the same tile, P^T comes from LDS
+// Two barriers per tile; the next tile's global loads are issued first and stored to the other buffer
+// between them, when no wave can still be reading it.
+template <int R64, int MR>
+__global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __restrict__ q,
+                                                            const uint16_t* __restrict__ cache, LatArgs a,
+                                                            uint16_t* __restrict__ out) {
+  constexpr int CH = R64 / 8;                     // 16-byte chunks per key
+  constexpr int XM = R64 % 128 == 0 ? 15 : 7;
+  constexpr int KS = R64 / 32;                    // MFMA steps over the rank
+  constexpr int NL = CH / 8;                      // chunks per thread of a 64-key tile
+  constexpr int KG = MR == 4 ? 2 : 1;             // 16-key groups per wave
+  constexpr int SL = 4 / KG;                      // waves per row group
+  constexpr int RT = R64 / 16;                    // 16-column output tiles
+  constexpr int NO = (RT + 7) / 8;                // per wave
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  char* kbuf = smem;                                            // [2][64][R64] bf16
+  uint16_t* sp = reinterpret_cast<uint16_t*>(smem + 2 * 64 * R64 * 2);   // [16 MR][LP]
+  float* smax = reinterpret_cast<float*>(sp + 16 * MR * LP);    // [MR][4][16]
+  float* salpha = smax + MR * 64;                               // [16 MR]
+
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int col = lane & 15, kq = lane >> 4;
+  const LatTile tl = lat_tile(a, blockIdx.x, blockIdx.y, 16 * MR);
+  const int RS = a.RS;
+
+  // score role: row group and key groups of this wave (MR = 1: waves 4-7 have none)
+  const int rg = MR == 1 ? 0 : w % MR, slot = MR == 1 ? w : w / MR;
+  const bool scorer = slot < SL;
+  const int gm = min(tl.m0 + 16 * rg + col, tl.rows - 1);
+  const int limit = tl.pos_base + gm / a.H + 1;   // keys this row sees
+  uint4 qf[KS];
+  if (scorer) {
+    const uint16_t* qr = q + (size_t)(tl.q_row + gm) * RS + 8 * kq;
+#pragma unroll
+    for (int k = 0; k < KS; ++k)
+      qf[k] = 32 * k < RS ? *reinterpret_cast<const uint4*>(qr + 32 * k) : make_uint4(0, 0, 0, 0);
+  }
+
+  const int nb = (tl.kend + CFC_KV_BS - 1) / CFC_KV_BS;
+  uint4 st[NL];
+  auto gload = [&](int kt) {
+    const int b0 = tl.bt[min(2 * kt, nb - 1)], b1 = tl.bt[min(2 * kt + 1, nb - 1)];
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = tid + 512 * i, key = e / CH, c = e % CH;
+      st[i] = 8 * c < RS ? *reinterpret_cast<const uint4*>(cache + ((size_t)(key < 32 ? b0 : b1) * 32 + (key & 31)) * RS + 8 * c)
+                         : make_uint4(0, 0, 0, 0);
+    }
+  };
+  auto lwrite = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = tid + 512 * i, key = e / CH, c = e % CH;
+      *reinterpret_cast<uint4*>(kbuf + buf * (64 * R64 * 2) + key * (R64 * 2) + ((c ^ (key & XM)) << 4)) = st[i];
+    }
+  };
+
+  f32x4_t o[NO][MR];
+#pragma unroll
+  for (int j = 0; j < NO; ++j)
+#pragma unroll
+    for (int r = 0; r < MR; ++r) o[j][r] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+
+  if (tl.kt0 < tl.kt1) {
+    gload(tl.kt0);
+    lwrite(0);
+  }
+  __syncthreads();
+  for (int kt = tl.kt0; kt < tl.kt1; ++kt) {
+    const int cur = (kt - tl.kt0) & 1;
+    const char* kb = kbuf + cur * (64 * R64 * 2);
+    const bool more = kt + 1 < tl.kt1;
+    if (more) gload(kt + 1);
+    f32x4_t s[KG];
+    if (scorer) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int g = 0; g < KG; ++g) {
+        const int key = 16 * (slot * KG + g) + col;
+        const char* kr = kb + key * (R64 * 2);
+        f32x4_t s0{0.f, 0.f, 0.f, 0.f}, s1{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < KS; k += 2) {
+          s0 = mfma16(*reinterpret_cast<const uint4*>(kr + (((4 * k + kq) ^ (key & XM)) << 4)), qf[k], s0);
+          if (k + 1 < KS)
+            s1 = mfma16(*reinterpret_cast<const uint4*>(kr + (((4 * k + 4 + kq) ^ (key & XM)) << 4)), qf[k + 1], s1);
+        }
+        const int k0 = kt * 64 + 16 * (slot * KG + g) + 4 * kq;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          s[g][i] = k0 + i < limit ? (s0[i] + s1[i]) * a.scale : -INFINITY;
+          mx = fmaxf(mx, s[g][i]);
+        }
+      }
+      mx = xor32_max(xor16_max(mx));
+      if (lane < 16) smax[(rg * 4 + slot) * 16 + lane] = mx;
+    }
+    __syncthreads();
+    if (scorer) {
+      float mn = m;
+#pragma unroll
+      for (int u = 0; u < SL; ++u) mn = fmaxf(mn, smax[(rg * 4 + u) * 16 + col]);
+      const float ref = mn == -INFINITY ? 0.f : mn;
+      const float alpha = __builtin_amdgcn_exp2f(m - ref);      // m = -inf: 0
+      m = mn;
+      l *= alpha;
+#pragma unroll
+      for (int g = 0; g < KG; ++g) {
+        float e[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          e[i] = __builtin_amdgcn_exp2f(s[g][i] - ref);
+          l += e[i];
+        }
+        *reinterpret_cast<uint2*>(sp + (16 * rg + col) * LP + 16 * (slot * KG + g) + 4 * kq) =
+            make_uint2(cvt_pk_bf16_f32(e[0], e[1]), cvt_pk_bf16_f32(e[2], e[3]));
+      }
+      if (slot == 0 && lane < 16) salpha[16 * rg + lane] = alpha;
+    }
+    if (more) lwrite(cur ^ 1);
+    __syncthreads();
+    uint4 pf[2][MR];
+#pragma unroll
+    for (int r = 0; r < MR; ++r) {
+      const float al = salpha[16 * r + col];
+      if (!__all(al == 1.f)) {
+#pragma unroll
+        for (int j = 0; j < NO; ++j) o[j][r] *= al;
+      }
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk)
+        pf[kk][r] = *reinterpret_cast<const uint4*>(sp + (16 * r + col) * LP + 32 * kk + 8 * kq);
+    }
+#pragma unroll
+    for (int j = 0; j < NO; ++j) {
+      const int rt = w + 8 * j;
+      if (rt < RT) {
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+          // lane i of a 16-lane group addresses 4 latent columns of key 8 kq + i / 4 and receives one
+          // column's 4 keys
+          uint32_t f[4];
+#pragma unroll
+          for (int u = 0; u < 2; ++u) {
+            const int key = 32 * kk + 8 * kq + 4 * u + (col >> 2), c = 2 * rt + ((col & 3) >> 1);
+            const char* p = kb + key * (R64 * 2) + ((c ^ (key & XM)) << 4) + 8 * (col & 1);
+            const i16x4_t v = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                (lds_i16x4_t*)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) const char*)p);
+            const uint2 vv = __builtin_bit_cast(uint2, v);
+            f[2 * u] = vv.x;
+            f[2 * u + 1] = vv.y;
+          }
+          const uint4 cf = make_uint4(f[0], f[1], f[2], f[3]);
+#pragma unroll
+          for (int r = 0; r < MR; ++r) o[j][r] = mfma16(cf, pf[kk][r], o[j][r]);
+        }
+      }
+    }
+  }
+  // row sums over the lane groups and the row group's waves
+  __syncthreads();
+  if (scorer) {
+    l = xor32_sum(xor16_sum(l));
+    if (lane < 16) {
+      smax[(rg * 4 + slot) * 16 + lane] = l;
+      if (slot == 0) salpha[16 * rg + lane] = m;
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int r = 0; r < MR; ++r) {
+    const int mrow = tl.m0 + 16 * r + col;
+    if (mrow >= tl.rows) continue;
+    float lt = 0.f;
+#pragma unroll
+    for (int u = 0; u < SL; ++u) lt += smax[(r * 4 + u) * 16 + col];
+    const size_t grow = (size_t)tl.q_row + mrow;
+    if (a.P > 1) {
+      float* po = a.part_o + (grow * a.P + blockIdx.y) * RS;
+#pragma unroll
+      for (int j = 0; j < NO; ++j) {
+        const int n = 16 * (w + 8 * j) + 4 * kq;
+        if (w + 8 * j < RT && n < RS) *reinterpret_cast<float4*>(po + n) = make_float4(o[j][r][0], o[j][r][1], o[j][r][2], o[j][r][3]);
+      }
+      if (w == 0 && kq == 0) {
+        float* ml = a.part_ml + (grow * a.P + blockIdx.y) * 2;
+        ml[0] = salpha[16 * r + col];
+        ml[1] = lt;
+      }
+    } else {
+      const float inv = lt > 0.f ? 1.f / lt : 0.f;
+      uint16_t* po = out + grow * RS;
+#pragma unroll
+      for (int j = 0; j < NO; ++j) {
+        const int n = 16 * (w + 8 * j) + 4 * kq;
+        if (w + 8 * j < RT && n < RS)
+          *reinterpret_cast<uint2*>(po + n) = make_uint2(cvt_pk_bf16_f32(o[j][r][0] * inv, o[j][r][1] * inv),
+                                                         cvt_pk_bf16_f32(o[j][r][2] * inv, o[j][r][3] * inv));
+      }
+    }
+  }
+}
+
+// Any rank up to 1024 and both activation types, one wave per (token, head) row and key slice: a lane
+// scores one key of 64, then owns every 64th latent column of the output.  The 32-bit path.
+constexpr int LG_C = 16;    // columns per lane
+template <typename ACT>
+__global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restrict__ q, const ACT* __restrict__ cache,
+                                                             LatArgs a, ACT* __restrict__ out) {
+  extern __shared__ float sq[];                 // [4][RS] q' rows, then [4][64] weights
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, RS = a.RS;
+  const LatTile tl = lat_tile(a, blockIdx.x, blockIdx.y, 4);
+  float* myq = sq + w * RS;
+  float* pw = sq + 4 * RS + 64 * w;
+  const int mrow = tl.m0 + w;
+  const bool live = mrow < tl.rows;             // the other waves of the tile go on: barriers below are the tile's
+  const size_t grow = (size_t)tl.q_row + (live ? mrow : tl.rows - 1);
+  for (int c = lane; c < RS; c += 64) myq[c] = ldf(q + grow * RS + c);
+  __syncthreads();
+  const int limit = tl.pos_base + (live ? mrow : tl.rows - 1) / a.H + 1;
+  float o[LG_C];
+#pragma unroll
+  for (int j = 0; j < LG_C; ++j) o[j] = 0.f;
+  float m = -INFINITY, l = 0.f;
+  for (int kt = tl.kt0; kt < tl.kt1; ++kt) {
+    const int key = kt * 64 + lane;
+    float s = -INFINITY;
+    if (key < limit) {
+      const ACT* c = cache + ((size_t)tl.bt[key / CFC_KV_BS] * CFC_KV_BS + key % CFC_KV_BS) * RS;
+      float s4[4] = {0.f, 0.f, 0.f, 0.f};
+      for (int r = 0; r < RS; r += 4)
+#pragma unroll
+        for (int u = 0; u < 4; ++u) s4[u] += myq[r + u] * ldf(c + r + u);
+      s = ((s4[0] + s4[1]) + (s4[2] + s4[3])) * a.scale;
+    }
+    const float mn = fmaxf(m, wave_max(s));
+    const float ref = mn == -INFINITY ? 0.f : mn;
+    const float alpha = exp2f(m - ref), p = exp2f(s - ref);
+    m = mn;
+    l = l * alpha + wave_sum(p);
+    pw[lane] = p;
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < LG_C; ++j) o[j] *= alpha;
+    const int nk = min(64, limit - kt * 64);
+    for (int k = 0; k < nk; ++k) {
+      const int kk = kt * 64 + k;
+      const ACT* c = cache + ((size_t)tl.bt[kk / CFC_KV_BS] * CFC_KV_BS + kk % CFC_KV_BS) * RS;
+      const float pk = pw[k];
+#pragma unroll
+      for (int j = 0; j < LG_C; ++j)
+        if (lane + 64 * j < RS) o[j] += pk * ldf(c + lane + 64 * j);
+    }
+    __syncthreads();
+  }
+  if (!live) return;
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+  for (int j = 0; j < LG_C; ++j) {
+    const int c = lane + 64 * j;
+    if (c >= RS) continue;
+    if (a.P > 1) a.part_o[(grow * a.P + blockIdx.y) * RS + c] = o[j];
+    else stf(out + grow * RS + c, o[j] * inv);
+  }
+  if (a.P > 1 && lane == 0) {
+    a.part_ml[(grow * a.P + blockIdx.y) * 2] = m;
+    a.part_ml[(grow * a.P + blockIdx.y) * 2 + 1] = l;
+  }
+}
+
+// one workgroup of 128 threads per (token, head) row
+template <typename ACT>
+__global__ void __launch_bounds__(128) latent_combine_kernel(const float* __restrict__ part_o,
+                                                            const float* __restrict__ part_ml, int P, int RS,
+                                                            ACT* __restrict__ out) {
+  const size_t row = blockIdx.x;
+  const float* ml = part_ml + row * P * 2;
+  float m = -INFINITY;
+  for (int p = 0; p < P; ++p) m = fmaxf(m, ml[2 * p]);
+  const float ref = m == -INFINITY ? 0.f : m;
+  float l = 0.f;
+  for (int p = 0; p < P; ++p) l += ml[2 * p + 1] * exp2f(ml[2 * p] - ref);
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  for (int c = threadIdx.x * 4; c < RS; c += 512) {
+    float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+    for (int p = 0; p < P; ++p) {
+      const float e = exp2f(ml[2 * p] - ref) * inv;
+      const float4 v = *reinterpret_cast<const float4*>(part_o + (row * P + p) * RS + c);
+      s.x += e * v.x; s.y += e * v.y; s.z += e * v.z; s.w += e * v.w;
+    }
+    ACT* o = out + row * RS + c;
+    stf(o, s.x); stf(o + 1, s.y); stf(o + 2, s.z); stf(o + 3, s.w);
+  }
+}
+
+template <int R64, int MR>
+int lat_go(dim3 grid, hipStream_t s, const void* q, const void* cache, const LatArgs& a, void* out) {
+  constexpr int lds = 2 * 64 * R64 * 2 + 16 * MR * LP * 2 + (MR * 64 + 16 * MR) * 4;
+  static bool raised = false;
+  if (lds > 65536 && !raised) {
+    hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<R64, MR>),
+                        hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    raised = true;
+  }
+  latent_attn_kernel<R64, MR><<<grid, 512, lds, s>>>((const uint16_t*)q, (const uint16_t*)cache, a, (uint16_t*)out);
+  return CFC_CHECK_LAUNCH();
+}
+
+template <int R64>
+int lat_mr(int mr, dim3 grid, hipStream_t s, const void* q, const void* cache, const LatArgs& a, void* out) {
+  switch (mr) {
+    case 1: return lat_go<R64, 1>(grid, s, q, cache, a, out);
+    case 2: return lat_go<R64, 2>(grid, s, q, cache, a, out);
+    case 4: return lat_go<R64, 4>(grid, s, q, cache, a, out);
+  }
+  return -3;
+}
+
+}  // namespace
+
+CFC_API int cfc_latent_norm(int f32, const float* part, int split, int T, int NQ, int NC, const float* wq, const float* wc,
+                            float eps, const int32_t* slots, void* q_out, int ldq, void* cache, int RS,
+                            hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (split < 1 || NQ < 1 || NC < 1 || NC > RS || ldq < NQ || (NQ + NC) * 4 > 60000) return -1;
+  const size_t lds = (size_t)(NQ + NC) * 4;
+  if (f32)
+    latent_norm_kernel<float><<<T, 256, lds, stream>>>(part, split, T, NQ, NC, wq, wc, eps, slots, (float*)q_out, ldq,
+                                                       (float*)cache, RS);
+  else
+    latent_norm_kernel<uint16_t><<<T, 256, lds, stream>>>(part, split, T, NQ, NC, wq, wc, eps, slots, (uint16_t*)q_out,
+                                                          ldq, (uint16_t*)cache, RS);
+  return CFC_CHECK_LAUNCH();
+}
+
+// x row (t, h) at t ldx + h hsx (K values), out at t ldo + h hso (N values); W [H][NP][KP] zero-padded
+CFC_API int cfc_head_linear(int f32, const void* x, int64_t ldx, int64_t hsx, const void* w, int NP, int KP, int T, int H,
+                            int N, int K, void* out, int64_t ldo, int64_t hso, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (H < 1 || H > 65535 || N < 1 || K < 1 || N > NP || K > KP || NP % 64 || KP % 32) return -1;
+  if (f32) {
+    const dim3 grid(T, (N + 255) / 256, H);
+    head_linear_f32_kernel<<<grid, 256, 0, stream>>>((const float*)x, ldx, hsx, (const float*)w, NP, KP, N, K, (float*)out,
+                                                     ldo, hso);
+    return CFC_CHECK_LAUNCH();
+  }
+  const bool vec = K % 8 == 0 && ldx % 8 == 0 && hsx % 8 == 0 && ((uintptr_t)x & 15) == 0 && N % 4 == 0 && ldo % 4 == 0 &&
+                   hso % 4 == 0 && ((uintptr_t)out & 7) == 0;
+#define HL(TT, NT, V)                                                                                                 \
+  head_linear_kernel<TT, NT, V><<<dim3((T + 16 * TT - 1) / (16 * TT), (NP + 64 * NT - 1) / (64 * NT), H), 256, 0, stream>>>( \
+      (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso)
+  if (!vec) HL(4, 1, false);
+  else if (T <= 16) HL(1, 1, true);
+  else if (T <= 256) HL(4, 1, true);
+  else HL(4, 2, true);
+#undef HL
+  return CFC_CHECK_LAUNCH();
+}
+
+// rows_per_tile: 16 / 32 / 64 on the MFMA kernel (bf16, rank <= 512), 4 on the general one
+CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, const int32_t* block_tables,
+                                 const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tile_seq,
+                                 const int32_t* tile_m0, int n_tiles, int tiles_per_seq, int rows_per_tile, int H, int RS,
+                                 int max_blocks, float scale, int P, int total_rows, float* part_o, float* part_ml,
+                                 void* out, hipStream_t stream) {
+  if (n_tiles <= 0) return 0;
+  if (H < 1 || RS < 32 || RS % 32 || P < 1 || P > 65535 || max_blocks < 1) return -1;
+  if ((tile_seq == nullptr) != (tile_m0 == nullptr) || (!tile_seq && tiles_per_seq < 1)) return -1;
+  if (P > 1 && (!part_o || !part_ml)) return -2;
+  LatArgs a{block_tables, cu_q, ctx_lens, tile_seq, tile_m0, tiles_per_seq, H, RS, max_blocks, P,
+            scale * 1.4426950408889634f, part_o, part_ml};
+  const dim3 grid(n_tiles, P);
+  int rc = -3;
+  if (rows_per_tile == 4) {
+    if (RS > 64 * LG_C) return -4;
+    const size_t lds = (size_t)(4 * RS + 256) * 4;
+    if (f32) latent_attn_any_kernel<float><<<grid, 256, lds, stream>>>((const float*)q, (const float*)cache, a, (float*)out);
+    else latent_attn_any_kernel<uint16_t><<<grid, 256, lds, stream>>>((const uint16_t*)q, (const uint16_t*)cache, a, (uint16_t*)out);
+    rc = CFC_CHECK_LAUNCH();
+  } else {
+    if (f32 || RS > 512) return -4;
+    const int mr = rows_per_tile / 16;
+    switch ((RS + 63) / 64) {
+      case 1: rc = lat_mr<64>(mr, grid, stream, q, cache, a, out); break;
+      case 2: rc = lat_mr<128>(mr, grid, stream, q, cache, a, out); break;
+      case 3: rc = lat_mr<192>(mr, grid, stream, q, cache, a, out); break;
+      case 4: rc = lat_mr<256>(mr, grid, stream, q, cache, a, out); break;
+      case 5: case 6: rc = lat_mr<384>(mr, grid, stream, q, cache, a, out); break;
+      default: rc = lat_mr<512>(mr, grid, stream, q, cache, a, out); break;
+    }
+  }
+  if (rc || P == 1) return rc;
+  if (f32) latent_combine_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RS, (float*)out);
+  else latent_combine_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RS, (uint16_t*)out);
+  return CFC_CHECK_LAUNCH();
+}
