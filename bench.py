@@ -82,11 +82,25 @@ def parse_args(argv=None):
     ap.add_argument("--pipeline", choices=["bench", "node"], default="bench",
                     help="bench: the stage code with a static LLM batch (headline); node: the real services "
                          "(Node, in-proc bus, continuous summarization engine), pipeline/node_bench.py")
+    ap.add_argument("--compare", default=None, metavar="PRESET[,PRESET...]",
+                    help="instead of the headline: prefill / decode throughput of these model presets side by side "
+                         "(random weights, pipeline/model_bench.py), e.g. vofosun-7b,mistral-7b")
+    ap.add_argument("--compare-layers", type=int, default=0, help="--compare with only this many layers of each model")
+    ap.add_argument("--compare-shapes", default=None, metavar="BxPxG[,BxPxG...]",
+                    help="--compare shapes: prompts x prompt tokens x generated tokens")
     return ap.parse_args(argv)
 
 
 def main(argv=None):
     args = parse_args(argv)
+    if args.compare:
+        from copilot_for_consensus_amd.pipeline.model_bench import SHAPES, bench_model
+        shapes = tuple(tuple(int(v) for v in s.split("x")) for s in args.compare_shapes.split(",")) \
+            if args.compare_shapes else SHAPES
+        for name in args.compare.split(","):
+            bench_model(name, shapes, layers=args.compare_layers or None, prefill_tokens=args.prefill_tokens,
+                        emit=lambda line: print(line, flush=True))
+        return 0
     import torch
     import torch.distributed as dist
 
