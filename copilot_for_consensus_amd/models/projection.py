@@ -13,23 +13,30 @@ import torch
 import torch.nn.functional as F
 
 from ..ops import kernels as K
+from ..ops.stream import clamped_glu
 
 
 class Projection:
     """y = x W^T for W [N, K], sharded by the caller.  bf16 on the GPU: packed when the shape fits."""
 
+    # swiglu: interleaved gate / up rows, tiled for a product without split (its epilogue gates)
     __slots__ = ("w", "packed", "N", "K", "min_tiles")
 
-    def __init__(self, w: torch.Tensor, decode_rows: int = 128):
+    def __init__(self, w: torch.Tensor, decode_rows: int = 128, swiglu: bool = False):
         self.N, self.K = w.shape
         self.packed = None
         self.w = w.contiguous()
         # fewer 256 x 256 output tiles than this run on the decode GEMM (DecoderModel.PGEMM_MIN_TILES)
         self.min_tiles = 96
-        if (w.is_cuda and w.dtype == torch.bfloat16 and self.N % 64 == 0 and self.K % 64 == 0
-                and os.environ.get("CFC_DECODE_PACKED", "auto") != "0"):
-            self.packed = K.pack_dgemm_weight(self.w, m=decode_rows)
+        if self.packs(w, self.N, self.K):
+            self.packed = K.pack_dgemm_weight(self.w, swiglu=swiglu, m=decode_rows)
             self.w = None
+
+    @staticmethod
+    def packs(w: torch.Tensor, N: int, K: int) -> bool:
+        """Whether an [N, K] matrix like ``w`` is packed for the hand-written products."""
+        return (w.is_cuda and w.dtype == torch.bfloat16 and N % 64 == 0 and K % 64 == 0
+                and os.environ.get("CFC_DECODE_PACKED", "auto") != "0")
 
     def rowmajor(self) -> torch.Tensor:
         return self.w if self.w is not None else K._rowmajor(self.packed)
@@ -73,6 +80,17 @@ class Projection:
         if x.is_cuda and x.dtype == torch.bfloat16:
             return torch.mm(x, w.t(), out_dtype=torch.float32)[None]
         return F.linear(x.float(), w.float())[None]
+
+    def glu(self, x: torch.Tensor, out: torch.Tensor, limit: float, alpha: float, beta: float) -> torch.Tensor:
+        """W = 8-row interleaved gate / up rows, packed: the clamped GLU of the product into ``out`` [M, N / 2]
+        (row-strided), in the product's epilogue where one pass over W fills the chip."""
+        k, M = self._kernel(x), x.shape[0]
+        if k == "pgemm" and self.K >= 128 and out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0:
+            return K.pgemm_glu(x, self.packed, out, limit, alpha, beta)
+        if k in ("pgemm", "dgemm") and self.N // self.packed.bn * -(-M // 256) >= K.DGEMM_CUS // 2 \
+                and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0:
+            return K.dgemm_glu(x, self.packed, out, limit, alpha, beta)
+        return clamped_glu(self.slabs(x), out, limit, alpha, beta, interleaved=True)
 
     def f32(self, x: torch.Tensor) -> torch.Tensor:
         """[M, N] fp32, a tensor of its own."""

@@ -37,6 +37,7 @@ from .projection import Projection
 
 GLU_ALPHA = 1.702     # slope of the gate's sigmoid
 GLU_SHIFT = 1.0       # added to the clamped up projection
+BIAS_COLS = 64        # input columns added for the gate / up biases on the packed path (one K step)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -245,7 +246,7 @@ class VofosunWeights:
             uv = mat(rows(get(p + "mix.uv"))).view(H, m.vdim, m.kv_rank)
             out = [mat(cols(get(p + "mix.o")))]
             lw = {
-                "H": H, "norm": 1.0 + vec(get(p + "norm1")), "convs": [vec(get(p + "canon1"))], "dwa": vec(get(p + "dwa")),
+                "H": H, "norm": 1.0 + vec(get(p + "norm1")), "convs": [vec(get(p + "canon1")).t().contiguous()], "dwa": vec(get(p + "dwa")),
                 "down_in": Projection(torch.cat([mat(get(p + "mix.dq")), mat(get(p + "mix.dkv"))])),
                 "dq_norm": vec(get(p + "mix.dq.norm")), "dkv_norm": vec(get(p + "mix.dkv.norm")),
                 "uq": Projection(mat(rows(get(p + "mix.uq")))),
@@ -253,12 +254,27 @@ class VofosunWeights:
                 "uk": L.HeadWeight(uk.transpose(1, 2), n_out=L.padded_rank(m.kv_rank)),
                 "uv": L.HeadWeight(uv), "bias": None,
             }
+            rs = L.padded_rank(m.kv_rank)
+            if (m.dim == m.vdim == L.EXPANDED_DIM and rs == m.kv_rank and Projection.packs(uk, H * m.dim, rs)
+                    and K.prefill_rows(H, H) == 256):
+                # long portions: keys and values per head from two products (ops.latent.expand)
+                lw["uk_full"] = K.pack_dgemm_weight(uk.reshape(H * m.dim, rs).contiguous())
+                lw["uv_full"] = uv.reshape(H * m.vdim, rs).contiguous()
             if s.mlp is not None:
                 gu = torch.cat([mat(rows(get(p + "mlp.gate"))), mat(rows(get(p + "mlp.up")))])
                 lw["interleaved"] = (s.mlp.ff // tp_size) % 8 == 0
-                lw["gate_up"] = Projection(interleave_gate_up(gu) if lw["interleaved"] else gu)
-                lw["gate_b"], lw["up_b"] = vec(rows(get(p + "mlp.gate.b"))), vec(rows(get(p + "mlp.up.b")))
-                lw["convs"].append(vec(get(p + "canon2")))
+                gb, ub = rows(get(p + "mlp.gate.b")), rows(get(p + "mlp.up.b"))
+                # packed: the biases are one more column of W (the input carries a constant 1 there), so
+                # the product's epilogue has only the gate to do
+                lw["fused_glu"] = lw["interleaved"] and Projection.packs(gu, gu.shape[0], cfg.hidden + BIAS_COLS)
+                if lw["fused_glu"]:
+                    pad = gu.new_zeros(gu.shape[0], BIAS_COLS)
+                    pad[:, 0] = mat(torch.cat([gb, ub]))
+                    gu = torch.cat([gu, pad], 1)
+                else:
+                    lw["gate_b"], lw["up_b"] = vec(gb), vec(ub)
+                lw["gate_up"] = Projection(interleave_gate_up(gu) if lw["interleaved"] else gu, swiglu=lw["fused_glu"])
+                lw["convs"].append(vec(get(p + "canon2")).t().contiguous())
                 out.append(mat(cols(get(p + "mlp.down"))))
                 lw["bias"] = vec(get(p + "mlp.down.b"))
             lw["out"] = Projection(torch.cat(out, 1))
@@ -275,6 +291,7 @@ class VofosunWeights:
         for lw in self.layers:
             n += sum(lw[k].nbytes() for k in ("down_in", "uq", "uk", "uv", "out"))
             n += lw["gate_up"].nbytes() if "gate_up" in lw else 0
+            n += lw["uk_full"].nbytes() + lw["uv_full"].numel() * 2 if "uk_full" in lw else 0
         return n
 
 
@@ -283,7 +300,7 @@ class VofosunModel:
 
     # leading blocks are shared with other sequences only once computed: a portion reads the
     # convolution tail of the block before it in the launch that writes the tails
-    kernel_sources = ("elementwise", "stream", "latent", "gemm", "dgemm", "pgemm")
+    kernel_sources = ("elementwise", "stream", "latent", "gemm", "dgemm", "pgemm", "attention")
 
     def __init__(self, weights: VofosunWeights, tp_group=None, custom_ar=None):
         self.w = weights
@@ -320,7 +337,27 @@ class VofosunModel:
             if key not in plan:
                 plan[key] = np.asarray(L.attn_tiles(cu, lw["H"], self._rows(i, False), ctx), np.int32).reshape(2, -1)
         plan["max_ctx"] = max(ctx)
+        for i, lw in enumerate(self.w.layers):
+            rs = self._rs(i)
+            if "uk_full" in lw and f"expand_{rs}" not in plan:
+                plan[f"expand_{rs}"] = self._expand_pays(cu, ctx, rs)
+                if plan[f"expand_{rs}"] and "gather" not in plan:
+                    gt, base = L.gather_tiles(ctx)
+                    plan["gather"], plan["tok_base"] = np.asarray(gt, np.int32), np.asarray(base, np.int32)
+                    plan["pf_tiles"] = np.asarray(K.prefill_tiles(cu, 256, ctx), np.int32)
         return plan
+
+    @staticmethod
+    def _expand_pays(cu, ctx, rs) -> bool:
+        """Whether per-head keys and values of the pass's contexts cost fewer flops (per head, halved) than
+        attention in the latent space with its two per-head products."""
+        d, latent, dense = 2 * L.EXPANDED_DIM, 0.0, 0.0
+        for s in range(len(ctx)):
+            n = cu[s + 1] - cu[s]
+            pairs = n * (ctx[s] - n / 2)
+            latent += pairs * 2 * rs + n * rs * d
+            dense += pairs * d + -(-ctx[s] // 64) * 64 * rs * d
+        return dense < latent
 
     # ---------------------------------------------------------------- forward
     def forward_prefill(self, ids, positions, slots, cu_q, ctx_lens, block_tables, kv, last_idx=None, plan=None):
@@ -332,17 +369,18 @@ class VofosunModel:
         hist, x = self._embed(ids)
         T = ids.numel()
         rstd = torch.empty(T, dtype=torch.float32, device=ids.device)
-        cur, up = hist[0], None
+        cur, up, bufs = hist[0], None, {}
         for i, lw in enumerate(self.w.layers):
             S.depth_stats(cur, hist, up, self.cfg.norm_eps, x, rstd)
             cur = x
-            hs = self._inputs(T, lw, ids.device)
+            hs = self._inputs(T, lw, ids.device, bufs)
             S.input_conv(x, rstd, lw["norm"], lw["convs"], plan["conv_tiles"], S.Tail(kv.tails[i], block_tables), hs)
             rows = self._rows(i, False)
             tiles = plan[f"attn_{lw['H']}_{rows}"]
             attn = dict(cu_q=cu_q, tiles=(tiles[0], tiles[1]), rows=rows,
                         P=L.partitions(tiles.shape[1], plan["max_ctx"]))
-            up = self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn)
+            dense = plan if "uk_full" in lw and plan[f"expand_{self._rs(i)}"] else None
+            up = self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn, dense)
         return S.depth_norm(cur, hist, up, self.w.final_norm, self.cfg.norm_eps, self.w.dtype,
                             None if last_idx is None else last_idx.to(torch.int32))
 
@@ -352,9 +390,9 @@ class VofosunModel:
         slices per sequence (the engine's form); ``shared_blocks`` is not used (latents are read once per
         token for all heads, through the caches)."""
         hist, x = self._embed(ids)
-        cur, up = hist[0], None
+        cur, up, bufs = hist[0], None, {}
         for i, lw in enumerate(self.w.layers):
-            hs = self._inputs(ids.numel(), lw, ids.device)
+            hs = self._inputs(ids.numel(), lw, ids.device, bufs)
             S.depth_conv_decode(cur, hist, up, lw["norm"], self.cfg.norm_eps, lw["convs"], positions,
                                 S.Tail(kv.tails[i], block_tables), x, hs)
             cur = x
@@ -368,26 +406,47 @@ class VofosunModel:
         S.embed_f32(self.w.embed, ids, hist[0])
         return hist, torch.empty_like(hist[0])
 
-    def _inputs(self, T, lw, device):
-        """Activation buffers of the sublayers' inputs."""
-        return [torch.empty(T, self.cfg.hidden, dtype=self.w.dtype, device=device) for _ in lw["convs"]]
+    def _inputs(self, T, lw, device, bufs):
+        """Activation buffers of the sublayers' inputs (the feed-forward's with its constant bias columns),
+        one set per forward pass, kept in ``bufs``."""
+        W, two = self.cfg.hidden, len(lw["convs"]) > 1
+        wide = two and lw["fused_glu"]
+        if (two, wide) not in bufs:
+            hs = [torch.empty(T, W, dtype=self.w.dtype, device=device)]
+            if two:
+                hs.append(torch.empty(T, W + (BIAS_COLS if wide else 0), dtype=self.w.dtype, device=device))
+            if wide:
+                hs[1][:, W:].zero_()
+                hs[1][:, W].fill_(1.0)
+            bufs[two, wide] = hs
+        return bufs[two, wide]
 
-    def _layer(self, i, hs, slots, ctx_lens, block_tables, kv, attn) -> S.Update:
-        """Both sublayers of layer i on their inputs: what the layer adds to the stream."""
+    def _layer(self, i, hs, slots, ctx_lens, block_tables, kv, attn, dense=None) -> S.Update:
+        """Both sublayers of layer i on their inputs: what the layer adds to the stream.  ``dense``: the launch
+        plan of a pass whose keys and values are expanded per head."""
         lw, spec = self.w.layers[i], self.cfg.specs[i]
         m, H = spec.mixer, lw["H"]
         T, dt, dev = hs[0].shape[0], self.w.dtype, hs[0].device
         cq = L.latent_norm(lw["down_in"].slabs(hs[0]), m.q_rank, lw["dq_norm"], lw["dkv_norm"], self.cfg.norm_eps, slots,
                            kv.latents[i], dt)
         q = lw["uq"].act(cq).view(T, H, m.dim)
-        ql = L.head_linear(q, lw["uk"], torch.empty(T, H, self._rs(i), dtype=dt, device=dev))
-        ol = L.latent_attention(ql, kv.latents[i], block_tables, ctx_lens=ctx_lens, scale=m.scale, **attn)
         F = spec.mlp.ff // self.w.tp_size if spec.mlp is not None else 0
         cat = torch.empty(T, H * m.vdim + F, dtype=dt, device=dev)
-        L.head_linear(ol, lw["uv"], cat[:, :H * m.vdim].unflatten(1, (H, m.vdim)))
+        o = cat[:, :H * m.vdim].unflatten(1, (H, m.vdim))
+        if dense is not None:
+            k, vt = L.expand(kv.latents[i], block_tables, ctx_lens, dense["gather"], lw["uk_full"], lw["uv_full"])
+            L.expanded_attention(q, k, vt, dense["tok_base"], attn["cu_q"], ctx_lens, m.scale, dense["pf_tiles"], o)
+        else:
+            ql = L.head_linear(q, lw["uk"], torch.empty(T, H, self._rs(i), dtype=dt, device=dev))
+            ol = L.latent_attention(ql, kv.latents[i], block_tables, ctx_lens=ctx_lens, scale=m.scale, **attn)
+            L.head_linear(ol, lw["uv"], o)
         if F:
-            S.clamped_glu(lw["gate_up"].act(hs[1]), cat[:, H * m.vdim:], spec.mlp.limit, GLU_ALPHA, GLU_SHIFT,
-                          lw["gate_b"], lw["up_b"], lw["interleaved"])
+            a = cat[:, H * m.vdim:]
+            if lw["fused_glu"]:
+                lw["gate_up"].glu(hs[1], a, spec.mlp.limit, GLU_ALPHA, GLU_SHIFT)
+            else:
+                gu = lw["gate_up"].slabs(hs[1])
+                S.clamped_glu(gu, a, spec.mlp.limit, GLU_ALPHA, GLU_SHIFT, lw["gate_b"], lw["up_b"], lw["interleaved"])
         part = lw["out"].slabs(cat)
         if self.w.tp_size > 1:
             part = part.sum(0, keepdim=True)

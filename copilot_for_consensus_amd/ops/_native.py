@@ -56,11 +56,13 @@ _KERNEL_SIGS = {
     "cfc_embed_f32": [P, P, P, I, I, I, I, P],
     "cfc_depth_norm": [I, I, I, P, P, P, P, I, P, P, I, P, F, P, P, I, I, P, I, P, I, P, P, I, P, P, I, P, I, P],
     "cfc_input_conv": [I, I, P, P, P, P, P, P, I, P, I, P, I, I, P, I, P, I, P],
-    "cfc_clamped_glu": [I, I, P, I, P, P, P, I, I, I, F, F, F, P],
+    "cfc_clamped_glu": [I, I, P, I, P, I, P, P, I, I, I, F, F, F, P],
     "cfc_softcap": [P, c_int64, F, P],
     "cfc_latent_norm": [I, P, I, I, I, I, P, P, F, P, P, I, P, I, P],
     "cfc_head_linear": [I, P, c_int64, c_int64, P, I, I, I, I, I, I, P, c_int64, c_int64, P],
     "cfc_latent_attention": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, P, P, P],
+    "cfc_latent_gather": [P, P, I, P, P, I, I, P, P, P],
+    "cfc_prefill_attention_expanded": [P, P, P, P, c_int64, P, P, P, P, I, I, F, P, c_int64, P],
     "cfc_knn_scores": [P, P, I, I, I, P, P, P, P],
     "cfc_topk_pass": [P, P, I, I, I, I, P, P, P],
     "cfc_knn_topk": [P, P, I, I, I, I, P, P, P, I, P, P, P],
@@ -76,6 +78,8 @@ _KERNEL_SIGS = {
     "cfc_pgemm_ln": [P, P, P, P, P, P, P, I, I, I, F, P],
     "cfc_pgemm_probe": [P, P, P, I, I, I, I, I, I, P],
     "cfc_pgemm_ppp_probe": [P, P, P, I, I, I, I, I, I, I, P],
+    "cfc_pgemm_glu": [P, P, P, I, I, I, I, I, F, F, F, P],
+    "cfc_dgemm_glu": [P, P, I, I, I, I, P, I, F, F, F, P],
     "cfc_dgemm_bm": [I],
     "cfc_dgemm_pack": [P, P, I, I, I, P],
     "cfc_dgemm_ablate": [P, P, I, I, I, I, I, I, P, P],

@@ -674,6 +674,35 @@ def pgemm(x: torch.Tensor, w, epi: str = "bf16", bias: torch.Tensor | None = Non
     return out
 
 
+def _glu_out(x, w, out, name):
+    if not isinstance(w, PackedWeight) or out.shape != (x.shape[0], w.N // 2) or out.dtype != torch.bfloat16 \
+            or out.stride(1) != 1:
+        raise ValueError(f"{name}: x {tuple(x.shape)} w {tuple(w.shape)} out {tuple(out.shape)} {out.dtype}")
+
+
+def pgemm_glu(x: torch.Tensor, w: "PackedWeight", out: torch.Tensor, limit: float, alpha: float,
+              beta: float) -> torch.Tensor:
+    """pgemm over packed 8-row interleaved gate / up weights with the clamped GLU in its epilogue:
+    min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta) into ``out`` [M, N / 2] (row-strided)."""
+    _glu_out(x, w, out, "pgemm_glu")
+    if not pgemm_ok(x, w):
+        raise ValueError(f"pgemm_glu: x {tuple(x.shape)} {x.dtype} w {tuple(w.shape)}")
+    check(kernels().cfc_pgemm_glu(x.data_ptr(), w.data.data_ptr(), out.data_ptr(), x.shape[0], w.N, w.K, out.stride(0),
+                                  w.bn // 16, float(limit), float(alpha), float(beta), _stream(x)), "cfc_pgemm_glu")
+    return out
+
+
+def dgemm_glu(x: torch.Tensor, w: "PackedWeight", out: torch.Tensor, limit: float, alpha: float,
+              beta: float) -> torch.Tensor:
+    """:func:`pgemm_glu` on the decode GEMM (one pass over W, no split)."""
+    _glu_out(x, w, out, "dgemm_glu")
+    if not dgemm_ok(x, w):
+        raise ValueError(f"dgemm_glu: x {tuple(x.shape)} {x.dtype} w {tuple(w.shape)}")
+    check(kernels().cfc_dgemm_glu(x.data_ptr(), w.data.data_ptr(), x.shape[0], w.N, w.K, w.bn, out.data_ptr(),
+                                  out.stride(0), float(limit), float(alpha), float(beta), _stream(x)), "cfc_dgemm_glu")
+    return out
+
+
 PGEMM_LN_N = (384,)     # output widths the fused GEMM + LayerNorm kernel is built for
 
 

@@ -141,3 +141,48 @@ def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles
                                          block_tables.shape[1], float(scale), P, T * H, _p(po), _p(pm), out.data_ptr(),
                                          _stream(q)), "cfc_latent_attention")
     return out
+
+
+# ------------------------------------------------------- long portions: expanded keys and values
+EXPANDED_DIM = 128        # head size of the prefill attention kernel
+
+
+def gather_tiles(ctx_lens) -> tuple[list, list]:
+    """Dense layout of whole sequences, 64-token tiles: ([(sequence, first position)], first row per sequence)."""
+    tiles, base, n = [], [], 0
+    for s, ctx in enumerate(ctx_lens):
+        base.append(n)
+        m = -(-ctx // 64)
+        tiles += [(s, 64 * i) for i in range(m)]
+        n += 64 * m
+    return tiles, base
+
+
+def expand(cache, block_tables, ctx_lens, tiles, uk, uv):
+    """Keys [tokens, H * 128] and transposed, slot-ordered values [H * 128, tokens] (row stride padded) of the
+    sequences of ``tiles`` (:func:`gather_tiles`): uk a PackedWeight [H * 128, RS], uv row-major [H * 128, RS]."""
+    from . import kernels as K
+    n, RS = tiles.shape[0], cache.shape[-1]
+    rows = torch.empty(2, n * 64, RS, dtype=cache.dtype, device=cache.device)
+    check(kernels().cfc_latent_gather(cache.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], ctx_lens.data_ptr(),
+                                      tiles.data_ptr(), n, RS, rows[0].data_ptr(), rows[1].data_ptr(), _stream(cache)),
+          "cfc_latent_gather")
+    k = K.pgemm(rows[0], uk, variant="ppp")
+    # the values' rows are read side by side: an odd number of 128-byte lines apart, not a power of two
+    ldv = n * 64 + (64 if n % 2 == 0 else 128)
+    vt = torch.empty(uv.shape[0], ldv, dtype=cache.dtype, device=cache.device)[:, :n * 64]
+    K.pgemm(uv, rows[1], out=vt, variant="pp")
+    return k, vt
+
+
+def expanded_attention(q, k, vt, tok_base, cu_q, ctx_lens, scale: float, tiles, out) -> torch.Tensor:
+    """Causal attention of q [T, H, 128] over :func:`expand`'s keys and values into ``out`` [T, H, 128] (row stride
+    free, heads dense); ``tiles``: ops.kernels.prefill_tiles for 256-row tiles."""
+    T, H, D = q.shape
+    if D != EXPANDED_DIM or not q.is_contiguous() or out.stride(1) != D or out.stride(2) != 1:
+        raise ValueError(f"expanded_attention: q {tuple(q.shape)}, out strides {out.stride()}")
+    check(kernels().cfc_prefill_attention_expanded(q.data_ptr(), k.data_ptr(), vt.data_ptr(), tok_base.data_ptr(),
+                                                   vt.stride(0), cu_q.data_ptr(), ctx_lens.data_ptr(), tiles[0].data_ptr(),
+                                                   tiles[1].data_ptr(), tiles[0].numel(), H, float(scale), out.data_ptr(),
+                                                   out.stride(0), _stream(q)), "cfc_prefill_attention_expanded")
+    return out

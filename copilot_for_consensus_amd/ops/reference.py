@@ -336,9 +336,9 @@ def depth_norm(x, hist, part, bias, dwa, n, eps):
 def input_conv(h, portions, block_tables, tail, weights):
     """h [T, W] fp32 convolution inputs of packed portions [(first row, rows, first position, sequence)];
     tail [blocks, slots, W] read for positions before a portion and updated.  weights: per sublayer
-    [W, taps].  Returns one h + conv(h) per sublayer."""
+    [taps, W].  Returns one h + conv(h) per sublayer."""
     outs = [h.clone() for _ in weights]
-    taps = weights[0].shape[1]
+    taps = weights[0].shape[0]
     for row0, n, pos0, seq in portions:
         past = []
         for q in range(pos0 - taps + 1, pos0):
@@ -349,7 +349,7 @@ def input_conv(h, portions, block_tables, tail, weights):
         ext = torch.cat([torch.stack(past), h[row0:row0 + n]]) if past else h[row0:row0 + n]
         for o, w in zip(outs, weights):
             for j in range(taps):
-                o[row0:row0 + n] += w[:, j] * ext[j:j + n]
+                o[row0:row0 + n] += w[j] * ext[j:j + n]
         for r in range(n):
             q = pos0 + r
             # the last inputs of the portion and of every block it crosses

@@ -72,7 +72,7 @@ def _depth(mode, f32, nrows, rows, x, hist, up, norm_w, eps, x_out, rstd, h1, h2
         mode, f32, nrows, _p(rows), x.data_ptr(), hist.data_ptr(), _p(up.part) if up else None,
         up.part.shape[0] if up else 0, _p(up.bias) if up else None, _p(up.dwa) if up else None, up.n if up else 0,
         _p(norm_w), float(eps), _p(x_out), _p(rstd), T, W, _p(h1), h1.stride(0) if h1 is not None else 0, _p(h2),
-        h2.stride(0) if h2 is not None else 0, _p(w1), _p(w2), w1.shape[1] if w1 is not None else 1, _p(positions), *t,
+        h2.stride(0) if h2 is not None else 0, _p(w1), _p(w2), w1.shape[0] if w1 is not None else 1, _p(positions), *t,
         _stream(ref_t)), "cfc_depth_norm")
 
 
@@ -103,7 +103,7 @@ def depth_norm(x, hist, up: Update | None, norm_w, eps: float, dtype, rows=None)
 
 def depth_conv_decode(x, hist, up: Update | None, norm_w, eps: float, convs, positions, tail: Tail, x_out, outs) -> None:
     """One token per sequence: apply ``up``, norm, and run the row through each sublayer's input
-    convolution (``convs``: one or two [W, taps]) with the cached tail; results into ``outs``."""
+    convolution (``convs``: one or two [taps, W]) with the cached tail; results into ``outs``."""
     if not hist.is_cuda:
         y, r = ref.depth_norm(x, hist, up and up.part, up and up.bias, up and up.dwa, up.n if up else 0, eps)
         x_out.copy_(y)
@@ -150,29 +150,32 @@ def input_conv(x, rstd, norm_w, convs, tiles, tail: Tail, outs) -> None:
     two = len(convs) > 1
     check(kernels().cfc_input_conv(_act(outs[0].dtype), tiles.shape[1], tiles.data_ptr(), x.data_ptr(), rstd.data_ptr(),
                                    norm_w.data_ptr(), convs[0].data_ptr(), _p(convs[1]) if two else None,
-                                   convs[0].shape[1], *tail.args(), x.shape[1], outs[0].data_ptr(), outs[0].stride(0),
+                                   convs[0].shape[0], *tail.args(), x.shape[1], outs[0].data_ptr(), outs[0].stride(0),
                                    _p(outs[1]) if two else None, outs[1].stride(0) if two else 0, _stream(x)),
           "cfc_input_conv")
 
 
 def clamped_glu(gu, out, limit: float, alpha: float, beta: float, gate_bias=None, up_bias=None,
                 interleaved: bool = False) -> torch.Tensor:
-    """g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + beta) into ``out`` [T, F] (row-strided);
-    ``gu`` [T, 2F]: gate | up halves or the 8-column interleaved groups of ops.reference.interleave_gate_up."""
-    T, F2 = gu.shape
+    """g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + beta) into ``out`` [T, F] (row-strided).
+    ``gu`` [T, 2F], or fp32 slabs [split, T, 2F] to be summed: gate | up halves or the 8-column interleaved
+    groups of ops.reference.interleave_gate_up."""
+    T, F2 = gu.shape[-2:]
+    split = gu.shape[0] if gu.dim() == 3 else 1
     if not gu.is_cuda:
+        gu = gu.float().sum(0) if gu.dim() == 3 else gu.float()
         if interleaved:
             v = gu.view(T, -1, 2, ref.GU_GROUP)
             g, u = v[:, :, 0].reshape(T, -1), v[:, :, 1].reshape(T, -1)
         else:
             g, u = gu[:, :F2 // 2], gu[:, F2 // 2:]
-        g = g.float() + (gate_bias if gate_bias is not None else 0.0)
-        u = u.float() + (up_bias if up_bias is not None else 0.0)
+        g = g + (gate_bias if gate_bias is not None else 0.0)
+        u = u + (up_bias if up_bias is not None else 0.0)
         out.copy_(ref.clamped_glu(g, u, limit, alpha, beta))
         return out
-    if not gu.is_contiguous():
-        raise ValueError("clamped_glu: gate / up must be contiguous")
-    check(kernels().cfc_clamped_glu(_act(out.dtype), _act(gu.dtype), out.data_ptr(), out.stride(0), gu.data_ptr(),
+    if not gu.is_contiguous() or out.shape != (T, F2 // 2):
+        raise ValueError(f"clamped_glu: gate / up {tuple(gu.shape)} (contiguous), out {tuple(out.shape)}")
+    check(kernels().cfc_clamped_glu(_act(out.dtype), _act(gu.dtype), out.data_ptr(), out.stride(0), gu.data_ptr(), split,
                                     _p(gate_bias), _p(up_bias), T, F2 // 2, int(interleaved), float(limit), float(alpha),
                                     float(beta), _stream(gu)), "cfc_clamped_glu")
     return out

@@ -891,12 +891,16 @@ __device__ __forceinline__ float quad_sum(float x) {
 }
 __device__ __forceinline__ int v5_off(int d, int c) { return d * 128 + ((c ^ ((d >> 1) & 7) ^ ((d & 1) << 2)) << 4); }
 
-template <int G, bool F8 = false>
+// EXP: keys and values are not in the paged cache but dense (a latent cache's, expanded for this pass):
+// K [tokens][Hkv][128] and V^T [Hkv][128][ldv] with each 32 tokens in the cache's slot order, sequence s
+// at tokens tok_base[s] .. (rounded up to 64, zero-filled); outputs leave with row stride ldo.
+template <int G, bool F8 = false, bool EXP = false>
 __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
     const uint16_t* __restrict__ q, const void* __restrict__ kc, const void* __restrict__ vc,
     const int32_t* __restrict__ block_tables, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ ctx_lens,
     const int32_t* __restrict__ tile_seq, const int32_t* __restrict__ tile_q0, float scale_log2, int Hq, int Hkv,
-    int max_blocks, int window, float v_scale, int xcd_local, uint16_t* __restrict__ out) {
+    int max_blocks, int window, float v_scale, int xcd_local, uint16_t* __restrict__ out,
+    const int32_t* __restrict__ tok_base = nullptr, int64_t ldv = 0, int64_t ldo = 0) {
   // F8: e4m3 caches (K / k_scale folded into scale_log2 by the host, V / v_scale rescaled at the
   // output); tiles are widened to bf16 at the LDS write, so the MFMA loop is the bf16 one
   constexpr int D = 128;
@@ -958,7 +962,18 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
   // the tile's MFMAs.
   const int nb_need = (kend + KV_BS - 1) / KV_BS;
   uint4 ks0, ks1, vs0, vs1;     // named (not an array): an array here is kept in scratch
+  const int64_t tok0 = EXP ? tok_base[s] : 0;
   auto gload = [&](int kt) {
+    if constexpr (EXP) {
+      const int64_t t0 = tok0 + kt * PF_KT;
+      const uint16_t* kp = reinterpret_cast<const uint16_t*>(kc) + ((t0 + (tid >> 4)) * Hkv + hk) * D + 8 * (tid & 15);
+      const uint16_t* vp = reinterpret_cast<const uint16_t*>(vc) + ((int64_t)hk * D + (tid >> 3)) * ldv + t0 + 8 * (tid & 7);
+      ks0 = *reinterpret_cast<const uint4*>(kp);
+      vs0 = *reinterpret_cast<const uint4*>(vp);
+      ks1 = *reinterpret_cast<const uint4*>(kp + (int64_t)32 * Hkv * D);
+      vs1 = *reinterpret_cast<const uint4*>(vp + 64 * ldv);
+      return;
+    }
     const int b0 = bt[min(2 * kt, nb_need - 1)], b1 = bt[min(2 * kt + 1, nb_need - 1)];
     if constexpr (F8) {
       // 8 KB of K and 8 KB of V per tile: one 16-B piece of each per thread; block = tid >> 8
@@ -977,6 +992,13 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
   auto lwrite = [&](int buf, int kt) {
     char* kb = smem + buf * 16384;
     char* vb = smem + 32768 + buf * 16384;
+    if constexpr (EXP) {
+      *reinterpret_cast<uint4*>(kb + k_lds_off(tid >> 4, tid & 15)) = ks0;
+      *reinterpret_cast<uint4*>(kb + k_lds_off((tid >> 4) + 32, tid & 15)) = ks1;
+      *reinterpret_cast<uint4*>(vb + v5_off(tid >> 3, tid & 7)) = vs0;
+      *reinterpret_cast<uint4*>(vb + v5_off((tid >> 3) + 64, tid & 7)) = vs1;
+      return;
+    }
     const bool z0 = kt * PF_KT >= kend, z1 = kt * PF_KT + KV_BS >= kend;
     if constexpr (F8) {
       const int b = tid >> 8, e = tid & 255;
@@ -1149,7 +1171,7 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
   l = pair_sum((lp[0] + lp[1]) + (lp[2] + lp[3]));
   if (my_row < q_len) {
     const float inv = l > 0.f ? v_scale / l : 0.f;
-    uint16_t* orow = out + ((size_t)(q_begin + my_row) * Hq + hq) * D;
+    uint16_t* orow = EXP ? out + (q_begin + my_row) * ldo + hq * D : out + ((size_t)(q_begin + my_row) * Hq + hq) * D;
 #pragma unroll
     for (int dt = 0; dt < 4; ++dt)
 #pragma unroll
@@ -1509,6 +1531,20 @@ CFC_API int cfc_prefill_attention(const void* q, const void* k_cache, const void
   else prefill_paged_kernel<4><<<dim3(n_tiles, Hq), 512, lds, stream>>>(PF_ARGS);
 #undef PF_ARGS
 #undef PF5_ARGS
+  return CFC_CHECK_LAUNCH();
+}
+
+// Causal prefill attention over dense K [tokens][H][128] / V^T [H][128][ldv] (prefill_gqa_kernel's EXP
+// layout), one kv head per query head, 256-row tiles; out row t, head h at t ldo + 128 h.
+CFC_API int cfc_prefill_attention_expanded(const void* q, const void* k, const void* vt, const int32_t* tok_base,
+                                           int64_t ldv, const int32_t* cu_q, const int32_t* ctx_lens,
+                                           const int32_t* tile_seq, const int32_t* tile_q0, int n_tiles, int H, float scale,
+                                           void* out, int64_t ldo, hipStream_t stream) {
+  if (n_tiles <= 0) return 0;
+  if (H < 1 || H > 65535 || ldv % 8 || ldo % 4 || ldo < (int64_t)128 * H || ((uintptr_t)vt & 15) || ((uintptr_t)out & 7)) return -1;
+  prefill_gqa_kernel<1, false, true><<<dim3(n_tiles, H), 512, 65536, stream>>>(
+      (const uint16_t*)q, k, vt, nullptr, cu_q, ctx_lens, tile_seq, tile_q0, scale * LOG2E, H, H, 0, 0, 1.f,
+      prefill_xcd_local(), (uint16_t*)out, tok_base, ldv, ldo);
   return CFC_CHECK_LAUNCH();
 }
 

@@ -48,7 +48,10 @@ constexpr int dg_loaders() { return BN / 16 >= 7 ? 1 : 8 - BN / 16 > 2 ? 2 : 8 -
 // runs instead of as dirty L2 lines the kernel boundary must write back before the consumer (the
 // residual + RMSNorm reduce, rope_kv) may start -- MI355X_MICROARCH "boundary": +B / 6 TB/s behind
 // B dirty bytes, 2.8-3.8 us behind 12.6-16.8 MB of fp32 partials.
-enum { DG_PART = 0, DG_BF16 = 1, DG_SILU = 2, DG_PART_WT = 3 };
+enum { DG_PART = 0, DG_BF16 = 1, DG_SILU = 2, DG_PART_WT = 3, DG_GLU = 4 };
+
+// constants of the DG_GLU epilogue: min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta)
+struct DgGlu { float limit = 0.f, alpha = 1.f, beta = 0.f; };
 
 // MX (ablation 64): two X-loader waves and an 8-slot X ring whatever BN -- one loader wave's
 // vmcnt window (63 pieces = 3 stages at BM = 128) may cap the X stream of the wide-BN shapes.
@@ -145,7 +148,7 @@ __device__ __forceinline__ uint4 dg_ldw(const uint16_t* p) {
 template <int BM, int BN, int EPI, bool NTW, int ABL = 0, bool PACKED = true>
 __global__ void __launch_bounds__((64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES), 1)
     dgemm_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, int M, int N, int K, int ntiles,
-                 int split, float* __restrict__ part, uint16_t* __restrict__ out, int ldo) {
+                 int split, float* __restrict__ part, uint16_t* __restrict__ out, int ldo, DgGlu gp) {
   using S = DgShape<BM, BN, (ABL & 64) != 0>;
   constexpr int NW = S::NW;
   constexpr int D = S::D;
@@ -302,14 +305,18 @@ __global__ void __launch_bounds__((64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES)
     // per lane: 4x the store instructions, the epilogue's store-issue tail of a small-N projection)
     const int mr = m0 + (lane & 15);
     const int nq = n0 + 16 * w + 4 * kq;
-    if constexpr (EPI == DG_SILU) {
+    if constexpr (EPI == DG_SILU || EPI == DG_GLU) {
       // 8-row interleave: W rows 0-7 of each 16-row group are gate, 8-15 the matching up rows, so the
       // lanes with kq < 2 hold gate rows and lane ^ 32 the up rows of the same output columns.  One
       // VALU lane swap (v_permlane32_swap) of (acc[0], acc[2]) hands every lane a (gate, up) pair --
       // column 0 in lanes kq < 2, column 2 in lanes kq >= 2 -- and one of (acc[1], acc[3]) columns
       // 1 / 3: each lane computes and stores two outputs
       const int oc = (n0 >> 1) + 8 * w + 4 * (kq & 1) + 2 * (kq >> 1);
-      auto silu_mul = [](float gate, float up) {
+      auto silu_mul = [&](float gate, float up) {
+        if constexpr (EPI == DG_GLU) {
+          const float gg = fminf(gate, gp.limit), uu = fminf(fmaxf(up, -gp.limit), gp.limit);
+          return gg / (1.f + __expf(-gp.alpha * gg)) * (uu + gp.beta);
+        }
         const float gt = bf2f(f2bf(gate)), u = bf2f(f2bf(up));
         return gt / (1.f + __expf(-gt)) * u;
       };
@@ -400,7 +407,7 @@ int dgemm_launch_bn(const void* x, const void* w, int M, int N, int K, int split
   const int ntiles = N / BN;
   const dim3 grid(ntiles * split, (M + BM - 1) / BM);
   const int threads = 64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES;
-#define DG_ARGS (const uint16_t*)x, (const uint16_t*)w, M, N, K, ntiles, split, part, (uint16_t*)out, ldo
+#define DG_ARGS (const uint16_t*)x, (const uint16_t*)w, M, N, K, ntiles, split, part, (uint16_t*)out, ldo, DgGlu{}
   switch (epi) {
     case DG_PART: dgemm_kernel<BM, BN, DG_PART, NTW, ABL, PK><<<grid, threads, 0, stream>>>(DG_ARGS); break;
     case DG_PART_WT: dgemm_kernel<BM, BN, DG_PART_WT, NTW, ABL, PK><<<grid, threads, 0, stream>>>(DG_ARGS); break;
@@ -485,6 +492,40 @@ CFC_API int cfc_dgemm(const void* x, const void* w, int M, int N, int K, int spl
 
 // Row-major W[N][K] bf16 -> the fragment-packed layout for bn-row workgroups (same size; the
 // packed weight is only valid with that bn).  N % bn == 0, bn % 16 == 0, K % 64 == 0.
+namespace {
+template <int BM, int BN>
+void dgemm_glu_go(const void* x, const void* w, int M, int N, int K, void* out, int ldo, const DgGlu& gp, hipStream_t stream) {
+  dgemm_kernel<BM, BN, DG_GLU, DG_NT, 0, true><<<dim3(N / BN, (M + BM - 1) / BM), 64 * DgShape<BM, BN>::WAVES, 0, stream>>>(
+      (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, nullptr, (uint16_t*)out, ldo, gp);
+}
+template <int BM>
+int dgemm_glu_bn(const void* x, const void* w, int M, int N, int K, int bn, void* out, int ldo, const DgGlu& gp,
+                 hipStream_t stream) {
+  switch (bn) {
+    case 64: dgemm_glu_go<BM, 64>(x, w, M, N, K, out, ldo, gp, stream); return 0;
+    case 96: dgemm_glu_go<BM, 96>(x, w, M, N, K, out, ldo, gp, stream); return 0;
+    case 112: dgemm_glu_go<BM, 112>(x, w, M, N, K, out, ldo, gp, stream); return 0;
+    case 128: dgemm_glu_go<BM, 128>(x, w, M, N, K, out, ldo, gp, stream); return 0;
+  }
+  return -5;
+}
+}  // namespace
+
+// Clamped GLU epilogue over packed, 8-row interleaved gate / up weights: out [M, N / 2] (row stride ldo)
+CFC_API int cfc_dgemm_glu(const void* x, const void* w, int M, int N, int K, int bn, void* out, int ldo, float limit,
+                          float alpha, float beta, hipStream_t stream) {
+  if (const int e = dgemm_check(M, N, K, 1, DG_GLU, bn, nullptr, out, ldo)) return e;
+  DgGlu gp;
+  gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
+  int rc;
+  switch (cfc_dgemm_bm(M)) {
+    case 64: rc = dgemm_glu_bn<64>(x, w, M, N, K, bn, out, ldo, gp, stream); break;
+    case 128: rc = dgemm_glu_bn<128>(x, w, M, N, K, bn, out, ldo, gp, stream); break;
+    default: rc = dgemm_glu_bn<256>(x, w, M, N, K, bn, out, ldo, gp, stream); break;
+  }
+  return rc ? rc : CFC_CHECK_LAUNCH();
+}
+
 CFC_API int cfc_dgemm_pack(const void* w, void* wp, int N, int K, int bn, hipStream_t stream) {
   if (N <= 0 || K <= 0 || bn <= 0 || bn % 16 || N % bn || K % 64 || w == wp) return -1;
   const size_t pieces = (size_t)N * K / 8;

@@ -11,8 +11,9 @@
 //                     flattened (token, head) rows of one sequence -- one decoded token's heads and a
 //                     prompt portion's rows are the same thing to it -- and a slice of its keys
 //   * latent_combine  merges the slices
-//   * latent_expand   a sequence's latents as per-head K / V blocks in the layout of the paged prefill
-//                     attention (attention.hip), for long portions where that costs fewer flops
+//   * latent_gather   the latents of whole sequences as dense rows, in token order and in the slot order
+//                     of the prefill attention's V^T: two products turn them into per-head keys and
+//                     values for long portions, where that costs fewer flops (attention.hip, EXP)
 #include "common.h"
 
 namespace {
@@ -453,6 +454,26 @@ __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restr
   }
 }
 
+// tiles [n][2]: {sequence, first position} of 64 tokens each, at dense rows 64 blockIdx.x ..; positions past
+// the context are zero rows
+__global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __restrict__ cache,
+                                                           const int32_t* __restrict__ block_tables, int max_blocks,
+                                                           const int32_t* __restrict__ ctx_lens,
+                                                           const int32_t* __restrict__ tiles, int RS,
+                                                           uint16_t* __restrict__ rows, uint16_t* __restrict__ slot_rows) {
+  const int s = tiles[2 * blockIdx.x], p0 = tiles[2 * blockIdx.x + 1], ctx = ctx_lens[s], ch = RS / 8;
+  const int32_t* bt = block_tables + (size_t)s * max_blocks;
+  for (int e = threadIdx.x; e < 64 * ch; e += 256) {
+    const int r = e / ch, c = e % ch, p = p0 + r;
+    const uint4 v = p < ctx ? *reinterpret_cast<const uint4*>(
+                                  cache + ((size_t)bt[p / CFC_KV_BS] * CFC_KV_BS + p % CFC_KV_BS) * RS + 8 * c)
+                            : make_uint4(0, 0, 0, 0);
+    const size_t base = (size_t)blockIdx.x * 64;
+    reinterpret_cast<uint4*>(rows + (base + r) * RS)[c] = v;
+    reinterpret_cast<uint4*>(slot_rows + (base + (r & 32) + kv_v_slot(r & 31)) * RS)[c] = v;
+  }
+}
+
 // one workgroup of 128 threads per (token, head) row
 template <typename ACT>
 __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __restrict__ part_o,
@@ -577,5 +598,14 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
   if (rc || P == 1) return rc;
   if (f32) latent_combine_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RS, (float*)out);
   else latent_combine_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RS, (uint16_t*)out);
+  return CFC_CHECK_LAUNCH();
+}
+
+CFC_API int cfc_latent_gather(const void* cache, const int32_t* block_tables, int max_blocks, const int32_t* ctx_lens,
+                              const int32_t* tiles, int n_tiles, int RS, void* rows, void* slot_rows, hipStream_t stream) {
+  if (n_tiles <= 0) return 0;
+  if (RS < 32 || RS % 32 || max_blocks < 1) return -1;
+  latent_gather_kernel<<<n_tiles, 256, 0, stream>>>((const uint16_t*)cache, block_tables, max_blocks, ctx_lens, tiles, RS,
+                                                    (uint16_t*)rows, (uint16_t*)slot_rows);
   return CFC_CHECK_LAUNCH();
 }

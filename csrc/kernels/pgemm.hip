@@ -39,7 +39,7 @@ typedef __attribute__((address_space(3))) void pg_lds_t;
 
 // PG_F32: the fp32 accumulators themselves (row stride ldo in floats): a tensor-parallel row-parallel
 // projection's partial, all-reduced in fp32 and rounded to bf16 once, as TP = 1 rounds the full sum
-enum { PG_BF16 = 0, PG_BIAS = 1, PG_BIAS_GELU = 2, PG_SWIGLU = 3, PG_F32 = 4 };
+enum { PG_BF16 = 0, PG_BIAS = 1, PG_BIAS_GELU = 2, PG_SWIGLU = 3, PG_F32 = 4, PG_GLU = 5 };
 
 constexpr int PG_BM = 256, PG_BN = 256, PG_BK = 64;
 constexpr int PG_STAGE = (PG_BM + PG_BN) * PG_BK * 2;   // 64 KB: A image then B image
@@ -61,17 +61,30 @@ __device__ __forceinline__ float pg_gelu(float v) { return 0.5f * v * (1.f + erf
 
 __device__ __forceinline__ float pg_bfr(float v) { return bf2f(f2bf(v)); }
 
+// Gated epilogues over 8-row interleaved gate / up weights: PG_SWIGLU silu(g) * u, and PG_GLU
+// min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta) with the constants of PgGlu.
+struct PgGlu { float limit = 0.f, alpha = 1.f, beta = 0.f; };
+constexpr bool pg_gated(int epi) { return epi == PG_SWIGLU || epi == PG_GLU; }
+
 // SwiGLU of one 4-value accumulator group (16-row n-tile = 8 gate rows then 8 up rows: lanes
 // g = 0, 1 hold gate columns, lanes g = 2, 3 -- lane ^ 32 -- the matching up columns).  One VALU lane
 // swap (v_permlane32_swap, common.h) of (v[0], v[2]) gives every lane a (gate, up) pair -- element 0
 // in lanes g < 2, element 2 in lanes g >= 2 -- and one of (v[1], v[3]) elements 1 / 3, so every lane
 // computes two outputs (no idle lane half, no LDS-crossbar shuffles) and returns them packed: output
-// columns pg_swiglu_col(g) + {0, 1} of the n-tile's 8.  Same values and rounding as the unfused
+// columns pg_gate_col(g) + {0, 1} of the n-tile's 8.  Same values and rounding as the unfused
 // GEMM -> silu_mul path: bf16 of gate and up, silu(g) * u in fp32.
-__device__ __forceinline__ uint32_t pg_swiglu2(const float (&v)[4]) {
+template <int EPI>
+__device__ __forceinline__ uint32_t pg_gate2(const float (&v)[4], const PgGlu& p) {
   float g0 = v[0], u0 = v[2], g1 = v[1], u1 = v[3];
   swap32(g0, u0);
   swap32(g1, u1);
+  if constexpr (EPI == PG_GLU) {
+    auto glu = [&](float gate, float up) {
+      const float gg = fminf(gate, p.limit), uu = fminf(fmaxf(up, -p.limit), p.limit);
+      return gg * __builtin_amdgcn_rcpf(1.f + __expf(-p.alpha * gg)) * (uu + p.beta);
+    };
+    return pack2bf(glu(g0, u0), glu(g1, u1));
+  }
   auto f = [](float gate, float up) {
     const float gg = pg_bfr(gate);
     return gg * __builtin_amdgcn_rcpf(1.f + __expf(-gg)) * pg_bfr(up);
@@ -79,13 +92,14 @@ __device__ __forceinline__ uint32_t pg_swiglu2(const float (&v)[4]) {
   return pack2bf(f(g0, u0), f(g1, u1));
 }
 
-__device__ __forceinline__ int pg_swiglu_col(int g) { return 4 * (g & 1) + 2 * (g >> 1); }
+__device__ __forceinline__ int pg_gate_col(int g) { return 4 * (g & 1) + 2 * (g >> 1); }
 
 // Epilogue of every kernel here: lane holds rows m = mw + 16 i + (lane & 15), columns
 // n = nw + 16 j + 4 (lane >> 4) + 0..3 of the wave's 128 x 16 NJ block.
 template <int EPI, int NJ>
 __device__ __forceinline__ void pg_epilogue(const f32x4_t (&acc)[8][NJ], const uint16_t* __restrict__ bias,
-                                            uint16_t* __restrict__ out, int M, int N, int ldo, int mw, int nw) {
+                                            uint16_t* __restrict__ out, int M, int N, int ldo, int mw, int nw,
+                                            const PgGlu& gp = PgGlu{}) {
   const int lane = threadIdx.x & 63;
   const int g = lane >> 4;
 #pragma unroll
@@ -96,10 +110,10 @@ __device__ __forceinline__ void pg_epilogue(const f32x4_t (&acc)[8][NJ], const u
       const int nb = nw + j * 16;   // n-tile base
       const int n = nb + 4 * g;
       float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
-      if constexpr (EPI == PG_SWIGLU) {
+      if constexpr (pg_gated(EPI)) {
         // bf16 rounding of g and u as the unfused GEMM -> silu_mul path
-        const uint32_t y = pg_swiglu2(v);
-        if (m < M && nb < N) *reinterpret_cast<uint32_t*>(out + (size_t)m * ldo + nb / 2 + pg_swiglu_col(g)) = y;
+        const uint32_t y = pg_gate2<EPI>(v, gp);
+        if (m < M && nb < N) *reinterpret_cast<uint32_t*>(out + (size_t)m * ldo + nb / 2 + pg_gate_col(g)) = y;
       } else if constexpr (EPI == PG_F32) {
         if (m < M && n < N)
           *reinterpret_cast<float4*>(reinterpret_cast<float*>(out) + (size_t)m * ldo + n) = make_float4(v[0], v[1], v[2], v[3]);
@@ -144,9 +158,9 @@ __device__ __forceinline__ void pg_epilogue_staged(const f32x4_t (&acc)[8][4], u
     for (int j = 0; j < 4; ++j) {
       float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
       if constexpr (EPI == PG_SWIGLU) {
-        // output columns 8 j + pg_swiglu_col(g) .. +1: unit j
+        // output columns 8 j + pg_gate_col(g) .. +1: unit j
         const int unit = j ^ (r & (UPR - 1));
-        *reinterpret_cast<uint32_t*>(region + r * RB + unit * 16 + 2 * pg_swiglu_col(g)) = pg_swiglu2(v);
+        *reinterpret_cast<uint32_t*>(region + r * RB + unit * 16 + 2 * pg_gate_col(g)) = pg_gate2<EPI>(v, PgGlu{});
       } else {
         // columns 16 j + 4 g .. +3: unit 2 j + (g >> 1), half g & 1
         const int unit = (2 * j + (g >> 1)) ^ (r & (UPR - 1));
@@ -689,11 +703,11 @@ __device__ __forceinline__ void ppp_st16(void* p, uint4 v) { *reinterpret_cast<u
 template <int EPI, bool STG = false>
 __global__ void __launch_bounds__(512, 1)
     pgemm_ppp_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, uint16_t* __restrict__ out,
-                     int M, int N, int K, int ldo, int tiles_m, int tiles_n, int wnw, int gm) {
-  static_assert(EPI == PG_BF16 || EPI == PG_SWIGLU, "bf16 / SwiGLU epilogues");
+                     int M, int N, int K, int ldo, int tiles_m, int tiles_n, int wnw, int gm, PgGlu gp) {
+  static_assert(EPI == PG_BF16 || pg_gated(EPI), "bf16 / gated epilogues");
   // epilogue store instructions per wave in the interior (counted in the next tile's first waits):
   // staged bf16 16 x 16 B (128 rows x 128 B), staged SwiGLU 8 x 16 B (128 rows x 64 B), else 32
-  constexpr int PPP_S = STG ? (EPI == PG_SWIGLU ? 8 : 16) : 32;
+  constexpr int PPP_S = STG ? (pg_gated(EPI) ? 8 : 16) : 32;
   __shared__ __attribute__((aligned(16))) char smem[2 * PP_BUF + (STG ? 8 * PPP_REGION : 0)];
   const int lane = threadIdx.x & 63;
   const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -864,17 +878,17 @@ __global__ void __launch_bounds__(512, 1)
         for (int j = 0; j < 4; ++j) {
           const int nb = nw0 + j * 16;
           float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
-          if constexpr (EPI == PG_SWIGLU && !STG) {
-            ppp_st4(out + (size_t)m * ldo + nb / 2 + pg_swiglu_col(g), pg_swiglu2(v));
+          if constexpr (pg_gated(EPI) && !STG) {
+            ppp_st4(out + (size_t)m * ldo + nb / 2 + pg_gate_col(g), pg_gate2<EPI>(v, gp));
           } else if constexpr (!STG) {
             ppp_st8(out + (size_t)m * ldo + nb + 4 * g, make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3])));
           }
         }
       }
-      if constexpr (STG && EPI == PG_SWIGLU) {
+      if constexpr (STG && pg_gated(EPI)) {
         // 2 chunks of 64 rows (m-tiles 4q .. 4q+3): 64-byte rows (32 output columns), 16-byte units
         // XOR-swizzled by the row (4 per row); each lane's two outputs (4 bytes) land at column
-        // 8 j + pg_swiglu_col(g) of the chunk row, read back as whole units, stored as 64-byte row
+        // 8 j + pg_gate_col(g) of the chunk row, read back as whole units, stored as 64-byte row
         // segments (8 x 16 B per wave instead of 32 x 4 B)
         char* region = smem + 2 * PP_BUF + w * PPP_REGION;
         const int rl = lane & 15;
@@ -887,8 +901,8 @@ __global__ void __launch_bounds__(512, 1)
             for (int j = 0; j < 4; ++j) {
               const f32x4_t& a = acc[4 * q + ii][j];
               const float v[4] = {a[0], a[1], a[2], a[3]};
-              *reinterpret_cast<uint32_t*>(region + r * 64 + ((j ^ (r & 3)) << 4) + 2 * pg_swiglu_col(g)) =
-                  pg_swiglu2(v);
+              *reinterpret_cast<uint32_t*>(region + r * 64 + ((j ^ (r & 3)) << 4) + 2 * pg_gate_col(g)) =
+                  pg_gate2<EPI>(v, gp);
             }
           }
           __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -940,7 +954,7 @@ __global__ void __launch_bounds__(512, 1)
       }
       st = true;
     } else {
-      pg_epilogue<EPI>(acc, nullptr, out, M, N, ldo, mw, nw0);
+      pg_epilogue<EPI>(acc, nullptr, out, M, N, ldo, mw, nw0, gp);
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
       st = false;
     }
@@ -1275,12 +1289,12 @@ int ppp_group_m(int tiles_n, int K) { return (K >= 8192 && tiles_n <= 16) ? 4 : 
 
 template <int EPI>
 int ppp_launch(const uint16_t* xp, const uint16_t* wp, uint16_t* op, int M, int N, int K, int ldo, int wnw, int gm,
-               bool stg, hipStream_t stream) {
+               bool stg, hipStream_t stream, const PgGlu& gp = PgGlu{}) {
   const int tm = (M + PG_BM - 1) / PG_BM, tn = (N + PG_BN - 1) / PG_BN;
   if (stg)
-    pgemm_ppp_kernel<EPI, true><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(xp, wp, op, M, N, K, ldo, tm, tn, wnw, gm);
+    pgemm_ppp_kernel<EPI, true><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(xp, wp, op, M, N, K, ldo, tm, tn, wnw, gm, gp);
   else
-    pgemm_ppp_kernel<EPI, false><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(xp, wp, op, M, N, K, ldo, tm, tn, wnw, gm);
+    pgemm_ppp_kernel<EPI, false><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(xp, wp, op, M, N, K, ldo, tm, tn, wnw, gm, gp);
   return (int)hipGetLastError();
 }
 
@@ -1351,6 +1365,21 @@ CFC_API int cfc_pgemm(const void* x, const void* w, const void* bias, void* out,
     case 4: return pgemm_launch_f32(x, w, out, M, N, K, ldo, wnw, stream);
     default: return (int)hipErrorInvalidValue;
   }
+}
+
+// Clamped GLU epilogue over packed, 8-row interleaved gate / up weights on the persistent kernel:
+// out [M, N / 2] (row stride ldo) = min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta).
+CFC_API int cfc_pgemm_glu(const void* x, const void* w, void* out, int M, int N, int K, int ldo, int wnw, float limit,
+                          float alpha, float beta, hipStream_t stream) {
+  if (M < 1 || N < 64 || K < 2 * PG_BK || K % 64 || N % 64 || ldo % 8 || ldo < N / 2 || ((uintptr_t)out & 15) || wnw < 1 ||
+      N % (16 * wnw) || (uint64_t)M * K * 2 >= (1ull << 32) || (uint64_t)N * K * 2 >= (1ull << 32))
+    return (int)hipErrorInvalidValue;
+  const int tm = (M + PG_BM - 1) / PG_BM, tn = (N + PG_BN - 1) / PG_BN;
+  PgGlu gp;
+  gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
+  pgemm_ppp_kernel<PG_GLU, true><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(
+      (const uint16_t*)x, (const uint16_t*)w, (uint16_t*)out, M, N, K, ldo, tm, tn, wnw, ppp_group_m(tn, K), gp);
+  return (int)hipGetLastError();
 }
 
 // Timing probe only (scripts/bench_pgemm.py --probe): the ping-pong kernel, bf16 epilogue, packed W

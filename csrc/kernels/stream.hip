@@ -86,15 +86,15 @@ struct DepthArgs {
   int T, W, split, n;
   float eps;
   // DN_CONV
-  const float* w1; const float* w2;   // [W][taps]; w2 null: one sublayer
+  const float* w1; const float* w2;   // [taps][W]; w2 null: one sublayer
   const int32_t* positions;
   TailArg tail;
   int taps, ld1_, ld2_;
 };
 
-// one workgroup per row; a thread holds NV vectors of V channels, NV * V * 256 >= W
-template <typename ACT, int V, int NV, int MODE>
-__global__ void __launch_bounds__(256) depth_norm_kernel(DepthArgs a, ACT* __restrict__ h1, ACT* __restrict__ h2) {
+// one workgroup of BT threads per row; a thread holds NV vectors of V channels, NV * V * BT >= W
+template <typename ACT, int V, int NV, int MODE, int BT>
+__global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __restrict__ h1, ACT* __restrict__ h2) {
   __shared__ float red[16];
   const int b = blockIdx.x, t = a.rows ? a.rows[b] : b;
   const size_t row = (size_t)t * a.W, plane = (size_t)a.T * a.W;
@@ -102,16 +102,21 @@ __global__ void __launch_bounds__(256) depth_norm_kernel(DepthArgs a, ACT* __res
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
-    const int c = (k * 256 + threadIdx.x) * V;
+    const int c = (k * BT + threadIdx.x) * V;
 #pragma unroll
     for (int e = 0; e < V; ++e) x[k].v[e] = 0.f;
     if (c >= a.W) continue;
     Vec<V> cur = ldv<V>(a.x_in + row + c);
     if (a.part) {
-      for (int p = 0; p < a.split; ++p) {
-        const Vec<V> y = ldv<V>(a.part + (size_t)p * plane + row + c);
+      for (int p0 = 0; p0 < a.split; p0 += 4) {      // four slabs in flight (past the last: re-read, not added)
+        Vec<V> y[4];
 #pragma unroll
-        for (int e = 0; e < V; ++e) cur.v[e] += y.v[e];
+        for (int u = 0; u < 4; ++u) y[u] = ldv<V>(a.part + (size_t)min(p0 + u, a.split - 1) * plane + row + c);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (p0 + u < a.split)
+#pragma unroll
+            for (int e = 0; e < V; ++e) cur.v[e] += y[u].v[e];
       }
       if (a.bias) {
         const Vec<V> y = ldv<V>(a.bias + c);
@@ -123,20 +128,16 @@ __global__ void __launch_bounds__(256) depth_norm_kernel(DepthArgs a, ACT* __res
       const float an = a.dwa[a.n];
 #pragma unroll
       for (int e = 0; e < V; ++e) acc.v[e] = an * cur.v[e];
-      int j = 0;
-      for (; j + 4 <= a.n; j += 4) {     // four rows of the history in flight
-        Vec<V> y[4];
+      for (int j = 0; j < a.n; j += 8) {     // eight rows of the history in flight
+        Vec<V> y[8];
 #pragma unroll
-        for (int u = 0; u < 4; ++u) y[u] = ldv<V>(a.hist + (size_t)(j + u) * plane + row + c);
+        for (int u = 0; u < 8; ++u) y[u] = ldv<V>(a.hist + (size_t)min(j + u, a.n - 1) * plane + row + c);
 #pragma unroll
-        for (int u = 0; u < 4; ++u)
+        for (int u = 0; u < 8; ++u) {
+          const float wj = j + u < a.n ? a.dwa[j + u] : 0.f;
 #pragma unroll
-          for (int e = 0; e < V; ++e) acc.v[e] += a.dwa[j + u] * y[u].v[e];
-      }
-      for (; j < a.n; ++j) {
-        const Vec<V> y = ldv<V>(a.hist + (size_t)j * plane + row + c);
-#pragma unroll
-        for (int e = 0; e < V; ++e) acc.v[e] += a.dwa[j] * y.v[e];
+          for (int e = 0; e < V; ++e) acc.v[e] += wj * y[u].v[e];
+        }
       }
       cur = acc;
     }
@@ -153,7 +154,7 @@ __global__ void __launch_bounds__(256) depth_norm_kernel(DepthArgs a, ACT* __res
     const int pos = MODE == DN_CONV ? a.positions[b] : 0;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
-      const int c = (k * 256 + threadIdx.x) * V;
+      const int c = (k * BT + threadIdx.x) * V;
       if (c >= a.W) continue;
       const Vec<V> g = ldv<V>(a.norm_w + c);
       Vec<V> h;
@@ -167,10 +168,13 @@ __global__ void __launch_bounds__(256) depth_norm_kernel(DepthArgs a, ACT* __res
           const int q = pos - a.taps + 1 + j;
           if (q < 0) continue;
           const Vec<V> s = j == a.taps - 1 ? h : ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+          const Vec<V> k1 = ldv<V>(a.w1 + (size_t)j * a.W + c);
 #pragma unroll
-          for (int e = 0; e < V; ++e) {
-            y1.v[e] += a.w1[(size_t)(c + e) * a.taps + j] * s.v[e];
-            if (a.w2) y2.v[e] += a.w2[(size_t)(c + e) * a.taps + j] * s.v[e];
+          for (int e = 0; e < V; ++e) y1.v[e] += k1.v[e] * s.v[e];
+          if (a.w2) {
+            const Vec<V> k2 = ldv<V>(a.w2 + (size_t)j * a.W + c);
+#pragma unroll
+            for (int e = 0; e < V; ++e) y2.v[e] += k2.v[e] * s.v[e];
           }
         }
         if (a.taps > 1) stv<V>(tail_row(a.tail, b, pos, a.W) + c, h);
@@ -227,8 +231,8 @@ __global__ void __launch_bounds__(256) input_conv_kernel(const float* __restrict
     for (int j = 0; j < TAPS; ++j)
 #pragma unroll
       for (int e = 0; e < V; ++e) {
-        k1[j][e] = w1[(size_t)(c + e) * TAPS + j];
-        k2[j][e] = w2 ? w2[(size_t)(c + e) * TAPS + j] : 0.f;
+        k1[j][e] = w1[(size_t)j * W + c + e];
+        k2[j][e] = w2 ? w2[(size_t)j * W + c + e] : 0.f;
       }
     Vec<V> win[TAPS];
 #pragma unroll
@@ -255,8 +259,8 @@ __global__ void __launch_bounds__(256) input_conv_kernel(const float* __restrict
         const Vec<V> s = j == taps - 1 ? h : input(r - taps + 1 + j);
 #pragma unroll
         for (int e = 0; e < V; ++e) {
-          y1.v[e] += w1[(size_t)(c + e) * taps + j] * s.v[e];
-          if (w2) y2.v[e] += w2[(size_t)(c + e) * taps + j] * s.v[e];
+          y1.v[e] += w1[(size_t)j * W + c + e] * s.v[e];
+          if (w2) y2.v[e] += w2[(size_t)j * W + c + e] * s.v[e];
         }
       }
       put(r, h, y1, y2);
@@ -277,16 +281,22 @@ __device__ __forceinline__ float glu<float>(float g, float u, float limit, float
   return g / (1.f + expf(-alpha * g)) * (u + beta);
 }
 
-// gu [T][2F] (ACT or fp32): gate | up halves, or 8-column interleaved groups
+// gu [split][T][2F] (ACT, or fp32 slabs whose sum is the product): gate | up halves, or 8-column
+// interleaved groups
 template <typename ACT, typename IN>
 __global__ void __launch_bounds__(256) clamped_glu_kernel(ACT* __restrict__ out, int ldo, const IN* __restrict__ gu,
                                                          const float* __restrict__ gb, const float* __restrict__ ub,
-                                                         int F, int interleaved, float limit, float alpha, float beta) {
+                                                         int F, int interleaved, float limit, float alpha, float beta, int split,
+                                                         size_t slab) {
   const int t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
   if (c >= F) return;
   const IN* r = gu + (size_t)t * 2 * F;
   const int gc = interleaved ? 16 * (c >> 3) + (c & 7) : c, uc = interleaved ? gc + 8 : F + c;
-  const float g = ld1(r + gc) + (gb ? gb[c] : 0.f), u = ld1(r + uc) + (ub ? ub[c] : 0.f);
+  float g = gb ? gb[c] : 0.f, u = ub ? ub[c] : 0.f;
+  for (int p = 0; p < split; ++p) {
+    g += ld1(r + p * slab + gc);
+    u += ld1(r + p * slab + uc);
+  }
   st1(out + (size_t)t * ldo + c, glu<ACT>(g, u, limit, alpha, beta));
 }
 
@@ -295,14 +305,19 @@ __global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ x, siz
   for (size_t i = blockIdx.x * (size_t)256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) x[i] = cap * tanhf(x[i] * inv);
 }
 
+// few rows (a decode step): the widest workgroup the row fills, one vector per thread
 template <typename ACT, int V, int MODE>
-int depth_nv(int nv, dim3 grid, hipStream_t s, const DepthArgs& a, void* h1, void* h2) {
-#define DN_GO(NV) depth_norm_kernel<ACT, V, NV, MODE><<<grid, 256, 0, s>>>(a, (ACT*)h1, (ACT*)h2)
-  if (nv <= 1) DN_GO(1);
-  else if (nv <= 2) DN_GO(2);
-  else if (nv <= 4) DN_GO(4);
-  else if (nv <= 8) DN_GO(8);
-  else if (nv <= 16) DN_GO(16);
+int depth_nv(int W, dim3 grid, hipStream_t s, const DepthArgs& a, void* h1, void* h2) {
+#define DN_GO(NV, BT) depth_norm_kernel<ACT, V, NV, MODE, BT><<<grid, BT, 0, s>>>(a, (ACT*)h1, (ACT*)h2)
+  const int vecs = (W + V - 1) / V;
+  const bool few = grid.x <= 512 && vecs > 256;
+  if (vecs <= 256) DN_GO(1, 256);
+  else if (few && vecs <= 1024) DN_GO(1, 1024);
+  else if (few && vecs <= 2048) DN_GO(2, 1024);
+  else if (vecs <= 512) DN_GO(2, 256);
+  else if (vecs <= 1024) DN_GO(4, 256);
+  else if (vecs <= 4096) DN_GO(4, 1024);
+  else if (vecs <= 8192) DN_GO(8, 1024);
   else return -4;
 #undef DN_GO
   return CFC_CHECK_LAUNCH();
@@ -313,8 +328,7 @@ int depth_launch(int mode, int nrows, hipStream_t s, const DepthArgs& a, void* h
   const bool v4 = a.W % 4 == 0 && (mode == DN_RSTD || (a.ld1_ % 4 == 0 && (!a.w2 || a.ld2_ % 4 == 0)));
   const dim3 grid(nrows);
 #define DN_MODE(M)                                                                             \
-  return v4 ? depth_nv<ACT, 4, M>((a.W + 1023) / 1024, grid, s, a, h1, h2)                      \
-            : depth_nv<ACT, 1, M>((a.W + 255) / 256, grid, s, a, h1, h2)
+  return v4 ? depth_nv<ACT, 4, M>(a.W, grid, s, a, h1, h2) : depth_nv<ACT, 1, M>(a.W, grid, s, a, h1, h2)
   switch (mode) {
     case DN_RSTD: DN_MODE(DN_RSTD);
     case DN_NORM: DN_MODE(DN_NORM);
@@ -391,24 +405,24 @@ CFC_API int cfc_input_conv(int f32, int n_tiles, const int32_t* tiles, const flo
 }
 
 // in_f32: gu is fp32 (else the activation type)
-CFC_API int cfc_clamped_glu(int f32, int in_f32, void* out, int ldo, const void* gu, const float* gb, const float* ub, int T,
-                            int F, int interleaved, float limit, float alpha, float beta, hipStream_t stream) {
+CFC_API int cfc_clamped_glu(int f32, int in_f32, void* out, int ldo, const void* gu, int split, const float* gb,
+                            const float* ub, int T, int F, int interleaved, float limit, float alpha, float beta, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (F <= 0 || (interleaved && F % 8) || T > 65535 * 16) return -1;
+  if (F <= 0 || (interleaved && F % 8) || split < 1 || (split > 1 && !f32 && !in_f32) || T > 65535 * 16) return -1;
   const int rows = T > 65535 ? 65535 : T;
   for (int t0 = 0; t0 < T; t0 += rows) {
     const int n = T - t0 < rows ? T - t0 : rows;
     const dim3 grid((F + 255) / 256, n);
-    const size_t go = (size_t)t0 * 2 * F, oo = (size_t)t0 * ldo;
+    const size_t slab = (size_t)T * 2 * F, go = (size_t)t0 * 2 * F, oo = (size_t)t0 * ldo;
     if (f32)
       clamped_glu_kernel<float, float><<<grid, 256, 0, stream>>>((float*)out + oo, ldo, (const float*)gu + go, gb, ub, F,
-                                                                 interleaved, limit, alpha, beta);
+                                                                 interleaved, limit, alpha, beta, split, slab);
     else if (in_f32)
       clamped_glu_kernel<uint16_t, float><<<grid, 256, 0, stream>>>((uint16_t*)out + oo, ldo, (const float*)gu + go, gb, ub,
-                                                                    F, interleaved, limit, alpha, beta);
+                                                                    F, interleaved, limit, alpha, beta, split, slab);
     else
       clamped_glu_kernel<uint16_t, uint16_t><<<grid, 256, 0, stream>>>((uint16_t*)out + oo, ldo, (const uint16_t*)gu + go,
-                                                                       gb, ub, F, interleaved, limit, alpha, beta);
+                                                                       gb, ub, F, interleaved, limit, alpha, beta, split, slab);
   }
   return CFC_CHECK_LAUNCH();
 }

@@ -23,6 +23,7 @@ EXPECTED = {
     ("0", "1"): {"global_store_dwordx4": 16, "global_store_dwordx2": 32, "global_store_dword": 0},   # bf16, staged
     ("0", "0"): {"global_store_dwordx4": 0, "global_store_dwordx2": 64, "global_store_dword": 0},    # bf16, direct
     ("3", "1"): {"global_store_dwordx4": 8, "global_store_dwordx2": 0, "global_store_dword": 32},    # SwiGLU, staged
+    ("5", "1"): {"global_store_dwordx4": 8, "global_store_dwordx2": 0, "global_store_dword": 32},    # clamped GLU, staged
     ("3", "0"): {"global_store_dwordx4": 0, "global_store_dwordx2": 0, "global_store_dword": 64},    # SwiGLU, direct
 }
 
