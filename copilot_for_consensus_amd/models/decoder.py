@@ -507,9 +507,14 @@ class DecoderModel:
         return PagedKVCache(self.cfg.layers, num_blocks, self.w.kv_heads, self.cfg.head_dim, device or self.w.device,
                             dtype=dtype or torch.bfloat16)
 
-    def decode_groups(self) -> int:
-        """Attention workgroups per sequence and KV partition of a decode step."""
-        return self.w.kv_heads
+    def decode_partitions(self, B: int, max_blocks: int) -> int:
+        """KV partitions per sequence of a B-row decode step: the smallest P giving >= CFC_DECODE_WGS
+        workgroups (default 512, two per CU).  Long KV runs per workgroup win: at B=128 P=1 streams
+        6.5 TB/s vs 5.0-5.4 for fixed 26-block partitions (scripts/bench_decode_attn.py,
+        profiles/decode_attn_partitions_r01.log)."""
+        target = int(os.environ.get("CFC_DECODE_WGS", "512"))
+        P = max(1, math.ceil(target / max(1, B * self.w.kv_heads)))
+        return min(P, max(1, max_blocks // 2))
 
     def decode_workspace(self, B: int, P: int) -> int:
         """fp32 elements of the split-KV partials of a B-row decode step over P partitions."""

@@ -30,7 +30,7 @@ import torch
 from ..ops import kernels as K
 from ..ops import latent as L
 from ..ops import stream as S
-from ..ops.reference import interleave_gate_up, tail_slots
+from ..ops.reference import KV_BLOCK, interleave_gate_up, tail_slots
 from ..runtime.kv_cache import LatentKVCache
 from .decoder import argmax_keys
 from .projection import Projection
@@ -315,9 +315,11 @@ class VofosunModel:
         return LatentKVCache([s.mixer.kv_rank for s in self.cfg.specs], num_blocks, self.cfg.hidden, tail_slots(self.cfg.taps),
                              device or self.w.device, self.w.dtype)
 
-    def decode_groups(self) -> int:
-        """Attention workgroups per sequence and key slice of a decode step."""
-        return min(math.ceil(lw["H"] / self._rows(i, True)) for i, lw in enumerate(self.w.layers))
+    def decode_partitions(self, B: int, max_blocks: int) -> int:
+        """Key slices per sequence of a B-row decode step over block tables ``max_blocks`` wide."""
+        if self.w.dtype != torch.bfloat16:
+            return max(1, min(math.ceil(512 / B), max_blocks // 8))
+        return max(L.decode_plan(B, lw["H"], self._rs(i), max_blocks * KV_BLOCK)[1] for i, lw in enumerate(self.w.layers))
 
     def decode_workspace(self, B: int, P: int) -> int:
         return max(B * lw["H"] * P * (self._rs(i) + 2) for i, lw in enumerate(self.w.layers)) if P > 1 else 1
@@ -325,17 +327,19 @@ class VofosunModel:
     def _rs(self, i: int) -> int:
         return L.padded_rank(self.cfg.specs[i].mixer.kv_rank)
 
-    def _rows(self, i: int, decode: bool) -> int:
-        return L.rows_per_tile(self.w.dtype, self._rs(i), self.w.layers[i]["H"], decode)
+    def _rows(self, i: int, decode: tuple | None = None) -> int:
+        """Rows per attention work item of layer i; ``decode``: (B, key slices, context bound) of a decode step."""
+        rs, H = self._rs(i), self.w.layers[i]["H"]
+        return L.rows_per_tile(self.w.dtype, rs, L.decode_plan(decode[0], H, rs, decode[2], decode[1]) if decode else None)
 
     def plan_prefill(self, cu, ctx, slots) -> dict:
         """Host-side launch plan of a packed pass over portions cu / ctx: int32 arrays for the device."""
         por = [(cu[s], cu[s + 1] - cu[s], ctx[s] - (cu[s + 1] - cu[s]), s) for s in range(len(ctx))]
         plan = {"conv_tiles": S.conv_tiles(por)}
         for i, lw in enumerate(self.w.layers):
-            key = f"attn_{lw['H']}_{self._rows(i, False)}"
+            key = f"attn_{lw['H']}_{self._rows(i)}"
             if key not in plan:
-                plan[key] = np.asarray(L.attn_tiles(cu, lw["H"], self._rows(i, False), ctx), np.int32).reshape(2, -1)
+                plan[key] = np.asarray(L.attn_tiles(cu, lw["H"], self._rows(i), ctx), np.int32).reshape(2, -1)
         plan["max_ctx"] = max(ctx)
         for i, lw in enumerate(self.w.layers):
             rs = self._rs(i)
@@ -375,7 +379,7 @@ class VofosunModel:
             cur = x
             hs = self._inputs(T, lw, ids.device, bufs)
             S.input_conv(x, rstd, lw["norm"], lw["convs"], plan["conv_tiles"], S.Tail(kv.tails[i], block_tables), hs)
-            rows = self._rows(i, False)
+            rows = self._rows(i)
             tiles = plan[f"attn_{lw['H']}_{rows}"]
             attn = dict(cu_q=cu_q, tiles=(tiles[0], tiles[1]), rows=rows,
                         P=L.partitions(tiles.shape[1], plan["max_ctx"]))
@@ -389,6 +393,7 @@ class VofosunModel:
         """One token per sequence.  Returns the final-normed hidden states [B, W].  ``part_blocks``: -P, P key
         slices per sequence (the engine's form); ``shared_blocks`` is not used (latents are read once per
         token for all heads, through the caches)."""
+        P = max(1, -part_blocks)
         hist, x = self._embed(ids)
         cur, up, bufs = hist[0], None, {}
         for i, lw in enumerate(self.w.layers):
@@ -396,7 +401,8 @@ class VofosunModel:
             S.depth_conv_decode(cur, hist, up, lw["norm"], self.cfg.norm_eps, lw["convs"], positions,
                                 S.Tail(kv.tails[i], block_tables), x, hs)
             cur = x
-            attn = dict(cu_q=None, rows=self._rows(i, True), P=max(1, -part_blocks), workspace=attn_workspace)
+            attn = dict(cu_q=None, rows=self._rows(i, (ids.numel(), P, block_tables.shape[1] * KV_BLOCK)), P=P,
+                        workspace=attn_workspace)
             up = self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn)
         return S.depth_norm(cur, hist, up, self.w.final_norm, self.cfg.norm_eps, self.w.dtype)
 

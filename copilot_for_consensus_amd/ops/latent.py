@@ -75,13 +75,38 @@ def latent_norm(part, nq: int, wq, wc, eps: float, slots, cache, dtype) -> torch
     return out
 
 
-def rows_per_tile(dtype, RS: int, heads: int, decode: bool) -> int:
+def rows_per_tile(dtype, RS: int, decode_plan: tuple | None = None) -> int:
     """(token, head) rows of one attention work item: the general kernel's 4, or 16 / 32 / 64 on MFMA."""
     if dtype != torch.bfloat16 or RS > MFMA_MAX_RANK:
         return ANY_ROWS
-    if not decode:
-        return 64
-    return 16 if heads <= 16 else (32 if heads <= 32 else 64)
+    return decode_plan[0] if decode_plan else 64
+
+
+MAX_PARTITIONS = 256
+_TILE_US = {16: 1.7, 32: 2.1, 64: 3.9}     # one 64-key tile at rank 512, by rows per work item (one workgroup alone)
+
+
+def decode_plan(B: int, heads: int, RS: int, max_ctx: int, P: int | None = None) -> tuple[int, int]:
+    """(rows per work item, key slices) of a decode step, from the time of its longest workgroup plus the
+    slices' partials (written and merged in fp32) against the time to stream the latents, which
+    workgroups of one sequence each read: measured per-tile times, one MI355X (64-key tiles)."""
+    scale = max(0.35, RS / 512)
+    per_cu = max(1, min(4, (160 * 1024) // (2 * 64 * 64 * math.ceil(RS / 64) * 2 + 12 * 1024)))
+    nt, best = max(1, math.ceil(max_ctx / 64)), None
+    cand = [P] if P else sorted({p for p in (1, 2, 3, 4, 5, 6, 8, 10, 12, 16, 20, 24, 32, 48, 64, 96, 128) if p <= nt})
+    for rows in (16, 32, 64):
+        if rows > 16 and rows >= 2 * heads:
+            continue
+        g = math.ceil(heads / rows)
+        for p in cand:
+            rounds = math.ceil(B * g * p / (256 * per_cu))
+            t = max(rounds * (4 + math.ceil(nt / p) * _TILE_US[rows] * scale * min(per_cu, math.ceil(B * g * p / 256))),
+                    B * max_ctx * RS * 2 * g / 7e6)
+            if p > 1:
+                t += 5 + 2 * B * heads * p * RS * 4 / 5e6
+            if best is None or t < best[0]:
+                best = (t, rows, p)
+    return best[1], best[2]
 
 
 def attn_tiles(cu_q, heads: int, rows: int, ctx_lens=None):
@@ -100,7 +125,7 @@ def attn_tiles(cu_q, heads: int, rows: int, ctx_lens=None):
 
 def partitions(n_tiles: int, max_ctx: int, target: int = 512) -> int:
     """Key slices per work item: enough workgroups to fill the chip, at least four 64-key tiles each."""
-    return max(1, min(math.ceil(target / max(1, n_tiles)), math.ceil(max_ctx / 256)))
+    return max(1, min(math.ceil(target / max(1, n_tiles)), math.ceil(max_ctx / 256), MAX_PARTITIONS))
 
 
 def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles=None, rows: int | None = None,
@@ -117,7 +142,7 @@ def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles
         raise ValueError(f"latent_attention: q {tuple(q.shape)} {q.dtype}, cache {tuple(cache.shape)} {cache.dtype}")
     for name, t in (("block_tables", block_tables), ("ctx_lens", ctx_lens)):
         _req(t, torch.int32, name)
-    rows = rows or rows_per_tile(q.dtype, RS, H, cu_q is None)
+    rows = rows or rows_per_tile(q.dtype, RS, decode_plan(B, H, RS, 64, P) if cu_q is None else None)
     if cu_q is None:
         if T != B:
             raise ValueError(f"latent_attention: {T} rows for {B} sequences")

@@ -148,12 +148,8 @@ class LLMEngine:
     # ------------------------------------------------------------------ helpers
     def _part_blocks(self, B, max_blocks):
         """Split-KV partitioning of the decode attention, as ``-P``: each sequence's own blocks in
-        P balanced ranges, P the smallest giving >= CFC_DECODE_WGS workgroups (default 512, two per
-        CU).  Long KV runs per workgroup win: at B=128 P=1 streams 6.5 TB/s vs 5.0-5.4 for fixed
-        26-block partitions (scripts/bench_decode_attn.py, profiles/decode_attn_partitions_r01.log)."""
-        target = int(os.environ.get("CFC_DECODE_WGS", "512"))
-        P = max(1, math.ceil(target / max(1, B * self.model.decode_groups())))
-        return -min(P, max(1, max_blocks // 2))
+        P balanced ranges, P the model's pick (DecoderModel.decode_partitions)."""
+        return -self.model.decode_partitions(B, max_blocks)
 
     def _i32(self, x):
         return torch.tensor(x, dtype=torch.int32, device=self.device)

@@ -174,6 +174,13 @@ __device__ __forceinline__ LatTile lat_tile(const LatArgs& a, int tile, int p, i
   return r;
 }
 
+// workgroup barrier that orders LDS only (__syncthreads also waits for every global load issued before it)
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 constexpr int LP = 72;      // P row stride in LDS, elements (64 keys + 8 against bank conflicts)
 
 // Eight waves, a 64-key x R64 tile of latents double-buffered in LDS (row-major, 16-byte chunks
@@ -183,8 +190,9 @@ constexpr int LP = 72;      // P row stride in LDS, elements (64 keys + 8 agains
 //   softmax  per row across the lane groups by lane swaps, across the waves of a row group through LDS
 //   output   O^T += C^T P^T: wave w owns latent columns 16 (w + 8 j) of every row; the C^T fragments
 //            are transposing LDS reads (ds_read_b64_tr_b16) of the same tile, P^T comes from LDS
-// Two barriers per tile; the next tile's global loads are issued first and stored to the other buffer
-// between them, when no wave can still be reading it.
+// Two barriers per tile.  Between them, when no wave can still be reading the other buffer, the next tile
+// is stored to it from registers and the loads of the one after are issued; the barriers order LDS only, so
+// those loads stay in flight across a whole tile.
 template <int R64, int MR>
 __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __restrict__ q,
                                                             const uint16_t* __restrict__ cache, LatArgs a,
@@ -205,7 +213,8 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
 
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int col = lane & 15, kq = lane >> 4;
-  const LatTile tl = lat_tile(a, blockIdx.x, blockIdx.y, 16 * MR);
+  // one XCD takes neighbouring tiles: a sequence's tiles read the same latents through one L2
+  const LatTile tl = lat_tile(a, a.P == 1 ? xcd_remap(blockIdx.x, gridDim.x) : blockIdx.x, blockIdx.y, 16 * MR);
   const int RS = a.RS;
 
   // score role: row group and key groups of this wave (MR = 1: waves 4-7 have none)
@@ -250,13 +259,12 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
   if (tl.kt0 < tl.kt1) {
     gload(tl.kt0);
     lwrite(0);
+    if (tl.kt0 + 1 < tl.kt1) gload(tl.kt0 + 1);
   }
   __syncthreads();
   for (int kt = tl.kt0; kt < tl.kt1; ++kt) {
     const int cur = (kt - tl.kt0) & 1;
     const char* kb = kbuf + cur * (64 * R64 * 2);
-    const bool more = kt + 1 < tl.kt1;
-    if (more) gload(kt + 1);
     f32x4_t s[KG];
     if (scorer) {
       float mx = -INFINITY;
@@ -281,7 +289,7 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
       mx = xor32_max(xor16_max(mx));
       if (lane < 16) smax[(rg * 4 + slot) * 16 + lane] = mx;
     }
-    __syncthreads();
+    lds_barrier();
     if (scorer) {
       float mn = m;
 #pragma unroll
@@ -303,8 +311,11 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
       }
       if (slot == 0 && lane < 16) salpha[16 * rg + lane] = alpha;
     }
-    if (more) lwrite(cur ^ 1);
-    __syncthreads();
+    if (kt + 1 < tl.kt1) {
+      lwrite(cur ^ 1);
+      if (kt + 2 < tl.kt1) gload(kt + 2);      // in flight for a whole tile
+    }
+    lds_barrier();
     uint4 pf[2][MR];
 #pragma unroll
     for (int r = 0; r < MR; ++r) {
@@ -474,25 +485,52 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __re
   }
 }
 
-// one workgroup of 128 threads per (token, head) row
+// one workgroup of 128 threads per (token, head) row; P <= LC_MAXP
+constexpr int LC_MAXP = 256;
 template <typename ACT>
 __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __restrict__ part_o,
                                                             const float* __restrict__ part_ml, int P, int RS,
                                                             ACT* __restrict__ out) {
+  __shared__ float wt[LC_MAXP];
   const size_t row = blockIdx.x;
   const float* ml = part_ml + row * P * 2;
-  float m = -INFINITY;
-  for (int p = 0; p < P; ++p) m = fmaxf(m, ml[2 * p]);
-  const float ref = m == -INFINITY ? 0.f : m;
-  float l = 0.f;
-  for (int p = 0; p < P; ++p) l += ml[2 * p + 1] * exp2f(ml[2 * p] - ref);
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  // every wave computes the weights (at most four slices per lane), the first stores them
+  const int lane = threadIdx.x & 63;
+  float m[LC_MAXP / 64], l[LC_MAXP / 64], mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < LC_MAXP / 64; ++i) {
+    const int p = lane + 64 * i;
+    m[i] = p < P ? ml[2 * p] : -INFINITY;
+    l[i] = p < P ? ml[2 * p + 1] : 0.f;
+    mx = fmaxf(mx, m[i]);
+  }
+  mx = wave_max(mx);
+  const float ref = mx == -INFINITY ? 0.f : mx;
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < LC_MAXP / 64; ++i) {
+    m[i] = exp2f(m[i] - ref);
+    sum += m[i] * l[i];
+  }
+  sum = wave_sum(sum);
+  const float inv = sum > 0.f ? 1.f / sum : 0.f;
+  if (threadIdx.x < 64) {
+#pragma unroll
+    for (int i = 0; i < LC_MAXP / 64; ++i)
+      if (lane + 64 * i < P) wt[lane + 64 * i] = m[i] * inv;
+  }
+  __syncthreads();
   for (int c = threadIdx.x * 4; c < RS; c += 512) {
     float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
-    for (int p = 0; p < P; ++p) {
-      const float e = exp2f(ml[2 * p] - ref) * inv;
-      const float4 v = *reinterpret_cast<const float4*>(part_o + (row * P + p) * RS + c);
-      s.x += e * v.x; s.y += e * v.y; s.z += e * v.z; s.w += e * v.w;
+    for (int p0 = 0; p0 < P; p0 += 8) {          // eight slices in flight (past the last: re-read, weight 0)
+      float4 v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const float4*>(part_o + (row * P + min(p0 + u, P - 1)) * RS + c);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const float e = p0 + u < P ? wt[p0 + u] : 0.f;
+        s.x += e * v[u].x; s.y += e * v[u].y; s.z += e * v[u].z; s.w += e * v[u].w;
+      }
     }
     ACT* o = out + row * RS + c;
     stf(o, s.x); stf(o + 1, s.y); stf(o + 2, s.z); stf(o + 3, s.w);
@@ -570,7 +608,7 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
                                  int max_blocks, float scale, int P, int total_rows, float* part_o, float* part_ml,
                                  void* out, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (H < 1 || RS < 32 || RS % 32 || P < 1 || P > 65535 || max_blocks < 1) return -1;
+  if (H < 1 || RS < 32 || RS % 32 || P < 1 || P > LC_MAXP || max_blocks < 1) return -1;
   if ((tile_seq == nullptr) != (tile_m0 == nullptr) || (!tile_seq && tiles_per_seq < 1)) return -1;
   if (P > 1 && (!part_o || !part_ml)) return -2;
   LatArgs a{block_tables, cu_q, ctx_lens, tile_seq, tile_m0, tiles_per_seq, H, RS, max_blocks, P,
