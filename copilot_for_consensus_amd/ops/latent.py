@@ -196,7 +196,7 @@ def expand(cache, block_tables, ctx_lens, tiles, uk, uv):
     # the values' rows are read side by side: an odd number of 128-byte lines apart, not a power of two
     ldv = n * 64 + (64 if n % 2 == 0 else 128)
     vt = torch.empty(uv.shape[0], ldv, dtype=cache.dtype, device=cache.device)[:, :n * 64]
-    K.pgemm(uv, rows[1], out=vt, variant="pp")
+    K.pgemm(uv, K.PackedWeight(rows[1].view(-1), n * 64, RS, 64), out=vt, variant="ppp")
     return k, vt
 
 

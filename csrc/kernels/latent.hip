@@ -27,33 +27,88 @@ __device__ __forceinline__ void stf(uint16_t* p, float v) { *p = f2bf(v); }
 __device__ __forceinline__ void stf(float* p, float v) { *p = v; }
 
 // ---------------------------------------------------------------------------------- latent_norm
-// part: fp32 slabs [split][T][NQ + NC] of the joint projection (query latent | cached latent).
-// One workgroup per row; the row's sums are kept in LDS.
-template <typename ACT>
-__global__ void __launch_bounds__(256) latent_norm_kernel(const float* __restrict__ part, int split, int T, int NQ, int NC,
-                                                         const float* __restrict__ wq, const float* __restrict__ wc,
-                                                         float eps, const int32_t* __restrict__ slots,
-                                                         ACT* __restrict__ q_out, int ldq, ACT* __restrict__ cache,
-                                                         int RS) {
-  extern __shared__ float row[];
+// part: fp32 slabs [split][T][NQ + NC] of the joint projection (query latent | cached latent).  One
+// workgroup per row, a thread holds up to NV vectors of V columns (V divides NQ).
+template <typename ACT, int V>
+__device__ __forceinline__ void st_vec(ACT* p, const float* v) {
+  if constexpr (V == 1) stf(p, v[0]);
+  else if constexpr (sizeof(ACT) == 2) *reinterpret_cast<uint2*>(p) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
+  else *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+
+template <typename ACT, int V, int NV, int BT>
+__global__ void __launch_bounds__(BT) latent_norm_kernel(const float* __restrict__ part, int split, int T, int NQ, int NC,
+                                                        const float* __restrict__ wq, const float* __restrict__ wc,
+                                                        float eps, const int32_t* __restrict__ slots,
+                                                        ACT* __restrict__ q_out, int ldq, ACT* __restrict__ cache, int RS) {
   __shared__ float red[16];
   const int t = blockIdx.x, N = NQ + NC;
-  float sq = 0.f, sc = 0.f;
-  for (int c = threadIdx.x; c < N; c += 256) {
-    float v = 0.f;
-    for (int p = 0; p < split; ++p) v += part[((size_t)p * T + t) * N + c];
-    row[c] = v;
-    if (c < NQ) sq += v * v;
-    else sc += v * v;
+  const size_t plane = (size_t)T * N;
+  const float* src = part + (size_t)t * N;
+  const int slot = slots[t];
+  float x[NV][V], sq = 0.f, sc = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = (k * BT + threadIdx.x) * V;
+#pragma unroll
+    for (int e = 0; e < V; ++e) x[k][e] = 0.f;
+    if (c >= N) continue;
+    for (int p0 = 0; p0 < split; p0 += 8) {       // eight slabs in flight (past the last: re-read, not added)
+      float y[8][V];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const float* s = src + (size_t)min(p0 + u, split - 1) * plane + c;
+        if constexpr (V == 4) {
+          const float4 f = *reinterpret_cast<const float4*>(s);
+          y[u][0] = f.x; y[u][1] = f.y; y[u][2] = f.z; y[u][3] = f.w;
+        } else {
+          y[u][0] = *s;
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
+        if (p0 + u < split)
+#pragma unroll
+          for (int e = 0; e < V; ++e) x[k][e] += y[u][e];
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss += x[k][e] * x[k][e];
+    if (c < NQ) sq += ss;
+    else sc += ss;
   }
   sq = block_sum(sq, red);
   sc = block_sum(sc, red);
   const float rq = 1.f / sqrtf(sq / (float)NQ + eps), rc = 1.f / sqrtf(sc / (float)NC + eps);
-  ACT* dst = cache + (size_t)slots[t] * RS;
-  for (int c = threadIdx.x; c < N; c += 256) {      // each thread reads back only what it wrote
-    if (c < NQ) stf(q_out + (size_t)t * ldq + c, row[c] * rq * wq[c]);
-    else stf(dst + (c - NQ), row[c] * rc * wc[c - NQ]);
+  ACT* dst = cache + (size_t)slot * RS;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = (k * BT + threadIdx.x) * V;
+    if (c >= N) continue;
+    const bool isq = c < NQ;
+    const float* w = isq ? wq + c : wc + (c - NQ);
+    const float r = isq ? rq : rc;
+    float v[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = x[k][e] * r * w[e];
+    st_vec<ACT, V>(isq ? q_out + (size_t)t * ldq + c : dst + (c - NQ), v);
   }
+}
+
+template <typename ACT, int V>
+int latent_norm_go(hipStream_t st, const float* part, int split, int T, int NQ, int NC, const float* wq, const float* wc,
+                   float eps, const int32_t* slots, void* q_out, int ldq, void* cache, int RS) {
+  const int vecs = (NQ + NC + V - 1) / V;
+#define LN_GO(NV, BT) \
+  latent_norm_kernel<ACT, V, NV, BT><<<T, BT, 0, st>>>(part, split, T, NQ, NC, wq, wc, eps, slots, (ACT*)q_out, ldq, (ACT*)cache, RS)
+  if (vecs <= 256) LN_GO(1, 256);
+  else if (vecs <= 512) LN_GO(1, 512);
+  else if (vecs <= 1024) LN_GO(1, 1024);
+  else if (vecs <= 4096) LN_GO(4, 1024);
+  else if (vecs <= 16384) LN_GO(16, 1024);
+  else return -4;
+#undef LN_GO
+  return CFC_CHECK_LAUNCH();
 }
 
 // ---------------------------------------------------------------------------------- head_linear
@@ -127,6 +182,58 @@ __global__ void __launch_bounds__(256) head_linear_kernel(const uint16_t* __rest
         }
       }
     }
+  }
+}
+
+// few tokens: the four waves of a workgroup share 16 outputs of 16 TT tokens, each a quarter of K with
+// all its loads in flight in rounds of four steps, and their sums meet in LDS
+template <int TT>
+__global__ void __launch_bounds__(256) head_linear_ks_kernel(const uint16_t* __restrict__ x, int64_t ldx, int64_t hsx,
+                                                            const uint16_t* __restrict__ w, int NP, int KP, int T, int N,
+                                                            int K, uint16_t* __restrict__ out, int64_t ldo, int64_t hso) {
+  __shared__ float4 red[3][TT][64];
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
+  const int h = blockIdx.z, t0 = blockIdx.x * 16 * TT, n0 = blockIdx.y * 16;
+  const int ks = KP / 32, k0 = ks * wv / 4, k1 = ks * (wv + 1) / 4;
+  const uint16_t* wp = w + ((size_t)h * NP + n0 + col) * KP + 8 * kq;
+  const uint16_t* xp[TT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) xp[i] = x + (int64_t)min(t0 + 16 * i + col, T - 1) * ldx + h * hsx;
+  f32x4_t acc[TT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k = k0; k < k1; k += 4) {
+    uint4 a[4], b[4][TT];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int kk = 32 * min(k + u, k1 - 1);
+      a[u] = *reinterpret_cast<const uint4*>(wp + kk);
+#pragma unroll
+      for (int i = 0; i < TT; ++i) b[u][i] = ld_frag<true>(xp[i], kk + 8 * kq, K);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      if (k + u < k1)
+#pragma unroll
+        for (int i = 0; i < TT; ++i) acc[i] = mfma16(a[u], b[u][i], acc[i]);
+  }
+  if (wv) {
+#pragma unroll
+    for (int i = 0; i < TT; ++i) red[wv - 1][i][lane] = make_float4(acc[i][0], acc[i][1], acc[i][2], acc[i][3]);
+  }
+  __syncthreads();
+  if (wv) return;
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    float v[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+#pragma unroll
+    for (int u = 0; u < 3; ++u) {
+      const float4 r = red[u][i][lane];
+      v[0] += r.x; v[1] += r.y; v[2] += r.z; v[3] += r.w;
+    }
+    const int t = t0 + 16 * i + col, n = n0 + 4 * kq;
+    if (t < T && n < N)
+      *reinterpret_cast<uint2*>(out + (int64_t)t * ldo + h * hso + n) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
   }
 }
 
@@ -466,7 +573,8 @@ __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restr
 }
 
 // tiles [n][2]: {sequence, first position} of 64 tokens each, at dense rows 64 blockIdx.x ..; positions past
-// the context are zero rows
+// the context are zero rows.  The slot-ordered copy is a product's W operand in the fragment-packed layout
+// of cfc_dgemm_pack for 64-row workgroups ([rows / 64][RS / 32][4][64 lanes][8])
 __global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __restrict__ cache,
                                                            const int32_t* __restrict__ block_tables, int max_blocks,
                                                            const int32_t* __restrict__ ctx_lens,
@@ -481,7 +589,9 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __re
                             : make_uint4(0, 0, 0, 0);
     const size_t base = (size_t)blockIdx.x * 64;
     reinterpret_cast<uint4*>(rows + (base + r) * RS)[c] = v;
-    reinterpret_cast<uint4*>(slot_rows + (base + (r & 32) + kv_v_slot(r & 31)) * RS)[c] = v;
+    const int sr = (r & 32) + kv_v_slot(r & 31);
+    reinterpret_cast<uint4*>(slot_rows)[(((size_t)blockIdx.x * (RS / 32) + (c >> 2)) * 4 + (sr >> 4)) * 64 + (sr & 15) +
+                                        16 * (c & 3)] = v;
   }
 }
 
@@ -566,15 +676,12 @@ CFC_API int cfc_latent_norm(int f32, const float* part, int split, int T, int NQ
                             float eps, const int32_t* slots, void* q_out, int ldq, void* cache, int RS,
                             hipStream_t stream) {
   if (T <= 0) return 0;
-  if (split < 1 || NQ < 1 || NC < 1 || NC > RS || ldq < NQ || (NQ + NC) * 4 > 60000) return -1;
-  const size_t lds = (size_t)(NQ + NC) * 4;
-  if (f32)
-    latent_norm_kernel<float><<<T, 256, lds, stream>>>(part, split, T, NQ, NC, wq, wc, eps, slots, (float*)q_out, ldq,
-                                                       (float*)cache, RS);
-  else
-    latent_norm_kernel<uint16_t><<<T, 256, lds, stream>>>(part, split, T, NQ, NC, wq, wc, eps, slots, (uint16_t*)q_out,
-                                                          ldq, (uint16_t*)cache, RS);
-  return CFC_CHECK_LAUNCH();
+  if (split < 1 || NQ < 1 || NC < 1 || NC > RS || ldq < NQ) return -1;
+  const bool v4 = NQ % 4 == 0 && NC % 4 == 0 && ldq % 4 == 0;
+#define LN_ARGS stream, part, split, T, NQ, NC, wq, wc, eps, slots, q_out, ldq, cache, RS
+  if (f32) return v4 ? latent_norm_go<float, 4>(LN_ARGS) : latent_norm_go<float, 1>(LN_ARGS);
+  return v4 ? latent_norm_go<uint16_t, 4>(LN_ARGS) : latent_norm_go<uint16_t, 1>(LN_ARGS);
+#undef LN_ARGS
 }
 
 // x row (t, h) at t ldx + h hsx (K values), out at t ldo + h hso (N values); W [H][NP][KP] zero-padded
@@ -593,11 +700,17 @@ CFC_API int cfc_head_linear(int f32, const void* x, int64_t ldx, int64_t hsx, co
 #define HL(TT, NT, V)                                                                                                 \
   head_linear_kernel<TT, NT, V><<<dim3((T + 16 * TT - 1) / (16 * TT), (NP + 64 * NT - 1) / (64 * NT), H), 256, 0, stream>>>( \
       (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso)
+#define HK(TT)                                                                                                   \
+  head_linear_ks_kernel<TT><<<dim3((T + 16 * TT - 1) / (16 * TT), (N + 15) / 16, H), 256, 0, stream>>>(          \
+      (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso)
   if (!vec) HL(4, 1, false);
+  else if (T <= 256 && KP >= 256 && T <= 16) HK(1);
+  else if (T <= 256 && KP >= 256) HK(2);
   else if (T <= 16) HL(1, 1, true);
   else if (T <= 256) HL(4, 1, true);
   else HL(4, 2, true);
 #undef HL
+#undef HK
   return CFC_CHECK_LAUNCH();
 }
 

@@ -100,6 +100,20 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
   const size_t row = (size_t)t * a.W, plane = (size_t)a.T * a.W;
   Vec<V> x[NV];
   float ss = 0.f;
+  // the first inputs of the convolution's past, requested ahead of everything that does not depend on them
+  constexpr int PRE = MODE == DN_CONV && NV == 1 ? 3 : 0;
+  Vec<V> past[PRE ? PRE : 1];
+  const int pos = MODE == DN_CONV ? a.positions[b] : 0;
+  if constexpr (PRE > 0) {
+    const int c = threadIdx.x * V;
+#pragma unroll
+    for (int u = 0; u < PRE; ++u) {
+      const int q = pos - 1 - u;
+#pragma unroll
+      for (int e = 0; e < V; ++e) past[u].v[e] = 0.f;
+      if (u < a.taps - 1 && q >= 0 && c < a.W) past[u] = ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+    }
+  }
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
     const int c = (k * BT + threadIdx.x) * V;
@@ -128,12 +142,13 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
       const float an = a.dwa[a.n];
 #pragma unroll
       for (int e = 0; e < V; ++e) acc.v[e] = an * cur.v[e];
-      for (int j = 0; j < a.n; j += 8) {     // eight rows of the history in flight
-        Vec<V> y[8];
+      constexpr int HU = NV == 1 ? 16 : 8;       // rows of the history in flight
+      for (int j = 0; j < a.n; j += HU) {
+        Vec<V> y[HU];
 #pragma unroll
-        for (int u = 0; u < 8; ++u) y[u] = ldv<V>(a.hist + (size_t)min(j + u, a.n - 1) * plane + row + c);
+        for (int u = 0; u < HU; ++u) y[u] = ldv<V>(a.hist + (size_t)min(j + u, a.n - 1) * plane + row + c);
 #pragma unroll
-        for (int u = 0; u < 8; ++u) {
+        for (int u = 0; u < HU; ++u) {
           const float wj = j + u < a.n ? a.dwa[j + u] : 0.f;
 #pragma unroll
           for (int e = 0; e < V; ++e) acc.v[e] += wj * y[u].v[e];
@@ -151,7 +166,6 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
   if constexpr (MODE == DN_RSTD) {
     if (threadIdx.x == 0) a.rstd[t] = rstd;
   } else {
-    const int pos = MODE == DN_CONV ? a.positions[b] : 0;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
       const int c = (k * BT + threadIdx.x) * V;
@@ -167,7 +181,12 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
         for (int j = 0; j < a.taps; ++j) {
           const int q = pos - a.taps + 1 + j;
           if (q < 0) continue;
-          const Vec<V> s = j == a.taps - 1 ? h : ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+          Vec<V> s = h;
+          if (j < a.taps - 1) {
+            const int u = a.taps - 2 - j;          // positions back, less one
+            if (u < PRE) s = u == 0 ? past[0] : u == 1 ? past[PRE > 1 ? 1 : 0] : past[PRE > 2 ? 2 : 0];
+            else s = ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+          }
           const Vec<V> k1 = ldv<V>(a.w1 + (size_t)j * a.W + c);
 #pragma unroll
           for (int e = 0; e < V; ++e) y1.v[e] += k1.v[e] * s.v[e];
