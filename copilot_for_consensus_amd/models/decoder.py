@@ -499,8 +499,10 @@ class DecoderModel:
             self.prefill_gemm = "hip"
 
     # ---------------------------------------------------------------- engine interface
-    # kernel sources (csrc/kernels/<name>.hip) a run of this family loads
-    kernel_sources = None        # the whole library
+    @staticmethod
+    def kernel_sources(cfg, dtype):
+        """csrc/kernels sources a run of this configuration launches kernels from (None: any of them)."""
+        return None
 
     def new_cache(self, num_blocks: int, dtype=None, device=None):
         from ..runtime.kv_cache import PagedKVCache

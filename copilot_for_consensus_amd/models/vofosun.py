@@ -298,9 +298,15 @@ class VofosunWeights:
 class VofosunModel:
     """Stateless forward functions over :class:`VofosunWeights` + a :class:`LatentKVCache`."""
 
-    # leading blocks are shared with other sequences only once computed: a portion reads the
-    # convolution tail of the block before it in the launch that writes the tails
-    kernel_sources = ("elementwise", "stream", "latent", "gemm", "dgemm", "pgemm", "attention")
+    @staticmethod
+    def kernel_sources(cfg, dtype) -> tuple:
+        """csrc/kernels sources a run of this configuration launches kernels from."""
+        src = ("elementwise", "stream", "latent")
+        if dtype == torch.bfloat16:
+            src += ("gemm", "dgemm", "pgemm")
+            if any(s.mixer.dim == s.mixer.vdim == L.EXPANDED_DIM for s in cfg.specs):
+                src += ("attention",)
+        return src
 
     def __init__(self, weights: VofosunWeights, tp_group=None, custom_ar=None):
         self.w = weights
@@ -384,7 +390,7 @@ class VofosunModel:
             attn = dict(cu_q=cu_q, tiles=(tiles[0], tiles[1]), rows=rows,
                         P=L.partitions(tiles.shape[1], plan["max_ctx"]))
             dense = plan if "uk_full" in lw and plan[f"expand_{self._rs(i)}"] else None
-            up = self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn, dense)
+            up = self._average(i, self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn, dense), hist, bufs)
         return S.depth_norm(cur, hist, up, self.w.final_norm, self.cfg.norm_eps, self.w.dtype,
                             None if last_idx is None else last_idx.to(torch.int32))
 
@@ -403,7 +409,7 @@ class VofosunModel:
             cur = x
             attn = dict(cu_q=None, rows=self._rows(i, (ids.numel(), P, block_tables.shape[1] * KV_BLOCK)), P=P,
                         workspace=attn_workspace)
-            up = self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn)
+            up = self._average(i, self._layer(i, hs, slots, ctx_lens, block_tables, kv, attn), hist, bufs)
         return S.depth_norm(cur, hist, up, self.w.final_norm, self.cfg.norm_eps, self.w.dtype)
 
     def _embed(self, ids):
@@ -427,9 +433,21 @@ class VofosunModel:
             bufs[two, wide] = hs
         return bufs[two, wide]
 
-    def _layer(self, i, hs, slots, ctx_lens, block_tables, kv, attn, dense=None) -> S.Update:
-        """Both sublayers of layer i on their inputs: what the layer adds to the stream.  ``dense``: the launch
-        plan of a pass whose keys and values are expanded per head."""
+    def _average(self, i, part, hist, bufs) -> S.Update:
+        """What layer i adds to the stream and the average that follows.  Every few layers the results so far
+        are summed once for all the averages of the run (S.depth_pre)."""
+        lw, run = self.w.layers[i], S.DEPTH_RUN
+        g = i - i % run
+        if g == 0:
+            return S.Update(part, lw["bias"], lw["dwa"], i + 1)
+        if i == g:
+            bufs["pre"] = S.depth_pre(hist, g + 1, [w["dwa"] for w in self.w.layers[g:g + run]])
+        return S.Update(part, lw["bias"], lw["dwa"], i + 1, bufs["pre"][i - g], g + 1)
+
+    def _layer(self, i, hs, slots, ctx_lens, block_tables, kv, attn, dense=None) -> torch.Tensor:
+        """Both sublayers of layer i on their inputs: the fp32 slabs [split, T, W] of what the layer adds to
+        the stream (without the feed-forward's output bias).  ``dense``: the launch plan of a pass whose keys
+        and values are expanded per head."""
         lw, spec = self.w.layers[i], self.cfg.specs[i]
         m, H = spec.mixer, lw["H"]
         T, dt, dev = hs[0].shape[0], self.w.dtype, hs[0].device
@@ -457,7 +475,7 @@ class VofosunModel:
         if self.w.tp_size > 1:
             part = part.sum(0, keepdim=True)
             torch.distributed.all_reduce(part, group=self.tp_group)
-        return S.Update(part, lw["bias"], lw["dwa"], i + 1)
+        return part
 
     # ---------------------------------------------------------------- output
     def _local_logits(self, hidden):

@@ -54,7 +54,8 @@ _KERNEL_SIGS = {
     "cfc_sample_truncated": [P, I, I, I, F, I, F, F, c_uint32, P, P, P],
     "cfc_decode_advance": [P, P, I, P, P, P, P, P, P, I, P, P, I, I] + [P] * 6 + [I] * 4 + [P] * 4,
     "cfc_embed_f32": [P, P, P, I, I, I, I, P],
-    "cfc_depth_norm": [I, I, I, P, P, P, P, I, P, P, I, P, F, P, P, I, I, P, I, P, I, P, P, I, P, P, I, P, I, P],
+    "cfc_depth_pre": [P, c_int64, I, I, P, P, P, P, P, P],
+    "cfc_depth_norm": [I, I, I, P, P, P, P, I, P, P, I, P, I, P, F, P, P, I, I, P, I, P, I, P, P, I, P, P, I, P, I, P],
     "cfc_input_conv": [I, I, P, P, P, P, P, P, I, P, I, P, I, I, P, I, P, I, P],
     "cfc_clamped_glu": [I, I, P, I, P, I, P, P, I, I, I, F, F, F, P],
     "cfc_softcap": [P, c_int64, F, P],

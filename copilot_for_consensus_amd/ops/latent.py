@@ -103,7 +103,7 @@ def decode_plan(B: int, heads: int, RS: int, max_ctx: int, P: int | None = None)
             t = max(rounds * (4 + math.ceil(nt / p) * _TILE_US[rows] * scale * min(per_cu, math.ceil(B * g * p / 256))),
                     B * max_ctx * RS * 2 * g / 7e6)
             if p > 1:
-                t += 5 + 2 * B * heads * p * RS * 4 / 5e6
+                t += 8 + 2 * B * heads * p * RS * 4 / 5e6
             if best is None or t < best[0]:
                 best = (t, rows, p)
     return best[1], best[2]

@@ -324,12 +324,15 @@ def tail_slots(taps: int) -> int:
     return 0 if taps <= 1 else min(taps + 1, KV_BLOCK)
 
 
-def depth_norm(x, hist, part, bias, dwa, n, eps):
-    """X_n = x + sum of part slabs + bias into hist[n]; returns (sum_j dwa[j] X_j, 1 / rms of it)."""
+def depth_norm(x, hist, part, bias, dwa, n, eps, pre=None, j0=0):
+    """X_n = x + sum of part slabs + bias into hist[n]; returns (sum_j dwa[j] X_j, 1 / rms of it); ``pre``
+    is the sum of the first j0 terms."""
     if part is not None:
         new = x + part.sum(0) + (bias if bias is not None else 0.0)
         hist[n].copy_(new)
-        x = torch.einsum("j,jtw->tw", dwa[:n + 1].float(), hist[:n + 1])
+        j0 = j0 if pre is not None else 0
+        x = torch.einsum("j,jtw->tw", dwa[j0:n + 1].float(), hist[j0:n + 1])
+        x = x if pre is None else x + pre
     return x, 1.0 / torch.sqrt((x * x).mean(-1) + eps)
 
 

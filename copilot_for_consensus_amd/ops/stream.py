@@ -51,12 +51,39 @@ class Tail:
 
 class Update:
     """What a layer adds to the stream: fp32 slabs [split, T, W] of its sublayers' sum, an optional bias
-    and the depth weights over X_0 .. X_n (n results so far, the new one becomes X_n)."""
+    and the depth weights over X_0 .. X_n (n results so far, the new one becomes X_n).  ``pre`` [T, W]: the
+    first ``j0`` terms of the average, already summed (:func:`depth_pre`)."""
 
-    __slots__ = ("part", "bias", "dwa", "n")
+    __slots__ = ("part", "bias", "dwa", "n", "pre", "j0")
 
-    def __init__(self, part, bias, dwa, n):
-        self.part, self.bias, self.dwa, self.n = part, bias, dwa, n
+    def __init__(self, part, bias, dwa, n, pre=None, j0=0):
+        self.part, self.bias, self.dwa, self.n, self.pre, self.j0 = part, bias, dwa, n, pre, j0
+
+    def terms(self, x, hist, eps):
+        """CPU: the averaged stream and its 1 / rms."""
+        return ref.depth_norm(x, hist, self.part, self.bias, self.dwa, self.n, eps, self.pre, self.j0)
+
+
+DEPTH_RUN = 4       # layers per depth_pre pass
+
+
+def depth_pre(hist, n: int, dwas) -> torch.Tensor:
+    """[len(dwas), T, W]: sum over j < n of dwa[j] X_j for each of (up to four) weight vectors."""
+    pre = torch.empty(len(dwas), *hist.shape[1:], dtype=torch.float32, device=hist.device)
+    if not hist.is_cuda:
+        for p, w in zip(pre, dwas):
+            p.copy_(torch.einsum("j,jtw->tw", w[:n].float(), hist[:n]))
+        return pre
+    if len(dwas) > DEPTH_RUN or any(w.numel() < n for w in dwas) or hist.shape[0] < n:
+        raise ValueError(f"depth_pre: {len(dwas)} weight vectors over {n} of {hist.shape[0]} results")
+    ptrs = [w.data_ptr() for w in dwas] + [None] * (DEPTH_RUN - len(dwas))
+    check(kernels().cfc_depth_pre(hist.data_ptr(), hist[0].numel(), n, len(dwas), *ptrs, pre.data_ptr(), _stream(hist)),
+          "cfc_depth_pre")
+    return pre
+
+
+def _stats_ref(x, hist, up, eps):
+    return up.terms(x, hist, eps) if up else ref.depth_norm(x, hist, None, None, None, 0, eps)
 
 
 def _depth(mode, f32, nrows, rows, x, hist, up, norm_w, eps, x_out, rstd, h1, h2, w1, w2, positions, tail, ref_t):
@@ -71,7 +98,7 @@ def _depth(mode, f32, nrows, rows, x, hist, up, norm_w, eps, x_out, rstd, h1, h2
     check(kernels().cfc_depth_norm(
         mode, f32, nrows, _p(rows), x.data_ptr(), hist.data_ptr(), _p(up.part) if up else None,
         up.part.shape[0] if up else 0, _p(up.bias) if up else None, _p(up.dwa) if up else None, up.n if up else 0,
-        _p(norm_w), float(eps), _p(x_out), _p(rstd), T, W, _p(h1), h1.stride(0) if h1 is not None else 0, _p(h2),
+        _p(up.pre) if up else None, up.j0 if up else 0, _p(norm_w), float(eps), _p(x_out), _p(rstd), T, W, _p(h1), h1.stride(0) if h1 is not None else 0, _p(h2),
         h2.stride(0) if h2 is not None else 0, _p(w1), _p(w2), w1.shape[0] if w1 is not None else 1, _p(positions), *t,
         _stream(ref_t)), "cfc_depth_norm")
 
@@ -79,7 +106,7 @@ def _depth(mode, f32, nrows, rows, x, hist, up, norm_w, eps, x_out, rstd, h1, h2
 def depth_stats(x, hist, up: Update | None, eps: float, x_out, rstd) -> None:
     """Apply ``up`` (if any) and leave the averaged stream in ``x_out`` and 1 / rms per row in ``rstd``."""
     if not hist.is_cuda:
-        y, r = ref.depth_norm(x, hist, up and up.part, up and up.bias, up and up.dwa, up.n if up else 0, eps)
+        y, r = _stats_ref(x, hist, up, eps)
         x_out.copy_(y)
         rstd.copy_(r)
         return
@@ -91,7 +118,7 @@ def depth_norm(x, hist, up: Update | None, norm_w, eps: float, dtype, rows=None)
     stream itself is not stored (the model's last norm)."""
     n = rows.numel() if rows is not None else hist.shape[1]
     if not hist.is_cuda:
-        y, r = ref.depth_norm(x, hist, up and up.part, up and up.bias, up and up.dwa, up.n if up else 0, eps)
+        y, r = _stats_ref(x, hist, up, eps)
         h = y * r[:, None] * norm_w
         return (h if rows is None else h[rows.long()]).to(dtype)
     out = torch.empty(n, hist.shape[2], dtype=dtype, device=hist.device)
@@ -105,7 +132,7 @@ def depth_conv_decode(x, hist, up: Update | None, norm_w, eps: float, convs, pos
     """One token per sequence: apply ``up``, norm, and run the row through each sublayer's input
     convolution (``convs``: one or two [taps, W]) with the cached tail; results into ``outs``."""
     if not hist.is_cuda:
-        y, r = ref.depth_norm(x, hist, up and up.part, up and up.bias, up and up.dwa, up.n if up else 0, eps)
+        y, r = _stats_ref(x, hist, up, eps)
         x_out.copy_(y)
         h = y * r[:, None] * norm_w
         por = [(b, 1, int(positions[b]), b) for b in range(h.shape[0])]

@@ -74,7 +74,7 @@ def open_session(model_dir, dtype: str, max_tokens: int, device="cuda:0") -> Tra
         if not torch.cuda.is_available():
             raise RuntimeError("no GPU")
         from ..ops import _native
-        _native.ensure_kernels(family.model.kernel_sources)
+        _native.ensure_kernels(family.model.kernel_sources(cfg, want))
     torch.set_float32_matmul_precision("highest")
     model = registry.build_model(registry.load_weights(cfg, model_dir, dev, dtype=want))
     kv = model.new_cache(blocks_needed(max_tokens))

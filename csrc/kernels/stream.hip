@@ -6,6 +6,7 @@
 //                        workgroup.  Three endings: the norm's 1 / rms only (a prompt's rows, before
 //                        input_conv), the normed row (the model's last norm), or the normed row run
 //                        through both sublayers' input convolutions with the cached tail (decode)
+//   * depth_pre          the older results' share of the next few layers' averages, in one pass over them
 //   * input_conv         h + conv(h) over time on each channel, for both sublayers at once, over a packed
 //                        batch of prompt portions
 //   * clamped_glu        min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta), optional biases
@@ -19,6 +20,8 @@
 //
 // ACT is the activation type the matrix products read: uint16_t (bf16 bits) or float.
 #include "common.h"
+
+#include <type_traits>
 
 namespace {
 
@@ -79,6 +82,8 @@ struct DepthArgs {
   const float* part;      // fp32 slabs [split][T][W] of the sublayers' sum, or null (no update)
   const float* bias;      // [W] fp32 or null
   const float* dwa;       // [n + 1]
+  const float* pre;       // [T][W] sum of the first j0 terms of the average (null: j0 = 0)
+  int j0;
   const float* norm_w;    // [W] fp32: the multiplier itself (1 + stored weight where the design stores it so)
   float* x_out;           // [T][W] (may be x_in), not written when null
   float* rstd;            // DN_RSTD: [T]
@@ -100,18 +105,20 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
   const size_t row = (size_t)t * a.W, plane = (size_t)a.T * a.W;
   Vec<V> x[NV];
   float ss = 0.f;
-  // the first inputs of the convolution's past, requested ahead of everything that does not depend on them
-  constexpr int PRE = MODE == DN_CONV && NV == 1 ? 3 : 0;
-  Vec<V> past[PRE ? PRE : 1];
+  // the last row's convolution past and every weight, requested ahead of the stream they wait for
+  constexpr int PRE = MODE == DN_CONV && NV == 1 ? 4 : 0;
+  Vec<V> past[PRE ? PRE : 1], k1[PRE ? PRE : 1], k2[PRE ? PRE : 1], gw;
   const int pos = MODE == DN_CONV ? a.positions[b] : 0;
+  const bool pre_ok = PRE > 0 && a.taps <= PRE;
   if constexpr (PRE > 0) {
-    const int c = threadIdx.x * V;
+    const int c = min((int)threadIdx.x * V, a.W - V);
+    gw = ldv<V>(a.norm_w + c);
 #pragma unroll
-    for (int u = 0; u < PRE; ++u) {
-      const int q = pos - 1 - u;
-#pragma unroll
-      for (int e = 0; e < V; ++e) past[u].v[e] = 0.f;
-      if (u < a.taps - 1 && q >= 0 && c < a.W) past[u] = ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+    for (int u = 0; u < PRE; ++u) {          // tap taps - 1 - u: u positions back
+      const int j = max(a.taps - 1 - u, 0);
+      k1[u] = ldv<V>(a.w1 + (size_t)j * a.W + c);
+      k2[u] = ldv<V>((a.w2 ? a.w2 : a.w1) + (size_t)j * a.W + c);
+      if (u && a.taps > 1) past[u] = ldv<V>(tail_row(a.tail, b, max(pos - u, 0), a.W) + c);
     }
   }
 #pragma unroll
@@ -122,12 +129,15 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
     if (c >= a.W) continue;
     Vec<V> cur = ldv<V>(a.x_in + row + c);
     if (a.part) {
-      for (int p0 = 0; p0 < a.split; p0 += 4) {      // four slabs in flight (past the last: re-read, not added)
-        Vec<V> y[4];
+      Vec<V> pre;
+      if (a.pre) pre = ldv<V>(a.pre + row + c);
+      constexpr int SU = NV == 1 ? 8 : 4;             // slabs in flight (past the last: re-read, not added)
+      for (int p0 = 0; p0 < a.split; p0 += SU) {
+        Vec<V> y[SU];
 #pragma unroll
-        for (int u = 0; u < 4; ++u) y[u] = ldv<V>(a.part + (size_t)min(p0 + u, a.split - 1) * plane + row + c);
+        for (int u = 0; u < SU; ++u) y[u] = ldv<V>(a.part + (size_t)min(p0 + u, a.split - 1) * plane + row + c);
 #pragma unroll
-        for (int u = 0; u < 4; ++u)
+        for (int u = 0; u < SU; ++u)
           if (p0 + u < a.split)
 #pragma unroll
             for (int e = 0; e < V; ++e) cur.v[e] += y[u].v[e];
@@ -142,17 +152,20 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
       const float an = a.dwa[a.n];
 #pragma unroll
       for (int e = 0; e < V; ++e) acc.v[e] = an * cur.v[e];
-      constexpr int HU = NV == 1 ? 16 : 8;       // rows of the history in flight
-      for (int j = 0; j < a.n; j += HU) {
-        Vec<V> y[HU];
+      for (int j = a.j0; j < a.n; j += 4) {      // four rows of the history in flight
+        Vec<V> y[4];
 #pragma unroll
-        for (int u = 0; u < HU; ++u) y[u] = ldv<V>(a.hist + (size_t)min(j + u, a.n - 1) * plane + row + c);
+        for (int u = 0; u < 4; ++u) y[u] = ldv<V>(a.hist + (size_t)min(j + u, a.n - 1) * plane + row + c);
 #pragma unroll
-        for (int u = 0; u < HU; ++u) {
+        for (int u = 0; u < 4; ++u) {
           const float wj = j + u < a.n ? a.dwa[j + u] : 0.f;
 #pragma unroll
           for (int e = 0; e < V; ++e) acc.v[e] += wj * y[u].v[e];
         }
+      }
+      if (a.pre) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) acc.v[e] += pre.v[e];
       }
       cur = acc;
     }
@@ -170,7 +183,7 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
     for (int k = 0; k < NV; ++k) {
       const int c = (k * BT + threadIdx.x) * V;
       if (c >= a.W) continue;
-      const Vec<V> g = ldv<V>(a.norm_w + c);
+      const Vec<V> g = PRE > 0 ? gw : ldv<V>(a.norm_w + c);
       Vec<V> h;
 #pragma unroll
       for (int e = 0; e < V; ++e) h.v[e] = x[k].v[e] * rstd * g.v[e];
@@ -178,22 +191,32 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
         stv<V>(h1 + (size_t)b * a.ld1_ + c, h);
       } else {
         Vec<V> y1 = h, y2 = h;
-        for (int j = 0; j < a.taps; ++j) {
-          const int q = pos - a.taps + 1 + j;
-          if (q < 0) continue;
-          Vec<V> s = h;
-          if (j < a.taps - 1) {
-            const int u = a.taps - 2 - j;          // positions back, less one
-            if (u < PRE) s = u == 0 ? past[0] : u == 1 ? past[PRE > 1 ? 1 : 0] : past[PRE > 2 ? 2 : 0];
-            else s = ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+        if (pre_ok) {
+          if constexpr (PRE > 0) {
+#pragma unroll
+            for (int u = PRE - 1; u >= 0; --u) {
+              if (u >= a.taps || pos - u < 0) continue;
+#pragma unroll
+              for (int e = 0; e < V; ++e) {
+                const float s = u ? past[u].v[e] : h.v[e];
+                y1.v[e] += k1[u].v[e] * s;
+                y2.v[e] += k2[u].v[e] * s;
+              }
+            }
           }
-          const Vec<V> k1 = ldv<V>(a.w1 + (size_t)j * a.W + c);
+        } else {
+          for (int j = 0; j < a.taps; ++j) {
+            const int q = pos - a.taps + 1 + j;
+            if (q < 0) continue;
+            const Vec<V> s = j == a.taps - 1 ? h : ldv<V>(tail_row(a.tail, b, q, a.W) + c);
+            const Vec<V> c1 = ldv<V>(a.w1 + (size_t)j * a.W + c);
 #pragma unroll
-          for (int e = 0; e < V; ++e) y1.v[e] += k1.v[e] * s.v[e];
-          if (a.w2) {
-            const Vec<V> k2 = ldv<V>(a.w2 + (size_t)j * a.W + c);
+            for (int e = 0; e < V; ++e) y1.v[e] += c1.v[e] * s.v[e];
+            if (a.w2) {
+              const Vec<V> c2 = ldv<V>(a.w2 + (size_t)j * a.W + c);
 #pragma unroll
-            for (int e = 0; e < V; ++e) y2.v[e] += k2.v[e] * s.v[e];
+              for (int e = 0; e < V; ++e) y2.v[e] += c2.v[e] * s.v[e];
+            }
           }
         }
         if (a.taps > 1) stv<V>(tail_row(a.tail, b, pos, a.W) + c, h);
@@ -202,6 +225,43 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
       }
     }
   }
+}
+
+// The oldest n results' share of the averages after up to DP_MAX consecutive layers, in one pass over the
+// history: pre[l] = sum_{j < n} dwa_l[j] X_j.  The averages of a run of layers then read only what that run
+// has added, instead of the whole history each.
+constexpr int DP_MAX = 4;
+struct PreArgs { const float* dwa[DP_MAX]; };
+
+template <int V, int CNT>
+__global__ void __launch_bounds__(256) depth_pre_kernel(const float* __restrict__ hist, size_t plane, int n, PreArgs w,
+                                                       float* __restrict__ pre) {
+  const size_t c = ((size_t)blockIdx.x * 256 + threadIdx.x) * V;
+  if (c >= plane) return;
+  Vec<V> acc[CNT];
+#pragma unroll
+  for (int l = 0; l < CNT; ++l)
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[l].v[e] = 0.f;
+  int j = 0;
+  auto step = [&](auto nu) {
+    constexpr int U = decltype(nu)::value;
+    Vec<V> y[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) y[u] = ldv<V>(hist + (size_t)(j + u) * plane + c);
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int l = 0; l < CNT; ++l)
+#pragma unroll
+        for (int e = 0; e < V; ++e) acc[l].v[e] += w.dwa[l][j + u] * y[u].v[e];
+    j += U;
+  };
+  while (j + 8 <= n) step(std::integral_constant<int, 8>{});
+  if (j + 4 <= n) step(std::integral_constant<int, 4>{});
+  while (j < n) step(std::integral_constant<int, 1>{});
+#pragma unroll
+  for (int l = 0; l < CNT; ++l) stv<V>(pre + (size_t)l * plane + c, acc[l]);
 }
 
 // Packed prompt portions.  A tile is the rows of one portion inside ONE cache block: {first row, rows,
@@ -390,19 +450,35 @@ CFC_API int cfc_embed_f32(float* out, const void* table, const int32_t* ids, int
 // normed outputs are fp32 (else bf16).  nrows workgroups; rows null: row b of T.
 CFC_API int cfc_depth_norm(int mode, int f32, int nrows, const int32_t* rows, const float* x_in, float* hist,
                            const float* part, int split, const float* bias, const float* dwa, int n,
+                           const float* pre, int j0,
                            const float* norm_w, float eps, float* x_out, float* rstd, int T, int W, void* h1, int ld1,
                            void* h2, int ld2, const float* w1, const float* w2, int taps, const int32_t* positions,
                            float* tail, int slots, const int32_t* block_tables, int max_blocks, hipStream_t stream) {
   if (nrows <= 0) return 0;
-  if (W <= 0 || T <= 0 || n < 0 || (part && (split < 1 || !hist || !dwa))) return -1;
+  if (W <= 0 || T <= 0 || n < 0 || (pre && (j0 < 0 || j0 > n)) || (part && (split < 1 || !hist || !dwa))) return -1;
   if (mode == DN_RSTD && !rstd) return -2;
   if (mode != DN_RSTD && (!h1 || !norm_w)) return -2;
   if (mode == DN_CONV && (!w1 || taps < 1 || !positions || (w2 && !h2) || rows ||
                           (taps > 1 && (!tail || slots < (taps - 1 < CFC_KV_BS ? taps - 1 : CFC_KV_BS) || !block_tables))))
     return -2;
-  DepthArgs a{x_in, hist, part, bias, dwa, norm_w, x_out, rstd, rows, T, W, split, n, eps, w1, w2, positions,
+  DepthArgs a{x_in, hist, part, bias, dwa, pre, pre ? j0 : 0, norm_w, x_out, rstd, rows, T, W, split, n, eps, w1, w2, positions,
               TailArg{tail, block_tables, max_blocks, slots > 0 ? slots : 1}, taps, ld1, ld2};
   return f32 ? depth_launch<float>(mode, nrows, stream, a, h1, h2) : depth_launch<uint16_t>(mode, nrows, stream, a, h1, h2);
+}
+
+// pre [count][T][W] (count <= 4): sums of the first n planes of hist [.][T][W] weighted by dwa0 .. dwa3
+CFC_API int cfc_depth_pre(const float* hist, int64_t plane, int n, int count, const float* dwa0, const float* dwa1,
+                          const float* dwa2, const float* dwa3, float* pre, hipStream_t stream) {
+  if (plane <= 0) return 0;
+  if (n < 1 || count < 1 || count > DP_MAX || !pre || !hist) return -1;
+  const PreArgs w{{dwa0, dwa1, dwa2, dwa3}};
+  const bool v4 = plane % 4 == 0 && ((uintptr_t)hist & 15) == 0 && ((uintptr_t)pre & 15) == 0;
+  const unsigned grid = (unsigned)((plane + (v4 ? 1023 : 255)) / (v4 ? 1024 : 256));
+#define DP_GO(V, C) depth_pre_kernel<V, C><<<grid, 256, 0, stream>>>(hist, (size_t)plane, n, w, pre); break
+  if (v4) switch (count) { case 1: DP_GO(4, 1); case 2: DP_GO(4, 2); case 3: DP_GO(4, 3); default: DP_GO(4, 4); }
+  else switch (count) { case 1: DP_GO(1, 1); case 2: DP_GO(1, 2); case 3: DP_GO(1, 3); default: DP_GO(1, 4); }
+#undef DP_GO
+  return CFC_CHECK_LAUNCH();
 }
 
 // tiles [2][n_tiles][4]: {first row, rows, first position, sequence}, then {portion rows before the tile, 0, 0, 0}
