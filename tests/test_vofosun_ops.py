@@ -1,0 +1,348 @@
+"""Each mechanism of the Vofosun decoder alone, against the plain implementation."""
+import math
+
+import numpy as np
+import pytest
+import torch
+
+import vofosun_oracle as oracle
+from copilot_for_consensus_amd.ops import kernels as K
+from copilot_for_consensus_amd.ops import latent as L
+from copilot_for_consensus_amd.ops import stream as S
+from copilot_for_consensus_amd.ops.reference import interleave_gate_up, tail_slots
+
+DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+DTYPES = [torch.float32, torch.bfloat16]
+
+
+def rnd(*shape, seed=0, scale=1.0):
+    return scale * torch.randn(*shape, generator=torch.Generator().manual_seed(seed + 31 * len(shape) + sum(shape)))
+
+
+def close(got, want, tol):
+    got, want = got.float().cpu(), want.float()
+    assert torch.isfinite(got).all()
+    assert float((got - want).abs().max()) <= tol * max(1.0, float(want.abs().max())), float((got - want).abs().max())
+
+
+def tol(dtype):
+    return 2e-5 if dtype == torch.float32 else 1e-2
+
+
+# ------------------------------------------------------------------ stream
+@pytest.mark.parametrize("device", DEVICES)
+def test_embedding_rows_as_fp32(device):
+    table, ids = rnd(37, 21).to(torch.bfloat16), torch.tensor([36, 0, 5, 5], dtype=torch.int32)
+    out = torch.empty(4, 21, device=device)
+    S.embed_f32(table.to(device), ids.to(device), out)
+    assert torch.equal(out.cpu(), table[ids.long()].float())
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("W,T,n,split", [(104, 5, 3, 1), (65, 3, 1, 4), (1500, 2, 9, 3), (4096, 3, 6, 9), (5000, 700, 2, 1)])
+@pytest.mark.parametrize("pre", [False, True])
+def test_depth_average_and_norm(device, W, T, n, split, pre):
+    hist, x, part = rnd(n + 1, T, W), rnd(T, W, seed=1), rnd(split, T, W, seed=2, scale=0.3)
+    bias, dwa, nw, eps = rnd(W, seed=3), rnd(n + 1, seed=4), rnd(W, seed=5), 1e-3
+    hist[n] = 0
+    new = x + part.sum(0) + bias
+    avg = oracle.depth_average([*hist[:n], new], dwa)
+    want = oracle.centred_norm(avg, nw, eps)
+    h, d = hist.to(device), lambda t: t.to(device).contiguous()
+    j0 = n // 2 if pre else 0
+    p = S.depth_pre(h, j0, [d(dwa)] * 2)[1] if j0 else None
+    up = S.Update(d(part), d(bias), d(dwa), n, p, j0)
+    xo, rstd = torch.empty(T, W, device=device), torch.empty(T, device=device)
+    S.depth_stats(d(x), h, up, eps, xo, rstd)
+    close(xo, avg, 3e-6)
+    close(h[n], new, 3e-6)
+    close(xo * rstd[:, None] * d(1 + nw), want, 3e-5)
+    rows = torch.tensor([T - 1, 0], dtype=torch.int32, device=device)
+    for dt in DTYPES:
+        close(S.depth_norm(d(x), h, up, d(1 + nw), eps, dt, rows), want[[T - 1, 0]], tol(dt))
+        close(S.depth_norm(d(x), h, up, d(1 + nw), eps, dt), want, tol(dt))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("count", [1, 3, 4])
+@pytest.mark.parametrize("n,W", [(1, 20), (5, 33), (13, 64)])
+def test_depth_pre_sums_for_several_layers(device, n, W, count):
+    hist, ws = rnd(n + 2, 3, W), [rnd(n + 1 + i, seed=i) for i in range(count)]
+    got = S.depth_pre(hist.to(device), n, [w.to(device) for w in ws])
+    for g, w in zip(got, ws):
+        close(g, oracle.depth_average(list(hist[:n]), w[:n]), 1e-5)
+
+
+class Pages:
+    """Block tables of several sequences over a shuffled pool."""
+
+    def __init__(self, ctxs, device, seed=0):
+        n = [max(1, -(-c // 32)) for c in ctxs]
+        perm = torch.randperm(sum(n) + 2, generator=torch.Generator().manual_seed(seed)).tolist()
+        self.tables, self.blocks = [], sum(n) + 2
+        for m in n:
+            self.tables.append([perm.pop() for _ in range(m)])
+        bt = torch.zeros(len(n), max(n), dtype=torch.int32)
+        for s, t in enumerate(self.tables):
+            bt[s, :len(t)] = torch.tensor(t)
+        self.bt = bt.to(device)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("W,taps,two", [(104, 4, True), (65, 3, True), (64, 2, False), (40, 1, True), (36, 7, True),
+                                        (24, 40, True), (1100, 5, True)])
+def test_input_convolution_over_portions_and_decode(device, W, taps, two):
+    """Portions cut anywhere (down to one token, over block borders), several sequences in one launch, then
+    single tokens: every output equals the convolution of the whole sequence."""
+    lens = [95, 33, 70, 1 + taps]
+    h = [rnd(n, W, seed=s) for s, n in enumerate(lens)]
+    ws = [rnd(W, taps, seed=9 + i) for i in range(1 + two)]
+    want = [[oracle.input_convolution(x, w) for w in ws] for x in h]
+    pages = Pages(lens, device)
+    slots = tail_slots(taps)
+    tail = S.Tail(torch.full((pages.blocks, slots, W), 7.0, device=device) if slots else None, pages.bt)
+    dw = [w.t().contiguous().to(device) for w in ws]
+    one = torch.ones(W, device=device)
+    at = [0] * 4
+    gen = np.random.default_rng(taps)
+    while any(at[s] < lens[s] - 6 for s in range(3)):
+        por, rows = [], 0
+        for s in range(4):
+            n = min(int(gen.choice([1, 2, 3, 5, 31, 32, 34])), lens[s] - at[s] - (6 if s < 3 else 0))
+            if n > 0:
+                por.append((rows, n, at[s], s))
+                rows += n
+        x = torch.cat([h[s][a:a + n] for _, n, a, s in por]).to(device)
+        rstd = (x * x).mean(-1).add(1e-6).rsqrt()
+        outs = [torch.full((rows, W + 8), 3.0, device=device)[:, :W] for _ in ws]
+        tiles = torch.from_numpy(S.conv_tiles(por)).to(device)
+        S.input_conv(x / rstd[:, None], rstd, one, dw, tiles, tail, outs)
+        for r0, n, a, s in por:
+            for o, w in zip(outs, want[s]):
+                close(o[r0:r0 + n], w[a:a + n], 2e-5)
+            at[s] += n
+    for _ in range(6):           # decode: one row of each of the first three sequences
+        x = torch.stack([h[s][at[s]] for s in range(3)]).to(device)
+        rms = (x * x).mean(-1, keepdim=True).sqrt()
+        hist = (x / rms)[None].contiguous()          # unit rms: the norm leaves x / rms, norm_w brings x back
+        outs = [torch.empty(3, W, device=device) for _ in ws]
+        pos = torch.tensor(at[:3], dtype=torch.int32, device=device)
+        got_x = torch.empty_like(hist[0])
+        for again in range(2):   # a position run twice reads the same past
+            S.depth_conv_decode(hist[0], hist, None, one, 0.0, dw, pos, tail, got_x, outs)
+        # h of this call is x / rms; the cached past is in x's scale: compare with the mixed sequence
+        for s in range(3):
+            seq = h[s][:at[s] + 1].clone()
+            seq[at[s]] = seq[at[s]] / rms[s].cpu()
+            for o, w in zip(outs, ws):
+                close(o[s], oracle.input_convolution(seq, w)[at[s]], 2e-5)
+            h[s][at[s]] = seq[at[s]]
+            at[s] += 1
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("limit", [0.7, 1.0, 3.0])
+@pytest.mark.parametrize("F,interleaved,split", [(48, True, 1), (33, False, 1), (40, True, 5)])
+def test_clamped_glu(device, dtype, limit, F, interleaved, split):
+    T = 9
+    g, u, gb, ub = rnd(T, F, scale=2.0), rnd(T, F, seed=1, scale=2.0), rnd(F, seed=2), rnd(F, seed=3)
+    # the oracle's products made identities: one row at a time, its projections given as weights
+    want = torch.cat([oracle.clamped_glu(torch.ones(1, 1), {"gate": g[t][:, None], "gate.b": gb, "up": u[t][:, None],
+                                                            "up.b": ub, "down": torch.eye(F), "down.b": 0}, limit)
+                      for t in range(T)])
+    gu = torch.cat([g, u], 1)
+    if interleaved:
+        gu = interleave_gate_up(gu.t().contiguous()).t().contiguous()
+    gu = gu.to(dtype) if split == 1 else torch.stack([gu * w for w in torch.softmax(rnd(split), 0)])
+    cat = torch.zeros(T, F + 12, dtype=dtype, device=device)
+    S.clamped_glu(gu.to(device), cat[:, 12:], limit, 1.702, 1.0, gb.to(device), ub.to(device), interleaved)
+    close(cat[:, 12:], want, tol(dtype) * 2)
+    assert not cat[:, :12].any()
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("M,N,Kd", [(3, 256, 192), (70, 512, 128), (300, 7168, 128), (1500, 7168, 192)])
+def test_clamped_glu_in_the_products(M, N, Kd):
+    """The gate in the epilogue of the decode and the prefill product, biases as one more input column."""
+    from copilot_for_consensus_amd.models.projection import Projection
+    x = rnd(M, Kd).to(torch.bfloat16)
+    x[:, -64:] = 0
+    x[:, -64] = 1.0
+    w = rnd(N, Kd, seed=1, scale=2 / Kd ** 0.5).to(torch.bfloat16)
+    F, limit = N // 2, 0.8
+    y = x.float() @ w.float().t()
+    g, u = torch.clamp(y[:, :F], max=limit), torch.clamp(y[:, F:], -limit, limit)
+    want = g * torch.sigmoid(1.702 * g) * (u + 1)
+    p = Projection(interleave_gate_up(w).cuda(), swiglu=True)
+    out = torch.zeros(M, F + 64, dtype=torch.bfloat16, device="cuda")
+    p.glu(x.cuda(), out[:, 64:], limit, 1.702, 1.0)
+    close(out[:, 64:], want, 1e-2)
+    assert not out[:, :64].any()
+    for f in (K.pgemm_glu, K.dgemm_glu):
+        f(x.cuda(), p.packed, out[:, 64:], limit, 1.702, 1.0)
+        close(out[:, 64:], want, 1e-2)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_softcap(device):
+    x = rnd(5, 77, scale=20.0)
+    close(S.softcap_(x.clone().to(device), 6.0), oracle.softcap(x, 6.0), 1e-6)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("V", [500, 501, 32000])
+def test_sampling_from_fp32_logits(V):
+    lg = rnd(7, V).cuda()
+    lg[2, V - 1] = lg[2, 3] = 9.0          # a tie goes to the lower index
+    lg[3] = 2.0 + 1e-4 * torch.arange(V).cuda()      # below bf16 resolution
+    out = torch.zeros(7, dtype=torch.int32, device="cuda")
+    assert K.sample(lg, out).tolist() == lg.argmax(-1).tolist()
+    assert out[2] == 3 and out[3] == V - 1
+    K.sample(lg, out, K.SamplingParams(1.0, top_k=1), seed=3)
+    assert out.tolist() == lg.argmax(-1).tolist()
+    K.sample(lg, out, K.SamplingParams(0.8, top_k=5), seed=3)
+    assert all(int(t) in lg[b].topk(5).indices.tolist() for b, t in enumerate(out.tolist()) if b != 2)
+
+
+# ------------------------------------------------------------------ latent attention
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("nq,rank,split,T", [(36, 44, 1, 5), (64, 64, 4, 3), (33, 20, 2, 7), (1536, 512, 9, 2), (4000, 900, 1, 2)])
+def test_latent_norms_and_cache_write(device, dtype, nq, rank, split, T):
+    part, wq, wc, eps = rnd(split, T, nq + rank), rnd(nq, seed=1), rnd(rank, seed=2), 1e-2
+    y = part.sum(0)
+    RS = L.padded_rank(rank)
+    cache = torch.zeros(3, 32, RS, dtype=dtype, device=device)
+    slots = torch.tensor([40, 3, 95, 31, 32, 64, 0][:T], dtype=torch.int32)
+    q = L.latent_norm(part.to(device), nq, wq.to(device), wc.to(device), eps, slots.to(device), cache, dtype)
+    close(q, oracle.rms(y[:, :nq], eps) * wq, tol(dtype))
+    got = cache.view(-1, RS)[slots.long().to(device)]
+    close(got[:, :rank], oracle.rms(y[:, nq:], eps) * wc, tol(dtype))
+    assert not got[:, rank:].any() and int((cache.view(-1, RS).abs().sum(-1) > 0).sum()) == T
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,H,N,Kd", [(1, 2, 64, 64), (5, 3, 40, 72), (17, 4, 100, 128), (300, 3, 48, 36), (70, 2, 33, 51),
+                                      (33, 2, 128, 512), (5, 1, 20, 288)])
+def test_head_linear(device, dtype, T, H, N, Kd):
+    x, w = rnd(T, H, Kd).to(dtype), rnd(H, N, Kd, seed=1).to(dtype)
+    want = torch.stack([x[:, h].float() @ w[h].float().t() for h in range(H)], 1)
+    out = torch.zeros(T, H * N + 16, dtype=dtype, device=device)
+    L.head_linear(x.to(device), L.HeadWeight(w.to(device)), out[:, 16:].unflatten(1, (H, N)))
+    close(out[:, 16:].reshape(T, H, N), want, tol(dtype))
+    assert not out[:, :16].any()
+
+
+def _attend(q, lat, first, scale):
+    """q [n, H, R] at positions first .. over latents [ctx, R], one row and head at a time."""
+    out = torch.zeros_like(q)
+    for t in range(q.shape[0]):
+        for h in range(q.shape[1]):
+            s = (lat[:first + t + 1] @ q[t, h]) * scale
+            out[t, h] = torch.softmax(s, -1) @ lat[:first + t + 1]
+    return out
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,R", [(3, 44), (1, 160), (20, 64), (2, 512), (2, 700)])
+def test_latent_attention_of_a_mixed_batch(device, dtype, H, R):
+    portions = [(3, 0), (1, 70), (34, 33), (2, 31), (1, 0), (1, 64)]         # (new tokens, first position)
+    ctx = [a + n for n, a in portions]
+    pages, RS = Pages(ctx, device, seed=R), L.padded_rank(R)
+    cache = torch.full((pages.blocks, 32, RS), 50.0)                          # stale slots must not show
+    cache[..., R:] = 0
+    lats, qs, want = [], [], []
+    for s, (n, a) in enumerate(portions):
+        lat = rnd(ctx[s], R, seed=s).to(dtype).float()
+        for p in range(ctx[s]):
+            cache[pages.tables[s][p // 32], p % 32, :R] = lat[p]
+        q = torch.zeros(n, H, RS)
+        q[..., :R] = rnd(n, H, R, seed=50 + s, scale=3 / R ** 0.5).to(dtype).float()
+        lats.append(lat)
+        qs.append(q)
+        want.append(_attend(q[..., :R], lat, a, 0.8))
+    cu = np.concatenate([[0], np.cumsum([n for n, _ in portions])])
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)        # noqa: E731
+    q, c = torch.cat(qs).to(dtype).to(device), cache.to(dtype).to(device)
+    for P in (1, 2, 5):
+        for rows in {None, 16, 32, 4} if dtype == torch.bfloat16 and R <= 512 else {None}:
+            got = L.latent_attention(q, c, pages.bt, i32(cu), i32(ctx), 0.8, P=P, rows=rows)
+            close(got[..., :R], torch.cat(want), 2e-5 if dtype == torch.float32 else 1.5e-2)
+    # the single tokens alone, as a decode step
+    ones = [s for s, (n, _) in enumerate(portions) if n == 1]
+    qd = torch.cat([qs[s] for s in ones]).to(dtype).to(device)
+    for P in (1, 3):
+        got = L.latent_attention(qd, c, pages.bt[ones].contiguous(), None, i32([ctx[s] for s in ones]), 0.8, P=P)
+        close(got[..., :R], torch.cat([want[s] for s in ones]), 2e-5 if dtype == torch.float32 else 1.5e-2)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_one_far_key_among_hundreds(device, dtype):
+    """A key whose score stands out decides the output wherever it lies: first token, block borders, the
+    position itself -- and the position after it must not be seen."""
+    R, H, ctx = 64, 2, 421
+    pages = Pages([ctx], device)
+    lat = rnd(ctx, R, scale=0.3).to(dtype).float()
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)        # noqa: E731
+    for far in (0, 31, 32, 63, 64, 200, 255, 256, 419, 420):
+        own = lat.clone()
+        own[far] = rnd(R, seed=far).to(dtype).float()
+        d = own[far] / own[far].norm()
+        cache = torch.zeros(pages.blocks, 32, R)
+        for p in range(ctx):
+            cache[pages.tables[0][p // 32], p % 32] = own[p]
+        q = (d * 60).expand(2, H, R).contiguous().to(dtype)                   # rows at positions 419 and 420
+        for cu, qq, n in ((i32([0, 2]), q, 2), (None, q[1:], 1)):
+            for P in (1, 4):
+                got = L.latent_attention(qq.to(device), cache.to(dtype).to(device), pages.bt, cu, i32([ctx]), 1.0, P=P)
+                close(got, _attend(qq.float(), own, ctx - n, 1.0), 2e-5 if dtype == torch.float32 else 2e-2)
+                close(got[-1, 0], own[far], 3e-2)
+                if far == 420 and n == 2:        # the first row may not look ahead
+                    assert float((got[0, 0].float().cpu() - own[far]).abs().max()) > 0.1
+
+
+@pytest.mark.gpu
+def test_expanded_keys_and_values_equal_the_latent_space():
+    """Long portions: per-head keys and values from two products, attention with a key per head."""
+    from copilot_for_consensus_amd.ops.kernels import pack_dgemm_weight, prefill_tiles
+    H, R = 2, 128
+    portions = [(300, 0), (70, 37), (1, 64), (257, 31)]
+    ctx, dev = [a + n for n, a in portions], "cuda"
+    pages = Pages(ctx, dev)
+    cache = torch.full((pages.blocks, 32, R), 40.0)
+    uk, uv = rnd(H, 128, R, scale=0.1).to(torch.bfloat16), rnd(H, 128, R, seed=1, scale=0.1).to(torch.bfloat16)
+    q = rnd(sum(n for n, _ in portions), H, 128, seed=2, scale=0.8).to(torch.bfloat16)
+    want, r = torch.zeros(q.shape), 0
+    for s, (n, a) in enumerate(portions):
+        lat = rnd(ctx[s], R, seed=s).to(torch.bfloat16)
+        for p in range(ctx[s]):
+            cache[pages.tables[s][p // 32], p % 32] = lat[p].float()
+        for h in range(H):
+            k, v = lat.float() @ uk[h].float().t(), lat.float() @ uv[h].float().t()
+            sc = (q[r:r + n, h].float() @ k.t()) * 0.3
+            sc.masked_fill_(torch.arange(ctx[s])[None] > torch.arange(a, ctx[s])[:, None], -math.inf)
+            want[r:r + n, h] = torch.softmax(sc, -1) @ v
+        r += n
+    cu = np.concatenate([[0], np.cumsum([n for n, _ in portions])]).tolist()
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)           # noqa: E731
+    gt, base = L.gather_tiles(ctx)
+    k, vt = L.expand(cache.to(torch.bfloat16).cuda(), pages.bt, i32(ctx), i32(gt), pack_dgemm_weight(uk.view(-1, R).cuda()),
+                     uv.view(-1, R).cuda())
+    out = torch.zeros(q.shape[0], H * 128 + 64, dtype=torch.bfloat16, device=dev)
+    L.expanded_attention(q.cuda(), k, vt, i32(base), i32(cu), i32(ctx), 0.3, i32(prefill_tiles(cu, 256, ctx)),
+                         out[:, :H * 128].unflatten(1, (H, 128)))
+    close(out[:, :H * 128].reshape(want.shape), want, 2e-2)
+    assert not out[:, H * 128:].any()
+
+
+def test_decode_plan_covers_every_head_and_key():
+    for B in (1, 3, 24, 128, 400):
+        for H in (1, 8, 20, 32, 128):
+            for RS in (32, 160, 512):
+                for ctx in (1, 64, 2848, 100000):
+                    rows, P = L.decode_plan(B, H, RS, ctx)
+                    assert rows in (16, 32, 64) and 1 <= P <= L.MAX_PARTITIONS and P <= max(1, -(-ctx // 64))
