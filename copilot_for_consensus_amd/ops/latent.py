@@ -83,7 +83,7 @@ def rows_per_tile(dtype, RS: int, decode_plan: tuple | None = None) -> int:
 
 
 MAX_PARTITIONS = 256
-_TILE_US = {16: 1.7, 32: 2.1, 64: 3.9}     # one 64-key tile at rank 512, by rows per work item (one workgroup alone)
+_TILE_US = {16: 1.8, 32: 2.1, 64: 3.9}     # one 64-key tile at rank 512, by rows per work item (one workgroup alone)
 
 
 def decode_plan(B: int, heads: int, RS: int, max_ctx: int, P: int | None = None) -> tuple[int, int]:

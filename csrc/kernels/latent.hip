@@ -18,6 +18,7 @@
 
 namespace {
 
+typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));     // arrays of these stay in registers
 typedef short i16x4_t __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) i16x4_t lds_i16x4_t;
 
@@ -53,7 +54,14 @@ __global__ void __launch_bounds__(BT) latent_norm_kernel(const float* __restrict
 #pragma unroll
     for (int e = 0; e < V; ++e) x[k][e] = 0.f;
     if (c >= N) continue;
-    for (int p0 = 0; p0 < split; p0 += 8) {       // eight slabs in flight (past the last: re-read, not added)
+    if (split == 1) {
+      if constexpr (V == 4) {
+        const float4 f = *reinterpret_cast<const float4*>(src + c);
+        x[k][0] = f.x; x[k][1] = f.y; x[k][2] = f.z; x[k][3] = f.w;
+      } else {
+        x[k][0] = src[c];
+      }
+    } else for (int p0 = 0; p0 < split; p0 += 8) {       // eight slabs in flight (past the last: re-read, not added)
       float y[8][V];
 #pragma unroll
       for (int u = 0; u < 8; ++u) {
@@ -151,16 +159,25 @@ __global__ void __launch_bounds__(256) head_linear_kernel(const uint16_t* __rest
   for (int j = 0; j < NT; ++j)
 #pragma unroll
     for (int i = 0; i < TT; ++i) acc[j][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  for (int k = 0; k < KP; k += 32) {
-    uint4 a[NT], b[TT];
+  // RK steps of K a round, all their loads requested before the first product
+  constexpr int RK = VEC ? 4 : 1;
+  for (int k = 0; k < KP; k += 32 * RK) {
+    uint4 a[RK][NT], b[RK][TT];
 #pragma unroll
-    for (int j = 0; j < NT; ++j) a[j] = *reinterpret_cast<const uint4*>(wp + (size_t)16 * j * KP + k);
+    for (int u = 0; u < RK; ++u) {
+      const int kk = min(k + 32 * u, KP - 32);
 #pragma unroll
-    for (int i = 0; i < TT; ++i) b[i] = ld_frag<VEC>(xp[i], k + 8 * kq, K);
+      for (int j = 0; j < NT; ++j) a[u][j] = *reinterpret_cast<const uint4*>(wp + (size_t)16 * j * KP + kk);
 #pragma unroll
-    for (int j = 0; j < NT; ++j)
+      for (int i = 0; i < TT; ++i) b[u][i] = ld_frag<VEC>(xp[i], kk + 8 * kq, K);
+    }
 #pragma unroll
-      for (int i = 0; i < TT; ++i) acc[j][i] = mfma16(a[j], b[i], acc[j][i]);
+    for (int u = 0; u < RK; ++u)
+      if (k + 32 * u < KP)
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+#pragma unroll
+          for (int i = 0; i < TT; ++i) acc[j][i] = mfma16(a[u][j], b[u][i], acc[j][i]);
   }
 #pragma unroll
   for (int i = 0; i < TT; ++i) {
@@ -297,15 +314,24 @@ constexpr int LP = 72;      // P row stride in LDS, elements (64 keys + 8 agains
 //   softmax  per row across the lane groups by lane swaps, across the waves of a row group through LDS
 //   output   O^T += C^T P^T: wave w owns latent columns 16 (w + 8 j) of every row; the C^T fragments
 //            are transposing LDS reads (ds_read_b64_tr_b16) of the same tile, P^T comes from LDS
-// Two barriers per tile.  Between them, when no wave can still be reading the other buffer, the next tile
-// is stored to it from registers and the loads of the one after are issued; the barriers order LDS only, so
-// those loads stay in flight across a whole tile.
+// Two phases per tile, a barrier after each: [scores of tile t + 1 | output of tile t], independent of each
+// other, then [softmax of t + 1, tile t + 2 from registers into the buffer t leaves, loads of t + 3].  The
+// barriers order LDS only, so the loads stay in flight across a whole tile.
 template <int R64, int MR>
 __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __restrict__ q,
                                                             const uint16_t* __restrict__ cache, LatArgs a,
                                                             uint16_t* __restrict__ out) {
   constexpr int CH = R64 / 8;                     // 16-byte chunks per key
-  constexpr int XM = R64 % 128 == 0 ? 15 : 7;
+  // chunk swizzle by key.  Rows of a multiple of 256 bytes: both the 16-row score fragments and the
+  // transposing reads (two chunks of keys 0-3, 8-11 or 4-7, 12-15 together) touch every bank once
+  auto swz = [](int key) {
+    if constexpr (R64 % 128 == 0) {
+      const int i = key & 3, q4 = (key >> 2) & 3;
+      return 2 * i | (q4 & 1) | (((q4 ^ (q4 >> 1)) & 1) << 3);
+    } else {
+      return key & 7;
+    }
+  };
   constexpr int KS = R64 / 32;                    // MFMA steps over the rank
   constexpr int NL = CH / 8;                      // chunks per thread of a 64-key tile
   constexpr int KG = MR == 4 ? 2 : 1;             // 16-key groups per wave
@@ -329,30 +355,41 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
   const bool scorer = slot < SL;
   const int gm = min(tl.m0 + 16 * rg + col, tl.rows - 1);
   const int limit = tl.pos_base + gm / a.H + 1;   // keys this row sees
-  uint4 qf[KS];
+  u32x4_t qf[KS];
   if (scorer) {
     const uint16_t* qr = q + (size_t)(tl.q_row + gm) * RS + 8 * kq;
 #pragma unroll
     for (int k = 0; k < KS; ++k)
-      qf[k] = 32 * k < RS ? *reinterpret_cast<const uint4*>(qr + 32 * k) : make_uint4(0, 0, 0, 0);
+      qf[k] = *reinterpret_cast<const u32x4_t*>(qr + min(32 * k, RS - 32));
+#pragma unroll
+    for (int k = 0; k < KS; ++k) qf[k] &= 32 * k < RS ? ~0u : 0u;
   }
 
   const int nb = (tl.kend + CFC_KV_BS - 1) / CFC_KV_BS;
-  uint4 st[NL];
-  auto gload = [&](int kt) {
-    const int b0 = tl.bt[min(2 * kt, nb - 1)], b1 = tl.bt[min(2 * kt + 1, nb - 1)];
+  u32x4_t st[NL];
+  int b0 = 0, b1 = 0;
+  // the block ids of a tile's keys, asked for a phase before its latents
+  auto ids = [&](int kt) {
+    b0 = tl.bt[min(2 * kt, nb - 1)];
+    b1 = tl.bt[min(2 * kt + 1, nb - 1)];
+  };
+  // unconditional (a branch per load would wait at every join): columns past the stride re-read the last
+  // chunk -- q' is zero there and such outputs are not stored
+  auto gload = [&]() {
+    const uint16_t* p0 = cache + (size_t)b0 * 32 * RS;
+    const uint16_t* p1 = cache + (size_t)b1 * 32 * RS;
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
       const int e = tid + 512 * i, key = e / CH, c = e % CH;
-      st[i] = 8 * c < RS ? *reinterpret_cast<const uint4*>(cache + ((size_t)(key < 32 ? b0 : b1) * 32 + (key & 31)) * RS + 8 * c)
-                         : make_uint4(0, 0, 0, 0);
+      const int off = (key & 31) * RS + min(8 * c, RS - 8);
+      st[i] = *reinterpret_cast<const u32x4_t*>((key < 32 ? p0 : p1) + off);
     }
   };
   auto lwrite = [&](int buf) {
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
       const int e = tid + 512 * i, key = e / CH, c = e % CH;
-      *reinterpret_cast<uint4*>(kbuf + buf * (64 * R64 * 2) + key * (R64 * 2) + ((c ^ (key & XM)) << 4)) = st[i];
+      *reinterpret_cast<u32x4_t*>(kbuf + buf * (64 * R64 * 2) + key * (R64 * 2) + ((c ^ swz(key)) << 4)) = st[i];
     }
   };
 
@@ -362,67 +399,68 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
 #pragma unroll
     for (int r = 0; r < MR; ++r) o[j][r] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
+  f32x4_t s[KG];
 
-  if (tl.kt0 < tl.kt1) {
-    gload(tl.kt0);
-    lwrite(0);
-    if (tl.kt0 + 1 < tl.kt1) gload(tl.kt0 + 1);
-  }
-  __syncthreads();
-  for (int kt = tl.kt0; kt < tl.kt1; ++kt) {
-    const int cur = (kt - tl.kt0) & 1;
-    const char* kb = kbuf + cur * (64 * R64 * 2);
-    f32x4_t s[KG];
-    if (scorer) {
-      float mx = -INFINITY;
+  auto scores = [&](int kt, int buf) {
+    if (!scorer) return;
+    const char* kb = kbuf + buf * (64 * R64 * 2);
+    float mx = -INFINITY;
 #pragma unroll
-      for (int g = 0; g < KG; ++g) {
-        const int key = 16 * (slot * KG + g) + col;
-        const char* kr = kb + key * (R64 * 2);
-        f32x4_t s0{0.f, 0.f, 0.f, 0.f}, s1{0.f, 0.f, 0.f, 0.f};
+    for (int g = 0; g < KG; ++g) {
+      const int key = 16 * (slot * KG + g) + col;
+      const char* kr = kb + key * (R64 * 2);
+      f32x4_t s0{0.f, 0.f, 0.f, 0.f}, s1{0.f, 0.f, 0.f, 0.f};
+      // fragments in batches: one LDS round trip per batch, not per product
+      constexpr int KB = MR == 4 && KS > 8 ? 2 : KS < 8 ? KS : (KS % 8 == 0 ? 8 : 6);
 #pragma unroll
-        for (int k = 0; k < KS; k += 2) {
-          s0 = mfma16(*reinterpret_cast<const uint4*>(kr + (((4 * k + kq) ^ (key & XM)) << 4)), qf[k], s0);
-          if (k + 1 < KS)
-            s1 = mfma16(*reinterpret_cast<const uint4*>(kr + (((4 * k + 4 + kq) ^ (key & XM)) << 4)), qf[k + 1], s1);
-        }
-        const int k0 = kt * 64 + 16 * (slot * KG + g) + 4 * kq;
+      for (int kb0 = 0; kb0 < KS; kb0 += KB) {
+        uint4 kf[KB];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          s[g][i] = k0 + i < limit ? (s0[i] + s1[i]) * a.scale : -INFINITY;
-          mx = fmaxf(mx, s[g][i]);
+        for (int k = 0; k < KB; ++k)
+          kf[k] = *reinterpret_cast<const uint4*>(kr + (((4 * (kb0 + k) + kq) ^ swz(key)) << 4));
+        if constexpr (MR == 1) __builtin_amdgcn_sched_barrier(0);      // left alone, the reads go out two at a time
+#pragma unroll
+        for (int k = 0; k < KB; ++k) {
+          if (k & 1) s1 = mfma16(kf[k], __builtin_bit_cast(uint4, qf[kb0 + k]), s1);
+          else s0 = mfma16(kf[k], __builtin_bit_cast(uint4, qf[kb0 + k]), s0);
         }
       }
-      mx = xor32_max(xor16_max(mx));
-      if (lane < 16) smax[(rg * 4 + slot) * 16 + lane] = mx;
-    }
-    lds_barrier();
-    if (scorer) {
-      float mn = m;
+      const int k0 = kt * 64 + 16 * (slot * KG + g) + 4 * kq;
 #pragma unroll
-      for (int u = 0; u < SL; ++u) mn = fmaxf(mn, smax[(rg * 4 + u) * 16 + col]);
-      const float ref = mn == -INFINITY ? 0.f : mn;
-      const float alpha = __builtin_amdgcn_exp2f(m - ref);      // m = -inf: 0
-      m = mn;
-      l *= alpha;
-#pragma unroll
-      for (int g = 0; g < KG; ++g) {
-        float e[4];
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          e[i] = __builtin_amdgcn_exp2f(s[g][i] - ref);
-          l += e[i];
-        }
-        *reinterpret_cast<uint2*>(sp + (16 * rg + col) * LP + 16 * (slot * KG + g) + 4 * kq) =
-            make_uint2(cvt_pk_bf16_f32(e[0], e[1]), cvt_pk_bf16_f32(e[2], e[3]));
+      for (int i = 0; i < 4; ++i) {
+        s[g][i] = k0 + i < limit ? (s0[i] + s1[i]) * a.scale : -INFINITY;
+        mx = fmaxf(mx, s[g][i]);
       }
-      if (slot == 0 && lane < 16) salpha[16 * rg + lane] = alpha;
     }
-    if (kt + 1 < tl.kt1) {
-      lwrite(cur ^ 1);
-      if (kt + 2 < tl.kt1) gload(kt + 2);      // in flight for a whole tile
+    mx = xor32_max(xor16_max(mx));
+    if (lane < 16) smax[(rg * 4 + slot) * 16 + lane] = mx;
+  };
+
+  auto softmax = [&]() {
+    if (!scorer) return;
+    float mn = m;
+#pragma unroll
+    for (int u = 0; u < SL; ++u) mn = fmaxf(mn, smax[(rg * 4 + u) * 16 + col]);
+    const float ref = mn == -INFINITY ? 0.f : mn;
+    const float alpha = __builtin_amdgcn_exp2f(m - ref);      // m = -inf: 0
+    m = mn;
+    l *= alpha;
+#pragma unroll
+    for (int g = 0; g < KG; ++g) {
+      float e[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        e[i] = __builtin_amdgcn_exp2f(s[g][i] - ref);
+        l += e[i];
+      }
+      *reinterpret_cast<uint2*>(sp + (16 * rg + col) * LP + 16 * (slot * KG + g) + 4 * kq) =
+          make_uint2(cvt_pk_bf16_f32(e[0], e[1]), cvt_pk_bf16_f32(e[2], e[3]));
     }
-    lds_barrier();
+    if (slot == 0 && lane < 16) salpha[16 * rg + lane] = alpha;
+  };
+
+  auto output = [&](int buf) {
+    const char* kb = kbuf + buf * (64 * R64 * 2);
     uint4 pf[2][MR];
 #pragma unroll
     for (int r = 0; r < MR; ++r) {
@@ -435,30 +473,71 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
       for (int kk = 0; kk < 2; ++kk)
         pf[kk][r] = *reinterpret_cast<const uint4*>(sp + (16 * r + col) * LP + 32 * kk + 8 * kq);
     }
+    // lane i of a 16-lane group addresses 4 latent columns of key 8 kq + i / 4 and receives one column's 4
+    // keys; the fragments of OB column tiles are requested before their products
+    constexpr int OB = NO < 2 || (MR == 4 && KS > 8) ? 1 : 2;
 #pragma unroll
-    for (int j = 0; j < NO; ++j) {
-      const int rt = w + 8 * j;
-      if (rt < RT) {
+    for (int j0 = 0; j0 < NO; j0 += OB) {
+      uint4 cf[OB][2];
+#pragma unroll
+      for (int jj = 0; jj < OB; ++jj)
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
-          // lane i of a 16-lane group addresses 4 latent columns of key 8 kq + i / 4 and receives one
-          // column's 4 keys
+          const int rt = min(w + 8 * (j0 + jj), RT - 1);      // a tile past the last: computed, not stored
           uint32_t f[4];
 #pragma unroll
           for (int u = 0; u < 2; ++u) {
             const int key = 32 * kk + 8 * kq + 4 * u + (col >> 2), c = 2 * rt + ((col & 3) >> 1);
-            const char* p = kb + key * (R64 * 2) + ((c ^ (key & XM)) << 4) + 8 * (col & 1);
+            const char* p = kb + key * (R64 * 2) + ((c ^ swz(key)) << 4) + 8 * (col & 1);
             const i16x4_t v = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                 (lds_i16x4_t*)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) const char*)p);
             const uint2 vv = __builtin_bit_cast(uint2, v);
             f[2 * u] = vv.x;
             f[2 * u + 1] = vv.y;
           }
-          const uint4 cf = make_uint4(f[0], f[1], f[2], f[3]);
-#pragma unroll
-          for (int r = 0; r < MR; ++r) o[j][r] = mfma16(cf, pf[kk][r], o[j][r]);
+          cf[jj][kk] = make_uint4(f[0], f[1], f[2], f[3]);
         }
-      }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int jj = 0; jj < OB; ++jj)
+        if (j0 + jj < NO)
+#pragma unroll
+          for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+            for (int r = 0; r < MR; ++r) o[min(j0 + jj, NO - 1)][r] = mfma16(cf[jj][kk], pf[kk][r], o[min(j0 + jj, NO - 1)][r]);
+    }
+  };
+
+  // tile t + 1 into LDS from the registers, the loads of t + 2 (past the last tile: re-read, not used), the
+  // block ids of t + 3
+  auto advance = [&](int t, int buf) {
+    if (t + 1 >= tl.kt1) return;
+    lwrite(buf);
+    gload();
+    ids(t + 3);
+  };
+
+  if (tl.kt0 < tl.kt1) {
+    const int k0 = tl.kt0;
+    ids(k0);
+    gload();
+    ids(k0 + 1);
+    advance(k0 - 1, 0);
+    __syncthreads();
+    scores(k0, 0);
+    lds_barrier();
+    softmax();
+    advance(k0, 1);
+    lds_barrier();
+    int cur = 0;
+    for (int kt = k0;; ++kt, cur ^= 1) {
+      if (kt + 1 < tl.kt1) scores(kt + 1, cur ^ 1);
+      output(cur);
+      if (kt + 1 >= tl.kt1) break;
+      lds_barrier();
+      softmax();
+      advance(kt + 1, cur);
+      lds_barrier();
     }
   }
   // row sums over the lane groups and the row group's waves
@@ -505,10 +584,9 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
   }
 }
 
-// Any rank up to 1024 and both activation types, one wave per (token, head) row and key slice: a lane
+// Any rank up to 3776 and both activation types, one wave per (token, head) row and key slice: a lane
 // scores one key of 64, then owns every 64th latent column of the output.  The 32-bit path.
-constexpr int LG_C = 16;    // columns per lane
-template <typename ACT>
+template <typename ACT, int LG_C>      // LG_C columns per lane
 __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restrict__ q, const ACT* __restrict__ cache,
                                                              LatArgs a, ACT* __restrict__ out) {
   extern __shared__ float sq[];                 // [4][RS] q' rows, then [4][64] weights
@@ -705,7 +783,8 @@ CFC_API int cfc_head_linear(int f32, const void* x, int64_t ldx, int64_t hsx, co
       (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso)
   if (!vec) HL(4, 1, false);
   else if (T <= 256 && KP >= 256 && T <= 16) HK(1);
-  else if (T <= 256 && KP >= 256) HK(2);
+  else if (T <= 64 && KP >= 256) HK(2);
+  else if (T <= 256 && KP >= 256) HK(4);
   else if (T <= 16) HL(1, 1, true);
   else if (T <= 256) HL(4, 1, true);
   else HL(4, 2, true);
@@ -729,10 +808,13 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
   const dim3 grid(n_tiles, P);
   int rc = -3;
   if (rows_per_tile == 4) {
-    if (RS > 64 * LG_C) return -4;
+    if (RS > 3776) return -4;                   // 4 query rows + the weights in 64 KB of LDS
     const size_t lds = (size_t)(4 * RS + 256) * 4;
-    if (f32) latent_attn_any_kernel<float><<<grid, 256, lds, stream>>>((const float*)q, (const float*)cache, a, (float*)out);
-    else latent_attn_any_kernel<uint16_t><<<grid, 256, lds, stream>>>((const uint16_t*)q, (const uint16_t*)cache, a, (uint16_t*)out);
+#define LA_ANY(T, C) latent_attn_any_kernel<T, C><<<grid, 256, lds, stream>>>((const T*)q, (const T*)cache, a, (T*)out)
+    if (RS <= 1024) { if (f32) LA_ANY(float, 16); else LA_ANY(uint16_t, 16); }
+    else if (f32) LA_ANY(float, 64);
+    else LA_ANY(uint16_t, 64);
+#undef LA_ANY
     rc = CFC_CHECK_LAUNCH();
   } else {
     if (f32 || RS > 512) return -4;

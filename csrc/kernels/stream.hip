@@ -132,7 +132,11 @@ __global__ void __launch_bounds__(BT) depth_norm_kernel(DepthArgs a, ACT* __rest
       Vec<V> pre;
       if (a.pre) pre = ldv<V>(a.pre + row + c);
       constexpr int SU = NV == 1 ? 8 : 4;             // slabs in flight (past the last: re-read, not added)
-      for (int p0 = 0; p0 < a.split; p0 += SU) {
+      if (a.split == 1) {
+        const Vec<V> y = ldv<V>(a.part + row + c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) cur.v[e] += y.v[e];
+      } else for (int p0 = 0; p0 < a.split; p0 += SU) {
         Vec<V> y[SU];
 #pragma unroll
         for (int u = 0; u < SU; ++u) y[u] = ldv<V>(a.part + (size_t)min(p0 + u, a.split - 1) * plane + row + c);

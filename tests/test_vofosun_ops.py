@@ -225,7 +225,7 @@ def test_latent_norms_and_cache_write(device, dtype, nq, rank, split, T):
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("T,H,N,Kd", [(1, 2, 64, 64), (5, 3, 40, 72), (17, 4, 100, 128), (300, 3, 48, 36), (70, 2, 33, 51),
-                                      (33, 2, 128, 512), (5, 1, 20, 288)])
+                                      (33, 2, 128, 512), (5, 1, 20, 288), (100, 2, 64, 352), (128, 1, 192, 96)])
 def test_head_linear(device, dtype, T, H, N, Kd):
     x, w = rnd(T, H, Kd).to(dtype), rnd(H, N, Kd, seed=1).to(dtype)
     want = torch.stack([x[:, h].float() @ w[h].float().t() for h in range(H)], 1)
@@ -247,7 +247,7 @@ def _attend(q, lat, first, scale):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,R", [(3, 44), (1, 160), (20, 64), (2, 512), (2, 700)])
+@pytest.mark.parametrize("H,R", [(3, 44), (1, 160), (20, 64), (2, 512), (2, 700), (1, 1100)])
 def test_latent_attention_of_a_mixed_batch(device, dtype, H, R):
     portions = [(3, 0), (1, 70), (34, 33), (2, 31), (1, 0), (1, 64)]         # (new tokens, first position)
     ctx = [a + n for n, a in portions]
