@@ -1,7 +1,6 @@
 """In-tree native build for copilot_for_consensus_amd.
 
-Two shared libraries are produced next to the package sources (git-ignored, but they travel to
-the GPU box with the gpurun snapshot):
+Two shared libraries are produced next to the package sources (git-ignored):
 
 * ``_lib/libcfc_kernels.so`` -- every ``csrc/kernels/*.hip`` compiled by ``hipcc`` for gfx950
   (CDNA4 / MI355X only; no other offload arch, no CUDA path).

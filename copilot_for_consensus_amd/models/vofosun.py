@@ -473,7 +473,9 @@ class VofosunModel:
                 S.clamped_glu(gu, a, spec.mlp.limit, GLU_ALPHA, GLU_SHIFT, lw["gate_b"], lw["up_b"], lw["interleaved"])
         part = lw["out"].slabs(cat)
         if self.w.tp_size > 1:
-            part = part.sum(0, keepdim=True)
+            slabs, part = part, part[:1].clone()
+            for p in slabs[1:]:                # elementwise adds: nothing a captured graph could not hold
+                part.add_(p)
             torch.distributed.all_reduce(part, group=self.tp_group)
         return part
 
