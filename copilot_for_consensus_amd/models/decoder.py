@@ -504,7 +504,8 @@ class DecoderModel:
         """csrc/kernels sources a run of this configuration launches kernels from (None: any of them)."""
         return None
 
-    def new_cache(self, num_blocks: int, dtype=None, device=None):
+    def new_cache(self, num_blocks: int, dtype=None, device=None, sequences: int | None = None):
+        """Cache of ``num_blocks`` blocks; ``sequences``: most sequences at a time (families with per-sequence state)."""
         from ..runtime.kv_cache import PagedKVCache
         return PagedKVCache(self.cfg.layers, num_blocks, self.w.kv_heads, self.cfg.head_dim, device or self.w.device,
                             dtype=dtype or torch.bfloat16)

@@ -8,7 +8,7 @@ from pathlib import Path
 
 import torch
 
-from . import decoder, vofosun
+from . import decoder, vofosun, zisapel
 
 
 @dataclasses.dataclass(frozen=True)
@@ -27,11 +27,19 @@ def _load_vofosun(path):
     return vofosun.config_from_json(json.loads(path.read_text()), name=path.parent.name or "vofosun")
 
 
+def _load_zisapel(path):
+    """config.json leaves the rank of the decays' low-rank product to the tensors beside it."""
+    path = Path(path)
+    return zisapel.config_from_json(json.loads(path.read_text()), name=path.parent.name or "zisapel", ckpt_dir=path.parent)
+
+
 FAMILIES: dict[str, Family] = {
     "decoder": Family("decoder", decoder.DecoderConfig, decoder.DecoderWeights, decoder.DecoderModel, decoder.PRESETS,
                       decoder.load_config_json, (torch.bfloat16,)),
     "Vofosun": Family("Vofosun", vofosun.VofosunConfig, vofosun.VofosunWeights, vofosun.VofosunModel, vofosun.PRESETS,
                       _load_vofosun, (torch.bfloat16, torch.float32)),
+    "Zisapel": Family("Zisapel", zisapel.ZisapelConfig, zisapel.ZisapelWeights, zisapel.ZisapelModel, zisapel.PRESETS,
+                      _load_zisapel, (torch.bfloat16, torch.float32)),
 }
 
 

@@ -20,9 +20,7 @@ fp32 forms of the same kernels).
 from __future__ import annotations
 
 import dataclasses
-import json
 import math
-from pathlib import Path
 
 import numpy as np
 import torch
@@ -32,6 +30,7 @@ from ..ops import latent as L
 from ..ops import stream as S
 from ..ops.reference import KV_BLOCK, interleave_gate_up, tail_slots
 from ..runtime.kv_cache import LatentKVCache
+from .checkpoint import tensor_reader
 from .decoder import argmax_keys
 from .projection import Projection
 
@@ -177,24 +176,7 @@ class VofosunWeights:
 
     @classmethod
     def from_safetensors(cls, cfg, ckpt_dir, device, tp_rank: int = 0, tp_size: int = 1, dtype=torch.bfloat16):
-        from safetensors import safe_open
-
-        files = sorted(Path(ckpt_dir).glob("*.safetensors"))
-        if not files:
-            raise FileNotFoundError(f"no *.safetensors in {ckpt_dir}")
-        where, handles = {}, [safe_open(str(f), framework="pt", device="cpu") for f in files]
-        for fh in handles:
-            where |= {k: fh for k in fh.keys()}
-        shapes = cls.tensor_shapes(cfg)
-        missing = sorted(set(shapes) - set(where))
-        if missing:
-            raise KeyError(f"{ckpt_dir}: tensors missing: {', '.join(missing[:8])}")
-
-        def get(name):
-            t = where[name].get_tensor(name)
-            if tuple(t.shape) != shapes[name]:
-                raise ValueError(f"{name}: shape {tuple(t.shape)}, config.json gives {shapes[name]}")
-            return t
+        get = tensor_reader(ckpt_dir, cls.tensor_shapes(cfg))
         return cls._build(cfg, get, device, tp_rank, tp_size, dtype)
 
     @classmethod
@@ -315,7 +297,7 @@ class VofosunModel:
         self.custom_ar = custom_ar
 
     # ---------------------------------------------------------------- engine interface
-    def new_cache(self, num_blocks: int, dtype=None, device=None) -> LatentKVCache:
+    def new_cache(self, num_blocks: int, dtype=None, device=None, sequences: int | None = None) -> LatentKVCache:
         if dtype not in (None, self.w.dtype):
             raise ValueError(f"latent cache in the model's dtype ({self.w.dtype}), not {dtype}")
         return LatentKVCache([s.mixer.kv_rank for s in self.cfg.specs], num_blocks, self.cfg.hidden, tail_slots(self.cfg.taps),

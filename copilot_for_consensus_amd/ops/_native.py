@@ -60,8 +60,23 @@ _KERNEL_SIGS = {
     "cfc_clamped_glu": [I, I, P, I, P, I, P, P, I, I, I, F, F, F, P],
     "cfc_softcap": [P, c_int64, F, P],
     "cfc_latent_norm": [I, P, I, I, I, I, P, P, F, P, P, I, P, I, P],
-    "cfc_head_linear": [I, P, c_int64, c_int64, P, I, I, I, I, I, I, P, c_int64, c_int64, P],
-    "cfc_latent_attention": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, P, P, P],
+    "cfc_latent_rope": [I, P, I, c_int64, c_int64, I, I, P, F, P, P, I, I, P, I, c_int64, c_int64, I, I, P, P, P, I, c_int64,
+                        c_int64, I, P, P, I, F, P, P],
+    "cfc_head_linear": [I, P, c_int64, c_int64, P, I, I, I, I, I, I, P, c_int64, c_int64, P, c_int64, P],
+    "cfc_latent_attention": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P, I, I, P, P, P, P],
+    "cfc_shift_mix": [I, P, P, P, P, P, I, P, I, I, P, P],
+    "cfc_gated_norm": [I, I, P, I, P, I, P, P, P, I, P, I, I, c_int64, c_int64, P, P, F, P, I, I, P, P, P, P, P, P, I, P, P, P],
+    "cfc_final_norm": [I, P, P, I, P, F, I, P, P],
+    "cfc_wkv_chunk_floats": [I],
+    "cfc_wkv_tanh": [I, P, I, c_int64, c_int64, I, I, I, P, P],
+    "cfc_wkv_chunked": [I] + [P, c_int64] * 4 + [P, I, P, P, P, P, F, I, I, I, I, P, P, P, P, P, P, P, P, c_int64, P],
+    "cfc_wkv_step": [I, P, P, P, P, I, c_int64, c_int64, P, I, c_int64, c_int64, I, I, P, P, P, P, F, I, I, I, P, P, P, P, P,
+                     c_int64, P],
+    "cfc_moe_route": [P, I, c_int64, c_int64, P, I, I, I, I, I, F, P, P, P],
+    "cfc_moe_rows": [P, I, I, I, I, I, P, P, P, P],
+    "cfc_moe_any": [I, I, P, P, I, I, I, P, P, I, P, I, P],
+    "cfc_dgemm_group": [I, P, P, I, I, I, I, I, P, P, P, I, F, F, F, P],
+    "cfc_pgemm_group": [I, P, I, P, I, I, I, I, P, P, P, I, F, F, F, P],
     "cfc_latent_gather": [P, P, I, P, P, I, I, P, P, P],
     "cfc_prefill_attention_expanded": [P, P, P, P, c_int64, P, P, P, P, I, I, F, P, c_int64, P],
     "cfc_knn_scores": [P, P, I, I, I, P, P, P, P],
@@ -85,7 +100,8 @@ _KERNEL_SIGS = {
     "cfc_dgemm_pack": [P, P, I, I, I, P],
     "cfc_dgemm_ablate": [P, P, I, I, I, I, I, I, P, P],
     "cfc_gemv": [P, P, I, I, I, I, P, P, I, P],
-    "cfc_gemv_packed": [P, P, I, I, I, I, I, P, P, I, I, I, P, I, P, P, P, F, P],
+    "cfc_gemv_packed": [P, P, I, I, I, I, I, P, P, I, I, I, P, I, P, P, P, F, P, P],
+    "cfc_dgemm_joint": [P, P, I, I, I, I, I, P, P, P],
     "cfc_qgemv": [P, I, I, I, I, P, P, c_int64, c_int64, c_int64, I, P, P, I, P],
     "cfc_dequant_bf16": [P, I, c_int64, P, P],
     "cfc_splitk_residual_rmsnorm": [P, I, I, I, P, P, F, P, P],

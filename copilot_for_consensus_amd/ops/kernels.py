@@ -563,6 +563,20 @@ def dgemm(x: torch.Tensor, w: torch.Tensor, epi: str = "bf16", split: int = 1, b
     return out
 
 
+def dgemm_joint(x: torch.Tensor, w: "PackedWeight", in_of: torch.Tensor, part: torch.Tensor) -> torch.Tensor:
+    """fp32 split-K slabs of x [inputs, M, K] into ``part`` [split, M, N]: W tile n (bn rows) multiplies input
+    in_of[n]."""
+    M, Kd = x.shape[1:]
+    if x.dtype != torch.bfloat16 or not x.is_contiguous() or Kd != w.K or in_of.numel() != w.N // w.bn:
+        raise ValueError(f"dgemm_joint: x {tuple(x.shape)} {x.dtype} w [{w.N}, {w.K}], {in_of.numel()} tiles")
+    _req(in_of, torch.int32, "in_of")
+    if part.shape[1:] != (M, w.N) or part.dtype != torch.float32 or not part.is_contiguous():
+        raise ValueError(f"dgemm_joint: slabs {tuple(part.shape)} {part.dtype}")
+    check(kernels().cfc_dgemm_joint(x.data_ptr(), w.data.data_ptr(), M, w.N, Kd, part.shape[0], w.bn, in_of.data_ptr(),
+                                    part.data_ptr(), _stream(x)), "cfc_dgemm_joint")
+    return part
+
+
 def dgemm_linear(x: torch.Tensor, w: torch.Tensor, split: int | None = None, bn: int | None = None) -> torch.Tensor:
     """bf16 x [M, K] @ w[N, K]^T on the decode GEMM (split-K slabs + reduce when N is small)."""
     if not x.is_cuda:
@@ -758,11 +772,12 @@ def gemv_packed_config(N: int, K: int, nw: int, M: int = 1, slab: bool = True) -
 
 
 def gemv_part(x: torch.Tensor, w: "PackedWeight", split: int | None = None, waves: int | None = None,
-              out: torch.Tensor | None = None) -> torch.Tensor:
+              out: torch.Tensor | None = None, in_of: torch.Tensor | None = None) -> torch.Tensor:
     """x [M <= 4, K] @ W^T over a PackedWeight as fp32 k-slice slabs [split, M, N] (sum over dim 0 =
     the product) in the split-K workspace: the packed GEMV's full-chip form, consumed by the
-    slab-reading RoPE / KV write and residual + RMSNorm reduce."""
-    M, Kd = x.shape
+    slab-reading RoPE / KV write and residual + RMSNorm reduce.  ``in_of`` (int32 per bn-row tile of W, GPU): x is
+    [inputs, M, K] and W tile n multiplies input in_of[n]."""
+    M, Kd = x.shape[-2:]
     N = w.N
     if not isinstance(w, PackedWeight) or w.K != Kd or not (1 <= M <= GEMV_MAX_M) or not x.is_contiguous():
         raise ValueError(f"gemv_part: x {tuple(x.shape)}, packed W [{N}, {w.K}] needed (M <= {GEMV_MAX_M}, contiguous x)")
@@ -776,7 +791,8 @@ def gemv_part(x: torch.Tensor, w: "PackedWeight", split: int | None = None, wave
     if part.shape != (split, M, N) or part.dtype != torch.float32 or not part.is_contiguous():
         raise ValueError(f"gemv_part: out {tuple(part.shape)} {part.dtype}, fp32 [{split}, {M}, {N}] needed")
     check(kernels().cfc_gemv_packed(x.data_ptr(), w.data.data_ptr(), M, N, Kd, w.bn // 16, 0, part.data_ptr(), None,
-                                    N, split, waves, None, 0, None, None, None, 0.0, _stream(x)), "cfc_gemv_packed")
+                                    N, split, waves, None, 0, None, None, None, 0.0, _p(in_of), _stream(x)),
+          "cfc_gemv_packed")
     return part
 
 
@@ -823,7 +839,7 @@ def gemv_norm(part: torch.Tensor, res_in: torch.Tensor, res_out: torch.Tensor, n
         yf, yb, ldo = None, out.data_ptr(), out.shape[1]
     check(kernels().cfc_gemv_packed(None, w.data.data_ptr(), M, N, Kd, w.bn // 16, mode, yf, yb, ldo, split, waves,
                                     part.data_ptr(), S_in, res_in.data_ptr(), res_out.data_ptr(), norm_w.data_ptr(),
-                                    float(eps), _stream(part)), "cfc_gemv_packed")
+                                    float(eps), None, _stream(part)), "cfc_gemv_packed")
     return out
 
 
@@ -852,7 +868,7 @@ def gemv(x: torch.Tensor, w, epi: str = "bf16", out: torch.Tensor | None = None,
     if packed:
         waves = waves or gemv_packed_config(N, Kd, w.bn // 16, M, slab=False)[1]
         check(kernels().cfc_gemv_packed(x.data_ptr(), w.data.data_ptr(), M, N, Kd, w.bn // 16, mode, yf, yb,
-                                        out.shape[1], 1, waves, None, 0, None, None, None, 0.0, _stream(x)),
+                                        out.shape[1], 1, waves, None, 0, None, None, None, 0.0, None, _stream(x)),
               "cfc_gemv_packed")
     else:
         check(kernels().cfc_gemv(x.data_ptr(), w.data_ptr(), M, N, Kd, mode, yf, yb, out.shape[1], _stream(x)),

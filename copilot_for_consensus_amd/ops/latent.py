@@ -5,16 +5,20 @@ GPU tensors go to the native library (which must be built), CPU tensors to the f
 """
 from __future__ import annotations
 
+import dataclasses
 import math
 
+import numpy as np
 import torch
 
 from . import reference as ref
 from ._native import check, kernels
+from .cols import Cols
 from .kernels import _p, _req, _stream, _workspace
 from .stream import _act
 
 MFMA_MAX_RANK = 512       # latent ranks the MFMA attention kernel is built for
+MFMA_MAX_KEY = 576        # and key columns (the latent and what follows it in the row)
 ANY_ROWS = 4              # rows per tile of the general kernel
 
 
@@ -38,20 +42,27 @@ class HeadWeight:
         return self.data.numel() * self.data.element_size()
 
 
-def head_linear(x: torch.Tensor, w: HeadWeight, out: torch.Tensor) -> torch.Tensor:
-    """out[t, h, :N] = w[h] x[t, h, :K].  x [T, H, >= K], out [T, H, >= N]: any row / head strides, last dim dense."""
+def head_linear(x: torch.Tensor, w: HeadWeight, out: torch.Tensor, gate: torch.Tensor | None = None) -> torch.Tensor:
+    """out[t, h, :N] = w[h] x[t, h, :K], times sigmoid(gate[t, h N + n]) when given ([T, H N], row-strided).
+    x [T, H, >= K], out [T, H, >= N]: any row / head strides, last dim dense."""
     T, H = x.shape[0], x.shape[1]
     if H != w.H or out.shape[:2] != (T, H) or x.shape[2] < w.K or out.shape[2] < w.N:
         raise ValueError(f"head_linear: x {tuple(x.shape)} w {w.H} x {w.N} x {w.K} out {tuple(out.shape)}")
     if not x.is_cuda:
         y = torch.matmul(x[:, :, :w.K].float().transpose(0, 1), w.data[:, :w.N, :w.K].float().transpose(1, 2))
-        out[:, :, :w.N] = y.transpose(0, 1).to(out.dtype)
+        y = y.transpose(0, 1)
+        if gate is not None:
+            y = y * torch.sigmoid(gate.float().view(T, H, w.N))
+        out[:, :, :w.N] = y.to(out.dtype)
         return out
     if x.stride(2) != 1 or out.stride(2) != 1 or x.dtype != out.dtype or x.dtype != w.data.dtype:
         raise ValueError("head_linear: dense last dimensions and one dtype needed")
+    if gate is not None and (gate.shape != (T, H * w.N) or gate.stride(1) != 1 or gate.dtype != x.dtype):
+        raise ValueError(f"head_linear: gate {tuple(gate.shape)} {gate.dtype}")
     check(kernels().cfc_head_linear(_act(x.dtype), x.data_ptr(), x.stride(0), x.stride(1), w.data.data_ptr(),
                                     w.data.shape[1], w.data.shape[2], T, H, w.N, w.K, out.data_ptr(), out.stride(0),
-                                    out.stride(1), _stream(x)), "cfc_head_linear")
+                                    out.stride(1), _p(gate), gate.stride(0) if gate is not None else 0, _stream(x)),
+          "cfc_head_linear")
     return out
 
 
@@ -75,9 +86,71 @@ def latent_norm(part, nq: int, wq, wc, eps: float, slots, cache, dtype) -> torch
     return out
 
 
-def rows_per_tile(dtype, RS: int, decode_plan: tuple | None = None) -> int:
+@dataclasses.dataclass
+class Rope:
+    """Rotary positions on neighbouring pairs of ``2 len(freq)`` dimensions: angle = position * freq, cos and sin
+    times ``mag``."""
+    freq: torch.Tensor            # fp32
+    mag: float
+
+    @property
+    def dims(self) -> int:
+        return 2 * self.freq.numel()
+
+
+def yarn_rope(dims: int, base: float, scaling: dict | None, device) -> Rope:
+    """Frequencies base^(-2i / dims); with ``scaling`` (factor, original, fast, slow) those of slow dimensions divided
+    by the factor, a linear ramp between, and the length's magnitude on cos and sin."""
+    i = np.arange(dims // 2, dtype=np.float64)
+    f, mag = base ** (-2.0 * i / dims), 1.0
+    if scaling:
+        at = [dims * math.log(scaling["original"] / (2 * math.pi * scaling[k])) / (2 * math.log(base)) for k in ("fast", "slow")]
+        lo, hi = max(math.floor(at[0]), 0), min(math.ceil(at[1]), dims - 1)
+        ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+        f = f / scaling["factor"] * ramp + f * (1.0 - ramp)
+        mag = 0.1 * math.log(scaling["factor"]) + 1.0
+    return Rope(torch.tensor(f, dtype=torch.float32, device=device), mag)
+
+
+def latent_rope(kv: Cols, rank: int, wc, eps: float, slots, cache, q: Cols, heads: int, dim: int, rope: Rope, positions, ql,
+                vdim: int = 0, gate: Cols | None = None):
+    """The normed latent (``rank`` columns of ``kv``) and the rotated shared key part behind it into ``cache``
+    [blocks, 32, RS] at ``slots``; each head's rotated query part into ql [T, heads, RS] (columns after the latent's).
+    ``q`` columns per head [dim | rot].  Returns (unrotated queries [T, heads, dim], output gate's pre-activations
+    [T, heads vdim] or None) as activations."""
+    T, RS, RV, dt = ql.shape[0], cache.shape[-1], padded_rank(rank), ql.dtype
+    if not ql.is_cuda:
+        y = kv.value()
+        c = y[:, :rank]
+        c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * wc
+        rows = cache.view(-1, RS)
+        rows[slots.long(), :rank] = c.to(dt)
+        rows[slots.long(), RV:RV + rope.dims] = ref.rotate_pairs(y[:, rank:], positions, rope.freq, rope.mag).to(dt)
+        qv = q.value().view(T, heads, dim + rope.dims)
+        ql[:, :, RV:] = 0
+        ql[:, :, RV:RV + rope.dims] = ref.rotate_pairs(qv[:, :, dim:], positions, rope.freq, rope.mag).to(dt)
+        return qv[:, :, :dim].to(dt), gate.value().to(dt) if gate is not None else None
+    if cache.dtype != dt or not ql.is_contiguous() or ql.shape[1:] != (heads, RS) or q.n != heads * (dim + rope.dims):
+        raise ValueError(f"latent_rope: ql {tuple(ql.shape)} {dt}, cache rows of {RS} {cache.dtype}, {q.n} query columns")
+    for name, t in (("slots", slots), ("positions", positions)):
+        _req(t, torch.int32, name)
+    qn = torch.empty(T, heads, dim, dtype=dt, device=ql.device) if q.slabs else None
+    gt = torch.empty(T, heads * vdim, dtype=dt, device=ql.device) if gate is not None and gate.slabs else None
+    g = gate.args(dt) if gt is not None else [None, 0, 0, 0]
+    check(kernels().cfc_latent_rope(_act(dt), *kv.args(dt), T, rank, wc.data_ptr(), float(eps), slots.data_ptr(),
+                                    cache.data_ptr(), RS, RV, *q.args(dt), heads, dim, ql.data_ptr(), _p(qn), *g, vdim, _p(gt),
+                                    rope.freq.data_ptr(), rope.dims, float(rope.mag), positions.data_ptr(), _stream(ql)),
+          "cfc_latent_rope")
+    if qn is None:
+        qn = q.t[:, q.c0:q.c0 + q.n].unflatten(1, (heads, dim + rope.dims))[:, :, :dim]
+    if gate is not None and gt is None:
+        gt = gate.t[:, gate.c0:gate.c0 + gate.n]
+    return qn, gt
+
+
+def rows_per_tile(dtype, RS: int, decode_plan: tuple | None = None, RV: int | None = None) -> int:
     """(token, head) rows of one attention work item: the general kernel's 4, or 16 / 32 / 64 on MFMA."""
-    if dtype != torch.bfloat16 or RS > MFMA_MAX_RANK:
+    if dtype != torch.bfloat16 or (RV or RS) > MFMA_MAX_RANK or RS > MFMA_MAX_KEY:
         return ANY_ROWS
     return decode_plan[0] if decode_plan else 64
 
@@ -109,15 +182,16 @@ def decode_plan(B: int, heads: int, RS: int, max_ctx: int, P: int | None = None)
     return best[1], best[2]
 
 
-def attn_tiles(cu_q, heads: int, rows: int, ctx_lens=None):
+def attn_tiles(cu_q, heads: int, rows: int, ctx_lens=None, window: int = 0):
     """(sequence, first row) of every work item of a packed batch; with ``ctx_lens`` those with the most
-    keys first, so the long ones do not end the grid alone."""
+    keys (at most about ``window``) first, so the long ones do not end the grid alone."""
     tiles = []
     for s in range(len(cu_q) - 1):
         n = cu_q[s + 1] - cu_q[s]
         base = ctx_lens[s] - n if ctx_lens is not None else 0
         for m0 in range(0, n * heads, rows):
-            tiles.append((base + (min(m0 + rows, n * heads) - 1) // heads, s, m0))
+            keys = base + (min(m0 + rows, n * heads) - 1) // heads
+            tiles.append((min(keys, window) if window else keys, s, m0))
     if ctx_lens is not None:
         tiles.sort(key=lambda t: -t[0])
     return [t[1] for t in tiles], [t[2] for t in tiles]
@@ -129,20 +203,23 @@ def partitions(n_tiles: int, max_ctx: int, target: int = 512) -> int:
 
 
 def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles=None, rows: int | None = None,
-                     P: int = 1, workspace=None) -> torch.Tensor:
-    """Softmax attention of q [T, H, RS] over the paged latents [blocks, 32, RS], causal inside each
-    sequence's portion.  ``cu_q`` None: one token per sequence.  ``tiles``: device (tile_seq, tile_m0) of
-    :func:`attn_tiles` cut for ``rows``; P key slices per tile merged at the end."""
+                     P: int = 1, workspace=None, window: int = 0, sink=None, RV: int | None = None) -> torch.Tensor:
+    """Softmax attention of q [T, H, RS] over the paged rows [blocks, 32, RS], causal inside each sequence's
+    portion; the value is a row's first ``RV`` columns (None: all).  ``window``: keys a token sees, itself included
+    (0: all before it).  ``sink`` [H] fp32: exp(sink) joins each denominator once.  ``cu_q`` None: one token per
+    sequence.  ``tiles``: device (tile_seq, tile_m0) of :func:`attn_tiles` cut for ``rows``; P key slices per tile
+    merged at the end."""
     T, H, RS = q.shape
+    RV = RV or RS
     B = ctx_lens.numel()
     if not q.is_cuda:
         cu = cu_q if cu_q is not None else torch.arange(B + 1)
-        return ref.latent_attention(q, cache, block_tables, cu, ctx_lens, scale)
+        return ref.latent_attention(q, cache, block_tables, cu, ctx_lens, scale, window, sink, RV)
     if not q.is_contiguous() or not cache.is_contiguous() or cache.shape[-1] != RS or cache.dtype != q.dtype:
         raise ValueError(f"latent_attention: q {tuple(q.shape)} {q.dtype}, cache {tuple(cache.shape)} {cache.dtype}")
     for name, t in (("block_tables", block_tables), ("ctx_lens", ctx_lens)):
         _req(t, torch.int32, name)
-    rows = rows or rows_per_tile(q.dtype, RS, decode_plan(B, H, RS, 64, P) if cu_q is None else None)
+    rows = rows or rows_per_tile(q.dtype, RS, decode_plan(B, H, RS, 64, P) if cu_q is None else None, RV)
     if cu_q is None:
         if T != B:
             raise ValueError(f"latent_attention: {T} rows for {B} sequences")
@@ -155,15 +232,17 @@ def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles
             tiles = tuple(torch.tensor(v, dtype=torch.int32, device=q.device) for v in (a, b))
         ts, tm = tiles
         per_seq, n_tiles = 0, ts.numel()
-    out = torch.empty_like(q)
+    if sink is not None:
+        _req(sink, torch.float32, "sink")
+    out = torch.empty(T, H, RV, dtype=q.dtype, device=q.device)
     po = pm = None
     if P > 1:
-        need = T * H * P * (RS + 2)
+        need = T * H * P * (RV + 2)
         ws = workspace if workspace is not None and workspace.numel() >= need else _workspace(q.device, need)
-        po, pm = ws[:T * H * P * RS], ws[T * H * P * RS:need]
+        po, pm = ws[:T * H * P * RV], ws[T * H * P * RV:need]
     check(kernels().cfc_latent_attention(_act(q.dtype), q.data_ptr(), cache.data_ptr(), block_tables.data_ptr(), _p(cu_q),
-                                         ctx_lens.data_ptr(), _p(ts), _p(tm), n_tiles, per_seq, rows, H, RS,
-                                         block_tables.shape[1], float(scale), P, T * H, _p(po), _p(pm), out.data_ptr(),
+                                         ctx_lens.data_ptr(), _p(ts), _p(tm), n_tiles, per_seq, rows, H, RS, RV,
+                                         block_tables.shape[1], float(scale), int(window), _p(sink), P, T * H, _p(po), _p(pm), out.data_ptr(),
                                          _stream(q)), "cfc_latent_attention")
     return out
 

@@ -12,6 +12,7 @@ from __future__ import annotations
 
 import math
 
+import numpy as np
 import torch
 
 KV_BLOCK = 32
@@ -377,15 +378,135 @@ def latent_norm(part, nq, wq, wc, eps):
     return q, c
 
 
-def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale):
-    """q [T, H, RS]; cache [blocks, 32, RS]: softmax over the sequence's latents, per row causal."""
-    out = torch.empty_like(q)
+def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale, window=0, sink=None, vcols=None):
+    """q [T, H, RS]; cache [blocks, 32, RS]: softmax over the sequence's cached rows, per row causal and at most
+    ``window`` keys back (0: all), exp(sink[h]) added to the denominator; the value is a row's first ``vcols``
+    columns."""
+    vcols = vcols or q.shape[2]
+    out = torch.empty(*q.shape[:2], vcols, dtype=q.dtype)
     for s in range(len(ctx_lens)):
         a, b, ctx = int(cu_q[s]), int(cu_q[s + 1]), int(ctx_lens[s])
         nb = -(-ctx // KV_BLOCK)
         c = cache[block_tables[s, :nb].long()].reshape(nb * KV_BLOCK, -1)[:ctx].float()
         sc = torch.matmul(q[a:b].float(), c.t()) * scale                        # [n, H, ctx]
-        pos = torch.arange(ctx - (b - a), ctx)
-        sc.masked_fill_((torch.arange(ctx)[None] > pos[:, None])[:, None], float("-inf"))
-        out[a:b] = torch.matmul(torch.softmax(sc, -1), c).to(q.dtype)
+        back = torch.arange(ctx - (b - a), ctx)[:, None] - torch.arange(ctx)[None]
+        hidden = (back < 0) | (back >= window) if window else back < 0
+        sc.masked_fill_(hidden[:, None], float("-inf"))
+        if sink is not None:
+            sc = torch.cat([sc, sink.float().view(1, -1, 1).expand(b - a, -1, 1)], -1)
+        p = torch.softmax(sc, -1)[..., :ctx]
+        out[a:b] = torch.matmul(p, c[:, :vcols]).to(q.dtype)
     return out
+
+
+# ----------------------------------------------------- rotary tables
+def rotate_pairs(x, positions, freq, mag):
+    """Neighbouring dimensions (2i, 2i + 1) of x [T, ..., 2n] rotated by positions * freq[i], scaled by mag."""
+    a = positions.to(torch.float32)[:, None] * freq
+    shape = (x.shape[0],) + (1,) * (x.dim() - 2) + (-1,)
+    c, s = (a.cos() * mag).view(shape), (a.sin() * mag).view(shape)
+    u, v = x[..., 0::2].float(), x[..., 1::2].float()
+    return torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+
+
+# ----------------------------------------------------- gated, post-normed branches (gated.hip)
+META_TAIL, META_SLOT = 4, 3        # row word: rows before it in its portion (0, 1, 2 = more) | last two rows | slot << 3
+
+
+def row_meta(portions) -> np.ndarray:
+    """Row words of packed portions [(rows, state slot)]."""
+    out = []
+    for n, slot in portions:
+        r = np.arange(n)
+        out.append(np.minimum(r, 2) | np.where(r >= n - 2, META_TAIL, 0) | (slot << META_SLOT))
+    return np.concatenate(out).astype(np.int32)
+
+
+def layernorm_rows(y, w, eps):
+    d = y - y.mean(-1, keepdim=True)
+    return d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * w
+
+
+def before_rows(x, meta, positions, prev):
+    """(x of the token before, x of the one before that) per row; prev [slots, 2, W] holds the rows of positions
+    before a portion at position % 2; zeros before the first token."""
+    xp, xpp = torch.zeros_like(x), torch.zeros_like(x)
+    for t, (m, p) in enumerate(zip(meta.tolist(), positions.tolist())):
+        lead, slot = m & 3, m >> META_SLOT
+        if p >= 1:
+            xp[t] = x[t - 1] if lead >= 1 else prev[slot, (p - 1) % 2]
+        if p >= 2:
+            xpp[t] = x[t - 2] if lead >= 2 else prev[slot, p % 2]
+    return xp, xpp
+
+
+def shift_mix(x, xp, xpp, positions, shift, mus):
+    """Token shift of x, then (``mus`` [n, W]) each mix of the shifted row with the one before it."""
+    h = x + (xp - x) * shift
+    if mus is None:
+        return [h]
+    hp = (xp + (xpp - xp) * shift) * (positions >= 1).to(x.dtype)[:, None]
+    return [h + (hp - h) * mu for mu in mus]
+
+
+# ----------------------------------------------------- per-channel decay recurrence (wkv.hip)
+LOG_DECAY_MIN = -104.0             # exp(-104) is 0 in fp32
+
+
+def wkv(r, k, v, w, u, S):
+    """r, k, v, w [T, H, D] fp32, u [H, D], S [H, D, D] (updated): o_t = (S + u k v^T)^T r, S = w S + k v^T."""
+    out = torch.empty_like(v)
+    for t in range(r.shape[0]):
+        kv = k[t][:, :, None] * v[t][:, None, :]
+        out[t] = torch.einsum("hij,hi->hj", S + u[:, :, None] * kv, r[t])
+        S.mul_(w[t][:, :, None]).add_(kv)
+    return out
+
+
+def wkv_decay(w1, w2, w0):
+    """w1 [T, R]: exp(-exp(tanh(w1) w2^T + w0))."""
+    return torch.exp(torch.clamp(-torch.exp(torch.tanh(w1) @ w2.float().t() + w0), min=LOG_DECAY_MIN))
+
+
+def wkv_out(o, norm, gate, eps):
+    """o [T, H, D] over its root mean square per head, times norm and silu(gate) [T, H D]."""
+    o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps)
+    return o.flatten(1) * norm * (gate * torch.sigmoid(gate))
+
+
+# ----------------------------------------------------- routed experts (moe.hip)
+def route(logits, correction, groups, keep, top, scale):
+    """logits [T, E] fp32: (ids [T, top], weights [T, top]).  Sigmoid scores; the choice adds ``correction``; a
+    group counts by its two largest choice scores and only the best ``keep`` groups take part."""
+    s = torch.sigmoid(logits)
+    c = s + correction
+    T, E = c.shape
+    g = c.view(T, groups, E // groups)
+    best = g.topk(min(2, E // groups), -1).values.sum(-1)
+    kept = torch.zeros_like(best, dtype=torch.bool).scatter_(1, best.topk(keep, -1).indices, True)
+    c = c.masked_fill(~kept.repeat_interleave(E // groups, 1), float("-inf"))
+    ids = c.topk(top, -1).indices
+    w = s.gather(1, ids)
+    return ids.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
+
+
+def moe_rows(ids, experts, tile):
+    """Rows of (token, choice) pairs sorted by expert, every expert's rows padded to whole tiles: (token per row
+    [M], row per pair [T, top], expert per tile [M / tile]), pad rows token 0, tiles past the last -1."""
+    T, top = ids.shape
+    n_tiles = moe_max_tiles(T * top, experts, tile)
+    rows, pos, te = np.zeros(n_tiles * tile, np.int32), np.zeros((T, top), np.int32), np.full(n_tiles, -1, np.int32)
+    at = 0
+    for e in range(experts):
+        pairs = [(t, c) for t in range(T) for c in range(top) if int(ids[t, c]) == e]
+        for i, (t, c) in enumerate(pairs):
+            rows[at + i], pos[t, c] = t, at + i
+        m = -(-len(pairs) // tile)
+        te[at // tile:at // tile + m] = e
+        at += m * tile
+    return rows, pos, te
+
+
+def moe_max_tiles(pairs: int, experts: int, tile: int) -> int:
+    """Most tiles that ``pairs`` rows over ``experts`` experts can take."""
+    return min(pairs, pairs // tile + min(experts, pairs))

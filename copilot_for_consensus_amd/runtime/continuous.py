@@ -96,6 +96,9 @@ class ContinuousEngine:
         self.ctx_lens = torch.ones(B, **i32)
         self.slots = torch.full((B,), self.scratch * KV_BLOCK, **i32)
         self.block_tables = torch.full((B, self.max_blocks), self.scratch, **i32)
+        # state slot per row (caches with per-sequence state): the scratch slot when empty
+        self.states = None if self.kv.states is None else torch.full((B,), self.kv.states.scratch, **i32)
+        self.slot_state: list[int | None] = [None] * B
         self.tokens = torch.zeros(B, self.cap, **i32)
         self.gen = torch.zeros(B, **i32)
         self.limit = torch.ones(B, **i32)
@@ -250,11 +253,14 @@ class ContinuousEngine:
         idle = all(r is None for r in self.slot_req)
         pc = self.engine.prefix_cache
         tables, fresh, start = [], [], []
+        states = None if self.kv.states is None else []
         try:
             for i, r in enumerate(take):
                 n = blocks_needed(len(r.prompt) + r.max_new)
                 shared = pc.acquire(r.prompt) if pc is not None else []
                 try:
+                    if states is not None and not self.kv.states.num_free():
+                        raise MemoryError("no free state slot")
                     new = pc.alloc(n - len(shared)) if pc is not None else self.kv.pool.alloc(n)
                 except MemoryError:
                     # KV cache full: admit what fits, the rest waits in the queue for running slots to
@@ -265,13 +271,15 @@ class ContinuousEngine:
                     self.queue.extendleft(reversed(take[i:]))
                     take = take[:i]
                     break
+                if states is not None:
+                    states += self.kv.states.alloc(1)
                 tables.append(shared + new)
                 fresh.append(new)
                 start.append(len(shared) * KV_BLOCK)
                 if pc is not None and not self.engine.share_late:
                     pc.insert(r.prompt, tables[-1])
         except BaseException:
-            self.engine._release(tables, fresh, failed=True)
+            self.engine._release(tables, fresh, failed=True, states=states)
             self.queue.extendleft(reversed(take))
             raise
         if not take:
@@ -282,12 +290,13 @@ class ContinuousEngine:
             # A stable sort on the admitted list, so TP followers replaying it place the same slots.
             order = sorted(range(len(take)), key=lambda i: -len(take[i].prompt))
             take, tables, fresh, start = ([v[i] for i in order] for v in (take, tables, fresh, start))
+            states = states if states is None else [states[i] for i in order]
         t = time.perf_counter()
         try:
-            first = self.engine._prefill([r.prompt for r in take], tables, self.sampling, self.seed, start)
+            first = self.engine._prefill([r.prompt for r in take], tables, self.sampling, self.seed, start, states)
         except BaseException:
             # nothing was installed in a slot yet: return the blocks, put the requests back in front
-            self.engine._release(tables, fresh, failed=True)
+            self.engine._release(tables, fresh, failed=True, states=states)
             self.queue.extendleft(reversed(take))
             raise
         self.engine._share_computed([r.prompt for r in take], tables)
@@ -310,6 +319,7 @@ class ContinuousEngine:
             self.slot_req[s] = r
             r.slot = s
             self.slot_tables[s] = (tbl, fresh[i])
+            self.slot_state[s] = states[i] if states is not None else None
             self._slot_shared[s] = start[i] // KV_BLOCK
         occupied = [self._slot_shared[q] for q in range(self.B) if self.slot_req[q] is not None]
         self.shared.fill_(min(occupied) if occupied and self.engine.shared_cached else 0)
@@ -318,6 +328,8 @@ class ContinuousEngine:
         self.block_tables.index_copy_(0, idx, torch.from_numpy(bt).to(self.device))
         for j, dst in enumerate((self.ids, self.positions, self.ctx_lens, self.slots, self.limit, self.done)):
             dst.index_copy_(0, idx, rows_t[:, j].contiguous())
+        if states is not None:
+            self.states.index_copy_(0, idx, torch.tensor(states, dtype=torch.int32, device=self.device))
         self.gen.index_fill_(0, idx, 1)
         if self.stop_state is not None:
             self.stop_state.set_slots(slots, sstates)
@@ -337,7 +349,8 @@ class ContinuousEngine:
         ss = self.stop_state.view(W) if self.stop_state is not None else None
         hidden = self.model.forward_decode(self.ids[:W], self.positions[:W], self.slots[:W], self.ctx_lens[:W],
                                            self.block_tables[:W], self.kv, attn_workspace=self.workspace,
-                                           part_blocks=self._pb[W], shared_blocks=self.shared)
+                                           part_blocks=self._pb[W], shared_blocks=self.shared,
+                                           **self.engine._state_kw(self.states[:W] if self.states is not None else None))
         self.engine._next_tokens(hidden, self.next_ids[:W], self.sampling, self.seed, self.step_t)
         K.decode_advance_cb(self.next_ids[:W], self.tokens[:W], self.gen[:W], self.limit[:W], self.ids[:W],
                             self.positions[:W], self.ctx_lens[:W], self.slots[:W], self.block_tables[:W],
@@ -346,6 +359,7 @@ class ContinuousEngine:
 
     def _state(self):
         extra = [self.stop_state.win, self.stop_state.wlen, self.stop_state.keep] if self.stop_state else []
+        extra += [self.states] if self.states is not None else []
         return [self.ids, self.positions, self.ctx_lens, self.slots, self.tokens, self.gen, self.done,
                 self.next_ids, self.step_t] + extra
 
@@ -353,6 +367,8 @@ class ContinuousEngine:
         W = self._width()          # no admission inside a burst: the occupied slots only shrink
         if self.use_graph and W not in self.graphs:
             saved = [t.clone() for t in self._state()]
+            if self.states is not None:      # the warm-up step runs on the scratch state
+                self.states.fill_(self.kv.states.scratch)
             s = self.engine.capture_stream()
             s.wait_stream(torch.cuda.current_stream(self.device))
             with torch.cuda.stream(s):
@@ -403,13 +419,15 @@ class ContinuousEngine:
         self.slots.index_fill_(0, idx, self.scratch * KV_BLOCK)
         self.positions.index_fill_(0, idx, 0)
         self.ctx_lens.index_fill_(0, idx, 1)
+        if self.states is not None:
+            self.states.index_fill_(0, idx, self.kv.states.scratch)
         self.stats["finished"] += len(out)
         return out
 
     def _release_slot(self, s: int) -> None:
         tbl, fresh = self.slot_tables[s]
-        self.engine._release([tbl], [fresh])
-        self.slot_tables[s] = None
+        self.engine._release([tbl], [fresh], states=[self.slot_state[s]] if self.states is not None else None)
+        self.slot_tables[s] = self.slot_state[s] = None
         self.slot_req[s] = None
         self.free.append(s)
         self.free.sort(reverse=True)     # pop() takes the lowest free slot: the decode width stays small

@@ -61,6 +61,7 @@ class _Job:
     temperature: object
     seed: int
     prefill_s: float
+    states: list | None = None    # state slots of the batch's rows (caches with per-sequence state)
     ready: object = None          # event recorded after the state setup (stream handoff)
     order: list | None = None     # slot s holds caller prompt order[s] (longest-first slots)
 
@@ -68,7 +69,7 @@ class _Job:
 class _DecodeState:
     """Static device buffers a captured decode graph reads and writes."""
 
-    def __init__(self, B, max_blocks, max_new, device, n_part_ws):
+    def __init__(self, B, max_blocks, max_new, device, n_part_ws, states=None):
         i32 = dict(dtype=torch.int32, device=device)
         self.ids = torch.zeros(B, **i32)
         self.positions = torch.zeros(B, **i32)
@@ -81,12 +82,15 @@ class _DecodeState:
         self.done = torch.zeros(B, **i32)
         self.next_ids = torch.zeros(B, **i32)
         self.stop_ids = torch.zeros(0, **i32)
+        # state slot per row (caches with per-sequence state); the scratch slot outside a run
+        self.states = torch.full((B,), states.scratch, **i32) if states is not None else None
         self.stop_state = None     # runtime.stops.StopState when the request has stop strings
         self.workspace = torch.empty(max(1, n_part_ws), dtype=torch.float32, device=device)
         self.graph = None
 
     def tensors(self):
         extra = [self.stop_state.win, self.stop_state.wlen, self.stop_state.keep] if self.stop_state else []
+        extra += [self.states] if self.states is not None else []
         return [self.ids, self.positions, self.ctx_lens, self.slots, self.block_tables, self.step, self.tokens,
                 self.done, self.next_ids] + extra
 
@@ -116,6 +120,8 @@ class LLMEngine:
         self._states: dict[tuple, _DecodeState] = {}
         self._alloc_lock = threading.RLock()     # KV / prefix-cache bookkeeping of start / finish
         # shared-prefix reuse of whole KV blocks (system prompt + template head of every thread)
+        if not getattr(kv, "share_prefix", True):
+            prefix_cache = False
         if prefix_cache is None:
             prefix_cache = os.environ.get("CFC_PREFIX_CACHE", "1") != "0"
         self.prefix_cache = PrefixCache(kv.pool) if prefix_cache else None
@@ -163,7 +169,11 @@ class LLMEngine:
             print(f"[ar-debug] rank {ar.rank} {tag}: errors={ar.errors()} epochs[0:4]={ep[:4]} "
                   f"epochs[32]={ep[32]} key={ep[-1]} distinct={sorted(set(ep))[:6]}", flush=True)
 
-    def _prefill(self, prompts, tables, temperature, seed, start=None):
+    def _state_kw(self, states) -> dict:
+        """The model's keyword for the state slots of a batch (nothing without per-sequence state)."""
+        return {} if states is None else {"states": states}
+
+    def _prefill(self, prompts, tables, temperature, seed, start=None, states=None):
         """Chunked packed prefill; returns first sampled token per prompt.  ``start[s]`` tokens of
         prompt s are already in the cache (shared prefix blocks)."""
         n = len(prompts)
@@ -183,7 +193,7 @@ class LLMEngine:
                 else:
                     break  # a split sequence ends the chunk
             halves = self._overlap_split(chunk)
-            metas = [self._chunk_meta(prompts, tables, part) for part in halves]
+            metas = [self._chunk_meta(prompts, tables, part, states) for part in halves]
             if len(metas) == 2:
                 hiddens = self.model.forward_prefill_overlap([m[0] for m in metas], self.kv)
             else:
@@ -216,7 +226,7 @@ class LLMEngine:
         k = best[1]
         return [chunk[:k], chunk[k:]]
 
-    def _chunk_meta(self, prompts, tables, chunk):
+    def _chunk_meta(self, prompts, tables, chunk, states=None):
         """Device metadata of one packed prefill pass over ``chunk`` [(seq, first, end)]: the
         forward_prefill keyword arguments, the sequences finishing in it, and their ids on device."""
         finishing, last_rows, row = [], [], 0
@@ -226,13 +236,14 @@ class LLMEngine:
                 last_rows.append(row - 1)
                 finishing.append(s)
         kw, extra = self._pass_meta([(prompts[s][a:b], a) for (s, a, b) in chunk], [tables[s] for (s, _, _) in chunk],
-                                    last_rows, np.asarray(finishing, np.int32))
+                                    last_rows, np.asarray(finishing, np.int32),
+                                    [states[s] for (s, _, _) in chunk] if states is not None else None)
         return kw, finishing, extra
 
-    def _pass_meta(self, portions, tables, last_rows, extra=np.zeros(0, np.int32)):
+    def _pass_meta(self, portions, tables, last_rows, extra=np.zeros(0, np.int32), states=None):
         """Device metadata of one packed pass over ``portions`` [(tokens, first position)] with their block
-        tables: the forward_prefill keyword arguments for the rows ``last_rows``, and ``extra`` (int32) on
-        the device."""
+        tables (and state slots): the forward_prefill keyword arguments for the rows ``last_rows``, and ``extra``
+        (int32) on the device."""
         cu, ctx = [0], []
         ids_np, pos_np, slot_np = [], [], []
         for (toks, a), tbl in zip(portions, tables):
@@ -250,7 +261,7 @@ class LLMEngine:
         # pageable torch.tensor(..., device=cuda) synchronises the stream, so the GPU would idle
         # while the host builds the next chunk
         slots_np = np.concatenate(slot_np)
-        plan = self.model.plan_prefill(cu, ctx, slots_np)
+        plan = self.model.plan_prefill(cu, ctx, slots_np, **self._state_kw(states))
         arrays = [k for k, v in plan.items() if isinstance(v, np.ndarray)]
         parts = [np.concatenate(ids_np), np.concatenate(pos_np), slots_np,
                  np.asarray(cu, np.int32), np.asarray(ctx, np.int32), np.asarray(last_rows, np.int32), extra,
@@ -272,10 +283,12 @@ class LLMEngine:
     @torch.inference_mode()
     def forward_step(self, entries) -> torch.Tensor | None:
         """One forward pass over a mixed batch: ``entries`` [(tokens, first position, block table, wanted
-        rows)], portions of prompts beside single decoded tokens, the tables already holding a block for
+        rows, state slot or None)], portions of prompts beside single decoded tokens, the tables already holding a block for
         every position.  Returns the logits at the wanted rows, in order (None if there are none).  A batch
         of single later tokens takes the decode step's kernels, any other the packed pass."""
         rows, base = [], 0
+        states = [e[4] for e in entries] if self.kv.states is not None else None
+        entries = [e[:4] for e in entries]
         for toks, _, _, want in entries:
             rows += [base + r for r in want]
             base += len(toks)
@@ -283,21 +296,24 @@ class LLMEngine:
             B = len(entries)
             maxb = 8 * math.ceil(max(len(t) for _, _, t, _ in entries) / 8)
             bt = np.zeros((B, maxb), np.int32)
-            meta = np.zeros((4, B), np.int32)
+            meta = np.zeros((5, B), np.int32)
+            if states is not None:
+                meta[4] = states
             for b, (toks, first, tbl, _) in enumerate(entries):
                 bt[b, :len(tbl)] = tbl
-                meta[:, b] = (toks[0], first, tbl[first // KV_BLOCK] * KV_BLOCK + first % KV_BLOCK, first + 1)
+                meta[:4, b] = (toks[0], first, tbl[first // KV_BLOCK] * KV_BLOCK + first % KV_BLOCK, first + 1)
             dev = self._h2d(np.concatenate([bt.reshape(-1), meta.reshape(-1)]))
-            d_bt, d_meta = dev[:B * maxb].view(B, maxb), dev[B * maxb:].view(4, B).clone()
+            d_bt, d_meta = dev[:B * maxb].view(B, maxb), dev[B * maxb:].view(5, B).clone()
             pb = self._part_blocks(B, maxb)
             ws = torch.empty(max(1, self.model.decode_workspace(B, -pb)), dtype=torch.float32, device=self.device)
             hidden = self.model.forward_decode(d_meta[0], d_meta[1], d_meta[2], d_meta[3], d_bt, self.kv,
-                                               attn_workspace=ws, part_blocks=pb)
+                                               attn_workspace=ws, part_blocks=pb,
+                                               **self._state_kw(d_meta[4] if states is not None else None))
             if len(rows) < B:
                 hidden = hidden.index_select(0, torch.tensor(rows, dtype=torch.long, device=self.device)) if rows else None
         else:
             kw, _ = self._pass_meta([(toks, first) for toks, first, _, _ in entries], [t for _, _, t, _ in entries],
-                                    rows or [base - 1])
+                                    rows or [base - 1], states=states)
             hidden = self.model.forward_prefill(**kw, kv=self.kv)
         self.progress += 1
         return self.model.logits(hidden) if rows else None
@@ -328,7 +344,7 @@ class LLMEngine:
     def _decode_step(self, st: _DecodeState, part_blocks, temperature, seed):
         hidden = self.model.forward_decode(st.ids, st.positions, st.slots, st.ctx_lens, st.block_tables, self.kv,
                                            attn_workspace=st.workspace, part_blocks=part_blocks,
-                                           shared_blocks=st.shared)
+                                           shared_blocks=st.shared, **self._state_kw(st.states))
         self._next_tokens(hidden, st.next_ids, temperature, seed, st.step)
         K.decode_advance(st.next_ids, st.tokens, st.step, st.ids, st.positions, st.ctx_lens, st.slots,
                          st.block_tables, st.done, st.stop_ids, st.stop_state)
@@ -338,7 +354,7 @@ class LLMEngine:
         st = self._states.get(key)
         if st is None:
             P = -part_blocks if part_blocks < 0 else math.ceil(max_blocks / part_blocks)
-            st = _DecodeState(B, max_blocks, max_new, self.device, self.model.decode_workspace(B, P))
+            st = _DecodeState(B, max_blocks, max_new, self.device, self.model.decode_workspace(B, P), self.kv.states)
             # persistent: a captured graph holds these pointers
             st.stop_ids = torch.tensor(list(stop_ids), dtype=torch.int32, device=self.device)
             if stop_strings is not None:
@@ -357,6 +373,8 @@ class LLMEngine:
 
     def _capture(self, st, part_blocks, temperature, seed):
         saved = [t.clone() for t in st.tensors()]
+        if st.states is not None:        # the warm-up steps run on the scratch state
+            st.states.fill_(self.kv.states.scratch)
         s = self.capture_stream()
         s.wait_stream(torch.cuda.current_stream(self.device))
         with torch.cuda.stream(s):
@@ -427,9 +445,11 @@ class LLMEngine:
         need = [blocks_needed(n + max_new_tokens) for n in lens]
         max_blocks = 8 * math.ceil(max(need) / 8)
         pc = self.prefix_cache
-        tables, start, fresh = [], [], []
+        tables, start, fresh, states = [], [], [], None
         with self._alloc_lock:
             try:
+                if self.kv.states is not None:
+                    states = self.kv.states.alloc(B)
                 for p, n in zip(prompts, need):
                     shared = pc.acquire(p) if pc is not None else []
                     tables.append(shared)       # registered before alloc so a failure releases it
@@ -440,7 +460,7 @@ class LLMEngine:
                     if pc is not None and not self.share_late:
                         pc.insert(p, tables[-1])
             except BaseException:
-                self._release(tables, fresh, failed=True)
+                self._release(tables, fresh, failed=True, states=states)
                 raise
         sync = self.device.type == "cuda"
 
@@ -454,7 +474,7 @@ class LLMEngine:
             barrier()
             t0 = time.perf_counter()
             with span("llm.prefill"):
-                first = self._prefill(prompts, tables, temperature, seed, start)
+                first = self._prefill(prompts, tables, temperature, seed, start, states)
             barrier()
             self._share_computed(prompts, tables)
             t1 = time.perf_counter()
@@ -473,6 +493,8 @@ class LLMEngine:
             st.positions.copy_(lens_t)
             st.ctx_lens.copy_(lens_t + 1)
             pos = lens_t.long()
+            if states is not None:
+                st.states.copy_(torch.tensor(states, dtype=torch.int32))
             st.slots.copy_(bt[torch.arange(B), pos // KV_BLOCK] * KV_BLOCK + pos % KV_BLOCK)
             st.tokens.zero_()
             st.tokens[:, 0].copy_(f)
@@ -498,10 +520,10 @@ class LLMEngine:
                 ready.record(torch.cuda.current_stream(self.device))
         except BaseException:
             with self._alloc_lock:
-                self._release(tables, fresh, failed=True)
+                self._release(tables, fresh, failed=True, states=states)
             raise
         return _Job(st, tables, fresh, lens, start, B, max_new_tokens, tuple(stop_ids), stop_strings, part_blocks,
-                    temperature, seed, t1 - t0, ready, order)
+                    temperature, seed, t1 - t0, states, ready, order)
 
     @torch.inference_mode()
     def finish(self, job: _Job, switch=None) -> GenerationResult:
@@ -560,7 +582,7 @@ class LLMEngine:
             ok = True
         finally:
             with self._alloc_lock:
-                self._release(job.tables, job.fresh, failed=not ok)
+                self._release(job.tables, job.fresh, failed=not ok, states=job.states)
         out = []
         stop = set(stop_ids)
         for b in range(B):
@@ -586,7 +608,9 @@ class LLMEngine:
                 for p, t in zip(prompts, tables):
                     self.prefix_cache.insert(p, t)
 
-    def _release(self, tables, fresh, failed: bool = False):
+    def _release(self, tables, fresh, failed: bool = False, states=None):
+        if states:
+            self.kv.states.free(states)
         if self.prefix_cache is None:
             for t in tables:
                 self.kv.pool.free(t)

@@ -73,6 +73,25 @@ class BlockPool:
         self._free.extend(reversed(blocks))
 
 
+class StateSlots:
+    """Per-sequence state slots 0 .. n - 1 and one scratch slot (n): rows of a decode batch that hold no sequence, and
+    a captured step's warm-up, work on the scratch."""
+
+    def __init__(self, n: int):
+        self.n, self.scratch, self._free = n, n, list(range(n - 1, -1, -1))
+
+    def num_free(self) -> int:
+        return len(self._free)
+
+    def alloc(self, n: int) -> list[int]:
+        if n > len(self._free):
+            raise MemoryError(f"state slots exhausted: need {n}, {len(self._free)} free")
+        return [self._free.pop() for _ in range(n)]
+
+    def free(self, slots: list[int]) -> None:
+        self._free.extend(reversed(slots))
+
+
 class PagedKVCache:
     """K [layers][blocks, kv_heads, 32, D] and V^T [layers][blocks, kv_heads, D, 32] (slot-permuted,
     stored as [4 slot groups][D][8] per block and head: ops.reference.v_groups).
@@ -80,6 +99,8 @@ class PagedKVCache:
     ``dtype`` bf16 (default) or ``torch.float8_e4m3fn``: the FP8 cache halves the bytes the decode
     attention streams; it holds K / ``k_scale`` and V / ``v_scale`` (clamped to +-448) and the
     kernels scale back.  Opt-in: it is a precision trade-off, not the default."""
+
+    states = None               # no state beside the blocks
 
     def __init__(self, layers: int, num_blocks: int, kv_heads: int, head_dim: int, device, dtype=torch.bfloat16,
                  k_scale: float = 1.0, v_scale: float = 1.0):
@@ -116,6 +137,7 @@ class LatentKVCache:
                                                     block, row = position % slots (None without history)
     A block holds all a sequence continuing after it needs, so prefix sharing works on whole blocks."""
 
+    states = None
     # another sequence may map a block only after the pass that computes it (its tail is read in the
     # launch that writes tails)
     share_after_compute = True
@@ -132,6 +154,34 @@ class LatentKVCache:
 
     def nbytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (*self.latents, *self.tails) if t is not None)
+
+
+class HybridCache:
+    """Cache of a decoder whose layers are of several kinds: paged rows for those that attend, on the same blocks and
+    :class:`BlockPool` as :class:`PagedKVCache`, and a state of fixed size per sequence (``states``: its slots) for
+    those that recur and for what every layer remembers of the tokens before.  Per layer:
+      rows   [blocks, 32, columns] or None     attention: latent and rotated key part, pad columns zero
+      recur  [slots + 1, *shape] fp32 or None  recurrent state
+      prev   [slots + 1, 2, width] fp32        the layer's input rows of the last two tokens, at position % 2
+    A sequence's state is not in its blocks, so blocks cannot be shared between sequences.  A slot needs no clearing:
+    what lies before a sequence's first token is never read."""
+
+    share_prefix = False
+
+    def __init__(self, columns: list[int | None], recurrent: list[tuple | None], num_blocks: int, sequences: int, width: int,
+                 device, dtype=torch.bfloat16):
+        self.layers, self.num_blocks, self.width = len(columns), num_blocks, width
+        self.dtype, self.device = dtype, torch.device(device)
+        self.states = StateSlots(sequences)
+        n, f32 = sequences + 1, dict(dtype=torch.float32, device=self.device)
+        # zero-initialised: the slots of a partly filled block are read (then masked)
+        self.rows = [torch.zeros(num_blocks, KV_BLOCK, c, dtype=dtype, device=self.device) if c else None for c in columns]
+        self.recur = [torch.zeros(n, *s, **f32) if s else None for s in recurrent]
+        self.prev = [torch.zeros(n, 2, width, **f32) for _ in columns]
+        self.pool = BlockPool(num_blocks)
+
+    def nbytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in (*self.rows, *self.recur, *self.prev) if t is not None)
 
 
 def blocks_needed(n_tokens: int) -> int:

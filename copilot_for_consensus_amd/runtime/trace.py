@@ -20,6 +20,7 @@ from pathlib import Path
 import numpy as np
 
 EXIT_DTYPE = 3
+LIVE_REQUESTS = 4         # most requests live at a time (per-sequence state slots)
 
 
 class TraceSession:
@@ -27,7 +28,8 @@ class TraceSession:
 
     def __init__(self, engine):
         self.engine = engine
-        self.live: dict[str, tuple[list[int], list[int]]] = {}     # id -> (block table, [tokens so far])
+        # id -> (block table, [tokens so far], state slot)
+        self.live: dict[str, tuple[list[int], list[int], int | None]] = {}
 
     def step(self, entries) -> np.ndarray | None:
         """``entries``: [(id, tokens, wanted places)].  The wanted logits [n, vocab], or None."""
@@ -40,20 +42,25 @@ class TraceSession:
         for rid, toks, want in entries:
             if not toks or any(not 0 <= t < vocab for t in toks) or any(not 0 <= w < len(toks) for w in want):
                 raise ValueError(f"request {rid}: tokens or wanted places out of range")
-            table, n = self.live.setdefault(rid, ([], [0]))
+            if rid not in self.live:
+                states = self.engine.kv.states
+                self.live[rid] = ([], [0], states.alloc(1)[0] if states is not None else None)
+            table, n, slot = self.live[rid]
             grow = blocks_needed(n[0] + len(toks)) - len(table)
             if grow > 0:
                 table += self.engine.kv.pool.alloc(grow)
             assert len(table) * KV_BLOCK >= n[0] + len(toks)
-            batch.append((toks, n[0], table, want))
+            batch.append((toks, n[0], table, want, slot))
         logits = self.engine.forward_step(batch) if batch else None
         for rid, toks, _ in entries:
             self.live[rid][1][0] += len(toks)
         return None if logits is None else logits.float().cpu().numpy()
 
     def end(self, rid: str) -> None:
-        table, _ = self.live.pop(rid)
+        table, _, slot = self.live.pop(rid)
         self.engine.kv.pool.free(table)
+        if slot is not None:
+            self.engine.kv.states.free([slot])
 
 
 def open_session(model_dir, dtype: str, max_tokens: int, device="cuda:0") -> TraceSession | None:
@@ -77,7 +84,7 @@ def open_session(model_dir, dtype: str, max_tokens: int, device="cuda:0") -> Tra
         _native.ensure_kernels(family.model.kernel_sources(cfg, want))
     torch.set_float32_matmul_precision("highest")
     model = registry.build_model(registry.load_weights(cfg, model_dir, dev, dtype=want))
-    kv = model.new_cache(blocks_needed(max_tokens))
+    kv = model.new_cache(blocks_needed(max_tokens), sequences=LIVE_REQUESTS)
     return TraceSession(LLMEngine(model, kv, use_graph=False, prefix_cache=False))
 
 

@@ -145,10 +145,25 @@ __device__ __forceinline__ uint4 dg_ldw(const uint16_t* p) {
 // 6.0 TB/s from the same 224-256 workgroups.  Packed loads are buffer loads (32-bit offsets into
 // the workgroup's span) so the cache policy can be set: NTW = nontemporal for these once-read
 // bytes (guide "nt-weights").
-template <int BM, int BN, int EPI, bool NTW, int ABL = 0, bool PACKED = true>
+// GRP 1: one matrix per expert, W[experts][N][K] packed one after the other.  grid.y walks the row tiles of a
+// batch sorted by expert: tile y multiplies rows y BM .. by matrix tile_expert[y] (negative: no such tile, the
+// workgroup leaves), row m of it being row rows[m] of X (rows null: m itself); M counts the sorted rows.
+// GRP 2: several inputs, X[inputs][M][K]: the BN rows of W tile n multiply input in_of[n].
+struct DgGroup {
+  const int32_t* rows = nullptr;
+  const int32_t* tile_expert = nullptr;
+  const int32_t* in_of = nullptr;
+};
+
+template <int BM, int BN, int EPI, bool NTW, int ABL = 0, bool PACKED = true, int GRP = 0>
 __global__ void __launch_bounds__((64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES), 1)
     dgemm_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, int M, int N, int K, int ntiles,
-                 int split, float* __restrict__ part, uint16_t* __restrict__ out, int ldo, DgGlu gp) {
+                 int split, float* __restrict__ part, uint16_t* __restrict__ out, int ldo, DgGlu gp, DgGroup grp) {
+  if constexpr (GRP == 1) {
+    const int e = __builtin_amdgcn_readfirstlane(grp.tile_expert[blockIdx.y]);
+    if (e < 0) return;
+    W += (size_t)e * N * K;
+  }
   using S = DgShape<BM, BN, (ABL & 64) != 0>;
   constexpr int NW = S::NW;
   constexpr int D = S::D;
@@ -160,6 +175,7 @@ __global__ void __launch_bounds__((64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES)
   const int lid = xcd_remap(blockIdx.x, gridDim.x);
   const int ks = lid / ntiles, tile = lid % ntiles;
   const int n0 = tile * BN, m0 = blockIdx.y * BM;
+  if constexpr (GRP == 2) X += (size_t)__builtin_amdgcn_readfirstlane(grp.in_of[tile]) * M * K;
   const int nks = K >> 6;
   const int kb = (int)((long)ks * nks / split), ke = (int)((long)(ks + 1) * nks / split);
   const int nst = ke - kb;
@@ -183,7 +199,9 @@ __global__ void __launch_bounds__((64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES)
     const uint16_t* xsrc[S::XP];
 #pragma unroll
     for (int i = 0; i < S::XP; ++i) {
-      const int m = min(m0 + 8 * S::XP * l + 8 * i + prow, M - 1);   // rows past M: results dropped
+      int m = min(m0 + 8 * S::XP * l + 8 * i + prow, M - 1);   // rows past M: results dropped
+      if constexpr (GRP == 1)
+        if (grp.rows) m = grp.rows[m];
       xsrc[i] = X + (size_t)m * K + (size_t)kb * 64 + 8 * pch;
     }
     const uint32_t lds0 =
@@ -407,7 +425,7 @@ int dgemm_launch_bn(const void* x, const void* w, int M, int N, int K, int split
   const int ntiles = N / BN;
   const dim3 grid(ntiles * split, (M + BM - 1) / BM);
   const int threads = 64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES;
-#define DG_ARGS (const uint16_t*)x, (const uint16_t*)w, M, N, K, ntiles, split, part, (uint16_t*)out, ldo, DgGlu{}
+#define DG_ARGS (const uint16_t*)x, (const uint16_t*)w, M, N, K, ntiles, split, part, (uint16_t*)out, ldo, DgGlu{}, DgGroup{}
   switch (epi) {
     case DG_PART: dgemm_kernel<BM, BN, DG_PART, NTW, ABL, PK><<<grid, threads, 0, stream>>>(DG_ARGS); break;
     case DG_PART_WT: dgemm_kernel<BM, BN, DG_PART_WT, NTW, ABL, PK><<<grid, threads, 0, stream>>>(DG_ARGS); break;
@@ -496,7 +514,7 @@ namespace {
 template <int BM, int BN>
 void dgemm_glu_go(const void* x, const void* w, int M, int N, int K, void* out, int ldo, const DgGlu& gp, hipStream_t stream) {
   dgemm_kernel<BM, BN, DG_GLU, DG_NT, 0, true><<<dim3(N / BN, (M + BM - 1) / BM), 64 * DgShape<BM, BN>::WAVES, 0, stream>>>(
-      (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, nullptr, (uint16_t*)out, ldo, gp);
+      (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, nullptr, (uint16_t*)out, ldo, gp, DgGroup{});
 }
 template <int BM>
 int dgemm_glu_bn(const void* x, const void* w, int M, int N, int K, int bn, void* out, int ldo, const DgGlu& gp,
@@ -522,6 +540,80 @@ CFC_API int cfc_dgemm_glu(const void* x, const void* w, int M, int N, int K, int
     case 64: rc = dgemm_glu_bn<64>(x, w, M, N, K, bn, out, ldo, gp, stream); break;
     case 128: rc = dgemm_glu_bn<128>(x, w, M, N, K, bn, out, ldo, gp, stream); break;
     default: rc = dgemm_glu_bn<256>(x, w, M, N, K, bn, out, ldo, gp, stream); break;
+  }
+  return rc ? rc : CFC_CHECK_LAUNCH();
+}
+
+namespace {
+template <int BM, int BN>
+void dgemm_group_go(int glu, const void* x, const void* w, int M, int N, int K, void* out, int ldo, const DgGlu& gp,
+                    const DgGroup& g, hipStream_t stream) {
+  const dim3 grid(N / BN, M / BM);
+  constexpr int threads = 64 * DgShape<BM, BN>::WAVES;
+  if (glu)
+    dgemm_kernel<BM, BN, DG_GLU, DG_NT, 0, true, 1><<<grid, threads, 0, stream>>>(
+        (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, nullptr, (uint16_t*)out, ldo, gp, g);
+  else
+    dgemm_kernel<BM, BN, DG_PART, DG_NT, 0, true, 1><<<grid, threads, 0, stream>>>(
+        (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, (float*)out, nullptr, 0, gp, g);
+}
+template <int BM>
+int dgemm_group_bn(int glu, const void* x, const void* w, int M, int N, int K, int bn, void* out, int ldo, const DgGlu& gp,
+                   const DgGroup& g, hipStream_t stream) {
+  switch (bn) {
+    case 64: dgemm_group_go<BM, 64>(glu, x, w, M, N, K, out, ldo, gp, g, stream); return 0;
+    case 128: dgemm_group_go<BM, 128>(glu, x, w, M, N, K, out, ldo, gp, g, stream); return 0;
+  }
+  return -5;
+}
+}  // namespace
+
+// Products of rows sorted by expert with W[experts][N][K] (each packed for bn): M sorted rows in tiles of bm = 64 or
+// 128, rows / tile_expert as in DgGroup.  glu 0: fp32 out [M][N]; 1: the clamped GLU of 8-row interleaved gate / up
+// rows, bf16 [M][N / 2] (row stride ldo)
+CFC_API int cfc_dgemm_group(int glu, const void* x, const void* w, int M, int N, int K, int bn, int bm, const int32_t* rows,
+                            const int32_t* tile_expert, void* out, int ldo, float limit, float alpha, float beta,
+                            hipStream_t stream) {
+  if (M == 0) return 0;
+  if (const int e = dgemm_check(M, N, K, 1, glu ? DG_GLU : DG_PART, bn, (const float*)out, out, glu ? ldo : N)) return e;
+  if (!tile_expert || (bm != 64 && bm != 128) || M % bm) return -1;
+  DgGlu gp;
+  gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
+  DgGroup g;
+  g.rows = rows; g.tile_expert = tile_expert;
+  const int rc = bm == 64 ? dgemm_group_bn<64>(glu, x, w, M, N, K, bn, out, ldo, gp, g, stream)
+                          : dgemm_group_bn<128>(glu, x, w, M, N, K, bn, out, ldo, gp, g, stream);
+  return rc ? rc : CFC_CHECK_LAUNCH();
+}
+
+namespace {
+template <int BM>
+int dgemm_joint_bn(const void* x, const void* w, int M, int N, int K, int split, int bn, float* part, const DgGroup& g,
+                   hipStream_t stream) {
+#define DJ(BN)                                                                                                       \
+  case BN:                                                                                                           \
+    dgemm_kernel<BM, BN, DG_PART_WT, DG_NT, 0, true, 2>                                                              \
+        <<<dim3(N / BN * split, (M + BM - 1) / BM), 64 * DgShape<BM, BN>::WAVES, 0, stream>>>(                       \
+            (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, split, part, nullptr, 0, DgGlu{}, g);           \
+    return 0;
+  switch (bn) { DJ(64) DJ(128) }
+#undef DJ
+  return -5;
+}
+}  // namespace
+
+// fp32 split-K slabs part[split][M][N] of X[inputs][M][K], the bn rows of W tile n multiplying input in_of[n]
+CFC_API int cfc_dgemm_joint(const void* x, const void* w, int M, int N, int K, int split, int bn, const int32_t* in_of,
+                            float* part, hipStream_t stream) {
+  if (const int e = dgemm_check(M, N, K, split, DG_PART_WT, bn, part, nullptr, N)) return e;
+  if (!in_of) return -1;
+  DgGroup g;
+  g.in_of = in_of;
+  int rc;
+  switch (cfc_dgemm_bm(M)) {
+    case 64: rc = dgemm_joint_bn<64>(x, w, M, N, K, split, bn, part, g, stream); break;
+    case 128: rc = dgemm_joint_bn<128>(x, w, M, N, K, split, bn, part, g, stream); break;
+    default: rc = dgemm_joint_bn<256>(x, w, M, N, K, split, bn, part, g, stream); break;
   }
   return rc ? rc : CFC_CHECK_LAUNCH();
 }

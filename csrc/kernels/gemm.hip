@@ -243,17 +243,20 @@ struct GvNorm {
   float eps;
 };
 
+// in_of: several inputs X[inputs][M][K], W tile n multiplying input in_of[n] (null: one input)
 template <int NW, int MT, int WAVES, bool XN>
 __global__ void __launch_bounds__(64 * WAVES) gemv_tile_kernel(const uint16_t* __restrict__ X,
                                                         const uint16_t* __restrict__ Wp, int N, int K, int S, int epi,
                                                         float* __restrict__ yf, uint16_t* __restrict__ yb, int ldo,
-                                                        GvNorm nm) {
+                                                        GvNorm nm, const int32_t* __restrict__ in_of) {
   constexpr int U = MT > 2 ? 2 : (NW >= 7 ? 3 : 4);
   constexpr int R = NW * MT * 16;                  // (group, m, row) values of one tile
   __shared__ float red[WAVES][R];
   extern __shared__ uint4 xs[];                    // XN: the normalised rows [MT][K] (bf16)
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, q = lane >> 4;
   const int tile = blockIdx.x / S, s = blockIdx.x - tile * S;
+  if constexpr (!XN)
+    if (in_of) X += (size_t)in_of[tile] * MT * K;
   const int KG = K / 32;
   const int kb = s * KG / S, ke = (s + 1) * KG / S;
   const uint16_t* base = Wp + (size_t)tile * KG * NW * 512;
@@ -445,7 +448,7 @@ CFC_API int cfc_gemv(const void* x, const void* w, int M, int N, int K, int epi,
 namespace {
 template <int NW, int MT, int WAVES, bool XN>
 void gemv_tile_go(dim3 grid, hipStream_t stream, const uint16_t* x, const uint16_t* wp, int N, int K, int split, int epi,
-                  float* yf, uint16_t* yb, int ldo, const GvNorm& nm) {
+                  float* yf, uint16_t* yb, int ldo, const GvNorm& nm, const int32_t* in_of) {
   const size_t lds = XN ? (size_t)MT * K * 2 : 0;
   if constexpr (XN) {
     static bool raised = false;                    // dynamic LDS past 64 KB (Llama-70B rows at M = 4)
@@ -455,16 +458,16 @@ void gemv_tile_go(dim3 grid, hipStream_t stream, const uint16_t* x, const uint16
       raised = true;
     }
   }
-  gemv_tile_kernel<NW, MT, WAVES, XN><<<grid, 64 * WAVES, lds, stream>>>(x, wp, N, K, split, epi, yf, yb, ldo, nm);
+  gemv_tile_kernel<NW, MT, WAVES, XN><<<grid, 64 * WAVES, lds, stream>>>(x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of);
 }
 
 template <int NW, int MT>
 void gemv_tile_launch(dim3 grid, int waves, hipStream_t stream, const uint16_t* x, const uint16_t* wp, int N, int K,
-                      int split, int epi, float* yf, uint16_t* yb, int ldo, const GvNorm& nm) {
+                      int split, int epi, float* yf, uint16_t* yb, int ldo, const GvNorm& nm, const int32_t* in_of) {
   const bool xn = nm.part != nullptr;
 #define GVT(WV)                                                                                    \
-  if (xn) gemv_tile_go<NW, MT, WV, true>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm);  \
-  else gemv_tile_go<NW, MT, WV, false>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm);
+  if (xn) gemv_tile_go<NW, MT, WV, true>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of);  \
+  else gemv_tile_go<NW, MT, WV, false>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of);
   if (waves == 4) { GVT(4) }
   else if (waves == 8) { GVT(8) }
   else if constexpr (MT == 1) { GVT(16) }         // 16 waves: 4 per SIMD, so <= 128 VGPRs -- single-row only
@@ -474,10 +477,11 @@ void gemv_tile_launch(dim3 grid, int waves, hipStream_t stream, const uint16_t* 
 
 // M <= 4 GEMV over a fragment-packed W (cfc_dgemm_pack layout for bn = 16 nw, nw in {4, 6, 7, 8}):
 // epilogues as cfc_gemv; split > 1 (fp32 only): yf = slabs [split, M, N] of the k-slice partial
-// sums.  N % (16 nw) == 0, K % 32 == 0, 1 <= split <= K / 32.
+// sums.  in_of (may be null): X[inputs][M][K], W tile n multiplying input in_of[n].  N % (16 nw) == 0, K % 32 == 0, 1 <= split <= K / 32.
 CFC_API int cfc_gemv_packed(const void* x, const void* wp, int M, int N, int K, int nw, int epi, float* yf, void* yb,
                             int ldo, int split, int waves, const float* xpart, int xsplit, const void* res_in,
-                            void* res_out, const void* norm_w, float eps, hipStream_t stream) {
+                            void* res_out, const void* norm_w, float eps, const int32_t* in_of,
+                            hipStream_t stream) {
   if (M < 1 || M > 4 || N <= 0 || nw <= 0 || N % (16 * nw) || K <= 0 || K % 32) return -1;
   if ((epi == GV_F32 && !yf) || (epi != GV_F32 && !yb) || epi < 0 || epi > 2) return -2;
   if (split < 1 || split > K / 32 || (split > 1 && epi != GV_F32)) return -4;
@@ -485,9 +489,10 @@ CFC_API int cfc_gemv_packed(const void* x, const void* wp, int M, int N, int K, 
   // the fused-norm prologue holds the first step's weights across the slab sums: <= 8 waves (VGPRs)
   if (xpart ? (xsplit < 1 || !res_in || !res_out || !norm_w || res_in == res_out || K > 8192 || waves > 8) : !x)
     return -6;
+  if (in_of && xpart) return -6;
   const GvNorm nm{xpart, xsplit, (const uint16_t*)res_in, (uint16_t*)res_out, (const uint16_t*)norm_w, eps};
   const dim3 grid((N / (16 * nw)) * split);
-#define GVP_ARGS (const uint16_t*)x, (const uint16_t*)wp, N, K, split, epi, yf, (uint16_t*)yb, ldo, nm
+#define GVP_ARGS (const uint16_t*)x, (const uint16_t*)wp, N, K, split, epi, yf, (uint16_t*)yb, ldo, nm, in_of
 #define GVP_CASE(NW)                                                                         \
   case NW:                                                                                   \
     switch (M) {                                                                             \

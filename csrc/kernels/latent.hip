@@ -6,6 +6,8 @@
 //
 //   * latent_norm     RMS norms of the query latent and the cached latent from the fp32 slabs of the
 //                     joint down projection; the latter goes straight into the cache slot
+//   * latent_rope     the same for designs with rotary positions: the normed latent and, behind it in the
+//                     row, the rotated key part all heads share; the heads' rotated query parts
 //   * head_linear     out[t][h] = W[h] in[t][h], the per-head products on both sides of the attention
 //   * latent_attn     flash-style attention over the paged latents.  A work item is 16 MR rows of the
 //                     flattened (token, head) rows of one sequence -- one decoded token's heads and a
@@ -119,6 +121,101 @@ int latent_norm_go(hipStream_t st, const float* part, int split, int T, int NQ, 
   return CFC_CHECK_LAUNCH();
 }
 
+// ---------------------------------------------------------------------------------- latent_rope
+// Columns of a product: activations (split 0) or fp32 slabs.
+struct LatCols { const void* p; int split; int64_t ld, plane; };
+
+template <typename ACT>
+__device__ __forceinline__ float ldcol(const LatCols& a, int64_t t, int c) {
+  const int64_t o = t * a.ld + c;
+  if (a.split == 0) return ldf(reinterpret_cast<const ACT*>(a.p) + o);
+  const float* p = reinterpret_cast<const float*>(a.p) + o;
+  float s = 0.f;
+  for (int i0 = 0; i0 < a.split; i0 += 8) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v[u] = p[(int64_t)min(i0 + u, a.split - 1) * a.plane];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) s += i0 + u < a.split ? v[u] : 0.f;
+  }
+  return s;
+}
+
+struct RopeArgs {
+  const float* freq;          // [rot / 2]
+  float mag;                  // on cos and sin
+  const int32_t* positions;
+  int rot;
+};
+
+__device__ __forceinline__ void rope_pair(const RopeArgs& r, int pos, int i, float& u, float& v) {
+  float sn, cs;
+  sincosf((float)pos * r.freq[i], &sn, &cs);
+  cs *= r.mag;
+  sn *= r.mag;
+  const float a = u * cs - v * sn, b = v * cs + u * sn;
+  u = a;
+  v = b;
+}
+
+// grid (rows, 1 + heads).  y = 0: RMS norm of the NC latent columns, the rotated key part behind them
+// (from column RV of the cache row).  y = 1 + h: head h's rotated query part at columns RV .. RS of its row of
+// ql (the pad zeroed); where q comes as slabs its unrotated part goes to qn [T][H][dim] as activations, and the
+// output gate's columns to gate [T][H vdim].
+template <typename ACT>
+__global__ void __launch_bounds__(256) latent_rope_kernel(LatCols kv, int NC, const float* __restrict__ wc, float eps,
+                                                         const int32_t* __restrict__ slots, ACT* __restrict__ cache, int RS,
+                                                         int RV, LatCols q, int dim, ACT* __restrict__ ql,
+                                                         ACT* __restrict__ qn, LatCols g, int vdim, ACT* __restrict__ gate,
+                                                         RopeArgs r) {
+  __shared__ float red[16];
+  const int t = blockIdx.x, tid = threadIdx.x, H = gridDim.y - 1, pos = r.positions[t];
+  if (blockIdx.y == 0) {
+    ACT* dst = cache + (size_t)slots[t] * RS;
+    float x[4], s = 0.f;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int c = k * 256 + tid;
+      x[k] = c < NC ? ldcol<ACT>(kv, t, c) : 0.f;
+      s += x[k] * x[k];
+    }
+    for (int c = 1024 + tid; c < NC; c += 256) {
+      const float v = ldcol<ACT>(kv, t, c);
+      s += v * v;
+    }
+    const float rs = 1.f / sqrtf(block_sum(s, red) / (float)NC + eps);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int c = k * 256 + tid;
+      if (c < NC) stf(dst + c, x[k] * rs * wc[c]);
+    }
+    for (int c = 1024 + tid; c < NC; c += 256) stf(dst + c, ldcol<ACT>(kv, t, c) * rs * wc[c]);
+    for (int i = tid; i < r.rot / 2; i += 256) {
+      float u = ldcol<ACT>(kv, t, NC + 2 * i), v = ldcol<ACT>(kv, t, NC + 2 * i + 1);
+      rope_pair(r, pos, i, u, v);
+      stf(dst + RV + 2 * i, u);
+      stf(dst + RV + 2 * i + 1, v);
+    }
+    return;
+  }
+  const int h = blockIdx.y - 1, q0 = h * (dim + r.rot);
+  ACT* row = ql + ((size_t)t * H + h) * RS;
+  for (int i = tid; i < (RS - RV) / 2; i += 256) {
+    float u = 0.f, v = 0.f;
+    if (i < r.rot / 2) {
+      u = ldcol<ACT>(q, t, q0 + dim + 2 * i);
+      v = ldcol<ACT>(q, t, q0 + dim + 2 * i + 1);
+      rope_pair(r, pos, i, u, v);
+    }
+    stf(row + RV + 2 * i, u);
+    stf(row + RV + 2 * i + 1, v);
+  }
+  if (qn)
+    for (int c = tid; c < dim; c += 256) stf(qn + ((size_t)t * H + h) * dim + c, ldcol<ACT>(q, t, q0 + c));
+  if (gate)
+    for (int c = tid; c < vdim; c += 256) stf(gate + ((size_t)t * H + h) * vdim + c, ldcol<ACT>(g, t, h * vdim + c));
+}
+
 // ---------------------------------------------------------------------------------- head_linear
 // W [H][NP][KP] zero-padded (NP % 64 == 0, KP % 32 == 0).  Operands: A = W rows, B = token rows, so a
 // lane ends with four consecutive outputs of one token.  grid (token tiles, NP / (16 NT 4), H), four
@@ -126,6 +223,17 @@ int latent_norm_go(hipStream_t st, const float* part, int split, int T, int NQ, 
 __device__ __forceinline__ f32x4_t mfma16(uint4 a, uint4 b, f32x4_t c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0,
                                                  0, 0);
+}
+
+__device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + __expf(-z)); }
+
+// four consecutive outputs times the sigmoid of their gates
+__device__ __forceinline__ void gate4(float (&v)[4], const uint16_t* g) {
+  const uint2 u = *reinterpret_cast<const uint2*>(g);
+  v[0] *= sigmoid(__uint_as_float(u.x << 16));
+  v[1] *= sigmoid(__uint_as_float(u.x & 0xffff0000u));
+  v[2] *= sigmoid(__uint_as_float(u.y << 16));
+  v[3] *= sigmoid(__uint_as_float(u.y & 0xffff0000u));
 }
 
 template <bool VEC>
@@ -146,7 +254,8 @@ __device__ __forceinline__ uint4 ld_frag(const uint16_t* p, int k, int K) {
 template <int TT, int NT, bool VEC>
 __global__ void __launch_bounds__(256) head_linear_kernel(const uint16_t* __restrict__ x, int64_t ldx, int64_t hsx,
                                                          const uint16_t* __restrict__ w, int NP, int KP, int T, int N,
-                                                         int K, uint16_t* __restrict__ out, int64_t ldo, int64_t hso) {
+                                                         int K, uint16_t* __restrict__ out, int64_t ldo, int64_t hso,
+                                                         const uint16_t* __restrict__ gate, int64_t ldg) {
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
   const int h = blockIdx.z, t0 = blockIdx.x * 16 * TT, n0 = (blockIdx.y * 4 + wv) * 16 * NT;
   if (n0 >= NP) return;
@@ -188,14 +297,16 @@ __global__ void __launch_bounds__(256) head_linear_kernel(const uint16_t* __rest
     for (int j = 0; j < NT; ++j) {
       const int n = n0 + 16 * j + 4 * kq;
       if constexpr (VEC) {
-        if (n < N)
-          *reinterpret_cast<uint2*>(o + n) =
-              make_uint2(pack2bf(acc[j][i][0], acc[j][i][1]), pack2bf(acc[j][i][2], acc[j][i][3]));
+        if (n < N) {
+          float v[4] = {acc[j][i][0], acc[j][i][1], acc[j][i][2], acc[j][i][3]};
+          if (gate) gate4(v, gate + (int64_t)t * ldg + (size_t)h * N + n);
+          *reinterpret_cast<uint2*>(o + n) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
+        }
       } else {
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const float v = acc[j][i][e];
-          if (n + e < N) o[n + e] = f2bf(v);
+          if (n + e < N) o[n + e] = f2bf(gate ? v * sigmoid(bf2f(gate[(int64_t)t * ldg + (size_t)h * N + n + e])) : v);
         }
       }
     }
@@ -207,7 +318,8 @@ __global__ void __launch_bounds__(256) head_linear_kernel(const uint16_t* __rest
 template <int TT>
 __global__ void __launch_bounds__(256) head_linear_ks_kernel(const uint16_t* __restrict__ x, int64_t ldx, int64_t hsx,
                                                             const uint16_t* __restrict__ w, int NP, int KP, int T, int N,
-                                                            int K, uint16_t* __restrict__ out, int64_t ldo, int64_t hso) {
+                                                            int K, uint16_t* __restrict__ out, int64_t ldo, int64_t hso,
+                                                         const uint16_t* __restrict__ gate, int64_t ldg) {
   __shared__ float4 red[3][TT][64];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
   const int h = blockIdx.z, t0 = blockIdx.x * 16 * TT, n0 = blockIdx.y * 16;
@@ -249,20 +361,24 @@ __global__ void __launch_bounds__(256) head_linear_ks_kernel(const uint16_t* __r
       v[0] += r.x; v[1] += r.y; v[2] += r.z; v[3] += r.w;
     }
     const int t = t0 + 16 * i + col, n = n0 + 4 * kq;
-    if (t < T && n < N)
+    if (t < T && n < N) {
+      if (gate) gate4(v, gate + (int64_t)t * ldg + (size_t)h * N + n);
       *reinterpret_cast<uint2*>(out + (int64_t)t * ldo + h * hso + n) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
+    }
   }
 }
 
 __global__ void __launch_bounds__(256) head_linear_f32_kernel(const float* __restrict__ x, int64_t ldx, int64_t hsx,
                                                              const float* __restrict__ w, int NP, int KP, int N, int K,
-                                                             float* __restrict__ out, int64_t ldo, int64_t hso) {
+                                                             float* __restrict__ out, int64_t ldo, int64_t hso,
+                                                             const float* __restrict__ gate, int64_t ldg) {
   const int n = blockIdx.y * 256 + threadIdx.x, t = blockIdx.x, h = blockIdx.z;
   if (n >= N) return;
   const float* xr = x + t * ldx + h * hsx;
   const float* wr = w + ((size_t)h * NP + n) * KP;
   float s = 0.f;
   for (int k = 0; k < K; ++k) s += xr[k] * wr[k];
+  if (gate) s *= sigmoid(gate[t * ldg + (size_t)h * N + n]);
   out[t * ldo + h * hso + n] = s;
 }
 
@@ -273,13 +389,25 @@ struct LatArgs {
   const int32_t* ctx_lens;    // cached + new tokens
   const int32_t* tile_seq;    // null: tile b is rows 16 MR (b % tiles_per_seq) of sequence b / tiles_per_seq
   const int32_t* tile_m0;
-  int tiles_per_seq, H, RS, max_blocks, P;
+  int tiles_per_seq, H, RS, RV, max_blocks, P;   // RS: columns of a key, RV: of them the value
   float scale;
-  float* part_o;              // [rows][P][RS], unnormalised
+  int window;                 // keys a row sees, itself included (0: all before it)
+  const float* sink;          // [H] or null: exp(sink) joins the denominator once
+  float* part_o;              // [rows][P][RV], unnormalised
   float* part_ml;             // [rows][P][2]: running maximum (log2 domain), sum
 };
 
 struct LatTile { int m0, rows, q_row, pos_base, kt0, kt1, kend; const int32_t* bt; };
+
+// first key a row with ``limit`` keys before its end sees
+__device__ __forceinline__ int lat_low(const LatArgs& a, int limit) { return a.window > 0 ? max(limit - a.window, 0) : 0; }
+
+// running maximum m (log2 domain) and sum l with the row's sink: what to scale the output by
+__device__ __forceinline__ float lat_inv(const LatArgs& a, int row, float m, float l) {
+  if (!a.sink) return l > 0.f ? 1.f / l : 0.f;
+  const float sk = a.sink[row % a.H] * 1.4426950408889634f, M = fmaxf(m, sk), f = exp2f(m - M);
+  return f / (l * f + exp2f(sk - M));
+}
 
 // the tile's rows and its slice of 64-key tiles
 __device__ __forceinline__ LatTile lat_tile(const LatArgs& a, int tile, int p, int rows_per_tile) {
@@ -291,9 +419,9 @@ __device__ __forceinline__ LatTile lat_tile(const LatArgs& a, int tile, int p, i
   r.q_row = q0 * a.H;
   r.pos_base = a.ctx_lens[s] - n;
   r.kend = r.pos_base + (min(r.m0 + rows_per_tile, r.rows) - 1) / a.H + 1;
-  const int nt = (r.kend + 63) / 64;
-  r.kt0 = (int)((int64_t)nt * p / a.P);
-  r.kt1 = (int)((int64_t)nt * (p + 1) / a.P);
+  const int t0 = lat_low(a, r.pos_base + r.m0 / a.H + 1) / 64, nt = (r.kend + 63) / 64 - t0;
+  r.kt0 = t0 + (int)((int64_t)nt * p / a.P);
+  r.kt1 = t0 + (int)((int64_t)nt * (p + 1) / a.P);
   r.bt = a.block_tables + (size_t)s * a.max_blocks;
   return r;
 }
@@ -317,7 +445,7 @@ constexpr int LP = 72;      // P row stride in LDS, elements (64 keys + 8 agains
 // Two phases per tile, a barrier after each: [scores of tile t + 1 | output of tile t], independent of each
 // other, then [softmax of t + 1, tile t + 2 from registers into the buffer t leaves, loads of t + 3].  The
 // barriers order LDS only, so the loads stay in flight across a whole tile.
-template <int R64, int MR>
+template <int R64, int V64, int MR>
 __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __restrict__ q,
                                                             const uint16_t* __restrict__ cache, LatArgs a,
                                                             uint16_t* __restrict__ out) {
@@ -336,7 +464,7 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
   constexpr int NL = CH / 8;                      // chunks per thread of a 64-key tile
   constexpr int KG = MR == 4 ? 2 : 1;             // 16-key groups per wave
   constexpr int SL = 4 / KG;                      // waves per row group
-  constexpr int RT = R64 / 16;                    // 16-column output tiles
+  constexpr int RT = V64 / 16;                    // 16-column output tiles
   constexpr int NO = (RT + 7) / 8;                // per wave
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char* kbuf = smem;                                            // [2][64][R64] bf16
@@ -354,7 +482,8 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
   const int rg = MR == 1 ? 0 : w % MR, slot = MR == 1 ? w : w / MR;
   const bool scorer = slot < SL;
   const int gm = min(tl.m0 + 16 * rg + col, tl.rows - 1);
-  const int limit = tl.pos_base + gm / a.H + 1;   // keys this row sees
+  const int limit = tl.pos_base + gm / a.H + 1;   // keys this row sees: low .. limit - 1
+  const int low = lat_low(a, limit);
   u32x4_t qf[KS];
   if (scorer) {
     const uint16_t* qr = q + (size_t)(tl.q_row + gm) * RS + 8 * kq;
@@ -428,7 +557,7 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
       const int k0 = kt * 64 + 16 * (slot * KG + g) + 4 * kq;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        s[g][i] = k0 + i < limit ? (s0[i] + s1[i]) * a.scale : -INFINITY;
+        s[g][i] = (unsigned)(k0 + i - low) < (unsigned)(limit - low) ? (s0[i] + s1[i]) * a.scale : -INFINITY;
         mx = fmaxf(mx, s[g][i]);
       }
     }
@@ -559,11 +688,11 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
     for (int u = 0; u < SL; ++u) lt += smax[(r * 4 + u) * 16 + col];
     const size_t grow = (size_t)tl.q_row + mrow;
     if (a.P > 1) {
-      float* po = a.part_o + (grow * a.P + blockIdx.y) * RS;
+      float* po = a.part_o + (grow * a.P + blockIdx.y) * a.RV;
 #pragma unroll
       for (int j = 0; j < NO; ++j) {
         const int n = 16 * (w + 8 * j) + 4 * kq;
-        if (w + 8 * j < RT && n < RS) *reinterpret_cast<float4*>(po + n) = make_float4(o[j][r][0], o[j][r][1], o[j][r][2], o[j][r][3]);
+        if (w + 8 * j < RT && n < a.RV) *reinterpret_cast<float4*>(po + n) = make_float4(o[j][r][0], o[j][r][1], o[j][r][2], o[j][r][3]);
       }
       if (w == 0 && kq == 0) {
         float* ml = a.part_ml + (grow * a.P + blockIdx.y) * 2;
@@ -571,12 +700,12 @@ __global__ void __launch_bounds__(512, 1) latent_attn_kernel(const uint16_t* __r
         ml[1] = lt;
       }
     } else {
-      const float inv = lt > 0.f ? 1.f / lt : 0.f;
-      uint16_t* po = out + grow * RS;
+      const float inv = lat_inv(a, mrow, salpha[16 * r + col], lt);
+      uint16_t* po = out + grow * a.RV;
 #pragma unroll
       for (int j = 0; j < NO; ++j) {
         const int n = 16 * (w + 8 * j) + 4 * kq;
-        if (w + 8 * j < RT && n < RS)
+        if (w + 8 * j < RT && n < a.RV)
           *reinterpret_cast<uint2*>(po + n) = make_uint2(cvt_pk_bf16_f32(o[j][r][0] * inv, o[j][r][1] * inv),
                                                          cvt_pk_bf16_f32(o[j][r][2] * inv, o[j][r][3] * inv));
       }
@@ -599,7 +728,7 @@ __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restr
   const size_t grow = (size_t)tl.q_row + (live ? mrow : tl.rows - 1);
   for (int c = lane; c < RS; c += 64) myq[c] = ldf(q + grow * RS + c);
   __syncthreads();
-  const int limit = tl.pos_base + (live ? mrow : tl.rows - 1) / a.H + 1;
+  const int limit = tl.pos_base + (live ? mrow : tl.rows - 1) / a.H + 1, low = lat_low(a, limit);
   float o[LG_C];
 #pragma unroll
   for (int j = 0; j < LG_C; ++j) o[j] = 0.f;
@@ -607,7 +736,7 @@ __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restr
   for (int kt = tl.kt0; kt < tl.kt1; ++kt) {
     const int key = kt * 64 + lane;
     float s = -INFINITY;
-    if (key < limit) {
+    if (key < limit && key >= low) {
       const ACT* c = cache + ((size_t)tl.bt[key / CFC_KV_BS] * CFC_KV_BS + key % CFC_KV_BS) * RS;
       float s4[4] = {0.f, 0.f, 0.f, 0.f};
       for (int r = 0; r < RS; r += 4)
@@ -625,24 +754,24 @@ __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restr
 #pragma unroll
     for (int j = 0; j < LG_C; ++j) o[j] *= alpha;
     const int nk = min(64, limit - kt * 64);
-    for (int k = 0; k < nk; ++k) {
+    for (int k = max(0, low - kt * 64); k < nk; ++k) {
       const int kk = kt * 64 + k;
       const ACT* c = cache + ((size_t)tl.bt[kk / CFC_KV_BS] * CFC_KV_BS + kk % CFC_KV_BS) * RS;
       const float pk = pw[k];
 #pragma unroll
       for (int j = 0; j < LG_C; ++j)
-        if (lane + 64 * j < RS) o[j] += pk * ldf(c + lane + 64 * j);
+        if (lane + 64 * j < a.RV) o[j] += pk * ldf(c + lane + 64 * j);
     }
     __syncthreads();
   }
   if (!live) return;
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv = lat_inv(a, mrow, m, l);
 #pragma unroll
   for (int j = 0; j < LG_C; ++j) {
     const int c = lane + 64 * j;
-    if (c >= RS) continue;
-    if (a.P > 1) a.part_o[(grow * a.P + blockIdx.y) * RS + c] = o[j];
-    else stf(out + grow * RS + c, o[j] * inv);
+    if (c >= a.RV) continue;
+    if (a.P > 1) a.part_o[(grow * a.P + blockIdx.y) * a.RV + c] = o[j];
+    else stf(out + grow * a.RV + c, o[j] * inv);
   }
   if (a.P > 1 && lane == 0) {
     a.part_ml[(grow * a.P + blockIdx.y) * 2] = m;
@@ -678,7 +807,7 @@ constexpr int LC_MAXP = 256;
 template <typename ACT>
 __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __restrict__ part_o,
                                                             const float* __restrict__ part_ml, int P, int RS,
-                                                            ACT* __restrict__ out) {
+                                                            const float* __restrict__ sink, int H, ACT* __restrict__ out) {
   __shared__ float wt[LC_MAXP];
   const size_t row = blockIdx.x;
   const float* ml = part_ml + row * P * 2;
@@ -693,6 +822,8 @@ __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __rest
     mx = fmaxf(mx, m[i]);
   }
   mx = wave_max(mx);
+  const float sk = sink ? sink[row % H] * 1.4426950408889634f : -INFINITY;
+  mx = fmaxf(mx, sk);
   const float ref = mx == -INFINITY ? 0.f : mx;
   float sum = 0.f;
 #pragma unroll
@@ -700,7 +831,7 @@ __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __rest
     m[i] = exp2f(m[i] - ref);
     sum += m[i] * l[i];
   }
-  sum = wave_sum(sum);
+  sum = wave_sum(sum) + exp2f(sk - ref);          // no sink: 0
   const float inv = sum > 0.f ? 1.f / sum : 0.f;
   if (threadIdx.x < 64) {
 #pragma unroll
@@ -725,25 +856,25 @@ __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __rest
   }
 }
 
-template <int R64, int MR>
+template <int R64, int V64, int MR>
 int lat_go(dim3 grid, hipStream_t s, const void* q, const void* cache, const LatArgs& a, void* out) {
   constexpr int lds = 2 * 64 * R64 * 2 + 16 * MR * LP * 2 + (MR * 64 + 16 * MR) * 4;
   static bool raised = false;
   if (lds > 65536 && !raised) {
-    hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<R64, MR>),
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<R64, V64, MR>),
                         hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     raised = true;
   }
-  latent_attn_kernel<R64, MR><<<grid, 512, lds, s>>>((const uint16_t*)q, (const uint16_t*)cache, a, (uint16_t*)out);
+  latent_attn_kernel<R64, V64, MR><<<grid, 512, lds, s>>>((const uint16_t*)q, (const uint16_t*)cache, a, (uint16_t*)out);
   return CFC_CHECK_LAUNCH();
 }
 
-template <int R64>
+template <int R64, int V64>
 int lat_mr(int mr, dim3 grid, hipStream_t s, const void* q, const void* cache, const LatArgs& a, void* out) {
   switch (mr) {
-    case 1: return lat_go<R64, 1>(grid, s, q, cache, a, out);
-    case 2: return lat_go<R64, 2>(grid, s, q, cache, a, out);
-    case 4: return lat_go<R64, 4>(grid, s, q, cache, a, out);
+    case 1: return lat_go<R64, V64, 1>(grid, s, q, cache, a, out);
+    case 2: return lat_go<R64, V64, 2>(grid, s, q, cache, a, out);
+    case 4: return lat_go<R64, V64, 4>(grid, s, q, cache, a, out);
   }
   return -3;
 }
@@ -762,25 +893,47 @@ CFC_API int cfc_latent_norm(int f32, const float* part, int split, int T, int NQ
 #undef LN_ARGS
 }
 
-// x row (t, h) at t ldx + h hsx (K values), out at t ldo + h hso (N values); W [H][NP][KP] zero-padded
+// kv columns [NC latent | rot key part], q columns per head [dim | rot]; each operand: pointer, split (0:
+// activations, else fp32 slabs), row stride, slab stride.  ql [T][H][RS]; qn, gate may be null
+CFC_API int cfc_latent_rope(int f32, const void* kv, int kv_split, int64_t kv_ld, int64_t kv_plane, int T, int NC,
+                            const float* wc, float eps, const int32_t* slots, void* cache, int RS, int RV, const void* q,
+                            int q_split, int64_t q_ld, int64_t q_plane, int H, int dim, void* ql, void* qn, const void* g,
+                            int g_split, int64_t g_ld, int64_t g_plane, int vdim, void* gate, const float* freq, int rot,
+                            float mag, const int32_t* positions, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (NC < 1 || NC > RV || RV % 2 || rot < 0 || rot % 2 || RV + rot > RS || RS % 2 || H < 1 || H > 65534 || dim < 1) return -1;
+  const LatCols ckv{kv, kv_split, kv_ld, kv_plane}, cq{q, q_split, q_ld, q_plane}, cg{g, g_split, g_ld, g_plane};
+  const RopeArgs r{freq, mag, positions, rot};
+#define LR(ACT)                                                                                                         \
+  latent_rope_kernel<ACT><<<dim3(T, 1 + H), 256, 0, stream>>>(ckv, NC, wc, eps, slots, (ACT*)cache, RS, RV, cq, dim, (ACT*)ql, \
+                                                             (ACT*)qn, cg, vdim, (ACT*)gate, r)
+  if (f32) LR(float);
+  else LR(uint16_t);
+#undef LR
+  return CFC_CHECK_LAUNCH();
+}
+
+// x row (t, h) at t ldx + h hsx (K values), out at t ldo + h hso (N values); W [H][NP][KP] zero-padded.
+// gate (may be null): output n of head h is multiplied by the sigmoid of gate[t ldg + h N + n]
 CFC_API int cfc_head_linear(int f32, const void* x, int64_t ldx, int64_t hsx, const void* w, int NP, int KP, int T, int H,
-                            int N, int K, void* out, int64_t ldo, int64_t hso, hipStream_t stream) {
+                            int N, int K, void* out, int64_t ldo, int64_t hso, const void* gate, int64_t ldg,
+                            hipStream_t stream) {
   if (T <= 0) return 0;
   if (H < 1 || H > 65535 || N < 1 || K < 1 || N > NP || K > KP || NP % 64 || KP % 32) return -1;
   if (f32) {
     const dim3 grid(T, (N + 255) / 256, H);
     head_linear_f32_kernel<<<grid, 256, 0, stream>>>((const float*)x, ldx, hsx, (const float*)w, NP, KP, N, K, (float*)out,
-                                                     ldo, hso);
+                                                     ldo, hso, (const float*)gate, ldg);
     return CFC_CHECK_LAUNCH();
   }
   const bool vec = K % 8 == 0 && ldx % 8 == 0 && hsx % 8 == 0 && ((uintptr_t)x & 15) == 0 && N % 4 == 0 && ldo % 4 == 0 &&
-                   hso % 4 == 0 && ((uintptr_t)out & 7) == 0;
+                   hso % 4 == 0 && ((uintptr_t)out & 7) == 0 && ldg % 4 == 0 && ((uintptr_t)gate & 7) == 0;
 #define HL(TT, NT, V)                                                                                                 \
   head_linear_kernel<TT, NT, V><<<dim3((T + 16 * TT - 1) / (16 * TT), (NP + 64 * NT - 1) / (64 * NT), H), 256, 0, stream>>>( \
-      (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso)
+      (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso, (const uint16_t*)gate, ldg)
 #define HK(TT)                                                                                                   \
   head_linear_ks_kernel<TT><<<dim3((T + 16 * TT - 1) / (16 * TT), (N + 15) / 16, H), 256, 0, stream>>>(          \
-      (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso)
+      (const uint16_t*)x, ldx, hsx, (const uint16_t*)w, NP, KP, T, N, K, (uint16_t*)out, ldo, hso, (const uint16_t*)gate, ldg)
   if (!vec) HL(4, 1, false);
   else if (T <= 256 && KP >= 256 && T <= 16) HK(1);
   else if (T <= 64 && KP >= 256) HK(2);
@@ -793,18 +946,20 @@ CFC_API int cfc_head_linear(int f32, const void* x, int64_t ldx, int64_t hsx, co
   return CFC_CHECK_LAUNCH();
 }
 
-// rows_per_tile: 16 / 32 / 64 on the MFMA kernel (bf16, rank <= 512), 4 on the general one
+// rows_per_tile: 16 / 32 / 64 on the MFMA kernel (bf16, RS <= 512, or RS <= 576 with RV <= 512), 4 on the general
+// one.  A cached row's RS columns are the key, its first RV the value; out [rows][RV]
 CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, const int32_t* block_tables,
                                  const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tile_seq,
                                  const int32_t* tile_m0, int n_tiles, int tiles_per_seq, int rows_per_tile, int H, int RS,
-                                 int max_blocks, float scale, int P, int total_rows, float* part_o, float* part_ml,
+                                 int RV, int max_blocks, float scale, int window, const float* sink, int P, int total_rows, float* part_o, float* part_ml,
                                  void* out, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (H < 1 || RS < 32 || RS % 32 || P < 1 || P > LC_MAXP || max_blocks < 1) return -1;
+  if (H < 1 || RS < 32 || RS % 32 || RV < 32 || RV % 32 || RV > RS || P < 1 || P > LC_MAXP || max_blocks < 1 || window < 0)
+    return -1;
   if ((tile_seq == nullptr) != (tile_m0 == nullptr) || (!tile_seq && tiles_per_seq < 1)) return -1;
   if (P > 1 && (!part_o || !part_ml)) return -2;
-  LatArgs a{block_tables, cu_q, ctx_lens, tile_seq, tile_m0, tiles_per_seq, H, RS, max_blocks, P,
-            scale * 1.4426950408889634f, part_o, part_ml};
+  LatArgs a{block_tables, cu_q, ctx_lens, tile_seq, tile_m0, tiles_per_seq, H, RS, RV, max_blocks, P,
+            scale * 1.4426950408889634f, window, sink, part_o, part_ml};
   const dim3 grid(n_tiles, P);
   int rc = -3;
   if (rows_per_tile == 4) {
@@ -817,20 +972,23 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
 #undef LA_ANY
     rc = CFC_CHECK_LAUNCH();
   } else {
-    if (f32 || RS > 512) return -4;
-    const int mr = rows_per_tile / 16;
+    if (f32 || RV > 512 || RS > 576) return -4;
+    const int mr = rows_per_tile / 16, rv = (RV + 63) / 64;
+#define LAT(R, V) rc = lat_mr<R, V>(mr, grid, stream, q, cache, a, out); break
     switch ((RS + 63) / 64) {
-      case 1: rc = lat_mr<64>(mr, grid, stream, q, cache, a, out); break;
-      case 2: rc = lat_mr<128>(mr, grid, stream, q, cache, a, out); break;
-      case 3: rc = lat_mr<192>(mr, grid, stream, q, cache, a, out); break;
-      case 4: rc = lat_mr<256>(mr, grid, stream, q, cache, a, out); break;
-      case 5: case 6: rc = lat_mr<384>(mr, grid, stream, q, cache, a, out); break;
-      default: rc = lat_mr<512>(mr, grid, stream, q, cache, a, out); break;
+      case 1: LAT(64, 64);
+      case 2: if (rv == 1) { LAT(128, 64); } else { LAT(128, 128); }
+      case 3: if (rv <= 2) { LAT(192, 128); } else { LAT(192, 192); }
+      case 4: if (rv <= 2) { LAT(256, 128); } else { LAT(256, 256); }
+      case 5: case 6: if (rv <= 4) { LAT(384, 256); } else { LAT(384, 384); }
+      case 7: case 8: if (rv <= 6) { LAT(512, 384); } else { LAT(512, 512); }
+      default: LAT(576, 512);
     }
+#undef LAT
   }
   if (rc || P == 1) return rc;
-  if (f32) latent_combine_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RS, (float*)out);
-  else latent_combine_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RS, (uint16_t*)out);
+  if (f32) latent_combine_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, sink, H, (float*)out);
+  else latent_combine_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, sink, H, (uint16_t*)out);
   return CFC_CHECK_LAUNCH();
 }
 

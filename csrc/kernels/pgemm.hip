@@ -437,11 +437,15 @@ __device__ __forceinline__ void pp_wait_barrier() {
 
 // PF: probe flags (scripts/bench_pgemm.py --probe; 0 in production): 1 = no s_setprio, 2 = static
 // priority 1 for group 1 instead of per-segment flips.  gm = M-tiles per N sweep of the tile order.
-template <int EPI, bool PACKED, int PF = 0>
+// GRP: one packed matrix per expert, W[experts][N][K]: M-tile y multiplies its rows by matrix tile_expert[y]
+// (negative: no such tile), row m being row rows[m] of X (rows null: m itself).
+struct PgGroup { const int32_t* rows = nullptr; const int32_t* tile_expert = nullptr; };
+
+template <int EPI, bool PACKED, int PF = 0, bool GRP = false>
 __global__ void __launch_bounds__(512, 1)
     pgemm_pp_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, const uint16_t* __restrict__ bias,
                     uint16_t* __restrict__ out, int M, int N, int K, int ldo, int tiles_m, int tiles_n, int wnw,
-                    int gm = PG_GROUP_M) {
+                    int gm = PG_GROUP_M, PgGlu gp = PgGlu{}, PgGroup pgrp = PgGroup{}) {
   __shared__ __attribute__((aligned(16))) char smem[2 * PP_BUF];
   const int lane = threadIdx.x & 63;
   const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -455,6 +459,11 @@ __global__ void __launch_bounds__(512, 1)
   const int in_group = id % per_group;
   const int m0 = (first_m + in_group % gsz) * PG_BM;
   const int n0 = (in_group / gsz) * PG_BN;
+  if constexpr (GRP) {
+    const int e = __builtin_amdgcn_readfirstlane(pgrp.tile_expert[m0 / PG_BM]);
+    if (e < 0) return;
+    W += (size_t)e * N * K;
+  }
   const int nk = K / PG_BK;
 
   // ---- DMA sources.  X: pieces w and w + 8 of half h = image rows 8 p .. 8 p + 7 (lane: row
@@ -467,7 +476,10 @@ __global__ void __launch_bounds__(512, 1)
       const int r = 8 * (w + 8 * i) + (lane >> 3);
       const int trow = (r >> 6) * 128 + 64 * h + (r & 63);
       const int c = (lane & 7) ^ (r & 7);
-      vx[h][i] = ((uint32_t)min(m0 + trow, M - 1) * (uint32_t)K + 8u * c) * 2u;
+      int xr = min(m0 + trow, M - 1);
+      if constexpr (GRP)
+        if (pgrp.rows) xr = pgrp.rows[xr];
+      vx[h][i] = ((uint32_t)xr * (uint32_t)K + 8u * c) * 2u;
     }
   // W half h, pieces w and w + 8.  Packed: piece f = fragment (n-tile f >> 1 of the half, k group
   // f & 1 of the K-tile); its 1 KB sits at ((g / wnw) * K/32 + kg) * wnw + g % wnw fragments
@@ -663,7 +675,7 @@ __global__ void __launch_bounds__(512, 1)
   if constexpr (STG)
     pg_epilogue_staged<EPI>(acc, out, M, N, ldo, m0 + grp * 128, n0 + wc * 64, smem + w * 16384);
   else
-    pg_epilogue<EPI>(acc, bias, out, M, N, ldo, m0 + grp * 128, n0 + wc * 64);
+    pg_epilogue<EPI>(acc, bias, out, M, N, ldo, m0 + grp * 128, n0 + wc * 64, gp);
   if (grp == 0) pp_barrier();   // matches group 1's stagger barrier
 }
 
@@ -1379,6 +1391,31 @@ CFC_API int cfc_pgemm_glu(const void* x, const void* w, void* out, int M, int N,
   gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
   pgemm_ppp_kernel<PG_GLU, true><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(
       (const uint16_t*)x, (const uint16_t*)w, (uint16_t*)out, M, N, K, ldo, tm, tn, wnw, ppp_group_m(tn, K), gp);
+  return (int)hipGetLastError();
+}
+
+// Products of rows sorted by expert with W[experts][N][K] (each packed for bn = 16 wnw): M sorted rows in tiles of
+// 256, rows / tile_expert as in PgGroup (rows of an x_rows-row X).  glu 0: fp32 out [M][N]; 1: the clamped GLU of
+// 8-row interleaved gate / up rows, bf16 [M][N / 2] (row stride ldo)
+CFC_API int cfc_pgemm_group(int glu, const void* x, int x_rows, const void* w, int M, int N, int K, int wnw, const int32_t* rows,
+                            const int32_t* tile_expert, void* out, int ldo, float limit, float alpha, float beta,
+                            hipStream_t stream) {
+  if (M == 0) return 0;
+  if (M < 1 || M % PG_BM || N < 64 || K < 64 || K % 64 || N % 64 || ldo % 4 || ldo < (glu ? N / 2 : N) || wnw < 1 ||
+      N % (16 * wnw) || !tile_expert || x_rows < 1 || (!rows && x_rows < M) || (uint64_t)x_rows * K * 2 >= (1ull << 32) ||
+      (uint64_t)N * K * 2 >= (1ull << 32))
+    return (int)hipErrorInvalidValue;
+  const int tm = M / PG_BM, tn = (N + PG_BN - 1) / PG_BN;
+  PgGlu gp;
+  gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
+  PgGroup g;
+  g.rows = rows; g.tile_expert = tile_expert;
+  const uint16_t *xp = (const uint16_t*)x, *wp = (const uint16_t*)w;
+  uint16_t* op = (uint16_t*)out;
+  if (glu)
+    pgemm_pp_kernel<PG_GLU, true, PP_PF, true><<<tm * tn, 512, 0, stream>>>(xp, wp, nullptr, op, M, N, K, ldo, tm, tn, wnw, PG_GROUP_M, gp, g);
+  else
+    pgemm_pp_kernel<PG_F32, true, PP_PF, true><<<tm * tn, 512, 0, stream>>>(xp, wp, nullptr, op, M, N, K, ldo, tm, tn, wnw, PG_GROUP_M, gp, g);
   return (int)hipGetLastError();
 }
 

@@ -1,0 +1,571 @@
+// Linear recurrence with a per-channel, data-dependent decay (the RWKV kind of time mixing), per head:
+//   o_t = (S + diag(u) k_t v_t^T)^T r_t,   S <- diag(w_t) S + k_t v_t^T,   w_t = exp(-exp(z_t))
+// with z_t = W2 tanh(low-rank projection) + w0; then o over its root mean square, times norm, times silu(gate).
+// S [slots][H][D][D] fp32 (key channel, value channel); a sequence at position 0 starts from zeros.
+//
+// Prompt portions run in chunks of 16 tokens.  With L_t the running sum of log w inside a chunk, token i's
+// output is  (r_i exp(L_(i-1)))^T S_chunk  +  sum_(j<i) [sum_c r_i k_j exp(L_(i-1) - L_j)] v_j  +  the bonus
+// term, and the chunk's state step is  S <- exp(L_15) S + sum_j (k_j exp(L_15 - L_j)) v_j^T.  Every exponent
+// is <= 0, whatever the decays, so nothing over- or underflows that the plain recurrence would keep.
+//   * wkv_tanh   the low-rank activations as three bf16 parts (24 bits: W2's product on the bf16 matrix
+//                cores is exact to fp32)
+//   * wkv_prep   one wave per (chunk, head), all chunks in parallel: decays, the scaled r and k and the 16 x 16
+//                coefficients, written in the fragment order of the scan's fp32 MFMAs
+//   * wkv_scan   one workgroup per (sequence, head), a wave per 16 value channels: the state stays in the
+//                accumulators over all chunks and is the B operand of the next one as it lies
+//   * wkv_step   token by token: decoded tokens (one pass over the state: read, output, update), and prompt
+//                portions of head sizes the chunked kernels are not built for
+#include "common.h"
+
+namespace {
+
+__device__ __forceinline__ float ld1(const uint16_t* p) { return bf2f(*p); }
+__device__ __forceinline__ float ld1(const float* p) { return *p; }
+__device__ __forceinline__ void st1(uint16_t* p, float v) { *p = f2bf(v); }
+__device__ __forceinline__ void st1(float* p, float v) { *p = v; }
+
+constexpr float LOG_DECAY_MIN = -104.f;      // exp(-104) is 0 in fp32
+constexpr int CT = 16;                       // tokens per chunk
+
+__device__ __forceinline__ float log_decay(float z) { return fmaxf(-expf(z), LOG_DECAY_MIN); }
+
+// columns of a product: activations (split 0) or fp32 slabs
+struct Cols {
+  const void* p;
+  int split;                // 0: activations
+  int64_t ld, plane;
+};
+
+template <typename ACT>
+__device__ __forceinline__ float ldc(const Cols& a, int64_t t, int c) {
+  const int64_t o = t * a.ld + c;
+  if (a.split == 0) return ld1(reinterpret_cast<const ACT*>(a.p) + o);
+  const float* p = reinterpret_cast<const float*>(a.p) + o;
+  float s = 0.f;
+  for (int i0 = 0; i0 < a.split; i0 += 8) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v[u] = p[(int64_t)min(i0 + u, a.split - 1) * a.plane];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) s += i0 + u < a.split ? v[u] : 0.f;
+  }
+  return s;
+}
+
+// out [T][3][RP]: high, middle and low bf16 parts of tanh(w1); columns past R zero
+template <typename ACT>
+__global__ void __launch_bounds__(256) wkv_tanh_kernel(Cols w1, int T, int R, int RP, uint16_t* __restrict__ out) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (int64_t)T * RP) return;
+  const int64_t t = i / RP;
+  const int c = (int)(i % RP);
+  const float v = c < R ? tanhf(ldc<ACT>(w1, t, c)) : 0.f;
+  const uint16_t hi = f2bf(v);
+  const float r1 = v - bf2f(hi);
+  const uint16_t mid = f2bf(r1);
+  uint16_t* o = out + t * 3 * RP + c;
+  o[0] = hi;
+  o[RP] = mid;
+  o[2 * RP] = f2bf(r1 - bf2f(mid));
+}
+
+// ---------------------------------------------------------------------------------- chunked prompt portions
+// per (chunk, head): [ND][64][4] scaled r, [ND][64][4] scaled k, [64][4] coefficients, [16 ND] decays
+template <int ND>
+struct ChunkRec {
+  static constexpr int R = 0, K = ND * 256, A = 2 * ND * 256, DEC = A + 256, SIZE = DEC + 16 * ND;
+};
+
+template <typename ACT, int ND, int WV>
+__global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const uint16_t* __restrict__ th, int RP,
+                                                          const uint16_t* __restrict__ w2, const float* __restrict__ w0,
+                                                          const float* __restrict__ u, const int32_t* __restrict__ chunks,
+                                                          int H, int D, float* __restrict__ rec) {
+  constexpr int DP = 16 * ND, LD = DP + 4;
+  using Rec = ChunkRec<ND>;
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, col = lane & 15, q = lane >> 4;
+  const int h = blockIdx.y * WV + wv;
+  if (h >= H) return;                             // waves share nothing below
+  float* L = smem + wv * (49 * LD);               // [17][LD]: L[t] = sum of log w before token t
+  float* rs = L + 17 * LD;                        // [16][LD]
+  float* ks = rs + 16 * LD;                       // [16][LD], then the coefficients [16][17] in its place
+  const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
+  const int hc = h * D;
+  // r and k, channel per lane
+#pragma unroll
+  for (int c0 = 0; c0 < DP; c0 += 64) {
+    const int c = c0 + lane;
+    if (c < DP) {
+      const bool live = c < D;
+      float a[CT], b[CT];
+#pragma unroll
+      for (int t = 0; t < CT; ++t) {
+        const int tt = row0 + min(t, n - 1), cc = hc + (live ? c : 0);
+        a[t] = ld1(reinterpret_cast<const ACT*>(r.p) + tt * r.ld + cc);
+        b[t] = ld1(reinterpret_cast<const ACT*>(k.p) + tt * k.ld + cc);
+      }
+#pragma unroll
+      for (int t = 0; t < CT; ++t) {
+        rs[t * LD + c] = live && t < n ? a[t] : 0.f;
+        ks[t * LD + c] = live && t < n ? b[t] : 0.f;
+      }
+    }
+  }
+  // z^T = W2 tanh^T: lane holds channels 16 T + 4 q + i of token col
+  f32x4_t z[ND];
+#pragma unroll
+  for (int T = 0; T < ND; ++T) z[T] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const uint16_t* tr = th + (size_t)(row0 + min(col, n - 1)) * 3 * RP + 8 * q;
+  for (int kk = 0; kk < RP; kk += 32) {
+    bf16x8_t b[3];
+#pragma unroll
+    for (int p = 0; p < 3; ++p) b[p] = *reinterpret_cast<const bf16x8_t*>(tr + p * RP + kk);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) {
+      const int ch = min(16 * T + col, D - 1);
+      const bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(w2 + (size_t)(hc + ch) * RP + kk + 8 * q);
+#pragma unroll
+      for (int p = 0; p < 3; ++p) z[T] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b[p], z[T], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int T = 0; T < ND; ++T) {
+    float v[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = 16 * T + 4 * q + i;
+      v[i] = c < D && col < n ? log_decay(z[T][i] + w0[hc + min(c, D - 1)]) : 0.f;
+    }
+    *reinterpret_cast<float4*>(L + (col + 1) * LD + 16 * T + 4 * q) = make_float4(v[0], v[1], v[2], v[3]);
+  }
+  auto sync = [] {                                // the wave's own LDS writes are visible to its lanes
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  };
+  sync();
+  float* out = rec + ((size_t)blockIdx.x * H + h) * Rec::SIZE;
+#pragma unroll
+  for (int c0 = 0; c0 < DP; c0 += 64) {
+    const int c = c0 + lane;
+    if (c < DP) {
+      float s = 0.f;
+      L[c] = 0.f;
+#pragma unroll
+      for (int t = 1; t <= CT; ++t) {
+        s += L[t * LD + c];
+        L[t * LD + c] = s;
+      }
+      out[Rec::DEC + c] = __expf(s);
+    }
+  }
+  sync();
+  // scaled r (row col, channels 16 T + 4 q ..) and scaled k (tokens 4 q + s, channel 16 T + col)
+#pragma unroll
+  for (int T = 0; T < ND; ++T) {
+    const int c = 16 * T + 4 * q;
+    const float4 rv = *reinterpret_cast<const float4*>(rs + col * LD + c), lv = *reinterpret_cast<const float4*>(L + col * LD + c);
+    reinterpret_cast<float4*>(out + Rec::R)[T * 64 + lane] =
+        make_float4(rv.x * __expf(lv.x), rv.y * __expf(lv.y), rv.z * __expf(lv.z), rv.w * __expf(lv.w));
+    float kv[4];
+    const float le = L[16 * LD + 16 * T + col];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) kv[s] = ks[(4 * q + s) * LD + 16 * T + col] * __expf(le - L[(4 * q + s + 1) * LD + 16 * T + col]);
+    reinterpret_cast<float4*>(out + Rec::K)[T * 64 + lane] = make_float4(kv[0], kv[1], kv[2], kv[3]);
+  }
+  // coefficients below the diagonal: two of the 120 pairs (i, j < i) per lane
+  int pi[2], pj[2];
+#pragma unroll
+  for (int e = 0; e < 2; ++e) {
+    const int p = min(lane + 64 * e, 119);
+    int i = (int)((1.f + sqrtf(1.f + 8.f * p)) * 0.5f);
+    if (i * (i - 1) / 2 > p) --i;
+    if ((i + 1) * i / 2 <= p) ++i;
+    pi[e] = i;
+    pj[e] = p - i * (i - 1) / 2;
+  }
+  float acc[2] = {0.f, 0.f};
+  for (int c = 0; c < DP; c += 4)
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+      const float4 a = *reinterpret_cast<const float4*>(L + pi[e] * LD + c), b = *reinterpret_cast<const float4*>(L + (pj[e] + 1) * LD + c);
+      const float4 x = *reinterpret_cast<const float4*>(rs + pi[e] * LD + c), y = *reinterpret_cast<const float4*>(ks + pj[e] * LD + c);
+      acc[e] += x.x * y.x * __expf(a.x - b.x) + x.y * y.y * __expf(a.y - b.y) + x.z * y.z * __expf(a.z - b.z) +
+                x.w * y.w * __expf(a.w - b.w);
+    }
+  // the diagonal: row lane / 4, a quarter of the channels
+  float dg = 0.f;
+  {
+    const int i = lane >> 2;
+    for (int c = (lane & 3) * 4; c < DP; c += 16)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float uu = c + e < D ? u[hc + c + e] : 0.f;
+        dg += uu * rs[i * LD + c + e] * ks[i * LD + c + e];
+      }
+    dg += __shfl_xor(dg, 1, 64);
+    dg += __shfl_xor(dg, 2, 64);
+  }
+  sync();
+  float* am = ks;                                 // every read of k is done
+#pragma unroll
+  for (int e = 0; e < 4; ++e) am[(lane >> 2) * 17 + 4 * (lane & 3) + e] = 0.f;
+  sync();
+#pragma unroll
+  for (int e = 0; e < 2; ++e)
+    if (lane + 64 * e < 120) am[pi[e] * 17 + pj[e]] = acc[e];
+  if ((lane & 3) == 0) am[(lane >> 2) * 17 + (lane >> 2)] = dg;
+  sync();
+  float av[4];
+#pragma unroll
+  for (int s = 0; s < 4; ++s) av[s] = am[col * 17 + 4 * q + s];
+  reinterpret_cast<float4*>(out + Rec::A)[lane] = make_float4(av[0], av[1], av[2], av[3]);
+}
+
+struct ScanSeq {
+  const int32_t* chunk_cu;    // [sequences + 1]
+  const int32_t* chunks;      // [chunks][2]: first row, rows
+  const int32_t* slots;       // [sequences]
+  const int32_t* cu_q;
+  const int32_t* ctx_lens;
+};
+
+__device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+template <typename ACT, int ND>
+__global__ void __launch_bounds__(64 * ND) wkv_scan_kernel(const float* __restrict__ rec, Cols v, Cols g, ScanSeq sq, int H,
+                                                          int D, const float* __restrict__ norm, float eps,
+                                                          float* __restrict__ state, ACT* __restrict__ out, int64_t ldo) {
+  using Rec = ChunkRec<ND>;
+  __shared__ float red[2][ND][16];
+  const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), col = lane & 15, q = lane >> 4;
+  const int h = blockIdx.x, s = blockIdx.y;
+  const int c0 = sq.chunk_cu[s], c1 = sq.chunk_cu[s + 1];
+  const bool fresh = sq.ctx_lens[s] == sq.cu_q[s + 1] - sq.cu_q[s];
+  const int vc = 16 * w + col;                    // value channel of this lane
+  const bool live = vc < D;
+  const int hv = h * D + min(vc, D - 1);
+  float* st = state + (((size_t)sq.slots[s] * H + h) * D) * D + min(vc, D - 1);
+  f32x4_t S[ND];
+#pragma unroll
+  for (int T = 0; T < ND; ++T)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int kc = 16 * T + 4 * q + i;
+      S[T][i] = !fresh && live && kc < D ? st[(size_t)min(kc, D - 1) * D] : 0.f;
+    }
+  const float nw = norm[hv];
+  struct Frag {
+    float4 r[ND], k[ND], dec[ND], a;
+    float v[4], g[4];
+    int row0, n;
+  };
+  auto load = [&](int c, Frag& f) {
+    const float4* p = reinterpret_cast<const float4*>(rec + ((size_t)c * H + h) * Rec::SIZE);
+    f.row0 = sq.chunks[2 * c];
+    f.n = sq.chunks[2 * c + 1];
+#pragma unroll
+    for (int T = 0; T < ND; ++T) {
+      f.r[T] = p[T * 64 + lane];
+      f.k[T] = p[Rec::K / 4 + T * 64 + lane];
+      f.dec[T] = p[Rec::DEC / 4 + 4 * T + q];
+    }
+    f.a = p[Rec::A / 4 + lane];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int64_t t = f.row0 + min(4 * q + i, f.n - 1);
+      f.v[i] = ld1(reinterpret_cast<const ACT*>(v.p) + t * v.ld + hv);
+      f.g[i] = ld1(reinterpret_cast<const ACT*>(g.p) + t * g.ld + hv);
+    }
+  };
+  Frag f[2];
+  if (c0 < c1) load(c0, f[0]);
+  auto chunk = [&](int c, Frag& cur, Frag& nxt, int par) {
+    load(min(c + 1, c1 - 1), nxt);
+    f32x4_t o0{0.f, 0.f, 0.f, 0.f}, o1{0.f, 0.f, 0.f, 0.f};
+    float vv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) vv[i] = live && 4 * q + i < cur.n ? cur.v[i] : 0.f;
+#pragma unroll
+    for (int T = 0; T < ND; ++T) {
+      o0 = mfma4(cur.r[T].x, S[T][0], o0);
+      o1 = mfma4(cur.r[T].y, S[T][1], o1);
+      o0 = mfma4(cur.r[T].z, S[T][2], o0);
+      o1 = mfma4(cur.r[T].w, S[T][3], o1);
+    }
+    o0 = mfma4(cur.a.x, vv[0], o0);
+    o1 = mfma4(cur.a.y, vv[1], o1);
+    o0 = mfma4(cur.a.z, vv[2], o0);
+    o1 = mfma4(cur.a.w, vv[3], o1);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) {
+      S[T][0] *= cur.dec[T].x; S[T][1] *= cur.dec[T].y; S[T][2] *= cur.dec[T].z; S[T][3] *= cur.dec[T].w;
+    }
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].x, vv[0], S[T]);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].y, vv[1], S[T]);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].z, vv[2], S[T]);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].w, vv[3], S[T]);
+    // rms over the head: the wave's 16 channels, then the waves
+    const f32x4_t o = o0 + o1;
+    float ss[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      ss[i] = live ? o[i] * o[i] : 0.f;
+#pragma unroll
+      for (int m = 8; m > 0; m >>= 1) ss[i] += __shfl_xor(ss[i], m, 64);
+    }
+    if (col == 0) *reinterpret_cast<float4*>(&red[par][w][4 * q]) = make_float4(ss[0], ss[1], ss[2], ss[3]);
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+    __builtin_amdgcn_s_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+    float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int j = 0; j < ND; ++j) {
+      const float4 a = *reinterpret_cast<const float4*>(&red[par][j][4 * q]);
+      sum.x += a.x; sum.y += a.y; sum.z += a.z; sum.w += a.w;
+    }
+    const float sv[4] = {sum.x, sum.y, sum.z, sum.w};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float gg = cur.g[i];
+      const float y = o[i] * (1.f / sqrtf(sv[i] / (float)D + eps)) * nw * (gg / (1.f + __expf(-gg)));
+      if (live && 4 * q + i < cur.n) st1(out + (int64_t)(cur.row0 + 4 * q + i) * ldo + hv, y);
+    }
+  };
+  int c = c0;
+  for (; c + 2 <= c1; c += 2) {
+    chunk(c, f[0], f[1], 0);
+    chunk(c + 1, f[1], f[0], 1);
+  }
+  if (c < c1) chunk(c, f[0], f[1], 0);
+  if (live && c0 < c1) {
+#pragma unroll
+    for (int T = 0; T < ND; ++T)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int kc = 16 * T + 4 * q + i;
+        if (kc < D) st[(size_t)kc * D] = S[T][i];
+      }
+  }
+}
+
+// ---------------------------------------------------------------------------------- token by token
+// one workgroup per (head, sequence); a thread owns V value channels of every NG-th key channel, so the
+// state needs no synchronisation between tokens
+constexpr int WS_T = 256, WS_NR = 4;
+template <typename ACT, int V>
+__global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, Cols g, Cols w1, int R, int RP,
+                                                       const uint16_t* __restrict__ w2, const float* __restrict__ w0,
+                                                       const float* __restrict__ u, const float* __restrict__ norm, float eps,
+                                                       int H, int D, const int32_t* __restrict__ slots,
+                                                       const int32_t* __restrict__ cu_q, const int32_t* __restrict__ ctx_lens,
+                                                       float* __restrict__ state, ACT* __restrict__ out, int64_t ldo) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  __shared__ float red[16];
+  const int nvec = (D + V - 1) / V, ng = WS_T / nvec;
+  float* rs = sm;              // [D] each
+  float* kk = rs + D;
+  float* vs = kk + D;
+  float* gs = vs + D;
+  float* ws = gs + D;
+  float* th = ws + D;          // [RP]
+  float* part = th + RP;       // [ng][D]
+  const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x;
+  const int q0 = cu_q ? cu_q[s] : s, n = cu_q ? cu_q[s + 1] - q0 : 1;
+  const bool fresh = ctx_lens[s] == n;
+  float* st = state + ((size_t)slots[s] * H + h) * D * D;
+  const int vx = tid % nvec, gy = tid / nvec, hc = h * D;
+  const bool own = gy < ng;
+  for (int t = 0; t < n; ++t) {
+    const bool zero = fresh && t == 0;
+    float S[WS_NR][V];
+    auto ldS = [&](int i0) {
+#pragma unroll
+      for (int a = 0; a < WS_NR; ++a) {
+        const int i = i0 + gy + a * ng;
+#pragma unroll
+        for (int e = 0; e < V; ++e) S[a][e] = 0.f;
+        if (own && i < D && !zero) {
+          if constexpr (V == 4) {
+            const float4 f = *reinterpret_cast<const float4*>(st + (size_t)i * D + 4 * vx);
+            S[a][0] = f.x; S[a][1] = f.y; S[a][2] = f.z; S[a][3] = f.w;
+          } else {
+            S[a][0] = st[(size_t)i * D + vx];
+          }
+        }
+      }
+    };
+    ldS(0);
+    const int64_t row = q0 + t;
+    for (int e = tid; e < 4 * D; e += WS_T) {
+      const int c = e % D;
+      const int w = e / D;
+      const Cols& src = w == 0 ? r : w == 1 ? k : w == 2 ? v : g;
+      rs[e] = ldc<ACT>(src, row, hc + c);
+    }
+    for (int c = tid; c < RP; c += WS_T) th[c] = c < R ? tanhf(ldc<ACT>(w1, row, c)) : 0.f;
+    __syncthreads();
+    // four threads per channel over the low rank
+    for (int c0 = 0; c0 < D; c0 += WS_T / 4) {
+      const int c = c0 + (tid >> 2), p = tid & 3;
+      float z = 0.f;
+      if (c < D)
+        for (int x = 8 * p; x < RP; x += 32) {
+          float wv[8];
+          unpack8(*reinterpret_cast<const uint4*>(w2 + (size_t)(hc + c) * RP + x), wv);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) z += wv[e] * th[x + e];
+        }
+      z += __shfl_xor(z, 1, 64);
+      z += __shfl_xor(z, 2, 64);
+      if (c < D && p == 0) ws[c] = expf(log_decay(z + w0[hc + c]));
+    }
+    float bonus = 0.f;
+    for (int c = tid; c < D; c += WS_T) bonus += u[hc + c] * rs[c] * kk[c];
+    bonus = block_sum(bonus, red);               // its barriers also publish ws
+    float o[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) o[e] = 0.f;
+    float vv[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) vv[e] = own ? vs[min(V * vx + e, D - 1)] : 0.f;
+    for (int i0 = 0; i0 < D; i0 += WS_NR * ng) {
+      if (i0) ldS(i0);
+#pragma unroll
+      for (int a = 0; a < WS_NR; ++a) {
+        const int i = i0 + gy + a * ng;
+        if (!own || i >= D) continue;
+        const float ri = rs[i], ki = kk[i], wi = ws[i];
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          o[e] += ri * S[a][e];
+          S[a][e] = wi * S[a][e] + ki * vv[e];
+        }
+        if constexpr (V == 4) *reinterpret_cast<float4*>(st + (size_t)i * D + 4 * vx) = make_float4(S[a][0], S[a][1], S[a][2], S[a][3]);
+        else st[(size_t)i * D + vx] = S[a][0];
+      }
+    }
+    if (own)
+#pragma unroll
+      for (int e = 0; e < V; ++e)
+        if (V * vx + e < D) part[gy * D + V * vx + e] = o[e];
+    __syncthreads();
+    float y[2], ss = 0.f;                        // D <= 2 WS_T
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const int c = tid + m * WS_T;
+      y[m] = 0.f;
+      if (c < D) {
+        for (int a = 0; a < ng; ++a) y[m] += part[a * D + c];
+        y[m] += bonus * vs[c];
+        ss += y[m] * y[m];
+      }
+    }
+    const float rr = 1.f / sqrtf(block_sum(ss, red) / (float)D + eps);
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const int c = tid + m * WS_T;
+      if (c < D) {
+        const float gg = gs[c];
+        st1(out + row * ldo + hc + c, y[m] * rr * norm[hc + c] * (gg / (1.f + expf(-gg))));
+      }
+    }
+    __syncthreads();                             // the next token overwrites what this one read
+  }
+}
+
+template <typename ACT, int ND>
+int chunked_go(hipStream_t s, const Cols& r, const Cols& k, const Cols& v, const Cols& g, const uint16_t* th, int RP,
+               const uint16_t* w2, const float* w0, const float* u, const float* norm, float eps, int H, int D, int n_chunks,
+               int n_seq, const ScanSeq& sq, float* rec, float* state, void* out, int64_t ldo) {
+  constexpr int WV = ND <= 4 ? 4 : 2;
+  constexpr int lds = WV * 49 * (16 * ND + 4) * 4;
+  wkv_prep_kernel<ACT, ND, WV><<<dim3(n_chunks, (H + WV - 1) / WV), 64 * WV, lds, s>>>(r, k, th, RP, w2, w0, u, sq.chunks, H, D, rec);
+  if (const int e = (int)hipGetLastError()) return e;
+  wkv_scan_kernel<ACT, ND><<<dim3(H, n_seq), 64 * ND, 0, s>>>(rec, v, g, sq, H, D, norm, eps, state, (ACT*)out, ldo);
+  return CFC_CHECK_LAUNCH();
+}
+
+}  // namespace
+
+constexpr int WKV_MAX_CHUNKED = 128;
+
+// floats of scratch per (chunk, head); 0: no chunked kernel for this head size
+CFC_API int cfc_wkv_chunk_floats(int D) {
+  if (D < 1 || D > WKV_MAX_CHUNKED) return 0;
+  const int nd = D <= 64 ? (D + 15) / 16 : D <= 96 ? 6 : 8;
+  return 2 * nd * 256 + 256 + 16 * nd;
+}
+
+// out [T][3][RP] bf16 parts of tanh(w1) (split 0: w1 are activations)
+CFC_API int cfc_wkv_tanh(int f32, const void* w1, int split, int64_t ld, int64_t plane, int T, int R, int RP, void* out,
+                         hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (R < 1 || RP < R || RP % 32 || split < 0) return -1;
+  const Cols c{w1, split, ld, plane};
+  const int64_t n = ((int64_t)T * RP + 255) / 256;
+  if (f32) wkv_tanh_kernel<float><<<(unsigned)n, 256, 0, stream>>>(c, T, R, RP, (uint16_t*)out);
+  else wkv_tanh_kernel<uint16_t><<<(unsigned)n, 256, 0, stream>>>(c, T, R, RP, (uint16_t*)out);
+  return CFC_CHECK_LAUNCH();
+}
+
+// r, k, v, g: activations with row strides; th from cfc_wkv_tanh; chunks [n][2] = {first row, rows <= 16} in
+// sequence order, chunk_cu [sequences + 1]; rec: cfc_wkv_chunk_floats(D) floats per (chunk, head)
+CFC_API int cfc_wkv_chunked(int f32, const void* r, int64_t ldr, const void* k, int64_t ldk, const void* v, int64_t ldv,
+                            const void* g, int64_t ldg, const void* th, int RP, const void* w2, const float* w0,
+                            const float* u, const float* norm, float eps, int H, int D, int n_chunks, int n_seq,
+                            const int32_t* chunk_cu, const int32_t* chunks, const int32_t* slots, const int32_t* cu_q,
+                            const int32_t* ctx_lens, float* rec, float* state, void* out, int64_t ldo, hipStream_t stream) {
+  if (n_seq <= 0 || n_chunks <= 0) return 0;
+  if (H < 1 || D < 1 || D > WKV_MAX_CHUNKED || RP < 32 || RP % 32 || n_seq > 65535) return -1;
+  const Cols cr{r, 0, ldr, 0}, ck{k, 0, ldk, 0}, cv{v, 0, ldv, 0}, cg{g, 0, ldg, 0};
+  const ScanSeq sq{chunk_cu, chunks, slots, cu_q, ctx_lens};
+#define WC(ACT, ND)                                                                                                      \
+  return chunked_go<ACT, ND>(stream, cr, ck, cv, cg, (const uint16_t*)th, RP, (const uint16_t*)w2, w0, u, norm, eps, H, \
+                             D, n_chunks, n_seq, sq, rec, state, out, ldo)
+#define WN(ACT)                                      \
+  switch (D <= 64 ? (D + 15) / 16 : D <= 96 ? 6 : 8) { \
+    case 1: WC(ACT, 1);                              \
+    case 2: WC(ACT, 2);                              \
+    case 3: WC(ACT, 3);                              \
+    case 4: WC(ACT, 4);                              \
+    case 6: WC(ACT, 6);                              \
+    default: WC(ACT, 8);                             \
+  }
+  if (f32) WN(float)
+  WN(uint16_t)
+#undef WN
+#undef WC
+}
+
+// one token per sequence (cu_q null) or portions, token by token.  Each operand: pointer, split (0:
+// activations, else fp32 slabs), row stride, slab stride
+CFC_API int cfc_wkv_step(int f32, const void* r, const void* k, const void* v, const void* g, int split, int64_t ld,
+                         int64_t plane, const void* w1, int split1, int64_t ld1, int64_t plane1, int R, int RP,
+                         const void* w2, const float* w0, const float* u, const float* norm, float eps, int H, int D, int n_seq,
+                         const int32_t* slots, const int32_t* cu_q, const int32_t* ctx_lens, float* state, void* out,
+                         int64_t ldo, hipStream_t stream) {
+  if (n_seq <= 0) return 0;
+  if (H < 1 || D < 1 || D > 2 * WS_T || R < 1 || RP < R || RP % 32 || RP > 2048 || split < 0 || split1 < 0 || n_seq > 65535) return -1;
+  const int V = D % 4 == 0 ? 4 : 1;
+  if ((D + V - 1) / V > WS_T) return -1;
+  const int ng = WS_T / ((D + V - 1) / V);
+  const size_t lds = (size_t)(5 * D + RP + ng * D) * 4;
+  const Cols cr{r, split, ld, plane}, ck{k, split, ld, plane}, cv{v, split, ld, plane}, cg{g, split, ld, plane},
+      c1{w1, split1, ld1, plane1};
+#define ST(ACT, VV)                                                                                                      \
+  wkv_step_kernel<ACT, VV><<<dim3(H, n_seq), WS_T, lds, stream>>>(cr, ck, cv, cg, c1, R, RP, (const uint16_t*)w2, w0, u, \
+                                                                 norm, eps, H, D, slots, cu_q, ctx_lens, state, (ACT*)out, ldo)
+  if (f32) { if (V == 4) ST(float, 4); else ST(float, 1); }
+  else if (V == 4) ST(uint16_t, 4);
+  else ST(uint16_t, 1);
+#undef ST
+  return CFC_CHECK_LAUNCH();
+}
