@@ -323,6 +323,11 @@ class ZisapelWeights:
                 uk = mat(rows(get(x + "uk"))).view(H, m.dim, m.kv_rank)
                 lw["uk"] = L.HeadWeight(uk.transpose(1, 2), n_out=L.padded_rank(m.kv_rank))
                 lw["uv"] = L.HeadWeight(mat(rows(get(x + "uv"))).view(H, m.vdim, m.kv_rank))
+                if (m.dim == m.vdim == L.EXPANDED_DIM and m.rot_dim <= L.ROT_COLS and m.rot_dim % 8 == 0
+                        and Projection.packs(uk, H * m.dim, m.kv_rank) and K.prefill_rows(H, H) == 256):
+                    # long portions: keys and values per head from two products (ops.latent.expand)
+                    lw["uk_full"] = K.pack_dgemm_weight(uk.reshape(H * m.dim, m.kv_rank).contiguous())
+                    lw["uv_full"] = mat(rows(get(x + "uv"))).contiguous()
                 lw["rope"] = L.yarn_rope(m.rot_dim, m.base, dict(m.scaling) if m.scaling else None, w.device)
             if f is not None:
                 lw["norm2"], lw["rg2_b"] = vec(get(p + "norm2")), vec(get(p + "rg2.b"))
@@ -354,7 +359,8 @@ class ZisapelWeights:
     def nbytes(self) -> int:
         n = self.embed.numel() * self.embed.element_size() + self.head.nbytes()
         for lw in self.layers:
-            n += sum(lw[k].nbytes() for k in ("o", "in", "uk", "uv", "rg2", "router_w", "experts") if k in lw)
+            n += sum(lw[k].nbytes() for k in ("o", "in", "uk", "uv", "uk_full", "rg2", "router_w", "experts") if k in lw)
+            n += lw["uv_full"].numel() * 2 if "uv_full" in lw else 0
             for k in ("glu", "shared"):
                 if lw.get(k):
                     n += lw[k]["gate_up"].nbytes() + lw[k]["down"].nbytes()
@@ -372,6 +378,8 @@ class ZisapelModel:
             src.add("wkv" if isinstance(s.mixer, WkvSpec) else "latent")
             if isinstance(s.mlp, MoeSpec):
                 src.add("moe")
+            if dtype == torch.bfloat16 and isinstance(s.mixer, WindowSpec) and s.mixer.dim == s.mixer.vdim == L.EXPANDED_DIM:
+                src.add("attention")
         if dtype == torch.bfloat16:
             src |= {"gemm", "dgemm", "pgemm"}
         return tuple(sorted(src))
@@ -437,7 +445,33 @@ class ZisapelModel:
             key = f"attn_{H}_{self._rows(i)}_{m.window}"
             if key not in plan:
                 plan[key] = np.asarray(L.attn_tiles(cu, H, self._rows(i), ctx, m.window), np.int32).reshape(2, -1)
+        for i, m, _, _, rv in self._windows():
+            key = f"expand_{rv}_{m.window}"
+            if "uk_full" in self.w.layers[i] and key not in plan:
+                plan[key] = self._expand_pays(cu, ctx, rv, m.window)
+                if plan[key] and f"gather_{m.window}" not in plan:
+                    starts = [self._first_key(c - (b - a), m.window) for a, b, c in zip(cu, cu[1:], ctx)]
+                    gt, base = L.gather_tiles(ctx, starts)
+                    plan[f"gather_{m.window}"], plan[f"base_{m.window}"] = np.asarray(gt, np.int32), np.asarray(base, np.int32)
+                    plan["pf_tiles"] = np.asarray(K.prefill_tiles(cu, 256, ctx), np.int32)
         return plan
+
+    @staticmethod
+    def _first_key(pos: int, window: int) -> int:
+        return max(0, pos - window + 1) if window else 0
+
+    @staticmethod
+    def _expand_pays(cu, ctx, rv, window) -> bool:
+        """Whether per-head keys and values of what the pass can see take less time than attention in the latent space
+        with its two per-head products: flops per head (halved) over the rates measured on one MI355X."""
+        d, latent, dense = 2 * L.EXPANDED_DIM, 0.0, 0.0
+        for a, b, c in zip(cu, cu[1:], ctx):
+            n, pos = b - a, c - (b - a)
+            full = max(0, min(n, c - window)) if window else 0          # rows that see a whole window
+            pairs = full * window + (n - full) * (pos + (n - full + 1) / 2)
+            latent += pairs * (2 * rv + L.ROT_COLS) / 0.22 + n * rv * d / 0.14
+            dense += pairs * (d + L.ROT_COLS) / 0.6 + (c - ZisapelModel._first_key(pos, window) + 32) * rv * d / 0.7
+        return dense < latent
 
     # ---------------------------------------------------------------- forward
     def forward_prefill(self, ids, positions, slots, cu_q, ctx_lens, block_tables, kv, last_idx=None, plan=None):
@@ -462,7 +496,7 @@ class ZisapelModel:
                 keys = self._visible(s.mixer, plan["max_ctx"])
                 o = self._attend(i, part.act(1, acts), part.slabs(2, acts), part.act(3, acts), positions, slots, ctx_lens,
                                  block_tables, kv, dict(cu_q=cu_q, tiles=(tiles[0], tiles[1]), rows=rows,
-                                                        P=L.partitions(tiles.shape[1], keys)))
+                                                        P=L.partitions(tiles.shape[1], keys)), plan)
             b = G.Branch(gate, lw["rg1_b"], lw["norm1"], self.cfg.norm_eps, y=self._sum(lw["o"].slabs(o)))
             G.gated_norm(x, b, dt, h if s.mlp is not None else None, kv.prev[i], plan["meta"], positions)
             if s.mlp is not None:
@@ -525,14 +559,24 @@ class ZisapelModel:
         torch.distributed.all_reduce(part, group=self.tp_group)
         return part
 
-    def _attend(self, i, q, kv_cols, g, positions, slots, ctx_lens, block_tables, kv, attn) -> torch.Tensor:
-        """Latent attention of layer i: the gated heads [T, H vdim]."""
+    def _attend(self, i, q, kv_cols, g, positions, slots, ctx_lens, block_tables, kv, attn, plan=None) -> torch.Tensor:
+        """Latent attention of layer i: the gated heads [T, H vdim].  ``plan``: the launch plan of a packed pass."""
         lw, m = self.w.layers[i], self.cfg.specs[i].mixer
         T, H, dt, dev = q.rows, lw["H"], self.w.dtype, positions.device
         rs, rv = self._cols(m)
+
+        def rope(qr):
+            return L.latent_rope(kv_cols, m.kv_rank, lw["dkv_norm"], self.cfg.norm_eps, slots, kv.rows[i], q, H, m.dim,
+                                 lw["rope"], positions, qr, m.vdim, g)
+        if plan is not None and plan.get(f"expand_{rv}_{m.window}") and "uk_full" in lw:
+            q2 = torch.empty(T, H, L.ROT_COLS, dtype=dt, device=dev)
+            _, gate = rope(q2)
+            k, vt, k2 = L.expand(kv.rows[i], block_tables, ctx_lens, plan[f"gather_{m.window}"], lw["uk_full"], lw["uv_full"], rv)
+            return L.expanded_window_attention(q, q2, k, k2, vt, plan[f"base_{m.window}"], attn["cu_q"], ctx_lens, m.scale,
+                                               plan["pf_tiles"], m.window, lw["sink"], gate,
+                                               torch.empty(T, H * m.vdim, dtype=dt, device=dev))
         ql = torch.empty(T, H, rs, dtype=dt, device=dev)
-        qn, gate = L.latent_rope(kv_cols, m.kv_rank, lw["dkv_norm"], self.cfg.norm_eps, slots, kv.rows[i], q, H, m.dim,
-                                 lw["rope"], positions, ql, m.vdim, g)
+        qn, gate = rope(ql[:, :, rv:])
         L.head_linear(qn, lw["uk"], ql)
         ol = L.latent_attention(ql, kv.rows[i], block_tables, ctx_lens=ctx_lens, scale=m.scale, window=m.window,
                                 sink=lw["sink"], RV=rv, **attn)
@@ -562,7 +606,7 @@ class ZisapelModel:
         if self.w.tp_size == 1:
             b.y, b.routed = shared, (rows, pos, wt)
         else:
-            y = (rows[pos.long()] * wt[..., None]).sum(1)[None]
+            y = (rows[pos.long()].float() * wt[..., None]).sum(1)[None]
             b.y = self._sum(torch.cat([y, shared]) if shared is not None else y)
         return b
 

@@ -60,8 +60,8 @@ _KERNEL_SIGS = {
     "cfc_clamped_glu": [I, I, P, I, P, I, P, P, I, I, I, F, F, F, P],
     "cfc_softcap": [P, c_int64, F, P],
     "cfc_latent_norm": [I, P, I, I, I, I, P, P, F, P, P, I, P, I, P],
-    "cfc_latent_rope": [I, P, I, c_int64, c_int64, I, I, P, F, P, P, I, I, P, I, c_int64, c_int64, I, I, P, P, P, I, c_int64,
-                        c_int64, I, P, P, I, F, P, P],
+    "cfc_latent_rope": [I, P, I, c_int64, c_int64, I, I, P, F, P, P, I, I, P, I, c_int64, c_int64, I, I, P, I, I, P, P, I,
+                        c_int64, c_int64, I, P, P, I, F, P, P],
     "cfc_head_linear": [I, P, c_int64, c_int64, P, I, I, I, I, I, I, P, c_int64, c_int64, P, c_int64, P],
     "cfc_latent_attention": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P, I, I, P, P, P, P],
     "cfc_shift_mix": [I, P, P, P, P, P, I, P, I, I, P, P],
@@ -77,7 +77,9 @@ _KERNEL_SIGS = {
     "cfc_moe_any": [I, I, P, P, I, I, I, P, P, I, P, I, P],
     "cfc_dgemm_group": [I, P, P, I, I, I, I, I, P, P, P, I, F, F, F, P],
     "cfc_pgemm_group": [I, P, I, P, I, I, I, I, P, P, P, I, F, F, F, P],
-    "cfc_latent_gather": [P, P, I, P, P, I, I, P, P, P],
+    "cfc_latent_gather": [P, P, I, P, P, I, I, I, P, P, P, P],
+    "cfc_prefill_attention_expanded2": [P, c_int64, c_int64, P, P, P, P, P, c_int64, P, P, P, P, I, I, F, I, P, P, c_int64, P,
+                                        c_int64, P],
     "cfc_prefill_attention_expanded": [P, P, P, P, c_int64, P, P, P, P, I, I, F, P, c_int64, P],
     "cfc_knn_scores": [P, P, I, I, I, P, P, P, P],
     "cfc_topk_pass": [P, P, I, I, I, I, P, P, P],

@@ -19,8 +19,8 @@ from .stream import _act
 @dataclasses.dataclass
 class Branch:
     """A sublayer's result on its way into the stream: x += LayerNorm((y + y2 + routed rows) * sigmoid(gate + bias)) w.
-    ``y``, ``y2``: fp32 slabs [split, T, W]; ``routed``: (rows [M, W] fp32, row per (token, choice), weight per
-    (token, choice)); ``gate``: pre-sigmoid columns."""
+    ``y``, ``y2``: fp32 slabs [split, T, W]; ``routed``: (rows [M, W] activations, row per (token, choice), weight
+    per (token, choice)); ``gate``: pre-sigmoid columns."""
     gate: Cols
     gate_bias: torch.Tensor
     norm_w: torch.Tensor
@@ -34,7 +34,7 @@ class Branch:
         y = sum(p.sum(0) for p in (self.y, self.y2) if p is not None)
         if self.routed is not None:
             rows, pos, wt = self.routed
-            y = y + (rows[pos.long()] * wt[..., None]).sum(1)
+            y = y + (rows[pos.long()].float() * wt[..., None]).sum(1)
         return ref.layernorm_rows(y * torch.sigmoid(self.gate.value() + self.gate_bias), self.norm_w, self.eps)
 
 
@@ -89,7 +89,7 @@ def _gated(mode, x, b: Branch | None, h, prev, meta, positions, sh: Shift | None
         rows = pos = wt = None
         if b.routed is not None:
             rows, pos, wt = b.routed
-            _req(rows, torch.float32, "routed rows")
+            _req(rows, dtype, "routed rows")
             _req(pos, torch.int32, "routed positions")
             _req(wt, torch.float32, "routed weights")
         g = b.gate.args(dtype)

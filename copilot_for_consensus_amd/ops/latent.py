@@ -112,14 +112,14 @@ def yarn_rope(dims: int, base: float, scaling: dict | None, device) -> Rope:
     return Rope(torch.tensor(f, dtype=torch.float32, device=device), mag)
 
 
-def latent_rope(kv: Cols, rank: int, wc, eps: float, slots, cache, q: Cols, heads: int, dim: int, rope: Rope, positions, ql,
+def latent_rope(kv: Cols, rank: int, wc, eps: float, slots, cache, q: Cols, heads: int, dim: int, rope: Rope, positions, qr,
                 vdim: int = 0, gate: Cols | None = None):
     """The normed latent (``rank`` columns of ``kv``) and the rotated shared key part behind it into ``cache``
-    [blocks, 32, RS] at ``slots``; each head's rotated query part into ql [T, heads, RS] (columns after the latent's).
-    ``q`` columns per head [dim | rot].  Returns (unrotated queries [T, heads, dim], output gate's pre-activations
+    [blocks, 32, RS] at ``slots``; each head's rotated query part into ``qr`` [T, heads, >= rot] (heads at an even
+    stride; the pad zeroed).  ``q`` columns per head [dim | rot].  Returns (unrotated queries [T, heads, dim], output gate's pre-activations
     [T, heads vdim] or None) as activations."""
-    T, RS, RV, dt = ql.shape[0], cache.shape[-1], padded_rank(rank), ql.dtype
-    if not ql.is_cuda:
+    T, RS, RV, dt = qr.shape[0], cache.shape[-1], padded_rank(rank), qr.dtype
+    if not qr.is_cuda:
         y = kv.value()
         c = y[:, :rank]
         c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * wc
@@ -127,19 +127,21 @@ def latent_rope(kv: Cols, rank: int, wc, eps: float, slots, cache, q: Cols, head
         rows[slots.long(), :rank] = c.to(dt)
         rows[slots.long(), RV:RV + rope.dims] = ref.rotate_pairs(y[:, rank:], positions, rope.freq, rope.mag).to(dt)
         qv = q.value().view(T, heads, dim + rope.dims)
-        ql[:, :, RV:] = 0
-        ql[:, :, RV:RV + rope.dims] = ref.rotate_pairs(qv[:, :, dim:], positions, rope.freq, rope.mag).to(dt)
+        qr.zero_()
+        qr[:, :, :rope.dims] = ref.rotate_pairs(qv[:, :, dim:], positions, rope.freq, rope.mag).to(dt)
         return qv[:, :, :dim].to(dt), gate.value().to(dt) if gate is not None else None
-    if cache.dtype != dt or not ql.is_contiguous() or ql.shape[1:] != (heads, RS) or q.n != heads * (dim + rope.dims):
-        raise ValueError(f"latent_rope: ql {tuple(ql.shape)} {dt}, cache rows of {RS} {cache.dtype}, {q.n} query columns")
+    if cache.dtype != dt or qr.stride(2) != 1 or qr.stride(0) != heads * qr.stride(1) or qr.shape[1] != heads \
+            or q.n != heads * (dim + rope.dims):
+        raise ValueError(f"latent_rope: qr {tuple(qr.shape)} {dt}, cache rows of {RS} {cache.dtype}, {q.n} query columns")
     for name, t in (("slots", slots), ("positions", positions)):
         _req(t, torch.int32, name)
-    qn = torch.empty(T, heads, dim, dtype=dt, device=ql.device) if q.slabs else None
-    gt = torch.empty(T, heads * vdim, dtype=dt, device=ql.device) if gate is not None and gate.slabs else None
+    qn = torch.empty(T, heads, dim, dtype=dt, device=qr.device) if q.slabs else None
+    gt = torch.empty(T, heads * vdim, dtype=dt, device=qr.device) if gate is not None and gate.slabs else None
     g = gate.args(dt) if gt is not None else [None, 0, 0, 0]
     check(kernels().cfc_latent_rope(_act(dt), *kv.args(dt), T, rank, wc.data_ptr(), float(eps), slots.data_ptr(),
-                                    cache.data_ptr(), RS, RV, *q.args(dt), heads, dim, ql.data_ptr(), _p(qn), *g, vdim, _p(gt),
-                                    rope.freq.data_ptr(), rope.dims, float(rope.mag), positions.data_ptr(), _stream(ql)),
+                                    cache.data_ptr(), RS, RV, *q.args(dt), heads, dim, qr.data_ptr(), qr.stride(1),
+                                    qr.shape[2], _p(qn), *g, vdim, _p(gt), rope.freq.data_ptr(), rope.dims, float(rope.mag),
+                                    positions.data_ptr(), _stream(qr)),
           "cfc_latent_rope")
     if qn is None:
         qn = q.t[:, q.c0:q.c0 + q.n].unflatten(1, (heads, dim + rope.dims))[:, :, :dim]
@@ -152,7 +154,12 @@ def rows_per_tile(dtype, RS: int, decode_plan: tuple | None = None, RV: int | No
     """(token, head) rows of one attention work item: the general kernel's 4, or 16 / 32 / 64 on MFMA."""
     if dtype != torch.bfloat16 or (RV or RS) > MFMA_MAX_RANK or RS > MFMA_MAX_KEY:
         return ANY_ROWS
-    return decode_plan[0] if decode_plan else 64
+    return decode_plan[0] if decode_plan else most_rows(RS)
+
+
+def most_rows(RS: int) -> int:
+    """Rows of the largest work item whose registers hold: longer rows leave room for 32."""
+    return 64 if RS <= MFMA_MAX_RANK else 32
 
 
 MAX_PARTITIONS = 256
@@ -168,7 +175,7 @@ def decode_plan(B: int, heads: int, RS: int, max_ctx: int, P: int | None = None)
     nt, best = max(1, math.ceil(max_ctx / 64)), None
     cand = [P] if P else sorted({p for p in (1, 2, 3, 4, 5, 6, 8, 10, 12, 16, 20, 24, 32, 48, 64, 96, 128) if p <= nt})
     for rows in (16, 32, 64):
-        if rows > 16 and rows >= 2 * heads:
+        if rows > 16 and (rows >= 2 * heads or rows > most_rows(RS)):
             continue
         g = math.ceil(heads / rows)
         for p in cand:
@@ -249,34 +256,39 @@ def latent_attention(q, cache, block_tables, cu_q, ctx_lens, scale: float, tiles
 
 # ------------------------------------------------------- long portions: expanded keys and values
 EXPANDED_DIM = 128        # head size of the prefill attention kernel
+ROT_COLS = 64             # columns of its second key part
 
 
-def gather_tiles(ctx_lens) -> tuple[list, list]:
-    """Dense layout of whole sequences, 64-token tiles: ([(sequence, first position)], first row per sequence)."""
+def gather_tiles(ctx_lens, starts=None) -> tuple[list, list]:
+    """Dense layout of sequences (from the 64-token tile of position ``starts[s]`` on), 64-token tiles: ([(sequence,
+    first position)], row of position 0 per sequence -- negative where the layout starts later)."""
     tiles, base, n = [], [], 0
     for s, ctx in enumerate(ctx_lens):
-        base.append(n)
-        m = -(-ctx // 64)
-        tiles += [(s, 64 * i) for i in range(m)]
-        n += 64 * m
+        lo, hi = starts[s] // 64 if starts is not None else 0, -(-ctx // 64)
+        base.append(n - 64 * lo)
+        tiles += [(s, 64 * i) for i in range(lo, hi)]
+        n += 64 * (hi - lo)
     return tiles, base
 
 
-def expand(cache, block_tables, ctx_lens, tiles, uk, uv):
+def expand(cache, block_tables, ctx_lens, tiles, uk, uv, RV: int | None = None):
     """Keys [tokens, H * 128] and transposed, slot-ordered values [H * 128, tokens] (row stride padded) of the
-    sequences of ``tiles`` (:func:`gather_tiles`): uk a PackedWeight [H * 128, RS], uv row-major [H * 128, RS]."""
+    sequences of ``tiles`` (:func:`gather_tiles`): uk a PackedWeight [H * 128, RV], uv row-major [H * 128, RV].  ``RV``:
+    latent columns of a row, where a rotated key part follows: it comes third, [tokens, 64]."""
     from . import kernels as K
     n, RS = tiles.shape[0], cache.shape[-1]
-    rows = torch.empty(2, n * 64, RS, dtype=cache.dtype, device=cache.device)
+    k2 = torch.empty(n * 64, ROT_COLS, dtype=cache.dtype, device=cache.device) if RV is not None else None
+    RV = RV or RS
+    rows = torch.empty(2, n * 64, RV, dtype=cache.dtype, device=cache.device)
     check(kernels().cfc_latent_gather(cache.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], ctx_lens.data_ptr(),
-                                      tiles.data_ptr(), n, RS, rows[0].data_ptr(), rows[1].data_ptr(), _stream(cache)),
+                                      tiles.data_ptr(), n, RS, RV, rows[0].data_ptr(), rows[1].data_ptr(), _p(k2), _stream(cache)),
           "cfc_latent_gather")
     k = K.pgemm(rows[0], uk, variant="ppp")
     # the values' rows are read side by side: an odd number of 128-byte lines apart, not a power of two
     ldv = n * 64 + (64 if n % 2 == 0 else 128)
     vt = torch.empty(uv.shape[0], ldv, dtype=cache.dtype, device=cache.device)[:, :n * 64]
-    K.pgemm(uv, K.PackedWeight(rows[1].view(-1), n * 64, RS, 64), out=vt, variant="ppp")
-    return k, vt
+    K.pgemm(uv, K.PackedWeight(rows[1].view(-1), n * 64, RV, 64), out=vt, variant="ppp")
+    return (k, vt) if k2 is None else (k, vt, k2)
 
 
 def expanded_attention(q, k, vt, tok_base, cu_q, ctx_lens, scale: float, tiles, out) -> torch.Tensor:
@@ -289,4 +301,21 @@ def expanded_attention(q, k, vt, tok_base, cu_q, ctx_lens, scale: float, tiles, 
                                                    vt.stride(0), cu_q.data_ptr(), ctx_lens.data_ptr(), tiles[0].data_ptr(),
                                                    tiles[1].data_ptr(), tiles[0].numel(), H, float(scale), out.data_ptr(),
                                                    out.stride(0), _stream(q)), "cfc_prefill_attention_expanded")
+    return out
+
+
+def expanded_window_attention(q: Cols, q2, k, k2, vt, tok_base, cu_q, ctx_lens, scale: float, tiles, window: int, sink, gate, out):
+    """The same with a second key part k2 [tokens, 64] shared by all heads and the heads' q2 [T, H, 64], a sliding
+    ``window`` (0: none), a ``sink`` per head and an output ``gate`` [T, H * 128].  ``q``: columns of which head h's 128
+    start at h * (columns per head)."""
+    T, H = q2.shape[:2]
+    p, _, q_ld, _ = q.args(out.dtype)
+    if q2.shape[2] != ROT_COLS or not q2.is_contiguous() or out.shape != (T, H * EXPANDED_DIM) or out.stride(1) != 1 \
+            or gate.shape != out.shape or gate.stride(1) != 1:
+        raise ValueError(f"expanded_window_attention: q2 {tuple(q2.shape)}, gate {tuple(gate.shape)}, out {tuple(out.shape)}")
+    check(kernels().cfc_prefill_attention_expanded2(p, q_ld, q.n // H, q2.data_ptr(), k.data_ptr(), k2.data_ptr(), vt.data_ptr(),
+                                                    tok_base.data_ptr(), vt.stride(0), cu_q.data_ptr(), ctx_lens.data_ptr(),
+                                                    tiles[0].data_ptr(), tiles[1].data_ptr(), tiles[0].numel(), H, float(scale),
+                                                    int(window), _p(sink), gate.data_ptr(), gate.stride(0), out.data_ptr(),
+                                                    out.stride(0), _stream(q2)), "cfc_prefill_attention_expanded2")
     return out

@@ -113,11 +113,11 @@ def _grouped(glu, x, w, E, N, bn, tile, rows, te, out):
 
 
 def experts(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
-    """W_down (silu(W_gate x) * W_up x) of every (token, choice): (fp32 rows [M, W], row per pair [T, top])."""
+    """W_down (silu(W_gate x) * W_up x) of every (token, choice): (rows [M, W] in x's dtype, row per pair [T, top])."""
     tile = w.tile(ids.numel())
     rows, pos, te = sort_rows(ids, w.E, tile)
     M = te.numel() * tile
-    y = torch.empty(M, w.W, dtype=torch.float32, device=x.device)
+    y = torch.empty(M, w.W, dtype=x.dtype, device=x.device)
     if not x.is_cuda:
         y.zero_()
         for i, e in enumerate(te.tolist()):
@@ -127,7 +127,7 @@ def experts(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
             gu = x[rows[s].long()].float() @ w.gu[e].float().t()
             g, u = gu.chunk(2, -1)
             a = (g * torch.sigmoid(g) * u).to(x.dtype)
-            y[s] = a.float() @ w.down[e].float().t()
+            y[s] = (a.float() @ w.down[e].float().t()).to(x.dtype)
         return y, pos
     a = torch.empty(M, w.F, dtype=x.dtype, device=x.device)
     if w.packed:

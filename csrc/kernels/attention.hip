@@ -889,18 +889,30 @@ __device__ __forceinline__ float quad_sum(float x) {
   const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
   return pair_sum(__uint_as_float(r[0]) + __uint_as_float(r[1]));
 }
+// 64 x 128-byte rows of the second key part: chunk c of row r, swizzled
+__device__ __forceinline__ int k2_lds_off(int r, int c) { return r * 128 + ((c ^ (r & 7)) << 4); }
 __device__ __forceinline__ int v5_off(int d, int c) { return d * 128 + ((c ^ ((d >> 1) & 7) ^ ((d & 1) << 2)) << 4); }
 
 // EXP: keys and values are not in the paged cache but dense (a latent cache's, expanded for this pass):
 // K [tokens][Hkv][128] and V^T [Hkv][128][ldv] with each 32 tokens in the cache's slot order, sequence s
 // at tokens tok_base[s] .. (rounded up to 64, zero-filled); outputs leave with row stride ldo.
-template <int G, bool F8 = false, bool EXP = false>
+// RD = 64 (with EXP): a second key part shared by all heads, K2 [tokens][64], with the heads' q2 [rows][H][64];
+// a sink per head in the denominator; outputs times sigmoid(gate) (row stride ldg, columns as out).
+struct PfExtra {
+  int64_t q_ld = 0, q_hs = 0;         // q strides per row and head
+  const uint16_t* q2 = nullptr;
+  const uint16_t* k2 = nullptr;
+  const float* sink = nullptr;
+  const uint16_t* gate = nullptr;
+  int64_t ldg = 0;
+};
+template <int G, bool F8 = false, bool EXP = false, int RD = 0>
 __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
     const uint16_t* __restrict__ q, const void* __restrict__ kc, const void* __restrict__ vc,
     const int32_t* __restrict__ block_tables, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ ctx_lens,
     const int32_t* __restrict__ tile_seq, const int32_t* __restrict__ tile_q0, float scale_log2, int Hq, int Hkv,
     int max_blocks, int window, float v_scale, int xcd_local, uint16_t* __restrict__ out,
-    const int32_t* __restrict__ tok_base = nullptr, int64_t ldv = 0, int64_t ldo = 0) {
+    const int32_t* __restrict__ tok_base = nullptr, int64_t ldv = 0, int64_t ldo = 0, PfExtra ex = PfExtra{}) {
   // F8: e4m3 caches (K / k_scale folded into scale_log2 by the host, V / v_scale rescaled at the
   // output); tiles are widened to bf16 at the LDS write, so the MFMA loop is the bf16 one
   constexpr int D = 128;
@@ -937,20 +949,26 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
   const int my_pos = pos_base + my_row;
   const int wave_min_pos = pos_base + qs + 32 * rsub;
   // Q^T B-operand, pre-scaled: k-step ks holds Q[row][16ks + 8hi .. +7]
-  bf16x8_t qf[8];
+  bf16x8_t qf[8], qf2[RD ? RD / 16 : 1];
   {
     const int rr = min(my_row, q_len - 1);
-    const uint16_t* qr = q + ((size_t)(q_begin + rr) * Hq + hq) * D;
-#pragma unroll
-    for (int ks = 0; ks < 8; ++ks) {
+    const uint16_t* qr = RD ? q + (q_begin + rr) * ex.q_ld + hq * ex.q_hs : q + ((size_t)(q_begin + rr) * Hq + hq) * D;
+    auto scaled = [&](const uint16_t* p) {
       float f[8];
-      unpack8(*reinterpret_cast<const uint4*>(qr + 16 * ks + 8 * hi), f);
+      unpack8(*reinterpret_cast<const uint4*>(p), f);
       uint4 u;
       u.x = cvt_pk_bf16(f[0] * scale_log2, f[1] * scale_log2);
       u.y = cvt_pk_bf16(f[2] * scale_log2, f[3] * scale_log2);
       u.z = cvt_pk_bf16(f[4] * scale_log2, f[5] * scale_log2);
       u.w = cvt_pk_bf16(f[6] * scale_log2, f[7] * scale_log2);
-      qf[ks] = as_bf16x8(u);
+      return as_bf16x8(u);
+    };
+#pragma unroll
+    for (int ks = 0; ks < 8; ++ks) qf[ks] = scaled(qr + 16 * ks + 8 * hi);
+    if constexpr (RD) {
+      const uint16_t* q2 = ex.q2 + ((size_t)(q_begin + rr) * Hq + hq) * RD;
+#pragma unroll
+      for (int ks = 0; ks < RD / 16; ++ks) qf2[ks] = scaled(q2 + 16 * ks + 8 * hi);
     }
   }
 
@@ -961,7 +979,7 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
   // makes the compiler wait for the loads inside the issue sequence -- they stay in flight across
   // the tile's MFMAs.
   const int nb_need = (kend + KV_BS - 1) / KV_BS;
-  uint4 ks0, ks1, vs0, vs1;     // named (not an array): an array here is kept in scratch
+  uint4 ks0, ks1, vs0, vs1, k2s;     // named (not an array): an array here is kept in scratch
   const int64_t tok0 = EXP ? tok_base[s] : 0;
   auto gload = [&](int kt) {
     if constexpr (EXP) {
@@ -972,6 +990,7 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
       vs0 = *reinterpret_cast<const uint4*>(vp);
       ks1 = *reinterpret_cast<const uint4*>(kp + (int64_t)32 * Hkv * D);
       vs1 = *reinterpret_cast<const uint4*>(vp + 64 * ldv);
+      if constexpr (RD) k2s = *reinterpret_cast<const uint4*>(ex.k2 + (t0 + (tid >> 3)) * RD + 8 * (tid & 7));
       return;
     }
     const int b0 = bt[min(2 * kt, nb_need - 1)], b1 = bt[min(2 * kt + 1, nb_need - 1)];
@@ -997,6 +1016,7 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
       *reinterpret_cast<uint4*>(kb + k_lds_off((tid >> 4) + 32, tid & 15)) = ks1;
       *reinterpret_cast<uint4*>(vb + v5_off(tid >> 3, tid & 7)) = vs0;
       *reinterpret_cast<uint4*>(vb + v5_off((tid >> 3) + 64, tid & 7)) = vs1;
+      if constexpr (RD) *reinterpret_cast<uint4*>(smem + 65536 + buf * 8192 + k2_lds_off(tid >> 3, tid & 7)) = k2s;
       return;
     }
     const bool z0 = kt * PF_KT >= kend, z1 = kt * PF_KT + KV_BS >= kend;
@@ -1079,8 +1099,16 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
           for (int ks = 0; ks < 8; ++ks) kf[ks] = *reinterpret_cast<const uint4*>(kb + k_lds_off(row, 2 * ks + hi));
 #pragma unroll
           for (int ks = 0; ks < 8; ++ks) sc[hf] = mfma32(as_bf16x8(kf[ks]), qf[ks], sc[hf]);
-          __builtin_amdgcn_sched_group_barrier(0x100, 8, 0);   // 8 DS reads, then
-          __builtin_amdgcn_sched_group_barrier(0x008, 8, 0);   // the 8 MFMAs (counted lgkmcnt waits)
+          if constexpr (RD) {
+            uint4 kr[RD / 16];
+#pragma unroll
+            for (int ks = 0; ks < RD / 16; ++ks)
+              kr[ks] = *reinterpret_cast<const uint4*>(smem + 65536 + cur * 8192 + k2_lds_off(row, 2 * ks + hi));
+#pragma unroll
+            for (int ks = 0; ks < RD / 16; ++ks) sc[hf] = mfma32(as_bf16x8(kr[ks]), qf2[ks], sc[hf]);
+          }
+          __builtin_amdgcn_sched_group_barrier(0x100, 8 + RD / 16, 0);   // the DS reads, then
+          __builtin_amdgcn_sched_group_barrier(0x008, 8 + RD / 16, 0);   // the MFMAs (counted lgkmcnt waits)
         } else {
 #pragma unroll
           for (int ks = 0; ks < 8; ++ks)
@@ -1170,15 +1198,31 @@ __global__ void __launch_bounds__(512, 2) prefill_gqa_kernel(
 
   l = pair_sum((lp[0] + lp[1]) + (lp[2] + lp[3]));
   if (my_row < q_len) {
-    const float inv = l > 0.f ? v_scale / l : 0.f;
+    float inv = l > 0.f ? v_scale / l : 0.f;
+    if constexpr (RD != 0) {
+      if (ex.sink) {
+        const float sk = ex.sink[hq] * LOG2E, M = fmaxf(m, sk), f = __builtin_amdgcn_exp2f(m - M);
+        inv = f / (l * f + __builtin_amdgcn_exp2f(sk - M));
+      }
+    }
     uint16_t* orow = EXP ? out + (q_begin + my_row) * ldo + hq * D : out + ((size_t)(q_begin + my_row) * Hq + hq) * D;
 #pragma unroll
     for (int dt = 0; dt < 4; ++dt)
 #pragma unroll
       for (int rg = 0; rg < 4; ++rg) {   // registers 4rg..4rg+3 = d 32dt + 8rg + 4hi + 0..3
+        float y[4] = {o[dt][4 * rg] * inv, o[dt][4 * rg + 1] * inv, o[dt][4 * rg + 2] * inv, o[dt][4 * rg + 3] * inv};
+        if constexpr (RD != 0) {
+          if (ex.gate) {
+            const uint2 gv = *reinterpret_cast<const uint2*>(ex.gate + (q_begin + my_row) * ex.ldg + hq * D + 32 * dt + 8 * rg + 4 * hi);
+            const float gz[4] = {__uint_as_float(gv.x << 16), __uint_as_float(gv.x & 0xffff0000u),
+                                 __uint_as_float(gv.y << 16), __uint_as_float(gv.y & 0xffff0000u)};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) y[e] *= 1.f / (1.f + __expf(-gz[e]));
+          }
+        }
         uint2 pk;
-        pk.x = cvt_pk_bf16(o[dt][4 * rg] * inv, o[dt][4 * rg + 1] * inv);
-        pk.y = cvt_pk_bf16(o[dt][4 * rg + 2] * inv, o[dt][4 * rg + 3] * inv);
+        pk.x = cvt_pk_bf16(y[0], y[1]);
+        pk.y = cvt_pk_bf16(y[2], y[3]);
         *reinterpret_cast<uint2*>(orow + 32 * dt + 8 * rg + 4 * hi) = pk;
       }
   }
@@ -1545,6 +1589,34 @@ CFC_API int cfc_prefill_attention_expanded(const void* q, const void* k, const v
   prefill_gqa_kernel<1, false, true><<<dim3(n_tiles, H), 512, 65536, stream>>>(
       (const uint16_t*)q, k, vt, nullptr, cu_q, ctx_lens, tile_seq, tile_q0, scale * LOG2E, H, H, 0, 0, 1.f,
       prefill_xcd_local(), (uint16_t*)out, tok_base, ldv, ldo);
+  return CFC_CHECK_LAUNCH();
+}
+
+// The same with a second key part of 64 dimensions shared by all heads (K2 [tokens][64]; q2 [rows][H][64]), a sliding
+// window (0: none), a sink per head (may be null) and an output gate (may be null); q row t, head h at
+// t q_ld + h q_hs.
+CFC_API int cfc_prefill_attention_expanded2(const void* q, int64_t q_ld, int64_t q_hs, const void* q2, const void* k,
+                                            const void* k2, const void* vt, const int32_t* tok_base, int64_t ldv,
+                                            const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tile_seq,
+                                            const int32_t* tile_q0, int n_tiles, int H, float scale, int window,
+                                            const float* sink, const void* gate, int64_t ldg, void* out, int64_t ldo,
+                                            hipStream_t stream) {
+  if (n_tiles <= 0) return 0;
+  if (H < 1 || H > 65535 || ldv % 8 || ldo % 4 || ldo < (int64_t)128 * H || ((uintptr_t)vt & 15) || ((uintptr_t)out & 7) ||
+      q_ld % 8 || q_hs % 8 || ((uintptr_t)q & 15) || ldg % 4 || ((uintptr_t)gate & 7) || window < 0 || !q2 || !k2)
+    return -1;
+  PfExtra ex;
+  ex.q_ld = q_ld; ex.q_hs = q_hs; ex.q2 = (const uint16_t*)q2; ex.k2 = (const uint16_t*)k2;
+  ex.sink = sink; ex.gate = (const uint16_t*)gate; ex.ldg = ldg;
+  static bool raised = false;
+  if (!raised) {
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&prefill_gqa_kernel<1, false, true, 64>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, 65536 + 16384);
+    raised = true;
+  }
+  prefill_gqa_kernel<1, false, true, 64><<<dim3(n_tiles, H), 512, 65536 + 16384, stream>>>(
+      (const uint16_t*)q, k, vt, nullptr, cu_q, ctx_lens, tile_seq, tile_q0, scale * LOG2E, H, H, 0, window, 1.f,
+      prefill_xcd_local(), (uint16_t*)out, tok_base, ldv, ldo, ex);
   return CFC_CHECK_LAUNCH();
 }
 

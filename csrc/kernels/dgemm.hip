@@ -554,8 +554,8 @@ void dgemm_group_go(int glu, const void* x, const void* w, int M, int N, int K, 
     dgemm_kernel<BM, BN, DG_GLU, DG_NT, 0, true, 1><<<grid, threads, 0, stream>>>(
         (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, nullptr, (uint16_t*)out, ldo, gp, g);
   else
-    dgemm_kernel<BM, BN, DG_PART, DG_NT, 0, true, 1><<<grid, threads, 0, stream>>>(
-        (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, (float*)out, nullptr, 0, gp, g);
+    dgemm_kernel<BM, BN, DG_BF16, DG_NT, 0, true, 1><<<grid, threads, 0, stream>>>(
+        (const uint16_t*)x, (const uint16_t*)w, M, N, K, N / BN, 1, nullptr, (uint16_t*)out, ldo, gp, g);
 }
 template <int BM>
 int dgemm_group_bn(int glu, const void* x, const void* w, int M, int N, int K, int bn, void* out, int ldo, const DgGlu& gp,
@@ -569,13 +569,13 @@ int dgemm_group_bn(int glu, const void* x, const void* w, int M, int N, int K, i
 }  // namespace
 
 // Products of rows sorted by expert with W[experts][N][K] (each packed for bn): M sorted rows in tiles of bm = 64 or
-// 128, rows / tile_expert as in DgGroup.  glu 0: fp32 out [M][N]; 1: the clamped GLU of 8-row interleaved gate / up
-// rows, bf16 [M][N / 2] (row stride ldo)
+// 128, rows / tile_expert as in DgGroup.  bf16 out of row stride ldo: [M][N], or (glu) the clamped GLU of 8-row
+// interleaved gate / up rows [M][N / 2]
 CFC_API int cfc_dgemm_group(int glu, const void* x, const void* w, int M, int N, int K, int bn, int bm, const int32_t* rows,
                             const int32_t* tile_expert, void* out, int ldo, float limit, float alpha, float beta,
                             hipStream_t stream) {
   if (M == 0) return 0;
-  if (const int e = dgemm_check(M, N, K, 1, glu ? DG_GLU : DG_PART, bn, (const float*)out, out, glu ? ldo : N)) return e;
+  if (const int e = dgemm_check(M, N, K, 1, glu ? DG_GLU : DG_BF16, bn, nullptr, out, ldo)) return e;
   if (!tile_expert || (bm != 64 && bm != 128) || M % bm) return -1;
   DgGlu gp;
   gp.limit = limit; gp.alpha = alpha; gp.beta = beta;

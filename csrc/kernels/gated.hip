@@ -151,7 +151,7 @@ __global__ void __launch_bounds__(256) shift_mix_kernel(const float* __restrict_
 struct BranchArgs {
   const float* y;  int ysplit;            // slabs [ysplit][T][W] (null: none)
   const float* y2; int y2split;           // a second product's
-  const float* ym; const int32_t* mrow; const float* mwt; int top;   // routed rows [*][W], row and weight per (token, choice)
+  const void* ym; const int32_t* mrow; const float* mwt; int top;   // routed rows [*][W] (activations), row and weight per (token, choice)
   const void* gate; int gate_act, gsplit; int64_t gld, gplane;       // pre-sigmoid: slabs, or activations (gate_act)
   const float* gbias;                     // [W]
   const float* norm_w;                    // [W]
@@ -204,7 +204,7 @@ __global__ void __launch_bounds__(BT) gated_norm_kernel(BranchArgs b, float* __r
       if (b.ym)
         for (int i = 0; i < b.top; ++i) {
           const float wt = b.mwt[(size_t)t * b.top + i];
-          const Vec<V> r = ldv<V>(b.ym + (size_t)b.mrow[(size_t)t * b.top + i] * W + c);
+          const Vec<V> r = ldv<V>(reinterpret_cast<const ACT*>(b.ym) + (size_t)b.mrow[(size_t)t * b.top + i] * W + c);
 #pragma unroll
           for (int e = 0; e < V; ++e) y[k].v[e] += wt * r.v[e];
         }
@@ -349,7 +349,7 @@ CFC_API int cfc_shift_mix(int f32, const float* x, const int32_t* meta, const in
 
 // mode 0: prompt rows (h: the updated row as an activation, prev: store the portion's last rows of x as they
 // were); mode 1: decoded rows (acts null: no shift follows; norm_w null: no branch comes first)
-CFC_API int cfc_gated_norm(int mode, int f32, const float* y, int ysplit, const float* y2, int y2split, const float* ym,
+CFC_API int cfc_gated_norm(int mode, int f32, const float* y, int ysplit, const float* y2, int y2split, const void* ym,
                            const int32_t* mrow, const float* mwt, int top, const void* gate, int gate_act, int gsplit,
                            int64_t gld, int64_t gplane, const float* gbias, const float* norm_w, float eps, float* x, int T,
                            int W, void* h, float* prev, const int32_t* meta, const int32_t* positions, const float* shift,

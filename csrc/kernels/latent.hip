@@ -148,28 +148,33 @@ struct RopeArgs {
   int rot;
 };
 
-__device__ __forceinline__ void rope_pair(const RopeArgs& r, int pos, int i, float& u, float& v) {
-  float sn, cs;
-  sincosf((float)pos * r.freq[i], &sn, &cs);
-  cs *= r.mag;
-  sn *= r.mag;
-  const float a = u * cs - v * sn, b = v * cs + u * sn;
-  u = a;
-  v = b;
-}
+constexpr int ROPE_MAX = 1024;
 
-// grid (rows, 1 + heads).  y = 0: RMS norm of the NC latent columns, the rotated key part behind them
-// (from column RV of the cache row).  y = 1 + h: head h's rotated query part at columns RV .. RS of its row of
-// ql (the pad zeroed); where q comes as slabs its unrotated part goes to qn [T][H][dim] as activations, and the
+// grid (rows, 1 + NB).  y = 0: RMS norm of the NC latent columns, the rotated key part behind them
+// (from column RV of the cache row).  y > 0: a run of heads' rotated query parts, PQ columns (the pad zeroed) at
+// qr + (t H + h) qs; where q comes as slabs its unrotated part goes to qn [T][H][dim] as activations, and the
 // output gate's columns to gate [T][H vdim].
 template <typename ACT>
 __global__ void __launch_bounds__(256) latent_rope_kernel(LatCols kv, int NC, const float* __restrict__ wc, float eps,
                                                          const int32_t* __restrict__ slots, ACT* __restrict__ cache, int RS,
-                                                         int RV, LatCols q, int dim, ACT* __restrict__ ql,
-                                                         ACT* __restrict__ qn, LatCols g, int vdim, ACT* __restrict__ gate,
+                                                         int RV, LatCols q, int H, int dim, ACT* __restrict__ qr, int qs,
+                                                         int PQ, ACT* __restrict__ qn, LatCols g, int vdim, ACT* __restrict__ gate,
                                                          RopeArgs r) {
   __shared__ float red[16];
-  const int t = blockIdx.x, tid = threadIdx.x, H = gridDim.y - 1, pos = r.positions[t];
+  __shared__ float2 cs[ROPE_MAX / 2];
+  const int t = blockIdx.x, tid = threadIdx.x, pos = r.positions[t];
+  for (int i = tid; i < r.rot / 2; i += 256) {
+    float sn, co;
+    sincosf((float)pos * r.freq[i], &sn, &co);
+    cs[i] = make_float2(co * r.mag, sn * r.mag);
+  }
+  __syncthreads();
+  auto rotate = [&](int i, float& u, float& v) {
+    const float2 c = cs[i];
+    const float a = u * c.x - v * c.y, b = v * c.x + u * c.y;
+    u = a;
+    v = b;
+  };
   if (blockIdx.y == 0) {
     ACT* dst = cache + (size_t)slots[t] * RS;
     float x[4], s = 0.f;
@@ -192,28 +197,31 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatCols kv, int NC, co
     for (int c = 1024 + tid; c < NC; c += 256) stf(dst + c, ldcol<ACT>(kv, t, c) * rs * wc[c]);
     for (int i = tid; i < r.rot / 2; i += 256) {
       float u = ldcol<ACT>(kv, t, NC + 2 * i), v = ldcol<ACT>(kv, t, NC + 2 * i + 1);
-      rope_pair(r, pos, i, u, v);
+      rotate(i, u, v);
       stf(dst + RV + 2 * i, u);
       stf(dst + RV + 2 * i + 1, v);
     }
     return;
   }
-  const int h = blockIdx.y - 1, q0 = h * (dim + r.rot);
-  ACT* row = ql + ((size_t)t * H + h) * RS;
-  for (int i = tid; i < (RS - RV) / 2; i += 256) {
+  const int NB = gridDim.y - 1, h0 = H * (blockIdx.y - 1) / NB, h1 = H * blockIdx.y / NB, hp = PQ / 2;
+  for (int e = tid; e < (h1 - h0) * hp; e += 256) {
+    const int h = h0 + e / hp, i = e % hp;
     float u = 0.f, v = 0.f;
     if (i < r.rot / 2) {
-      u = ldcol<ACT>(q, t, q0 + dim + 2 * i);
-      v = ldcol<ACT>(q, t, q0 + dim + 2 * i + 1);
-      rope_pair(r, pos, i, u, v);
+      const int c = h * (dim + r.rot) + dim + 2 * i;
+      u = ldcol<ACT>(q, t, c);
+      v = ldcol<ACT>(q, t, c + 1);
+      rotate(i, u, v);
     }
-    stf(row + RV + 2 * i, u);
-    stf(row + RV + 2 * i + 1, v);
+    ACT* row = qr + ((size_t)t * H + h) * qs + 2 * i;
+    stf(row, u);
+    stf(row + 1, v);
   }
   if (qn)
-    for (int c = tid; c < dim; c += 256) stf(qn + ((size_t)t * H + h) * dim + c, ldcol<ACT>(q, t, q0 + c));
+    for (int e = h0 * dim + tid; e < h1 * dim; e += 256)
+      stf(qn + (size_t)t * H * dim + e, ldcol<ACT>(q, t, e / dim * (dim + r.rot) + e % dim));
   if (gate)
-    for (int c = tid; c < vdim; c += 256) stf(gate + ((size_t)t * H + h) * vdim + c, ldcol<ACT>(g, t, h * vdim + c));
+    for (int e = h0 * vdim + tid; e < h1 * vdim; e += 256) stf(gate + (size_t)t * H * vdim + e, ldcol<ACT>(g, t, e));
 }
 
 // ---------------------------------------------------------------------------------- head_linear
@@ -785,9 +793,10 @@ __global__ void __launch_bounds__(256) latent_attn_any_kernel(const ACT* __restr
 __global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __restrict__ cache,
                                                            const int32_t* __restrict__ block_tables, int max_blocks,
                                                            const int32_t* __restrict__ ctx_lens,
-                                                           const int32_t* __restrict__ tiles, int RS,
-                                                           uint16_t* __restrict__ rows, uint16_t* __restrict__ slot_rows) {
-  const int s = tiles[2 * blockIdx.x], p0 = tiles[2 * blockIdx.x + 1], ctx = ctx_lens[s], ch = RS / 8;
+                                                           const int32_t* __restrict__ tiles, int RS, int RV,
+                                                           uint16_t* __restrict__ rows, uint16_t* __restrict__ slot_rows,
+                                                           uint16_t* __restrict__ k2) {
+  const int s = tiles[2 * blockIdx.x], p0 = tiles[2 * blockIdx.x + 1], ctx = ctx_lens[s], ch = RV / 8;
   const int32_t* bt = block_tables + (size_t)s * max_blocks;
   for (int e = threadIdx.x; e < 64 * ch; e += 256) {
     const int r = e / ch, c = e % ch, p = p0 + r;
@@ -795,11 +804,19 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __re
                                   cache + ((size_t)bt[p / CFC_KV_BS] * CFC_KV_BS + p % CFC_KV_BS) * RS + 8 * c)
                             : make_uint4(0, 0, 0, 0);
     const size_t base = (size_t)blockIdx.x * 64;
-    reinterpret_cast<uint4*>(rows + (base + r) * RS)[c] = v;
+    reinterpret_cast<uint4*>(rows + (base + r) * RV)[c] = v;
     const int sr = (r & 32) + kv_v_slot(r & 31);
-    reinterpret_cast<uint4*>(slot_rows)[(((size_t)blockIdx.x * (RS / 32) + (c >> 2)) * 4 + (sr >> 4)) * 64 + (sr & 15) +
+    reinterpret_cast<uint4*>(slot_rows)[(((size_t)blockIdx.x * (RV / 32) + (c >> 2)) * 4 + (sr >> 4)) * 64 + (sr & 15) +
                                         16 * (c & 3)] = v;
   }
+  if (k2)
+    for (int e = threadIdx.x; e < 64 * 8; e += 256) {      // the rest of the row, padded to 64 columns
+      const int r = e >> 3, c = e & 7, p = p0 + r;
+      const uint4 v = p < ctx && RV + 8 * c < RS
+                          ? *reinterpret_cast<const uint4*>(cache + ((size_t)bt[p / CFC_KV_BS] * CFC_KV_BS + p % CFC_KV_BS) * RS + RV + 8 * c)
+                          : make_uint4(0, 0, 0, 0);
+      reinterpret_cast<uint4*>(k2 + ((size_t)blockIdx.x * 64 + r) * 64)[c] = v;
+    }
 }
 
 // one workgroup of 128 threads per (token, head) row; P <= LC_MAXP
@@ -874,7 +891,8 @@ int lat_mr(int mr, dim3 grid, hipStream_t s, const void* q, const void* cache, c
   switch (mr) {
     case 1: return lat_go<R64, V64, 1>(grid, s, q, cache, a, out);
     case 2: return lat_go<R64, V64, 2>(grid, s, q, cache, a, out);
-    case 4: return lat_go<R64, V64, 4>(grid, s, q, cache, a, out);
+    case 4:
+      if constexpr (R64 <= 512) return lat_go<R64, V64, 4>(grid, s, q, cache, a, out);      // past that the registers spill
   }
   return -3;
 }
@@ -894,19 +912,24 @@ CFC_API int cfc_latent_norm(int f32, const float* part, int split, int T, int NQ
 }
 
 // kv columns [NC latent | rot key part], q columns per head [dim | rot]; each operand: pointer, split (0:
-// activations, else fp32 slabs), row stride, slab stride.  ql [T][H][RS]; qn, gate may be null
+// activations, else fp32 slabs), row stride, slab stride.  Rotated queries: PQ columns of row t H + h at qr (row stride
+// qs); qn, gate may be null
 CFC_API int cfc_latent_rope(int f32, const void* kv, int kv_split, int64_t kv_ld, int64_t kv_plane, int T, int NC,
                             const float* wc, float eps, const int32_t* slots, void* cache, int RS, int RV, const void* q,
-                            int q_split, int64_t q_ld, int64_t q_plane, int H, int dim, void* ql, void* qn, const void* g,
+                            int q_split, int64_t q_ld, int64_t q_plane, int H, int dim, void* qr, int qs, int PQ, void* qn, const void* g,
                             int g_split, int64_t g_ld, int64_t g_plane, int vdim, void* gate, const float* freq, int rot,
                             float mag, const int32_t* positions, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (NC < 1 || NC > RV || RV % 2 || rot < 0 || rot % 2 || RV + rot > RS || RS % 2 || H < 1 || H > 65534 || dim < 1) return -1;
+  if (NC < 1 || NC > RV || RV % 2 || rot < 0 || rot % 2 || rot > ROPE_MAX || RV + rot > RS || PQ < rot || PQ % 2 || qs < PQ ||
+      H < 1 || dim < 1)
+    return -1;
+  // few rows: one workgroup per head, so their slab sums do not follow one another
+  const int NB = T >= 512 ? 1 : H < 64 ? H : 64;
   const LatCols ckv{kv, kv_split, kv_ld, kv_plane}, cq{q, q_split, q_ld, q_plane}, cg{g, g_split, g_ld, g_plane};
   const RopeArgs r{freq, mag, positions, rot};
 #define LR(ACT)                                                                                                         \
-  latent_rope_kernel<ACT><<<dim3(T, 1 + H), 256, 0, stream>>>(ckv, NC, wc, eps, slots, (ACT*)cache, RS, RV, cq, dim, (ACT*)ql, \
-                                                             (ACT*)qn, cg, vdim, (ACT*)gate, r)
+  latent_rope_kernel<ACT><<<dim3(T, 1 + NB), 256, 0, stream>>>(ckv, NC, wc, eps, slots, (ACT*)cache, RS, RV, cq, H, dim, \
+                                                              (ACT*)qr, qs, PQ, (ACT*)qn, cg, vdim, (ACT*)gate, r)
   if (f32) LR(float);
   else LR(uint16_t);
 #undef LR
@@ -946,8 +969,8 @@ CFC_API int cfc_head_linear(int f32, const void* x, int64_t ldx, int64_t hsx, co
   return CFC_CHECK_LAUNCH();
 }
 
-// rows_per_tile: 16 / 32 / 64 on the MFMA kernel (bf16, RS <= 512, or RS <= 576 with RV <= 512), 4 on the general
-// one.  A cached row's RS columns are the key, its first RV the value; out [rows][RV]
+// rows_per_tile: 16 / 32 / 64 on the MFMA kernel (bf16, RS <= 512; 16 / 32 for RS <= 576 with RV <= 512), 4 on the
+// general one.  A cached row's RS columns are the key, its first RV the value; out [rows][RV]
 CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, const int32_t* block_tables,
                                  const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tile_seq,
                                  const int32_t* tile_m0, int n_tiles, int tiles_per_seq, int rows_per_tile, int H, int RS,
@@ -993,10 +1016,11 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
 }
 
 CFC_API int cfc_latent_gather(const void* cache, const int32_t* block_tables, int max_blocks, const int32_t* ctx_lens,
-                              const int32_t* tiles, int n_tiles, int RS, void* rows, void* slot_rows, hipStream_t stream) {
+                              const int32_t* tiles, int n_tiles, int RS, int RV, void* rows, void* slot_rows, void* k2,
+                              hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (RS < 32 || RS % 32 || max_blocks < 1) return -1;
+  if (RV < 32 || RV % 32 || RS < RV || RS % 8 || (k2 && RS - RV > 64) || max_blocks < 1) return -1;
   latent_gather_kernel<<<n_tiles, 256, 0, stream>>>((const uint16_t*)cache, block_tables, max_blocks, ctx_lens, tiles, RS,
-                                                    (uint16_t*)rows, (uint16_t*)slot_rows);
+                                                    RV, (uint16_t*)rows, (uint16_t*)slot_rows, (uint16_t*)k2);
   return CFC_CHECK_LAUNCH();
 }

@@ -31,7 +31,13 @@ __global__ void __launch_bounds__(256) moe_route_kernel(const float* __restrict_
     const int e = lane + 64 * i;
     float z = 0.f;
     if (e < E && t < T)
-      for (int p = 0; p < split; ++p) z += logits[(int64_t)p * plane + (int64_t)t * ld + e];
+      for (int p0 = 0; p0 < split; p0 += 16) {         // sixteen slabs in flight (past the last: re-read, not added)
+        float v[16];
+#pragma unroll
+        for (int u = 0; u < 16; ++u) v[u] = logits[(int64_t)min(p0 + u, split - 1) * plane + (int64_t)t * ld + e];
+#pragma unroll
+        for (int u = 0; u < 16; ++u) z += p0 + u < split ? v[u] : 0.f;
+      }
     s[i] = 1.f / (1.f + expf(-z));
     c[i] = e < E ? s[i] + correction[min(e, E - 1)] : -INFINITY;
     choice[w][e] = c[i];
@@ -130,7 +136,7 @@ __global__ void __launch_bounds__(1024) moe_rows_kernel(const int32_t* __restric
 }
 
 // Row-major W [experts][GLU ? 2 N : N][K]; 32 rows x 64 columns per workgroup, K in steps of 16 through LDS.
-// GLU: columns n of the gate rows 0 .. N - 1 and of the up rows N .. 2 N - 1, silu(g) u; else the product, fp32
+// GLU: columns n of the gate rows 0 .. N - 1 and of the up rows N .. 2 N - 1, silu(g) u; else the product
 template <typename ACT, bool GLU>
 __global__ void __launch_bounds__(256) moe_any_kernel(const ACT* __restrict__ x, const ACT* __restrict__ W, int N, int K,
                                                      const int32_t* __restrict__ rows, const int32_t* __restrict__ tile_expert,
@@ -174,7 +180,7 @@ __global__ void __launch_bounds__(256) moe_any_kernel(const ACT* __restrict__ x,
         const float g = acc[0][a][b];
         st1(reinterpret_cast<ACT*>(out) + (size_t)m * ldo + n, g / (1.f + expf(-g)) * acc[NM - 1][a][b]);
       } else {
-        reinterpret_cast<float*>(out)[(size_t)m * ldo + n] = acc[0][a][b];
+        st1(reinterpret_cast<ACT*>(out) + (size_t)m * ldo + n, acc[0][a][b]);
       }
     }
 }
@@ -207,7 +213,7 @@ CFC_API int cfc_moe_rows(const int32_t* ids, int pairs, int top, int E, int tile
   return CFC_CHECK_LAUNCH();
 }
 
-// M sorted rows in tiles of `tile` (a multiple of 32).  glu: activations [M][N], else fp32 [M][N]; row stride ldo
+// M sorted rows in tiles of `tile` (a multiple of 32), activations [M][N] of row stride ldo
 CFC_API int cfc_moe_any(int f32, int glu, const void* x, const void* w, int M, int N, int K, const int32_t* rows,
                         const int32_t* tile_expert, int tile, void* out, int ldo, hipStream_t stream) {
   if (M == 0) return 0;

@@ -1395,13 +1395,13 @@ CFC_API int cfc_pgemm_glu(const void* x, const void* w, void* out, int M, int N,
 }
 
 // Products of rows sorted by expert with W[experts][N][K] (each packed for bn = 16 wnw): M sorted rows in tiles of
-// 256, rows / tile_expert as in PgGroup (rows of an x_rows-row X).  glu 0: fp32 out [M][N]; 1: the clamped GLU of
-// 8-row interleaved gate / up rows, bf16 [M][N / 2] (row stride ldo)
+// 256, rows / tile_expert as in PgGroup (rows of an x_rows-row X).  bf16 out of row stride ldo: [M][N], or (glu) the
+// clamped GLU of 8-row interleaved gate / up rows [M][N / 2]
 CFC_API int cfc_pgemm_group(int glu, const void* x, int x_rows, const void* w, int M, int N, int K, int wnw, const int32_t* rows,
                             const int32_t* tile_expert, void* out, int ldo, float limit, float alpha, float beta,
                             hipStream_t stream) {
   if (M == 0) return 0;
-  if (M < 1 || M % PG_BM || N < 64 || K < 64 || K % 64 || N % 64 || ldo % 4 || ldo < (glu ? N / 2 : N) || wnw < 1 ||
+  if (M < 1 || M % PG_BM || N < 64 || K < 64 || K % 64 || N % 64 || ldo % 8 || ((uintptr_t)out & 15) || ldo < (glu ? N / 2 : N) || wnw < 1 ||
       N % (16 * wnw) || !tile_expert || x_rows < 1 || (!rows && x_rows < M) || (uint64_t)x_rows * K * 2 >= (1ull << 32) ||
       (uint64_t)N * K * 2 >= (1ull << 32))
     return (int)hipErrorInvalidValue;
@@ -1415,7 +1415,7 @@ CFC_API int cfc_pgemm_group(int glu, const void* x, int x_rows, const void* w, i
   if (glu)
     pgemm_pp_kernel<PG_GLU, true, PP_PF, true><<<tm * tn, 512, 0, stream>>>(xp, wp, nullptr, op, M, N, K, ldo, tm, tn, wnw, PG_GROUP_M, gp, g);
   else
-    pgemm_pp_kernel<PG_F32, true, PP_PF, true><<<tm * tn, 512, 0, stream>>>(xp, wp, nullptr, op, M, N, K, ldo, tm, tn, wnw, PG_GROUP_M, gp, g);
+    pgemm_pp_kernel<PG_BF16, true, PP_PF | 64, true><<<tm * tn, 512, 0, stream>>>(xp, wp, nullptr, op, M, N, K, ldo, tm, tn, wnw, PG_GROUP_M, gp, g);
   return (int)hipGetLastError();
 }
 

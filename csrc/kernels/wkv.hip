@@ -186,6 +186,7 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
     pj[e] = p - i * (i - 1) / 2;
   }
   float acc[2] = {0.f, 0.f};
+#pragma unroll 2
   for (int c = 0; c < DP; c += 4)
 #pragma unroll
     for (int e = 0; e < 2; ++e) {
@@ -235,16 +236,24 @@ __device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 
+// Records, v and g of the next SCAN_AHEAD chunks are on their way in registers while a chunk runs from LDS (two
+// buffers, one barrier per chunk); a chunk's outputs wait for the head's mean square until the next barrier.
+constexpr int SCAN_AHEAD = 4;
+
 template <typename ACT, int ND>
-__global__ void __launch_bounds__(64 * ND) wkv_scan_kernel(const float* __restrict__ rec, Cols v, Cols g, ScanSeq sq, int H,
-                                                          int D, const float* __restrict__ norm, float eps,
-                                                          float* __restrict__ state, ACT* __restrict__ out, int64_t ldo) {
+__global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __restrict__ rec, Cols v, Cols g, ScanSeq sq, int H,
+                                                             int D, const float* __restrict__ norm, float eps,
+                                                             float* __restrict__ state, ACT* __restrict__ out, int64_t ldo) {
   using Rec = ChunkRec<ND>;
-  __shared__ float red[2][ND][16];
-  const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), col = lane & 15, q = lane >> 4;
+  constexpr int NV4 = Rec::SIZE / 4, NT = 64 * ND, NLD = (NV4 + NT - 1) / NT;
+  __shared__ __attribute__((aligned(16))) float buf[2][Rec::SIZE];
+  __shared__ __attribute__((aligned(16))) float red[2][ND][16];
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, q = lane >> 4;
   const int h = blockIdx.x, s = blockIdx.y;
-  const int c0 = sq.chunk_cu[s], c1 = sq.chunk_cu[s + 1];
-  const bool fresh = sq.ctx_lens[s] == sq.cu_q[s + 1] - sq.cu_q[s];
+  const int c0 = sq.chunk_cu[s], nc = sq.chunk_cu[s + 1] - c0;
+  if (nc <= 0) return;
+  const int row0 = sq.cu_q[s], len = sq.cu_q[s + 1] - row0;
+  const bool fresh = sq.ctx_lens[s] == len;
   const int vc = 16 * w + col;                    // value channel of this lane
   const bool live = vc < D;
   const int hv = h * D + min(vc, D - 1);
@@ -258,94 +267,115 @@ __global__ void __launch_bounds__(64 * ND) wkv_scan_kernel(const float* __restri
       S[T][i] = !fresh && live && kc < D ? st[(size_t)min(kc, D - 1) * D] : 0.f;
     }
   const float nw = norm[hv];
-  struct Frag {
-    float4 r[ND], k[ND], dec[ND], a;
-    float v[4], g[4];
-    int row0, n;
-  };
-  auto load = [&](int c, Frag& f) {
-    const float4* p = reinterpret_cast<const float4*>(rec + ((size_t)c * H + h) * Rec::SIZE);
-    f.row0 = sq.chunks[2 * c];
-    f.n = sq.chunks[2 * c + 1];
+  typedef float f4_t __attribute__((ext_vector_type(4)));      // arrays of these stay in registers
+  f4_t rr[SCAN_AHEAD][NLD];
+  float rv[SCAN_AHEAD][4], rg[SCAN_AHEAD][4];
+  const ACT* vp = reinterpret_cast<const ACT*>(v.p) + hv;
+  const ACT* gp = reinterpret_cast<const ACT*>(g.p) + hv;
+  // chunk c (past the last: re-read, not used)
+  auto load = [&](int c, int u) {
+    c = min(c, nc - 1);
+    const f4_t* p = reinterpret_cast<const f4_t*>(rec + ((size_t)(c0 + c) * H + h) * Rec::SIZE);
 #pragma unroll
-    for (int T = 0; T < ND; ++T) {
-      f.r[T] = p[T * 64 + lane];
-      f.k[T] = p[Rec::K / 4 + T * 64 + lane];
-      f.dec[T] = p[Rec::DEC / 4 + 4 * T + q];
-    }
-    f.a = p[Rec::A / 4 + lane];
+    for (int i = 0; i < NLD; ++i) rr[u][i] = p[min(tid + NT * i, NV4 - 1)];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int64_t t = f.row0 + min(4 * q + i, f.n - 1);
-      f.v[i] = ld1(reinterpret_cast<const ACT*>(v.p) + t * v.ld + hv);
-      f.g[i] = ld1(reinterpret_cast<const ACT*>(g.p) + t * g.ld + hv);
+      const int64_t t = row0 + min(CT * c + 4 * q + i, len - 1);
+      rv[u][i] = ld1(vp + t * v.ld);
+      rg[u][i] = ld1(gp + t * g.ld);
     }
   };
-  Frag f[2];
-  if (c0 < c1) load(c0, f[0]);
-  auto chunk = [&](int c, Frag& cur, Frag& nxt, int par) {
-    load(min(c + 1, c1 - 1), nxt);
-    f32x4_t o0{0.f, 0.f, 0.f, 0.f}, o1{0.f, 0.f, 0.f, 0.f};
-    float vv[4];
+  auto store = [&](int b, int u) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) vv[i] = live && 4 * q + i < cur.n ? cur.v[i] : 0.f;
-#pragma unroll
-    for (int T = 0; T < ND; ++T) {
-      o0 = mfma4(cur.r[T].x, S[T][0], o0);
-      o1 = mfma4(cur.r[T].y, S[T][1], o1);
-      o0 = mfma4(cur.r[T].z, S[T][2], o0);
-      o1 = mfma4(cur.r[T].w, S[T][3], o1);
-    }
-    o0 = mfma4(cur.a.x, vv[0], o0);
-    o1 = mfma4(cur.a.y, vv[1], o1);
-    o0 = mfma4(cur.a.z, vv[2], o0);
-    o1 = mfma4(cur.a.w, vv[3], o1);
-#pragma unroll
-    for (int T = 0; T < ND; ++T) {
-      S[T][0] *= cur.dec[T].x; S[T][1] *= cur.dec[T].y; S[T][2] *= cur.dec[T].z; S[T][3] *= cur.dec[T].w;
-    }
-#pragma unroll
-    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].x, vv[0], S[T]);
-#pragma unroll
-    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].y, vv[1], S[T]);
-#pragma unroll
-    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].z, vv[2], S[T]);
-#pragma unroll
-    for (int T = 0; T < ND; ++T) S[T] = mfma4(cur.k[T].w, vv[3], S[T]);
-    // rms over the head: the wave's 16 channels, then the waves
-    const f32x4_t o = o0 + o1;
-    float ss[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      ss[i] = live ? o[i] * o[i] : 0.f;
-#pragma unroll
-      for (int m = 8; m > 0; m >>= 1) ss[i] += __shfl_xor(ss[i], m, 64);
-    }
-    if (col == 0) *reinterpret_cast<float4*>(&red[par][w][4 * q]) = make_float4(ss[0], ss[1], ss[2], ss[3]);
+    for (int i = 0; i < NLD; ++i)
+      if (NT * (i + 1) <= NV4 || tid + NT * i < NV4) reinterpret_cast<f4_t*>(buf[b])[tid + NT * i] = rr[u][i];
+  };
+  auto barrier = [] {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
     __builtin_amdgcn_s_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
-    float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
+  };
+  f32x4_t o_prev{0.f, 0.f, 0.f, 0.f};
+  float g_prev[4] = {0.f, 0.f, 0.f, 0.f};
+  // outputs of chunk c from the mean squares in red[b]
+  auto finish = [&](int c, int b) {
+    float sv[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int j = 0; j < ND; ++j) {
-      const float4 a = *reinterpret_cast<const float4*>(&red[par][j][4 * q]);
-      sum.x += a.x; sum.y += a.y; sum.z += a.z; sum.w += a.w;
+      const float4 a = *reinterpret_cast<const float4*>(&red[b][j][4 * q]);
+      sv[0] += a.x; sv[1] += a.y; sv[2] += a.z; sv[3] += a.w;
     }
-    const float sv[4] = {sum.x, sum.y, sum.z, sum.w};
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const float gg = cur.g[i];
-      const float y = o[i] * (1.f / sqrtf(sv[i] / (float)D + eps)) * nw * (gg / (1.f + __expf(-gg)));
-      if (live && 4 * q + i < cur.n) st1(out + (int64_t)(cur.row0 + 4 * q + i) * ldo + hv, y);
+      const int t = CT * c + 4 * q + i;
+      const float y = o_prev[i] * (1.f / sqrtf(sv[i] / (float)D + eps)) * nw * (g_prev[i] / (1.f + __expf(-g_prev[i])));
+      if (live && t < len) st1(out + (int64_t)(row0 + t) * ldo + hv, y);
     }
   };
-  int c = c0;
-  for (; c + 2 <= c1; c += 2) {
-    chunk(c, f[0], f[1], 0);
-    chunk(c + 1, f[1], f[0], 1);
-  }
-  if (c < c1) chunk(c, f[0], f[1], 0);
-  if (live && c0 < c1) {
+#pragma unroll
+  for (int u = 0; u < SCAN_AHEAD; ++u) load(u, u);
+  store(0, 0);
+  // chunk c from buf[u & 1] (its v and g in slot u); slot u then takes chunk c + SCAN_AHEAD
+  auto chunk = [&](int c, int u) {
+    barrier();
+    const int b = u & 1;
+    if (c > 0) finish(c - 1, b ^ 1);
+    float vv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      vv[i] = live && CT * c + 4 * q + i < len ? rv[u][i] : 0.f;
+      g_prev[i] = rg[u][i];
+    }
+    load(c + SCAN_AHEAD, u);
+    const float4* p = reinterpret_cast<const float4*>(buf[b]);
+    f32x4_t o0{0.f, 0.f, 0.f, 0.f}, o1{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int T = 0; T < ND; ++T) {
+      const float4 r = p[T * 64 + lane];
+      o0 = mfma4(r.x, S[T][0], o0);
+      o1 = mfma4(r.y, S[T][1], o1);
+      o0 = mfma4(r.z, S[T][2], o0);
+      o1 = mfma4(r.w, S[T][3], o1);
+    }
+    const float4 a = p[Rec::A / 4 + lane];
+    o0 = mfma4(a.x, vv[0], o0);
+    o1 = mfma4(a.y, vv[1], o1);
+    o0 = mfma4(a.z, vv[2], o0);
+    o1 = mfma4(a.w, vv[3], o1);
+    float4 k[ND];
+#pragma unroll
+    for (int T = 0; T < ND; ++T) {
+      const float4 d = p[Rec::DEC / 4 + 4 * T + q];
+      k[T] = p[Rec::K / 4 + T * 64 + lane];
+      S[T][0] *= d.x; S[T][1] *= d.y; S[T][2] *= d.z; S[T][3] *= d.w;
+    }
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(k[T].x, vv[0], S[T]);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(k[T].y, vv[1], S[T]);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(k[T].z, vv[2], S[T]);
+#pragma unroll
+    for (int T = 0; T < ND; ++T) S[T] = mfma4(k[T].w, vv[3], S[T]);
+    // sums of squares over the wave's 16 channels
+    o_prev = o0 + o1;
+    float ss[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      ss[i] = live ? o_prev[i] * o_prev[i] : 0.f;
+#pragma unroll
+      for (int m = 8; m > 0; m >>= 1) ss[i] += __shfl_xor(ss[i], m, 64);
+    }
+    if (col == 0) *reinterpret_cast<float4*>(&red[b][w][4 * q]) = make_float4(ss[0], ss[1], ss[2], ss[3]);
+    store(b ^ 1, (u + 1) % SCAN_AHEAD);
+  };
+  for (int c = 0; c < nc; c += SCAN_AHEAD)
+#pragma unroll
+    for (int u = 0; u < SCAN_AHEAD; ++u)
+      if (c + u < nc) chunk(c + u, u);
+  barrier();
+  finish(nc - 1, (nc - 1) & 1);
+  if (live) {
 #pragma unroll
     for (int T = 0; T < ND; ++T)
 #pragma unroll
