@@ -100,10 +100,11 @@ struct ShiftArgs {
   const int32_t* positions;
 };
 
-// the row's outputs at p, p + stride, ..: x itself (when first), then the shifted row or its mixes
-template <typename ACT, int V>
+// the row's outputs at p, p + stride, ..: x itself, then the shifted row or its mixes.  NM: their number, the mixes'
+// weights given in registers (0: read as they come)
+template <typename ACT, int V, int NM = 0>
 __device__ __forceinline__ void shift_row(const ShiftArgs& a, const Vec<V>& x, const Vec<V>& xp, const Vec<V>& xpp, bool any,
-                                          const Vec<V>& sh, int W, int c, ACT* p, size_t stride) {
+                                          const Vec<V>& sh, int W, int c, ACT* p, size_t stride, const Vec<V>* mu_r = nullptr) {
   stv<V>(p, x);
   Vec<V> h, hp;
 #pragma unroll
@@ -113,6 +114,16 @@ __device__ __forceinline__ void shift_row(const ShiftArgs& a, const Vec<V>& x, c
   }
   if (!a.mus) {
     stv<V>(p + stride, h);
+    return;
+  }
+  if constexpr (NM > 0) {
+#pragma unroll
+    for (int s = 0; s < NM; ++s) {
+      Vec<V> m;
+#pragma unroll
+      for (int e = 0; e < V; ++e) m.v[e] = h.v[e] + (hp.v[e] - h.v[e]) * mu_r[s].v[e];
+      stv<V>(p + (size_t)(1 + s) * stride, m);
+    }
     return;
   }
   for (int s = 0; s < a.n_mix; ++s) {
@@ -126,13 +137,15 @@ __device__ __forceinline__ void shift_row(const ShiftArgs& a, const Vec<V>& x, c
 
 // prompt rows: ROWS consecutive rows of 256 V channels per workgroup; acts [1 + outputs][T][W]
 constexpr int SM_ROWS = 8;
-template <typename ACT, int V>
+template <typename ACT, int V, int NM>
 __global__ void __launch_bounds__(256) shift_mix_kernel(const float* __restrict__ x, const int32_t* __restrict__ meta,
                                                        ShiftArgs a, int T, int W, ACT* __restrict__ acts) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * V, t0 = blockIdx.x * SM_ROWS;
   if (c >= W) return;
   const Vec<V> sh = ldv<V>(a.shift + c);
-  Vec<V> xp = zerov<V>(), xpp = zerov<V>();
+  Vec<V> xp = zerov<V>(), xpp = zerov<V>(), mu[NM ? NM : 1];
+#pragma unroll
+  for (int s = 0; s < NM; ++s) mu[s] = ldv<V>(a.mus + (size_t)s * W + c);
   for (int t = t0; t < min(t0 + SM_ROWS, T); ++t) {
     const int m = meta[t], lead = m & 3, pos = a.positions[t];
     const size_t row = (size_t)t * W + c;
@@ -142,7 +155,7 @@ __global__ void __launch_bounds__(256) shift_mix_kernel(const float* __restrict_
       xpp = pos < 2 ? zerov<V>() : ldv<V>(lead >= 2 ? x + row - 2 * (size_t)W : st + (size_t)(pos & 1) * W);
     }
     const Vec<V> xt = ldv<V>(x + row);
-    shift_row<ACT, V>(a, xt, xp, xpp, pos >= 1, sh, W, c, acts + row, (size_t)T * W);
+    shift_row<ACT, V, NM>(a, xt, xp, xpp, pos >= 1, sh, W, c, acts + row, (size_t)T * W, mu);
     xpp = xp;
     xp = xt;
   }
@@ -339,7 +352,11 @@ CFC_API int cfc_shift_mix(int f32, const float* x, const int32_t* meta, const in
   const ShiftArgs a{shift, mus, n_mix, prev, positions};
   const int V = W % 4 == 0 ? 4 : 1;
   const dim3 grid((T + SM_ROWS - 1) / SM_ROWS, (W + 256 * V - 1) / (256 * V));
-#define SM(ACT, VV) shift_mix_kernel<ACT, VV><<<grid, 256, 0, stream>>>(x, meta, a, T, W, (ACT*)acts)
+#define SM(ACT, VV)                                                                               \
+  do {                                                                                            \
+    if (n_mix == 5) shift_mix_kernel<ACT, VV, 5><<<grid, 256, 0, stream>>>(x, meta, a, T, W, (ACT*)acts); \
+    else shift_mix_kernel<ACT, VV, 0><<<grid, 256, 0, stream>>>(x, meta, a, T, W, (ACT*)acts);    \
+  } while (0)
   if (f32) { if (V == 4) SM(float, 4); else SM(float, 1); }
   else if (V == 4) SM(uint16_t, 4);
   else SM(uint16_t, 1);

@@ -203,19 +203,32 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatCols kv, int NC, co
     }
     return;
   }
+  // bf16 pairs as one word
+  const bool pairs = sizeof(ACT) == 2 && q.split == 0 && dim % 2 == 0 && q.ld % 2 == 0 && ((uintptr_t)q.p & 3) == 0 &&
+                     qs % 2 == 0 && ((uintptr_t)qr & 3) == 0;
   const int NB = gridDim.y - 1, h0 = H * (blockIdx.y - 1) / NB, h1 = H * blockIdx.y / NB, hp = PQ / 2;
   for (int e = tid; e < (h1 - h0) * hp; e += 256) {
     const int h = h0 + e / hp, i = e % hp;
     float u = 0.f, v = 0.f;
     if (i < r.rot / 2) {
       const int c = h * (dim + r.rot) + dim + 2 * i;
-      u = ldcol<ACT>(q, t, c);
-      v = ldcol<ACT>(q, t, c + 1);
+      if (pairs) {
+        const uint32_t w = *reinterpret_cast<const uint32_t*>(reinterpret_cast<const uint16_t*>(q.p) + t * q.ld + c);
+        u = __uint_as_float(w << 16);
+        v = __uint_as_float(w & 0xffff0000u);
+      } else {
+        u = ldcol<ACT>(q, t, c);
+        v = ldcol<ACT>(q, t, c + 1);
+      }
       rotate(i, u, v);
     }
     ACT* row = qr + ((size_t)t * H + h) * qs + 2 * i;
-    stf(row, u);
-    stf(row + 1, v);
+    if (pairs) {
+      *reinterpret_cast<uint32_t*>(row) = pack2bf(u, v);
+    } else {
+      stf(row, u);
+      stf(row + 1, v);
+    }
   }
   if (qn)
     for (int e = h0 * dim + tid; e < h1 * dim; e += 256)

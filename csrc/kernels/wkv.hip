@@ -36,20 +36,33 @@ struct Cols {
   int64_t ld, plane;
 };
 
+// in two steps, so that other loads can go out between the request and the wait: the first (up to) eight slabs,
+// then their sum and the rest
+template <typename ACT>
+__device__ __forceinline__ void ldc_ask(const Cols& a, int64_t t, int c, float (&v)[8]) {
+  const int64_t o = t * a.ld + c;
+  if (a.split == 0) {
+    v[0] = ld1(reinterpret_cast<const ACT*>(a.p) + o);
+    return;
+  }
+  const float* p = reinterpret_cast<const float*>(a.p) + o;
+#pragma unroll
+  for (int u = 0; u < 8; ++u) v[u] = p[(int64_t)min(u, a.split - 1) * a.plane];
+}
+template <typename ACT>
+__device__ __forceinline__ float ldc_sum(const Cols& a, int64_t t, int c, const float (&v)[8]) {
+  float s = v[0];
+#pragma unroll
+  for (int u = 1; u < 8; ++u) s += u < a.split ? v[u] : 0.f;
+  const float* p = reinterpret_cast<const float*>(a.p) + t * a.ld + c;
+  for (int u = 8; u < a.split; ++u) s += p[(int64_t)u * a.plane];
+  return s;
+}
 template <typename ACT>
 __device__ __forceinline__ float ldc(const Cols& a, int64_t t, int c) {
-  const int64_t o = t * a.ld + c;
-  if (a.split == 0) return ld1(reinterpret_cast<const ACT*>(a.p) + o);
-  const float* p = reinterpret_cast<const float*>(a.p) + o;
-  float s = 0.f;
-  for (int i0 = 0; i0 < a.split; i0 += 8) {
-    float v[8];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) v[u] = p[(int64_t)min(i0 + u, a.split - 1) * a.plane];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) s += i0 + u < a.split ? v[u] : 0.f;
-  }
-  return s;
+  float v[8];
+  ldc_ask<ACT>(a, t, c, v);
+  return ldc_sum<ACT>(a, t, c, v);
 }
 
 // out [T][3][RP]: high, middle and low bf16 parts of tanh(w1); columns past R zero
@@ -246,7 +259,7 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
                                                              float* __restrict__ state, ACT* __restrict__ out, int64_t ldo) {
   using Rec = ChunkRec<ND>;
   constexpr int NV4 = Rec::SIZE / 4, NT = 64 * ND, NLD = (NV4 + NT - 1) / NT;
-  __shared__ __attribute__((aligned(16))) float buf[2][Rec::SIZE];
+  __shared__ __attribute__((aligned(16))) float buf[2][NLD * NT * 4];   // the last piece past the record: not read
   __shared__ __attribute__((aligned(16))) float red[2][ND][16];
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, q = lane >> 4;
   const int h = blockIdx.x, s = blockIdx.y;
@@ -269,7 +282,7 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
   const float nw = norm[hv];
   typedef float f4_t __attribute__((ext_vector_type(4)));      // arrays of these stay in registers
   f4_t rr[SCAN_AHEAD][NLD];
-  float rv[SCAN_AHEAD][4], rg[SCAN_AHEAD][4];
+  ACT rv[SCAN_AHEAD][4], rg[SCAN_AHEAD][4];         // as loaded: a conversion would wait for them
   const ACT* vp = reinterpret_cast<const ACT*>(v.p) + hv;
   const ACT* gp = reinterpret_cast<const ACT*>(g.p) + hv;
   // chunk c (past the last: re-read, not used)
@@ -281,20 +294,24 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int64_t t = row0 + min(CT * c + 4 * q + i, len - 1);
-      rv[u][i] = ld1(vp + t * v.ld);
-      rg[u][i] = ld1(gp + t * g.ld);
+      rv[u][i] = vp[t * v.ld];
+      rg[u][i] = gp[t * g.ld];
     }
   };
   auto store = [&](int b, int u) {
 #pragma unroll
-    for (int i = 0; i < NLD; ++i)
-      if (NT * (i + 1) <= NV4 || tid + NT * i < NV4) reinterpret_cast<f4_t*>(buf[b])[tid + NT * i] = rr[u][i];
+    for (int i = 0; i < NLD; ++i) reinterpret_cast<f4_t*>(buf[b])[tid + NT * i] = rr[u][i];
   };
   auto barrier = [] {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
     __builtin_amdgcn_s_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
   };
+  const uintptr_t ob = (uintptr_t)(out + (int64_t)row0 * ldo);
+  // unsigned halves: readfirstlane returns int, whose sign would run into the upper half
+  const uint32_t ob_lo = __builtin_amdgcn_readfirstlane((uint32_t)ob), ob_hi = __builtin_amdgcn_readfirstlane((uint32_t)(ob >> 32));
+  const __amdgpu_buffer_rsrc_t ors = __builtin_amdgcn_make_buffer_rsrc((void*)(((uintptr_t)ob_hi << 32) | ob_lo), (short)0,
+                                                                       0x7fffffe0, 0x00020000);
   f32x4_t o_prev{0.f, 0.f, 0.f, 0.f};
   float g_prev[4] = {0.f, 0.f, 0.f, 0.f};
   // outputs of chunk c from the mean squares in red[b]
@@ -309,7 +326,10 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
     for (int i = 0; i < 4; ++i) {
       const int t = CT * c + 4 * q + i;
       const float y = o_prev[i] * (1.f / sqrtf(sv[i] / (float)D + eps)) * nw * (g_prev[i] / (1.f + __expf(-g_prev[i])));
-      if (live && t < len) st1(out + (int64_t)(row0 + t) * ldo + hv, y);
+      // without a branch (a join would wait for every load in flight): offsets past the range store nothing
+      const int off = live && t >= 0 && t < len ? (int)((t * ldo + hv) * (int64_t)sizeof(ACT)) : 0x7ffffff0;
+      if constexpr (sizeof(ACT) == 2) __builtin_amdgcn_raw_buffer_store_b16((short)f2bf(y), ors, off, 0, 0);
+      else __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(y), ors, off, 0, 0);
     }
   };
 #pragma unroll
@@ -319,12 +339,13 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
   auto chunk = [&](int c, int u) {
     barrier();
     const int b = u & 1;
-    if (c > 0) finish(c - 1, b ^ 1);
+    finish(c - 1, b ^ 1);
+    const float keep = c < nc ? 0.f : 1.f;        // past the last chunk: the state stays as it is
     float vv[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      vv[i] = live && CT * c + 4 * q + i < len ? rv[u][i] : 0.f;
-      g_prev[i] = rg[u][i];
+      vv[i] = live && CT * c + 4 * q + i < len ? ld1(&rv[u][i]) : 0.f;
+      g_prev[i] = ld1(&rg[u][i]);
     }
     load(c + SCAN_AHEAD, u);
     const float4* p = reinterpret_cast<const float4*>(buf[b]);
@@ -345,7 +366,8 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
     float4 k[ND];
 #pragma unroll
     for (int T = 0; T < ND; ++T) {
-      const float4 d = p[Rec::DEC / 4 + 4 * T + q];
+      float4 d = p[Rec::DEC / 4 + 4 * T + q];       // decays are at most 1
+      d = make_float4(fmaxf(d.x, keep), fmaxf(d.y, keep), fmaxf(d.z, keep), fmaxf(d.w, keep));
       k[T] = p[Rec::K / 4 + T * 64 + lane];
       S[T][0] *= d.x; S[T][1] *= d.y; S[T][2] *= d.z; S[T][3] *= d.w;
     }
@@ -371,10 +393,10 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
   };
   for (int c = 0; c < nc; c += SCAN_AHEAD)
 #pragma unroll
-    for (int u = 0; u < SCAN_AHEAD; ++u)
-      if (c + u < nc) chunk(c + u, u);
+    for (int u = 0; u < SCAN_AHEAD; ++u) chunk(c + u, u);
+  const int last = (nc + SCAN_AHEAD - 1) / SCAN_AHEAD * SCAN_AHEAD - 1;
   barrier();
-  finish(nc - 1, (nc - 1) & 1);
+  finish(last, last & 1);
   if (live) {
 #pragma unroll
     for (int T = 0; T < ND; ++T)
@@ -432,30 +454,50 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
         }
       }
     };
-    ldS(0);
     const int64_t row = q0 + t;
-    for (int e = tid; e < 4 * D; e += WS_T) {
-      const int c = e % D;
+    auto pick = [&](int e) {
+      Cols s = r;
       const int w = e / D;
-      const Cols& src = w == 0 ? r : w == 1 ? k : w == 2 ? v : g;
-      rs[e] = ldc<ACT>(src, row, hc + c);
-    }
-    for (int c = tid; c < RP; c += WS_T) th[c] = c < R ? tanhf(ldc<ACT>(w1, row, c)) : 0.f;
+      s.p = w == 0 ? r.p : w == 1 ? k.p : w == 2 ? v.p : g.p;
+      return s;
+    };
+    // the small operands are asked for ahead of the state: loads return in order
+    float ask[8], ask1[8];
+    const int e0 = min(tid, 4 * D - 1), z0 = min(tid, R - 1), wc = min(tid >> 2, D - 1);
+    uint4 wq[2];
+    ldc_ask<ACT>(pick(e0), row, hc + e0 % D, ask);
+    ldc_ask<ACT>(w1, row, z0, ask1);
+#pragma unroll
+    for (int y = 0; y < 2; ++y)
+      wq[y] = *reinterpret_cast<const uint4*>(w2 + (size_t)(hc + wc) * RP + min(8 * (tid & 3) + 32 * y, RP - 8));
+    const float w0v = w0[hc + wc];
+    ldS(0);
+    if (tid < 4 * D) rs[tid] = ldc_sum<ACT>(pick(e0), row, hc + e0 % D, ask);
+    if (tid < RP) th[tid] = tid < R ? tanhf(ldc_sum<ACT>(w1, row, z0, ask1)) : 0.f;
+    for (int e = tid + WS_T; e < 4 * D; e += WS_T) rs[e] = ldc<ACT>(pick(e), row, hc + e % D);
+    for (int c = tid + WS_T; c < RP; c += WS_T) th[c] = c < R ? tanhf(ldc<ACT>(w1, row, c)) : 0.f;
     __syncthreads();
     // four threads per channel over the low rank
     for (int c0 = 0; c0 < D; c0 += WS_T / 4) {
       const int c = c0 + (tid >> 2), p = tid & 3;
       float z = 0.f;
-      if (c < D)
-        for (int x = 8 * p; x < RP; x += 32) {
-          float wv[8];
-          unpack8(*reinterpret_cast<const uint4*>(w2 + (size_t)(hc + c) * RP + x), wv);
+      auto dot = [&](const uint4& w, int x) {
+        float wv[8];
+        unpack8(w, wv);
 #pragma unroll
-          for (int e = 0; e < 8; ++e) z += wv[e] * th[x + e];
+        for (int e = 0; e < 8; ++e) z += wv[e] * th[x + e];
+      };
+      if (c < D) {
+        if (c0 == 0) {
+          dot(wq[0], 8 * p);
+          if (RP > 32) dot(wq[1], 8 * p + 32);
         }
+        for (int x = 8 * p + (c0 == 0 ? 64 : 0); x < RP; x += 32)
+          dot(*reinterpret_cast<const uint4*>(w2 + (size_t)(hc + c) * RP + x), x);
+      }
       z += __shfl_xor(z, 1, 64);
       z += __shfl_xor(z, 2, 64);
-      if (c < D && p == 0) ws[c] = expf(log_decay(z + w0[hc + c]));
+      if (c < D && p == 0) ws[c] = expf(log_decay(z + (c0 == 0 ? w0v : w0[hc + c])));
     }
     float bonus = 0.f;
     for (int c = tid; c < D; c += WS_T) bonus += u[hc + c] * rs[c] * kk[c];
@@ -555,6 +597,8 @@ CFC_API int cfc_wkv_chunked(int f32, const void* r, int64_t ldr, const void* k, 
                             const int32_t* ctx_lens, float* rec, float* state, void* out, int64_t ldo, hipStream_t stream) {
   if (n_seq <= 0 || n_chunks <= 0) return 0;
   if (H < 1 || D < 1 || D > WKV_MAX_CHUNKED || RP < 32 || RP % 32 || n_seq > 65535) return -1;
+  // 32-bit store offsets within a portion
+  if ((int64_t)n_chunks * CT * ldo * (f32 ? 4 : 2) >= 0x7fffffe0ll) return -4;
   const Cols cr{r, 0, ldr, 0}, ck{k, 0, ldk, 0}, cv{v, 0, ldv, 0}, cg{g, 0, ldg, 0};
   const ScanSeq sq{chunk_cu, chunks, slots, cu_q, ctx_lens};
 #define WC(ACT, ND)                                                                                                      \

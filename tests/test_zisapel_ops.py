@@ -1,0 +1,444 @@
+"""Each mechanism of the Zisapel decoder alone, against the plain implementation."""
+import math
+
+import numpy as np
+import pytest
+import torch
+
+import zisapel_oracle as oracle
+from copilot_for_consensus_amd.models.projection import JointProjection
+from copilot_for_consensus_amd.ops import gated as G
+from copilot_for_consensus_amd.ops import latent as L
+from copilot_for_consensus_amd.ops import moe as M
+from copilot_for_consensus_amd.ops import wkv as R
+from copilot_for_consensus_amd.ops.cols import Cols
+from copilot_for_consensus_amd.ops.reference import moe_rows, row_meta
+
+DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+DTYPES = [torch.float32, torch.bfloat16]
+
+
+def rnd(*shape, seed=0, scale=1.0):
+    return scale * torch.randn(*shape, generator=torch.Generator().manual_seed(seed + 31 * len(shape) + sum(shape)))
+
+
+def close(got, want, tol):
+    got, want = got.float().cpu(), want.float()
+    assert torch.isfinite(got).all()
+    assert float((got - want).abs().max()) <= tol * max(1.0, float(want.abs().max())), float((got - want).abs().max())
+
+
+def tol(dtype):
+    return 2e-5 if dtype == torch.float32 else 1.2e-2
+
+
+def i32(x, device="cpu"):
+    return torch.tensor(np.asarray(x), dtype=torch.int32, device=device)
+
+
+def slabs(x, n, seed=7):
+    """fp32 parts whose sum is x."""
+    parts = rnd(n, *x.shape, seed=seed)
+    parts[-1] = x - parts[:-1].sum(0)
+    return parts
+
+
+# ------------------------------------------------------------------ token shift, gated branches
+PORTIONS = [(1, 0), (5, 0), (2, 1), (9, 2), (3, 7), (17, 30), (1, 40)]      # rows, first position
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W,mixes", [(104, 5), (65, 0), (1500, 1), (260, 5)])
+def test_shift_and_mixes(device, dtype, W, mixes):
+    shift, mus = rnd(W, seed=1), rnd(mixes, W, seed=2) if mixes else None
+    n = len(PORTIONS)
+    prev = rnd(n + 2, 2, W, seed=9)                       # stale rows everywhere
+    xs, rows, want = [], [], []
+    for s, (k, pos) in enumerate(PORTIONS):
+        seq = rnd(pos + k, W, seed=20 + s)
+        for p in (pos - 1, pos - 2):
+            if p >= 0:
+                prev[n - s, p % 2] = seq[p]
+        h = oracle.mix(seq, shift)
+        outs = [seq, h] if mus is None else [seq] + [oracle.mix(h, mu) for mu in mus]
+        want.append(torch.stack(outs)[:, pos:])
+        xs.append(seq[pos:])
+        rows.append((k, n - s))
+    want, x = torch.cat(want, 1), torch.cat(xs).to(device)
+    pos = i32([p + r for k, p in PORTIONS for r in range(k)], device)
+    sh = G.Shift(shift.to(device), mus.to(device) if mixes else None, prev.to(device))
+    acts = sh.acts(x.shape[0], dtype)
+    G.shift_mix(x, sh, torch.from_numpy(row_meta(rows)).to(device), pos, acts)
+    close(acts, want, tol(dtype))
+    # the same rows decoded one per sequence: only the portions of one row
+    one = [i for i, (k, _) in enumerate(PORTIONS) if k == 1]
+    at = [sum(k for k, _ in PORTIONS[:i]) for i in one]
+    xd, a1 = x[at].clone(), sh.acts(len(one), dtype)
+    G.gated_shift(xd, None, dtype, None, sh, pos[at].contiguous(), i32([n - i for i in one], device), a1)
+    close(a1, want[:, at], tol(dtype))
+    for i, t in zip(one, at):
+        close(sh.prev[n - i, int(pos[t]) % 2], want[0, t], 1e-6)          # the state moved on
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W,T,split,top", [(104, 5, 1, 0), (65, 3, 3, 2), (1500, 4, 9, 3), (5000, 2, 1, 1)])
+@pytest.mark.parametrize("slab_gate", [False, True])
+def test_gated_branch(device, dtype, W, T, split, top, slab_gate):
+    x, y, z, b, w, eps = rnd(T, W), rnd(T, W, seed=1), rnd(T, W + 8, seed=2), rnd(W, seed=3), rnd(W, seed=4), 1e-3
+    gate = z[:, 4:4 + W] if slab_gate else z[:, :W].to(dtype).float()
+    total, routed = y.clone(), None
+    if top:
+        rows, pos, wt = rnd(3 * T, W, seed=5).to(dtype), torch.randint(0, 3 * T, (T, top), generator=torch.Generator().manual_seed(0)), rnd(T, top, seed=6)
+        total = total + (rows.float()[pos] * wt[..., None]).sum(1)
+        routed = (rows.to(device), i32(pos, device), wt.to(device))
+    want = x + oracle.layer_norm(total * torch.sigmoid(gate + b), w, eps)
+    d = lambda t: t.to(device).contiguous()
+    cols = Cols(d(slabs(z, 2)), 4, W) if slab_gate else Cols(d(z[:, :W].to(dtype)))
+    br = G.Branch(cols, d(b), d(w), eps, y=d(slabs(y, split)), routed=routed)
+    prev, meta, pos = torch.zeros(3, 2, W, device=device), torch.from_numpy(row_meta([(T, 2)])).to(device), i32(range(10, 10 + T), device)
+    xg, h = d(x).clone(), torch.empty(T, W, dtype=dtype, device=device)
+    G.gated_norm(xg, br, dtype, h, prev, meta, pos)
+    close(xg, want, 3e-5)
+    close(h, want, tol(dtype))
+    for t in (T - 2, T - 1):
+        assert torch.equal(prev[2, (10 + t) % 2].cpu(), x[t])
+    assert not prev[:2].any()
+    xg = d(x).clone()
+    br.y2, br.y = br.y, None
+    G.gated_shift(xg, br, dtype, h)
+    close(xg, want, 3e-5)
+    close(h, want, tol(dtype))
+    close(G.final_norm(xg, d(w), eps, dtype, i32([T - 1, 0], device)), oracle.layer_norm(want, w, eps)[[T - 1, 0]], tol(dtype))
+    close(G.final_norm(xg, d(w), eps, dtype), oracle.layer_norm(want, w, eps), tol(dtype))
+
+
+# ------------------------------------------------------------------ recurrence
+def wkv_case(H, D, rank, T, seed, w0=-1.0, spread=1.5):
+    p = {"w2": rnd(H * D, rank, seed=seed, scale=0.6 / rank ** 0.5).to(torch.bfloat16), "w0": rnd(H * D, seed=seed + 1, scale=spread) + w0,
+         "u": rnd(H, D, seed=seed + 2), "norm": rnd(H * D, seed=seed + 3)}
+    x = {k: rnd(T, H * D, seed=seed + 10 + j) for j, k in enumerate("rkvg")}
+    return p, x, rnd(T, rank, seed=seed + 20)
+
+
+def wkv_want(p, x, w1, H, D, eps):
+    T = w1.shape[0]
+    w = torch.exp(-torch.exp(torch.tanh(w1.double()) @ p["w2"].double().T + p["w0"].double()))
+    r, k, v = (x[c].double().view(T, H, D) for c in "rkv")
+    o = oracle.rms(oracle.wkv_recurrence(r, k, v, w.view(T, H, D), p["u"].double()), eps).reshape(T, H * D)
+    g = x["g"].double()
+    return (o * p["norm"].double() * g * torch.sigmoid(g)).float()
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,D,rank", [(2, 64, 24), (3, 24, 1), (1, 17, 33), (2, 48, 70), (5, 16, 8), (2, 96, 16), (3, 72, 5), (1, 128, 64),
+                                      (2, 160, 12), (1, 9, 3)])
+def test_recurrence_in_portions_and_decoded(device, dtype, H, D, rank):
+    """Whole, in portions down to one token that carry the state, and token by token: other slots untouched."""
+    T, eps = 71, 1e-4
+    p, x, w1 = wkv_case(H, D, rank, T, seed=H + D)
+    x = {k: v.to(dtype).float() for k, v in x.items()}
+    want = wkv_want(p, x, w1, H, D, eps)
+    d = lambda t: t.to(device).contiguous()
+    mix = R.Wkv(H, D, rank, d(p["w2"]), d(p["w0"]), d(p["u"]), d(p["norm"]), eps)
+    for cuts in ([T], [16, 32, 23], [1, 2, 15, 17, 31, 3, 2], [1] * T):
+        state = torch.full((4, H, D, D), 7.0, device=device)
+        out = torch.empty(T, H * D, dtype=dtype, device=device)
+        a = 0
+        for n in cuts:
+            ops = [Cols(d(x[k][a:a + n].to(dtype))) for k in "rkvg"]
+            cu, ctx = [0, n], i32([a + n], device)
+            ch, ccu = R.chunk_plan(cu)
+            if len(cuts) == T:
+                s = d(slabs(torch.cat([x[k][a:a + n] for k in "rkvg"], 1), 3))
+                R.step(mix, *(Cols(s, j * H * D, H * D) for j in range(4)), Cols(d(slabs(w1[a:a + n], 2))), i32([2], device), ctx, state,
+                       out[a:a + n])
+            else:
+                R.prefill(mix, *ops, Cols(d(slabs(w1[a:a + n], 2))), i32([2], device), i32(cu, device), ctx, d(torch.from_numpy(ch)),
+                          d(torch.from_numpy(ccu)), state, out[a:a + n])
+            a += n
+        close(out, want, tol(dtype))
+        assert (state[[0, 1, 3]] == 7.0).all()
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("w0,spread", [(-9.0, 0.1), (3.0, 0.5), (0.0, 6.0)])
+def test_recurrence_from_no_decay_to_immediate(device, w0, spread):
+    """Decays next to one, decays of exp(-20) a token, and both side by side: nothing over- or underflows."""
+    H, D, T, eps = 2, 64, 150, 1e-5
+    p, x, w1 = wkv_case(H, D, 12, T, seed=3, w0=w0, spread=spread)
+    d = lambda t: t.to(device).contiguous()
+    mix = R.Wkv(H, D, 12, d(p["w2"]), d(p["w0"]), d(p["u"]), d(p["norm"]), eps)
+    out, state = torch.empty(T, H * D, device=device), torch.zeros(1, H, D, D, device=device)
+    ch, ccu = R.chunk_plan([0, T])
+    R.prefill(mix, *(Cols(d(x[k])) for k in "rkvg"), Cols(d(w1)[None]), i32([0], device), i32([0, T], device), i32([T], device),
+              d(torch.from_numpy(ch)), d(torch.from_numpy(ccu)), state, out)
+    close(out, wkv_want(p, x, w1, H, D, eps), 3e-5)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_recurrence_of_a_packed_batch(device):
+    """Several sequences in one pass, fresh and continued, from one row to many chunks."""
+    H, D, rank, eps = 2, 32, 6, 1e-4
+    lens, old = [40, 1, 16, 33, 2], [0, 5, 17, 0, 1]
+    d = lambda t: t.to(device).contiguous()
+    cases = [wkv_case(H, D, rank, a + b, seed=60)[:1] + wkv_case(H, D, rank, a + b, seed=60 + 7 * i)[1:] for i, (a, b) in enumerate(zip(old, lens))]
+    p = cases[0][0]
+    mix = R.Wkv(H, D, rank, d(p["w2"]), d(p["w0"]), d(p["u"]), d(p["norm"]), eps)
+    state = torch.full((6, H, D, D), 3.0, device=device)
+
+    def go(parts, ctx, slots):
+        cu = np.concatenate([[0], np.cumsum([b - a for _, a, b in parts])]).tolist()
+        ch, ccu = R.chunk_plan(cu)
+        cat = {k: torch.cat([cases[i][1][k][a:b] for i, a, b in parts]) for k in "rkvg"}
+        out = torch.empty(cu[-1], H * D, device=device)
+        R.prefill(mix, *(Cols(d(cat[k])) for k in "rkvg"), Cols(d(torch.cat([cases[i][2][a:b] for i, a, b in parts]))[None]),
+                  i32(slots, device), i32(cu, device), i32(ctx, device), d(torch.from_numpy(ch)), d(torch.from_numpy(ccu)), state, out)
+        return out
+    first = [(i, 0, o) for i, o in enumerate(old) if o]
+    go(first, [o for _, _, o in first], [5 - i for i, _, _ in first])
+    out = go([(i, o, o + n) for i, (o, n) in enumerate(zip(old, lens))], [o + n for o, n in zip(old, lens)], [5 - i for i in range(5)])
+    at = 0
+    for i, (o, n) in enumerate(zip(old, lens)):
+        close(out[at:at + n], wkv_want(p, cases[i][1], cases[i][2], H, D, eps)[o:], 2e-5)
+        at += n
+
+
+# ------------------------------------------------------------------ latent attention
+SCALING = {"factor": 4.0, "original": 64, "fast": 8.0, "slow": 1.0}
+
+
+@pytest.mark.parametrize("dims,base,scaling", [(16, 10000.0, SCALING), (16, 10000.0, None), (2, 50.0, SCALING), (64, 500.0, dict(SCALING, factor=1.0)),
+                                               (24, 1e6, dict(SCALING, original=4096, fast=32.0))])
+def test_rotary_frequencies(dims, base, scaling):
+    r = L.yarn_rope(dims, base, scaling, "cpu")
+    cos, sin = oracle.yarn_angles(300, {"dims": dims, "base": base, "scaling": scaling}, torch.float64)
+    a = torch.arange(300, dtype=torch.float64)[:, None] * r.freq.double()
+    close(a.cos() * r.mag, cos, 1e-4)
+    close(a.sin() * r.mag, sin, 1e-4)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,dim,rot,rank,vdim", [(3, 20, 12, 44, 28), (1, 8, 2, 20, 10), (4, 128, 64, 512, 128), (2, 32, 16, 1100, 16)])
+@pytest.mark.parametrize("split", [0, 1, 11])
+def test_latent_and_rotary_rows(device, dtype, H, dim, rot, rank, vdim, split):
+    T, eps = 6, 1e-3
+    kv, q, g, w = rnd(T, rank + rot), rnd(T, H * (dim + rot), seed=1), rnd(T, H * vdim, seed=2), rnd(rank, seed=3)
+    if not split:
+        kv, q, g = (t.to(dtype).float() for t in (kv, q, g))
+    d = lambda t: t.to(device).contiguous()
+    rope = L.yarn_rope(rot, 300.0, SCALING, device)
+    rv, pad = L.padded_rank(rank), L.padded_rank(rot)
+    cache = torch.zeros(4, 32, rv + pad, dtype=dtype, device=device)
+    slots, pos = i32([3, 40, 41, 100, 7, 64], device), i32([0, 1, 500, 31, 32, 9000], device)
+    ql = torch.full((T, H, rv + pad), 5.0, dtype=dtype, device=device)
+    c = [Cols(d(slabs(t, split))) if split else Cols(d(t.to(dtype))) for t in (kv, q, g)]
+    qn, gate = L.latent_rope(c[0], rank, d(w), eps, slots, cache, c[1], H, dim, rope, pos, ql[:, :, rv:], vdim, c[2])
+    a = pos.cpu().double()[:, None] * rope.freq.cpu().double()
+    cos, sin = (a.cos() * rope.mag).float(), (a.sin() * rope.mag).float()
+    rows = cache.view(-1, rv + pad)[slots.long()]
+    # positions in the thousands: one fp32 ulp of the angle
+    t = max(tol(dtype), 6e-4)
+    close(rows[:, :rank], oracle.rms(kv[:, :rank], eps) * w, tol(dtype))
+    close(rows[:, rv:rv + rot], oracle.rotate_pairs(kv[:, rank:], cos, sin), t)
+    assert not rows[:, rank:rv].any() and not rows[:, rv + rot:].any()
+    qv = q.view(T, H, dim + rot)
+    close(qn, qv[:, :, :dim], tol(dtype))
+    close(ql[:, :, rv:rv + rot], oracle.rotate_pairs(qv[:, :, dim:], cos, sin), t)
+    assert not ql[:, :, rv + rot:].any() and (ql[:, :, :rv] == 5.0).all()
+    close(gate, g, tol(dtype))
+
+
+class Pages:
+    """Block tables of several sequences over a shuffled pool, rows written position by position."""
+
+    def __init__(self, rows, device, dtype, seed=0):
+        n = [max(1, -(-r.shape[0] // 32)) for r in rows]
+        ids = torch.randperm(sum(n) + 3, generator=torch.Generator().manual_seed(seed)).tolist()
+        bt = np.zeros((len(rows), max(n)), np.int32)
+        cache = torch.full((sum(n) + 3, 32, rows[0].shape[1]), 3.0)          # stale values in unused places
+        for s, r in enumerate(rows):
+            for b in range(n[s]):
+                bt[s, b] = ids.pop()
+                part = r[32 * b:32 * b + 32]
+                cache[bt[s, b], :part.shape[0]] = part
+        self.tables, self.cache = i32(bt, device), cache.to(dtype).to(device)
+
+
+def window_case(H, rv, rot, ctxs, news, seed=0, peak=None):
+    rows = [rnd(c, rv + L.padded_rank(rot), seed=seed + 5 * i) for i, c in enumerate(ctxs)]
+    q = [rnd(n, H, rv + L.padded_rank(rot), seed=seed + 100 + i) for i, n in enumerate(news)]
+    if peak is not None:                       # the last row's query points at one key
+        for r, x in zip(rows, q):
+            x[-1, :] = 4.0 * r[max(0, r.shape[0] - 1 - peak)]
+    return rows, q
+
+
+def window_want(rows, q, scale, window, sink, rv):
+    out = []
+    for r, x in zip(rows, q):
+        c, n = r.shape[0], x.shape[0]
+        see = oracle.window_mask(c, window if window else c + 1)[c - n:]
+        o = torch.zeros(n, x.shape[1], rv)
+        for h in range(x.shape[1]):
+            s = (x[:, h] @ r.T * scale).masked_fill(~see, -math.inf)
+            p = oracle.softmax_with_sink(s, sink[h]) if sink is not None else torch.softmax(s, -1)
+            o[:, h] = p @ r[:, :rv]
+        out.append(o)
+    return torch.cat(out)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,rv,rot", [(3, 64, 12), (8, 128, 16), (5, 192, 64), (2, 512, 64), (1, 96, 8), (4, 320, 32), (2, 640, 16)])
+@pytest.mark.parametrize("window", [0, 1, 33, 72, 200])
+def test_window_attention_with_sinks(device, dtype, H, rv, rot, window):
+    ctxs, news = [300, 1, 64, 97, 65], [37, 1, 2, 1, 65]
+    sink, scale = rnd(H, seed=3) + 1.0, 1.5 / (rv + rot) ** 0.5
+    for peak in (None, 0, max(0, window - 1), window):
+        rows, q = window_case(H, rv, rot, ctxs, news, peak=peak)
+        rows, q = [r.to(dtype).float() for r in rows], [x.to(dtype).float() for x in q]
+        pg = Pages(rows, device, dtype)
+        cu = np.concatenate([[0], np.cumsum(news)]).tolist()
+        for sk in (None, sink):
+            got = L.latent_attention(torch.cat(q).to(dtype).to(device), pg.cache, pg.tables, i32(cu, device), i32(ctxs, device), scale,
+                                     P=1 if peak is None else 3, window=window, sink=sk.to(device) if sk is not None else None, RV=rv)
+            close(got, window_want(rows, q, scale, window, sk, rv), tol(dtype))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("P", [1, 4, 9])
+def test_window_attention_decoded(device, dtype, P):
+    H, rv, rot, window = 6, 128, 32, 100
+    ctxs = [1, 100, 101, 165, 500, 32]
+    rows, q = window_case(H, rv, rot, ctxs, [1] * 6, peak=window - 1)
+    rows, q = [r.to(dtype).float() for r in rows], [x.to(dtype).float() for x in q]
+    pg, sink = Pages(rows, device, dtype), rnd(H, seed=4)
+    got = L.latent_attention(torch.cat(q).to(dtype).to(device), pg.cache, pg.tables, None, i32(ctxs, device), 0.09, P=P, window=window,
+                             sink=sink.to(device), RV=rv)
+    close(got, window_want(rows, q, 0.09, window, sink, rv), tol(dtype))
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("window", [0, 1, 64, 150, 1000])
+@pytest.mark.parametrize("rot", [64, 32])
+def test_expanded_window_attention(window, rot):
+    """Per-head keys and values of 128 with the shared rotated part, window, sinks and output gate."""
+    H, D, rank, dt, scale = 3, 128, 128, torch.bfloat16, 0.1
+    ctxs, news = [600, 64, 333, 5], [600, 1, 70, 5]
+    rp = L.padded_rank(rot)
+    lat = [rnd(c, rank + rp, seed=i).to(dt) for i, c in enumerate(ctxs)]
+    uk, uv = rnd(H * D, rank, seed=8, scale=0.1).to(dt), rnd(H * D, rank, seed=9, scale=0.1).to(dt)
+    T = sum(news)
+    qn, q2, gate, sink = rnd(T, H * (D + rot), seed=10).to(dt), rnd(T, H, 64, seed=11).to(dt), rnd(T, H * D, seed=12).to(dt), rnd(H, seed=13)
+    q2[:, :, rp:] = 0
+    cu = np.concatenate([[0], np.cumsum(news)]).tolist()
+    want, at = torch.empty(T, H * D), 0
+    for r, c, n in zip(lat, ctxs, news):
+        rf = r.float()
+        k, v = (rf[:, :rank] @ uk.float().T).view(c, H, D), (rf[:, :rank] @ uv.float().T).view(c, H, D)
+        see = oracle.window_mask(c, window or c + 1)[c - n:]
+        for h in range(H):
+            s = (qn[at:at + n].float().view(n, H, -1)[:, h, :D] @ k[:, h].T + q2[at:at + n, h, :rp].float() @ rf[:, rank:].T) * scale
+            p = oracle.softmax_with_sink(s.masked_fill(~see, -math.inf), sink[h])
+            want[at:at + n, h * D:(h + 1) * D] = p @ v[:, h]
+        at += n
+    want = want * torch.sigmoid(gate.float())
+    from copilot_for_consensus_amd.ops import kernels as K
+    dev = "cuda"
+    pg = Pages([r.float() for r in lat], dev, dt)
+    starts = [max(0, c - n - window + 1) if window else 0 for c, n in zip(ctxs, news)]
+    gt, base = L.gather_tiles(ctxs, starts)
+    ctx = i32(ctxs, dev)
+    k, vt, k2 = L.expand(pg.cache, pg.tables, ctx, i32(gt, dev), K.pack_dgemm_weight(uk.to(dev)), uv.to(dev), rank)
+    out = torch.empty(T, H * D, dtype=dt, device=dev)
+    L.expanded_window_attention(Cols(qn.to(dev)), q2.to(dev), k, k2, vt, i32(base, dev), i32(cu, dev), ctx, scale,
+                                [i32(t, dev) for t in K.prefill_tiles(cu, 256, ctxs)], window, sink.to(dev), gate.to(dev), out)
+    close(out, want, 2e-2)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T", [1, 7, 40, 300])
+@pytest.mark.parametrize("H,N,K", [(3, 28, 44), (4, 64, 128), (2, 128, 512), (1, 10, 20)])
+def test_gated_head_products(device, dtype, T, H, N, K):
+    x, w, g = rnd(T, H, K).to(dtype).float(), rnd(H, N, K, seed=1, scale=K ** -0.5).to(dtype).float(), rnd(T, H * N, seed=2).to(dtype).float()
+    want = torch.einsum("thk,hnk->thn", x, w) * torch.sigmoid(g).view(T, H, N)
+    out = torch.empty(T, H, N, dtype=dtype, device=device)
+    L.head_linear(x.to(dtype).to(device), L.HeadWeight(w.to(dtype).to(device)), out, g.to(dtype).to(device))
+    close(out, want, tol(dtype))
+
+
+# ------------------------------------------------------------------ routed experts
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("E,top,groups,keep,split", [(12, 3, 4, 2, 1), (4, 1, 1, 1, 3), (64, 8, 8, 4, 17), (6, 2, 3, 3, 1), (130, 5, 10, 3, 2),
+                                                     (8, 4, 8, 4, 1), (300, 6, 1, 1, 1)])
+def test_routing(device, E, top, groups, keep, split):
+    T = 33
+    z, corr = rnd(T, E, scale=2.0), rnd(E, seed=1, scale=0.6) - 1.0          # choice scores mostly below zero
+    r = {"experts": E, "top": top, "groups": {"count": groups, "keep": keep}, "scale": 1.7}
+    ids, wts = _route_oracle(z, corr, r)
+    pad = torch.cat([z, torch.full((T, 5), 9.0)], 1)                         # columns past the experts are not theirs
+    got = M.route(Cols(slabs(pad, split).to(device), 0, E), M.Router(E, top, groups, keep, 1.7, corr.to(device)))
+    for t in range(T):
+        have = dict(zip(got[0][t].tolist(), got[1][t].tolist()))
+        assert sorted(have) == sorted(ids[t]), t
+        for e, w in zip(ids[t], wts[t].tolist()):
+            assert abs(have[e] - w) < 1e-5
+
+
+def _route_oracle(z, corr, r):
+    """The plain router fed logits: h = z through an identity."""
+    return oracle.route(z, {"router": torch.eye(z.shape[1]), "correction": corr}, r)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("T,top,E,tile", [(1, 2, 8, 32), (50, 3, 6, 32), (700, 4, 16, 64), (5, 1, 40, 64), (1500, 2, 3, 256)])
+def test_rows_sorted_by_expert(device, T, top, E, tile):
+    ids = torch.randint(0, E, (T, top), generator=torch.Generator().manual_seed(T), dtype=torch.int32)
+    ids[:, 0] = min(1, E - 1)                                                # one crowded, some empty
+    want = moe_rows(ids, E, tile)
+    for g, w in zip(M.sort_rows(ids.to(device), E, tile), want):
+        assert np.array_equal(g.cpu().numpy(), w)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,W,F,E,top", [(1, 104, 20, 6, 2), (37, 65, 31, 5, 3), (9, 128, 72, 8, 2), (300, 192, 64, 4, 2), (700, 64, 128, 4, 3)])
+def test_expert_products(device, dtype, T, W, F, E, top):
+    x = rnd(T, W).to(dtype)
+    g, u, dn = (rnd(E, *s, seed=i, scale=s[1] ** -0.5).to(dtype) for i, s in enumerate(((F, W), (F, W), (W, F))))
+    ids = torch.randint(0, E, (T, top), generator=torch.Generator().manual_seed(3), dtype=torch.int32)
+    rows, pos = M.experts(x.to(device), M.ExpertWeights(g.to(device), u.to(device), dn.to(device)), ids.to(device))
+    got = rows.float().cpu()[pos.cpu().long()]
+    want = torch.empty(T, top, W)
+    for t in range(T):
+        for c in range(top):
+            e = int(ids[t, c])
+            p = {"e.gate": g[e].float(), "e.up": u[e].float(), "e.down": dn[e].float()}
+            want[t, c] = oracle.expert(x[t].float(), p, "e")
+    close(got, want, tol(dtype))
+
+
+# ------------------------------------------------------------------ joint products
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T", [1, 3, 40, 130, 300])
+@pytest.mark.parametrize("K", [104, 192])
+def test_joint_products_of_several_inputs(device, dtype, T, K):
+    sizes, inputs = [K, 256, 72, 10], [0, 2, 2, 1]
+    ws = [rnd(n, K, seed=n, scale=K ** -0.5).to(dtype) for n in sizes]
+    acts = rnd(3, T, K).to(dtype)
+    j = JointProjection([(w.to(device), i) for w, i in zip(ws, inputs)])
+    a = acts.to(device)
+    for got, w, i in zip(j.joint(a), ws, inputs):
+        close(got.t.sum(0)[:, got.c0:got.c0 + got.n], acts[i].float() @ w.float().T, 2e-5 if dtype == torch.float32 else 2e-3)
+    for n in range(4):
+        want = acts[inputs[n]].float() @ ws[n].float().T
+        for c, t in ((j.act(n, a), tol(dtype)), (j.slabs(n, a), 2e-3)):
+            v = c.t.sum(0) if c.slabs else c.t
+            close(v[:, c.c0:c.c0 + c.n], want, t)
