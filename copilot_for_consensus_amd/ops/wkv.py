@@ -90,7 +90,8 @@ def prefill(p: Wkv, r: Cols, k: Cols, v: Cols, g: Cols, w1: Cols, slots, cu_q, c
     """Packed portions, in chunks of 16 tokens (``chunks``, ``chunk_cu`` of :func:`chunk_plan` on the device)."""
     if not out.is_cuda:
         return _ref(p, r, k, v, g, w1, slots, cu_q, ctx_lens, state, out)
-    if p.D > MAX_CHUNKED_DIM or chunks.shape[0] * CHUNK * out.stride(0) * out.element_size() >= 2 ** 31 - 64:
+    widest = max(out.stride(0), v.t.stride(-2), g.t.stride(-2)) * out.element_size()
+    if p.D > MAX_CHUNKED_DIM or (chunks.shape[0] + 4) * CHUNK * widest >= 2 ** 31 - 256:
         return step(p, r, k, v, g, w1, slots, ctx_lens, state, out, cu_q)
     T, RP, lib = out.shape[0], p.w2.shape[1], kernels()
     a = [c.args(out.dtype) for c in (r, k, v, g)]

@@ -26,6 +26,7 @@ __device__ __forceinline__ void st1(float* p, float v) { *p = v; }
 
 constexpr float LOG_DECAY_MIN = -104.f;      // exp(-104) is 0 in fp32
 constexpr int CT = 16;                       // tokens per chunk
+constexpr float LOG2E = 1.4426950408889634f;
 
 __device__ __forceinline__ float log_decay(float z) { return fmaxf(-expf(z), LOG_DECAY_MIN); }
 
@@ -36,10 +37,11 @@ struct Cols {
   int64_t ld, plane;
 };
 
-// in two steps, so that other loads can go out between the request and the wait: the first (up to) eight slabs,
+// in two steps, so that other loads can go out between the request and the wait: the first (up to) ASK slabs,
 // then their sum and the rest
+constexpr int ASK = 4;
 template <typename ACT>
-__device__ __forceinline__ void ldc_ask(const Cols& a, int64_t t, int c, float (&v)[8]) {
+__device__ __forceinline__ void ldc_ask(const Cols& a, int64_t t, int c, float (&v)[ASK]) {
   const int64_t o = t * a.ld + c;
   if (a.split == 0) {
     v[0] = ld1(reinterpret_cast<const ACT*>(a.p) + o);
@@ -47,20 +49,20 @@ __device__ __forceinline__ void ldc_ask(const Cols& a, int64_t t, int c, float (
   }
   const float* p = reinterpret_cast<const float*>(a.p) + o;
 #pragma unroll
-  for (int u = 0; u < 8; ++u) v[u] = p[(int64_t)min(u, a.split - 1) * a.plane];
+  for (int u = 0; u < ASK; ++u) v[u] = p[(int64_t)min(u, a.split - 1) * a.plane];
 }
 template <typename ACT>
-__device__ __forceinline__ float ldc_sum(const Cols& a, int64_t t, int c, const float (&v)[8]) {
+__device__ __forceinline__ float ldc_sum(const Cols& a, int64_t t, int c, const float (&v)[ASK]) {
   float s = v[0];
 #pragma unroll
-  for (int u = 1; u < 8; ++u) s += u < a.split ? v[u] : 0.f;
+  for (int u = 1; u < ASK; ++u) s += u < a.split ? v[u] : 0.f;
   const float* p = reinterpret_cast<const float*>(a.p) + t * a.ld + c;
-  for (int u = 8; u < a.split; ++u) s += p[(int64_t)u * a.plane];
+  for (int u = ASK; u < a.split; ++u) s += p[(int64_t)u * a.plane];
   return s;
 }
 template <typename ACT>
 __device__ __forceinline__ float ldc(const Cols& a, int64_t t, int c) {
-  float v[8];
+  float v[ASK];
   ldc_ask<ACT>(a, t, c, v);
   return ldc_sum<ACT>(a, t, c, v);
 }
@@ -100,7 +102,7 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, col = lane & 15, q = lane >> 4;
   const int h = blockIdx.y * WV + wv;
   if (h >= H) return;                             // waves share nothing below
-  float* L = smem + wv * (49 * LD);               // [17][LD]: L[t] = sum of log w before token t
+  float* L = smem + wv * (49 * LD);               // [17][LD]: L[t] = sum of log2 w before token t
   float* rs = L + 17 * LD;                        // [16][LD]
   float* ks = rs + 16 * LD;                       // [16][LD], then the coefficients [16][17] in its place
   const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
@@ -148,7 +150,7 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int c = 16 * T + 4 * q + i;
-      v[i] = c < D && col < n ? log_decay(z[T][i] + w0[hc + min(c, D - 1)]) : 0.f;
+      v[i] = c < D && col < n ? log_decay(z[T][i] + w0[hc + min(c, D - 1)]) * LOG2E : 0.f;
     }
     *reinterpret_cast<float4*>(L + (col + 1) * LD + 16 * T + 4 * q) = make_float4(v[0], v[1], v[2], v[3]);
   }
@@ -170,7 +172,7 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
         s += L[t * LD + c];
         L[t * LD + c] = s;
       }
-      out[Rec::DEC + c] = __expf(s);
+      out[Rec::DEC + c] = __builtin_amdgcn_exp2f(s);
     }
   }
   sync();
@@ -180,11 +182,11 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
     const int c = 16 * T + 4 * q;
     const float4 rv = *reinterpret_cast<const float4*>(rs + col * LD + c), lv = *reinterpret_cast<const float4*>(L + col * LD + c);
     reinterpret_cast<float4*>(out + Rec::R)[T * 64 + lane] =
-        make_float4(rv.x * __expf(lv.x), rv.y * __expf(lv.y), rv.z * __expf(lv.z), rv.w * __expf(lv.w));
+        make_float4(rv.x * __builtin_amdgcn_exp2f(lv.x), rv.y * __builtin_amdgcn_exp2f(lv.y), rv.z * __builtin_amdgcn_exp2f(lv.z), rv.w * __builtin_amdgcn_exp2f(lv.w));
     float kv[4];
     const float le = L[16 * LD + 16 * T + col];
 #pragma unroll
-    for (int s = 0; s < 4; ++s) kv[s] = ks[(4 * q + s) * LD + 16 * T + col] * __expf(le - L[(4 * q + s + 1) * LD + 16 * T + col]);
+    for (int s = 0; s < 4; ++s) kv[s] = ks[(4 * q + s) * LD + 16 * T + col] * __builtin_amdgcn_exp2f(le - L[(4 * q + s + 1) * LD + 16 * T + col]);
     reinterpret_cast<float4*>(out + Rec::K)[T * 64 + lane] = make_float4(kv[0], kv[1], kv[2], kv[3]);
   }
   // coefficients below the diagonal: two of the 120 pairs (i, j < i) per lane
@@ -205,8 +207,8 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
     for (int e = 0; e < 2; ++e) {
       const float4 a = *reinterpret_cast<const float4*>(L + pi[e] * LD + c), b = *reinterpret_cast<const float4*>(L + (pj[e] + 1) * LD + c);
       const float4 x = *reinterpret_cast<const float4*>(rs + pi[e] * LD + c), y = *reinterpret_cast<const float4*>(ks + pj[e] * LD + c);
-      acc[e] += x.x * y.x * __expf(a.x - b.x) + x.y * y.y * __expf(a.y - b.y) + x.z * y.z * __expf(a.z - b.z) +
-                x.w * y.w * __expf(a.w - b.w);
+      acc[e] += x.x * y.x * __builtin_amdgcn_exp2f(a.x - b.x) + x.y * y.y * __builtin_amdgcn_exp2f(a.y - b.y) + x.z * y.z * __builtin_amdgcn_exp2f(a.z - b.z) +
+                x.w * y.w * __builtin_amdgcn_exp2f(a.w - b.w);
     }
   // the diagonal: row lane / 4, a quarter of the channels
   float dg = 0.f;
@@ -253,11 +255,44 @@ __device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) {
 // buffers, one barrier per chunk); a chunk's outputs wait for the head's mean square until the next barrier.
 constexpr int SCAN_AHEAD = 4;
 
+typedef unsigned short raw16_t;
+template <typename ACT> struct RawOf { typedef uint32_t type; };
+template <> struct RawOf<uint16_t> { typedef raw16_t type; };
+template <typename ACT>
+__device__ __forceinline__ typename RawOf<ACT>::type ld_raw(__amdgpu_buffer_rsrc_t b, int vo, int so) {
+  if constexpr (sizeof(ACT) == 2) return __builtin_amdgcn_raw_buffer_load_b16(b, vo, so, 0);
+  else return __builtin_amdgcn_raw_buffer_load_b32(b, vo, so, 0);
+}
+template <typename ACT>
+__device__ __forceinline__ void st_raw(__amdgpu_buffer_rsrc_t b, int vo, int so, float y) {
+  if constexpr (sizeof(ACT) == 2) __builtin_amdgcn_raw_buffer_store_b16((raw16_t)(cvt_pk_bf16_f32(y, y) & 0xffff), b, vo, so, 0);
+  else __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(y), b, vo, so, 0);
+}
+template <typename ACT>
+__device__ __forceinline__ float raw2f(typename RawOf<ACT>::type v) {
+  return sizeof(ACT) == 2 ? __uint_as_float((uint32_t)v << 16) : __uint_as_float((uint32_t)v);
+}
+// buffer over `bytes` (< 2^31) from p, both uniform over the workgroup
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t rows_of(const void* p, int64_t bytes) {
+  // unsigned halves: readfirstlane returns int, whose sign would run into the upper half
+  const uint32_t lo = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)p), hi = __builtin_amdgcn_readfirstlane((uint32_t)((uintptr_t)p >> 32));
+  return __builtin_amdgcn_make_buffer_rsrc((void*)(((uintptr_t)hi << 32) | lo), (short)0, __builtin_amdgcn_readfirstlane((int)bytes), 0x00020000);
+}
+// sum over the 16 lanes of a row (four rotations within it)
+__device__ __forceinline__ float row16_sum(float x) {
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x128, 0xf, 0xf, false));   // row_ror:8
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x124, 0xf, 0xf, false));
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x122, 0xf, 0xf, false));
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x121, 0xf, 0xf, false));
+  return x;
+}
+
 template <typename ACT, int ND>
 __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __restrict__ rec, Cols v, Cols g, ScanSeq sq, int H,
                                                              int D, const float* __restrict__ norm, float eps,
                                                              float* __restrict__ state, ACT* __restrict__ out, int64_t ldo) {
   using Rec = ChunkRec<ND>;
+  using RAW = typename RawOf<ACT>::type;
   constexpr int NV4 = Rec::SIZE / 4, NT = 64 * ND, NLD = (NV4 + NT - 1) / NT;
   __shared__ __attribute__((aligned(16))) float buf[2][NLD * NT * 4];   // the last piece past the record: not read
   __shared__ __attribute__((aligned(16))) float red[2][ND][16];
@@ -279,23 +314,34 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
       const int kc = 16 * T + 4 * q + i;
       S[T][i] = !fresh && live && kc < D ? st[(size_t)min(kc, D - 1) * D] : 0.f;
     }
-  const float nw = norm[hv];
+  const float nw = norm[hv], rD = 1.f / (float)D;
   typedef float f4_t __attribute__((ext_vector_type(4)));      // arrays of these stay in registers
   f4_t rr[SCAN_AHEAD][NLD];
-  ACT rv[SCAN_AHEAD][4], rg[SCAN_AHEAD][4];         // as loaded: a conversion would wait for them
-  const ACT* vp = reinterpret_cast<const ACT*>(v.p) + hv;
-  const ACT* gp = reinterpret_cast<const ACT*>(g.p) + hv;
+  RAW rv[SCAN_AHEAD][4], rg[SCAN_AHEAD][4];         // as loaded: a conversion would wait for them
+  // buffers of the portion's rows: a chunk's place is a scalar offset, rows past the portion read as zero and are
+  // not stored -- no bounds arithmetic, and no branch whose join would wait for every load in flight
+  constexpr int EB = sizeof(ACT);
+  const __amdgpu_buffer_rsrc_t vb = rows_of(reinterpret_cast<const ACT*>(v.p) + row0 * v.ld, len * v.ld * EB);
+  const __amdgpu_buffer_rsrc_t gb = rows_of(reinterpret_cast<const ACT*>(g.p) + row0 * g.ld, len * g.ld * EB);
+  const __amdgpu_buffer_rsrc_t ob = rows_of(out + row0 * ldo, len * ldo * EB);
+  int vo[4], go[4], oo[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    vo[i] = ((4 * q + i) * (int)v.ld + hv) * EB;
+    go[i] = ((4 * q + i) * (int)g.ld + hv) * EB;
+    oo[i] = live ? ((4 * q + i) * (int)ldo + hv) * EB : 0x7ffffff0;
+  }
+  const float lm = live ? 1.f : 0.f;
   // chunk c (past the last: re-read, not used)
   auto load = [&](int c, int u) {
-    c = min(c, nc - 1);
+    c = __builtin_amdgcn_readfirstlane(min(c, nc - 1));
     const f4_t* p = reinterpret_cast<const f4_t*>(rec + ((size_t)(c0 + c) * H + h) * Rec::SIZE);
 #pragma unroll
     for (int i = 0; i < NLD; ++i) rr[u][i] = p[min(tid + NT * i, NV4 - 1)];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int64_t t = row0 + min(CT * c + 4 * q + i, len - 1);
-      rv[u][i] = vp[t * v.ld];
-      rg[u][i] = gp[t * g.ld];
+      rv[u][i] = ld_raw<ACT>(vb, vo[i], c * CT * (int)v.ld * EB);
+      rg[u][i] = ld_raw<ACT>(gb, go[i], c * CT * (int)g.ld * EB);
     }
   };
   auto store = [&](int b, int u) {
@@ -307,11 +353,6 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
     __builtin_amdgcn_s_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
   };
-  const uintptr_t ob = (uintptr_t)(out + (int64_t)row0 * ldo);
-  // unsigned halves: readfirstlane returns int, whose sign would run into the upper half
-  const uint32_t ob_lo = __builtin_amdgcn_readfirstlane((uint32_t)ob), ob_hi = __builtin_amdgcn_readfirstlane((uint32_t)(ob >> 32));
-  const __amdgpu_buffer_rsrc_t ors = __builtin_amdgcn_make_buffer_rsrc((void*)(((uintptr_t)ob_hi << 32) | ob_lo), (short)0,
-                                                                       0x7fffffe0, 0x00020000);
   f32x4_t o_prev{0.f, 0.f, 0.f, 0.f};
   float g_prev[4] = {0.f, 0.f, 0.f, 0.f};
   // outputs of chunk c from the mean squares in red[b]
@@ -322,14 +363,12 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
       const float4 a = *reinterpret_cast<const float4*>(&red[b][j][4 * q]);
       sv[0] += a.x; sv[1] += a.y; sv[2] += a.z; sv[3] += a.w;
     }
+    const int so = __builtin_amdgcn_readfirstlane(max(c, 0) * CT * (int)ldo * EB);   // before the first: overwritten by it
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int t = CT * c + 4 * q + i;
-      const float y = o_prev[i] * (1.f / sqrtf(sv[i] / (float)D + eps)) * nw * (g_prev[i] / (1.f + __expf(-g_prev[i])));
-      // without a branch (a join would wait for every load in flight): offsets past the range store nothing
-      const int off = live && t >= 0 && t < len ? (int)((t * ldo + hv) * (int64_t)sizeof(ACT)) : 0x7ffffff0;
-      if constexpr (sizeof(ACT) == 2) __builtin_amdgcn_raw_buffer_store_b16((short)f2bf(y), ors, off, 0, 0);
-      else __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(y), ors, off, 0, 0);
+      const float r = __builtin_amdgcn_rsqf(sv[i] * rD + eps);
+      const float y = o_prev[i] * r * nw * (g_prev[i] * __builtin_amdgcn_rcpf(1.f + __expf(-g_prev[i])));
+      st_raw<ACT>(ob, oo[i], so, y);
     }
   };
 #pragma unroll
@@ -340,12 +379,11 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
     barrier();
     const int b = u & 1;
     finish(c - 1, b ^ 1);
-    const float keep = c < nc ? 0.f : 1.f;        // past the last chunk: the state stays as it is
     float vv[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      vv[i] = live && CT * c + 4 * q + i < len ? ld1(&rv[u][i]) : 0.f;
-      g_prev[i] = ld1(&rg[u][i]);
+      vv[i] = raw2f<ACT>(rv[u][i]);
+      g_prev[i] = raw2f<ACT>(rg[u][i]);
     }
     load(c + SCAN_AHEAD, u);
     const float4* p = reinterpret_cast<const float4*>(buf[b]);
@@ -366,8 +404,7 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
     float4 k[ND];
 #pragma unroll
     for (int T = 0; T < ND; ++T) {
-      float4 d = p[Rec::DEC / 4 + 4 * T + q];       // decays are at most 1
-      d = make_float4(fmaxf(d.x, keep), fmaxf(d.y, keep), fmaxf(d.z, keep), fmaxf(d.w, keep));
+      const float4 d = p[Rec::DEC / 4 + 4 * T + q];
       k[T] = p[Rec::K / 4 + T * 64 + lane];
       S[T][0] *= d.x; S[T][1] *= d.y; S[T][2] *= d.z; S[T][3] *= d.w;
     }
@@ -384,19 +421,20 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
     float ss[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      ss[i] = live ? o_prev[i] * o_prev[i] : 0.f;
-#pragma unroll
-      for (int m = 8; m > 0; m >>= 1) ss[i] += __shfl_xor(ss[i], m, 64);
+      ss[i] = row16_sum(lm * o_prev[i] * o_prev[i]);
     }
     if (col == 0) *reinterpret_cast<float4*>(&red[b][w][4 * q]) = make_float4(ss[0], ss[1], ss[2], ss[3]);
     store(b ^ 1, (u + 1) % SCAN_AHEAD);
   };
-  for (int c = 0; c < nc; c += SCAN_AHEAD)
+  int c = 0;
+  for (; c + SCAN_AHEAD <= nc; c += SCAN_AHEAD)
 #pragma unroll
     for (int u = 0; u < SCAN_AHEAD; ++u) chunk(c + u, u);
-  const int last = (nc + SCAN_AHEAD - 1) / SCAN_AHEAD * SCAN_AHEAD - 1;
+#pragma unroll
+  for (int u = 0; u < SCAN_AHEAD - 1; ++u)
+    if (c + u < nc) chunk(c + u, u);
   barrier();
-  finish(last, last & 1);
+  finish(nc - 1, (nc - 1) & 1);
   if (live) {
 #pragma unroll
     for (int T = 0; T < ND; ++T)
@@ -412,8 +450,8 @@ __global__ void __launch_bounds__(64 * ND, 2) wkv_scan_kernel(const float* __res
 // one workgroup per (head, sequence); a thread owns V value channels of every NG-th key channel, so the
 // state needs no synchronisation between tokens
 constexpr int WS_T = 256, WS_NR = 4;
-template <typename ACT, int V>
-__global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, Cols g, Cols w1, int R, int RP,
+template <typename ACT, int V, bool ONE>      // ONE: a token per sequence
+__global__ void __launch_bounds__(WS_T, ONE ? 6 : 4) wkv_step_kernel(Cols r, Cols k, Cols v, Cols g, Cols w1, int R, int RP,
                                                        const uint16_t* __restrict__ w2, const float* __restrict__ w0,
                                                        const float* __restrict__ u, const float* __restrict__ norm, float eps,
                                                        int H, int D, const int32_t* __restrict__ slots,
@@ -427,10 +465,11 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
   float* vs = kk + D;
   float* gs = vs + D;
   float* ws = gs + D;
-  float* th = ws + D;          // [RP]
+  float* us = ws + D;          // u r k: the bonus
+  float* th = us + D;          // [RP]
   float* part = th + RP;       // [ng][D]
   const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x;
-  const int q0 = cu_q ? cu_q[s] : s, n = cu_q ? cu_q[s + 1] - q0 : 1;
+  const int q0 = ONE ? s : cu_q[s], n = ONE ? 1 : cu_q[s + 1] - q0;
   const bool fresh = ctx_lens[s] == n;
   float* st = state + ((size_t)slots[s] * H + h) * D * D;
   const int vx = tid % nvec, gy = tid / nvec, hc = h * D;
@@ -462,7 +501,7 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
       return s;
     };
     // the small operands are asked for ahead of the state: loads return in order
-    float ask[8], ask1[8];
+    float ask[ASK], ask1[ASK];
     const int e0 = min(tid, 4 * D - 1), z0 = min(tid, R - 1), wc = min(tid >> 2, D - 1);
     uint4 wq[2];
     ldc_ask<ACT>(pick(e0), row, hc + e0 % D, ask);
@@ -499,9 +538,8 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
       z += __shfl_xor(z, 2, 64);
       if (c < D && p == 0) ws[c] = expf(log_decay(z + (c0 == 0 ? w0v : w0[hc + c])));
     }
-    float bonus = 0.f;
-    for (int c = tid; c < D; c += WS_T) bonus += u[hc + c] * rs[c] * kk[c];
-    bonus = block_sum(bonus, red);               // its barriers also publish ws
+    for (int c = tid; c < D; c += WS_T) us[c] = u[hc + c] * rs[c] * kk[c];
+    __syncthreads();
     float o[V];
 #pragma unroll
     for (int e = 0; e < V; ++e) o[e] = 0.f;
@@ -514,10 +552,10 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
       for (int a = 0; a < WS_NR; ++a) {
         const int i = i0 + gy + a * ng;
         if (!own || i >= D) continue;
-        const float ri = rs[i], ki = kk[i], wi = ws[i];
+        const float ri = rs[i], ki = kk[i], wi = ws[i], bi = us[i];
 #pragma unroll
         for (int e = 0; e < V; ++e) {
-          o[e] += ri * S[a][e];
+          o[e] += ri * S[a][e] + bi * vv[e];
           S[a][e] = wi * S[a][e] + ki * vv[e];
         }
         if constexpr (V == 4) *reinterpret_cast<float4*>(st + (size_t)i * D + 4 * vx) = make_float4(S[a][0], S[a][1], S[a][2], S[a][3]);
@@ -536,11 +574,11 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
       y[m] = 0.f;
       if (c < D) {
         for (int a = 0; a < ng; ++a) y[m] += part[a * D + c];
-        y[m] += bonus * vs[c];
         ss += y[m] * y[m];
       }
     }
-    const float rr = 1.f / sqrtf(block_sum(ss, red) / (float)D + eps);
+    if (ONE && D <= 64 && tid >= 64) return;     // one wave holds the head
+    const float rr = 1.f / sqrtf((D <= 64 ? wave_sum(ss) : block_sum(ss, red)) / (float)D + eps);
 #pragma unroll
     for (int m = 0; m < 2; ++m) {
       const int c = tid + m * WS_T;
@@ -549,7 +587,7 @@ __global__ void __launch_bounds__(WS_T) wkv_step_kernel(Cols r, Cols k, Cols v, 
         st1(out + row * ldo + hc + c, y[m] * rr * norm[hc + c] * (gg / (1.f + expf(-gg))));
       }
     }
-    __syncthreads();                             // the next token overwrites what this one read
+    if constexpr (!ONE) __syncthreads();         // the next token overwrites what this one read
   }
 }
 
@@ -597,8 +635,9 @@ CFC_API int cfc_wkv_chunked(int f32, const void* r, int64_t ldr, const void* k, 
                             const int32_t* ctx_lens, float* rec, float* state, void* out, int64_t ldo, hipStream_t stream) {
   if (n_seq <= 0 || n_chunks <= 0) return 0;
   if (H < 1 || D < 1 || D > WKV_MAX_CHUNKED || RP < 32 || RP % 32 || n_seq > 65535) return -1;
-  // 32-bit store offsets within a portion
-  if ((int64_t)n_chunks * CT * ldo * (f32 ? 4 : 2) >= 0x7fffffe0ll) return -4;
+  // 32-bit offsets within a portion
+  const int64_t ldm = ldo > ldv ? (ldo > ldg ? ldo : ldg) : (ldv > ldg ? ldv : ldg);
+  if (((int64_t)n_chunks + 4) * CT * ldm * (f32 ? 4 : 2) >= 0x7fffff00ll) return -4;
   const Cols cr{r, 0, ldr, 0}, ck{k, 0, ldk, 0}, cv{v, 0, ldv, 0}, cg{g, 0, ldg, 0};
   const ScanSeq sq{chunk_cu, chunks, slots, cu_q, ctx_lens};
 #define WC(ACT, ND)                                                                                                      \
@@ -631,15 +670,21 @@ CFC_API int cfc_wkv_step(int f32, const void* r, const void* k, const void* v, c
   const int V = D % 4 == 0 ? 4 : 1;
   if ((D + V - 1) / V > WS_T) return -1;
   const int ng = WS_T / ((D + V - 1) / V);
-  const size_t lds = (size_t)(5 * D + RP + ng * D) * 4;
+  const size_t lds = (size_t)(6 * D + RP + ng * D) * 4;
   const Cols cr{r, split, ld, plane}, ck{k, split, ld, plane}, cv{v, split, ld, plane}, cg{g, split, ld, plane},
       c1{w1, split1, ld1, plane1};
-#define ST(ACT, VV)                                                                                                      \
-  wkv_step_kernel<ACT, VV><<<dim3(H, n_seq), WS_T, lds, stream>>>(cr, ck, cv, cg, c1, R, RP, (const uint16_t*)w2, w0, u, \
-                                                                 norm, eps, H, D, slots, cu_q, ctx_lens, state, (ACT*)out, ldo)
+#define ST1(ACT, VV, ONE)                                                                                                     \
+  wkv_step_kernel<ACT, VV, ONE><<<dim3(H, n_seq), WS_T, lds, stream>>>(cr, ck, cv, cg, c1, R, RP, (const uint16_t*)w2, w0, u, \
+                                                                      norm, eps, H, D, slots, cu_q, ctx_lens, state, (ACT*)out, ldo)
+#define ST(ACT, VV)                  \
+  do {                               \
+    if (cu_q) ST1(ACT, VV, false);   \
+    else ST1(ACT, VV, true);         \
+  } while (0)
   if (f32) { if (V == 4) ST(float, 4); else ST(float, 1); }
   else if (V == 4) ST(uint16_t, 4);
   else ST(uint16_t, 1);
 #undef ST
+#undef ST1
   return CFC_CHECK_LAUNCH();
 }
