@@ -331,12 +331,12 @@ class ZisapelWeights:
                 lw["rope"] = L.yarn_rope(m.rot_dim, m.base, dict(m.scaling) if m.scaling else None, w.device)
             if f is not None:
                 lw["norm2"], lw["rg2_b"] = vec(get(p + "norm2")), vec(get(p + "rg2.b"))
-                lw["rg2"] = Projection(mat(get(p + "rg2")))
             if isinstance(f, GluSpec):
                 lw["glu"], lw["limit"] = glu(p + "mlp.", f.ff), f.limit
+                lw["ff_in"] = JointProjection([(mat(get(p + "rg2")), 0)])
             elif f is not None:
                 y = p + "mlp."
-                lw["router_w"] = Projection(cls._whole_tiles(mat(get(y + "router"))))
+                lw["ff_in"] = JointProjection([(mat(get(p + "rg2")), 0), (mat(get(y + "router")), 0)])
                 lw["router"] = M.Router(f.experts, f.top, f.groups, f.keep, f.scale, vec(get(y + "correction")))
                 ex = [[mat(cut(get(f"{y}e{e}.{k}"))) for e in range(f.experts)]
                       for k, cut in (("gate", rows), ("up", rows), ("down", cols))]
@@ -350,16 +350,10 @@ class ZisapelWeights:
             torch.cuda.empty_cache()
         return w
 
-    @staticmethod
-    def _whole_tiles(t: torch.Tensor) -> torch.Tensor:
-        """A small matrix with zero rows up to whole 64-row tiles where that puts it on the packed products."""
-        n = -t.shape[0] % 64
-        return torch.cat([t, t.new_zeros(n, t.shape[1])]) if n and Projection.packs(t, 64, t.shape[1]) else t
-
     def nbytes(self) -> int:
         n = self.embed.numel() * self.embed.element_size() + self.head.nbytes()
         for lw in self.layers:
-            n += sum(lw[k].nbytes() for k in ("o", "in", "uk", "uv", "uk_full", "rg2", "router_w", "experts") if k in lw)
+            n += sum(lw[k].nbytes() for k in ("o", "in", "uk", "uv", "uk_full", "ff_in", "experts") if k in lw)
             n += lw["uv_full"].numel() * 2 if "uv_full" in lw else 0
             for k in ("glu", "shared"):
                 if lw.get(k):
@@ -500,7 +494,8 @@ class ZisapelModel:
             b = G.Branch(gate, lw["rg1_b"], lw["norm1"], self.cfg.norm_eps, y=self._sum(lw["o"].slabs(o)))
             G.gated_norm(x, b, dt, h if s.mlp is not None else None, kv.prev[i], plan["meta"], positions)
             if s.mlp is not None:
-                G.gated_norm(x, self._feed(i, h, G.Cols(lw["rg2"].act(h))), dt)
+                ff, hs = lw["ff_in"], h[None]
+                G.gated_norm(x, self._feed(i, h, ff.act(0, hs), ff.slabs(1, hs) if len(ff.sizes) > 1 else None), dt)
         return G.final_norm(x, self.w.final_norm, self.cfg.norm_eps, dt, None if last_idx is None else last_idx.to(torch.int32))
 
     def forward_decode(self, ids, positions, slots, ctx_lens, block_tables, kv, attn_workspace=None, part_blocks=-1,
@@ -536,7 +531,7 @@ class ZisapelModel:
                 acts = shift(b, i + 1)
             else:
                 G.gated_shift(x, b, dt, h)
-                acts = shift(self._feed(i, h, G.Cols(lw["rg2"].slabs(h, own=True))), i + 1)
+                acts = shift(self._feed(i, h, *lw["ff_in"].joint(h[None])), i + 1)
         return G.final_norm(x, self.w.final_norm, self.cfg.norm_eps, dt)
 
     def _shift(self, i, kv) -> G.Shift:
@@ -593,14 +588,14 @@ class ZisapelModel:
             S.clamped_glu(p["gate_up"].slabs(h), a, limit, alpha, beta)
         return p["down"].slabs(a, own=own)
 
-    def _feed(self, i, h, gate) -> G.Branch:
-        """Layer i's feed-forward of h as the branch it adds."""
+    def _feed(self, i, h, gate, router=None) -> G.Branch:
+        """Layer i's feed-forward of h as the branch it adds; ``router``: the router's logits (routed layers)."""
         lw, f = self.w.layers[i], self.cfg.specs[i].mlp
         b = G.Branch(gate, lw["rg2_b"], lw["norm2"], self.cfg.norm_eps)
         if isinstance(f, GluSpec):
             b.y = self._sum(self._glu(h, lw["glu"], lw["limit"], GLU_ALPHA, GLU_SHIFT))
             return b
-        ids, wt = M.route(G.Cols(lw["router_w"].slabs(h), 0, f.experts), lw["router"])
+        ids, wt = M.route(router, lw["router"])
         rows, pos = M.experts(h, lw["experts"], ids)
         shared = self._glu(h, lw["shared"], M.INF, 1.0, 0.0) if lw["shared"] else None
         if self.w.tp_size == 1:

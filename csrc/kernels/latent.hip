@@ -130,6 +130,7 @@ __device__ __forceinline__ float ldcol(const LatCols& a, int64_t t, int c) {
   const int64_t o = t * a.ld + c;
   if (a.split == 0) return ldf(reinterpret_cast<const ACT*>(a.p) + o);
   const float* p = reinterpret_cast<const float*>(a.p) + o;
+  if (a.split == 1) return *p;
   float s = 0.f;
   for (int i0 = 0; i0 < a.split; i0 += 8) {
     float v[8];
@@ -235,6 +236,72 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatCols kv, int NC, co
       stf(qn + (size_t)t * H * dim + e, ldcol<ACT>(q, t, e / dim * (dim + r.rot) + e % dim));
   if (gate)
     for (int e = h0 * vdim + tid; e < h1 * vdim; e += 256) stf(gate + (size_t)t * H * vdim + e, ldcol<ACT>(g, t, e));
+}
+
+// Prompt rows (q as activations): a wave per row, everything it reads requested before its first wait.  NK x 64
+// latent columns; rot <= 128
+template <typename ACT, int NK>
+__global__ void __launch_bounds__(256) latent_rope_rows_kernel(LatCols kv, int T, int NC, const float* __restrict__ wc, float eps,
+                                                              const int32_t* __restrict__ slots, ACT* __restrict__ cache,
+                                                              int RS, int RV, LatCols q, int H, int dim,
+                                                              ACT* __restrict__ qr, int qs, int PQ, RopeArgs r) {
+  __shared__ float2 cs[4][64];
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, hr = r.rot / 2;
+  const int t = min((int)blockIdx.x * 4 + w, T - 1);        // rows past the last: the last one again
+  const int pos = r.positions[t];
+  ACT* dst = cache + (size_t)slots[t] * RS;
+  float x[NK];
+#pragma unroll
+  for (int k = 0; k < NK; ++k) x[k] = ldcol<ACT>(kv, t, min(64 * k + lane, NC - 1));
+  const int pr = min(lane, max(hr - 1, 0));
+  float ku = ldcol<ACT>(kv, t, NC + 2 * pr), kw = ldcol<ACT>(kv, t, NC + 2 * pr + 1);
+  float sn, co;
+  sincosf((float)pos * r.freq[pr], &sn, &co);
+  const float2 mine = make_float2(co * r.mag, sn * r.mag);
+  cs[w][lane] = mine;
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  float s = 0.f;
+#pragma unroll
+  for (int k = 0; k < NK; ++k) s += 64 * k + lane < NC ? x[k] * x[k] : 0.f;
+  const float rs = 1.f / sqrtf(wave_sum(s) / (float)NC + eps);
+#pragma unroll
+  for (int k = 0; k < NK; ++k)
+    if (64 * k + lane < NC) stf(dst + 64 * k + lane, x[k] * rs * wc[64 * k + lane]);
+  if (lane < hr) {
+    stf(dst + RV + 2 * lane, ku * mine.x - kw * mine.y);
+    stf(dst + RV + 2 * lane + 1, kw * mine.x + ku * mine.y);
+  }
+  const int hp = PQ / 2, n = H * hp, step = dim + r.rot;
+  const ACT* qrow = reinterpret_cast<const ACT*>(q.p) + (int64_t)t * q.ld + dim;
+  ACT* orow = qr + (size_t)t * H * qs;
+  for (int e0 = 0; e0 < n; e0 += 512) {
+    float u[8], v[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const int e = min(e0 + 64 * k + lane, n - 1), h = e / hp, i = min(e % hp, hr - 1);
+      const ACT* p = qrow + h * step + 2 * i;
+      if constexpr (sizeof(ACT) == 2) {
+        const uint32_t b = *reinterpret_cast<const uint32_t*>(p);
+        u[k] = __uint_as_float(b << 16);
+        v[k] = __uint_as_float(b & 0xffff0000u);
+      } else {
+        u[k] = ldf(p);
+        v[k] = ldf(p + 1);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const int e = e0 + 64 * k + lane, h = min(e, n - 1) / hp, i = min(e, n - 1) % hp;
+      if (e >= n) continue;
+      const float2 c = cs[w][min(i, 63)];
+      const float a = i < hr ? u[k] * c.x - v[k] * c.y : 0.f, b = i < hr ? v[k] * c.x + u[k] * c.y : 0.f;
+      ACT* o = orow + h * qs + 2 * i;
+      if constexpr (sizeof(ACT) == 2) *reinterpret_cast<uint32_t*>(o) = pack2bf(a, b);
+      else { stf(o, a); stf(o + 1, b); }
+    }
+  }
 }
 
 // ---------------------------------------------------------------------------------- head_linear
@@ -940,6 +1007,18 @@ CFC_API int cfc_latent_rope(int f32, const void* kv, int kv_split, int64_t kv_ld
   const int NB = T >= 512 ? 1 : H < 64 ? H : 64;
   const LatCols ckv{kv, kv_split, kv_ld, kv_plane}, cq{q, q_split, q_ld, q_plane}, cg{g, g_split, g_ld, g_plane};
   const RopeArgs r{freq, mag, positions, rot};
+  // prompt rows whose pairs are words
+  if (T >= 512 && q_split == 0 && rot >= 2 && rot <= 128 && NC <= 1024 && !qn && !gate && dim % 2 == 0 && q_ld % 2 == 0 &&
+      qs % 2 == 0 && (((uintptr_t)q | (uintptr_t)qr) & 3) == 0) {
+#define LRR(ACT, NK)                                                                                                 \
+  latent_rope_rows_kernel<ACT, NK><<<(T + 3) / 4, 256, 0, stream>>>(ckv, T, NC, wc, eps, slots, (ACT*)cache, RS, RV, cq, H, \
+                                                                   dim, (ACT*)qr, qs, PQ, r)
+    if (NC <= 512) { if (f32) LRR(float, 8); else LRR(uint16_t, 8); }
+    else if (f32) LRR(float, 16);
+    else LRR(uint16_t, 16);
+#undef LRR
+    return CFC_CHECK_LAUNCH();
+  }
 #define LR(ACT)                                                                                                         \
   latent_rope_kernel<ACT><<<dim3(T, 1 + NB), 256, 0, stream>>>(ckv, NC, wc, eps, slots, (ACT*)cache, RS, RV, cq, H, dim, \
                                                               (ACT*)qr, qs, PQ, (ACT*)qn, cg, vdim, (ACT*)gate, r)

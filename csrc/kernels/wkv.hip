@@ -127,10 +127,17 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
       }
     }
   }
-  // z^T = W2 tanh^T: lane holds channels 16 T + 4 q + i of token col
+  // z^T = W2 tanh^T + w0: lane holds channels 16 T + 4 q + i of token col.  Every load unconditional: one under a
+  // branch would be waited for before the next goes out
   f32x4_t z[ND];
+  float ur[ND][4];                                // u of the lane's channels of the diagonal, below
 #pragma unroll
-  for (int T = 0; T < ND; ++T) z[T] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int T = 0; T < ND; ++T)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      z[T][i] = w0[hc + min(16 * T + 4 * q + i, D - 1)];
+      ur[T][i] = u[hc + min(16 * T + 4 * (lane & 3) + i, D - 1)];
+    }
   const uint16_t* tr = th + (size_t)(row0 + min(col, n - 1)) * 3 * RP + 8 * q;
   for (int kk = 0; kk < RP; kk += 32) {
     bf16x8_t b[3];
@@ -150,7 +157,8 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int c = 16 * T + 4 * q + i;
-      v[i] = c < D && col < n ? log_decay(z[T][i] + w0[hc + min(c, D - 1)]) * LOG2E : 0.f;
+      const float l = log_decay(z[T][i]) * LOG2E;
+      v[i] = c < D && col < n ? l : 0.f;
     }
     *reinterpret_cast<float4*>(L + (col + 1) * LD + 16 * T + 4 * q) = make_float4(v[0], v[1], v[2], v[3]);
   }
@@ -214,12 +222,12 @@ __global__ void __launch_bounds__(64 * WV) wkv_prep_kernel(Cols r, Cols k, const
   float dg = 0.f;
   {
     const int i = lane >> 2;
-    for (int c = (lane & 3) * 4; c < DP; c += 16)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const float uu = c + e < D ? u[hc + c + e] : 0.f;
-        dg += uu * rs[i * LD + c + e] * ks[i * LD + c + e];
-      }
+    for (int T = 0; T < ND; ++T) {                // r and k past D are zero
+      const int c = 16 * T + 4 * (lane & 3);
+      const float4 a = *reinterpret_cast<const float4*>(rs + i * LD + c), b = *reinterpret_cast<const float4*>(ks + i * LD + c);
+      dg += ur[T][0] * a.x * b.x + ur[T][1] * a.y * b.y + ur[T][2] * a.z * b.z + ur[T][3] * a.w * b.w;
+    }
     dg += __shfl_xor(dg, 1, 64);
     dg += __shfl_xor(dg, 2, 64);
   }

@@ -223,17 +223,19 @@ def test_rotary_frequencies(dims, base, scaling):
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,dim,rot,rank,vdim", [(3, 20, 12, 44, 28), (1, 8, 2, 20, 10), (4, 128, 64, 512, 128), (2, 32, 16, 1100, 16)])
-@pytest.mark.parametrize("split", [0, 1, 11])
-def test_latent_and_rotary_rows(device, dtype, H, dim, rot, rank, vdim, split):
-    T, eps = 6, 1e-3
+@pytest.mark.parametrize("split,T", [(0, 6), (1, 6), (11, 6), (0, 517)])
+def test_latent_and_rotary_rows(device, dtype, H, dim, rot, rank, vdim, split, T):
+    eps = 1e-3
     kv, q, g, w = rnd(T, rank + rot), rnd(T, H * (dim + rot), seed=1), rnd(T, H * vdim, seed=2), rnd(rank, seed=3)
     if not split:
         kv, q, g = (t.to(dtype).float() for t in (kv, q, g))
     d = lambda t: t.to(device).contiguous()
     rope = L.yarn_rope(rot, 300.0, SCALING, device)
     rv, pad = L.padded_rank(rank), L.padded_rank(rot)
-    cache = torch.zeros(4, 32, rv + pad, dtype=dtype, device=device)
-    slots, pos = i32([3, 40, 41, 100, 7, 64], device), i32([0, 1, 500, 31, 32, 9000], device)
+    blocks = 4 + T // 32
+    cache = torch.zeros(blocks, 32, rv + pad, dtype=dtype, device=device)
+    slots = i32(torch.randperm(32 * blocks, generator=torch.Generator().manual_seed(2))[:T], device)
+    pos = i32([0, 1, 500, 31, 32, 9000] + list(range(100, 94 + T)), device)
     ql = torch.full((T, H, rv + pad), 5.0, dtype=dtype, device=device)
     c = [Cols(d(slabs(t, split))) if split else Cols(d(t.to(dtype))) for t in (kv, q, g)]
     qn, gate = L.latent_rope(c[0], rank, d(w), eps, slots, cache, c[1], H, dim, rope, pos, ql[:, :, rv:], vdim, c[2])
