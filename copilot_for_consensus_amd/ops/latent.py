@@ -180,7 +180,8 @@ def decode_plan(B: int, heads: int, RS: int, max_ctx: int, P: int | None = None)
         g = math.ceil(heads / rows)
         for p in cand:
             rounds = math.ceil(B * g * p / (256 * per_cu))
-            t = max(rounds * (4 + math.ceil(nt / p) * _TILE_US[rows] * scale * min(per_cu, math.ceil(B * g * p / 256))),
+            us = _TILE_US[rows] * scale * (1.15 if rows > 16 and RS > MFMA_MAX_RANK else 1.0)
+            t = max(rounds * (4 + math.ceil(nt / p) * us * min(per_cu, math.ceil(B * g * p / 256))),
                     B * max_ctx * RS * 2 * g / 7e6)
             if p > 1:
                 t += 8 + 2 * B * heads * p * RS * 4 / 5e6

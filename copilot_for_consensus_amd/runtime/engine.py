@@ -505,14 +505,14 @@ class LLMEngine:
             done0 = torch.isin(f, st.stop_ids.cpu()).to(torch.int32) if stop_ids else torch.zeros(B, dtype=torch.int32)
             if stop_strings is not None:
                 # the prefill's token is the first of every sequence: fed on the host
-                states, keep = [], []
+                stop_states, keep = [], []
                 for b in range(B):
                     s0, hit = stop_strings.feed(stop_strings.initial(), int(first[b]))
-                    states.append(s0)
+                    stop_states.append(s0)
                     keep.append(1 if hit else st.stop_state.cap)
                     if hit:
                         done0[b] = 1
-                st.stop_state.set_slots(range(B), states, keep)
+                st.stop_state.set_slots(range(B), stop_states, keep)
             st.done.copy_(done0)
             ready = None
             if sync:

@@ -294,6 +294,27 @@ def test_greedy_generation_through_both_engines(device):
     assert eng.kv.states.num_free() == 6
 
 
+@pytest.mark.parametrize("device", DEVICES)
+def test_stop_strings_and_sampling(device):
+    """The engine's own stops and sampler over the family: a stopped row ends where its text does, its slot comes
+    back; the same seed draws the same tokens."""
+    from copilot_for_consensus_amd.runtime.stops import StopStringMatcher
+    from test_stops import STOPS, _vocab_tok
+    m = Model(config([wkv(heads=2, dim=16, mlp=dense(40)), attn(heads=2, mlp=None)], vocab=512, width=64), seed=5)
+    g = m.build(device)
+    eng = LLMEngine(g, g.new_cache(64, sequences=6))
+    matcher = StopStringMatcher.for_tokenizer(_vocab_tok(512), STOPS)
+    prompts = [m.tokens(20 + i, seed=i) for i in range(6)]
+    full = eng.generate(prompts, 40, temperature=1.5, seed=11, ignore_eos=True).tokens
+    assert eng.generate(prompts, 40, temperature=1.5, seed=11, ignore_eos=True).tokens == full
+    res = eng.generate(prompts, 40, temperature=1.5, seed=11, ignore_eos=True, stop_strings=matcher).tokens
+    cut = [matcher.match_tokens(t) for t in full]
+    assert any(c is not None for c in cut)
+    for whole, c, got in zip(full, cut, res):
+        assert got == (whole if c is None else whole[:c + 1])
+    assert eng.kv.states.num_free() == 6
+
+
 @pytest.mark.gpu
 def test_decode_graph_replays_equal_eager_steps():
     m = model("packed")
