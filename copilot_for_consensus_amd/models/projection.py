@@ -103,7 +103,7 @@ class Projection:
         k, M = self._kernel(x), x.shape[0]
         if k == "pgemm" and self.K >= 128 and out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0:
             return K.pgemm_glu(x, self.packed, out, limit, alpha, beta)
-        if k in ("pgemm", "dgemm") and self.N // self.packed.bn * -(-M // 256) >= K.DGEMM_CUS // 2 \
+        if k in ("pgemm", "dgemm") and self.N // self.packed.bn * -(-M // 256) > K.DGEMM_CUS // 2 \
                 and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0:
             return K.dgemm_glu(x, self.packed, out, limit, alpha, beta)
         return clamped_glu(self.slabs(x), out, limit, alpha, beta, interleaved=True)

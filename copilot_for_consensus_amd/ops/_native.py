@@ -102,6 +102,7 @@ _KERNEL_SIGS = {
     "cfc_dgemm_pack": [P, P, I, I, I, P],
     "cfc_dgemm_ablate": [P, P, I, I, I, I, I, I, P, P],
     "cfc_gemv": [P, P, I, I, I, I, P, P, I, P],
+    "cfc_gemv_group": [P, P, P, I, I, I, I, I, I, I, P, P, I, I, P],
     "cfc_gemv_packed": [P, P, I, I, I, I, I, P, P, I, I, I, P, I, P, P, P, F, P, P],
     "cfc_dgemm_joint": [P, P, I, I, I, I, I, P, P, P],
     "cfc_qgemv": [P, I, I, I, I, P, P, c_int64, c_int64, c_int64, I, P, P, I, P],

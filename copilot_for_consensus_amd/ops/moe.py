@@ -14,8 +14,9 @@ from . import reference as ref
 from ._native import check, kernels
 from .cols import Cols
 from .kernels import _p, _req, _stream
-from .stream import _act
+from .stream import _act, clamped_glu
 
+GEMV_PAIRS = 8          # at most so many (token, choice) pairs each stream their own expert
 ANY_TILE = 32           # rows per tile of the general products
 MAX_EXPERTS = 1024
 INF = float("inf")
@@ -40,6 +41,7 @@ class ExpertWeights:
         E, F, W = gate.shape
         self.E, self.F, self.W, self.dtype = E, F, W, gate.dtype
         self.packed = gate.is_cuda and gate.dtype == torch.bfloat16 and W % 64 == 0
+        self.pair_order = None if not self.packed else torch.arange(GEMV_PAIRS, dtype=torch.int32, device=gate.device)
         if not self.packed:
             self.gu = torch.cat([gate, up], 1).contiguous()
             self.down = down.contiguous()
@@ -113,8 +115,28 @@ def _grouped(glu, x, w, E, N, bn, tile, rows, te, out):
                                   out.stride(0), INF, 1.0, 0.0, _stream(x)), "cfc_dgemm_group")
 
 
+def _experts_gemv(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
+    """Few pairs: each streams its expert's matrices, in the pairs' own order."""
+    T, top = ids.shape
+    pairs, lib, dev = T * top, kernels(), x.device
+    split, waves = K.gemv_packed_config(pairs * 2 * w.F, w.W, w.bn_gu // 16)
+    part = K._workspace(dev, split * pairs * 2 * w.F)[:split * pairs * 2 * w.F].view(split, pairs, 2 * w.F)
+    check(lib.cfc_gemv_group(x.data_ptr(), w.gu.data_ptr(), ids.data_ptr(), pairs, top, w.E, 2 * w.F, w.W, w.bn_gu // 16, 0,
+                             part.data_ptr(), None, split, waves, _stream(x)), "cfc_gemv_group")
+    a = clamped_glu(part, torch.empty(pairs, w.F, dtype=x.dtype, device=dev), INF, 1.0, 0.0, interleaved=True)
+    y = torch.empty(pairs, w.W, dtype=x.dtype, device=dev)
+    _, waves = K.gemv_packed_config(pairs * w.W, w.F, w.bn_down // 16, slab=False)
+    check(lib.cfc_gemv_group(a.data_ptr(), w.down.data_ptr(), ids.data_ptr(), pairs, 1, w.E, w.W, w.F, w.bn_down // 16, 1, None,
+                             y.data_ptr(), 1, waves, _stream(x)), "cfc_gemv_group")
+    return y, w.pair_order[:pairs].view(T, top)
+
+
 def experts(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
     """W_down (silu(W_gate x) * W_up x) of every (token, choice): (rows [M, W] in x's dtype, row per pair [T, top])."""
+    if w.packed and ids.numel() <= GEMV_PAIRS and x.is_contiguous():
+        _req(x, torch.bfloat16, "x")
+        _req(ids, torch.int32, "ids")
+        return _experts_gemv(x, w, ids)
     tile = w.tile(ids.numel())
     rows, pos, te = sort_rows(ids, w.E, tile)
     M = te.numel() * tile

@@ -243,12 +243,18 @@ struct GvNorm {
   float eps;
 };
 
+// routed products: output run p (tiles tiles long) multiplies row p / per of X with matrix ids[p] of experts (null ids: none)
+struct GvGroup {
+  const int32_t* ids = nullptr;
+  int experts = 0, tiles = 1, per = 1;
+};
+
 // in_of: several inputs X[inputs][M][K], W tile n multiplying input in_of[n] (null: one input)
 template <int NW, int MT, int WAVES, bool XN>
 __global__ void __launch_bounds__(64 * WAVES) gemv_tile_kernel(const uint16_t* __restrict__ X,
                                                         const uint16_t* __restrict__ Wp, int N, int K, int S, int epi,
                                                         float* __restrict__ yf, uint16_t* __restrict__ yb, int ldo,
-                                                        GvNorm nm, const int32_t* __restrict__ in_of) {
+                                                        GvNorm nm, const int32_t* __restrict__ in_of, GvGroup gr) {
   constexpr int U = MT > 2 ? 2 : (NW >= 7 ? 3 : 4);
   constexpr int R = NW * MT * 16;                  // (group, m, row) values of one tile
   __shared__ float red[WAVES][R];
@@ -259,7 +265,14 @@ __global__ void __launch_bounds__(64 * WAVES) gemv_tile_kernel(const uint16_t* _
     if (in_of) X += (size_t)in_of[tile] * MT * K;
   const int KG = K / 32;
   const int kb = s * KG / S, ke = (s + 1) * KG / S;
-  const uint16_t* base = Wp + (size_t)tile * KG * NW * 512;
+  int wt = tile;
+  if constexpr (!XN && MT == 1)
+    if (gr.ids) {
+      const int p = tile / gr.tiles;
+      wt = min(max(gr.ids[p], 0), gr.experts - 1) * gr.tiles + tile - p * gr.tiles;
+      X += (size_t)(p / gr.per) * K;
+    }
+  const uint16_t* base = Wp + (size_t)wt * KG * NW * 512;
   const uint32_t lo = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)base);
   const uint32_t hi = __builtin_amdgcn_readfirstlane((uint32_t)((uintptr_t)base >> 32));
   const __amdgpu_buffer_rsrc_t rs = __builtin_amdgcn_make_buffer_rsrc(
@@ -448,7 +461,7 @@ CFC_API int cfc_gemv(const void* x, const void* w, int M, int N, int K, int epi,
 namespace {
 template <int NW, int MT, int WAVES, bool XN>
 void gemv_tile_go(dim3 grid, hipStream_t stream, const uint16_t* x, const uint16_t* wp, int N, int K, int split, int epi,
-                  float* yf, uint16_t* yb, int ldo, const GvNorm& nm, const int32_t* in_of) {
+                  float* yf, uint16_t* yb, int ldo, const GvNorm& nm, const int32_t* in_of, const GvGroup& gr) {
   const size_t lds = XN ? (size_t)MT * K * 2 : 0;
   if constexpr (XN) {
     static bool raised = false;                    // dynamic LDS past 64 KB (Llama-70B rows at M = 4)
@@ -458,16 +471,17 @@ void gemv_tile_go(dim3 grid, hipStream_t stream, const uint16_t* x, const uint16
       raised = true;
     }
   }
-  gemv_tile_kernel<NW, MT, WAVES, XN><<<grid, 64 * WAVES, lds, stream>>>(x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of);
+  gemv_tile_kernel<NW, MT, WAVES, XN><<<grid, 64 * WAVES, lds, stream>>>(x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of, gr);
 }
 
 template <int NW, int MT>
 void gemv_tile_launch(dim3 grid, int waves, hipStream_t stream, const uint16_t* x, const uint16_t* wp, int N, int K,
-                      int split, int epi, float* yf, uint16_t* yb, int ldo, const GvNorm& nm, const int32_t* in_of) {
+                      int split, int epi, float* yf, uint16_t* yb, int ldo, const GvNorm& nm, const int32_t* in_of,
+                      const GvGroup& gr = {}) {
   const bool xn = nm.part != nullptr;
 #define GVT(WV)                                                                                    \
-  if (xn) gemv_tile_go<NW, MT, WV, true>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of);  \
-  else gemv_tile_go<NW, MT, WV, false>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of);
+  if (xn) gemv_tile_go<NW, MT, WV, true>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of, gr);  \
+  else gemv_tile_go<NW, MT, WV, false>(grid, stream, x, wp, N, K, split, epi, yf, yb, ldo, nm, in_of, gr);
   if (waves == 4) { GVT(4) }
   else if (waves == 8) { GVT(8) }
   else if constexpr (MT == 1) { GVT(16) }         // 16 waves: 4 per SIMD, so <= 128 VGPRs -- single-row only
@@ -508,5 +522,28 @@ CFC_API int cfc_gemv_packed(const void* x, const void* wp, int M, int N, int K, 
   }
 #undef GVP_CASE
 #undef GVP_ARGS
+  return CFC_CHECK_LAUNCH();
+}
+
+// Routed products of few rows: pair p (a token's choice) multiplies row p / per of x [pairs / per][K] with matrix ids[p]
+// of wp [experts][N][K] (packed as above); out [pairs][N], fp32 slabs or bf16 (epi).  A pair reads its own matrix.
+CFC_API int cfc_gemv_group(const void* x, const void* wp, const int32_t* ids, int pairs, int per, int experts, int N, int K,
+                           int nw, int epi, float* yf, void* yb, int split, int waves, hipStream_t stream) {
+  if (pairs < 1 || per < 1 || pairs % per || experts < 1 || N <= 0 || (nw != 4 && nw != 8) || N % (16 * nw) || K <= 0 || K % 32)
+    return -1;
+  if ((epi == GV_F32 && !yf) || (epi != GV_F32 && !yb) || epi < 0 || epi > 1) return -2;
+  if (!x || !ids || split < 1 || split > K / 32 || (split > 1 && epi != GV_F32)) return -4;
+  if ((waves != 4 && waves != 8 && waves != 16) || (size_t)K / 32 * nw * 1024 >= (1u << 31)) return -5;
+  GvGroup gr;
+  gr.ids = ids; gr.experts = experts; gr.tiles = N / (16 * nw); gr.per = per;
+  const GvNorm nm{nullptr, 0, nullptr, nullptr, nullptr, 0.f};
+  const dim3 grid(pairs * gr.tiles * split);
+  const int NT = pairs * N;
+  if (nw == 4)
+    gemv_tile_launch<4, 1>(grid, waves, stream, (const uint16_t*)x, (const uint16_t*)wp, NT, K, split, epi, yf, (uint16_t*)yb,
+                           NT, nm, nullptr, gr);
+  else
+    gemv_tile_launch<8, 1>(grid, waves, stream, (const uint16_t*)x, (const uint16_t*)wp, NT, K, split, epi, yf, (uint16_t*)yb,
+                           NT, nm, nullptr, gr);
   return CFC_CHECK_LAUNCH();
 }

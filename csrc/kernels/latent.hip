@@ -1003,8 +1003,8 @@ CFC_API int cfc_latent_rope(int f32, const void* kv, int kv_split, int64_t kv_ld
   if (NC < 1 || NC > RV || RV % 2 || rot < 0 || rot % 2 || rot > ROPE_MAX || RV + rot > RS || PQ < rot || PQ % 2 || qs < PQ ||
       H < 1 || dim < 1)
     return -1;
-  // few rows: one workgroup per head, so their slab sums do not follow one another
-  const int NB = T >= 512 ? 1 : H < 64 ? H : 64;
+  // few rows: up to one workgroup per head, so their slab sums do not follow one another; no more than run at once
+  const int fit = T >= 512 ? 1 : max(2, 1024 / T), NB = H < fit ? H : fit < 64 ? fit : 64;
   const LatCols ckv{kv, kv_split, kv_ld, kv_plane}, cq{q, q_split, q_ld, q_plane}, cg{g, g_split, g_ld, g_plane};
   const RopeArgs r{freq, mag, positions, rot};
   // prompt rows whose pairs are words

@@ -410,7 +410,8 @@ def test_rows_sorted_by_expert(device, T, top, E, tile):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,W,F,E,top", [(1, 104, 20, 6, 2), (37, 65, 31, 5, 3), (9, 128, 72, 8, 2), (300, 192, 64, 4, 2), (700, 64, 128, 4, 3)])
+@pytest.mark.parametrize("T,W,F,E,top", [(1, 104, 20, 6, 2), (1, 128, 72, 8, 2), (2, 192, 64, 16, 4), (4, 64, 200, 3, 2),
+                                             (1, 2048, 320, 9, 8), (37, 65, 31, 5, 3), (9, 128, 72, 8, 2), (300, 192, 64, 4, 2), (700, 64, 128, 4, 3)])
 def test_expert_products(device, dtype, T, W, F, E, top):
     x = rnd(T, W).to(dtype)
     g, u, dn = (rnd(E, *s, seed=i, scale=s[1] ** -0.5).to(dtype) for i, s in enumerate(((F, W), (F, W), (W, F))))
