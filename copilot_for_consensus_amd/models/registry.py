@@ -8,7 +8,7 @@ from pathlib import Path
 
 import torch
 
-from . import decoder, vofosun, zisapel
+from . import decoder, pemolorn, vofosun, zisapel
 
 
 @dataclasses.dataclass(frozen=True)
@@ -33,6 +33,11 @@ def _load_zisapel(path):
     return zisapel.config_from_json(json.loads(path.read_text()), name=path.parent.name or "zisapel", ckpt_dir=path.parent)
 
 
+def _load_pemolorn(path):
+    path = Path(path)
+    return pemolorn.config_from_json(json.loads(path.read_text()), name=path.parent.name or "pemolorn")
+
+
 FAMILIES: dict[str, Family] = {
     "decoder": Family("decoder", decoder.DecoderConfig, decoder.DecoderWeights, decoder.DecoderModel, decoder.PRESETS,
                       decoder.load_config_json, (torch.bfloat16,)),
@@ -40,6 +45,8 @@ FAMILIES: dict[str, Family] = {
                       _load_vofosun, (torch.bfloat16, torch.float32)),
     "Zisapel": Family("Zisapel", zisapel.ZisapelConfig, zisapel.ZisapelWeights, zisapel.ZisapelModel, zisapel.PRESETS,
                       _load_zisapel, (torch.bfloat16, torch.float32)),
+    "Pemolorn": Family("Pemolorn", pemolorn.PemolornConfig, pemolorn.PemolornWeights, pemolorn.PemolornModel, pemolorn.PRESETS,
+                       _load_pemolorn, (torch.bfloat16, torch.float32)),
 }
 
 

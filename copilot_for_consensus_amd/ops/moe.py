@@ -30,6 +30,19 @@ class Router:
     keep: int
     scale: float
     correction: torch.Tensor      # [experts] fp32
+    softmax: bool = False         # scores: softmax over all outputs, else sigmoid
+    renorm: bool = True           # weights over their sum
+
+
+@dataclasses.dataclass(frozen=True)
+class Glu:
+    """Constants of an expert's gated activation: g = min(gate, limit), g sigmoid(alpha g) (clamp(up, +-limit) + beta)."""
+    limit: float = INF
+    alpha: float = 1.0
+    beta: float = 0.0
+
+    def args(self):
+        return [float(self.limit), float(self.alpha), float(self.beta)]
 
 
 class ExpertWeights:
@@ -75,7 +88,7 @@ class ExpertWeights:
 def route(logits: Cols, r: Router) -> tuple[torch.Tensor, torch.Tensor]:
     """(expert per (token, choice) int32, weight fp32) of the router logits' fp32 slabs."""
     if not logits.t.is_cuda:
-        return ref.route(logits.value(), r.correction, r.groups, r.keep, r.top, r.scale)
+        return ref.route(logits.value(), r.correction, r.groups, r.keep, r.top, r.scale, r.softmax, r.renorm)
     if not logits.slabs:
         raise ValueError("route: fp32 slabs needed")
     T = logits.rows
@@ -83,7 +96,8 @@ def route(logits: Cols, r: Router) -> tuple[torch.Tensor, torch.Tensor]:
     w = torch.empty(T, r.top, dtype=torch.float32, device=logits.t.device)
     p, split, ld, plane = logits.args()
     check(kernels().cfc_moe_route(p, split, ld, plane, r.correction.data_ptr(), T, r.experts, r.groups, r.keep, r.top,
-                                  float(r.scale), ids.data_ptr(), w.data_ptr(), _stream(ids)), "cfc_moe_route")
+                                  float(r.scale), int(r.softmax), int(r.renorm), ids.data_ptr(), w.data_ptr(), _stream(ids)),
+          "cfc_moe_route")
     return ids, w
 
 
@@ -102,20 +116,21 @@ def sort_rows(ids, experts: int, tile: int):
     return rows, pos, te
 
 
-def _grouped(glu, x, w, E, N, bn, tile, rows, te, out):
-    """One grouped product over packed weights."""
+def _grouped(glu: Glu | None, x, w, E, N, bn, tile, rows, te, out):
+    """One grouped product over packed weights, gated with ``glu``."""
     M, Kd, lib = te.numel() * tile, x.shape[1], kernels()
     if not x.is_contiguous() or out.shape[0] != M:
         raise ValueError(f"grouped product: x {tuple(x.shape)}, out {tuple(out.shape)} for {M} rows")
+    on, consts = int(glu is not None), (glu or Glu()).args()
     if tile == 256:
-        check(lib.cfc_pgemm_group(glu, x.data_ptr(), x.shape[0], w.data_ptr(), M, N, Kd, bn // 16, _p(rows), te.data_ptr(),
-                                  out.data_ptr(), out.stride(0), INF, 1.0, 0.0, _stream(x)), "cfc_pgemm_group")
+        check(lib.cfc_pgemm_group(on, x.data_ptr(), x.shape[0], w.data_ptr(), M, N, Kd, bn // 16, _p(rows), te.data_ptr(),
+                                  out.data_ptr(), out.stride(0), *consts, _stream(x)), "cfc_pgemm_group")
     else:
-        check(lib.cfc_dgemm_group(glu, x.data_ptr(), w.data_ptr(), M, N, Kd, bn, tile, _p(rows), te.data_ptr(), out.data_ptr(),
-                                  out.stride(0), INF, 1.0, 0.0, _stream(x)), "cfc_dgemm_group")
+        check(lib.cfc_dgemm_group(on, x.data_ptr(), w.data_ptr(), M, N, Kd, bn, tile, _p(rows), te.data_ptr(), out.data_ptr(),
+                                  out.stride(0), *consts, _stream(x)), "cfc_dgemm_group")
 
 
-def _experts_gemv(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
+def _experts_gemv(x, w: ExpertWeights, ids, glu: Glu) -> tuple[torch.Tensor, torch.Tensor]:
     """Few pairs: each streams its expert's matrices, in the pairs' own order."""
     T, top = ids.shape
     pairs, lib, dev = T * top, kernels(), x.device
@@ -123,7 +138,7 @@ def _experts_gemv(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]
     part = K._workspace(dev, split * pairs * 2 * w.F)[:split * pairs * 2 * w.F].view(split, pairs, 2 * w.F)
     check(lib.cfc_gemv_group(x.data_ptr(), w.gu.data_ptr(), ids.data_ptr(), pairs, top, w.E, 2 * w.F, w.W, w.bn_gu // 16, 0,
                              part.data_ptr(), None, split, waves, _stream(x)), "cfc_gemv_group")
-    a = clamped_glu(part, torch.empty(pairs, w.F, dtype=x.dtype, device=dev), INF, 1.0, 0.0, interleaved=True)
+    a = clamped_glu(part, torch.empty(pairs, w.F, dtype=x.dtype, device=dev), *glu.args(), interleaved=True)
     y = torch.empty(pairs, w.W, dtype=x.dtype, device=dev)
     _, waves = K.gemv_packed_config(pairs * w.W, w.F, w.bn_down // 16, slab=False)
     check(lib.cfc_gemv_group(a.data_ptr(), w.down.data_ptr(), ids.data_ptr(), pairs, 1, w.E, w.W, w.F, w.bn_down // 16, 1, None,
@@ -131,12 +146,13 @@ def _experts_gemv(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]
     return y, w.pair_order[:pairs].view(T, top)
 
 
-def experts(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
-    """W_down (silu(W_gate x) * W_up x) of every (token, choice): (rows [M, W] in x's dtype, row per pair [T, top])."""
+def experts(x, w: ExpertWeights, ids, glu: Glu = Glu()) -> tuple[torch.Tensor, torch.Tensor]:
+    """W_down glu(W_gate x, W_up x) of every (token, choice): (rows [M, W] in x's dtype, row per pair [T, top]).  Choices
+    past the last expert have no row of their own: what their place holds does not count."""
     if w.packed and ids.numel() <= GEMV_PAIRS and x.is_contiguous():
         _req(x, torch.bfloat16, "x")
         _req(ids, torch.int32, "ids")
-        return _experts_gemv(x, w, ids)
+        return _experts_gemv(x, w, ids, glu)
     tile = w.tile(ids.numel())
     rows, pos, te = sort_rows(ids, w.E, tile)
     M = te.numel() * tile
@@ -149,19 +165,19 @@ def experts(x, w: ExpertWeights, ids) -> tuple[torch.Tensor, torch.Tensor]:
             s = slice(i * tile, (i + 1) * tile)
             gu = x[rows[s].long()].float() @ w.gu[e].float().t()
             g, u = gu.chunk(2, -1)
-            a = (g * torch.sigmoid(g) * u).to(x.dtype)
+            a = ref.clamped_glu(g, u, *glu.args()).to(x.dtype)
             y[s] = (a.float() @ w.down[e].float().t()).to(x.dtype)
         return y, pos
     a = torch.empty(M, w.F, dtype=x.dtype, device=x.device)
     if w.packed:
-        _grouped(1, x, w.gu, w.E, 2 * w.F, w.bn_gu, tile, rows, te, a)
-        _grouped(0, a, w.down, w.E, w.W, w.bn_down, tile, None, te, y)
+        _grouped(glu, x, w.gu, w.E, 2 * w.F, w.bn_gu, tile, rows, te, a)
+        _grouped(None, a, w.down, w.E, w.W, w.bn_down, tile, None, te, y)
         return y, pos
     lib, f32 = kernels(), _act(x.dtype)
     if x.dtype != w.dtype or not x.is_contiguous():
         raise ValueError(f"experts: activations {x.dtype}, weights {w.dtype}")
     check(lib.cfc_moe_any(f32, 1, x.data_ptr(), w.gu.data_ptr(), M, w.F, w.W, rows.data_ptr(), te.data_ptr(), tile, a.data_ptr(),
-                          w.F, _stream(x)), "cfc_moe_any")
+                          w.F, *glu.args(), _stream(x)), "cfc_moe_any")
     check(lib.cfc_moe_any(f32, 0, a.data_ptr(), w.down.data_ptr(), M, w.W, w.F, None, te.data_ptr(), tile, y.data_ptr(), w.W,
-                          _stream(x)), "cfc_moe_any")
+                          *Glu().args(), _stream(x)), "cfc_moe_any")
     return y, pos

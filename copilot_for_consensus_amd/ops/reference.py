@@ -475,10 +475,11 @@ def wkv_out(o, norm, gate, eps):
 
 
 # ----------------------------------------------------- routed experts (moe.hip)
-def route(logits, correction, groups, keep, top, scale):
-    """logits [T, E] fp32: (ids [T, top], weights [T, top]).  Sigmoid scores; the choice adds ``correction``; a
-    group counts by its two largest choice scores and only the best ``keep`` groups take part."""
-    s = torch.sigmoid(logits)
+def route(logits, correction, groups, keep, top, scale, softmax=False, renorm=True):
+    """logits [T, E] fp32: (ids [T, top], weights [T, top]).  Sigmoid (or softmax) scores; the choice adds
+    ``correction``; a group counts by its two largest choice scores and only the best ``keep`` groups take part.  The
+    weights are the chosen scores, over their sum with ``renorm``."""
+    s = torch.softmax(logits, -1) if softmax else torch.sigmoid(logits)
     c = s + correction
     T, E = c.shape
     g = c.view(T, groups, E // groups)
@@ -487,18 +488,19 @@ def route(logits, correction, groups, keep, top, scale):
     c = c.masked_fill(~kept.repeat_interleave(E // groups, 1), float("-inf"))
     ids = c.topk(top, -1).indices
     w = s.gather(1, ids)
-    return ids.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
+    return ids.to(torch.int32), (w / (w.sum(-1, keepdim=True) + 1e-20) if renorm else w) * scale
 
 
 def moe_rows(ids, experts, tile):
     """Rows of (token, choice) pairs sorted by expert, every expert's rows padded to whole tiles: (token per row
-    [M], row per pair [T, top], expert per tile [M / tile]), pad rows token 0, tiles past the last -1."""
+    [M], row per pair [T, top], expert per tile [M / tile]), pad rows token 0, tiles past the last -1.  Choices past the
+    last expert take no row (their row per pair is 0)."""
     T, top = ids.shape
     n_tiles = moe_max_tiles(T * top, experts, tile)
     rows, pos, te = np.zeros(n_tiles * tile, np.int32), np.zeros((T, top), np.int32), np.full(n_tiles, -1, np.int32)
     at = 0
     for e in range(experts):
-        pairs = [(t, c) for t in range(T) for c in range(top) if int(ids[t, c]) == e]
+        pairs = (ids == e).nonzero().tolist()
         for i, (t, c) in enumerate(pairs):
             rows[at + i], pos[t, c] = t, at + i
         m = -(-len(pairs) // tile)
@@ -510,3 +512,79 @@ def moe_rows(ids, experts, tile):
 def moe_max_tiles(pairs: int, experts: int, tile: int) -> int:
     """Most tiles that ``pairs`` rows over ``experts`` experts can take."""
     return min(pairs, pairs // tile + min(experts, pairs))
+
+
+# ----------------------------------------------------- branches between two norms (branch.hip)
+def rms_rows(x, eps):
+    return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+
+def relu_sq(x):
+    return torch.clamp(x, min=0.0).square()
+
+
+# ----------------------------------------------------- minimal gated recurrence (gru.hip)
+def min_gru(z, u, S):
+    """Pre-activations of gate and candidate [T, C], S [C] (updated): the states S_t [T, C]."""
+    g, c = torch.sigmoid(z), torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    a, out = torch.sigmoid(-z), torch.empty_like(z)
+    for t in range(z.shape[0]):
+        S.mul_(a[t]).add_(g[t] * c[t])
+        out[t] = S
+    return out
+
+
+# ----------------------------------------------------- grouped attention over two key ranges (qkv.hip, gqa.hip)
+def conv_over_time(u, w, lead, positions, slots, tail):
+    """u [T, C] fp32, w [taps, C]: y_t = sum_d w[taps - 1 - d] u_(t - d) inside each sequence.  ``lead`` rows of the same
+    portion lie before a row; older inputs from ``tail`` [slots, taps - 1, C] (position p at row p % (taps - 1))."""
+    taps, y = w.shape[0], u * w[-1]
+    for t, (n, p) in enumerate(zip(lead.tolist(), positions.tolist())):
+        for d in range(1, min(taps - 1, p) + 1):
+            y[t] += w[taps - 1 - d] * (u[t - d] if d <= n else tail[int(slots[t]), (p - d) % (taps - 1)])
+    return y
+
+
+def head_norm(x, w, eps, per_head, heads):
+    """RMS norm of x [T, heads * dim] over all of it, or per head (``w`` [dim])."""
+    if not per_head:
+        return rms_rows(x, eps) * w
+    return (rms_rows(x.view(x.shape[0], heads, -1), eps) * w).flatten(1)
+
+
+def rotate_heads(x, positions, freq):
+    """The first 2 len(freq) dimensions of x [T, heads, dim] turned in neighbouring pairs."""
+    n = 2 * freq.numel()
+    return torch.cat([rotate_pairs(x[..., :n], positions, freq, 1.0), x[..., n:]], -1)
+
+
+def paged_rows(cache, table, n):
+    """The first n rows [n, G, D] of a sequence in a cache [blocks, G, entries, D]."""
+    e = cache.shape[2]
+    return cache[table[:-(-n // e)].long()].transpose(1, 2).reshape(-1, cache.shape[1], cache.shape[3])[:n]
+
+
+def grouped_attention(q, k, v, pooled, block_tables, cu_q, ctx_lens, size, keep, pool, sink, vdim):
+    """q [T, H, D] scaled by log2(e); k, v [blocks, G, 32, D], ``pooled`` their block means [blocks, G, E, D] (pool > 0).
+    A row sees its last ``size`` keys (0: all), the first ``keep``, and the means of blocks of ``pool`` keys wholly ahead
+    of the window; exp(sink) joins the denominator."""
+    T, H, D = q.shape
+    out = torch.empty(T, H * vdim, dtype=q.dtype)
+    for s in range(len(ctx_lens)):
+        a, b, ctx = int(cu_q[s]), int(cu_q[s + 1]), int(ctx_lens[s])
+        K, V = (paged_rows(c, block_tables[s], ctx).float() for c in (k, v))
+        pos, j = torch.arange(ctx - (b - a), ctx)[:, None], torch.arange(ctx)[None]
+        see = (j <= pos) & ((pos - j < size) | (j < keep)) if size else j <= pos
+        n = max(ctx - size, 0) // pool if pool else 0
+        if n:
+            PK, PV = (paged_rows(c, block_tables[s], n).float() for c in pooled)
+            K, V = torch.cat([K, PK]), torch.cat([V, PV])
+            see = torch.cat([see, torch.arange(n)[None] < (pos - size + 1).clamp(min=0) // pool], 1)
+        for h in range(H):
+            g = h * K.shape[1] // H
+            sc = (q[a:b, h].float() @ K[:, g].t() * math.log(2.0)).masked_fill(~see, float("-inf"))
+            if sink is not None:
+                sc = torch.cat([sc, sink[h].expand(b - a, 1)], 1)
+            p = torch.softmax(sc, -1)[:, :K.shape[0]]
+            out[a:b, h * vdim:(h + 1) * vdim] = (p @ V[:, g, :vdim]).to(q.dtype)
+    return out

@@ -184,5 +184,53 @@ class HybridCache:
         return sum(t.numel() * t.element_size() for t in (*self.rows, *self.recur, *self.prev) if t is not None)
 
 
+class PagedHeads:
+    """Keys and values of one attention layer, row-major: ``k``, ``v`` [blocks, G, 32, D]; with ``pool`` the mean keys and
+    values of blocks of ``pool`` tokens ``pk``, ``pv`` [blocks, G, entries, D], entry b of a sequence in block b // entries
+    of its table (ops.gqa.pool_entries: allocated by the time token block b is complete)."""
+
+    def __init__(self, num_blocks: int, heads: int, dim: int, pool: int, entries: int, device, dtype):
+        def zeros(n):
+            # the slots of a partly filled block are read (then masked)
+            return torch.zeros(num_blocks, heads, n, dim, dtype=dtype, device=device)
+        self.k, self.v, self.pool = zeros(KV_BLOCK), zeros(KV_BLOCK), pool
+        self.pk, self.pv = (zeros(entries), zeros(entries)) if pool else (None, None)
+        self.log2_entries = entries.bit_length() - 1 if pool else 0
+
+    def tensors(self):
+        return [t for t in (self.k, self.v, self.pk, self.pv) if t is not None]
+
+
+class GroupedCache:
+    """Cache of a decoder of grouped-query attention layers and recurrences, on the same blocks and :class:`BlockPool` as
+    :class:`PagedKVCache`, with state slots per sequence.  Per layer:
+      heads  :class:`PagedHeads`, or the very object of an earlier layer whose keys and values the layer uses
+      tail   [slots + 1, taps - 1, channels] fp32 or None   last inputs of the convolution, position p at p % (taps - 1)
+      recur  [slots + 1, width] fp32 or None                recurrent state
+    A sequence's state is not in its blocks, so blocks cannot be shared between sequences.  A slot needs no clearing:
+    what lies before a sequence's first token is never read."""
+
+    share_prefix = False
+
+    def __init__(self, layers: list[dict], num_blocks: int, sequences: int, device, dtype=torch.bfloat16):
+        """``layers``: per layer ``heads`` (G, D, pool, entries) or the index of the layer whose it uses, ``tail``
+        (taps - 1, channels) or None, ``recur`` width or None."""
+        self.layers, self.num_blocks = len(layers), num_blocks
+        self.dtype, self.device = dtype, torch.device(device)
+        self.states = StateSlots(sequences)
+        n, f32 = sequences + 1, dict(dtype=torch.float32, device=self.device)
+        self.heads: list[PagedHeads] = []
+        for c in layers:
+            h = c["heads"]
+            self.heads.append(self.heads[h] if isinstance(h, int) else PagedHeads(num_blocks, *h, self.device, dtype))
+        self.tail = [torch.zeros(n, *c["tail"], **f32) if c.get("tail") else None for c in layers]
+        self.recur = [torch.zeros(n, c["recur"], **f32) if c.get("recur") else None for c in layers]
+        self.pool = BlockPool(num_blocks)
+
+    def nbytes(self) -> int:
+        rows = [t for h in {id(h): h for h in self.heads}.values() for t in h.tensors()]
+        return sum(t.numel() * t.element_size() for t in (*rows, *self.tail, *self.recur) if t is not None)
+
+
 def blocks_needed(n_tokens: int) -> int:
     return math.ceil(n_tokens / KV_BLOCK)

@@ -1,0 +1,207 @@
+// Minimal gated recurrence: gate and candidate read the current token only, so the state is a linear recurrence
+//   S_t = (1 - z_t) S_(t-1) + z_t c_t,   z = sigmoid(pre_z + bz),   c = u + 1/2 (u >= 0) or sigmoid(u),  u = pre_x + bx
+// element by element, and the layer's output S_t silu(pre_g).  States are fp32, one row per sequence slot; a sequence's
+// first token starts from zero whatever the slot holds.
+//   * gru_step    one token per sequence, straight from a joint product's slabs
+//   * gru_chunk   prompt portions, chunks of 64 tokens in parallel: each chunk's decay (the product of 1 - z) and what
+//                 it adds to a state of zero
+//   * gru_carry   per sequence through its chunks: the state ahead of each, and the one the portion leaves
+//   * gru_apply   the chunks again from their states: outputs
+#include "rows.h"
+
+namespace {
+
+struct GruCols { const void* p; int split; int64_t ld, plane; };      // split 0: activations, else fp32 slabs
+
+template <typename ACT, int V>
+__device__ __forceinline__ Vec<V> gru_ld(const GruCols& a, int64_t t, int c) {
+  const int64_t o = t * a.ld + c;
+  if (a.split == 0) return ldv<V>(reinterpret_cast<const ACT*>(a.p) + o);
+  Vec<V> y = zerov<V>();
+  add_slabs<V>(y, reinterpret_cast<const float*>(a.p), a.split, a.plane, (size_t)o);
+  return y;
+}
+
+__device__ __forceinline__ float sigm(float z) { return 1.f / (1.f + expf(-z)); }
+
+// decay 1 - z and contribution z c of one token
+__device__ __forceinline__ void gru_gates(float pz, float u, float& a, float& b) {
+  a = sigm(-pz);
+  b = sigm(pz) * (u >= 0.f ? u + 0.5f : sigm(u));
+}
+
+template <typename ACT, int V>
+__global__ void __launch_bounds__(64) gru_step_kernel(GruCols z, GruCols u, GruCols g, const float* __restrict__ bz,
+                                                     const float* __restrict__ bx, const int32_t* __restrict__ slots,
+                                                     const int32_t* __restrict__ ctx_lens, int W, float* __restrict__ state,
+                                                     ACT* __restrict__ out) {
+  const int b = blockIdx.x, c = (blockIdx.y * 64 + threadIdx.x) * V;
+  if (c >= W) return;
+  float* sp = state + (size_t)slots[b] * W + c;
+  Vec<V> S = ctx_lens[b] > 1 ? ldv<V>(sp) : zerov<V>();
+  const Vec<V> zv = gru_ld<ACT, V>(z, b, c), uv = gru_ld<ACT, V>(u, b, c), gv = gru_ld<ACT, V>(g, b, c);
+  const Vec<V> vz = ldv<V>(bz + c), vx = ldv<V>(bx + c);
+  Vec<V> o;
+#pragma unroll
+  for (int e = 0; e < V; ++e) {
+    float a, k;
+    gru_gates(zv.v[e] + vz.v[e], uv.v[e] + vx.v[e], a, k);
+    S.v[e] = a * S.v[e] + k;
+    o.v[e] = S.v[e] * gv.v[e] * sigm(gv.v[e]);
+  }
+  stv<V>(sp, S);
+  stv<V>(out + (size_t)b * W + c, o);
+}
+
+constexpr int GRU_FLIGHT = 8;        // rows requested ahead of their use
+
+// chunks [n][2]: {first row, rows}; sums [n][2][W]: decay, contribution
+template <typename ACT, int V>
+__global__ void __launch_bounds__(64) gru_chunk_kernel(GruCols z, GruCols u, const float* __restrict__ bz,
+                                                      const float* __restrict__ bx, const int32_t* __restrict__ chunks, int W,
+                                                      float* __restrict__ sums) {
+  const int c = (blockIdx.y * 64 + threadIdx.x) * V;
+  if (c >= W) return;
+  const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
+  const Vec<V> vz = ldv<V>(bz + c), vx = ldv<V>(bx + c);
+  Vec<V> A, B = zerov<V>();
+#pragma unroll
+  for (int e = 0; e < V; ++e) A.v[e] = 1.f;
+  for (int r0 = 0; r0 < n; r0 += GRU_FLIGHT) {
+    Vec<V> zv[GRU_FLIGHT], uv[GRU_FLIGHT];
+#pragma unroll
+    for (int i = 0; i < GRU_FLIGHT; ++i) {
+      const int64_t t = row0 + min(r0 + i, n - 1);
+      zv[i] = gru_ld<ACT, V>(z, t, c);
+      uv[i] = gru_ld<ACT, V>(u, t, c);
+    }
+#pragma unroll
+    for (int i = 0; i < GRU_FLIGHT; ++i)
+      if (r0 + i < n)
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          float a, k;
+          gru_gates(zv[i].v[e] + vz.v[e], uv[i].v[e] + vx.v[e], a, k);
+          A.v[e] *= a;
+          B.v[e] = a * B.v[e] + k;
+        }
+  }
+  float* o = sums + (size_t)blockIdx.x * 2 * W + c;
+  stv<V>(o, A);
+  stv<V>(o + W, B);
+}
+
+// sums[chunk][0] becomes the state ahead of the chunk
+template <int V>
+__global__ void __launch_bounds__(64) gru_carry_kernel(const int32_t* __restrict__ chunk_cu, const int32_t* __restrict__ cu_q,
+                                                      const int32_t* __restrict__ ctx_lens, const int32_t* __restrict__ slots,
+                                                      int W, float* __restrict__ sums, float* __restrict__ state) {
+  const int s = blockIdx.x, c = (blockIdx.y * 64 + threadIdx.x) * V;
+  if (c >= W) return;
+  const int i0 = chunk_cu[s], i1 = chunk_cu[s + 1];
+  float* sp = state + (size_t)slots[s] * W + c;
+  Vec<V> S = ctx_lens[s] > cu_q[s + 1] - cu_q[s] ? ldv<V>(sp) : zerov<V>();
+  for (int i = i0; i < i1; i += GRU_FLIGHT) {
+    Vec<V> A[GRU_FLIGHT], B[GRU_FLIGHT];
+#pragma unroll
+    for (int k = 0; k < GRU_FLIGHT; ++k) {
+      const float* p = sums + (size_t)min(i + k, i1 - 1) * 2 * W + c;
+      A[k] = ldv<V>(p);
+      B[k] = ldv<V>(p + W);
+    }
+#pragma unroll
+    for (int k = 0; k < GRU_FLIGHT; ++k)
+      if (i + k < i1) {
+        stv<V>(sums + (size_t)(i + k) * 2 * W + c, S);
+#pragma unroll
+        for (int e = 0; e < V; ++e) S.v[e] = A[k].v[e] * S.v[e] + B[k].v[e];
+      }
+  }
+  stv<V>(sp, S);
+}
+
+template <typename ACT, int V>
+__global__ void __launch_bounds__(64) gru_apply_kernel(GruCols z, GruCols u, GruCols g, const float* __restrict__ bz,
+                                                      const float* __restrict__ bx, const int32_t* __restrict__ chunks, int W,
+                                                      const float* __restrict__ sums, ACT* __restrict__ out) {
+  const int c = (blockIdx.y * 64 + threadIdx.x) * V;
+  if (c >= W) return;
+  const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
+  const Vec<V> vz = ldv<V>(bz + c), vx = ldv<V>(bx + c);
+  Vec<V> S = ldv<V>(sums + (size_t)blockIdx.x * 2 * W + c);
+  for (int r0 = 0; r0 < n; r0 += GRU_FLIGHT) {
+    Vec<V> zv[GRU_FLIGHT], uv[GRU_FLIGHT], gv[GRU_FLIGHT];
+#pragma unroll
+    for (int i = 0; i < GRU_FLIGHT; ++i) {
+      const int64_t t = row0 + min(r0 + i, n - 1);
+      zv[i] = gru_ld<ACT, V>(z, t, c);
+      uv[i] = gru_ld<ACT, V>(u, t, c);
+      gv[i] = gru_ld<ACT, V>(g, t, c);
+    }
+#pragma unroll
+    for (int i = 0; i < GRU_FLIGHT; ++i)
+      if (r0 + i < n) {
+        Vec<V> o;
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          float a, k;
+          gru_gates(zv[i].v[e] + vz.v[e], uv[i].v[e] + vx.v[e], a, k);
+          S.v[e] = a * S.v[e] + k;
+          o.v[e] = S.v[e] * gv[i].v[e] * sigm(gv[i].v[e]);
+        }
+        stv<V>(out + (size_t)(row0 + r0 + i) * W + c, o);
+      }
+  }
+}
+
+// vectors of four where every operand's rows allow them
+bool gru_vec(const GruCols* a, int n, int W, int f32) {
+  bool v = W % 4 == 0;
+  for (int i = 0; i < n; ++i)
+    v = v && a[i].ld % 4 == 0 && a[i].plane % 4 == 0 && ((uintptr_t)a[i].p & (a[i].split == 0 && !f32 ? 7 : 15)) == 0;
+  return v;
+}
+
+}  // namespace
+
+// z, u, g: columns of products (pointer, split (0: activations, else fp32 slabs), row stride, slab stride)
+CFC_API int cfc_gru_step(int f32, const void* z, int z_split, int64_t z_ld, int64_t z_plane, const void* u, int u_split,
+                         int64_t u_ld, int64_t u_plane, const void* g, int g_split, int64_t g_ld, int64_t g_plane, const float* bz,
+                         const float* bx, const int32_t* slots, const int32_t* ctx_lens, int B, int W, float* state, void* out,
+                         hipStream_t stream) {
+  if (B <= 0) return 0;
+  if (W < 1 || !slots || !ctx_lens || !state) return -1;
+  const GruCols a[3] = {{z, z_split, z_ld, z_plane}, {u, u_split, u_ld, u_plane}, {g, g_split, g_ld, g_plane}};
+#define GS(ACT, V) \
+  gru_step_kernel<ACT, V><<<dim3(B, (W + 64 * V - 1) / (64 * V)), 64, 0, stream>>>(a[0], a[1], a[2], bz, bx, slots, ctx_lens, W, state, (ACT*)out)
+  const bool v4 = gru_vec(a, 3, W, f32);
+  if (f32) { if (v4) GS(float, 4); else GS(float, 1); }
+  else if (v4) GS(uint16_t, 4);
+  else GS(uint16_t, 1);
+#undef GS
+  return CFC_CHECK_LAUNCH();
+}
+
+// packed portions; chunks [n][2] {first row, rows}, chunk_cu [portions + 1]; sums scratch [n][2][W]
+CFC_API int cfc_gru_prefill(int f32, const void* z, int z_split, int64_t z_ld, int64_t z_plane, const void* u, int u_split,
+                            int64_t u_ld, int64_t u_plane, const void* g, int g_split, int64_t g_ld, int64_t g_plane,
+                            const float* bz, const float* bx, const int32_t* chunks, int n, const int32_t* chunk_cu,
+                            const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* slots, int portions, int W, float* sums,
+                            float* state, void* out, hipStream_t stream) {
+  if (n <= 0 || portions <= 0) return 0;
+  if (W < 1 || !chunks || !chunk_cu || !cu_q || !ctx_lens || !slots || !sums || !state) return -1;
+  const GruCols a[3] = {{z, z_split, z_ld, z_plane}, {u, u_split, u_ld, u_plane}, {g, g_split, g_ld, g_plane}};
+#define GP(ACT, V)                                                                                                    \
+  do {                                                                                                                \
+    const int gy = (W + 64 * V - 1) / (64 * V);                                                                       \
+    gru_chunk_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(a[0], a[1], bz, bx, chunks, W, sums);                    \
+    gru_carry_kernel<V><<<dim3(portions, gy), 64, 0, stream>>>(chunk_cu, cu_q, ctx_lens, slots, W, sums, state);      \
+    gru_apply_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(a[0], a[1], a[2], bz, bx, chunks, W, sums, (ACT*)out);   \
+  } while (0)
+  const bool v4 = gru_vec(a, 3, W, f32);
+  if (f32) { if (v4) GP(float, 4); else GP(float, 1); }
+  else if (v4) GP(uint16_t, 4);
+  else GP(uint16_t, 1);
+#undef GP
+  return CFC_CHECK_LAUNCH();
+}

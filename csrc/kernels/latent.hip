@@ -12,11 +12,11 @@
 //   * latent_attn     flash-style attention over the paged latents.  A work item is 16 MR rows of the
 //                     flattened (token, head) rows of one sequence -- one decoded token's heads and a
 //                     prompt portion's rows are the same thing to it -- and a slice of its keys
-//   * latent_combine  merges the slices
+//   * slice_merge     merges the slices (split_merge.h)
 //   * latent_gather   the latents of whole sequences as dense rows, in token order and in the slot order
 //                     of the prefill attention's V^T: two products turn them into per-head keys and
 //                     values for long portions, where that costs fewer flops (attention.hip, EXP)
-#include "common.h"
+#include "split_merge.h"
 
 namespace {
 
@@ -899,60 +899,6 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(const uint16_t* __re
     }
 }
 
-// one workgroup of 128 threads per (token, head) row; P <= LC_MAXP
-constexpr int LC_MAXP = 256;
-template <typename ACT>
-__global__ void __launch_bounds__(128) latent_combine_kernel(const float* __restrict__ part_o,
-                                                            const float* __restrict__ part_ml, int P, int RS,
-                                                            const float* __restrict__ sink, int H, ACT* __restrict__ out) {
-  __shared__ float wt[LC_MAXP];
-  const size_t row = blockIdx.x;
-  const float* ml = part_ml + row * P * 2;
-  // every wave computes the weights (at most four slices per lane), the first stores them
-  const int lane = threadIdx.x & 63;
-  float m[LC_MAXP / 64], l[LC_MAXP / 64], mx = -INFINITY;
-#pragma unroll
-  for (int i = 0; i < LC_MAXP / 64; ++i) {
-    const int p = lane + 64 * i;
-    m[i] = p < P ? ml[2 * p] : -INFINITY;
-    l[i] = p < P ? ml[2 * p + 1] : 0.f;
-    mx = fmaxf(mx, m[i]);
-  }
-  mx = wave_max(mx);
-  const float sk = sink ? sink[row % H] * 1.4426950408889634f : -INFINITY;
-  mx = fmaxf(mx, sk);
-  const float ref = mx == -INFINITY ? 0.f : mx;
-  float sum = 0.f;
-#pragma unroll
-  for (int i = 0; i < LC_MAXP / 64; ++i) {
-    m[i] = exp2f(m[i] - ref);
-    sum += m[i] * l[i];
-  }
-  sum = wave_sum(sum) + exp2f(sk - ref);          // no sink: 0
-  const float inv = sum > 0.f ? 1.f / sum : 0.f;
-  if (threadIdx.x < 64) {
-#pragma unroll
-    for (int i = 0; i < LC_MAXP / 64; ++i)
-      if (lane + 64 * i < P) wt[lane + 64 * i] = m[i] * inv;
-  }
-  __syncthreads();
-  for (int c = threadIdx.x * 4; c < RS; c += 512) {
-    float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
-    for (int p0 = 0; p0 < P; p0 += 8) {          // eight slices in flight (past the last: re-read, weight 0)
-      float4 v[8];
-#pragma unroll
-      for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const float4*>(part_o + (row * P + min(p0 + u, P - 1)) * RS + c);
-#pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const float e = p0 + u < P ? wt[p0 + u] : 0.f;
-        s.x += e * v[u].x; s.y += e * v[u].y; s.z += e * v[u].z; s.w += e * v[u].w;
-      }
-    }
-    ACT* o = out + row * RS + c;
-    stf(o, s.x); stf(o + 1, s.y); stf(o + 2, s.z); stf(o + 3, s.w);
-  }
-}
-
 template <int R64, int V64, int MR>
 int lat_go(dim3 grid, hipStream_t s, const void* q, const void* cache, const LatArgs& a, void* out) {
   constexpr int lds = 2 * 64 * R64 * 2 + 16 * MR * LP * 2 + (MR * 64 + 16 * MR) * 4;
@@ -1069,7 +1015,7 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
                                  int RV, int max_blocks, float scale, int window, const float* sink, int P, int total_rows, float* part_o, float* part_ml,
                                  void* out, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (H < 1 || RS < 32 || RS % 32 || RV < 32 || RV % 32 || RV > RS || P < 1 || P > LC_MAXP || max_blocks < 1 || window < 0)
+  if (H < 1 || RS < 32 || RS % 32 || RV < 32 || RV % 32 || RV > RS || P < 1 || P > MERGE_MAXP || max_blocks < 1 || window < 0)
     return -1;
   if ((tile_seq == nullptr) != (tile_m0 == nullptr) || (!tile_seq && tiles_per_seq < 1)) return -1;
   if (P > 1 && (!part_o || !part_ml)) return -2;
@@ -1102,8 +1048,8 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
 #undef LAT
   }
   if (rc || P == 1) return rc;
-  if (f32) latent_combine_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, sink, H, (float*)out);
-  else latent_combine_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, sink, H, (uint16_t*)out);
+  if (f32) slice_merge_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, RV, sink, H, (float*)out);
+  else slice_merge_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, RV, sink, H, (uint16_t*)out);
   return CFC_CHECK_LAUNCH();
 }
 

@@ -1,9 +1,10 @@
 // Routed experts (mixture of experts):
-//   * moe_route   sigmoid scores of the router logits; experts chosen by score + correction among the best
-//                 groups; weights from the scores alone.  One wave per token
+//   * moe_route   sigmoid or softmax scores of the router logits; experts chosen by score + correction among the
+//                 best groups; weights from the scores alone, over their sum or as they are.  One wave per token
 //   * moe_rows    the (token, choice) pairs sorted by expert, each expert's rows padded to whole tiles: what the
 //                 grouped products (dgemm.hip, pgemm.hip) and the gather of their results go by.  Nothing
-//                 comes back to the host, so a captured decode step routes anew on every replay
+//                 comes back to the host, so a captured decode step routes anew on every replay.  Choices past
+//                 the last expert (outputs of the router without matrices) take no row
 //   * moe_any     grouped products of any shape and both activation types (the 32-bit path, odd widths)
 #include "common.h"
 
@@ -20,7 +21,8 @@ constexpr int MR_MAXE = 1024;
 template <int NE>
 __global__ void __launch_bounds__(256) moe_route_kernel(const float* __restrict__ logits, int split, int64_t ld, int64_t plane,
                                                        const float* __restrict__ correction, int T, int E, int groups, int keep,
-                                                       int top, float scale, int32_t* __restrict__ ids, float* __restrict__ weights) {
+                                                       int top, float scale, int softmax, int renorm, int32_t* __restrict__ ids,
+                                                       float* __restrict__ weights) {
   __shared__ float choice[4][64 * NE], gscore[4][MR_MAXE];
   __shared__ int kept[4][MR_MAXE];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, t = blockIdx.x * 4 + w;
@@ -38,12 +40,30 @@ __global__ void __launch_bounds__(256) moe_route_kernel(const float* __restrict_
 #pragma unroll
         for (int u = 0; u < 16; ++u) z += p0 + u < split ? v[u] : 0.f;
       }
-    s[i] = 1.f / (1.f + expf(-z));
+    s[i] = softmax ? (e < E ? z : -INFINITY) : 1.f / (1.f + expf(-z));
+  }
+  if (softmax) {
+    float mx = -INFINITY, all = 0.f;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) mx = fmaxf(mx, s[i]);
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      s[i] = expf(s[i] - mx);
+      all += s[i];
+    }
+    all = wave_sum(all);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) s[i] /= all;
+  }
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
     c[i] = e < E ? s[i] + correction[min(e, E - 1)] : -INFINITY;
     choice[w][e] = c[i];
   }
   __syncthreads();
-  for (int g = lane; g < groups; g += 64) {
+  for (int g = keep < groups ? lane : groups; g < groups; g += 64) {
     float a = -INFINITY, b = -INFINITY;           // the two largest
     for (int i = 0; i < size; ++i) {
       const float v = choice[w][g * size + i];
@@ -53,7 +73,7 @@ __global__ void __launch_bounds__(256) moe_route_kernel(const float* __restrict_
     gscore[w][g] = size > 1 ? a + b : a;
   }
   __syncthreads();
-  for (int g = lane; g < groups; g += 64) {
+  for (int g = keep < groups ? lane : groups; g < groups; g += 64) {
     const float v = gscore[w][g];
     int better = 0;
     for (int o = 0; o < groups; ++o) better += gscore[w][o] > v || (gscore[w][o] == v && o < g);
@@ -63,7 +83,7 @@ __global__ void __launch_bounds__(256) moe_route_kernel(const float* __restrict_
 #pragma unroll
   for (int i = 0; i < NE; ++i) {
     const int e = lane + 64 * i;
-    if (e < E && !kept[w][e / size]) c[i] = -INFINITY;
+    if (keep < groups && e < E && !kept[w][e / size]) c[i] = -INFINITY;
   }
   float mine = 0.f, sum = 0.f;
   int mine_id = 0;
@@ -87,7 +107,7 @@ __global__ void __launch_bounds__(256) moe_route_kernel(const float* __restrict_
   }
   if (t < T && lane < top) {
     ids[(size_t)t * top + lane] = mine_id;
-    weights[(size_t)t * top + lane] = mine / (sum + 1e-20f) * scale;
+    weights[(size_t)t * top + lane] = (renorm ? mine / (sum + 1e-20f) : mine) * scale;
   }
 }
 
@@ -100,7 +120,11 @@ __global__ void __launch_bounds__(1024) moe_rows_kernel(const int32_t* __restric
   for (int i = tid; i < E; i += 1024) count[i] = 0;
   if (tid == 0) base_s = 0;
   __syncthreads();
-  for (int p = tid; p < pairs; p += 1024) atomicAdd(&count[ids[p]], 1);
+  for (int p = tid; p < pairs; p += 1024) {
+    const int i = ids[p];
+    if (i < E) atomicAdd(&count[i], 1);
+    else if (e == 0) pos[p] = 0;               // no row of its own: a place that exists
+  }
   __syncthreads();
   for (int i = tid; i < e; i += 1024) atomicAdd(&base_s, (count[i] + tile - 1) / tile);
   __syncthreads();
@@ -136,11 +160,13 @@ __global__ void __launch_bounds__(1024) moe_rows_kernel(const int32_t* __restric
 }
 
 // Row-major W [experts][GLU ? 2 N : N][K]; 32 rows x 64 columns per workgroup, K in steps of 16 through LDS.
-// GLU: columns n of the gate rows 0 .. N - 1 and of the up rows N .. 2 N - 1, silu(g) u; else the product
+// GLU: columns n of the gate rows 0 .. N - 1 and of the up rows N .. 2 N - 1, g = min(gate, limit):
+// g sigmoid(alpha g) (clamp(up, +-limit) + beta); else the product
 template <typename ACT, bool GLU>
 __global__ void __launch_bounds__(256) moe_any_kernel(const ACT* __restrict__ x, const ACT* __restrict__ W, int N, int K,
                                                      const int32_t* __restrict__ rows, const int32_t* __restrict__ tile_expert,
-                                                     int tile, void* __restrict__ out, int ldo) {
+                                                     int tile, void* __restrict__ out, int ldo, float limit, float alpha,
+                                                     float beta) {
   constexpr int NM = GLU ? 2 : 1;
   __shared__ float xs[16][33], wsm[NM][16][65];
   const int m0 = blockIdx.y * 32, n0 = blockIdx.x * 64, e = tile_expert[m0 / tile], tid = threadIdx.x;
@@ -177,8 +203,8 @@ __global__ void __launch_bounds__(256) moe_any_kernel(const ACT* __restrict__ x,
       const int m = m0 + 2 * tm + a, n = n0 + tn + 16 * b;
       if (n >= N) continue;
       if constexpr (GLU) {
-        const float g = acc[0][a][b];
-        st1(reinterpret_cast<ACT*>(out) + (size_t)m * ldo + n, g / (1.f + expf(-g)) * acc[NM - 1][a][b]);
+        const float g = fminf(acc[0][a][b], limit), u = fminf(fmaxf(acc[NM - 1][a][b], -limit), limit);
+        st1(reinterpret_cast<ACT*>(out) + (size_t)m * ldo + n, g / (1.f + expf(-alpha * g)) * (u + beta));
       } else {
         st1(reinterpret_cast<ACT*>(out) + (size_t)m * ldo + n, acc[0][a][b]);
       }
@@ -188,13 +214,14 @@ __global__ void __launch_bounds__(256) moe_any_kernel(const ACT* __restrict__ x,
 }  // namespace
 
 CFC_API int cfc_moe_route(const float* logits, int split, int64_t ld, int64_t plane, const float* correction, int T, int E,
-                          int groups, int keep, int top, float scale, int32_t* ids, float* weights, hipStream_t stream) {
+                          int groups, int keep, int top, float scale, int softmax, int renorm, int32_t* ids, float* weights,
+                          hipStream_t stream) {
   if (T <= 0) return 0;
   if (E < 1 || E > MR_MAXE || groups < 1 || E % groups || keep < 1 || keep > groups || top < 1 || top > 64 ||
       top > keep * (E / groups) || split < 1)
     return -1;
 #define MO(NE) \
-  moe_route_kernel<NE><<<(T + 3) / 4, 256, 0, stream>>>(logits, split, ld, plane, correction, T, E, groups, keep, top, scale, ids, weights)
+  moe_route_kernel<NE><<<(T + 3) / 4, 256, 0, stream>>>(logits, split, ld, plane, correction, T, E, groups, keep, top, scale, softmax, renorm, ids, weights)
   if (E <= 64) MO(1);
   else if (E <= 128) MO(2);
   else if (E <= 256) MO(4);
@@ -215,11 +242,11 @@ CFC_API int cfc_moe_rows(const int32_t* ids, int pairs, int top, int E, int tile
 
 // M sorted rows in tiles of `tile` (a multiple of 32), activations [M][N] of row stride ldo
 CFC_API int cfc_moe_any(int f32, int glu, const void* x, const void* w, int M, int N, int K, const int32_t* rows,
-                        const int32_t* tile_expert, int tile, void* out, int ldo, hipStream_t stream) {
+                        const int32_t* tile_expert, int tile, void* out, int ldo, float limit, float alpha, float beta, hipStream_t stream) {
   if (M == 0) return 0;
   if (M < 0 || N < 1 || K < 1 || tile < 32 || tile % 32 || M % tile || ldo < N || M / 32 > 65535 || !tile_expert) return -1;
   const dim3 grid((N + 63) / 64, M / 32);
-#define MA(ACT, G) moe_any_kernel<ACT, G><<<grid, 256, 0, stream>>>((const ACT*)x, (const ACT*)w, N, K, rows, tile_expert, tile, out, ldo)
+#define MA(ACT, G) moe_any_kernel<ACT, G><<<grid, 256, 0, stream>>>((const ACT*)x, (const ACT*)w, N, K, rows, tile_expert, tile, out, ldo, limit, alpha, beta)
   if (f32) { if (glu) MA(float, true); else MA(float, false); }
   else if (glu) MA(uint16_t, true);
   else MA(uint16_t, false);

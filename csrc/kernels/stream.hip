@@ -19,40 +19,14 @@
 // position that is run again (a decode graph's warm-up) from overwriting what it reads.
 //
 // ACT is the activation type the matrix products read: uint16_t (bf16 bits) or float.
-#include "common.h"
+#include "rows.h"
 
 #include <type_traits>
 
 namespace {
 
-__device__ __forceinline__ float ld1(const uint16_t* p) { return bf2f(*p); }
-__device__ __forceinline__ float ld1(const float* p) { return *p; }
 __device__ __forceinline__ void st1(uint16_t* p, float v) { *p = f2bf(v); }
 __device__ __forceinline__ void st1(float* p, float v) { *p = v; }
-
-template <int V> struct Vec { float v[V]; };
-
-template <int V>
-__device__ __forceinline__ Vec<V> ldv(const float* p) {
-  Vec<V> r;
-  if constexpr (V == 4) {
-    const float4 f = *reinterpret_cast<const float4*>(p);
-    r.v[0] = f.x; r.v[1] = f.y; r.v[2] = f.z; r.v[3] = f.w;
-  } else {
-    r.v[0] = *p;
-  }
-  return r;
-}
-template <int V>
-__device__ __forceinline__ void stv(float* p, const Vec<V>& r) {
-  if constexpr (V == 4) *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
-  else *p = r.v[0];
-}
-template <int V>
-__device__ __forceinline__ void stv(uint16_t* p, const Vec<V>& r) {
-  if constexpr (V == 4) *reinterpret_cast<uint2*>(p) = make_uint2(pack2bf(r.v[0], r.v[1]), pack2bf(r.v[2], r.v[3]));
-  else *p = f2bf(r.v[0]);
-}
 
 template <typename TAB>
 __global__ void __launch_bounds__(256) embed_f32_kernel(float* __restrict__ out, const TAB* __restrict__ table,
@@ -383,6 +357,25 @@ __global__ void __launch_bounds__(256) clamped_glu_kernel(ACT* __restrict__ out,
   st1(out + (size_t)t * ldo + c, glu<ACT>(g, u, limit, alpha, beta));
 }
 
+// relu(sum of slabs)^2 of n values (a multiple of V)
+template <typename ACT, typename IN, int V>
+__global__ void __launch_bounds__(256) relu_sq_kernel(ACT* __restrict__ out, const IN* __restrict__ x, int split, size_t n) {
+  for (size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V; i < n; i += (size_t)gridDim.x * 256 * V) {
+    Vec<V> v = ldv<V>(x + i);
+    if constexpr (sizeof(IN) == 4)
+      if (split > 1) {
+        v = zerov<V>();
+        add_slabs<V>(v, x, split, (int64_t)n, i);
+      }
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      v.v[e] = fmaxf(v.v[e], 0.f);
+      v.v[e] *= v.v[e];
+    }
+    stv<V>(out + i, v);
+  }
+}
+
 __global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ x, size_t n, float cap) {
   const float inv = 1.f / cap;
   for (size_t i = blockIdx.x * (size_t)256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) x[i] = cap * tanhf(x[i] * inv);
@@ -531,5 +524,22 @@ CFC_API int cfc_softcap(float* x, int64_t n, float cap, hipStream_t stream) {
   if (!(cap > 0.f)) return -1;
   const int64_t blocks = (n + 255) / 256;
   softcap_kernel<<<(unsigned)(blocks < 4096 ? blocks : 4096), 256, 0, stream>>>(x, (size_t)n, cap);
+  return CFC_CHECK_LAUNCH();
+}
+
+// x: fp32 slabs [split][n] (in_f32) or n activations; out n activations, may be x itself (one slab)
+CFC_API int cfc_relu_sq(int f32, int in_f32, void* out, const void* x, int split, int64_t n, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (split < 1 || (split > 1 && !in_f32) || (f32 && !in_f32)) return -1;
+  const bool v4 = n % 4 == 0;
+  const int64_t blocks = (n / (v4 ? 4 : 1) + 255) / 256;
+  const unsigned g = (unsigned)(blocks < 16384 ? blocks : 16384);
+#define RS(A, I) \
+  if (v4) relu_sq_kernel<A, I, 4><<<g, 256, 0, stream>>>((A*)out, (const I*)x, split, (size_t)n); \
+  else relu_sq_kernel<A, I, 1><<<g, 256, 0, stream>>>((A*)out, (const I*)x, split, (size_t)n)
+  if (f32) { RS(float, float); }
+  else if (in_f32) { RS(uint16_t, float); }
+  else { RS(uint16_t, uint16_t); }
+#undef RS
   return CFC_CHECK_LAUNCH();
 }
