@@ -122,9 +122,6 @@ class PemolornConfig:
     def layers(self) -> int:
         return len(self.specs)
 
-    def cut(self, layers: int) -> "PemolornConfig":
-        return dataclasses.replace(self, specs=self.specs[:layers])
-
     def num_params(self) -> int:
         return sum(math.prod(s) for s in PemolornWeights.tensor_shapes(self).values())
 

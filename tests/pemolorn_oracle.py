@@ -42,20 +42,14 @@ def rotate(x, positions, base, dims):
 
 def window_mask(T, size, keep=0):
     """True where token i sees token j: its last ``size`` tokens and the first ``keep``."""
-    see = torch.zeros(T, T, dtype=torch.bool)
-    for i in range(T):
-        for j in range(i + 1):
-            see[i, j] = i - j < size or j < keep
-    return see
+    i, j = torch.arange(T)[:, None], torch.arange(T)[None]
+    return (j <= i) & ((i - j < size) | (j < keep))
 
 
 def pooled_mask(T, size, pool):
     """True where token i sees block b (tokens b pool .. b pool + pool - 1)."""
-    see = torch.zeros(T, T // pool, dtype=torch.bool)
-    for i in range(T):
-        for b in range(T // pool):
-            see[i, b] = b * pool + pool - 1 <= i - size
-    return see
+    i, last = torch.arange(T)[:, None], torch.arange(T // pool)[None] * pool + pool - 1
+    return last <= i - size
 
 
 def pooled(x, pool):
