@@ -502,9 +502,7 @@ class PemolornModel:
         lw, f = self.w.layers[i], self.cfg.specs[i].mlp
         b = N.Branch(lw["norm2b"], self.cfg.norm_eps)
         if isinstance(f, DenseSpec):
-            up = lw["up"]
-            a = S.relu_sq(up.slabs(h) if h.shape[0] <= 256 else up.act(h), h.dtype)
-            b.y = self._sum(lw["down"].slabs(a))
+            b.y = self._sum(lw["down"].slabs(lw["up"].relu_sq(h)))
             return b
         ids, wt = M.route(lw["gate"].slabs(0, h[None]), lw["router"])
         rows, pos = M.experts(h, lw["experts"], ids, lw["glu"])

@@ -14,7 +14,7 @@ import torch.nn.functional as F
 
 from ..ops import kernels as K
 from ..ops.cols import Cols
-from ..ops.stream import clamped_glu
+from ..ops.stream import clamped_glu, relu_sq
 
 
 class Projection:
@@ -107,6 +107,13 @@ class Projection:
                 and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0:
             return K.dgemm_glu(x, self.packed, out, limit, alpha, beta)
         return clamped_glu(self.slabs(x), out, limit, alpha, beta, interleaved=True)
+
+    def relu_sq(self, x: torch.Tensor) -> torch.Tensor:
+        """relu(product)^2 [M, N] in x's dtype, in the prompt product's epilogue, else with the sum of the slabs."""
+        k = self._kernel(x)
+        if k == "pgemm" and self.K >= 128:
+            return K.pgemm(x, self.packed, "relu2", variant="ppp")
+        return relu_sq(self.slabs(x), x.dtype)
 
     def f32(self, x: torch.Tensor) -> torch.Tensor:
         """[M, N] fp32, a tensor of its own."""

@@ -77,13 +77,13 @@ _KERNEL_SIGS = {
     "cfc_moe_any": [I, I, P, P, I, I, I, P, P, I, P, I, F, F, F, P],
     "cfc_branch_norm": [I, I, P, I, P, P, I, P, F, P, P, P, P, I, I, P, P, I, F, P, I, I, P, I, P, P],
     "cfc_gru_step": [I] + [P, I, c_int64, c_int64] * 3 + [P, P, P, P, I, I, P, P, P],
-    "cfc_gru_prefill": [I] + [P, I, c_int64, c_int64] * 3 + [P, P, P, I, P, P, P, P, I, I, P, P, P, P],
+    "cfc_gru_prefill": [I] + [P, c_int64] * 3 + [P, P, P, I, P, P, P, P, I, I, P, P, P, P],
     "cfc_qkv_rows": [I, P, I, c_int64, c_int64, I, I, I, I, I, I, I, P, P, I, F, P, I, F, P, I] + [P] * 10 + [I, I, P, I, P],
     "cfc_conv_tail": [I, P, I, c_int64, c_int64, I, P, P, P, I, I, P, P],
     "cfc_pool_rows": [I, P, I, P, I, P, P, P, P, I, I, I, I, P],
     "cfc_gqa_prompt_rows": [I],
     "cfc_gqa_attention": [I, I] + [P] * 10 + [I] * 11 + [P, I, I, P, P, P, P],
-    "cfc_relu_sq": [I, I, P, P, I, c_int64, P],
+    "cfc_relu_sq": [I, P, P, I, c_int64, P],
     "cfc_dgemm_group": [I, P, P, I, I, I, I, I, P, P, P, I, F, F, F, P],
     "cfc_pgemm_group": [I, P, I, P, I, I, I, I, P, P, P, I, F, F, F, P],
     "cfc_latent_gather": [P, P, I, P, P, I, I, I, P, P, P, P],

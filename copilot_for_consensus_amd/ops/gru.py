@@ -48,10 +48,10 @@ def _ref(p: Gru, z, u, g, slots, cu, ctx, state, out):
     return out
 
 
-def _args(p: Gru, cols, out, state):
+def _fits(p: Gru, cols, out, state):
     if any(c.n != p.width for c in cols) or out.shape[1] != p.width or not out.is_contiguous() or state.shape[-1] != p.width:
         raise ValueError(f"gru: columns {[c.n for c in cols]}, out {tuple(out.shape)} for a width of {p.width}")
-    return [x for c in cols for x in c.args(out.dtype)] + [p.bz.data_ptr(), p.bx.data_ptr()]
+    return [c.args(out.dtype) for c in cols]
 
 
 def step(p: Gru, z: Cols, u: Cols, g: Cols, slots, ctx_lens, state, out) -> torch.Tensor:
@@ -60,20 +60,24 @@ def step(p: Gru, z: Cols, u: Cols, g: Cols, slots, ctx_lens, state, out) -> torc
         return _ref(p, z, u, g, slots, torch.arange(len(slots) + 1), ctx_lens, state, out)
     _req(slots, torch.int32, "slots")
     _req(ctx_lens, torch.int32, "ctx_lens")
-    check(kernels().cfc_gru_step(_act(out.dtype), *_args(p, (z, u, g), out, state), slots.data_ptr(), ctx_lens.data_ptr(),
-                                 out.shape[0], p.width, state.data_ptr(), out.data_ptr(), _stream(out)), "cfc_gru_step")
+    ops = [x for c in _fits(p, (z, u, g), out, state) for x in c]
+    check(kernels().cfc_gru_step(_act(out.dtype), *ops, p.bz.data_ptr(), p.bx.data_ptr(), slots.data_ptr(), ctx_lens.data_ptr(), out.shape[0],
+                                 p.width, state.data_ptr(), out.data_ptr(), _stream(out)), "cfc_gru_step")
     return out
 
 
 def prefill(p: Gru, z: Cols, u: Cols, g: Cols, slots, cu_q, ctx_lens, chunks, chunk_cu, state, out) -> torch.Tensor:
-    """Packed portions (``chunks``, ``chunk_cu`` of :func:`chunk_plan` on the device)."""
+    """Packed portions, ``z``, ``u``, ``g`` activations (``chunks``, ``chunk_cu`` of :func:`chunk_plan` on the device)."""
     if not out.is_cuda:
         return _ref(p, z, u, g, slots, cu_q, ctx_lens, state, out)
     for name, t in (("slots", slots), ("cu_q", cu_q), ("ctx_lens", ctx_lens), ("chunks", chunks), ("chunk_cu", chunk_cu)):
         _req(t, torch.int32, name)
+    ops = _fits(p, (z, u, g), out, state)
+    if any(c[1] for c in ops):
+        raise ValueError("gru prefill: z, u and g are activations")
     n = chunks.shape[0]
     sums = torch.empty(n * 2 * p.width, dtype=torch.float32, device=out.device)
-    check(kernels().cfc_gru_prefill(_act(out.dtype), *_args(p, (z, u, g), out, state), chunks.data_ptr(), n, chunk_cu.data_ptr(),
-                                    cu_q.data_ptr(), ctx_lens.data_ptr(), slots.data_ptr(), slots.numel(), p.width, sums.data_ptr(),
+    check(kernels().cfc_gru_prefill(_act(out.dtype), *(x for c in ops for x in (c[0], c[2])), p.bz.data_ptr(), p.bx.data_ptr(),
+                                    chunks.data_ptr(), n, chunk_cu.data_ptr(), cu_q.data_ptr(), ctx_lens.data_ptr(), slots.data_ptr(), slots.numel(), p.width, sums.data_ptr(),
                                     state.data_ptr(), out.data_ptr(), _stream(out)), "cfc_gru_prefill")
     return out

@@ -622,7 +622,7 @@ def dgemm_residual_rmsnorm(x: torch.Tensor, w: torch.Tensor, residual: torch.Ten
 
 
 # ------------------------------------------------------------------ prefill / encoder GEMM
-PGEMM_EPI = {"bf16": 0, "bias": 1, "bias_gelu": 2, "swiglu": 3, "f32": 4}
+PGEMM_EPI = {"bf16": 0, "bias": 1, "bias_gelu": 2, "swiglu": 3, "f32": 4, "relu2": 6}
 
 
 def pgemm_ok(x: torch.Tensor, w) -> bool:
@@ -647,7 +647,8 @@ def pgemm(x: torch.Tensor, w, epi: str = "bf16", bias: torch.Tensor | None = Non
     """Hand-written MFMA GEMM for prefill / encoder shapes: x [M, K] @ w[N, K]^T with the following
     elementwise op fused into the epilogue.  ``epi``: "bf16"; "bias" (+ bias[N]); "bias_gelu"
     (gelu_erf(y + bias)); "swiglu" (8-row interleaved gate/up weights -> [M, N/2] =
-    silu(gate) * up with the unfused path's bf16 rounding of gate and up).  ``w``: row-major bf16
+    silu(gate) * up with the unfused path's bf16 rounding of gate and up); "relu2" (relu(y)^2, a PackedWeight
+    with K >= 128 only).  ``w``: row-major bf16
     [N, K], or the decode GEMM's PackedWeight (one weight copy for prefill and decode: the "w4",
     "pps", "ppp" or, for any other variant, the "pp" kernel).  ``variant``: the K loop ("stage2": 2 LDS
     stages of BK=64; "ring5" / "ring4": BK=32 rings of 5 / 4 LDS slots; "pp": two wave groups
@@ -667,6 +668,8 @@ def pgemm(x: torch.Tensor, w, epi: str = "bf16", bias: torch.Tensor | None = Non
             return ref.silu_mul_interleaved(y.to(x.dtype))
         if mode == 4:
             return y
+        if mode == 6:
+            y = ref.relu_sq(y)
         return y.to(x.dtype)
     if not pgemm_ok(x, w):
         raise ValueError(f"pgemm: x {tuple(x.shape)} {x.dtype} w {tuple(w.shape)} {getattr(w, 'dtype', 'packed')}")
@@ -676,6 +679,8 @@ def pgemm(x: torch.Tensor, w, epi: str = "bf16", bias: torch.Tensor | None = Non
         _req(bias, torch.bfloat16, "bias")
         if bias.numel() != N:
             raise ValueError(f"pgemm: bias of {bias.numel()} for N = {N}")
+    if mode == 6 and not packed:
+        raise ValueError("pgemm: the squared relu epilogue takes a packed weight")
     if mode == 4 and (variant or PGEMM_VARIANT) not in ("pp", "pps", "ppp") and not packed:
         variant = "pp"              # the fp32 epilogue is built for the ping-pong kernel only
     if out is None:

@@ -218,13 +218,10 @@ def softcap_(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 def relu_sq(x: torch.Tensor, dtype) -> torch.Tensor:
-    """relu(x)^2 as activations [T, F]: x activations (in place), or fp32 slabs [split, T, F] to be summed."""
-    slabs = x.dim() == 3
+    """relu(sum of fp32 slabs [split, T, F])^2 as activations [T, F]."""
     if not x.is_cuda:
-        return ref.relu_sq(x.sum(0) if slabs else x.float()).to(dtype)
-    if not x.is_contiguous() or (slabs and x.dtype != torch.float32) or (not slabs and x.dtype != dtype):
-        raise ValueError(f"relu_sq: {tuple(x.shape)} {x.dtype} for {dtype}")
-    out = torch.empty(x.shape[-2:], dtype=dtype, device=x.device) if slabs else x
-    check(kernels().cfc_relu_sq(_act(dtype), _act(x.dtype), out.data_ptr(), x.data_ptr(), x.shape[0] if slabs else 1,
-                                out.numel(), _stream(x)), "cfc_relu_sq")
+        return ref.relu_sq(x.sum(0)).to(dtype)
+    _req(x, torch.float32, "x")
+    out = torch.empty(x.shape[1:], dtype=dtype, device=x.device)
+    check(kernels().cfc_relu_sq(_act(dtype), out.data_ptr(), x.data_ptr(), x.shape[0], out.numel(), _stream(x)), "cfc_relu_sq")
     return out

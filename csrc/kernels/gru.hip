@@ -22,13 +22,46 @@ __device__ __forceinline__ Vec<V> gru_ld(const GruCols& a, int64_t t, int c) {
   return y;
 }
 
-__device__ __forceinline__ float sigm(float z) { return 1.f / (1.f + expf(-z)); }
+// ACT decides the exponential and the reciprocal: the hardware's for bf16 activations, the library's on the 32-bit path
+template <typename ACT> __device__ __forceinline__ float exp_of(float x);
+template <> __device__ __forceinline__ float exp_of<uint16_t>(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+template <> __device__ __forceinline__ float exp_of<float>(float x) { return expf(x); }
+template <typename ACT> __device__ __forceinline__ float over1(float x);              // 1 / (1 + x)
+template <> __device__ __forceinline__ float over1<uint16_t>(float x) { return __builtin_amdgcn_rcpf(1.f + x); }
+template <> __device__ __forceinline__ float over1<float>(float x) { return 1.f / (1.f + x); }
 
-// decay 1 - z and contribution z c of one token
+// decay 1 - z and contribution z c of one token.  With t = exp(pre_z): 1 - z = 1 / (1 + t) and z = t / (1 + t), neither
+// the other's difference from 1, so that small ones keep their digits; sigmoid(min(u, 0)) is 1/2 where u >= 0
+template <typename ACT>
 __device__ __forceinline__ void gru_gates(float pz, float u, float& a, float& b) {
-  a = sigm(-pz);
-  b = sigm(pz) * (u >= 0.f ? u + 0.5f : sigm(u));
+  const float t = exp_of<ACT>(fminf(pz, 60.f)), v = exp_of<ACT>(fminf(u, 0.f));
+  a = over1<ACT>(t);
+  b = t * a * (fmaxf(u, 0.f) + v * over1<ACT>(v));
 }
+
+template <typename ACT>
+__device__ __forceinline__ float silu(float g) { return g * over1<ACT>(exp_of<ACT>(fminf(-g, 60.f))); }
+
+// V activations as loaded
+template <typename ACT, int V> struct Raw;
+template <> struct Raw<uint16_t, 4> {
+  uint2 u;
+  __device__ __forceinline__ void get(const uint16_t* p) { u = *reinterpret_cast<const uint2*>(p); }
+  __device__ __forceinline__ float at(int e) const {
+    const uint32_t w = e < 2 ? u.x : u.y;
+    return __uint_as_float(e & 1 ? w & 0xffff0000u : w << 16);
+  }
+};
+template <> struct Raw<float, 4> {
+  float4 f;
+  __device__ __forceinline__ void get(const float* p) { f = *reinterpret_cast<const float4*>(p); }
+  __device__ __forceinline__ float at(int e) const { return e == 0 ? f.x : e == 1 ? f.y : e == 2 ? f.z : f.w; }
+};
+template <typename ACT> struct Raw<ACT, 1> {
+  ACT u;
+  __device__ __forceinline__ void get(const ACT* p) { u = *p; }
+  __device__ __forceinline__ float at(int) const { return ld1(&u); }
+};
 
 template <typename ACT, int V>
 __global__ void __launch_bounds__(64) gru_step_kernel(GruCols z, GruCols u, GruCols g, const float* __restrict__ bz,
@@ -45,47 +78,52 @@ __global__ void __launch_bounds__(64) gru_step_kernel(GruCols z, GruCols u, GruC
 #pragma unroll
   for (int e = 0; e < V; ++e) {
     float a, k;
-    gru_gates(zv.v[e] + vz.v[e], uv.v[e] + vx.v[e], a, k);
+    gru_gates<ACT>(zv.v[e] + vz.v[e], uv.v[e] + vx.v[e], a, k);
     S.v[e] = a * S.v[e] + k;
-    o.v[e] = S.v[e] * gv.v[e] * sigm(gv.v[e]);
+    o.v[e] = S.v[e] * silu<ACT>(gv.v[e]);
   }
   stv<V>(sp, S);
   stv<V>(out + (size_t)b * W + c, o);
 }
 
 constexpr int GRU_FLIGHT = 8;        // rows requested ahead of their use
+struct GruRows { const void* p; int64_t ld; };      // activations
 
 // chunks [n][2]: {first row, rows}; sums [n][2][W]: decay, contribution
 template <typename ACT, int V>
-__global__ void __launch_bounds__(64) gru_chunk_kernel(GruCols z, GruCols u, const float* __restrict__ bz,
+__global__ void __launch_bounds__(64) gru_chunk_kernel(GruRows z, GruRows u, const float* __restrict__ bz,
                                                       const float* __restrict__ bx, const int32_t* __restrict__ chunks, int W,
                                                       float* __restrict__ sums) {
   const int c = (blockIdx.y * 64 + threadIdx.x) * V;
   if (c >= W) return;
   const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
   const Vec<V> vz = ldv<V>(bz + c), vx = ldv<V>(bx + c);
+  const ACT *zp = reinterpret_cast<const ACT*>(z.p) + row0 * z.ld + c, *up = reinterpret_cast<const ACT*>(u.p) + row0 * u.ld + c;
   Vec<V> A, B = zerov<V>();
 #pragma unroll
   for (int e = 0; e < V; ++e) A.v[e] = 1.f;
-  for (int r0 = 0; r0 < n; r0 += GRU_FLIGHT) {
-    Vec<V> zv[GRU_FLIGHT], uv[GRU_FLIGHT];
+  Raw<ACT, V> zv[GRU_FLIGHT], uv[GRU_FLIGHT];
+#pragma unroll
+  for (int i = 0; i < GRU_FLIGHT; ++i) {
+    zv[i].get(zp + min(i, n - 1) * z.ld);
+    uv[i].get(up + min(i, n - 1) * u.ld);
+  }
+  for (int r0 = 0; r0 < n; r0 += GRU_FLIGHT)
 #pragma unroll
     for (int i = 0; i < GRU_FLIGHT; ++i) {
-      const int64_t t = row0 + min(r0 + i, n - 1);
-      zv[i] = gru_ld<ACT, V>(z, t, c);
-      uv[i] = gru_ld<ACT, V>(u, t, c);
-    }
-#pragma unroll
-    for (int i = 0; i < GRU_FLIGHT; ++i)
+      const Raw<ACT, V> zr = zv[i], ur = uv[i];
+      const int64_t next = min(r0 + GRU_FLIGHT + i, n - 1);      // past the last: read again, not used
+      zv[i].get(zp + next * z.ld);
+      uv[i].get(up + next * u.ld);
       if (r0 + i < n)
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           float a, k;
-          gru_gates(zv[i].v[e] + vz.v[e], uv[i].v[e] + vx.v[e], a, k);
+          gru_gates<ACT>(zr.at(e) + vz.v[e], ur.at(e) + vx.v[e], a, k);
           A.v[e] *= a;
           B.v[e] = a * B.v[e] + k;
         }
-  }
+    }
   float* o = sums + (size_t)blockIdx.x * 2 * W + c;
   stv<V>(o, A);
   stv<V>(o + W, B);
@@ -121,37 +159,44 @@ __global__ void __launch_bounds__(64) gru_carry_kernel(const int32_t* __restrict
 }
 
 template <typename ACT, int V>
-__global__ void __launch_bounds__(64) gru_apply_kernel(GruCols z, GruCols u, GruCols g, const float* __restrict__ bz,
+__global__ void __launch_bounds__(64) gru_apply_kernel(GruRows z, GruRows u, GruRows g, const float* __restrict__ bz,
                                                       const float* __restrict__ bx, const int32_t* __restrict__ chunks, int W,
                                                       const float* __restrict__ sums, ACT* __restrict__ out) {
   const int c = (blockIdx.y * 64 + threadIdx.x) * V;
   if (c >= W) return;
   const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
   const Vec<V> vz = ldv<V>(bz + c), vx = ldv<V>(bx + c);
+  const ACT *zp = reinterpret_cast<const ACT*>(z.p) + row0 * z.ld + c, *up = reinterpret_cast<const ACT*>(u.p) + row0 * u.ld + c,
+            *gp = reinterpret_cast<const ACT*>(g.p) + row0 * g.ld + c;
   Vec<V> S = ldv<V>(sums + (size_t)blockIdx.x * 2 * W + c);
-  for (int r0 = 0; r0 < n; r0 += GRU_FLIGHT) {
-    Vec<V> zv[GRU_FLIGHT], uv[GRU_FLIGHT], gv[GRU_FLIGHT];
+  Raw<ACT, V> zv[GRU_FLIGHT], uv[GRU_FLIGHT], gv[GRU_FLIGHT];
+#pragma unroll
+  for (int i = 0; i < GRU_FLIGHT; ++i) {
+    const int64_t r = min(i, n - 1);
+    zv[i].get(zp + r * z.ld);
+    uv[i].get(up + r * u.ld);
+    gv[i].get(gp + r * g.ld);
+  }
+  for (int r0 = 0; r0 < n; r0 += GRU_FLIGHT)
 #pragma unroll
     for (int i = 0; i < GRU_FLIGHT; ++i) {
-      const int64_t t = row0 + min(r0 + i, n - 1);
-      zv[i] = gru_ld<ACT, V>(z, t, c);
-      uv[i] = gru_ld<ACT, V>(u, t, c);
-      gv[i] = gru_ld<ACT, V>(g, t, c);
-    }
-#pragma unroll
-    for (int i = 0; i < GRU_FLIGHT; ++i)
+      const Raw<ACT, V> zr = zv[i], ur = uv[i], gr = gv[i];
+      const int64_t next = min(r0 + GRU_FLIGHT + i, n - 1);
+      zv[i].get(zp + next * z.ld);
+      uv[i].get(up + next * u.ld);
+      gv[i].get(gp + next * g.ld);
       if (r0 + i < n) {
         Vec<V> o;
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           float a, k;
-          gru_gates(zv[i].v[e] + vz.v[e], uv[i].v[e] + vx.v[e], a, k);
+          gru_gates<ACT>(zr.at(e) + vz.v[e], ur.at(e) + vx.v[e], a, k);
           S.v[e] = a * S.v[e] + k;
-          o.v[e] = S.v[e] * gv[i].v[e] * sigm(gv[i].v[e]);
+          o.v[e] = S.v[e] * silu<ACT>(gr.at(e));
         }
         stv<V>(out + (size_t)(row0 + r0 + i) * W + c, o);
       }
-  }
+    }
 }
 
 // vectors of four where every operand's rows allow them
@@ -182,21 +227,22 @@ CFC_API int cfc_gru_step(int f32, const void* z, int z_split, int64_t z_ld, int6
   return CFC_CHECK_LAUNCH();
 }
 
-// packed portions; chunks [n][2] {first row, rows}, chunk_cu [portions + 1]; sums scratch [n][2][W]
-CFC_API int cfc_gru_prefill(int f32, const void* z, int z_split, int64_t z_ld, int64_t z_plane, const void* u, int u_split,
-                            int64_t u_ld, int64_t u_plane, const void* g, int g_split, int64_t g_ld, int64_t g_plane,
+// packed portions; z, u, g activations (pointer, row stride); chunks [n][2] {first row, rows}, chunk_cu [portions + 1]; sums
+// scratch [n][2][W]
+CFC_API int cfc_gru_prefill(int f32, const void* z, int64_t z_ld, const void* u, int64_t u_ld, const void* g, int64_t g_ld,
                             const float* bz, const float* bx, const int32_t* chunks, int n, const int32_t* chunk_cu,
                             const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* slots, int portions, int W, float* sums,
                             float* state, void* out, hipStream_t stream) {
   if (n <= 0 || portions <= 0) return 0;
   if (W < 1 || !chunks || !chunk_cu || !cu_q || !ctx_lens || !slots || !sums || !state) return -1;
-  const GruCols a[3] = {{z, z_split, z_ld, z_plane}, {u, u_split, u_ld, u_plane}, {g, g_split, g_ld, g_plane}};
+  const GruCols a[3] = {{z, 0, z_ld, 0}, {u, 0, u_ld, 0}, {g, 0, g_ld, 0}};
+  const GruRows r[3] = {{z, z_ld}, {u, u_ld}, {g, g_ld}};
 #define GP(ACT, V)                                                                                                    \
   do {                                                                                                                \
     const int gy = (W + 64 * V - 1) / (64 * V);                                                                       \
-    gru_chunk_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(a[0], a[1], bz, bx, chunks, W, sums);                    \
+    gru_chunk_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(r[0], r[1], bz, bx, chunks, W, sums);                    \
     gru_carry_kernel<V><<<dim3(portions, gy), 64, 0, stream>>>(chunk_cu, cu_q, ctx_lens, slots, W, sums, state);      \
-    gru_apply_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(a[0], a[1], a[2], bz, bx, chunks, W, sums, (ACT*)out);   \
+    gru_apply_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(r[0], r[1], r[2], bz, bx, chunks, W, sums, (ACT*)out);   \
   } while (0)
   const bool v4 = gru_vec(a, 3, W, f32);
   if (f32) { if (v4) GP(float, 4); else GP(float, 1); }

@@ -39,7 +39,7 @@ typedef __attribute__((address_space(3))) void pg_lds_t;
 
 // PG_F32: the fp32 accumulators themselves (row stride ldo in floats): a tensor-parallel row-parallel
 // projection's partial, all-reduced in fp32 and rounded to bf16 once, as TP = 1 rounds the full sum
-enum { PG_BF16 = 0, PG_BIAS = 1, PG_BIAS_GELU = 2, PG_SWIGLU = 3, PG_F32 = 4, PG_GLU = 5 };
+enum { PG_BF16 = 0, PG_BIAS = 1, PG_BIAS_GELU = 2, PG_SWIGLU = 3, PG_F32 = 4, PG_GLU = 5, PG_RELU2 = 6 };
 
 constexpr int PG_BM = 256, PG_BN = 256, PG_BK = 64;
 constexpr int PG_STAGE = (PG_BM + PG_BN) * PG_BK * 2;   // 64 KB: A image then B image
@@ -94,6 +94,16 @@ __device__ __forceinline__ uint32_t pg_gate2(const float (&v)[4], const PgGlu& p
 
 __device__ __forceinline__ int pg_gate_col(int g) { return 4 * (g & 1) + 2 * (g >> 1); }
 
+// what a value leaves as: PG_RELU2 its squared positive part
+template <int EPI>
+__device__ __forceinline__ float pg_out(float v) {
+  if constexpr (EPI == PG_RELU2) {
+    v = fmaxf(v, 0.f);
+    return v * v;
+  }
+  return v;
+}
+
 // Epilogue of every kernel here: lane holds rows m = mw + 16 i + (lane & 15), columns
 // n = nw + 16 j + 4 (lane >> 4) + 0..3 of the wave's 128 x 16 NJ block.
 template <int EPI, int NJ>
@@ -130,7 +140,8 @@ __device__ __forceinline__ void pg_epilogue(const f32x4_t (&acc)[8][NJ], const u
 #pragma unroll
             for (int e = 0; e < 4; ++e) v[e] = pg_gelu(v[e]);
           }
-          *reinterpret_cast<uint2*>(out + (size_t)m * ldo + n) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
+          *reinterpret_cast<uint2*>(out + (size_t)m * ldo + n) =
+              make_uint2(pack2bf(pg_out<EPI>(v[0]), pg_out<EPI>(v[1])), pack2bf(pg_out<EPI>(v[2]), pg_out<EPI>(v[3])));
         }
       }
     }
@@ -716,7 +727,7 @@ template <int EPI, bool STG = false>
 __global__ void __launch_bounds__(512, 1)
     pgemm_ppp_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, uint16_t* __restrict__ out,
                      int M, int N, int K, int ldo, int tiles_m, int tiles_n, int wnw, int gm, PgGlu gp) {
-  static_assert(EPI == PG_BF16 || pg_gated(EPI), "bf16 / gated epilogues");
+  static_assert(EPI == PG_BF16 || EPI == PG_RELU2 || pg_gated(EPI), "bf16 / gated epilogues");
   // epilogue store instructions per wave in the interior (counted in the next tile's first waits):
   // staged bf16 16 x 16 B (128 rows x 128 B), staged SwiGLU 8 x 16 B (128 rows x 64 B), else 32
   constexpr int PPP_S = STG ? (pg_gated(EPI) ? 8 : 16) : 32;
@@ -893,7 +904,8 @@ __global__ void __launch_bounds__(512, 1)
           if constexpr (pg_gated(EPI) && !STG) {
             ppp_st4(out + (size_t)m * ldo + nb / 2 + pg_gate_col(g), pg_gate2<EPI>(v, gp));
           } else if constexpr (!STG) {
-            ppp_st8(out + (size_t)m * ldo + nb + 4 * g, make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3])));
+            ppp_st8(out + (size_t)m * ldo + nb + 4 * g,
+                    make_uint2(pack2bf(pg_out<EPI>(v[0]), pg_out<EPI>(v[1])), pack2bf(pg_out<EPI>(v[2]), pg_out<EPI>(v[3]))));
           }
         }
       }
@@ -945,7 +957,7 @@ __global__ void __launch_bounds__(512, 1)
               const f32x4_t& a = acc[2 * q + ii][j];
               const int unit = (2 * j + (g >> 1)) ^ (r & 7);
               *reinterpret_cast<uint2*>(region + r * 128 + unit * 16 + (g & 1) * 8) =
-                  make_uint2(pack2bf(a[0], a[1]), pack2bf(a[2], a[3]));
+                  make_uint2(pack2bf(pg_out<EPI>(a[0]), pg_out<EPI>(a[1])), pack2bf(pg_out<EPI>(a[2]), pg_out<EPI>(a[3])));
             }
           }
           __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -1356,7 +1368,7 @@ int pgemm_launch_f32(const void* x, const void* w, void* out, int M, int N, int 
 
 }  // namespace
 
-// epi & 15: 0 bf16, 1 + bias, 2 + bias -> GELU, 3 SwiGLU (out [M, N/2]); epi >> 4: K-loop variant
+// epi & 15: 0 bf16, 1 + bias, 2 + bias -> GELU, 3 SwiGLU (out [M, N/2]), 4 fp32, 6 squared relu; epi >> 4: K-loop variant
 // for a row-major W (0 BK = 32 ring of 5 slots, 1 the 2-stage BK = 64 kernel, 2 ring of 4 slots,
 // 3 the ping-pong kernel, 5 the same with the LDS-staged bf16 / SwiGLU epilogue, 6 the persistent
 // ping-pong kernel for a packed W -- the ping-pong kernel otherwise); ldo = output row stride.  wnw > 0: W is in the decode GEMM's
@@ -1375,6 +1387,10 @@ CFC_API int cfc_pgemm(const void* x, const void* w, const void* bias, void* out,
     case 2: return pgemm_launch<PG_BIAS_GELU>(x, w, bias, out, M, N, K, ldo, variant, wnw, stream);
     case 3: return pgemm_launch<PG_SWIGLU>(x, w, bias, out, M, N, K, ldo, variant, wnw, stream);
     case 4: return pgemm_launch_f32(x, w, out, M, N, K, ldo, wnw, stream);
+    case 6:        // packed W, the persistent kernel
+      if (wnw < 1 || K < 2 * PG_BK || ldo % 8 || ((uintptr_t)out & 15)) return (int)hipErrorInvalidValue;
+      return ppp_launch<PG_RELU2>((const uint16_t*)x, (const uint16_t*)w, (uint16_t*)out, M, N, K, ldo, wnw,
+                                  ppp_group_m((N + PG_BN - 1) / PG_BN, K), PPP_STG, stream);
     default: return (int)hipErrorInvalidValue;
   }
 }

@@ -4,6 +4,7 @@
 //                 and values into the paged cache [blocks][G][32][D].  A row's queries, keys and values take a
 //                 workgroup each.  Decoded rows also store what the convolution remembers and, where a pooled block of
 //                 tokens ends, the block's mean key and value
+//   * qkv_prompt  the same for prompt rows of common shapes, many rows per workgroup
 //   * conv_tail   the last inputs of prompt portions' convolutions into the sequences' state (a launch of its own:
 //                 rows of the same portion read the old ones)
 //   * pool_rows   mean keys and values of the blocks that prompt portions end, from the cache as it holds them
@@ -44,6 +45,7 @@ __device__ __forceinline__ float round_act(float v, const uint16_t*) { return bf
 __device__ __forceinline__ float round_act(float v, const float*) { return v; }
 
 constexpr int ROT_MAX = 1024;
+constexpr int MAX_BACK = 3;          // convolution rows before the own that a thread holds in registers
 
 // grid (rows, parts).  Dynamic LDS: per-vector sums, and for V = 1 the row
 template <typename ACT, int V, int NV, int BT>
@@ -52,24 +54,53 @@ __global__ void __launch_bounds__(BT) qkv_rows_kernel(QkvArgs a) {
   __shared__ float2 cs[ROT_MAX / 2];
   extern __shared__ float dyn[];
   const int t = xcd_remap(blockIdx.x, gridDim.x), part = blockIdx.y, tid = threadIdx.x;
-  const int pos = a.positions[t], heads = part == 0 ? a.H : a.G, hd = part == 2 ? a.vdim : a.dim, C = heads * hd;
-  const int c0 = part == 0 ? 0 : part == 1 ? a.H * a.dim : (a.H + a.G) * a.dim;
+  // gridDim.z > 1: each takes a run of the heads
+  const int all_heads = part == 0 ? a.H : a.G, h0 = all_heads * blockIdx.z / gridDim.z, h1 = all_heads * (blockIdx.z + 1) / gridDim.z;
+  const int pos = a.positions[t], heads = h1 - h0, hd = part == 2 ? a.vdim : a.dim, C = heads * hd;
+  const int c0 = (part == 0 ? 0 : part == 1 ? a.H * a.dim : (a.H + a.G) * a.dim) + h0 * hd;
+  if (heads == 0) return;
   const int nvec = C / V, allc = a.H * a.dim + (a.parts > 1 ? a.G * (a.dim + a.vdim) : 0);
   const float* wn = part == 0 ? a.qn : part == 1 ? a.kn : nullptr;
   const int rot = part == 2 ? 0 : a.rot;
   Vec<V> x[NV];
+  if (!a.conv) {
 #pragma unroll
-  for (int k = 0; k < NV; ++k) {
-    const int c = (k * BT + tid) * V;
-    x[k] = c < C ? qkv_ld<ACT, V>(a, t, c0 + c) : zerov<V>();
-  }
-  if (a.conv) {
+    for (int k = 0; k < NV; ++k) {
+      const int c = (k * BT + tid) * V;
+      x[k] = c < C ? qkv_ld<ACT, V>(a, t, c0 + c) : zerov<V>();
+    }
+  } else {
+#pragma unroll
+    for (int k = 0; k < NV; ++k) x[k] = zerov<V>();
     const int back = a.taps - 1, lead = a.lead ? a.lead[t] : 0;
     float* st = back ? a.tail + (size_t)a.slots[t] * back * allc + c0 : nullptr;
+    if (!a.lead && back <= MAX_BACK) {
+      // decoded rows: what a vector needs is asked for together
+#pragma unroll
+      for (int k = 0; k < NV; ++k) {
+        const int c = min((k * BT + tid) * V, C - V);
+        Vec<V> o[MAX_BACK], w[MAX_BACK + 1];
+#pragma unroll
+        for (int d = 0; d <= MAX_BACK; ++d) w[d] = ldv<V>(a.conv + (size_t)max(back - d, 0) * allc + c0 + c);
+#pragma unroll
+        for (int d = 1; d <= MAX_BACK; ++d)
+          o[d - 1] = d <= back && d <= pos ? ldv<V>(st + (size_t)((pos - d) % max(back, 1)) * allc + c) : zerov<V>();
+        const Vec<V> u = qkv_ld<ACT, V>(a, t, c0 + c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          x[k].v[e] = u.v[e] * w[0].v[e];
+#pragma unroll
+          for (int d = 1; d <= MAX_BACK; ++d) x[k].v[e] += d <= back ? o[d - 1].v[e] * w[d].v[e] : 0.f;
+        }
+        if ((k * BT + tid) * V >= C) x[k] = zerov<V>();
+        else if (back > 0) stv<V>(st + (size_t)(pos % back) * allc + c, u);
+      }
+    } else
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
       const int c = (k * BT + tid) * V;
       if (c >= C) continue;
+      x[k] = qkv_ld<ACT, V>(a, t, c0 + c);
       const Vec<V> u = x[k], w = ldv<V>(a.conv + (size_t)back * allc + c0 + c);
 #pragma unroll
       for (int e = 0; e < V; ++e) x[k].v[e] *= w.v[e];
@@ -166,7 +197,7 @@ __global__ void __launch_bounds__(BT) qkv_rows_kernel(QkvArgs a) {
     }
   }
   if (part == 0) {
-    ACT* q = reinterpret_cast<ACT*>(a.q) + (size_t)t * a.H * a.D;
+    ACT* q = reinterpret_cast<ACT*>(a.q) + ((size_t)t * a.H + h0) * a.D;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
       const int c = (k * BT + tid) * V;
@@ -183,7 +214,7 @@ __global__ void __launch_bounds__(BT) qkv_rows_kernel(QkvArgs a) {
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
     const int c = (k * BT + tid) * V;
-    if (c < C) stv<V>(cache + row(slot / CFC_KV_BS, c / hd, slot % CFC_KV_BS) + c % hd, x[k]);
+    if (c < C) stv<V>(cache + row(slot / CFC_KV_BS, h0 + c / hd, slot % CFC_KV_BS) + c % hd, x[k]);
   }
   if (a.pool == 0 || (pos + 1) % a.pool) return;
   const int32_t* bt = a.bt + (size_t)t * a.max_blocks;
@@ -191,7 +222,7 @@ __global__ void __launch_bounds__(BT) qkv_rows_kernel(QkvArgs a) {
   ACT* pc = reinterpret_cast<ACT*>(part == 1 ? a.pk : a.pv) + (((size_t)bt[b >> a.le] * a.G) << a.le) * a.D;
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
-    const int c = (k * BT + tid) * V, g = c / hd;
+    const int c = (k * BT + tid) * V, g = h0 + c / hd;
     if (c >= C) continue;
     Vec<V> m;
 #pragma unroll
@@ -208,18 +239,226 @@ __global__ void __launch_bounds__(BT) qkv_rows_kernel(QkvArgs a) {
   }
 }
 
+// Prompt rows from activations: PR_ROWS consecutive rows of one part (0: queries, 1: keys and values) per workgroup, two or four
+// at a time, a vector of V channels per thread.  What the convolution reads back stays in registers, weights are read
+// once, the rows of a time share one reduction.  Heads of a power of two of vectors (per-head norms) and, with a
+// convolution, at most MAX_BACK + 1 taps.
+constexpr int PR_ROWS = 16;
+template <typename ACT, int V> struct Raw;
+template <> struct Raw<uint16_t, 8> {
+  uint4 u;
+  __device__ __forceinline__ void get(const void* p) { u = *reinterpret_cast<const uint4*>(p); }
+  __device__ __forceinline__ void zero() { u = make_uint4(0, 0, 0, 0); }
+  __device__ __forceinline__ Vec<8> val() const { Vec<8> r; unpack8(u, r.v); return r; }
+};
+template <> struct Raw<float, 4> {
+  float4 f;
+  __device__ __forceinline__ void get(const void* p) { f = *reinterpret_cast<const float4*>(p); }
+  __device__ __forceinline__ void zero() { f = make_float4(0.f, 0.f, 0.f, 0.f); }
+  __device__ __forceinline__ Vec<4> val() const { return Vec<4>{{f.x, f.y, f.z, f.w}}; }
+};
+template <int V>
+__device__ __forceinline__ Vec<V> ldw(const float* p) {
+  Vec<V> r;
+#pragma unroll
+  for (int e = 0; e < V; e += 4) {
+    const float4 f = *reinterpret_cast<const float4*>(p + e);
+    r.v[e] = f.x; r.v[e + 1] = f.y; r.v[e + 2] = f.z; r.v[e + 3] = f.w;
+  }
+  return r;
+}
+__device__ __forceinline__ void stw(uint16_t* p, const Vec<8>& r) { *reinterpret_cast<uint4*>(p) = pack8(r.v); }
+__device__ __forceinline__ void stw(float* p, const Vec<4>& r) { *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]); }
+
+template <typename ACT, int V, int BT, bool CONV>
+__global__ void __launch_bounds__(BT, BT <= 512 ? 4 : 1) qkv_prompt_kernel(QkvArgs a, int T) {
+  constexpr int RG = CONV ? 2 : 4, NW = BT / 64;
+  __shared__ float red[2][RG][NW];
+  __shared__ int4 meta[PR_ROWS];                       // position, rows before it in its portion, cache slot, state slot
+  extern __shared__ float2 cs[];                       // [PR_ROWS][rot / 2]
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, part = blockIdx.y;
+  const int t0 = xcd_remap(blockIdx.x, gridDim.x) * PR_ROWS, t1 = min(t0 + PR_ROWS, T);
+  const int allc = a.H * a.dim + (a.parts > 1 ? a.G * (a.dim + a.vdim) : 0), nk = a.G * a.dim, c = tid * V;
+  const int C = part == 0 ? a.H * a.dim : nk, cp = part == 0 ? 0 : a.H * a.dim;
+  const bool live = c < (part == 0 ? C : nk + a.G * a.vdim), isv = part == 1 && c >= nk;
+  const int hd = isv ? a.vdim : a.dim, ch = isv ? c - nk : c, head = ch / hd, cd = ch - head * hd;
+  const float* wn = isv || !live ? nullptr : part == 0 ? a.qn : a.kn;
+  const int back = CONV ? a.taps - 1 : 0, half = a.rot / 2;
+  const bool turn = !isv && live && cd < a.rot;
+  for (int i = tid; i < PR_ROWS; i += BT) {
+    const int t = min(t0 + i, T - 1);
+    meta[i] = make_int4(a.positions[t], a.lead[t], a.cslots ? a.cslots[t] : 0, back ? a.slots[t] : 0);
+  }
+  const ACT* src = reinterpret_cast<const ACT*>(a.p) + cp + (live ? c : 0);
+  Vec<V> nw, cw[MAX_BACK + 1];
+#pragma unroll
+  for (int e = 0; e < V; ++e) nw.v[e] = 1.f;
+  if (wn) nw = ldw<V>(wn + (a.per_head ? cd : c));
+  if (part == 0)
+#pragma unroll
+    for (int e = 0; e < V; ++e) nw.v[e] *= a.qscale;
+  if constexpr (CONV) {
+#pragma unroll
+    for (int d = 0; d <= MAX_BACK; ++d) {
+      cw[d] = ldw<V>(a.conv + (size_t)max(back - d, 0) * allc + cp + (live ? c : 0));
+      if (d > back)
+#pragma unroll
+        for (int e = 0; e < V; ++e) cw[d].v[e] = 0.f;
+    }
+  }
+  // win[MAX_BACK + r]: row r of the group
+  Raw<ACT, V> win[MAX_BACK + RG], nxt[RG];
+  if constexpr (CONV)
+#pragma unroll
+    for (int d = 1; d <= MAX_BACK; ++d) win[MAX_BACK - d].get(src + (int64_t)max(t0 - d, 0) * a.ld);
+#pragma unroll
+  for (int r = 0; r < RG; ++r) win[MAX_BACK + r].get(src + (int64_t)min(t0 + r, T - 1) * a.ld);
+  __syncthreads();
+  for (int i = tid; i < PR_ROWS * half; i += BT) {
+    float sn, co;
+    sincosf((float)meta[i / half].x * a.freq[i % half], &sn, &co);
+    cs[i] = make_float2(co, sn);
+  }
+  __syncthreads();
+  for (int g0 = t0, par = 0; g0 < t1; g0 += RG, par ^= 1) {
+    int4 mt[RG];
+    int least = MAX_BACK;
+#pragma unroll
+    for (int r = 0; r < RG; ++r) {
+      mt[r] = meta[g0 - t0 + r];
+      least = min(least, mt[r].y);
+    }
+    const bool inside = __builtin_amdgcn_readfirstlane(least) >= back;      // no row reads before its portion
+#pragma unroll
+    for (int r = 0; r < RG; ++r) nxt[r].get(src + (int64_t)min(g0 + RG + r, T - 1) * a.ld);
+    Vec<V> y[RG];
+    float ss[RG];
+#pragma unroll
+    for (int r = 0; r < RG; ++r) {
+      y[r] = win[MAX_BACK + r].val();
+      if constexpr (CONV) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[r].v[e] *= cw[0].v[e];
+        if (inside) {                          // weights past the taps are zero
+#pragma unroll
+          for (int d = 1; d <= MAX_BACK; ++d) {
+            const Vec<V> o = win[MAX_BACK + r - d].val();
+#pragma unroll
+            for (int e = 0; e < V; ++e) y[r].v[e] += cw[d].v[e] * o.v[e];
+          }
+        } else {
+          const int pos = __builtin_amdgcn_readfirstlane(mt[r].x), lead = __builtin_amdgcn_readfirstlane(mt[r].y);
+#pragma unroll
+          for (int d = 1; d <= MAX_BACK; ++d) {
+            if (d > back || d > pos) break;
+            const Vec<V> o = d <= lead ? win[MAX_BACK + r - d].val()
+                                       : ldw<V>(a.tail + ((size_t)mt[r].w * back + (pos - d) % back) * allc + cp + (live ? c : 0));
+#pragma unroll
+            for (int e = 0; e < V; ++e) y[r].v[e] += cw[d].v[e] * o.v[e];
+          }
+        }
+      }
+      ss[r] = 0.f;
+      if (wn)
+#pragma unroll
+        for (int e = 0; e < V; ++e) ss[r] += y[r].v[e] * y[r].v[e];
+    }
+    float inv[RG];
+    if (a.per_head) {
+      const int hv = a.dim / V;
+#pragma unroll
+      for (int r = 0; r < RG; ++r) {
+        for (int m = hv / 2; m > 0; m >>= 1) ss[r] += __shfl_xor(ss[r], m, 64);
+        inv[r] = 1.f / sqrtf(ss[r] / (float)a.dim + a.eps);
+      }
+    } else {
+#pragma unroll
+      for (int r = 0; r < RG; ++r) {
+        ss[r] = wave_sum(ss[r]);
+        if (lane == 0) red[par][r][w] = ss[r];
+      }
+      __syncthreads();
+#pragma unroll
+      for (int r = 0; r < RG; ++r) {
+        float s = 0.f;
+#pragma unroll
+        for (int i = 0; i < NW; ++i) s += red[par][r][i];
+        inv[r] = 1.f / sqrtf(s / (float)C + a.eps);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < RG; ++r) {
+      const int t = g0 + r;
+      if (t >= t1 || !live) continue;
+      const float f = wn ? inv[r] : 1.f;
+#pragma unroll
+      for (int e = 0; e < V; ++e) y[r].v[e] *= f * nw.v[e];
+      if (turn) {
+#pragma unroll
+        for (int e = 0; e < V; e += 2)
+          if (cd + e < a.rot) {
+            const float2 k = cs[(t - t0) * half + ((cd + e) >> 1)];
+            const float u = y[r].v[e], v = y[r].v[e + 1];
+            y[r].v[e] = u * k.x - v * k.y;
+            y[r].v[e + 1] = v * k.x + u * k.y;
+          }
+      }
+      if (part == 0) {
+        stw(reinterpret_cast<ACT*>(a.q) + ((size_t)t * a.H + head) * a.D + cd, y[r]);
+      } else {
+        const int slot = mt[r].z;
+        stw(reinterpret_cast<ACT*>(isv ? a.vc : a.kc) +
+                (((size_t)(slot / CFC_KV_BS) * a.G + head) * CFC_KV_BS + slot % CFC_KV_BS) * a.D + cd, y[r]);
+      }
+    }
+#pragma unroll
+    for (int d = 0; d < MAX_BACK; ++d) win[d] = win[d + RG];
+#pragma unroll
+    for (int r = 0; r < RG; ++r) win[MAX_BACK + r] = nxt[r];
+  }
+}
+
+// whether the prompt kernel takes the layer; its threads
+template <typename ACT, int V>
+int prompt_threads(const QkvArgs& a) {
+  if (!a.lead || a.split || a.dim % V || a.vdim % V || a.D % V || a.ld % V || ((uintptr_t)a.p & 15) || a.taps > MAX_BACK + 1 ||
+      a.rot > 512)
+    return 0;
+  if (a.per_head && (a.dim / V > 64 || (a.dim / V & (a.dim / V - 1)) || (64 % (a.dim / V)))) return 0;
+  const int vecs = max(a.H * a.dim, a.parts > 1 ? a.G * (a.dim + a.vdim) : 0) / V;
+  return vecs <= 64 ? 64 : vecs <= 256 ? 256 : vecs <= 512 ? 512 : vecs <= 1024 ? 1024 : 0;
+}
+
+template <typename ACT, int V>
+int qkv_prompt_go(hipStream_t s, int T, int threads, const QkvArgs& a) {
+  const dim3 grid((T + PR_ROWS - 1) / PR_ROWS, a.parts > 1 ? 2 : 1);
+  const size_t lds = (size_t)PR_ROWS * (a.rot / 2) * sizeof(float2) + 16;
+#define GO(BT)                                                                             \
+  if (a.conv) qkv_prompt_kernel<ACT, V, BT, true><<<grid, BT, lds, s>>>(a, T);             \
+  else qkv_prompt_kernel<ACT, V, BT, false><<<grid, BT, lds, s>>>(a, T)
+  if (threads == 64) { GO(64); }
+  else if (threads == 256) { GO(256); }
+  else if (threads == 512) { GO(512); }
+  else { GO(1024); }
+#undef GO
+  return CFC_CHECK_LAUNCH();
+}
+
 template <typename ACT, int V>
 int qkv_go(hipStream_t s, int T, const QkvArgs& a) {
-  int C = a.H * a.dim;
-  if (a.parts > 1) C = max(C, a.G * max(a.dim, a.vdim));
+  // few rows with norms per head: runs of heads beside each other, so their loads do not follow one another
+  const int most = max(a.H, a.parts > 1 ? a.G : 0);
+  const int z = a.per_head && T * a.parts < 512 ? max(1, min(min(most, 8), 512 / (T * a.parts))) : 1;
+  int C = (a.H + z - 1) / z * a.dim;
+  if (a.parts > 1) C = max(C, (a.G + z - 1) / z * max(a.dim, a.vdim));
   const int vecs = (C + V - 1) / V;
   const size_t lds = (size_t)(vecs + max(a.H, a.G)) * 4;
   if (lds > 49152) return -4;
-#define GO(NV, BT) qkv_rows_kernel<ACT, V, NV, BT><<<dim3(T, a.parts), BT, lds, s>>>(a)
+#define GO(NV, BT) qkv_rows_kernel<ACT, V, NV, BT><<<dim3(T, a.parts, z), BT, lds, s>>>(a)
   if (vecs <= 64) GO(1, 64);
   else if (vecs <= 256) GO(1, 256);
-  else if (vecs <= 512) GO(2, 256);
-  else if (vecs <= 1024) GO(4, 256);
+  else if (vecs <= 512) GO(1, 512);
+  else if (vecs <= 1024) GO(1, 1024);
   else if (vecs <= 4096) GO(4, 1024);
   else if (vecs <= 16384) GO(16, 1024);
   else return -4;
@@ -288,6 +527,8 @@ CFC_API int cfc_qkv_rows(int f32, const void* p, int split, int64_t ld, int64_t 
                   lead, slots, positions, cslots, q, kc, vc, pk, pv, lead ? 0 : pool, le, bt, max_blocks};
   const bool v4 = dim % 4 == 0 && vdim % 4 == 0 && D % 4 == 0 && ld % 4 == 0 && plane % 4 == 0 &&
                   ((uintptr_t)p & (split == 0 && !f32 ? 7 : 15)) == 0;
+  if (const int th = f32 ? prompt_threads<float, 4>(a) : prompt_threads<uint16_t, 8>(a))
+    return f32 ? qkv_prompt_go<float, 4>(stream, T, th, a) : qkv_prompt_go<uint16_t, 8>(stream, T, th, a);
   if (f32) return v4 ? qkv_go<float, 4>(stream, T, a) : qkv_go<float, 1>(stream, T, a);
   return v4 ? qkv_go<uint16_t, 4>(stream, T, a) : qkv_go<uint16_t, 1>(stream, T, a);
 }

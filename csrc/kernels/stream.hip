@@ -358,15 +358,11 @@ __global__ void __launch_bounds__(256) clamped_glu_kernel(ACT* __restrict__ out,
 }
 
 // relu(sum of slabs)^2 of n values (a multiple of V)
-template <typename ACT, typename IN, int V>
-__global__ void __launch_bounds__(256) relu_sq_kernel(ACT* __restrict__ out, const IN* __restrict__ x, int split, size_t n) {
+template <typename ACT, int V>
+__global__ void __launch_bounds__(256) relu_sq_kernel(ACT* __restrict__ out, const float* __restrict__ x, int split, size_t n) {
   for (size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V; i < n; i += (size_t)gridDim.x * 256 * V) {
-    Vec<V> v = ldv<V>(x + i);
-    if constexpr (sizeof(IN) == 4)
-      if (split > 1) {
-        v = zerov<V>();
-        add_slabs<V>(v, x, split, (int64_t)n, i);
-      }
+    Vec<V> v = zerov<V>();
+    add_slabs<V>(v, x, split, (int64_t)n, i);
 #pragma unroll
     for (int e = 0; e < V; ++e) {
       v.v[e] = fmaxf(v.v[e], 0.f);
@@ -527,19 +523,17 @@ CFC_API int cfc_softcap(float* x, int64_t n, float cap, hipStream_t stream) {
   return CFC_CHECK_LAUNCH();
 }
 
-// x: fp32 slabs [split][n] (in_f32) or n activations; out n activations, may be x itself (one slab)
-CFC_API int cfc_relu_sq(int f32, int in_f32, void* out, const void* x, int split, int64_t n, hipStream_t stream) {
+// x: fp32 slabs [split][n]; out n activations
+CFC_API int cfc_relu_sq(int f32, void* out, const float* x, int split, int64_t n, hipStream_t stream) {
   if (n <= 0) return 0;
-  if (split < 1 || (split > 1 && !in_f32) || (f32 && !in_f32)) return -1;
+  if (split < 1) return -1;
   const bool v4 = n % 4 == 0;
   const int64_t blocks = (n / (v4 ? 4 : 1) + 255) / 256;
   const unsigned g = (unsigned)(blocks < 16384 ? blocks : 16384);
-#define RS(A, I) \
-  if (v4) relu_sq_kernel<A, I, 4><<<g, 256, 0, stream>>>((A*)out, (const I*)x, split, (size_t)n); \
-  else relu_sq_kernel<A, I, 1><<<g, 256, 0, stream>>>((A*)out, (const I*)x, split, (size_t)n)
-  if (f32) { RS(float, float); }
-  else if (in_f32) { RS(uint16_t, float); }
-  else { RS(uint16_t, uint16_t); }
+#define RS(A, V) relu_sq_kernel<A, V><<<g, 256, 0, stream>>>((A*)out, x, split, (size_t)n)
+  if (f32) { if (v4) RS(float, 4); else RS(float, 1); }
+  else if (v4) RS(uint16_t, 4);
+  else RS(uint16_t, 1);
 #undef RS
   return CFC_CHECK_LAUNCH();
 }

@@ -6,6 +6,7 @@ import pytest
 import torch
 
 import pemolorn_oracle as oracle
+from copilot_for_consensus_amd.models.projection import Projection
 from copilot_for_consensus_amd.ops import branch as N
 from copilot_for_consensus_amd.ops import gqa as A
 from copilot_for_consensus_amd.ops import gru as R
@@ -86,10 +87,16 @@ def test_branch_and_norms(device, dtype, W, T, split, kind):
 @pytest.mark.parametrize("T,F,split", [(3, 65, 1), (5, 256, 3), (2, 1030, 11)])
 def test_squared_relu(device, dtype, T, F, split):
     x = rnd(T, F)
-    want = torch.clamp(x, min=0.0) ** 2
-    close(S.relu_sq(slabs(x, split).to(device), dtype), want, tol(dtype))
-    a = x.to(device, dtype)
-    close(S.relu_sq(a.clone(), dtype), torch.clamp(a.float().cpu(), min=0.0) ** 2, tol(dtype))
+    close(S.relu_sq(slabs(x, split).to(device), dtype), torch.clamp(x, min=0.0) ** 2, tol(dtype))
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("M,N,K", [(300, 24704, 128), (1, 192, 64), (513, 25600, 192), (100, 256, 320), (6200, 1024, 192)])
+def test_squared_relu_of_a_product(M, N, K):
+    """Every kernel a product takes, among them the prompt product's epilogue with whole and cut tiles."""
+    x, w = rnd(M, K).to(torch.bfloat16), rnd(N, K, seed=1, scale=K ** -0.5).to(torch.bfloat16)
+    got = Projection(w.cuda()).relu_sq(x.cuda())
+    close(got, torch.clamp(x.float() @ w.float().T, min=0.0) ** 2, 8e-3)
 
 
 # ------------------------------------------------------------------ recurrence
