@@ -196,10 +196,16 @@ def prompt_rows(dtype, D: int) -> int:
 
 
 def prompt_tiles(cu, ctx, H: int, G: int, rows: int) -> np.ndarray:
-    """[2, n] (sequence, first row) of the tiles of packed portions."""
+    """[2, n] (sequence, first row) of the tiles of packed portions, the latest positions (most keys) first."""
     per, step = (H // G, rows) if rows else (H, ANY_ROWS)
-    t = [(s, m) for s, (lo, hi) in enumerate(zip(cu, cu[1:])) for m in range(0, (hi - lo) * per, step)]
-    return np.ascontiguousarray(np.asarray(t, np.int32).reshape(-1, 2).T)
+    seq, m0, pos = [], [], []
+    for s, (lo, hi, c) in enumerate(zip(cu, cu[1:], ctx)):
+        m = np.arange(0, (hi - lo) * per, step)
+        seq.append(np.full(len(m), s))
+        m0.append(m)
+        pos.append(c - (hi - lo) + np.minimum(m + step, (hi - lo) * per) // per)
+    order = np.argsort(-np.concatenate(pos), kind="stable")
+    return np.stack([np.concatenate(seq)[order], np.concatenate(m0)[order]]).astype(np.int32)
 
 
 def decode_slices(B: int, H: int, G: int, D: int, visible: int, dtype) -> int:

@@ -278,7 +278,8 @@ __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) gqa_decode_kernel(const
 }
 
 // ------------------------------------------------------------------------------------------ prompt portions
-// 1-D grid of n_tiles * G, key head major and XCD-remapped: neighbouring tiles of one key head share an L2.
+// 1-D grid of n_tiles * G, tile major: in the tiles' order (those with the most keys first, so that long ones do not end
+// the grid alone), and an XCD takes one key head of eight, whose keys its L2 then holds.
 // A tile is 32 NW rows (row r of a portion and key head: token r / R, head r % R of the group).
 template <int D, int NW>
 __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(const uint16_t* __restrict__ q,
@@ -291,7 +292,7 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
   constexpr bool EVEN = 64 * CH % NT == 0;
   constexpr int TILE = 64 * D * 2;
   extern __shared__ __attribute__((aligned(16))) char smem[];          // [2][K | V]
-  const int lin = xcd_remap(blockIdx.x, gridDim.x), hk = lin / a.n_tiles, tile = lin - hk * a.n_tiles;
+  const int tile = blockIdx.x / a.G, hk = blockIdx.x - tile * a.G;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l32 = lane & 31, hi = lane >> 5;
   const int R = a.H / a.G, s = a.tile_seq[tile], m0 = a.tile_m0[tile];
   const int q0 = a.cu_q[s], n = a.cu_q[s + 1] - q0, rows = n * R, base = a.ctx_lens[s] - n;
