@@ -24,6 +24,8 @@ EXPECTED = {
     ("0", "0"): {"global_store_dwordx4": 0, "global_store_dwordx2": 64, "global_store_dword": 0},    # bf16, direct
     ("3", "1"): {"global_store_dwordx4": 8, "global_store_dwordx2": 0, "global_store_dword": 32},    # SwiGLU, staged
     ("5", "1"): {"global_store_dwordx4": 8, "global_store_dwordx2": 0, "global_store_dword": 32},    # clamped GLU, staged
+    ("6", "1"): {"global_store_dwordx4": 16, "global_store_dwordx2": 32, "global_store_dword": 0},   # squared relu, staged
+    ("6", "0"): {"global_store_dwordx4": 0, "global_store_dwordx2": 64, "global_store_dword": 0},    # squared relu, direct
     ("3", "0"): {"global_store_dwordx4": 0, "global_store_dwordx2": 0, "global_store_dword": 64},    # SwiGLU, direct
 }
 
