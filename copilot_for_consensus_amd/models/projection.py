@@ -97,16 +97,16 @@ class Projection:
             return torch.mm(x, w.t(), out_dtype=torch.float32)[None]
         return F.linear(x.float(), w.float())[None]
 
-    def glu(self, x: torch.Tensor, out: torch.Tensor, limit: float, alpha: float, beta: float) -> torch.Tensor:
-        """W = 8-row interleaved gate / up rows, packed: the clamped GLU of the product into ``out`` [M, N / 2]
-        (row-strided), in the product's epilogue where one pass over W fills the chip."""
+    def glu(self, x: torch.Tensor, out: torch.Tensor, limit: float, alpha: float, beta: float, cubic: float = 0.0) -> torch.Tensor:
+        """W = 8-row interleaved gate / up rows: the clamped GLU of the product into ``out`` [M, N / 2]
+        (row-strided), in the product's epilogue where one pass over (packed) W fills the chip."""
         k, M = self._kernel(x), x.shape[0]
         if k == "pgemm" and self.K >= 128 and out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0:
-            return K.pgemm_glu(x, self.packed, out, limit, alpha, beta)
+            return K.pgemm_glu(x, self.packed, out, limit, alpha, beta, cubic)
         if k in ("pgemm", "dgemm") and self.N // self.packed.bn * -(-M // 256) > K.DGEMM_CUS // 2 \
                 and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0:
-            return K.dgemm_glu(x, self.packed, out, limit, alpha, beta)
-        return clamped_glu(self.slabs(x), out, limit, alpha, beta, interleaved=True)
+            return K.dgemm_glu(x, self.packed, out, limit, alpha, beta, cubic)
+        return clamped_glu(self.slabs(x), out, limit, alpha, beta, interleaved=True, cubic=cubic)
 
     def relu_sq(self, x: torch.Tensor) -> torch.Tensor:
         """relu(product)^2 [M, N] in x's dtype, in the prompt product's epilogue, else with the sum of the slabs."""

@@ -8,7 +8,7 @@ from pathlib import Path
 
 import torch
 
-from . import decoder, pemolorn, vofosun, zisapel
+from . import decoder, pemolorn, tadolix, vofosun, zisapel
 
 
 @dataclasses.dataclass(frozen=True)
@@ -38,6 +38,12 @@ def _load_pemolorn(path):
     return pemolorn.config_from_json(json.loads(path.read_text()), name=path.parent.name or "pemolorn")
 
 
+def _load_tadolix(path):
+    """config.json leaves the rows of the distance biases to the tensors beside it."""
+    path = Path(path)
+    return tadolix.config_from_json(json.loads(path.read_text()), name=path.parent.name or "tadolix", ckpt_dir=path.parent)
+
+
 FAMILIES: dict[str, Family] = {
     "decoder": Family("decoder", decoder.DecoderConfig, decoder.DecoderWeights, decoder.DecoderModel, decoder.PRESETS,
                       decoder.load_config_json, (torch.bfloat16,)),
@@ -47,6 +53,8 @@ FAMILIES: dict[str, Family] = {
                       _load_zisapel, (torch.bfloat16, torch.float32)),
     "Pemolorn": Family("Pemolorn", pemolorn.PemolornConfig, pemolorn.PemolornWeights, pemolorn.PemolornModel, pemolorn.PRESETS,
                        _load_pemolorn, (torch.bfloat16, torch.float32)),
+    "Tadolix": Family("Tadolix", tadolix.TadolixConfig, tadolix.TadolixWeights, tadolix.TadolixModel, tadolix.PRESETS,
+                      _load_tadolix, (torch.bfloat16, torch.float32)),
 }
 
 

@@ -53,11 +53,11 @@ _KERNEL_SIGS = {
     "cfc_sample": [P, I, I, I, F, c_uint32, P, P, P],
     "cfc_sample_truncated": [P, I, I, I, F, I, F, F, c_uint32, P, P, P],
     "cfc_decode_advance": [P, P, I, P, P, P, P, P, P, I, P, P, I, I] + [P] * 6 + [I] * 4 + [P] * 4,
-    "cfc_embed_f32": [P, P, P, I, I, I, I, P],
+    "cfc_embed_f32": [P, P, P, I, I, I, I, F, P, P, P],
     "cfc_depth_pre": [P, c_int64, I, I, P, P, P, P, P, P],
     "cfc_depth_norm": [I, I, I, P, P, P, P, I, P, P, I, P, I, P, F, P, P, I, I, P, I, P, I, P, P, I, P, P, I, P, I, P],
     "cfc_input_conv": [I, I, P, P, P, P, P, P, I, P, I, P, I, I, P, I, P, I, P],
-    "cfc_clamped_glu": [I, I, P, I, P, I, P, P, I, I, I, F, F, F, P],
+    "cfc_clamped_glu": [I, I, P, I, P, I, P, P, I, I, I, F, F, F, F, P],
     "cfc_softcap": [P, c_int64, F, P],
     "cfc_latent_norm": [I, P, I, I, I, I, P, P, F, P, P, I, P, I, P],
     "cfc_latent_rope": [I, P, I, c_int64, c_int64, I, I, P, F, P, P, I, I, P, I, c_int64, c_int64, I, I, P, I, I, P, P, I,
@@ -76,13 +76,18 @@ _KERNEL_SIGS = {
     "cfc_moe_rows": [P, I, I, I, I, I, P, P, P, P],
     "cfc_moe_any": [I, I, P, P, I, I, I, P, P, I, P, I, F, F, F, P],
     "cfc_branch_norm": [I, I, P, I, P, P, I, P, F, P, P, P, P, I, I, P, P, I, F, P, I, I, P, I, P, P],
-    "cfc_gru_step": [I] + [P, I, c_int64, c_int64] * 3 + [P, P, P, P, I, I, P, P, P],
-    "cfc_gru_prefill": [I] + [P, c_int64] * 3 + [P, P, P, I, P, P, P, P, I, I, P, P, P, P],
+    "cfc_gru_step": [I] + [P, I, c_int64, c_int64] * 3 + [P, P, P, P, I, I, P, P, c_int64, F, P],
+    "cfc_gru_prefill": [I] + [P, c_int64] * 3 + [P, P, P, I, P, P, P, P, I, I, P, P, P, c_int64, F, P],
+    "cfc_hyper_norm": [I, I, I, P, P, c_int64, c_int64, P, P, I, P, P, P, P, F, I, I, I, P, P, P, I, P, P, P, I, P, P],
+    "cfc_rglru_segment": [],
+    "cfc_rglru_max_block": [],
+    "cfc_rglru_step": [I] + [P, I, c_int64, c_int64] * 2 + [P, P, P, I] + [P] * 5 + [I] * 4 + [P] * 5 + [I, P, P],
+    "cfc_rglru_prefill": [I] + [P, c_int64] * 2 + [P, P, P, I] + [P] * 5 + [I] * 4 + [P] * 4 + [I, P, I, P, P, P, I, I, P, P, P, P],
     "cfc_qkv_rows": [I, P, I, c_int64, c_int64, I, I, I, I, I, I, I, P, P, I, F, P, I, F, P, I] + [P] * 10 + [I, I, P, I, P],
     "cfc_conv_tail": [I, P, I, c_int64, c_int64, I, P, P, P, I, I, P, P],
     "cfc_pool_rows": [I, P, I, P, I, P, P, P, P, I, I, I, I, P],
     "cfc_gqa_prompt_rows": [I],
-    "cfc_gqa_attention": [I, I] + [P] * 10 + [I] * 11 + [P, I, I, P, P, P, P],
+    "cfc_gqa_attention": [I, I] + [P] * 10 + [I] * 13 + [F, P, I, P, P, I, c_int64, c_int64, F, I, I, P, P, P, c_int64, P],
     "cfc_relu_sq": [I, P, P, I, c_int64, P],
     "cfc_dgemm_group": [I, P, P, I, I, I, I, I, P, P, P, I, F, F, F, P],
     "cfc_pgemm_group": [I, P, I, P, I, I, I, I, P, P, P, I, F, F, F, P],
@@ -105,8 +110,8 @@ _KERNEL_SIGS = {
     "cfc_pgemm_ln": [P, P, P, P, P, P, P, I, I, I, F, P],
     "cfc_pgemm_probe": [P, P, P, I, I, I, I, I, I, P],
     "cfc_pgemm_ppp_probe": [P, P, P, I, I, I, I, I, I, I, P],
-    "cfc_pgemm_glu": [P, P, P, I, I, I, I, I, F, F, F, P],
-    "cfc_dgemm_glu": [P, P, I, I, I, I, P, I, F, F, F, P],
+    "cfc_pgemm_glu": [P, P, P, I, I, I, I, I, F, F, F, F, P],
+    "cfc_dgemm_glu": [P, P, I, I, I, I, P, I, F, F, F, F, P],
     "cfc_dgemm_bm": [I],
     "cfc_dgemm_pack": [P, P, I, I, I, P],
     "cfc_dgemm_ablate": [P, P, I, I, I, I, I, I, P, P],

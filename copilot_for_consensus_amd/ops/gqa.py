@@ -1,12 +1,15 @@
-"""Grouped-query attention over two key ranges: a sliding window, and either kept first tokens or mean keys and values of
-earlier blocks (csrc/kernels/qkv.hip, gqa.hip).
+"""Grouped-query attention over two key ranges: a sliding window or the own chunk of positions, and either kept first
+tokens or mean keys and values of earlier blocks; scores with a softcap and a bias by distance, outputs through a gate
+(csrc/kernels/qkv.hip, gqa.hip).
 
 GPU tensors go to the native library (which must be built), CPU tensors to the fp32 reference.
 """
 from __future__ import annotations
 
+import bisect
 import dataclasses
 import math
+from fractions import Fraction
 
 import numpy as np
 import torch
@@ -23,19 +26,23 @@ MAX_DIM = 1024
 ANY_ROWS = 4              # rows per tile of the general kernel
 MAX_PARTITIONS = 256
 LOG2E = 1.4426950408889634
+CAP_NEAR = 0.35           # scores up to this share of their cap take the cap's short form
 
 
 @dataclasses.dataclass(frozen=True)
 class Mask:
-    """What a token sees: its last ``size`` tokens (0: all), the first ``keep``, one mean per block of ``pool`` tokens
-    wholly ahead of the window (0: none)."""
+    """What a token sees: its last ``size`` tokens (0: all), or with ``chunked`` those of its own run of ``size`` positions
+    (counted from 0), the first ``keep``, one mean per block of ``pool`` tokens wholly ahead of the window (0: none)."""
     size: int
     keep: int = 0
     pool: int = 0
+    chunked: bool = False
 
     def __post_init__(self):
         if min(self.size, self.keep, self.pool) < 0 or (self.pool and (self.keep or not self.size)):
             raise ValueError(f"{self}: pooled blocks need a window and no kept tokens")
+        if self.chunked and (not self.size or self.pool):
+            raise ValueError(f"{self}: chunks have a size and no pooled blocks")
 
     def visible(self, ctx: int) -> int:
         """Keys and means the last of ``ctx`` tokens sees (about)."""
@@ -56,11 +63,42 @@ def pool_entries(pool: int) -> int:
     return 1 << math.ceil(math.log2(KV_BLOCK / pool)) if pool < KV_BLOCK else 1
 
 
+def distance_starts(rows: int, far) -> list[int]:
+    """First distance of each of a bias table's ``rows`` rows: one distance each in the first half, then steps of equal
+    ratio, the last row's one step short of ``far``: n is at or past the k-th when (n / half)^steps >= (far / half)^k."""
+    half = rows // 2
+    if rows < 2:
+        return [0] * rows
+    far = Fraction(far)
+    if far <= half:
+        raise ValueError(f"distance bias of {rows} rows up to a distance of {far}")
+    steps, out = rows - half, list(range(half + 1))
+    for k in range(1, steps):
+        n, level = math.floor(half * (float(far) / half) ** (k / steps)), far ** k * half ** (steps - k)
+        while n ** steps >= level:
+            n -= 1
+        while n ** steps < level:
+            n += 1
+        out.append(n)
+    return out
+
+
+def distance_bias(rel: torch.Tensor, far, limit: int) -> torch.Tensor:
+    """[H, n] biases by distance from a table ``rel`` [rows, H] (:func:`distance_starts`), the last entry for all distances
+    from there on; no more than ``limit`` (> 0) distances."""
+    starts = distance_starts(rel.shape[0], far)
+    n = starts[-1] + 1
+    row = [bisect.bisect_right(starts, d) - 1 for d in range(min(n, limit) if limit else n)]
+    return rel.float()[torch.tensor(row, dtype=torch.long, device=rel.device)].t().contiguous()
+
+
 @dataclasses.dataclass
 class Heads:
     """An attention layer between its projections and its output: ``H`` query heads in ``G`` groups.  Norm weights over the
     whole projection ([H dim], [G dim]) or per head ([dim]), fp32; ``conv`` [taps, (H + G) dim + G vdim] fp32 over time
-    ahead of the norms; ``freq`` the rotation of the first dimensions.  ``shared``: keys and values are another layer's."""
+    ahead of the norms; ``freq`` the rotation of the first dimensions.  ``shared``: keys and values are another layer's.
+    ``softcap`` of the scores (0: none), then ``bias`` [H, n] fp32 by distance (:func:`distance_bias`).  ``unit``: norms per
+    head with weights of 1, so that no score exceeds ``dim * scale``."""
     H: int
     G: int
     dim: int
@@ -75,9 +113,18 @@ class Heads:
     freq: torch.Tensor | None = None
     conv: torch.Tensor | None = None
     shared: bool = False
+    softcap: float = 0.0
+    bias: torch.Tensor | None = None
+    unit: bool = False
 
     def __post_init__(self):
         self.D = padded_dim(self.dim, self.vdim)
+        # queries carry the scale into the softmax's base 2, or into the cap's e^(2 score / cap)
+        self.q_scale = self.scale * LOG2E * (2.0 / self.softcap if self.softcap else 1.0)
+        self.capped = 0 if not self.softcap else 2 if self.unit and self.dim * abs(self.scale) <= 0.98 * CAP_NEAR * self.softcap else 1
+        self.bias2 = None if self.bias is None else (self.bias * LOG2E).contiguous()
+        if self.bias is not None and (self.bias.shape[0] != self.H or self.mask.pool):
+            raise ValueError(f"bias {tuple(self.bias.shape)} for {self.H} heads over {self.mask}")
         if self.H % self.G or self.D > MAX_DIM:
             raise ValueError(f"{self.H} heads in {self.G} groups, {self.D} columns")
 
@@ -100,7 +147,7 @@ def rope_freq(dims: int, base: float, device) -> torch.Tensor | None:
 
 
 def qkv_rows(a: Heads, cols: Cols, rows, positions, slots, states, block_tables, tail=None, lead=None) -> torch.Tensor:
-    """Projections [q | k | v] of packed rows to queries [T, H, D] (scaled by log2(e)) and rows of the cache ``rows``
+    """Projections [q | k | v] of packed rows to queries [T, H, D] (scaled by ``q_scale``) and rows of the cache ``rows``
     (runtime.kv_cache.PagedHeads) at ``slots``.  ``lead``: rows of the same portion before each row (prompts: afterwards
     :func:`conv_tail` and :func:`pool_rows`); None: one token per sequence, whose state in ``tail`` [states, taps - 1, C]
     and pooled entries are written here."""
@@ -114,7 +161,7 @@ def qkv_rows(a: Heads, cols: Cols, rows, positions, slots, states, block_tables,
     q = (torch.empty if a.D == a.dim else torch.zeros)(T, a.H, a.D, dtype=dt, device=rows.k.device)
     rot = 2 * a.freq.numel() if a.freq is not None else 0
     check(kernels().cfc_qkv_rows(_act(dt), *cols.args(dt), T, a.H, a.G, a.dim, a.vdim, a.D, 1 if a.shared else 3, _p(a.q_norm),
-                                 _p(a.k_norm), int(a.per_head), float(a.eps), _p(a.freq), rot, float(a.scale * LOG2E), _p(a.conv),
+                                 _p(a.k_norm), int(a.per_head), float(a.eps), _p(a.freq), rot, float(a.q_scale), _p(a.conv),
                                  a.taps, _p(tail), _p(lead), _p(states), positions.data_ptr(), slots.data_ptr(), q.data_ptr(),
                                  rows.k.data_ptr(), rows.v.data_ptr(), _p(rows.pk), _p(rows.pv), a.mask.pool, rows.log2_entries,
                                  block_tables.data_ptr(), block_tables.shape[1], _stream(q)), "cfc_qkv_rows")
@@ -137,7 +184,7 @@ def _qkv_ref(a, cols, rows, positions, slots, states, block_tables, tail, lead, 
         x = (ref.head_norm(x, w, a.eps, a.per_head, heads) if w is not None else x).view(T, heads, a.dim)
         return ref.rotate_heads(x, positions, a.freq) if a.freq is not None else x
     q = torch.zeros(T, a.H, a.D, dtype=dt)
-    q[..., :a.dim] = (turned(u[:, :nq], a.q_norm, a.H) * (a.scale * LOG2E)).to(dt)
+    q[..., :a.dim] = (turned(u[:, :nq], a.q_norm, a.H) * a.q_scale).to(dt)
     if a.shared:
         return q
     blk, off = (slots // KV_BLOCK).long(), (slots % KV_BLOCK).long()
@@ -216,16 +263,20 @@ def decode_slices(B: int, H: int, G: int, D: int, visible: int, dtype) -> int:
     return max(1, min(math.ceil(1024 / items), visible // 256, MAX_PARTITIONS))
 
 
-def attention(a: Heads, q, rows, block_tables, ctx_lens, cu_q=None, tiles=None, P: int = 1, workspace=None) -> torch.Tensor:
+def attention(a: Heads, q, rows, block_tables, ctx_lens, cu_q=None, tiles=None, P: int = 1, workspace=None, gate: Cols | None = None,
+              factor: float = 1.0, out: torch.Tensor | None = None) -> torch.Tensor:
     """Attention of :func:`qkv_rows`' queries over the paged rows: [T, H vdim].  ``cu_q`` None: one token per sequence, P key
-    slices each; else packed portions with ``tiles`` of :func:`prompt_tiles` (on the device)."""
+    slices each; else packed portions with ``tiles`` of :func:`prompt_tiles` (on the device).  ``gate`` [T, H vdim]: the
+    result times factor sigmoid(gate).  ``out``: where to (row-strided)."""
     T, H, D = q.shape
     m, dt = a.mask, q.dtype
     B = ctx_lens.numel()
     if not q.is_cuda:
         cu = cu_q if cu_q is not None else torch.arange(B + 1)
-        return ref.grouped_attention(q, rows.k, rows.v, (rows.pk, rows.pv), block_tables, cu, ctx_lens, m.size, m.keep, m.pool,
-                                     a.sink, a.vdim)
+        y = ref.grouped_attention(q, rows.k, rows.v, (rows.pk, rows.pv), block_tables, cu, ctx_lens, m.size, m.keep, m.pool,
+                                  a.sink, a.vdim, m.chunked, a.softcap, a.bias)
+        y = y * factor * torch.sigmoid(gate.value()) if gate is not None else y * factor
+        return y.to(dt) if out is None else out.copy_(y)
     if not q.is_contiguous() or rows.k.shape[1] != a.G or rows.k.shape[3] != D or rows.k.dtype != dt or H != a.H \
             or (m.pool and (rows.pk is None or rows.pool != m.pool)):
         raise ValueError(f"attention: q {tuple(q.shape)} {dt}, cache {tuple(rows.k.shape)} {rows.k.dtype}, {m}")
@@ -243,7 +294,12 @@ def attention(a: Heads, q, rows, block_tables, ctx_lens, cu_q=None, tiles=None, 
         _req(cu_q, torch.int32, "cu_q")
         _req(tiles, torch.int32, "tiles")
         ts, tm, n = tiles[0], tiles[1], tiles.shape[1]
-    out = torch.empty(T, H * a.vdim, dtype=dt, device=q.device)
+    if gate is not None and (gate.n != H * a.vdim or gate.rows != T):
+        raise ValueError(f"attention: gate of {gate.n} columns and {gate.rows} rows for {T} x {H * a.vdim}")
+    if out is None:
+        out = torch.empty(T, H * a.vdim, dtype=dt, device=q.device)
+    elif out.shape != (T, H * a.vdim) or out.stride(1) != 1 or out.dtype != dt:
+        raise ValueError(f"attention: out {tuple(out.shape)} {out.dtype}")
     po = pm = None
     if P > 1:
         need = T * H * P * (D + 2)
@@ -251,6 +307,8 @@ def attention(a: Heads, q, rows, block_tables, ctx_lens, cu_q=None, tiles=None, 
         po, pm = ws[:T * H * P * D], ws[T * H * P * D:need]
     check(kernels().cfc_gqa_attention(kind, _act(dt), q.data_ptr(), rows.k.data_ptr(), rows.v.data_ptr(), _p(rows.pk), _p(rows.pv),
                                       block_tables.data_ptr(), _p(cu_q), ctx_lens.data_ptr(), _p(ts), _p(tm), n, B, H, a.G, D, a.vdim,
-                                      block_tables.shape[1], m.size, m.keep, m.pool, rows.log2_entries, _p(a.sink), P, T * H, _p(po),
-                                      _p(pm), out.data_ptr(), _stream(q)), "cfc_gqa_attention")
+                                      block_tables.shape[1], m.size, m.keep, m.pool, rows.log2_entries, int(m.chunked), a.capped,
+                                      float(a.softcap * LOG2E), _p(a.bias2), a.bias2.shape[1] if a.bias2 is not None else 0, _p(a.sink),
+                                      *(gate.args(dt) if gate is not None else (None, 0, 0, 0)), float(factor), P, T * H, _p(po),
+                                      _p(pm), out.data_ptr(), out.stride(0), _stream(q)), "cfc_gqa_attention")
     return out

@@ -700,25 +700,25 @@ def _glu_out(x, w, out, name):
 
 
 def pgemm_glu(x: torch.Tensor, w: "PackedWeight", out: torch.Tensor, limit: float, alpha: float,
-              beta: float) -> torch.Tensor:
+              beta: float, cubic: float = 0.0) -> torch.Tensor:
     """pgemm over packed 8-row interleaved gate / up weights with the clamped GLU in its epilogue:
-    min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta) into ``out`` [M, N / 2] (row-strided)."""
+    min(g, limit) sigmoid(alpha g (1 + cubic g^2)) (clamp(u, +-limit) + beta) into ``out`` [M, N / 2] (row-strided)."""
     _glu_out(x, w, out, "pgemm_glu")
     if not pgemm_ok(x, w):
         raise ValueError(f"pgemm_glu: x {tuple(x.shape)} {x.dtype} w {tuple(w.shape)}")
     check(kernels().cfc_pgemm_glu(x.data_ptr(), w.data.data_ptr(), out.data_ptr(), x.shape[0], w.N, w.K, out.stride(0),
-                                  w.bn // 16, float(limit), float(alpha), float(beta), _stream(x)), "cfc_pgemm_glu")
+                                  w.bn // 16, float(limit), float(alpha), float(beta), float(cubic), _stream(x)), "cfc_pgemm_glu")
     return out
 
 
 def dgemm_glu(x: torch.Tensor, w: "PackedWeight", out: torch.Tensor, limit: float, alpha: float,
-              beta: float) -> torch.Tensor:
+              beta: float, cubic: float = 0.0) -> torch.Tensor:
     """:func:`pgemm_glu` on the decode GEMM (one pass over W, no split)."""
     _glu_out(x, w, out, "dgemm_glu")
     if not dgemm_ok(x, w):
         raise ValueError(f"dgemm_glu: x {tuple(x.shape)} {x.dtype} w {tuple(w.shape)}")
     check(kernels().cfc_dgemm_glu(x.data_ptr(), w.data.data_ptr(), x.shape[0], w.N, w.K, w.bn, out.data_ptr(),
-                                  out.stride(0), float(limit), float(alpha), float(beta), _stream(x)), "cfc_dgemm_glu")
+                                  out.stride(0), float(limit), float(alpha), float(beta), float(cubic), _stream(x)), "cfc_dgemm_glu")
     return out
 
 

@@ -325,6 +325,12 @@ def tail_slots(taps: int) -> int:
     return 0 if taps <= 1 else min(taps + 1, KV_BLOCK)
 
 
+def sinusoids(positions, turns, width):
+    """[T, width]: sine and cosine of positions * turns[i] turns at entries 2i and 2i + 1."""
+    a = positions.to(torch.float64)[:, None] * turns * (2.0 * math.pi)
+    return torch.stack([a.sin(), a.cos()], -1).flatten(1)[:, :width].to(torch.float32)
+
+
 def depth_norm(x, hist, part, bias, dwa, n, eps, pre=None, j0=0):
     """X_n = x + sum of part slabs + bias into hist[n]; returns (sum_j dwa[j] X_j, 1 / rms of it); ``pre``
     is the sum of the first j0 terms."""
@@ -339,17 +345,20 @@ def depth_norm(x, hist, part, bias, dwa, n, eps, pre=None, j0=0):
 
 def input_conv(h, portions, block_tables, tail, weights):
     """h [T, W] fp32 convolution inputs of packed portions [(first row, rows, first position, sequence)];
-    tail [blocks, slots, W] read for positions before a portion and updated.  weights: per sublayer
-    [taps, W].  Returns one h + conv(h) per sublayer."""
+    tail [blocks, slots, W] read for positions before a portion and updated (``block_tables`` [sequences]: one row of
+    slots per sequence).  weights: per sublayer [taps, W].  Returns one h + conv(h) per sublayer."""
     outs = [h.clone() for _ in weights]
     taps = weights[0].shape[0]
+
+    def block(seq, q):
+        return int(block_tables[seq, q // KV_BLOCK] if block_tables.dim() == 2 else block_tables[seq])
     for row0, n, pos0, seq in portions:
         past = []
         for q in range(pos0 - taps + 1, pos0):
             if q < 0:
                 past.append(torch.zeros_like(h[0]))
             else:
-                past.append(tail[int(block_tables[seq, q // KV_BLOCK]), q % tail.shape[1]])
+                past.append(tail[block(seq, q), q % tail.shape[1]])
         ext = torch.cat([torch.stack(past), h[row0:row0 + n]]) if past else h[row0:row0 + n]
         for o, w in zip(outs, weights):
             for j in range(taps):
@@ -358,14 +367,14 @@ def input_conv(h, portions, block_tables, tail, weights):
             q = pos0 + r
             # the last inputs of the portion and of every block it crosses
             if taps > 1 and (r >= n - (taps - 1) or KV_BLOCK - q % KV_BLOCK <= taps - 1):
-                tail[int(block_tables[seq, q // KV_BLOCK]), q % tail.shape[1]] = h[row0 + r]
+                tail[block(seq, q), q % tail.shape[1]] = h[row0 + r]
     return outs
 
 
-def clamped_glu(g, u, limit, alpha, beta):
+def clamped_glu(g, u, limit, alpha, beta, cubic=0.0):
     g = torch.clamp(g, max=limit)
     u = torch.clamp(u, min=-limit, max=limit)
-    return g * torch.sigmoid(alpha * g) * (u + beta)
+    return g * torch.sigmoid(alpha * g * (1.0 + cubic * g * g)) * (u + beta)
 
 
 # ----------------------------------------------------- latent attention (latent.hip)
@@ -534,6 +543,27 @@ def min_gru(z, u, S):
     return out
 
 
+# ----------------------------------------------------- hyper-connections (hyper.hip)
+def hyper_update(x, y, mix, out):
+    """x [T, S, W]: x_t <- sum_s mix[s, t] x_s + out[t] y."""
+    return torch.einsum("tsw,sq->tqw", x, mix) + out[:, None] * y[:, None]
+
+
+# ----------------------------------------------------- real-gated recurrence behind a short convolution (rglru.hip)
+def gelu_tanh(z):
+    return z * torch.sigmoid(2.0 * math.sqrt(2.0 / math.pi) * z * (1.0 + 0.044715 * z * z))
+
+
+def rglru(u, pr, pi, rate, S):
+    """u and the gates' pre-activations [T, C], S [C] (updated): the states S_t [T, C]."""
+    la, out = rate * torch.sigmoid(pr), torch.empty_like(u)
+    a, b = torch.exp(la), torch.sqrt(-torch.expm1(2.0 * la)) * torch.sigmoid(pi) * u
+    for t in range(u.shape[0]):
+        S.mul_(a[t]).add_(b[t])
+        out[t] = S
+    return out
+
+
 # ----------------------------------------------------- grouped attention over two key ranges (qkv.hip, gqa.hip)
 def conv_over_time(u, w, lead, positions, slots, tail):
     """u [T, C] fp32, w [taps, C]: y_t = sum_d w[taps - 1 - d] u_(t - d) inside each sequence.  ``lead`` rows of the same
@@ -564,17 +594,20 @@ def paged_rows(cache, table, n):
     return cache[table[:-(-n // e)].long()].transpose(1, 2).reshape(-1, cache.shape[1], cache.shape[3])[:n]
 
 
-def grouped_attention(q, k, v, pooled, block_tables, cu_q, ctx_lens, size, keep, pool, sink, vdim):
-    """q [T, H, D] scaled by log2(e); k, v [blocks, G, 32, D], ``pooled`` their block means [blocks, G, E, D] (pool > 0).
-    A row sees its last ``size`` keys (0: all), the first ``keep``, and the means of blocks of ``pool`` keys wholly ahead
-    of the window; exp(sink) joins the denominator."""
+def grouped_attention(q, k, v, pooled, block_tables, cu_q, ctx_lens, size, keep, pool, sink, vdim, chunked=False, softcap=0.0,
+                      bias=None):
+    """q [T, H, D] scaled by log2(e) (with a softcap: by 2 log2(e) / softcap); k, v [blocks, G, 32, D], ``pooled`` their block
+    means [blocks, G, E, D] (pool > 0).  A row sees its last ``size`` keys (0: all; ``chunked``: those of its own run of
+    ``size`` positions), the first ``keep``, and the means of blocks of ``pool`` keys wholly ahead of the window; ``bias``
+    [H, n] by distance joins the scores, exp(sink) the denominator.  fp32."""
     T, H, D = q.shape
-    out = torch.empty(T, H * vdim, dtype=q.dtype)
+    out = torch.empty(T, H * vdim, dtype=torch.float32)
     for s in range(len(ctx_lens)):
         a, b, ctx = int(cu_q[s]), int(cu_q[s + 1]), int(ctx_lens[s])
         K, V = (paged_rows(c, block_tables[s], ctx).float() for c in (k, v))
         pos, j = torch.arange(ctx - (b - a), ctx)[:, None], torch.arange(ctx)[None]
-        see = (j <= pos) & ((pos - j < size) | (j < keep)) if size else j <= pos
+        near = pos // size == j // size if chunked else pos - j < size
+        see = (j <= pos) & (near | (j < keep)) if size else j <= pos
         n = max(ctx - size, 0) // pool if pool else 0
         if n:
             PK, PV = (paged_rows(c, block_tables[s], n).float() for c in pooled)
@@ -582,9 +615,13 @@ def grouped_attention(q, k, v, pooled, block_tables, cu_q, ctx_lens, size, keep,
             see = torch.cat([see, torch.arange(n)[None] < (pos - size + 1).clamp(min=0) // pool], 1)
         for h in range(H):
             g = h * K.shape[1] // H
-            sc = (q[a:b, h].float() @ K[:, g].t() * math.log(2.0)).masked_fill(~see, float("-inf"))
+            sc = q[a:b, h].float() @ K[:, g].t()
+            sc = softcap * torch.tanh(sc * (0.5 * math.log(2.0))) if softcap else sc * math.log(2.0)
+            if bias is not None:
+                sc = sc + bias[h][(pos - j).clamp(0, bias.shape[1] - 1)]
+            sc = sc.masked_fill(~see, float("-inf"))
             if sink is not None:
                 sc = torch.cat([sc, sink[h].expand(b - a, 1)], 1)
             p = torch.softmax(sc, -1)[:, :K.shape[0]]
-            out[a:b, h * vdim:(h + 1) * vdim] = (p @ V[:, g, :vdim]).to(q.dtype)
+            out[a:b, h * vdim:(h + 1) * vdim] = p @ V[:, g, :vdim]
     return out

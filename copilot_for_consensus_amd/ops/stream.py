@@ -22,21 +22,36 @@ def _act(dtype) -> int:
     return int(dtype == torch.float32)
 
 
-def embed_f32(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
-    """Token rows as fp32 into ``out`` [T, W]."""
+def sinusoid_turns(width: int, base: float, device) -> torch.Tensor:
+    """Turns per position of the sinusoids of entries 2i and 2i + 1: base^(-2i / width) / 2 pi, in 64 bits."""
+    i = np.arange((width + 1) // 2, dtype=np.float64)
+    return torch.tensor(base ** (-2.0 * i / width) / (2.0 * np.pi), dtype=torch.float64, device=device)
+
+
+def embed_f32(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float = 1.0, positions=None, turns=None) -> torch.Tensor:
+    """Token rows times ``scale`` as fp32 into ``out`` [T, W]; with ``positions`` plus their sinusoids (``turns`` of
+    :func:`sinusoid_turns`)."""
     if not table.is_cuda:
         out.copy_(table[ids.long()])
+        if scale != 1.0:
+            out.mul_(scale)
+        if positions is not None:
+            out.add_(ref.sinusoids(positions, turns, out.shape[1]))
         return out
     _req(ids, torch.int32, "ids")
     _req(out, torch.float32, "out")
+    if positions is not None:
+        _req(positions, torch.int32, "positions")
+        _req(turns, torch.float64, "turns")
     check(kernels().cfc_embed_f32(out.data_ptr(), table.data_ptr(), ids.data_ptr(), ids.numel(), table.shape[1],
-                                  table.shape[0], _act(table.dtype), _stream(table)), "cfc_embed_f32")
+                                  table.shape[0], _act(table.dtype), float(scale), _p(positions), _p(turns), _stream(table)),
+          "cfc_embed_f32")
     return out
 
 
 class Tail:
-    """The input convolution's paged tail of one layer: rows [blocks, slots, W] fp32, addressed by the
-    batch's block tables."""
+    """The input convolution's tail of one layer: rows [blocks, slots, W] fp32, paged, addressed by the batch's block
+    tables; or (``block_tables`` one-dimensional) [sequence slots, ring, W], addressed by the batch's state slots."""
 
     __slots__ = ("rows", "block_tables")
 
@@ -46,7 +61,9 @@ class Tail:
     def args(self):
         if self.rows is None:
             return [None, 0, None, 1]
-        return [self.rows.data_ptr(), self.rows.shape[1], self.block_tables.data_ptr(), self.block_tables.shape[1]]
+        _req(self.block_tables, torch.int32, "block tables or slots")
+        paged = self.block_tables.dim() == 2
+        return [self.rows.data_ptr(), self.rows.shape[1], self.block_tables.data_ptr(), self.block_tables.shape[1] if paged else 0]
 
 
 class Update:
@@ -144,16 +161,17 @@ def depth_conv_decode(x, hist, up: Update | None, norm_w, eps: float, convs, pos
            outs[1] if two else None, convs[0], convs[1] if two else None, positions, tail, hist)
 
 
-def conv_tiles(portions) -> np.ndarray:
+def conv_tiles(portions, rows: int | None = None) -> np.ndarray:
     """[2, n, 4] int32 tiles of :func:`input_conv`: each portion (first row, rows, first position,
-    sequence) cut at the cache blocks' borders, then per tile the portion's rows before it."""
+    sequence) cut at the cache blocks' borders, or (tails in slots) after every ``rows`` of its rows, at least
+    taps - 1; then per tile the portion's rows before it and in all."""
     tiles, lead = [], []
     for row0, n, pos0, seq in portions:
         r = 0
         while r < n:
-            m = min(n - r, KV_BLOCK - (pos0 + r) % KV_BLOCK)
+            m = min(n - r, rows or KV_BLOCK - (pos0 + r) % KV_BLOCK)
             tiles.append((row0 + r, m, pos0 + r, seq))
-            lead.append((r, 0, 0, 0))
+            lead.append((r, n, 0, 0))
             r += m
     return np.asarray([tiles, lead], np.int32).reshape(2, -1, 4)
 
@@ -183,8 +201,9 @@ def input_conv(x, rstd, norm_w, convs, tiles, tail: Tail, outs) -> None:
 
 
 def clamped_glu(gu, out, limit: float, alpha: float, beta: float, gate_bias=None, up_bias=None,
-                interleaved: bool = False) -> torch.Tensor:
-    """g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + beta) into ``out`` [T, F] (row-strided).
+                interleaved: bool = False, cubic: float = 0.0) -> torch.Tensor:
+    """g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g (1 + cubic g^2)) (u + beta) into ``out`` [T, F]
+    (row-strided).
     ``gu`` [T, 2F], or fp32 slabs [split, T, 2F] to be summed: gate | up halves or the 8-column interleaved
     groups of ops.reference.interleave_gate_up."""
     T, F2 = gu.shape[-2:]
@@ -198,13 +217,13 @@ def clamped_glu(gu, out, limit: float, alpha: float, beta: float, gate_bias=None
             g, u = gu[:, :F2 // 2], gu[:, F2 // 2:]
         g = g + (gate_bias if gate_bias is not None else 0.0)
         u = u + (up_bias if up_bias is not None else 0.0)
-        out.copy_(ref.clamped_glu(g, u, limit, alpha, beta))
+        out.copy_(ref.clamped_glu(g, u, limit, alpha, beta, cubic))
         return out
     if not gu.is_contiguous() or out.shape != (T, F2 // 2):
         raise ValueError(f"clamped_glu: gate / up {tuple(gu.shape)} (contiguous), out {tuple(out.shape)}")
     check(kernels().cfc_clamped_glu(_act(out.dtype), _act(gu.dtype), out.data_ptr(), out.stride(0), gu.data_ptr(), split,
                                     _p(gate_bias), _p(up_bias), T, F2 // 2, int(interleaved), float(limit), float(alpha),
-                                    float(beta), _stream(gu)), "cfc_clamped_glu")
+                                    float(beta), float(cubic), _stream(gu)), "cfc_clamped_glu")
     return out
 
 

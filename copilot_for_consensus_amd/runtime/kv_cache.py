@@ -203,33 +203,35 @@ class PagedHeads:
 
 class GroupedCache:
     """Cache of a decoder of grouped-query attention layers and recurrences, on the same blocks and :class:`BlockPool` as
-    :class:`PagedKVCache`, with state slots per sequence.  Per layer:
-      heads  :class:`PagedHeads`, or the very object of an earlier layer whose keys and values the layer uses
-      tail   [slots + 1, taps - 1, channels] fp32 or None   last inputs of the convolution, position p at p % (taps - 1)
-      recur  [slots + 1, width] fp32 or None                recurrent state
+    :class:`PagedKVCache`, with state slots per sequence.  Per layer (a layer that runs several times: per run):
+      heads  :class:`PagedHeads`, or the very object of an earlier layer whose keys and values the layer uses, or None
+      tail   [slots + 1, rows, channels] fp32 or None   last inputs of the mixer's convolution, position p at p % rows
+      inputs [slots + 1, rows, width] fp32 or None      last inputs of the convolution ahead of the mixer, likewise
+      recur  [slots + 1, width] fp32 or None            recurrent state
     A sequence's state is not in its blocks, so blocks cannot be shared between sequences.  A slot needs no clearing:
     what lies before a sequence's first token is never read."""
 
     share_prefix = False
 
     def __init__(self, layers: list[dict], num_blocks: int, sequences: int, device, dtype=torch.bfloat16):
-        """``layers``: per layer ``heads`` (G, D, pool, entries) or the index of the layer whose it uses, ``tail``
-        (taps - 1, channels) or None, ``recur`` width or None."""
+        """``layers``: per layer ``heads`` (G, D, pool, entries) or the index of the layer whose it uses or None, ``tail`` and
+        ``inputs`` (rows, channels) or None, ``recur`` width or None."""
         self.layers, self.num_blocks = len(layers), num_blocks
         self.dtype, self.device = dtype, torch.device(device)
         self.states = StateSlots(sequences)
         n, f32 = sequences + 1, dict(dtype=torch.float32, device=self.device)
-        self.heads: list[PagedHeads] = []
+        self.heads: list[PagedHeads | None] = []
         for c in layers:
-            h = c["heads"]
-            self.heads.append(self.heads[h] if isinstance(h, int) else PagedHeads(num_blocks, *h, self.device, dtype))
-        self.tail = [torch.zeros(n, *c["tail"], **f32) if c.get("tail") else None for c in layers]
+            h = c.get("heads")
+            self.heads.append(None if h is None else self.heads[h] if isinstance(h, int) else
+                              PagedHeads(num_blocks, *h, self.device, dtype))
+        self.tail, self.inputs = ([torch.zeros(n, *c[k], **f32) if c.get(k) else None for c in layers] for k in ("tail", "inputs"))
         self.recur = [torch.zeros(n, c["recur"], **f32) if c.get("recur") else None for c in layers]
         self.pool = BlockPool(num_blocks)
 
     def nbytes(self) -> int:
-        rows = [t for h in {id(h): h for h in self.heads}.values() for t in h.tensors()]
-        return sum(t.numel() * t.element_size() for t in (*rows, *self.tail, *self.recur) if t is not None)
+        rows = [t for h in {id(h): h for h in self.heads if h is not None}.values() for t in h.tensors()]
+        return sum(t.numel() * t.element_size() for t in (*rows, *self.tail, *self.inputs, *self.recur) if t is not None)
 
 
 def blocks_needed(n_tokens: int) -> int:

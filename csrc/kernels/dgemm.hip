@@ -50,8 +50,8 @@ constexpr int dg_loaders() { return BN / 16 >= 7 ? 1 : 8 - BN / 16 > 2 ? 2 : 8 -
 // B dirty bytes, 2.8-3.8 us behind 12.6-16.8 MB of fp32 partials.
 enum { DG_PART = 0, DG_BF16 = 1, DG_SILU = 2, DG_PART_WT = 3, DG_GLU = 4 };
 
-// constants of the DG_GLU epilogue: min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta)
-struct DgGlu { float limit = 0.f, alpha = 1.f, beta = 0.f; };
+// constants of the DG_GLU epilogue: min(g, limit) sigmoid(alpha g (1 + cubic g^2)) (clamp(u, +-limit) + beta)
+struct DgGlu { float limit = 0.f, alpha = 1.f, beta = 0.f, cubic = 0.f; };
 
 // MX (ablation 64): two X-loader waves and an 8-slot X ring whatever BN -- one loader wave's
 // vmcnt window (63 pieces = 3 stages at BM = 128) may cap the X stream of the wide-BN shapes.
@@ -333,7 +333,7 @@ __global__ void __launch_bounds__((64 * DgShape<BM, BN, (ABL & 64) != 0>::WAVES)
       auto silu_mul = [&](float gate, float up) {
         if constexpr (EPI == DG_GLU) {
           const float gg = fminf(gate, gp.limit), uu = fminf(fmaxf(up, -gp.limit), gp.limit);
-          return gg / (1.f + __expf(-gp.alpha * gg)) * (uu + gp.beta);
+          return gg / (1.f + __expf(-gp.alpha * gg * (1.f + gp.cubic * gg * gg))) * (uu + gp.beta);
         }
         const float gt = bf2f(f2bf(gate)), u = bf2f(f2bf(up));
         return gt / (1.f + __expf(-gt)) * u;
@@ -531,10 +531,10 @@ int dgemm_glu_bn(const void* x, const void* w, int M, int N, int K, int bn, void
 
 // Clamped GLU epilogue over packed, 8-row interleaved gate / up weights: out [M, N / 2] (row stride ldo)
 CFC_API int cfc_dgemm_glu(const void* x, const void* w, int M, int N, int K, int bn, void* out, int ldo, float limit,
-                          float alpha, float beta, hipStream_t stream) {
+                          float alpha, float beta, float cubic, hipStream_t stream) {
   if (const int e = dgemm_check(M, N, K, 1, DG_GLU, bn, nullptr, out, ldo)) return e;
   DgGlu gp;
-  gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
+  gp.limit = limit; gp.alpha = alpha; gp.beta = beta; gp.cubic = cubic;
   int rc;
   switch (cfc_dgemm_bm(M)) {
     case 64: rc = dgemm_glu_bn<64>(x, w, M, N, K, bn, out, ldo, gp, stream); break;

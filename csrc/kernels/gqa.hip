@@ -1,9 +1,12 @@
 // Grouped-query attention over a paged cache where a token sees two ranges of keys under one softmax:
-//   * its window: the last `size` tokens (0: all), and
+//   * its window: the last `size` tokens (0: all), or with `chunk` those of its own run of `size` positions, and
 //   * far keys: the first `keep` tokens, or one mean key and value per block of `pool` tokens that lies wholly ahead
 //     of the window (pooled cache)
-// and a learned sink per head joins the denominator.  Keys and values lie row-major, [blocks][G][32][D]; pooled entries
-// [blocks][G][E][D], entry b of a sequence in page b / E.  Queries [T][H][D] arrive scaled into the exponent's base 2.
+// and a learned sink per head joins the denominator.  Scores may be shaped ahead of the softmax: cap tanh(score / cap),
+// then a bias per head and distance (a table, its last entry for all distances from there on).  Outputs may pass a gate
+// (split_merge.h) and go to rows of any stride.  Keys and values lie row-major, [blocks][G][32][D]; pooled entries
+// [blocks][G][E][D], entry b of a sequence in page b / E.  Queries [T][H][D] arrive scaled into the exponent's base 2,
+// with a cap so that exp2 of the score is e^(2 score / cap).
 // Heads h of G groups: R = H / G consecutive heads share a key / value head.
 //
 //   * gqa_decode   one token per sequence: a workgroup per (sequence, key head, slice of its keys), its four waves on
@@ -34,6 +37,10 @@ struct GqaArgs {
   int n_tiles;
   int H, G, D, DV, max_blocks, P;      // DV: value columns that leave
   int size, keep, pool, le;            // window; first tokens; tokens per pooled block, log2 of entries per page
+  int chunk;                           // size counts from multiples of it
+  int capped; float cap2;              // 0: no cap, 1: any score, 2: |score| <= CAP_NEAR cap; cap log2(e)
+  const float* bias; int nb;           // [H][nb] by distance, times log2(e) (null: none)
+  OutGate og;
   const float* sink;          // [H] or null
   float* part_o;              // [rows][P][D], unnormalised
   float* part_ml;             // [rows][P][2]
@@ -42,13 +49,32 @@ struct GqaArgs {
 // pooled blocks the token at pos sees
 __device__ __forceinline__ int pooled_seen(const GqaArgs& a, int pos) { return max(pos - a.size + 1, 0) / a.pool; }
 
+// the window's first key for the row at pos (size > 0)
+__device__ __forceinline__ int window_first(const GqaArgs& a, int pos) { return a.chunk ? pos - pos % a.size : max(0, pos - a.size + 1); }
+
+constexpr float LN2 = 0.69314718055994531f;
+constexpr float CAP_NEAR = 0.35f;
+
+// the capped score (base 2) of a score s = 2 log2(e) score / cap.  Near zero by the series of tanh in x = s ln(2) / 2 (its
+// next term, 62 / 2835 x^9, is below 3e-6 of x)
+template <typename ACT>
+__device__ __forceinline__ float cap_score(const GqaArgs& a, float s) {
+  if constexpr (sizeof(ACT) == 4) return a.cap2 * tanhf(s * (0.5f * LN2));
+  if (a.capped == 2) {
+    constexpr float h = 0.5f * LN2, h2 = h * h;
+    const float t = s * s;
+    return s * (a.cap2 * h) * (1.f + t * (-h2 / 3.f + t * (2.f * h2 * h2 / 15.f - t * (17.f * h2 * h2 * h2 / 315.f))));
+  }
+  return a.cap2 - 2.f * a.cap2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s));
+}
+
 // Tiles of KT keys for rows at positions pmin .. pmax: first `nat` of the far range (`na` keys), then the window's,
 // from key `lo` on
 struct KeyTiles { int na, nat, lo, nt; };
 template <int KT>
 __device__ __forceinline__ KeyTiles key_tiles(const GqaArgs& a, int pmin, int pmax) {
   KeyTiles r;
-  r.lo = a.size > 0 ? max(0, pmin - a.size + 1) / KT * KT : 0;
+  r.lo = a.size > 0 ? window_first(a, pmin) / KT * KT : 0;
   r.na = a.size == 0 ? 0 : a.pool ? pooled_seen(a, pmax) : min(a.keep, r.lo);
   r.nat = (r.na + KT - 1) / KT;
   r.nt = r.nat + pmax / KT - r.lo / KT + 1;
@@ -57,7 +83,7 @@ __device__ __forceinline__ KeyTiles key_tiles(const GqaArgs& a, int pmin, int pm
 
 // a window tile's key j for the row at pos
 __device__ __forceinline__ bool sees(const GqaArgs& a, int pos, int j) {
-  return j <= pos && (a.size == 0 || pos - j < a.size || j < a.keep);
+  return j <= pos && (a.size == 0 || j >= window_first(a, pos) || j < a.keep);
 }
 
 // where key e of a tile range lies: its table entry, then (with the page) its row of the [.][G][.] cache
@@ -109,7 +135,7 @@ __device__ __forceinline__ void wave_lds_fence() {
 
 // ------------------------------------------------------------------------------------------ decoded tokens
 // grid (B * G * ceil(R / 16), P)
-template <int D>
+template <int D, bool SHAPED>
 __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) gqa_decode_kernel(const uint16_t* __restrict__ q,
                                                                           const uint16_t* __restrict__ kc,
                                                                           const uint16_t* __restrict__ vc,
@@ -137,6 +163,8 @@ __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) gqa_decode_kernel(const
     qf[k] = *reinterpret_cast<const u32x4_t*>(q + (qrow + min(col, nr - 1)) * D + 32 * k + 8 * kq);
 
   char* vbuf = smem + w * 64 * D;
+  const float* bias = SHAPED && a.bias ? a.bias + (size_t)(hk * R + r0 + min(col, nr - 1)) * a.nb : nullptr;
+  const float far_bias = bias ? bias[a.nb - 1] : 0.f;
   u32x4_t kf[2][KS], vf[NV];
   // row of this lane's key (lane & 31) in a tile; tiles past the slice: its last
   auto rows_of = [&](int t) {
@@ -187,6 +215,25 @@ __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) gqa_decode_kernel(const
       load(t + 4, row);                      // past the slice: re-read, not used
       row = rows_of(t + 8);
       const bool far = t < kt.nat;
+      if constexpr (SHAPED) {
+        const int k0 = far ? 32 * t : kt.lo + 32 * (t - kt.nat);
+        float bt8[2][4];
+        if (bias && pos - k0 - 31 < a.nb - 1) {
+#pragma unroll
+          for (int g = 0; g < 2; ++g)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) bt8[g][i] = bias[min(max(pos - k0 - (16 * g + 4 * kq + i), 0), a.nb - 1)];
+        } else {
+#pragma unroll
+          for (int g = 0; g < 2; ++g)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) bt8[g][i] = far_bias;
+        }
+#pragma unroll
+        for (int g = 0; g < 2; ++g)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) sc[g][i] = (a.capped ? cap_score<uint16_t>(a, sc[g][i]) : sc[g][i]) + bt8[g][i];
+      }
       float mx = -INFINITY;
 #pragma unroll
       for (int g = 0; g < 2; ++g)
@@ -266,22 +313,31 @@ __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) gqa_decode_kernel(const
       continue;
     }
     const float inv = sink_inv(a, hk * R + r0 + r, M, L);
-    uint16_t* dst = out + grow * a.DV + c;
-    if (a.DV % 4 == 0) {
-      if (c < a.DV) *reinterpret_cast<uint2*>(dst) = make_uint2(cvt_pk_bf16_f32(y[0] * inv, y[1] * inv), cvt_pk_bf16_f32(y[2] * inv, y[3] * inv));
+    const int oc = (hk * R + r0 + r) * a.DV + c;
+    uint16_t* dst = out + s * a.og.ld + oc;
+    if (a.og.vec) {
+      if (c < a.DV) {
+        const f32x4_t f = inv * out_gate4<uint16_t>(a.og, s, oc);
+        *reinterpret_cast<uint2*>(dst) = make_uint2(cvt_pk_bf16_f32(y[0] * f[0], y[1] * f[1]), cvt_pk_bf16_f32(y[2] * f[2], y[3] * f[3]));
+      }
     } else {
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (c + i < a.DV) dst[i] = f2bf(y[i] * inv);
+        if (c + i < a.DV) dst[i] = f2bf(y[i] * inv * out_gate<uint16_t>(a.og, s, oc + i));
     }
   }
 }
 
 // ------------------------------------------------------------------------------------------ prompt portions
+// biases of one head in LDS, and whether a group's leave two workgroups a CU
+constexpr int BIAS_PAD = 3;
+__host__ __device__ __forceinline__ int bias_stride(int nb) { return (nb + 2 * BIAS_PAD) | 1; }
+__host__ __device__ __forceinline__ bool bias_in_lds(int R, int nb) { return (int64_t)R * bias_stride(nb) <= 4096; }
+
 // 1-D grid of n_tiles * G, tile major: in the tiles' order (those with the most keys first, so that long ones do not end
 // the grid alone), and an XCD takes one key head of eight, whose keys its L2 then holds.
 // A tile is 32 NW rows (row r of a portion and key head: token r / R, head r % R of the group).
-template <int D, int NW>
+template <int D, int NW, bool SHAPED>
 __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(const uint16_t* __restrict__ q,
                                                                               const uint16_t* __restrict__ kc,
                                                                               const uint16_t* __restrict__ vc,
@@ -291,7 +347,7 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
   constexpr int NT = 64 * NW, CH = D / 8, NL = (64 * CH + NT - 1) / NT, KS = D / 16, DT = D / 32;
   constexpr bool EVEN = 64 * CH % NT == 0;
   constexpr int TILE = 64 * D * 2;
-  extern __shared__ __attribute__((aligned(16))) char smem[];          // [2][K | V]
+  extern __shared__ __attribute__((aligned(16))) char smem[];          // [2][K | V], then the group's biases (bias_stride)
   const int tile = blockIdx.x / a.G, hk = blockIdx.x - tile * a.G;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l32 = lane & 31, hi = lane >> 5;
   const int R = a.H / a.G, s = a.tile_seq[tile], m0 = a.tile_m0[tile];
@@ -354,6 +410,23 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
   gload(0);
   ids(1);
   lwrite(0);
+  // biases by falling distance, the ends repeated BIAS_PAD times: four neighbouring keys' are four neighbours here
+  const int bs = SHAPED && a.bias ? bias_stride(a.nb) : 0;
+  const float* lb = nullptr;
+  float far_bias = 0.f;
+  if constexpr (SHAPED) {
+    if (a.bias) {
+      far_bias = a.bias[(size_t)head * a.nb + a.nb - 1];
+      float* tab = reinterpret_cast<float*>(smem + 4 * TILE);
+      if (bias_in_lds(R, a.nb)) {
+        for (int e = tid; e < R * bs; e += NT) {
+          const int r = e / bs, i = e - r * bs;
+          tab[e] = a.bias[(size_t)(hk * R + r) * a.nb + min(max(a.nb - 1 - (i - BIAS_PAD), 0), a.nb - 1)];
+        }
+        lb = tab + (head - hk * R) * bs + BIAS_PAD;
+      }
+    }
+  }
   __syncthreads();
   for (int t = 0; t < kt.nt; ++t) {
     gload(t + 1);
@@ -362,8 +435,8 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
     const int k0 = far ? 64 * t : kt.lo + 64 * (t - kt.nat);
     // what this wave's rows see of the tile: nothing, some, all
     const int seen0 = a.pool ? pooled_seen(a, wp0) : kt.na, seen1 = a.pool ? pooled_seen(a, wp1) : kt.na;
-    const bool none = far ? k0 >= seen1 : k0 > wp1 || (a.size > 0 && k0 + 63 <= wp0 - a.size && k0 >= a.keep);
-    const bool all = far ? k0 + 64 <= seen0 : k0 + 63 <= wp0 && (a.size == 0 || k0 > wp1 - a.size);
+    const bool none = far ? k0 >= seen1 : k0 > wp1 || (a.size > 0 && k0 + 63 < window_first(a, wp0) && k0 >= a.keep);
+    const bool all = far ? k0 + 64 <= seen0 : k0 + 63 <= wp0 && (a.size == 0 || k0 >= window_first(a, wp1));
     if (!none) {
       const char* kb = smem + (t & 1) * 2 * TILE;
       const char* vb = kb + TILE;
@@ -373,7 +446,7 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
       for (int h = 0; h < 2; ++h) {
         const int key = 32 * h + l32;
 #pragma unroll
-        for (int r = 0; r < 16; ++r) sc[h][r] = -ref0;
+        for (int r = 0; r < 16; ++r) sc[h][r] = SHAPED ? 0.f : -ref0;
         constexpr int KB = KS <= 8 ? KS : KS / 2;         // fragments in batches: one LDS round trip each
 #pragma unroll
         for (int b0 = 0; b0 < KS; b0 += KB) {
@@ -385,6 +458,35 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
           for (int k = 0; k < KB; ++k) sc[h] = mfma32(kf[k], qf[b0 + k], sc[h]);
           __builtin_amdgcn_sched_group_barrier(0x100, KB, 0);
           __builtin_amdgcn_sched_group_barrier(0x008, KB, 0);
+        }
+      }
+      if constexpr (SHAPED) {
+        if (a.capped)
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) sc[h][r] = cap_score<uint16_t>(a, sc[h][r]);
+        if (a.bias && wp0 - (k0 + 63) < a.nb - 1) {
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int g = 0; g < 4; ++g) {
+              const int n = my_pos - (k0 + 32 * h + 8 * g + 4 * hi);          // the first key's distance
+              if (lb) {
+                const float* b = lb + min(max(a.nb - 1 - n, -BIAS_PAD), a.nb - 1);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) sc[h][4 * g + i] += b[i] - ref0;
+              } else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                  sc[h][4 * g + i] += a.bias[(size_t)head * a.nb + min(max(n - i, 0), a.nb - 1)] - ref0;
+              }
+            }
+        } else {
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) sc[h][r] += far_bias - ref0;
         }
       }
       if (!all) {
@@ -453,20 +555,23 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
   const float l = xor32_sum((lp[0] + lp[1]) + (lp[2] + lp[3]));
   if (my >= rows) return;
   const float inv = sink_inv(a, head, m, l);
-  uint16_t* dst = out + ((size_t)(q0 + my_tok) * a.H + head) * a.DV;
+  const int token = q0 + my_tok, oc = head * a.DV;
+  uint16_t* dst = out + token * a.og.ld + oc;
 #pragma unroll
   for (int d = 0; d < DT; ++d)
 #pragma unroll
     for (int g = 0; g < 4; ++g) {
       const int c = 32 * d + 8 * g + 4 * hi;
-      if (a.DV % 4 == 0) {
-        if (c < a.DV)
-          *reinterpret_cast<uint2*>(dst + c) = make_uint2(cvt_pk_bf16_f32(o[d][4 * g] * inv, o[d][4 * g + 1] * inv),
-                                                          cvt_pk_bf16_f32(o[d][4 * g + 2] * inv, o[d][4 * g + 3] * inv));
+      if (a.og.vec) {
+        if (c < a.DV) {
+          const f32x4_t f = inv * out_gate4<uint16_t>(a.og, token, oc + c);
+          *reinterpret_cast<uint2*>(dst + c) = make_uint2(cvt_pk_bf16_f32(o[d][4 * g] * f[0], o[d][4 * g + 1] * f[1]),
+                                                          cvt_pk_bf16_f32(o[d][4 * g + 2] * f[2], o[d][4 * g + 3] * f[3]));
+        }
       } else {
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          if (c + i < a.DV) dst[c + i] = f2bf(o[d][4 * g + i] * inv);
+          if (c + i < a.DV) dst[c + i] = f2bf(o[d][4 * g + i] * inv * out_gate<uint16_t>(a.og, token, oc + c + i));
       }
     }
 }
@@ -515,6 +620,8 @@ __global__ void __launch_bounds__(256) gqa_any_kernel(const ACT* __restrict__ q,
 #pragma unroll
         for (int u = 0; u < 4; ++u) s4[u] += myq[r + u] * ldf(c + r + u);
       sc = (s4[0] + s4[1]) + (s4[2] + s4[3]);
+      if (a.capped) sc = cap_score<float>(a, sc);
+      if (a.bias) sc += a.bias[(size_t)head * a.nb + min(pos - e, a.nb - 1)];
     }
     const float mn = fmaxf(m, wave_max(sc)), ref = mn == -INFINITY ? 0.f : mn;
     const float alpha = exp2f(m - ref), p = exp2f(sc - ref);
@@ -544,7 +651,8 @@ __global__ void __launch_bounds__(256) gqa_any_kernel(const ACT* __restrict__ q,
     if (a.P > 1) {
       if (c < D) a.part_o[(grow * a.P + blockIdx.y) * D + c] = o[j];
     } else if (c < a.DV) {
-      stf(out + grow * a.DV + c, o[j] * inv);
+      const int token = q0 + mrow / a.H, oc = head * a.DV + c;
+      stf(out + token * a.og.ld + oc, o[j] * inv * out_gate<ACT>(a.og, token, oc));
     }
   }
   if (a.P > 1 && lane == 0) {
@@ -553,16 +661,17 @@ __global__ void __launch_bounds__(256) gqa_any_kernel(const ACT* __restrict__ q,
   }
 }
 
-template <int D, int NW>
+template <int D, int NW, bool SHAPED>
 int prompt_go(int grid, hipStream_t s, const void* q, const void* kc, const void* vc, const void* pk, const void* pv,
               const GqaArgs& a, void* out) {
-  constexpr int lds = 2 * 2 * 64 * D * 2;
+  constexpr int tiles = 2 * 2 * 64 * D * 2, most = tiles + (SHAPED ? 16384 : 0);
   static bool raised = false;
-  if (lds > 65536 && !raised) {
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&gqa_prompt_kernel<D, NW>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+  if (most > 65536 && !raised) {
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&gqa_prompt_kernel<D, NW, SHAPED>), hipFuncAttributeMaxDynamicSharedMemorySize, most);
     raised = true;
   }
-  gqa_prompt_kernel<D, NW><<<grid, 64 * NW, lds, s>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc,
+  const int R = a.H / a.G, lds = tiles + (SHAPED && a.bias && bias_in_lds(R, a.nb) ? 4 * R * bias_stride(a.nb) : 0);
+  gqa_prompt_kernel<D, NW, SHAPED><<<grid, 64 * NW, lds, s>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc,
                                                      (const uint16_t*)pk, (const uint16_t*)pv, a, (uint16_t*)out);
   return CFC_CHECK_LAUNCH();
 }
@@ -577,23 +686,40 @@ CFC_API int cfc_gqa_prompt_rows(int D) {
 }
 
 // q [T][H][D] scaled by log2(e); caches [blocks][G][32][D], pooled [blocks][G][1 << le][D]; out [T][H][DV].
-// kind 0: general (tiles of 4 rows over all heads; tile_seq null: one token per sequence), 1: decode, 2: prompt portions
+// kind 0: general (tiles of 4 rows over all heads; tile_seq null: one token per sequence), 1: decode, 2: prompt portions.
+// chunk: the window is the row's own run of size positions.  capped 1 or 2 (|score| <= 0.35 cap): q scaled by 2 log2(e) / cap
+// instead, cap2 = cap log2(e).  bias [H][nb] times log2(e), by distance.  gate: columns [T][H DV] of a product (gate_split 0:
+// activations, else fp32 slabs; null: none) that, as oscale sigmoid(gate), multiply the output, whose rows have stride ldo
 CFC_API int cfc_gqa_attention(int kind, int f32, const void* q, const void* kc, const void* vc, const void* pk, const void* pv,
                               const int32_t* block_tables, const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tile_seq,
                               const int32_t* tile_m0, int n_tiles, int B, int H, int G, int D, int DV, int max_blocks, int size,
-                              int keep, int pool, int le, const float* sink, int P, int total_rows, float* part_o, float* part_ml,
-                              void* out, hipStream_t stream) {
+                              int keep, int pool, int le, int chunk, int capped, float cap2, const float* bias, int nb,
+                              const float* sink, const void* gate, int gate_split, int64_t gate_ld, int64_t gate_plane, float oscale,
+                              int P, int total_rows, float* part_o, float* part_ml, void* out, int64_t ldo, hipStream_t stream) {
   if (B <= 0 || (kind != 1 && n_tiles <= 0)) return 0;
   if (H < 1 || G < 1 || H % G || D < 32 || D % 32 || D > 1024 || DV < 1 || DV > D || max_blocks < 1 || P < 1 || P > MERGE_MAXP) return -1;
   if (size < 0 || keep < 0 || pool < 0 || (pool && (keep || !pk || !pv || le < 0 || le > 5 || (pool << le) < CFC_KV_BS || size < 1))) return -2;
+  if (chunk && (size < 1 || pool)) return -2;
+  if (capped < 0 || capped > 2 || (capped && !(cap2 > 0.f)) || (bias && nb < 1) || (bias && pool)) return -7;
+  if (ldo < (int64_t)H * DV || (gate && (gate_split < 0 || gate_ld < (int64_t)H * DV))) return -8;
   if (P > 1 && (!part_o || !part_ml)) return -3;
   if (kind == 2 && (P != 1 || !cu_q || !tile_seq || !tile_m0)) return -4;
   if (kind != 0 && (f32 || cfc_gqa_prompt_rows(D) == 0)) return -5;
+  OutGate og;
+  og.p = gate; og.split = gate_split; og.pld = gate_ld; og.plane = gate_plane; og.scale = oscale; og.ld = ldo;
+  const int esz = f32 ? 4 : 2, gsz = gate_split ? 4 : esz;
+  og.vec = DV % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)out & (4 * esz - 1)) == 0 &&
+           (!gate || (gate_ld % 4 == 0 && gate_plane % 4 == 0 && ((uintptr_t)gate & (4 * gsz - 1)) == 0));
   const GqaArgs a{block_tables, cu_q, ctx_lens, tile_seq, tile_m0, n_tiles, H, G, D, DV, max_blocks, P, size, keep, pool, le,
-                  sink, part_o, part_ml};
+                  chunk, capped, cap2, bias, nb, og, sink, part_o, part_ml};
+  const bool shaped = capped || bias;
   int rc = -6;
   if (kind == 2) {
-#define GP(DD) case DD: rc = prompt_go<DD, prompt_waves(DD)>(n_tiles * G, stream, q, kc, vc, pk, pv, a, out); break
+#define GP(DD)                                                                                                       \
+  case DD:                                                                                                           \
+    rc = shaped ? prompt_go<DD, prompt_waves(DD), true>(n_tiles * G, stream, q, kc, vc, pk, pv, a, out)              \
+                : prompt_go<DD, prompt_waves(DD), false>(n_tiles * G, stream, q, kc, vc, pk, pv, a, out);            \
+    break
     switch (D) { GP(32); GP(64); GP(96); GP(128); GP(160); GP(192); GP(256); }
 #undef GP
     return rc;
@@ -602,8 +728,12 @@ CFC_API int cfc_gqa_attention(int kind, int f32, const void* q, const void* kc, 
     const dim3 grid(B * G * ((H / G + 15) / 16), P);
 #define GD(DD)                                                                                                            \
   case DD:                                                                                                                \
-    gqa_decode_kernel<DD><<<grid, 256, 0, stream>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc,         \
-                                                    (const uint16_t*)pk, (const uint16_t*)pv, a, (uint16_t*)out);         \
+    if (shaped)                                                                                                           \
+      gqa_decode_kernel<DD, true><<<grid, 256, 0, stream>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc, \
+                                                            (const uint16_t*)pk, (const uint16_t*)pv, a, (uint16_t*)out); \
+    else                                                                                                                  \
+      gqa_decode_kernel<DD, false><<<grid, 256, 0, stream>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc, \
+                                                             (const uint16_t*)pk, (const uint16_t*)pv, a, (uint16_t*)out); \
     rc = CFC_CHECK_LAUNCH();                                                                                              \
     break
     switch (D) { GD(32); GD(64); GD(96); GD(128); GD(160); GD(192); GD(256); }
@@ -620,7 +750,7 @@ CFC_API int cfc_gqa_attention(int kind, int f32, const void* q, const void* kc, 
     rc = CFC_CHECK_LAUNCH();
   }
   if (rc || P == 1) return rc;
-  if (f32) slice_merge_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, D, DV, sink, H, (float*)out);
-  else slice_merge_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, D, DV, sink, H, (uint16_t*)out);
+  if (f32) slice_merge_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, D, DV, sink, H, og, (float*)out);
+  else slice_merge_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, D, DV, sink, H, og, (uint16_t*)out);
   return CFC_CHECK_LAUNCH();
 }

@@ -5,9 +5,9 @@
 //   * gru_step    one token per sequence, straight from a joint product's slabs
 //   * gru_chunk   prompt portions, chunks of 64 tokens in parallel: each chunk's decay (the product of 1 - z) and what
 //                 it adds to a state of zero
-//   * gru_carry   per sequence through its chunks: the state ahead of each, and the one the portion leaves
+//   * carry       per sequence through its chunks: the state ahead of each, and the one the portion leaves (recur.h)
 //   * gru_apply   the chunks again from their states: outputs
-#include "rows.h"
+#include "recur.h"
 
 namespace {
 
@@ -21,14 +21,6 @@ __device__ __forceinline__ Vec<V> gru_ld(const GruCols& a, int64_t t, int c) {
   add_slabs<V>(y, reinterpret_cast<const float*>(a.p), a.split, a.plane, (size_t)o);
   return y;
 }
-
-// ACT decides the exponential and the reciprocal: the hardware's for bf16 activations, the library's on the 32-bit path
-template <typename ACT> __device__ __forceinline__ float exp_of(float x);
-template <> __device__ __forceinline__ float exp_of<uint16_t>(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
-template <> __device__ __forceinline__ float exp_of<float>(float x) { return expf(x); }
-template <typename ACT> __device__ __forceinline__ float over1(float x);              // 1 / (1 + x)
-template <> __device__ __forceinline__ float over1<uint16_t>(float x) { return __builtin_amdgcn_rcpf(1.f + x); }
-template <> __device__ __forceinline__ float over1<float>(float x) { return 1.f / (1.f + x); }
 
 // decay 1 - z and contribution z c of one token.  With t = exp(pre_z): 1 - z = 1 / (1 + t) and z = t / (1 + t), neither
 // the other's difference from 1, so that small ones keep their digits; sigmoid(min(u, 0)) is 1/2 where u >= 0
@@ -67,7 +59,7 @@ template <typename ACT, int V>
 __global__ void __launch_bounds__(64) gru_step_kernel(GruCols z, GruCols u, GruCols g, const float* __restrict__ bz,
                                                      const float* __restrict__ bx, const int32_t* __restrict__ slots,
                                                      const int32_t* __restrict__ ctx_lens, int W, float* __restrict__ state,
-                                                     ACT* __restrict__ out) {
+                                                     ACT* __restrict__ out, int64_t ldo, float oscale) {
   const int b = blockIdx.x, c = (blockIdx.y * 64 + threadIdx.x) * V;
   if (c >= W) return;
   float* sp = state + (size_t)slots[b] * W + c;
@@ -80,10 +72,10 @@ __global__ void __launch_bounds__(64) gru_step_kernel(GruCols z, GruCols u, GruC
     float a, k;
     gru_gates<ACT>(zv.v[e] + vz.v[e], uv.v[e] + vx.v[e], a, k);
     S.v[e] = a * S.v[e] + k;
-    o.v[e] = S.v[e] * silu<ACT>(gv.v[e]);
+    o.v[e] = S.v[e] * silu<ACT>(gv.v[e]) * oscale;
   }
   stv<V>(sp, S);
-  stv<V>(out + (size_t)b * W + c, o);
+  stv<V>(out + b * ldo + c, o);
 }
 
 constexpr int GRU_FLIGHT = 8;        // rows requested ahead of their use
@@ -129,39 +121,11 @@ __global__ void __launch_bounds__(64) gru_chunk_kernel(GruRows z, GruRows u, con
   stv<V>(o + W, B);
 }
 
-// sums[chunk][0] becomes the state ahead of the chunk
-template <int V>
-__global__ void __launch_bounds__(64) gru_carry_kernel(const int32_t* __restrict__ chunk_cu, const int32_t* __restrict__ cu_q,
-                                                      const int32_t* __restrict__ ctx_lens, const int32_t* __restrict__ slots,
-                                                      int W, float* __restrict__ sums, float* __restrict__ state) {
-  const int s = blockIdx.x, c = (blockIdx.y * 64 + threadIdx.x) * V;
-  if (c >= W) return;
-  const int i0 = chunk_cu[s], i1 = chunk_cu[s + 1];
-  float* sp = state + (size_t)slots[s] * W + c;
-  Vec<V> S = ctx_lens[s] > cu_q[s + 1] - cu_q[s] ? ldv<V>(sp) : zerov<V>();
-  for (int i = i0; i < i1; i += GRU_FLIGHT) {
-    Vec<V> A[GRU_FLIGHT], B[GRU_FLIGHT];
-#pragma unroll
-    for (int k = 0; k < GRU_FLIGHT; ++k) {
-      const float* p = sums + (size_t)min(i + k, i1 - 1) * 2 * W + c;
-      A[k] = ldv<V>(p);
-      B[k] = ldv<V>(p + W);
-    }
-#pragma unroll
-    for (int k = 0; k < GRU_FLIGHT; ++k)
-      if (i + k < i1) {
-        stv<V>(sums + (size_t)(i + k) * 2 * W + c, S);
-#pragma unroll
-        for (int e = 0; e < V; ++e) S.v[e] = A[k].v[e] * S.v[e] + B[k].v[e];
-      }
-  }
-  stv<V>(sp, S);
-}
-
 template <typename ACT, int V>
 __global__ void __launch_bounds__(64) gru_apply_kernel(GruRows z, GruRows u, GruRows g, const float* __restrict__ bz,
                                                       const float* __restrict__ bx, const int32_t* __restrict__ chunks, int W,
-                                                      const float* __restrict__ sums, ACT* __restrict__ out) {
+                                                      const float* __restrict__ sums, ACT* __restrict__ out, int64_t ldo,
+                                                      float oscale) {
   const int c = (blockIdx.y * 64 + threadIdx.x) * V;
   if (c >= W) return;
   const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1];
@@ -192,16 +156,16 @@ __global__ void __launch_bounds__(64) gru_apply_kernel(GruRows z, GruRows u, Gru
           float a, k;
           gru_gates<ACT>(zr.at(e) + vz.v[e], ur.at(e) + vx.v[e], a, k);
           S.v[e] = a * S.v[e] + k;
-          o.v[e] = S.v[e] * silu<ACT>(gr.at(e));
+          o.v[e] = S.v[e] * silu<ACT>(gr.at(e)) * oscale;
         }
-        stv<V>(out + (size_t)(row0 + r0 + i) * W + c, o);
+        stv<V>(out + (row0 + r0 + i) * ldo + c, o);
       }
     }
 }
 
 // vectors of four where every operand's rows allow them
-bool gru_vec(const GruCols* a, int n, int W, int f32) {
-  bool v = W % 4 == 0;
+bool gru_vec(const GruCols* a, int n, int W, int f32, const void* out, int64_t ldo) {
+  bool v = W % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)out & (f32 ? 15 : 7)) == 0;
   for (int i = 0; i < n; ++i)
     v = v && a[i].ld % 4 == 0 && a[i].plane % 4 == 0 && ((uintptr_t)a[i].p & (a[i].split == 0 && !f32 ? 7 : 15)) == 0;
   return v;
@@ -209,17 +173,18 @@ bool gru_vec(const GruCols* a, int n, int W, int f32) {
 
 }  // namespace
 
-// z, u, g: columns of products (pointer, split (0: activations, else fp32 slabs), row stride, slab stride)
+// z, u, g: columns of products (pointer, split (0: activations, else fp32 slabs), row stride, slab stride); out rows of stride
+// ldo, times oscale
 CFC_API int cfc_gru_step(int f32, const void* z, int z_split, int64_t z_ld, int64_t z_plane, const void* u, int u_split,
                          int64_t u_ld, int64_t u_plane, const void* g, int g_split, int64_t g_ld, int64_t g_plane, const float* bz,
                          const float* bx, const int32_t* slots, const int32_t* ctx_lens, int B, int W, float* state, void* out,
-                         hipStream_t stream) {
+                         int64_t ldo, float oscale, hipStream_t stream) {
   if (B <= 0) return 0;
-  if (W < 1 || !slots || !ctx_lens || !state) return -1;
+  if (W < 1 || !slots || !ctx_lens || !state || ldo < W) return -1;
   const GruCols a[3] = {{z, z_split, z_ld, z_plane}, {u, u_split, u_ld, u_plane}, {g, g_split, g_ld, g_plane}};
 #define GS(ACT, V) \
-  gru_step_kernel<ACT, V><<<dim3(B, (W + 64 * V - 1) / (64 * V)), 64, 0, stream>>>(a[0], a[1], a[2], bz, bx, slots, ctx_lens, W, state, (ACT*)out)
-  const bool v4 = gru_vec(a, 3, W, f32);
+  gru_step_kernel<ACT, V><<<dim3(B, (W + 64 * V - 1) / (64 * V)), 64, 0, stream>>>(a[0], a[1], a[2], bz, bx, slots, ctx_lens, W, state, (ACT*)out, ldo, oscale)
+  const bool v4 = gru_vec(a, 3, W, f32, out, ldo);
   if (f32) { if (v4) GS(float, 4); else GS(float, 1); }
   else if (v4) GS(uint16_t, 4);
   else GS(uint16_t, 1);
@@ -232,19 +197,19 @@ CFC_API int cfc_gru_step(int f32, const void* z, int z_split, int64_t z_ld, int6
 CFC_API int cfc_gru_prefill(int f32, const void* z, int64_t z_ld, const void* u, int64_t u_ld, const void* g, int64_t g_ld,
                             const float* bz, const float* bx, const int32_t* chunks, int n, const int32_t* chunk_cu,
                             const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* slots, int portions, int W, float* sums,
-                            float* state, void* out, hipStream_t stream) {
+                            float* state, void* out, int64_t ldo, float oscale, hipStream_t stream) {
   if (n <= 0 || portions <= 0) return 0;
-  if (W < 1 || !chunks || !chunk_cu || !cu_q || !ctx_lens || !slots || !sums || !state) return -1;
+  if (W < 1 || !chunks || !chunk_cu || !cu_q || !ctx_lens || !slots || !sums || !state || ldo < W) return -1;
   const GruCols a[3] = {{z, 0, z_ld, 0}, {u, 0, u_ld, 0}, {g, 0, g_ld, 0}};
   const GruRows r[3] = {{z, z_ld}, {u, u_ld}, {g, g_ld}};
 #define GP(ACT, V)                                                                                                    \
   do {                                                                                                                \
     const int gy = (W + 64 * V - 1) / (64 * V);                                                                       \
     gru_chunk_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(r[0], r[1], bz, bx, chunks, W, sums);                    \
-    gru_carry_kernel<V><<<dim3(portions, gy), 64, 0, stream>>>(chunk_cu, cu_q, ctx_lens, slots, W, sums, state);      \
-    gru_apply_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(r[0], r[1], r[2], bz, bx, chunks, W, sums, (ACT*)out);   \
+    carry_kernel<V><<<dim3(portions, gy), 64, 0, stream>>>(chunk_cu, cu_q, ctx_lens, slots, W, sums, state);      \
+    gru_apply_kernel<ACT, V><<<dim3(n, gy), 64, 0, stream>>>(r[0], r[1], r[2], bz, bx, chunks, W, sums, (ACT*)out, ldo, oscale);   \
   } while (0)
-  const bool v4 = gru_vec(a, 3, W, f32);
+  const bool v4 = gru_vec(a, 3, W, f32, out, ldo);
   if (f32) { if (v4) GP(float, 4); else GP(float, 1); }
   else if (v4) GP(uint16_t, 4);
   else GP(uint16_t, 1);

@@ -1048,8 +1048,10 @@ CFC_API int cfc_latent_attention(int f32, const void* q, const void* cache, cons
 #undef LAT
   }
   if (rc || P == 1) return rc;
-  if (f32) slice_merge_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, RV, sink, H, (float*)out);
-  else slice_merge_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, RV, sink, H, (uint16_t*)out);
+  OutGate g;
+  g.ld = (int64_t)H * RV;
+  if (f32) slice_merge_kernel<float><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, RV, sink, H, g, (float*)out);
+  else slice_merge_kernel<uint16_t><<<total_rows, 128, 0, stream>>>(part_o, part_ml, P, RV, RV, sink, H, g, (uint16_t*)out);
   return CFC_CHECK_LAUNCH();
 }
 

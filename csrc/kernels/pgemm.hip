@@ -62,8 +62,8 @@ __device__ __forceinline__ float pg_gelu(float v) { return 0.5f * v * (1.f + erf
 __device__ __forceinline__ float pg_bfr(float v) { return bf2f(f2bf(v)); }
 
 // Gated epilogues over 8-row interleaved gate / up weights: PG_SWIGLU silu(g) * u, and PG_GLU
-// min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta) with the constants of PgGlu.
-struct PgGlu { float limit = 0.f, alpha = 1.f, beta = 0.f; };
+// min(g, limit) sigmoid(alpha g (1 + cubic g^2)) (clamp(u, +-limit) + beta) with the constants of PgGlu.
+struct PgGlu { float limit = 0.f, alpha = 1.f, beta = 0.f, cubic = 0.f; };
 constexpr bool pg_gated(int epi) { return epi == PG_SWIGLU || epi == PG_GLU; }
 
 // SwiGLU of one 4-value accumulator group (16-row n-tile = 8 gate rows then 8 up rows: lanes
@@ -81,7 +81,7 @@ __device__ __forceinline__ uint32_t pg_gate2(const float (&v)[4], const PgGlu& p
   if constexpr (EPI == PG_GLU) {
     auto glu = [&](float gate, float up) {
       const float gg = fminf(gate, p.limit), uu = fminf(fmaxf(up, -p.limit), p.limit);
-      return gg * __builtin_amdgcn_rcpf(1.f + __expf(-p.alpha * gg)) * (uu + p.beta);
+      return gg * __builtin_amdgcn_rcpf(1.f + __expf(-p.alpha * gg * (1.f + p.cubic * gg * gg))) * (uu + p.beta);
     };
     return pack2bf(glu(g0, u0), glu(g1, u1));
   }
@@ -1396,15 +1396,15 @@ CFC_API int cfc_pgemm(const void* x, const void* w, const void* bias, void* out,
 }
 
 // Clamped GLU epilogue over packed, 8-row interleaved gate / up weights on the persistent kernel:
-// out [M, N / 2] (row stride ldo) = min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta).
+// out [M, N / 2] (row stride ldo) = min(g, limit) sigmoid(alpha g (1 + cubic g^2)) (clamp(u, +-limit) + beta).
 CFC_API int cfc_pgemm_glu(const void* x, const void* w, void* out, int M, int N, int K, int ldo, int wnw, float limit,
-                          float alpha, float beta, hipStream_t stream) {
+                          float alpha, float beta, float cubic, hipStream_t stream) {
   if (M < 1 || N < 64 || K < 2 * PG_BK || K % 64 || N % 64 || ldo % 8 || ldo < N / 2 || ((uintptr_t)out & 15) || wnw < 1 ||
       N % (16 * wnw) || (uint64_t)M * K * 2 >= (1ull << 32) || (uint64_t)N * K * 2 >= (1ull << 32))
     return (int)hipErrorInvalidValue;
   const int tm = (M + PG_BM - 1) / PG_BM, tn = (N + PG_BN - 1) / PG_BN;
   PgGlu gp;
-  gp.limit = limit; gp.alpha = alpha; gp.beta = beta;
+  gp.limit = limit; gp.alpha = alpha; gp.beta = beta; gp.cubic = cubic;
   pgemm_ppp_kernel<PG_GLU, true><<<min(tm * tn, pg_cus()), 512, 0, stream>>>(
       (const uint16_t*)x, (const uint16_t*)w, (uint16_t*)out, M, N, K, ldo, tm, tn, wnw, ppp_group_m(tn, K), gp);
   return (int)hipGetLastError();

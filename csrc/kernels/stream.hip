@@ -1,6 +1,6 @@
 // Residual-stream kernels for decoders that keep a 32-bit stream and look back in depth and in time:
 //
-//   * embed_f32          token rows of a bf16 / fp32 table as the fp32 stream
+//   * embed_f32          token rows of a bf16 / fp32 table as the fp32 stream, scaled, with the positions' sinusoids if asked
 //   * depth_norm         X_new = x + sublayer outputs (fp32 split-K slabs, bias), x' = sum_j a_j X_j over
 //                        the results of every earlier layer, and the RMS norm that follows, one row per
 //                        workgroup.  Three endings: the norm's 1 / rms only (a prompt's rows, before
@@ -9,7 +9,7 @@
 //   * depth_pre          the older results' share of the next few layers' averages, in one pass over them
 //   * input_conv         h + conv(h) over time on each channel, for both sublayers at once, over a packed
 //                        batch of prompt portions
-//   * clamped_glu        min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + beta), optional biases
+//   * clamped_glu        min(g, limit) sigmoid(alpha g (1 + cubic g^2)) (clamp(u, +-limit) + beta), optional biases
 //   * softcap            cap * tanh(x / cap), in place on fp32
 //
 // The tail of a sequence's convolution inputs lives in the paged cache, beside the KV block that holds
@@ -17,6 +17,8 @@
 // a sequence that continues (or shares) it needs, and freeing the block frees the tail.  slots is
 // taps + 1 (at most one block's 32 positions): taps - 1 inputs are live, and two spare rows keep a
 // position that is run again (a decode graph's warm-up) from overwriting what it reads.
+// Or it lives in a slot per sequence (max_blocks 0: block_tables holds each sequence's slot): then the tile that a portion
+// starts with also stores the portion's last inputs, after it has read the old ones.
 //
 // ACT is the activation type the matrix products read: uint16_t (bf16 bits) or float.
 #include "rows.h"
@@ -30,21 +32,32 @@ __device__ __forceinline__ void st1(float* p, float v) { *p = v; }
 
 template <typename TAB>
 __global__ void __launch_bounds__(256) embed_f32_kernel(float* __restrict__ out, const TAB* __restrict__ table,
-                                                       const int32_t* __restrict__ ids, int W, int vocab) {
+                                                       const int32_t* __restrict__ ids, int W, int vocab, float scale,
+                                                       const int32_t* __restrict__ positions, const double* __restrict__ turns) {
   const int t = blockIdx.x;
   const int id = min(max(ids[t], 0), vocab - 1);
-  for (int c = threadIdx.x; c < W; c += 256) out[(size_t)t * W + c] = ld1(table + (size_t)id * W + c);
+  const double pos = positions ? positions[t] : 0;
+  for (int c = threadIdx.x; c < W; c += 256) {
+    float v = scale * ld1(table + (size_t)id * W + c);
+    if (positions) {
+      // turns per position in 64 bits: the angle's fraction of a turn keeps its digits however far the position
+      const double n = pos * turns[c >> 1];
+      const float f = (float)(n - floor(n));
+      v += c & 1 ? cospif(2.f * f) : sinpif(2.f * f);
+    }
+    out[(size_t)t * W + c] = v;
+  }
 }
 
 // What a convolution input of an earlier step is read from.
 struct TailArg {
   float* tail;                    // [blocks][slots][W]
-  const int32_t* block_tables;    // [sequences][max_blocks]
+  const int32_t* block_tables;    // [sequences][max_blocks], or [sequences] slots
   int max_blocks, slots;
 };
 
 __device__ __forceinline__ float* tail_row(const TailArg& a, int seq, int pos, int W) {
-  const int blk = a.block_tables[(size_t)seq * a.max_blocks + pos / CFC_KV_BS];
+  const int blk = a.block_tables[a.max_blocks ? (size_t)seq * a.max_blocks + pos / CFC_KV_BS : (size_t)seq];
   return a.tail + ((size_t)blk * a.slots + pos % a.slots) * W;
 }
 
@@ -262,6 +275,7 @@ __global__ void __launch_bounds__(256) input_conv_kernel(const float* __restrict
   const Vec<V> g = ldv<V>(norm_w + c);
   // rows of this portion that precede the tile: tile_lead rows are in x, the rest in the tail
   const int lead = tiles[4 * (gridDim.x + blockIdx.x)];
+  const bool paged = ta.max_blocks != 0;
   auto input = [&](int r) -> Vec<V> {        // convolution input of row row0 + r (r may be negative)
     Vec<V> h;
     if (pos0 + r < 0) {
@@ -280,7 +294,7 @@ __global__ void __launch_bounds__(256) input_conv_kernel(const float* __restrict
   auto put = [&](int r, const Vec<V>& h, const Vec<V>& y1, const Vec<V>& y2) {
     stv<V>(h1 + (size_t)(row0 + r) * ld_1 + c, y1);
     if (w2) stv<V>(h2 + (size_t)(row0 + r) * ld_2 + c, y2);
-    if (r >= n - (taps - 1)) stv<V>(tail_row(ta, seq, pos0 + r, W) + c, h);
+    if (paged && r >= n - (taps - 1)) stv<V>(tail_row(ta, seq, pos0 + r, W) + c, h);
   };
   if constexpr (TAPS > 0) {
     float k1[TAPS][V], k2[TAPS][V];
@@ -323,19 +337,23 @@ __global__ void __launch_bounds__(256) input_conv_kernel(const float* __restrict
       put(r, h, y1, y2);
     }
   }
+  if (!paged && lead == 0) {
+    const int N = tiles[4 * (gridDim.x + blockIdx.x) + 1];
+    for (int r = max(0, N - (taps - 1)); r < N; ++r) stv<V>(tail_row(ta, seq, pos0 + r, W) + c, input(r));
+  }
 }
 
 template <typename ACT>
-__device__ __forceinline__ float glu(float g, float u, float limit, float alpha, float beta) {
+__device__ __forceinline__ float glu(float g, float u, float limit, float alpha, float beta, float cubic) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + __expf(-alpha * g)) * (u + beta);
+  return g / (1.f + __expf(-alpha * g * (1.f + cubic * g * g))) * (u + beta);
 }
 template <>
-__device__ __forceinline__ float glu<float>(float g, float u, float limit, float alpha, float beta) {
+__device__ __forceinline__ float glu<float>(float g, float u, float limit, float alpha, float beta, float cubic) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + beta);
+  return g / (1.f + expf(-alpha * g * (1.f + cubic * g * g))) * (u + beta);
 }
 
 // gu [split][T][2F] (ACT, or fp32 slabs whose sum is the product): gate | up halves, or 8-column
@@ -343,7 +361,7 @@ __device__ __forceinline__ float glu<float>(float g, float u, float limit, float
 template <typename ACT, typename IN>
 __global__ void __launch_bounds__(256) clamped_glu_kernel(ACT* __restrict__ out, int ldo, const IN* __restrict__ gu,
                                                          const float* __restrict__ gb, const float* __restrict__ ub,
-                                                         int F, int interleaved, float limit, float alpha, float beta, int split,
+                                                         int F, int interleaved, float limit, float alpha, float beta, float cubic, int split,
                                                          size_t slab) {
   const int t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
   if (c >= F) return;
@@ -354,7 +372,7 @@ __global__ void __launch_bounds__(256) clamped_glu_kernel(ACT* __restrict__ out,
     g += ld1(r + p * slab + gc);
     u += ld1(r + p * slab + uc);
   }
-  st1(out + (size_t)t * ldo + c, glu<ACT>(g, u, limit, alpha, beta));
+  st1(out + (size_t)t * ldo + c, glu<ACT>(g, u, limit, alpha, beta, cubic));
 }
 
 // relu(sum of slabs)^2 of n values (a multiple of V)
@@ -429,12 +447,13 @@ int conv_launch(dim3 grid, hipStream_t s, const float* x, const float* rstd, con
 }  // namespace
 
 // table: bf16 (f32 = 0) or fp32 rows; ids outside [0, vocab) are clamped
-CFC_API int cfc_embed_f32(float* out, const void* table, const int32_t* ids, int T, int W, int vocab, int f32,
-                          hipStream_t stream) {
+// positions (null: none): entries 2i and 2i + 1 get the sine and the cosine of positions * turns[i] turns
+CFC_API int cfc_embed_f32(float* out, const void* table, const int32_t* ids, int T, int W, int vocab, int f32, float scale,
+                          const int32_t* positions, const double* turns, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (W <= 0 || vocab <= 0) return -1;
-  if (f32) embed_f32_kernel<float><<<T, 256, 0, stream>>>(out, (const float*)table, ids, W, vocab);
-  else embed_f32_kernel<uint16_t><<<T, 256, 0, stream>>>(out, (const uint16_t*)table, ids, W, vocab);
+  if (W <= 0 || vocab <= 0 || (positions && !turns)) return -1;
+  if (f32) embed_f32_kernel<float><<<T, 256, 0, stream>>>(out, (const float*)table, ids, W, vocab, scale, positions, turns);
+  else embed_f32_kernel<uint16_t><<<T, 256, 0, stream>>>(out, (const uint16_t*)table, ids, W, vocab, scale, positions, turns);
   return CFC_CHECK_LAUNCH();
 }
 
@@ -474,7 +493,8 @@ CFC_API int cfc_depth_pre(const float* hist, int64_t plane, int n, int count, co
   return CFC_CHECK_LAUNCH();
 }
 
-// tiles [2][n_tiles][4]: {first row, rows, first position, sequence}, then {portion rows before the tile, 0, 0, 0}
+// tiles [2][n_tiles][4]: {first row, rows, first position, sequence}, then {portion rows before the tile, the portion's rows,
+// 0, 0}.  max_blocks 0: block_tables holds each sequence's slot, tail [slots][tail slots][W]
 CFC_API int cfc_input_conv(int f32, int n_tiles, const int32_t* tiles, const float* x, const float* rstd,
                            const float* norm_w, const float* w1, const float* w2, int taps, float* tail, int slots,
                            const int32_t* block_tables, int max_blocks, int W, void* h1, int ld1, void* h2, int ld2,
@@ -494,7 +514,8 @@ CFC_API int cfc_input_conv(int f32, int n_tiles, const int32_t* tiles, const flo
 
 // in_f32: gu is fp32 (else the activation type)
 CFC_API int cfc_clamped_glu(int f32, int in_f32, void* out, int ldo, const void* gu, int split, const float* gb,
-                            const float* ub, int T, int F, int interleaved, float limit, float alpha, float beta, hipStream_t stream) {
+                            const float* ub, int T, int F, int interleaved, float limit, float alpha, float beta, float cubic,
+                            hipStream_t stream) {
   if (T <= 0) return 0;
   if (F <= 0 || (interleaved && F % 8) || split < 1 || (split > 1 && !f32 && !in_f32) || T > 65535 * 16) return -1;
   const int rows = T > 65535 ? 65535 : T;
@@ -504,13 +525,13 @@ CFC_API int cfc_clamped_glu(int f32, int in_f32, void* out, int ldo, const void*
     const size_t slab = (size_t)T * 2 * F, go = (size_t)t0 * 2 * F, oo = (size_t)t0 * ldo;
     if (f32)
       clamped_glu_kernel<float, float><<<grid, 256, 0, stream>>>((float*)out + oo, ldo, (const float*)gu + go, gb, ub, F,
-                                                                 interleaved, limit, alpha, beta, split, slab);
+                                                                 interleaved, limit, alpha, beta, cubic, split, slab);
     else if (in_f32)
       clamped_glu_kernel<uint16_t, float><<<grid, 256, 0, stream>>>((uint16_t*)out + oo, ldo, (const float*)gu + go, gb, ub,
-                                                                    F, interleaved, limit, alpha, beta, split, slab);
+                                                                    F, interleaved, limit, alpha, beta, cubic, split, slab);
     else
       clamped_glu_kernel<uint16_t, uint16_t><<<grid, 256, 0, stream>>>((uint16_t*)out + oo, ldo, (const uint16_t*)gu + go,
-                                                                       gb, ub, F, interleaved, limit, alpha, beta, split, slab);
+                                                                       gb, ub, F, interleaved, limit, alpha, beta, cubic, split, slab);
   }
   return CFC_CHECK_LAUNCH();
 }
