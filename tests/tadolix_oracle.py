@@ -6,6 +6,7 @@ the dtype of their inputs (float32 or float64).
 """
 from __future__ import annotations
 
+import functools
 import math
 from fractions import Fraction
 
@@ -55,6 +56,7 @@ def write_streams(xs, y, mix, out):
     return [sum(mix[s, t] * xs[s] for s in range(len(xs))) + out[t] * y for t in range(len(xs))]
 
 
+@functools.cache
 def bucket(n, rows, far):
     """The table's row for a distance of n tokens: its own below half the rows, from there on logarithmically up to the
     last at ``far`` (compared exactly, in integers: the k-th step starts at half (far / half)^(k / steps))."""
