@@ -419,7 +419,7 @@ class TadolixModel:
                     plan[self._tiles(a)] = A.prompt_tiles(cu, ctx, a.H, a.G, A.prompt_rows(self.w.dtype, a.D))
                 if "chunks" not in plan:
                     plan["chunks"], plan["chunk_cu"] = R.chunk_plan(cu)
-            elif "segments" not in plan:
+            elif "segments" not in plan and not L.whole_portions(cu, lw["lru"].width):
                 plan["segments"], plan["segment_cu"] = R.chunk_plan(cu, L.SEGMENT)
         return plan
 
@@ -497,7 +497,8 @@ class TadolixModel:
         tail, state, p = io.kv.tail[run], io.kv.recur[run], io.plan
         if p is None:
             return L.step(r, x, y, io.states, io.positions, io.ctx_lens, tail, state, out)
-        return L.prefill(r, x, y, io.states, io.cu_q, io.ctx_lens, p["conv_tiles"], p["segments"], p["segment_cu"], tail, state, out)
+        # a pass that has segments for one layer's width runs all layers on them
+        return L.prefill(r, x, y, io.states, io.cu_q, io.ctx_lens, p["conv_tiles"], p.get("segments"), p.get("segment_cu"), tail, state, out)
 
     def _feed(self, i, h) -> torch.Tensor:
         """fp32 slabs of layer i's feed-forward."""

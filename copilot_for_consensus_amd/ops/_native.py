@@ -82,7 +82,7 @@ _KERNEL_SIGS = {
     "cfc_rglru_segment": [],
     "cfc_rglru_max_block": [],
     "cfc_rglru_step": [I] + [P, I, c_int64, c_int64] * 2 + [P, P, P, I] + [P] * 5 + [I] * 4 + [P] * 5 + [I, P, P],
-    "cfc_rglru_prefill": [I] + [P, c_int64] * 2 + [P, P, P, I] + [P] * 5 + [I] * 4 + [P] * 4 + [I, P, I, P, P, P, I, I, P, P, P, P],
+    "cfc_rglru_prefill": [I] + [P, c_int64] * 2 + [P, P, P, I] + [P] * 5 + [I] * 4 + [P] * 4 + [I, I, P, I, P, P, P, I, I, P, P, P, P],
     "cfc_qkv_rows": [I, P, I, c_int64, c_int64, I, I, I, I, I, I, I, P, P, I, F, P, I, F, P, I] + [P] * 10 + [I, I, P, I, P],
     "cfc_conv_tail": [I, P, I, c_int64, c_int64, I, P, P, P, I, I, P, P],
     "cfc_pool_rows": [I, P, I, P, I, P, P, P, P, I, I, I, I, P],

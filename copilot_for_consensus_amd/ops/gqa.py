@@ -26,7 +26,7 @@ MAX_DIM = 1024
 ANY_ROWS = 4              # rows per tile of the general kernel
 MAX_PARTITIONS = 256
 LOG2E = 1.4426950408889634
-CAP_NEAR = 0.35           # scores up to this share of their cap take the cap's short form
+CAP_NEAR = (0.25, 0.35)   # scores up to these shares of their cap take shorter forms of the cap
 
 
 @dataclasses.dataclass(frozen=True)
@@ -121,7 +121,8 @@ class Heads:
         self.D = padded_dim(self.dim, self.vdim)
         # queries carry the scale into the softmax's base 2, or into the cap's e^(2 score / cap)
         self.q_scale = self.scale * LOG2E * (2.0 / self.softcap if self.softcap else 1.0)
-        self.capped = 0 if not self.softcap else 2 if self.unit and self.dim * abs(self.scale) <= 0.98 * CAP_NEAR * self.softcap else 1
+        share = 1.02 * self.dim * abs(self.scale) / self.softcap if self.unit and self.softcap else 1.0
+        self.capped = 0 if not self.softcap else 3 if share <= CAP_NEAR[0] else 2 if share <= CAP_NEAR[1] else 1
         self.bias2 = None if self.bias is None else (self.bias * LOG2E).contiguous()
         if self.bias is not None and (self.bias.shape[0] != self.H or self.mask.pool):
             raise ValueError(f"bias {tuple(self.bias.shape)} for {self.H} heads over {self.mask}")

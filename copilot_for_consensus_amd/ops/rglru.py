@@ -13,11 +13,12 @@ import torch.nn.functional as F
 from . import reference as ref
 from ._native import check, kernels
 from .cols import Cols
-from .kernels import _req, _stream
+from .kernels import _p, _req, _stream
 from .stream import _act
 
 SEGMENT = 128            # tokens per segment of the prompt kernels
 MAX_BLOCK = 512          # block columns (padded) they take; wider ones and fp32: the general kernels
+FILL = 1024              # workgroups that fill the chip (four waves each)
 
 
 @dataclasses.dataclass
@@ -88,6 +89,13 @@ def _ref(p: RgLru, x, y, slots, positions, cu, tail, state, out):
     return out
 
 
+def whole_portions(cu, width: int) -> bool:
+    """Whether the portions of a pass are one segment each: those alone fill the chip and are about even, or none is longer
+    than a segment."""
+    n = [b - a for a, b in zip(cu, cu[1:])]
+    return max(n) <= SEGMENT or (len(n) * math.ceil(width / 64) >= FILL and max(n) * len(n) <= 2 * sum(n))
+
+
 def _fits(p: RgLru, x: Cols, y: Cols, tail, state, out):
     if x.n != p.width or y.n != p.width or out.shape != (x.rows, p.width) or not out.is_contiguous() or state.shape[-1] != p.width \
             or tail.shape[1:] != (p.ring, p.width) or p.f32 != (out.dtype == torch.float32):
@@ -113,20 +121,22 @@ def step(p: RgLru, x: Cols, y: Cols, slots, positions, ctx_lens, tail, state, ou
 
 def prefill(p: RgLru, x: Cols, y: Cols, slots, cu_q, ctx_lens, tiles, chunks, chunk_cu, tail, state, out) -> torch.Tensor:
     """Packed portions, ``x`` and ``y`` activations; ``tiles`` of ops.stream.conv_tiles (by rows), ``chunks`` and ``chunk_cu``
-    of ops.gru.chunk_plan with SEGMENT, on the device."""
+    of ops.gru.chunk_plan with SEGMENT, on the device; both None: every portion is one segment (:func:`whole_portions`)."""
     if not out.is_cuda:
         first = ctx_lens - (cu_q[1:] - cu_q[:-1])
         return _ref(p, x, y, slots, first, cu_q, tail, state, out)
-    for name, t in (("slots", slots), ("cu_q", cu_q), ("ctx_lens", ctx_lens), ("tiles", tiles), ("chunks", chunks), ("chunk_cu", chunk_cu)):
+    whole = chunks is None
+    for name, t in (("slots", slots), ("cu_q", cu_q), ("ctx_lens", ctx_lens), ("tiles", tiles)) + \
+            (() if whole else (("chunks", chunks), ("chunk_cu", chunk_cu))):
         _req(t, torch.int32, name)
     xa, ya = _fits(p, x, y, tail, state, out)
     if xa[1] or ya[1]:
         raise ValueError("rglru prefill: x and y are activations")
-    T, n = out.shape[0], chunks.shape[0]
+    T, n, mfma = out.shape[0], 0 if whole else chunks.shape[0], not p.f32 and p.KP <= MAX_BLOCK
     u = torch.empty(T, p.blocks * p.KP, dtype=out.dtype, device=out.device)
-    sums = torch.empty((n if not p.f32 and p.KP <= MAX_BLOCK else T) * 2 * p.width, dtype=torch.float32, device=out.device)
+    sums = None if mfma and whole else torch.empty((n if mfma else T) * 2 * p.width, dtype=torch.float32, device=out.device)
     check(kernels().cfc_rglru_prefill(_act(out.dtype), xa[0], xa[2], ya[0], ya[2], *p.weights(), tail.data_ptr(), state.data_ptr(),
-                                      slots.data_ptr(), tiles.data_ptr(), tiles.shape[1], chunks.data_ptr(), n, chunk_cu.data_ptr(),
-                                      cu_q.data_ptr(), ctx_lens.data_ptr(), slots.numel(), T, u.data_ptr(), sums.data_ptr(),
+                                      slots.data_ptr(), tiles.data_ptr(), tiles.shape[1], int(whole), _p(chunks), n, _p(chunk_cu),
+                                      cu_q.data_ptr(), ctx_lens.data_ptr(), slots.numel(), T, u.data_ptr(), _p(sums),
                                       out.data_ptr(), _stream(out)), "cfc_rglru_prefill")
     return out

@@ -38,7 +38,8 @@ struct GqaArgs {
   int H, G, D, DV, max_blocks, P;      // DV: value columns that leave
   int size, keep, pool, le;            // window; first tokens; tokens per pooled block, log2 of entries per page
   int chunk;                           // size counts from multiples of it
-  int capped; float cap2;              // 0: no cap, 1: any score, 2: |score| <= CAP_NEAR cap; cap log2(e)
+  int capped; float cap2;              // 0: no cap, 1: any score, 2, 3: |score| <= 0.35, 0.25 cap; cap log2(e)
+  float k0, k1, k2, k3;                // capped 2 and 3: s (k0 + t (k1 + t (k2 + t k3))), t = s^2
   const float* bias; int nb;           // [H][nb] by distance, times log2(e) (null: none)
   OutGate og;
   const float* sink;          // [H] or null
@@ -53,19 +54,17 @@ __device__ __forceinline__ int pooled_seen(const GqaArgs& a, int pos) { return m
 __device__ __forceinline__ int window_first(const GqaArgs& a, int pos) { return a.chunk ? pos - pos % a.size : max(0, pos - a.size + 1); }
 
 constexpr float LN2 = 0.69314718055994531f;
-constexpr float CAP_NEAR = 0.35f;
 
-// the capped score (base 2) of a score s = 2 log2(e) score / cap.  Near zero by the series of tanh in x = s ln(2) / 2 (its
-// next term, 62 / 2835 x^9, is below 3e-6 of x)
+// the capped score (base 2) of a score s = 2 log2(e) score / cap, plus b.  Near zero by the series of tanh in x = s ln(2) / 2
+// (its next term, 62 / 2835 x^9, is below 4e-6 of x; without the one before it, nearer zero, 17 / 315 x^7 below 1.4e-5)
 template <typename ACT>
-__device__ __forceinline__ float cap_score(const GqaArgs& a, float s) {
-  if constexpr (sizeof(ACT) == 4) return a.cap2 * tanhf(s * (0.5f * LN2));
-  if (a.capped == 2) {
-    constexpr float h = 0.5f * LN2, h2 = h * h;
+__device__ __forceinline__ float cap_score(const GqaArgs& a, float s, float b) {
+  if constexpr (sizeof(ACT) == 4) return a.cap2 * tanhf(s * (0.5f * LN2)) + b;
+  if (a.capped >= 2) {
     const float t = s * s;
-    return s * (a.cap2 * h) * (1.f + t * (-h2 / 3.f + t * (2.f * h2 * h2 / 15.f - t * (17.f * h2 * h2 * h2 / 315.f))));
+    return s * (a.k0 + t * (a.k1 + t * (a.k2 + t * a.k3))) + b;
   }
-  return a.cap2 - 2.f * a.cap2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s));
+  return a.cap2 + b - 2.f * a.cap2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s));
 }
 
 // Tiles of KT keys for rows at positions pmin .. pmax: first `nat` of the far range (`na` keys), then the window's,
@@ -232,7 +231,7 @@ __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) gqa_decode_kernel(const
 #pragma unroll
         for (int g = 0; g < 2; ++g)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) sc[g][i] = (a.capped ? cap_score<uint16_t>(a, sc[g][i]) : sc[g][i]) + bt8[g][i];
+          for (int i = 0; i < 4; ++i) sc[g][i] = a.capped ? cap_score<uint16_t>(a, sc[g][i], bt8[g][i]) : sc[g][i] + bt8[g][i];
       }
       float mx = -INFINITY;
 #pragma unroll
@@ -461,32 +460,39 @@ __global__ void __launch_bounds__(64 * NW, D <= 128 ? 2 : 1) gqa_prompt_kernel(c
         }
       }
       if constexpr (SHAPED) {
-        if (a.capped)
+        const float far0 = far_bias - ref0;
 #pragma unroll
-          for (int h = 0; h < 2; ++h)
+        for (int h = 0; h < 2; ++h) {
+          float bv[16];                        // the biases, less the running maximum
 #pragma unroll
-            for (int r = 0; r < 16; ++r) sc[h][r] = cap_score<uint16_t>(a, sc[h][r]);
-        if (a.bias && wp0 - (k0 + 63) < a.nb - 1) {
-#pragma unroll
-          for (int h = 0; h < 2; ++h)
+          for (int r = 0; r < 16; ++r) bv[r] = far0;
+          if (a.bias && wp0 - (k0 + 32 * h + 31) < a.nb - 1) {
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
               const int n = my_pos - (k0 + 32 * h + 8 * g + 4 * hi);          // the first key's distance
               if (lb) {
                 const float* b = lb + min(max(a.nb - 1 - n, -BIAS_PAD), a.nb - 1);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) sc[h][4 * g + i] += b[i] - ref0;
+                for (int i = 0; i < 4; ++i) bv[4 * g + i] = b[i] - ref0;
               } else {
 #pragma unroll
-                for (int i = 0; i < 4; ++i)
-                  sc[h][4 * g + i] += a.bias[(size_t)head * a.nb + min(max(n - i, 0), a.nb - 1)] - ref0;
+                for (int i = 0; i < 4; ++i) bv[4 * g + i] = a.bias[(size_t)head * a.nb + min(max(n - i, 0), a.nb - 1)] - ref0;
               }
             }
-        } else {
+          }
+          if (a.capped == 3) {
 #pragma unroll
-          for (int h = 0; h < 2; ++h)
+            for (int r = 0; r < 16; ++r) {
+              const float t = sc[h][r] * sc[h][r];
+              sc[h][r] = sc[h][r] * (a.k0 + t * (a.k1 + t * a.k2)) + bv[r];
+            }
+          } else if (a.capped) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) sc[h][r] += far_bias - ref0;
+            for (int r = 0; r < 16; ++r) sc[h][r] = cap_score<uint16_t>(a, sc[h][r], bv[r]);
+          } else {
+#pragma unroll
+            for (int r = 0; r < 16; ++r) sc[h][r] += bv[r];
+          }
         }
       }
       if (!all) {
@@ -620,7 +626,7 @@ __global__ void __launch_bounds__(256) gqa_any_kernel(const ACT* __restrict__ q,
 #pragma unroll
         for (int u = 0; u < 4; ++u) s4[u] += myq[r + u] * ldf(c + r + u);
       sc = (s4[0] + s4[1]) + (s4[2] + s4[3]);
-      if (a.capped) sc = cap_score<float>(a, sc);
+      if (a.capped) sc = cap_score<float>(a, sc, 0.f);
       if (a.bias) sc += a.bias[(size_t)head * a.nb + min(pos - e, a.nb - 1)];
     }
     const float mn = fmaxf(m, wave_max(sc)), ref = mn == -INFINITY ? 0.f : mn;
@@ -687,7 +693,7 @@ CFC_API int cfc_gqa_prompt_rows(int D) {
 
 // q [T][H][D] scaled by log2(e); caches [blocks][G][32][D], pooled [blocks][G][1 << le][D]; out [T][H][DV].
 // kind 0: general (tiles of 4 rows over all heads; tile_seq null: one token per sequence), 1: decode, 2: prompt portions.
-// chunk: the window is the row's own run of size positions.  capped 1 or 2 (|score| <= 0.35 cap): q scaled by 2 log2(e) / cap
+// chunk: the window is the row's own run of size positions.  capped 1, 2 or 3 (|score| <= 0.35, 0.25 cap): q scaled by 2 log2(e) / cap
 // instead, cap2 = cap log2(e).  bias [H][nb] times log2(e), by distance.  gate: columns [T][H DV] of a product (gate_split 0:
 // activations, else fp32 slabs; null: none) that, as oscale sigmoid(gate), multiply the output, whose rows have stride ldo
 CFC_API int cfc_gqa_attention(int kind, int f32, const void* q, const void* kc, const void* vc, const void* pk, const void* pv,
@@ -700,7 +706,7 @@ CFC_API int cfc_gqa_attention(int kind, int f32, const void* q, const void* kc, 
   if (H < 1 || G < 1 || H % G || D < 32 || D % 32 || D > 1024 || DV < 1 || DV > D || max_blocks < 1 || P < 1 || P > MERGE_MAXP) return -1;
   if (size < 0 || keep < 0 || pool < 0 || (pool && (keep || !pk || !pv || le < 0 || le > 5 || (pool << le) < CFC_KV_BS || size < 1))) return -2;
   if (chunk && (size < 1 || pool)) return -2;
-  if (capped < 0 || capped > 2 || (capped && !(cap2 > 0.f)) || (bias && nb < 1) || (bias && pool)) return -7;
+  if (capped < 0 || capped > 3 || (capped && !(cap2 > 0.f)) || (bias && nb < 1) || (bias && pool)) return -7;
   if (ldo < (int64_t)H * DV || (gate && (gate_split < 0 || gate_ld < (int64_t)H * DV))) return -8;
   if (P > 1 && (!part_o || !part_ml)) return -3;
   if (kind == 2 && (P != 1 || !cu_q || !tile_seq || !tile_m0)) return -4;
@@ -710,8 +716,10 @@ CFC_API int cfc_gqa_attention(int kind, int f32, const void* q, const void* kc, 
   const int esz = f32 ? 4 : 2, gsz = gate_split ? 4 : esz;
   og.vec = DV % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)out & (4 * esz - 1)) == 0 &&
            (!gate || (gate_ld % 4 == 0 && gate_plane % 4 == 0 && ((uintptr_t)gate & (4 * gsz - 1)) == 0));
+  const float h = 0.5f * LN2, h2 = h * h, h3 = h2 * h;
   const GqaArgs a{block_tables, cu_q, ctx_lens, tile_seq, tile_m0, n_tiles, H, G, D, DV, max_blocks, P, size, keep, pool, le,
-                  chunk, capped, cap2, bias, nb, og, sink, part_o, part_ml};
+                  chunk, capped, cap2, h * cap2, -h3 / 3.f * cap2, 2.f * h3 * h2 / 15.f * cap2, -17.f * h3 * h2 * h2 / 315.f * cap2,
+                  bias, nb, og, sink, part_o, part_ml};
   const bool shaped = capped || bias;
   int rc = -6;
   if (kind == 2) {

@@ -59,20 +59,25 @@ __global__ void __launch_bounds__(BT) hyper_norm_kernel(HyperArgs a, int mode, A
 #pragma unroll
       for (int d = 1; d <= PRE; ++d) past[d - 1] = d <= back && d <= pos ? ldv<V>(tail + (size_t)((pos - d) % a.ring) * W + c) : zerov<V>();
     }
-  __syncthreads();
-  Vec<V> u[NV];
+  Vec<V> u[NV], x[SM], y = zerov<V>();
   float ss = 0.f;
+  auto load = [&](int c) {
+#pragma unroll
+    for (int s = 0; s < SM; ++s) x[s] = ldv<V>(xr + min(s, S - 1) * a.lds + c);
+    if (a.y) {
+      y = zerov<V>();
+      add_slabs<V>(y, a.y, a.split, (int64_t)a.T * W, (size_t)t * W + c);
+    }
+  };
+  load(min((int)threadIdx.x * V, W - V));
+  __syncthreads();
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
     const int c = (k * BT + threadIdx.x) * V;
     u[k] = zerov<V>();
     if (c >= W) continue;
-    Vec<V> x[SM];
-#pragma unroll
-    for (int s = 0; s < SM; ++s) x[s] = ldv<V>(xr + min(s, S - 1) * a.lds + c);
+    if (k) load(c);
     if (a.y) {
-      Vec<V> y = zerov<V>();
-      add_slabs<V>(y, a.y, a.split, (int64_t)a.T * W, (size_t)t * W + c);
 #pragma unroll
       for (int q = 0; q < SM; ++q) {
         if (q >= S) break;

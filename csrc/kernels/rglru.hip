@@ -8,8 +8,9 @@
 //   * short_conv   prompt rows: u as rows [T][blocks][KP], a block's columns padded with zeros to whole operands
 //   * rglru_scan   segments of prompt portions on the matrix cores: a wave keeps the gate matrices of its 16 channels in
 //                  registers and takes 16 tokens at a time; a lane holds four neighbouring tokens of one channel, the four
-//                  lane groups are composed with shuffles.  Once for what each segment does to the state, then (behind
-//                  carry, recur.h) again from the states, for the outputs: cheaper than keeping 32-bit gates
+//                  lane groups are composed with lane swaps.  Once for what each segment does to the state, then (behind
+//                  carry, recur.h) again from the states, for the outputs: cheaper than keeping 32-bit gates.  Where the
+//                  portions alone fill the chip each is one segment, and the second pass does it all
 //   * rglru_step   one token per sequence, straight from a joint product's slabs: convolution, gates, state, output
 //   * rglru_any    any block size and the 32-bit path, prompt rows and decoded ones: gates a workgroup per (row, block),
 //                  then a thread per channel
@@ -39,7 +40,16 @@ __device__ __forceinline__ Vec<V> lru_ld(const LruCols& a, int64_t t, int c) {
   const int64_t o = t * a.ld + c;
   if (a.split == 0) return ldv<V>(reinterpret_cast<const ACT*>(a.p) + o);
   Vec<V> y = zerov<V>();
-  add_slabs<V>(y, reinterpret_cast<const float*>(a.p), a.split, a.plane, (size_t)o);
+  const float* p = reinterpret_cast<const float*>(a.p) + o;
+  for (int p0 = 0; p0 < a.split; p0 += 4) {            // four slabs in flight (past the last: re-read, not added)
+    Vec<V> v[4];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) v[s] = ldv<V>(p + min(p0 + s, a.split - 1) * a.plane);
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+#pragma unroll
+      for (int e = 0; e < V; ++e) y.v[e] += p0 + s < a.split ? v[s].v[e] : 0.f;
+  }
   return y;
 }
 
@@ -47,26 +57,27 @@ __device__ __forceinline__ f32x4_t mfma16(u32x4_t a, u32x4_t b, f32x4_t c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
-// -expm1(z) for z <= 0: 1 - e^z keeps its digits near zero
-template <typename ACT> __device__ __forceinline__ float one_minus_exp(float z);
-template <> __device__ __forceinline__ float one_minus_exp<float>(float z) { return -expm1f(z); }
-template <> __device__ __forceinline__ float one_minus_exp<uint16_t>(float z) {
-  const float s = -z * (1.f + z * (0.5f + z * (1.f / 6.f + z * (1.f / 24.f))));       // next term z^4 / 120
-  return z > -0.125f ? s : 1.f - exp_of<uint16_t>(z);
+// 1 - a^2 for a = e^la, la <= 0: near 1 by the series of -expm1(2 la), whose next term is la^3 / 3 of it
+template <typename ACT> __device__ __forceinline__ float one_minus_sq(float la, float a);
+template <> __device__ __forceinline__ float one_minus_sq<float>(float la, float) { return -expm1f(2.f * la); }
+template <> __device__ __forceinline__ float one_minus_sq<uint16_t>(float la, float a) {
+  const float s = la * (-2.f + la * (-2.f - la * (4.f / 3.f)));
+  return la > -0.015f ? s : 1.f - a * a;
 }
 template <typename ACT> __device__ __forceinline__ float root(float x);
 template <> __device__ __forceinline__ float root<float>(float x) { return sqrtf(x); }
 template <> __device__ __forceinline__ float root<uint16_t>(float x) { return __builtin_amdgcn_sqrtf(x); }
 
+// far below zero e^-x is infinite and 1 / (1 + e^-x) zero
 template <typename ACT>
-__device__ __forceinline__ float sigm(float x) { return over1<ACT>(exp_of<ACT>(fminf(-x, 80.f))); }
+__device__ __forceinline__ float sigm(float x) { return over1<ACT>(exp_of<ACT>(-x)); }
 
 // decay a and contribution of one token from the gates' pre-activations
 template <typename ACT>
 __device__ __forceinline__ void lru_gates(float pr, float pi, float u, float rate, float& a, float& b) {
   const float la = rate * sigm<ACT>(pr);
   a = exp_of<ACT>(la);
-  b = root<ACT>(fmaxf(one_minus_exp<ACT>(2.f * la), 0.f)) * sigm<ACT>(pi) * u;
+  b = root<ACT>(one_minus_sq<ACT>(la, a)) * sigm<ACT>(pi) * u;
 }
 
 // z / 2 (1 + tanh(k (z + 0.044715 z^3))) = z sigmoid(2 k (..)), k = sqrt(2 / pi)
@@ -144,152 +155,196 @@ __global__ void __launch_bounds__(256) short_conv_kernel(LruArgs a, const int32_
 }
 
 // ------------------------------------------------------------------------------------------ gates and scan, prompt rows
-// the segment's steps of 16 tokens; a lane's four tokens are 4 kq .. of one channel.  grid (segments, blocks * NP / 64
-// rounded up); chunks [n][2] {first row, rows}; sums [n][2][W]: decay and contribution, or (APPLY) the state ahead
-template <int KS, bool APPLY>
-__global__ void __launch_bounds__(256, KS <= 8 ? 2 : 1) rglru_scan_kernel(LruArgs a, const uint16_t* __restrict__ u,
+// grid (segments, blocks * NP / 64 rounded up); chunks [n][2] {first row, rows}.  Tiles of 32 tokens of u in LDS, double
+// buffered, in two steps of 16; a lane's four tokens of a step are 4 kq .. of one channel.
+//   SCAN_SUMS   sums [n][2][W]: what each segment does to the state
+//   SCAN_APPLY  outputs, from the state ahead of each segment in sums
+//   SCAN_WHOLE  a segment is a portion (chunks null: cu_q): outputs, from the sequence's state, which is updated
+enum { SCAN_SUMS = 0, SCAN_APPLY = 1, SCAN_WHOLE = 2 };
+constexpr int SCAN_TILE = 32;
+
+template <int KS, int MODE>
+__global__ void __launch_bounds__(256, KS <= 4 ? 4 : KS <= 8 ? 3 : 2) rglru_scan_kernel(LruArgs a, const uint16_t* __restrict__ u,
                                                                          const int32_t* __restrict__ chunks,
+                                                                         const int32_t* __restrict__ cu_q,
+                                                                         const int32_t* __restrict__ ctx_lens,
                                                                          float* __restrict__ sums, uint16_t* __restrict__ out) {
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
-  const int groups = (a.NP + 63) / 64, blk = blockIdx.y / groups, n0 = (blockIdx.y - blk * groups) * 64 + 16 * w;
-  if (n0 >= a.NP) return;
-  const int row0 = chunks[2 * blockIdx.x], n = chunks[2 * blockIdx.x + 1], UW = a.blocks * a.KP, W = a.W;
-  const bool live = n0 + col < a.bs;
-  const int c = blk * a.bs + min(n0 + col, a.bs - 1);
+  constexpr int LDU = 32 * KS + 8, NL = SCAN_TILE * 4 * KS / 256 > 0 ? SCAN_TILE * 4 * KS / 256 : 1;      // 16-byte pieces per thread
+  __shared__ __attribute__((aligned(16))) uint16_t tile[2][SCAN_TILE][LDU];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, col = lane & 15, kq = lane >> 4;
+  const int groups = (a.NP + 63) / 64, blk = blockIdx.y / groups, n0 = min((blockIdx.y - blk * groups) * 64 + 16 * w, a.NP - 16);
+  const bool mine = (blockIdx.y - blk * groups) * 64 + 16 * w < a.NP;      // else a wave that only loads
+  const int row0 = MODE == SCAN_WHOLE ? cu_q[blockIdx.x] : chunks[2 * blockIdx.x];
+  const int n = MODE == SCAN_WHOLE ? cu_q[blockIdx.x + 1] - row0 : chunks[2 * blockIdx.x + 1];
+  const int UW = a.blocks * a.KP, W = a.W, kb = a.KP / 32;
+  const bool live = mine && n0 + col < a.bs;
+  const int ku = min(n0 + col, a.bs - 1), c = blk * a.bs + ku;
   u32x4_t wr[KS], wi[KS];
   {
     const uint16_t* p = reinterpret_cast<const uint16_t*>(a.wg) + ((size_t)blk * a.NP + n0 + col) * a.KP + 8 * kq;
     const size_t second = (size_t)a.blocks * a.NP * a.KP;
 #pragma unroll
-    for (int k = 0; k < KS; ++k) {                     // steps past the block's: the last again, against zeros
-      const int o = 32 * min(k, a.KP / 32 - 1);
+    for (int k = 0; k < KS; ++k) {
+      const int o = 32 * min(k, kb - 1);
       wr[k] = *reinterpret_cast<const u32x4_t*>(p + o);
       wi[k] = *reinterpret_cast<const u32x4_t*>(p + second + o);
+      if (k >= kb) wr[k] = wi[k] = u32x4_t{0, 0, 0, 0};        // steps past the block's: its last columns against zeros
     }
   }
-  const float br = a.br[c], bi = a.bi[c], rate = a.rate[c], by = APPLY ? a.by[c] : 0.f;
+  const float br = a.br[c], bi = a.bi[c], rate = a.rate[c], by = MODE ? a.by[c] : 0.f;
   const uint16_t* ub = u + (size_t)row0 * UW + (size_t)blk * a.KP;
-  const uint16_t* yb = reinterpret_cast<const uint16_t*>(a.y.p) + (APPLY ? (int64_t)row0 * a.y.ld + c : 0);
-  const int ku = min(n0 + col, a.bs - 1);
-  float* sp = sums + (size_t)blockIdx.x * 2 * W + c;
-  float S = APPLY ? sp[0] : 0.f, A = 1.f;
-  u32x4_t uf[KS], un[KS];
-  uint16_t uo[4], uon[4], yo[4], yon[4];
-  auto load = [&](int t, u32x4_t* f, uint16_t* o, uint16_t* yv) {      // rows past the segment: its last
-    const uint16_t* p = ub + (size_t)min(t + col, n - 1) * UW + 8 * kq;
+  const uint16_t* yb = MODE ? reinterpret_cast<const uint16_t*>(a.y.p) + (int64_t)row0 * a.y.ld + c : nullptr;
+  float* sp = MODE == SCAN_WHOLE ? a.state + (size_t)a.slots[blockIdx.x] * W + c : sums + (size_t)blockIdx.x * 2 * W + c;
+  float S = 0.f, A = 1.f;
+  if (MODE == SCAN_APPLY || (MODE == SCAN_WHOLE && ctx_lens[blockIdx.x] > n)) S = sp[0];
+
+  u32x4_t pre[NL];
+  uint16_t yv[2][4], yn[2][4];
+  const int pieces = SCAN_TILE * 4 * kb;
+  int prow[NL], pk[NL];                                 // row and columns of this thread's pieces
 #pragma unroll
-    for (int k = 0; k < KS; ++k) f[k] = *reinterpret_cast<const u32x4_t*>(p + 32 * min(k, a.KP / 32 - 1));
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int r = min(t + 4 * kq + e, n - 1);
-      o[e] = ub[(size_t)r * UW + ku];
-      if (APPLY) yv[e] = yb[r * a.y.ld];
-    }
-  };
-  load(0, uf, uo, yo);
-  for (int t = 0; t < n; t += 16) {
-    load(t + 16, un, uon, yon);
-    f32x4_t pr{0.f, 0.f, 0.f, 0.f}, pi{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int k = 0; k < KS; ++k) {
-      if (32 * k < a.KP) {
-        pr = mfma16(uf[k], wr[k], pr);
-        pi = mfma16(uf[k], wi[k], pi);
-      }
-    }
-    float ta[4], tb[4], ga = 1.f, gb = 0.f;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      lru_gates<uint16_t>(pr[e] + br, pi[e] + bi, bf2f(uo[e]), rate, ta[e], tb[e]);
-      if (t + 4 * kq + e >= n) {
-        ta[e] = 1.f;
-        tb[e] = 0.f;
-      }
-      ga *= ta[e];
-      gb = ta[e] * gb + tb[e];
-    }
-    // composition over the four lane groups, up to and with the own one
-#pragma unroll
-    for (int d = 16; d <= 32; d *= 2) {
-      const float pa = __shfl(ga, lane - d, 64), pb = __shfl(gb, lane - d, 64);
-      if (lane >= d) {
-        gb = ga * pb + gb;
-        ga = ga * pa;
-      }
-    }
-    const float la = __shfl(ga, 48 + col, 64), lb = __shfl(gb, 48 + col, 64);
-    if constexpr (APPLY) {
-      float ea = __shfl(ga, lane - 16, 64), eb = __shfl(gb, lane - 16, 64);
-      if (kq == 0) {
-        ea = 1.f;
-        eb = 0.f;
-      }
-      float s = ea * S + eb;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        s = ta[e] * s + tb[e];
-        const int r = t + 4 * kq + e;
-        if (r < n && live) out[(size_t)(row0 + r) * W + c] = f2bf(s * gelu_tanh<uint16_t>(bf2f(yo[e]) + by));
-      }
-      S = la * S + lb;
-    } else {
-      S = la * S + lb;
-      A *= la;
-    }
-#pragma unroll
-    for (int k = 0; k < KS; ++k) uf[k] = un[k];
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      uo[e] = uon[e];
-      if (APPLY) yo[e] = yon[e];
-    }
+  for (int i = 0; i < NL; ++i) {
+    const int e = min(tid + 256 * i, pieces - 1);      // past the last: it again
+    prow[i] = e / (4 * kb);
+    pk[i] = 8 * (e - prow[i] * 4 * kb);
   }
-  if (!APPLY && kq == 0 && live) {
-    sp[0] = A;
-    sp[W] = S;
+  auto fetch = [&](int t) {                            // rows past the segment: its last
+#pragma unroll
+    for (int i = 0; i < NL; ++i) pre[i] = *reinterpret_cast<const u32x4_t*>(ub + (size_t)min(t + prow[i], n - 1) * UW + pk[i]);
+    if constexpr (MODE != SCAN_SUMS)
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) yn[h][e] = yb[min(t + 16 * h + 4 * kq + e, n - 1) * a.y.ld];
+  };
+  auto put = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < NL; ++i) *reinterpret_cast<u32x4_t*>(&tile[buf][prow[i]][pk[i]]) = pre[i];
+#pragma unroll
+    for (int h = 0; h < 2; ++h)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) yv[h][e] = yn[h][e];
+  };
+  fetch(0);
+  put(0);
+  __syncthreads();
+  for (int t = 0, buf = 0; t < n; t += SCAN_TILE, buf ^= 1) {
+    if (t + SCAN_TILE < n) fetch(t + SCAN_TILE);
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      f32x4_t pr{br, br, br, br}, pi{bi, bi, bi, bi};
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        const u32x4_t uf = *reinterpret_cast<const u32x4_t*>(&tile[buf][16 * h + col][32 * min(k, kb - 1) + 8 * kq]);
+        pr = mfma16(uf, wr[k], pr);
+        pi = mfma16(uf, wi[k], pi);
+      }
+      float ta[4], tb[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        lru_gates<uint16_t>(pr[e], pi[e], bf2f(tile[buf][16 * h + 4 * kq + e][ku]), rate, ta[e], tb[e]);
+      if (t + 16 * h + 16 > n)
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (t + 16 * h + 4 * kq + e >= n) {
+            ta[e] = 1.f;
+            tb[e] = 0.f;
+          }
+      float ga = ta[0], gb = tb[0];
+#pragma unroll
+      for (int e = 1; e < 4; ++e) {
+        ga *= ta[e];
+        gb = ta[e] * gb + tb[e];
+      }
+      // composition over the four lane groups: swaps leave every lane with both values of its pair of groups, then of the
+      // two pairs, in their order
+      float ea = ga, eb = gb, oa = ga, ob = gb;
+      swap16(ea, oa);
+      swap16(eb, ob);
+      float fa = ea * oa, fb = oa * eb + ob, la = fa, lb = fb;
+      swap32(fa, la);
+      swap32(fb, lb);
+      if constexpr (MODE != SCAN_SUMS) {
+        float s = kq & 2 ? fa * S + fb : S;
+        s = kq & 1 ? ea * s + eb : s;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          s = ta[e] * s + tb[e];
+          const int r = t + 16 * h + 4 * kq + e;
+          if (r < n && live) out[(size_t)(row0 + r) * W + c] = f2bf(s * gelu_tanh<uint16_t>(bf2f(yv[h][e]) + by));
+        }
+      } else {
+        A *= fa * la;
+      }
+      S = la * (fa * S + fb) + lb;
+    }
+    if (t + SCAN_TILE < n) put(buf ^ 1);
+    __syncthreads();
+  }
+  if (kq == 0 && live) {
+    if (MODE == SCAN_SUMS) {
+      sp[0] = A;
+      sp[W] = S;
+    } else if (MODE == SCAN_WHOLE) {
+      sp[0] = S;
+    }
   }
 }
 
 // ------------------------------------------------------------------------------------------ one token per sequence
-// u of 16 rows x a block's columns into LDS (row stride ldu), the block's raw inputs into the state by the workgroup whose
-// channels n0 .. n1 they are
+// u of up to 16 rows x a block's columns into LDS (row stride ldu), the block's raw inputs into the state by the workgroup
+// whose channels n0 .. n1 they are
 template <typename ACT, typename LT, int V>
-__device__ __forceinline__ void step_conv(const LruArgs& a, int b0, int nb, int rows, int blk, int n0, int n1,
-                                          const int32_t* positions, LT* ul, int ldu) {
-  const int nv = a.KP / V, back = a.taps - 1;
-  for (int i = threadIdx.x; i < rows * nv; i += blockDim.x) {
-    const int r = i / nv, k = (i - r * nv) * V;
-    Vec<V> y = zerov<V>();
-    if (r < nb && k < a.bs) {
-      const int b = b0 + r, c = blk * a.bs + k, pos = positions[b];
-      float* st = a.tail + (size_t)a.slots[b] * a.taps * a.W + c;
-      const Vec<V> x = lru_ld<ACT, V>(a.x, b, c), bx = ldv<V>(a.bx + c), w0 = ldv<V>(a.conv + (size_t)back * a.W + c);
-      y = ldv<V>(a.cb + c);
-      Vec<V> o[3], w[3];                               // three rows back asked for together
+__device__ __forceinline__ void step_conv(const LruArgs& a, int b0, int nb, int blk, int n0, int n1, const int32_t* positions, LT* ul,
+                                          int ldu) {
+  constexpr int IN = 2;                                // vectors a thread asks for together
+  const int nv = a.KP / V, back = a.taps - 1, items = nb * nv;
+  for (int i0 = threadIdx.x; i0 < items; i0 += IN * blockDim.x) {
+    Vec<V> x[IN], o[IN][3], y[IN], bx[IN], w[IN][4];
+    int64_t at[IN];
+    int ps[IN];
 #pragma unroll
-      for (int d = 1; d <= 3; ++d) {
-        const bool on = d <= back && d <= pos;
-        o[d - 1] = on ? ldv<V>(st + (size_t)((pos - d) % a.taps) * a.W) : zerov<V>();
-        w[d - 1] = on ? ldv<V>(a.conv + (size_t)(back - d) * a.W + c) : zerov<V>();
+    for (int j = 0; j < IN; ++j) {                     // past the last or in the pad: another's, not stored
+      const int i = min(i0 + j * (int)blockDim.x, items - 1), r = i / nv, k = (i - r * nv) * V, b = b0 + r;
+      const int c = blk * a.bs + min(k, a.bs - V);
+      ps[j] = positions[b];
+      at[j] = (int64_t)a.slots[b] * a.taps * a.W + c;
+      x[j] = lru_ld<ACT, V>(a.x, b, c);
+      bx[j] = ldv<V>(a.bx + c);
+      y[j] = ldv<V>(a.cb + c);
+#pragma unroll
+      for (int d = 0; d < 4; ++d) w[j][d] = ldv<V>(a.conv + (size_t)max(back - d, 0) * a.W + c);
+#pragma unroll
+      for (int d = 1; d <= 3; ++d) o[j][d - 1] = ldv<V>(a.tail + at[j] + (size_t)(max(ps[j] - d, 0) % a.taps) * a.W);
+    }
+#pragma unroll
+    for (int j = 0; j < IN; ++j) {
+      const int i = i0 + j * (int)blockDim.x, r = i / nv, k = (i - r * nv) * V, pos = ps[j];
+      if (i >= items) break;
+      if (k >= a.bs) {
+        stv<V>(ul + r * ldu + k, zerov<V>());
+        continue;
       }
 #pragma unroll
       for (int e = 0; e < V; ++e) {
-        y.v[e] += w0.v[e] * (x.v[e] + bx.v[e]);
+        y[j].v[e] += w[j][0].v[e] * (x[j].v[e] + bx[j].v[e]);
 #pragma unroll
-        for (int d = 0; d < 3; ++d) y.v[e] += w[d].v[e] * (o[d].v[e] + bx.v[e]);
+        for (int d = 1; d <= 3; ++d) y[j].v[e] += d <= back && d <= pos ? w[j][d].v[e] * (o[j][d - 1].v[e] + bx[j].v[e]) : 0.f;
       }
       for (int d = 4; d <= back && d <= pos; ++d) {
-        const Vec<V> od = ldv<V>(st + (size_t)((pos - d) % a.taps) * a.W), wd = ldv<V>(a.conv + (size_t)(back - d) * a.W + c);
+        const int c = blk * a.bs + k;
+        const Vec<V> od = ldv<V>(a.tail + at[j] + (size_t)((pos - d) % a.taps) * a.W), wd = ldv<V>(a.conv + (size_t)(back - d) * a.W + c);
 #pragma unroll
-        for (int e = 0; e < V; ++e) y.v[e] += wd.v[e] * (od.v[e] + bx.v[e]);
+        for (int e = 0; e < V; ++e) y[j].v[e] += wd.v[e] * (od.v[e] + bx[j].v[e]);
       }
-      if (back > 0 && k >= n0 && k < n1) stv<V>(st + (size_t)(pos % a.taps) * a.W, x);
+      if (back > 0 && k >= n0 && k < n1) stv<V>(a.tail + at[j] + (size_t)(pos % a.taps) * a.W, x[j]);
+      stv<V>(ul + r * ldu + k, y[j]);
     }
-    stv<V>(ul + r * ldu + k, y);
   }
 }
 
-// grid (rows / 16, blocks * NP / 64 rounded up); four waves of 16 channels.  V: vectors of channels (4 or 1)
+// 1-D grid of rows / 16 x blocks x NP / 64, rounded up each; where eight divides the blocks, an XCD takes all of a block's, so
+// that its matrices and inputs come into one L2.  Four waves of 16 channels.  V: vectors of channels (4 or 1)
 template <int V>
 __global__ void __launch_bounds__(256) rglru_step_kernel(LruArgs a, const int32_t* __restrict__ positions,
                                                         const int32_t* __restrict__ ctx_lens, int B, uint16_t* __restrict__ out) {
@@ -297,8 +352,15 @@ __global__ void __launch_bounds__(256) rglru_step_kernel(LruArgs a, const int32_
   uint16_t* ul = reinterpret_cast<uint16_t*>(smem);
   const int ldu = a.KP + 8, W = a.W;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
-  const int groups = (a.NP + 63) / 64, blk = blockIdx.y / groups, g0 = (blockIdx.y - blk * groups) * 64, n0 = g0 + 16 * w;
-  const int b0 = 16 * blockIdx.x, nb = min(16, B - b0), b = b0 + min(col, nb - 1);
+  const int groups = (a.NP + 63) / 64, per = groups * ((B + 15) / 16);
+  int blk = blockIdx.x / per, rest = blockIdx.x - blk * per;
+  if (a.blocks % 8 == 0) {
+    const int i = blockIdx.x / 8;
+    blk = blockIdx.x % 8 + 8 * (i / per);
+    rest = i % per;
+  }
+  const int g0 = rest % groups * 64, n0 = g0 + 16 * w, b0 = 16 * (rest / groups), nb = min(16, B - b0);
+  const int b = b0 + min(col, nb - 1);
   // this lane's row and channels 4 kq .. of the wave's: what the end needs, asked for first
   const int k0 = n0 + 4 * kq;
   const bool on = col < nb && k0 < a.bs;
@@ -325,24 +387,28 @@ __global__ void __launch_bounds__(256) rglru_step_kernel(LruArgs a, const int32_
 #pragma unroll
     for (int e = 0; e < 4; ++e) y.v[e] += by.v[e];
   }
-  step_conv<uint16_t, uint16_t, V>(a, b0, nb, 16, blk, g0, g0 + 64, positions, ul, ldu);
-  __syncthreads();
-  if (n0 >= a.NP) return;
-  f32x4_t pr{0.f, 0.f, 0.f, 0.f}, pi{0.f, 0.f, 0.f, 0.f};
-  const uint16_t* p = reinterpret_cast<const uint16_t*>(a.wg) + ((size_t)blk * a.NP + n0 + col) * a.KP + 8 * kq;
+  const uint16_t* p = reinterpret_cast<const uint16_t*>(a.wg) + ((size_t)blk * a.NP + min(n0, a.NP - 16) + col) * a.KP + 8 * kq;
   const size_t second = (size_t)a.blocks * a.NP * a.KP;
   const int KS = a.KP / 32;
-  for (int s0 = 0; s0 < KS; s0 += 4) {                 // four steps' matrices in flight (past the last: again, not used)
-    u32x4_t wr[4], wi[4];
+  u32x4_t wr[4], wi[4];                                // four steps' matrices in flight (past the last: again, not used)
+  auto matrices = [&](int s0) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int o = 32 * min(s0 + j, KS - 1);
       wr[j] = *reinterpret_cast<const u32x4_t*>(p + o);
       wi[j] = *reinterpret_cast<const u32x4_t*>(p + second + o);
     }
+  };
+  matrices(0);
+  step_conv<uint16_t, uint16_t, V>(a, b0, nb, blk, g0, g0 + 64, positions, ul, ldu);
+  __syncthreads();
+  if (n0 >= a.NP) return;
+  f32x4_t pr{0.f, 0.f, 0.f, 0.f}, pi{0.f, 0.f, 0.f, 0.f};
+  for (int s0 = 0; s0 < KS; s0 += 4) {
+    if (s0) matrices(s0);
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-      if (s0 + j < KS) {
+      if (s0 + j < KS) {                               // columns past the rows there are: not looked at
         const u32x4_t uf = *reinterpret_cast<const u32x4_t*>(ul + col * ldu + 32 * (s0 + j) + 8 * kq);
         pr = mfma16(wr[j], uf, pr);
         pi = mfma16(wi[j], uf, pi);
@@ -392,7 +458,7 @@ __global__ void __launch_bounds__(256) rglru_any_kernel(LruArgs a, const ACT* __
   if (u) {
     for (int k = threadIdx.x; k < a.bs; k += 256) ul[k] = ld1(u + (size_t)t * a.blocks * a.KP + blk * a.KP + k);
   } else {
-    step_conv<ACT, float, 1>(a, t, 1, 1, blk, 0, a.bs, positions, ul, a.KP);
+    step_conv<ACT, float, 1>(a, t, 1, blk, 0, a.bs, positions, ul, a.KP);
     __syncthreads();
     for (int k = threadIdx.x; k < a.bs; k += 256) ul[k] = round_act(ul[k], (const ACT*)nullptr);
   }
@@ -489,7 +555,7 @@ CFC_API int cfc_rglru_step(int f32, const void* x, int x_split, int64_t x_ld, in
   const LruArgs a{{x, x_split, x_ld, x_plane}, {y, y_split, y_ld, y_plane}, bx, conv, cb, taps, br, bi, rate, by, wg, blocks, bs, KP,
                   NP, blocks * bs, tail, state, slots};
   if (!f32 && KP <= 1024) {
-    const dim3 grid((B + 15) / 16, blocks * ((NP + 63) / 64));
+    const int grid = (B + 15) / 16 * blocks * ((NP + 63) / 64);
     const size_t lds = (size_t)16 * (KP + 8) * 2;
     const bool v4 = bs % 4 == 0 && lru_cols_vec(a.x, 0) && lru_cols_vec(a.y, 0) && ((uintptr_t)out & 7) == 0;
     if (v4) rglru_step_kernel<4><<<grid, 256, lds, stream>>>(a, positions, ctx_lens, B, (uint16_t*)out);
@@ -504,17 +570,19 @@ CFC_API int cfc_rglru_step(int f32, const void* x, int x_split, int64_t x_ld, in
 }
 
 // packed portions, x and y activations.  tiles as in short_conv; chunks [n][2] {first row, rows} (segments), chunk_cu
-// [portions + 1]; u scratch [T][blocks KP] activations; sums scratch, n or (general path) T times 2 W floats
+// [portions + 1], or whole: every portion one segment (both unused); u scratch [T][blocks KP] activations; sums scratch, n or (general path) T times 2 W floats
 CFC_API int cfc_rglru_prefill(int f32, const void* x, int64_t x_ld, const void* y, int64_t y_ld, const float* bx, const float* conv,
                               const float* cb, int taps, const float* br, const float* bi, const float* rate, const float* by,
                               const void* wg, int blocks, int bs, int KP, int NP, float* tail, float* state, const int32_t* slots,
-                              const int32_t* tiles, int n_tiles, const int32_t* chunks, int n_chunks, const int32_t* chunk_cu,
+                              const int32_t* tiles, int n_tiles, int whole, const int32_t* chunks, int n_chunks, const int32_t* chunk_cu,
                               const int32_t* cu_q, const int32_t* ctx_lens, int portions, int T, void* u, float* sums, void* out,
                               hipStream_t stream) {
   if (T <= 0 || portions <= 0) return 0;
-  if (blocks < 1 || bs < 1 || KP < bs || KP % 4 || taps < 1 || !wg || !tail || !state || !slots || !tiles || !chunks || !chunk_cu || !cu_q ||
-      !ctx_lens || !u || !sums || n_tiles < 1 || n_chunks < 1)
+  if (blocks < 1 || bs < 1 || KP < bs || KP % 4 || taps < 1 || !wg || !tail || !state || !slots || !tiles || !cu_q ||
+      !ctx_lens || !u || n_tiles < 1)
     return -1;
+  const bool mfma = !f32 && KP <= cfc_rglru_max_block();
+  if ((mfma && !whole && (!chunks || !chunk_cu || n_chunks < 1)) || (!(mfma && whole) && !sums)) return -1;
   if (!f32 && (KP % 32 || NP < bs || NP % 16)) return -2;
   const LruArgs a{{x, 0, x_ld, 0}, {y, 0, y_ld, 0}, bx, conv, cb, taps, br, bi, rate, by, wg, blocks, bs, KP, NP, blocks * bs, tail,
                   state, slots};
@@ -523,20 +591,24 @@ CFC_API int cfc_rglru_prefill(int f32, const void* x, int64_t x_ld, const void* 
   if (f32) rc = v4 ? conv_go<float, 4>(stream, n_tiles, a, tiles, u) : conv_go<float, 1>(stream, n_tiles, a, tiles, u);
   else rc = v4 ? conv_go<uint16_t, 4>(stream, n_tiles, a, tiles, u) : conv_go<uint16_t, 1>(stream, n_tiles, a, tiles, u);
   if (rc) return rc;
-  if (!f32 && KP <= cfc_rglru_max_block()) {
-    const dim3 grid(n_chunks, blocks * ((NP + 63) / 64));
+  if (mfma) {
+    const dim3 grid(whole ? portions : n_chunks, blocks * ((NP + 63) / 64));
     const uint16_t* up = (const uint16_t*)u;
-#define RS(KS, AP) rglru_scan_kernel<KS, AP><<<grid, 256, 0, stream>>>(a, up, chunks, sums, (uint16_t*)out)
-#define RP(AP)                \
-  if (KP <= 64) RS(2, AP);    \
-  else if (KP <= 128) RS(4, AP); \
-  else if (KP <= 256) RS(8, AP); \
-  else RS(16, AP)
-    RP(false);
+#define RS(KS, M) rglru_scan_kernel<KS, M><<<grid, 256, 0, stream>>>(a, up, chunks, cu_q, ctx_lens, sums, (uint16_t*)out)
+#define RP(M)                    \
+  if (KP <= 64) RS(2, M);        \
+  else if (KP <= 128) RS(4, M);  \
+  else if (KP <= 256) RS(8, M);  \
+  else RS(16, M)
+    if (whole) {
+      RP(SCAN_WHOLE);
+      return CFC_CHECK_LAUNCH();
+    }
+    RP(SCAN_SUMS);
     if (const int e = CFC_CHECK_LAUNCH()) return e;
     if (a.W % 4) carry_kernel<1><<<dim3(portions, (a.W + 63) / 64), 64, 0, stream>>>(chunk_cu, cu_q, ctx_lens, slots, a.W, sums, state);
     else carry_kernel<4><<<dim3(portions, (a.W + 255) / 256), 64, 0, stream>>>(chunk_cu, cu_q, ctx_lens, slots, a.W, sums, state);
-    RP(true);
+    RP(SCAN_APPLY);
 #undef RP
 #undef RS
     return CFC_CHECK_LAUNCH();

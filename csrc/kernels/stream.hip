@@ -37,15 +37,19 @@ __global__ void __launch_bounds__(256) embed_f32_kernel(float* __restrict__ out,
   const int t = blockIdx.x;
   const int id = min(max(ids[t], 0), vocab - 1);
   const double pos = positions ? positions[t] : 0;
-  for (int c = threadIdx.x; c < W; c += 256) {
-    float v = scale * ld1(table + (size_t)id * W + c);
-    if (positions) {
-      // turns per position in 64 bits: the angle's fraction of a turn keeps its digits however far the position
-      const double n = pos * turns[c >> 1];
-      const float f = (float)(n - floor(n));
-      v += c & 1 ? cospif(2.f * f) : sinpif(2.f * f);
-    }
-    out[(size_t)t * W + c] = v;
+  const TAB* row = table + (size_t)id * W;
+  float* o = out + (size_t)t * W;
+  if (!positions) {
+    for (int c = threadIdx.x; c < W; c += 256) o[c] = scale * ld1(row + c);
+    return;
+  }
+  for (int c = 2 * threadIdx.x; c < W; c += 512) {
+    // turns per position in 64 bits: the angle's fraction of a turn keeps its digits however far the position
+    const double n = pos * turns[c >> 1];
+    float sn, co;
+    sincospif(2.f * (float)(n - floor(n)), &sn, &co);
+    o[c] = scale * ld1(row + c) + sn;
+    if (c + 1 < W) o[c + 1] = scale * ld1(row + c + 1) + co;
   }
 }
 

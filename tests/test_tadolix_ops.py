@@ -194,7 +194,7 @@ def test_distance_table_rows():
 ATTN = [  # H, G, dim, vdim, scale, cap, rows of the table, its far end, chunk
     (4, 2, 64, 64, 0.2, 50.0, 32, 120, 100), (8, 2, 48, 48, 0.25, 45.0, 16, 50, 64), (3, 1, 18, 14, 1.0, 5.0, 7, 17, 17),
     (2, 2, 36, 9, 0.4, 0.0, 10, 40, 70), (20, 1, 128, 128, 0.09, 50.0, 32, 200, 290), (40, 1, 32, 32, 0.5, 3.0, 4, 6, 1),
-    (2, 1, 140, 160, 0.09, 40.0, 32, 500, 0), (2, 1, 192, 180, 0.1, 8.0, 2, 5, 65), (1, 1, 256, 256, 0.06, 50.0, 20, 90, 150),
+    (2, 1, 140, 160, 0.09, 40.0, 32, 500, 0), (4, 2, 64, 64, 0.2, 60.0, 12, 70, 128), (2, 1, 192, 180, 0.1, 8.0, 2, 5, 65), (1, 1, 256, 256, 0.06, 50.0, 20, 90, 150),
     (2, 2, 300, 33, 0.06, 30.0, 32, 100, 45), (24, 1, 64, 62, 0.2, 60.0, 40, 400, 0), (4, 4, 96, 96, 0.1, 30.0, 1, 9, 33)]
 
 
@@ -230,7 +230,7 @@ def test_attention_in_portions_and_decoded(device, dtype, case):
     several key slices; gated or not, into rows of another's width; garbage pages in the pool do not matter."""
     H, G, dim, vdim, scale, cap, _, far, chunk = case
     rel, a = attn_case(case, device)
-    assert a.capped == (0 if not cap else 2 if dim * scale <= 0.34 * cap else 1)
+    assert a.capped == (0 if not cap else 3 if dim * scale <= 0.24 * cap else 2 if dim * scale <= 0.34 * cap else 1)
     lens, tables = [300, 131], [[3, 9, 1, 14, 7, 5, 11, 0, 8, 2], [13, 4, 6, 12, 10]]
     rows = PagedHeads(16, G, a.D, 0, 0, device, dtype)
     for t, w in ((rows.k, dim), (rows.v, vdim)):
@@ -383,14 +383,14 @@ def test_linear_recurrence_in_portions_and_decoded(device, dtype, case):
     want, yx = want_lru(p, x, y, dtype), torch.cat([y, x], 1).to(device, dtype)
     limit = 5e-5 if dtype == torch.float32 else 2e-2
 
-    def portions(ranges, slots, tail, state):
+    def portions(ranges, slots, tail, state, whole=False):
         idx = torch.cat([torch.arange(lo, hi) for lo, hi in ranges])
         cu = np.cumsum([0] + [hi - lo for lo, hi in ranges]).tolist()
         por = [(cu[s], hi - lo, lo, s) for s, (lo, hi) in enumerate(ranges)]
-        seg, seg_cu = R.chunk_plan(cu, L.SEGMENT)
+        seg, seg_cu = (None, None) if whole else (i32(t, device) for t in R.chunk_plan(cu, L.SEGMENT))
         rows = yx[idx.to(device)].contiguous()
         out = L.prefill(r, Cols(rows, W, W), Cols(rows, 0, W), i32(slots, device), i32(cu, device), i32([hi for _, hi in ranges], device),
-                        i32(S.conv_tiles(por, 32), device), i32(seg, device), i32(seg_cu, device), tail, state,
+                        i32(S.conv_tiles(por, 32), device), seg, seg_cu, tail, state,
                         torch.empty(cu[-1], W, dtype=dtype, device=device))
         close(out, want[idx], limit)
 
@@ -410,8 +410,9 @@ def test_linear_recurrence_in_portions_and_decoded(device, dtype, case):
             close(out, want[both], limit)
         assert torch.equal(state[[1, 3]], before[1][[1, 3]]) and torch.equal(tail[[1, 3]], before[0][[1, 3]])
     tail, state = rnd(4, r.ring, W, seed=7).to(device), rnd(4, W, seed=8).to(device)
-    portions([(0, 150), (0, 1), (0, 257)], [3, 0, 2], tail, state)
-    portions([(150, 152), (1, 34), (257, 290)], [3, 0, 2], tail, state)
+    for whole in (False, True):
+        portions([(0, 150), (0, 1), (0, 257)], [3, 0, 2], tail, state, whole)
+        portions([(150, 152), (1, 34), (257, 290)], [3, 0, 2], tail, state, whole)
 
 
 @pytest.mark.parametrize("device", DEVICES)
@@ -429,6 +430,12 @@ def test_decays_near_one_keep_their_digits(device):
                         i32(S.conv_tiles([(0, T, 0, 0)], 32), device), i32(seg, device), i32(cu, device), torch.zeros(1, 1, W, device=device),
                         torch.zeros(1, W, device=device), torch.empty(T, W, dtype=dtype, device=device))
         close(out / want.abs().amax().to(device), want / want.abs().amax(), 1e-4 if dtype == torch.float32 else 2e-2)
+
+
+def test_portions_as_segments():
+    assert L.whole_portions([0, 1, 129], 64) and not L.whole_portions([0, 1, 130], 64)
+    assert L.whole_portions(list(range(0, 16 * 700 + 1, 700)), 4096) and not L.whole_portions(list(range(0, 15 * 700 + 1, 700)), 4096)
+    assert not L.whole_portions([0, 5000] + list(range(5001, 5016)), 4096)
 
 
 def test_segments_match_the_kernels():
