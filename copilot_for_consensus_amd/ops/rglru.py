@@ -18,7 +18,6 @@ from .stream import _act
 
 SEGMENT = 128            # tokens per segment of the prompt kernels
 MAX_BLOCK = 512          # block columns (padded) they take; wider ones and fp32: the general kernels
-FILL = 1024              # workgroups that fill the chip (four waves each)
 
 
 @dataclasses.dataclass
@@ -90,10 +89,9 @@ def _ref(p: RgLru, x, y, slots, positions, cu, tail, state, out):
 
 
 def whole_portions(cu, width: int) -> bool:
-    """Whether the portions of a pass are one segment each: those alone fill the chip and are about even, or none is longer
-    than a segment."""
-    n = [b - a for a, b in zip(cu, cu[1:])]
-    return max(n) <= SEGMENT or (len(n) * math.ceil(width / 64) >= FILL and max(n) * len(n) <= 2 * sum(n))
+    """Whether the portions of a pass are one segment each.  That takes as long as the longest one's tokens in turn; segments
+    take launches and two passes over all elements (microseconds measured on one MI355X)."""
+    return 0.1 * max(b - a for a, b in zip(cu, cu[1:])) <= 25.0 + 5.7e-6 * (cu[-1] - cu[0]) * width
 
 
 def _fits(p: RgLru, x: Cols, y: Cols, tail, state, out):

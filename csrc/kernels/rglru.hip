@@ -299,6 +299,7 @@ __device__ __forceinline__ void step_conv(const LruArgs& a, int b0, int nb, int 
                                           int ldu) {
   constexpr int IN = 2;                                // vectors a thread asks for together
   const int nv = a.KP / V, back = a.taps - 1, items = nb * nv;
+  const bool same = blockDim.x % nv == 0;              // a thread's vectors are of the same channels
   for (int i0 = threadIdx.x; i0 < items; i0 += IN * blockDim.x) {
     Vec<V> x[IN], o[IN][3], y[IN], bx[IN], w[IN][4];
     int64_t at[IN];
@@ -310,10 +311,17 @@ __device__ __forceinline__ void step_conv(const LruArgs& a, int b0, int nb, int 
       ps[j] = positions[b];
       at[j] = (int64_t)a.slots[b] * a.taps * a.W + c;
       x[j] = lru_ld<ACT, V>(a.x, b, c);
-      bx[j] = ldv<V>(a.bx + c);
-      y[j] = ldv<V>(a.cb + c);
+      if (j && same) {
+        bx[j] = bx[0];
+        y[j] = y[0];
 #pragma unroll
-      for (int d = 0; d < 4; ++d) w[j][d] = ldv<V>(a.conv + (size_t)max(back - d, 0) * a.W + c);
+        for (int d = 0; d < 4; ++d) w[j][d] = w[0][d];
+      } else {
+        bx[j] = ldv<V>(a.bx + c);
+        y[j] = ldv<V>(a.cb + c);
+#pragma unroll
+        for (int d = 0; d < 4; ++d) w[j][d] = ldv<V>(a.conv + (size_t)max(back - d, 0) * a.W + c);
+      }
 #pragma unroll
       for (int d = 1; d <= 3; ++d) o[j][d - 1] = ldv<V>(a.tail + at[j] + (size_t)(max(ps[j] - d, 0) % a.taps) * a.W);
     }
@@ -343,23 +351,23 @@ __device__ __forceinline__ void step_conv(const LruArgs& a, int b0, int nb, int 
   }
 }
 
-// 1-D grid of rows / 16 x blocks x NP / 64, rounded up each; where eight divides the blocks, an XCD takes all of a block's, so
-// that its matrices and inputs come into one L2.  Four waves of 16 channels.  V: vectors of channels (4 or 1)
-template <int V>
-__global__ void __launch_bounds__(256) rglru_step_kernel(LruArgs a, const int32_t* __restrict__ positions,
+// 1-D grid of rows / 16 x blocks x NP / 16 NW, rounded up each; where eight divides the blocks, an XCD takes all of a block's,
+// so that its matrices and inputs come into one L2.  NW waves of 16 channels.  V: vectors of channels (4 or 1)
+template <int V, int NW>
+__global__ void __launch_bounds__(64 * NW) rglru_step_kernel(LruArgs a, const int32_t* __restrict__ positions,
                                                         const int32_t* __restrict__ ctx_lens, int B, uint16_t* __restrict__ out) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* ul = reinterpret_cast<uint16_t*>(smem);
   const int ldu = a.KP + 8, W = a.W;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, col = lane & 15, kq = lane >> 4;
-  const int groups = (a.NP + 63) / 64, per = groups * ((B + 15) / 16);
+  const int groups = (a.NP + 16 * NW - 1) / (16 * NW), per = groups * ((B + 15) / 16);
   int blk = blockIdx.x / per, rest = blockIdx.x - blk * per;
   if (a.blocks % 8 == 0) {
     const int i = blockIdx.x / 8;
     blk = blockIdx.x % 8 + 8 * (i / per);
     rest = i % per;
   }
-  const int g0 = rest % groups * 64, n0 = g0 + 16 * w, b0 = 16 * (rest / groups), nb = min(16, B - b0);
+  const int g0 = rest % groups * (16 * NW), n0 = g0 + 16 * w, b0 = 16 * (rest / groups), nb = min(16, B - b0);
   const int b = b0 + min(col, nb - 1);
   // this lane's row and channels 4 kq .. of the wave's: what the end needs, asked for first
   const int k0 = n0 + 4 * kq;
@@ -400,7 +408,7 @@ __global__ void __launch_bounds__(256) rglru_step_kernel(LruArgs a, const int32_
     }
   };
   matrices(0);
-  step_conv<uint16_t, uint16_t, V>(a, b0, nb, blk, g0, g0 + 64, positions, ul, ldu);
+  step_conv<uint16_t, uint16_t, V>(a, b0, nb, blk, g0, g0 + 16 * NW, positions, ul, ldu);
   __syncthreads();
   if (n0 >= a.NP) return;
   f32x4_t pr{0.f, 0.f, 0.f, 0.f}, pi{0.f, 0.f, 0.f, 0.f};
@@ -555,11 +563,15 @@ CFC_API int cfc_rglru_step(int f32, const void* x, int x_split, int64_t x_ld, in
   const LruArgs a{{x, x_split, x_ld, x_plane}, {y, y_split, y_ld, y_plane}, bx, conv, cb, taps, br, bi, rate, by, wg, blocks, bs, KP,
                   NP, blocks * bs, tail, state, slots};
   if (!f32 && KP <= 1024) {
-    const int grid = (B + 15) / 16 * blocks * ((NP + 63) / 64);
+    // many rows: more channels per workgroup, so that fewer repeat a row's convolution
+    const int nw = B >= 32 && NP > 64 ? 8 : 4, grid = (B + 15) / 16 * blocks * ((NP + 16 * nw - 1) / (16 * nw));
     const size_t lds = (size_t)16 * (KP + 8) * 2;
     const bool v4 = bs % 4 == 0 && lru_cols_vec(a.x, 0) && lru_cols_vec(a.y, 0) && ((uintptr_t)out & 7) == 0;
-    if (v4) rglru_step_kernel<4><<<grid, 256, lds, stream>>>(a, positions, ctx_lens, B, (uint16_t*)out);
-    else rglru_step_kernel<1><<<grid, 256, lds, stream>>>(a, positions, ctx_lens, B, (uint16_t*)out);
+#define ST(V, NW) rglru_step_kernel<V, NW><<<grid, 64 * NW, lds, stream>>>(a, positions, ctx_lens, B, (uint16_t*)out)
+    if (nw == 8) { if (v4) ST(4, 8); else ST(1, 8); }
+    else if (v4) ST(4, 4);
+    else ST(1, 4);
+#undef ST
     return CFC_CHECK_LAUNCH();
   }
   if (KP > LRU_ANY_MAX) return -3;

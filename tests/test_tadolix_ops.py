@@ -416,6 +416,27 @@ def test_linear_recurrence_in_portions_and_decoded(device, dtype, case):
 
 
 @pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("case", [(35, 5, 3), (192, 2, 4), (800, 8, 5), (260, 1, 2)])
+def test_linear_recurrence_of_many_decoded_rows(device, dtype, case):
+    """More rows than a tile, each at another position of its own sequence, slots in any order."""
+    W, blocks, taps = case
+    B = 37
+    p, r = lru_case(W, blocks, taps, dtype, device)
+    seqs = [(rnd(9, W, seed=2 * b).to(dtype).float(), rnd(9, W, seed=2 * b + 1).to(dtype).float()) for b in range(B)]
+    want = [want_lru(p, x, y, dtype) for x, y in seqs]
+    slots = torch.randperm(B + 2, generator=torch.Generator().manual_seed(1))[:B].tolist()
+    tail, state = rnd(B + 2, r.ring, W, seed=6).to(device), rnd(B + 2, W, seed=7).to(device)
+    for t in range(9):
+        rows = [b for b in range(B) if b % 9 <= t]            # sequence b starts at step b % 9
+        at = [t - b % 9 for b in rows]
+        c = slabs(torch.stack([torch.cat([seqs[b][1][i], seqs[b][0][i]]) for b, i in zip(rows, at)]), 5, seed=t).to(device)
+        out = L.step(r, Cols(c, W, W), Cols(c, 0, W), i32([slots[b] for b in rows], device), i32(at, device), i32([i + 1 for i in at], device),
+                     tail, state, torch.empty(len(rows), W, dtype=dtype, device=device))
+        close(out, torch.stack([want[b][i] for b, i in zip(rows, at)]), 5e-5 if dtype == torch.float32 else 2e-2)
+
+
+@pytest.mark.parametrize("device", DEVICES)
 def test_decays_near_one_keep_their_digits(device):
     """The slowest decays: 1 - a^2 far below a's rounding, over a long portion."""
     T, W = 512, 64
@@ -433,9 +454,8 @@ def test_decays_near_one_keep_their_digits(device):
 
 
 def test_portions_as_segments():
-    assert L.whole_portions([0, 1, 129], 64) and not L.whole_portions([0, 1, 130], 64)
-    assert L.whole_portions(list(range(0, 16 * 700 + 1, 700)), 4096) and not L.whole_portions(list(range(0, 15 * 700 + 1, 700)), 4096)
-    assert not L.whole_portions([0, 5000] + list(range(5001, 5016)), 4096)
+    assert L.whole_portions([0, 1, 129], 64) and not L.whole_portions([0, 2800], 4096)
+    assert L.whole_portions(list(range(0, 6 * 2800 + 1, 2800)), 4096) and not L.whole_portions([0, 5000] + list(range(5001, 5016)), 4096)
 
 
 def test_segments_match_the_kernels():
