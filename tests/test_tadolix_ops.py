@@ -192,7 +192,7 @@ def test_distance_table_rows():
 
 # ------------------------------------------------------------------ attention
 ATTN = [  # H, G, dim, vdim, scale, cap, rows of the table, its far end, chunk
-    (4, 2, 64, 64, 0.2, 50.0, 32, 120, 100), (8, 2, 48, 48, 0.25, 45.0, 16, 50, 64), (3, 1, 18, 14, 1.0, 5.0, 7, 17, 17),
+    (4, 2, 64, 64, 0.2, 50.0, 32, 120, 100), (6, 2, 48, 40, 0.25, 45.0, 16, 50, 56), (3, 1, 18, 14, 1.0, 5.0, 7, 17, 17),
     (2, 2, 36, 9, 0.4, 0.0, 10, 40, 70), (20, 1, 128, 128, 0.09, 50.0, 32, 200, 290), (40, 1, 32, 32, 0.5, 3.0, 4, 6, 1),
     (2, 1, 140, 160, 0.09, 40.0, 32, 500, 0), (4, 2, 64, 64, 0.2, 60.0, 12, 70, 128), (2, 1, 192, 180, 0.1, 8.0, 2, 5, 65), (1, 1, 256, 256, 0.06, 50.0, 20, 90, 150),
     (2, 2, 300, 33, 0.06, 30.0, 32, 100, 45), (24, 1, 64, 62, 0.2, 60.0, 40, 400, 0), (4, 4, 96, 96, 0.1, 30.0, 1, 9, 33)]
